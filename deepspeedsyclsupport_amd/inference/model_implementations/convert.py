@@ -566,8 +566,17 @@ def _put(param, src):
 
 def load_layer(model: DSInferenceModel, idx, lw):
     """Canonical full weights of layer `idx` -> this rank's shard of the injected layer."""
+    layer = model.layers[idx]
+    if hasattr(model, "shard_layer"):  # models with layers of several kinds name their own parameters
+        for path, t in model.shard_layer(idx, lw).items():
+            p = layer.get_parameter(path)
+            if p.shape != t.shape:
+                raise ValueError(f"layer {idx}: {path} is {tuple(t.shape)} in the checkpoint, {tuple(p.shape)} by the "
+                                 f"configuration")
+            _put(p, t)
+        return
     for name, t in shard_layer(model.spec, lw, model.tp_rank, model.tp_size).items():
-        _put(getattr(model.layers[idx], name), t)
+        _put(getattr(layer, name), t)
 
 
 def load_top(model: DSInferenceModel, top):

@@ -60,6 +60,12 @@ class DSModelSpec:
     moe_top_k: int = 2
     moe_renormalize: bool = True     # renormalise the top-k routing weights to sum to 1
     moe_residual: bool = False       # PR-MoE: softmax(coefficient(x)) mixes the routed experts with a dense MLP
+    norm_bias: bool = True           # "ln" norms: with a bias
+    # decoders whose layers differ (`model_implementations/hybrid.py`): one dict per layer, {"type": mixer, "mixer":
+    # its sizes and constants, "mlp": the feed-forward's or None}; empty for the uniform decoders above
+    layer_specs: tuple = ()
+    streams: int = 1                 # residual streams (hyper-connections)
+    residual_mult: float = 1.0       # factor of every sublayer's output
 
     def __post_init__(self):
         if not self.head_dim:
@@ -157,15 +163,24 @@ class RaggedMeta:
     seq_ids: torch.Tensor            # [T] sequence of every token
     cu_q: torch.Tensor               # [S + 1] token offsets
     work: torch.Tensor               # [W, 2] (sequence, 128-row query block) for the prefill sequences
-    last_idx: torch.Tensor           # [S] row of each sequence's last token
+    last_idx: torch.Tensor           # rows whose logits are wanted: [S] each sequence's last token, or a list given
     n_decode: int                    # sequences [0, n_decode) are single-token decodes
     cu_host: List[int]
     start_host: List[int]
     max_len: int                     # host upper bound of seq_lens (decode split sizing)
     block_size: int
+    slots: Optional[torch.Tensor] = None     # [S] state slot of every sequence (models with recurrent layers)
+    seq_list: Optional[torch.Tensor] = None  # sequences whose portion is short: recurrent layers go token by token
+    chunk_seqs: Optional[torch.Tensor] = None  # the others, which go by chunks of `STATE_CHUNK` tokens
+    chunk_work: Optional[torch.Tensor] = None  # [N, 2] (sequence, chunk) of those
+
+    STATE_CHUNK = 64     # tokens per chunk of a recurrent layer's parallel form
+    STEP_TOKENS = 16     # portions up to this long pass a recurrent layer token by token
 
     @staticmethod
-    def build(starts, n_new, block_lists, n_decode, block_size, device):
+    def build(starts, n_new, block_lists, n_decode, block_size, device, slots=None, logit_rows=None):
+        """`slots`: state slots of the sequences; `logit_rows`: rows (of the concatenated tokens) whose logits are
+        wanted instead of every sequence's last."""
         S = len(starts)
         cu = [0]
         for n in n_new:
@@ -181,31 +196,100 @@ class RaggedMeta:
         for b in block_lists:
             bt.extend(list(b) + [0] * (width - len(b)))
         lens = [st + n for st, n in zip(starts, n_new)]
-        last = [c - 1 for c in cu[1:]]
-        flat = pos + sid + list(starts) + lens + cu + [x for w in work for x in w] + last + bt
+        last = [c - 1 for c in cu[1:]] if logit_rows is None else list(logit_rows)
+        slots = [] if slots is None else list(slots)
+        long = [i for i in range(S) if n_new[i] > RaggedMeta.STEP_TOKENS] if slots else []
+        short = [i for i in range(S) if n_new[i] <= RaggedMeta.STEP_TOKENS] if slots else []
+        chunks = [(i, c) for i in long for c in range(-(-n_new[i] // RaggedMeta.STATE_CHUNK))]
+        flat = pos + sid + list(starts) + lens + cu + [x for w in work for x in w] + last + bt + slots + short + long + \
+            [x for w in chunks for x in w]
         buf = torch.tensor(flat, dtype=torch.int32)
         if device is not None and torch.device(device).type == "cuda":
             buf = buf.pin_memory().to(device, non_blocking=True)
         views, o = [], 0
-        for n in (T, T, S, S, S + 1, 2 * len(work), S, S * width):
+        for n in (T, T, S, S, S + 1, 2 * len(work), len(last), S * width, len(slots), len(short), len(long),
+                  2 * len(chunks)):
             views.append(buf[o:o + n])
             o += n
-        pos_t, sid_t, st_t, len_t, cu_t, work_t, last_t, bt_t = views
+        pos_t, sid_t, st_t, len_t, cu_t, work_t, last_t, bt_t, slot_t, short_t, long_t, chunk_t = views
         return RaggedMeta(block_tables=bt_t.view(S, width), start_pos=st_t, seq_lens=len_t, pos_ids=pos_t,
                           seq_ids=sid_t, cu_q=cu_t, work=work_t.view(-1, 2), last_idx=last_t.long(),
                           n_decode=n_decode, cu_host=cu, start_host=list(starts), max_len=width * block_size,
-                          block_size=block_size)
+                          block_size=block_size, slots=slot_t, seq_list=short_t, chunk_seqs=long_t,
+                          chunk_work=chunk_t.view(-1, 2))
 
 
-class DSInferenceLayer(nn.Module):
+class ProjectionLayer(nn.Module):
+    """What decoder layers share: a set of named projection weights (row-major parameters, optionally group-quantised,
+    split, or doubled in the decode layout) and the tensor-parallel sum behind the row-parallel ones."""
 
-    def __init__(self, spec: DSModelSpec, layer_idx: int, tp_group=None, tp_size=1, dtype=torch.bfloat16,
-                 device=None):
+    def __init__(self, spec: DSModelSpec, layer_idx: int, tp_group=None, tp_size=1):
         super().__init__()
         self.spec = spec
         self.layer_idx = layer_idx
         self.tp_group = tp_group
         self.tp = tp_size
+        self.quant = {}
+        # bf16 weights ALSO held in the shuffled decode layout (name -> Bf16Weight), next to the row-major parameters:
+        # decode steps of SH_MIN_ROWS..16 token rows stream these, everything else uses the parameters
+        self.sh = {}
+        # split (aliased) projections: name -> list of weights / biases applied side by side (hybrid engine shares
+        # the training module's separate q/k/v and gate/up tensors instead of fusing copies)
+        self.split_w, self.split_b = {}, {}
+
+    def projection_names(self):
+        """The parameters that are quantised / re-laid together."""
+        raise NotImplementedError
+
+    def quantize_weights(self, bits=8, group_size=64):
+        self.sh = {}
+        for name in self.projection_names():
+            self.quant[name] = QuantLinearWeight(getattr(self, name).data, bits, group_size)
+            getattr(self, name).data = torch.empty(0, dtype=getattr(self, name).dtype,
+                                                   device=getattr(self, name).device)
+
+    SH_MIN_ROWS = 2  # measured on Llama-2-7B: the row-major stream wins at 1 token row, the shuffled one from 2 up
+
+    def add_decode_layout(self):
+        """Keep a second copy of the four projection weights in MFMA operand order (`ops/bf16_gemv.py`): twice the
+        weight memory — 288 GB of HBM is sized for it — for up to 1.2x on batched decode steps (2 - 16 token rows). No-op
+        for quantised, split or non-bf16 weights."""
+        from ...ops.bf16_gemv import Bf16Weight
+        if self.quant or self.split_w or self.spec.num_experts:
+            return False
+        ws = {n: getattr(self, n) for n in ("qkv_w", "o_w", "fc1_w", "fc2_w")}
+        if not all(w.is_cuda and Bf16Weight.supported(w.data) for w in ws.values()):
+            return False
+        self.sh = {n: Bf16Weight(w.data) for n, w in ws.items()}
+        return True
+
+    def _linear(self, x, name, bias=None):
+        """x . W^T (+ bias). Int8 weight-only layers run `Int8Weight.linear`: at decode sizes (<= 16 token rows) the
+        fused-dequant MFMA stream over the pre-shuffled weight (`csrc/gemv/skinny_int8.hip`, never materialises a
+        bf16 weight); larger batches dequantise into a bf16 temporary for a library GEMM (reference
+        `ds_vector_matmul_int8`)."""
+        if name in self.split_w:
+            bs = self.split_b.get(name) or [None] * len(self.split_w[name])
+            return torch.cat([F.linear(x, w, b) for w, b in zip(self.split_w[name], bs)], -1)
+        qw = self.quant.get(name)
+        if qw is not None and qw.i8 is not None:
+            return qw.i8.linear(x, bias)
+        return F.linear(x, self._w(name), bias)
+
+    def _w(self, name):
+        return self.quant[name].materialize() if name in self.quant else getattr(self, name)
+
+    def _allreduce(self, x):
+        if self.tp > 1:
+            dist.inference_all_reduce(x, group=self.tp_group)
+        return x
+
+
+class DSInferenceLayer(ProjectionLayer):
+
+    def __init__(self, spec: DSModelSpec, layer_idx: int, tp_group=None, tp_size=1, dtype=torch.bfloat16,
+                 device=None):
+        super().__init__(spec, layer_idx, tp_group, tp_size)
         assert spec.num_heads % tp_size == 0, "heads must divide tp size"
         self.hq = spec.num_heads // tp_size
         self.hk = max(spec.num_kv_heads // tp_size, 1)
@@ -245,62 +329,15 @@ class DSInferenceLayer(nn.Module):
             self.res_fc2_b = nn.Parameter(torch.zeros(H, **kw), requires_grad=False)
             self.coef_w = nn.Parameter(torch.empty(2, H, **kw), requires_grad=False)
             self.coef_b = nn.Parameter(torch.zeros(2, **kw), requires_grad=False)
-        self.quant = {}
-        # bf16 weights ALSO held in the shuffled decode layout (name -> Bf16Weight), next to the row-major parameters:
-        # decode steps of SH_MIN_ROWS..16 token rows stream these, everything else uses the parameters
-        self.sh = {}
-        # split (aliased) projections: name -> list of weights / biases applied side by side (hybrid engine shares
-        # the training module's separate q/k/v and gate/up tensors instead of fusing copies)
-        self.split_w, self.split_b = {}, {}
 
     # ------------------------------------------------------------------------------------------ helpers
-    def quantize_weights(self, bits=8, group_size=64):
-        self.sh = {}
-        for name in ("qkv_w", "o_w") + (() if self.spec.num_experts else ("fc1_w", "fc2_w")):
-            self.quant[name] = QuantLinearWeight(getattr(self, name).data, bits, group_size)
-            getattr(self, name).data = torch.empty(0, dtype=getattr(self, name).dtype,
-                                                   device=getattr(self, name).device)
-
-    SH_MIN_ROWS = 2  # measured on Llama-2-7B: the row-major stream wins at 1 token row, the shuffled one from 2 up
-
-    def add_decode_layout(self):
-        """Keep a second copy of the four projection weights in MFMA operand order (`ops/bf16_gemv.py`): twice the
-        weight memory — 288 GB of HBM is sized for it — for up to 1.2x on batched decode steps (2 - 16 token rows). No-op
-        for quantised, split or non-bf16 weights."""
-        from ...ops.bf16_gemv import Bf16Weight
-        if self.quant or self.split_w or self.spec.num_experts:
-            return False
-        ws = {n: getattr(self, n) for n in ("qkv_w", "o_w", "fc1_w", "fc2_w")}
-        if not all(w.is_cuda and Bf16Weight.supported(w.data) for w in ws.values()):
-            return False
-        self.sh = {n: Bf16Weight(w.data) for n, w in ws.items()}
-        return True
-
-    def _linear(self, x, name, bias=None):
-        """x . W^T (+ bias). Int8 weight-only layers run `Int8Weight.linear`: at decode sizes (<= 16 token rows) the
-        fused-dequant MFMA stream over the pre-shuffled weight (`csrc/gemv/skinny_int8.hip`, never materialises a
-        bf16 weight); larger batches dequantise into a bf16 temporary for a library GEMM (reference
-        `ds_vector_matmul_int8`)."""
-        if name in self.split_w:
-            bs = self.split_b.get(name) or [None] * len(self.split_w[name])
-            return torch.cat([F.linear(x, w, b) for w, b in zip(self.split_w[name], bs)], -1)
-        qw = self.quant.get(name)
-        if qw is not None and qw.i8 is not None:
-            return qw.i8.linear(x, bias)
-        return F.linear(x, self._w(name), bias)
-
-    def _w(self, name):
-        return self.quant[name].materialize() if name in self.quant else getattr(self, name)
+    def projection_names(self):
+        return ("qkv_w", "o_w") + (() if self.spec.num_experts else ("fc1_w", "fc2_w"))
 
     def _norm(self, x, w, b, residual=None):
         if self.spec.norm == "rms":
             return DF.rms_norm(x, w, self.spec.norm_eps, residual)
         return DF.layer_norm(x, w, b, self.spec.norm_eps, residual)
-
-    def _allreduce(self, x):
-        if self.tp > 1:
-            dist.inference_all_reduce(x, group=self.tp_group)
-        return x
 
     # ------------------------------------------------------------------------------------------ attention
     def _attend(self, qkv, meta: BatchMeta, cache, rope, alibi):
@@ -724,6 +761,7 @@ def _decode_attention(q, kc, vc, meta, scale, alibi, window):
 
 # ------------------------------------------------------------------------------------------------ model
 class DSInferenceModel(nn.Module):
+    layer_class = DSInferenceLayer
 
     def __init__(self, spec: DSModelSpec, tp_group=None, tp_size=1, tp_rank=0, dtype=torch.bfloat16, device=None):
         super().__init__()
@@ -739,10 +777,11 @@ class DSInferenceModel(nn.Module):
         if spec.embed_norm:
             self.embed_ln_w = nn.Parameter(torch.ones(H, **kw), requires_grad=False)
             self.embed_ln_b = nn.Parameter(torch.zeros(H, **kw), requires_grad=False)
-        self.layers = nn.ModuleList([DSInferenceLayer(spec, i, tp_group, tp_size, dtype, device)
+        self.layers = nn.ModuleList([self.layer_class(spec, i, tp_group, tp_size, dtype, device)
                                      for i in range(spec.num_layers)])
         self.norm_w = nn.Parameter(torch.ones(H, **kw), requires_grad=False)
-        self.norm_b = nn.Parameter(torch.zeros(H, **kw), requires_grad=False) if spec.norm == "ln" else None
+        self.norm_b = nn.Parameter(torch.zeros(H, **kw), requires_grad=False) \
+            if spec.norm == "ln" and spec.norm_bias else None
         vloc = (spec.vocab_size + tp_size - 1) // tp_size
         self.vocab_local = vloc
         self.lm_head = nn.Parameter(torch.empty(vloc, H, **kw), requires_grad=False)
@@ -764,11 +803,19 @@ class DSInferenceModel(nn.Module):
         self.cache = None
 
     # ------------------------------------------------------------------------------------------ cache
-    def allocate_cache(self, num_blocks, block_size=64):
-        from ..kv_cache import BlockedKVCache
+    def kv_geometry(self):
+        """Per layer (kv heads on this rank, key width, value width), or None for a layer without keys and values."""
         hk = max(self.spec.num_kv_heads // self.tp_size, 1)
-        self.cache = BlockedKVCache(self.spec.num_layers, num_blocks, hk, block_size, self.spec.head_dim, self.dtype,
-                                    self.device)
+        return [(hk, self.spec.head_dim, self.spec.head_dim)] * self.spec.num_layers
+
+    def state_geometry(self):
+        """Per layer {name: (shape, dtype)} of what one sequence carries from token to token, or None."""
+        return [None] * self.spec.num_layers
+
+    def allocate_cache(self, num_blocks, block_size=64, num_slots=0):
+        from ..kv_cache import BlockedKVCache
+        self.cache = BlockedKVCache.from_geometry(self.kv_geometry(), num_blocks, block_size, self.dtype, self.device,
+                                                  self.state_geometry(), num_slots)
         return self.cache
 
     # ------------------------------------------------------------------------------------------ forward
@@ -838,6 +885,8 @@ class DSInferenceModel(nn.Module):
         for layer in self.layers:
             h, residual = layer(h, residual, meta, self.cache, rope, self.alibi)
         h = materialize(h)
+        if meta.last_idx.numel() == 0:
+            return h.new_empty((0, self.spec.vocab_size))
         h = h[0].index_select(0, meta.last_idx)
         residual = residual[0].index_select(0, meta.last_idx) if residual is not None else None
         if (h.is_cuda and h.dtype == torch.bfloat16 and self.spec.final_norm and self.spec.norm == "rms"

@@ -7,6 +7,7 @@ shards are loaded with `torch.load(weights_only=True, mmap=True)`.
 """
 import json
 import os
+from types import SimpleNamespace
 
 import torch
 
@@ -21,6 +22,11 @@ class HuggingFaceCheckpointEngine(CheckpointEngineBase):
             raise FileNotFoundError(f"{model_name_or_path} is not a local checkpoint directory (checkpoints are "
                                     f"never downloaded)")
         self.model_name_or_path = model_name_or_path
+        self.model_config = self._own_config()
+        if self.model_config is not None:
+            self.generation_config = None
+            self._files = self._shards()
+            return
         from transformers import AutoConfig, GenerationConfig
         self.model_config = AutoConfig.from_pretrained(model_name_or_path, local_files_only=True)
         try:
@@ -28,6 +34,18 @@ class HuggingFaceCheckpointEngine(CheckpointEngineBase):
         except Exception:
             self.generation_config = None
         self._files = self._shards()
+
+    def _own_config(self):
+        """The config of a checkpoint whose config.json names an "architecture" of this package rather than a
+        transformers `model_type`: its JSON under attribute access, `model_type` being the lower-case name."""
+        path = os.path.join(self.model_name_or_path, "config.json")
+        if not os.path.exists(path):
+            return None
+        with open(path) as f:
+            raw = json.load(f)
+        if "model_type" in raw or not isinstance(raw.get("architecture"), str):
+            return None
+        return SimpleNamespace(model_type=raw["architecture"].lower(), **raw)
 
     def _shards(self):
         d = self.model_name_or_path

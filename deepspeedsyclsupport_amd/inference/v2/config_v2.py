@@ -28,6 +28,9 @@ class DSStateManagerConfig(DeepSpeedConfigModel):
     max_ragged_sequence_count: PositiveInt = 512
     max_context: PositiveInt = 8192
     memory_config: MemoryConfig = MemoryConfig()
+    # sequences whose carried state fits at once, for models with recurrent layers (0: `max_tracked_sequences`, or
+    # what a quarter of the free memory holds if that is less)
+    state_slots: int = 0
     offload: bool = False
 
     @model_validator(mode="after")

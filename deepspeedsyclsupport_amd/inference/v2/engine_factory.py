@@ -9,8 +9,8 @@ from .engine_v2 import InferenceEngineV2
 
 def build_hf_engine(path_or_model, engine_config: RaggedInferenceEngineConfig = None, debug_level=0,
                     dtype=torch.bfloat16, device=None):
-    """`path_or_model`: a local HF checkpoint directory (loaded with safetensors/transformers, no network) or an
-    already-instantiated HF / native model."""
+    """`path_or_model`: a local checkpoint directory (HF layout, or config.json + model.safetensors of one of this
+    package's own architectures; no network) or an already-instantiated HF / native model."""
     engine_config = engine_config or RaggedInferenceEngineConfig()
     if isinstance(path_or_model, str):
         import os
@@ -101,11 +101,13 @@ def build_engine_from_ds_checkpoint(path, engine_config: RaggedInferenceEngineCo
 
     from safetensors.torch import load_file
 
-    from ..model_implementations.transformer import DSInferenceModel, DSModelSpec
+    from ..model_implementations.hybrid import model_class
+    from ..model_implementations.transformer import DSModelSpec
     engine_config = engine_config or RaggedInferenceEngineConfig()
     with open(os.path.join(path, "ds_model_config.json")) as f:
         fields = json.load(f)
-    fields["layer_windows"] = tuple(fields.get("layer_windows", ()))
+    for name in ("layer_windows", "layer_specs"):
+        fields[name] = tuple(fields.get(name, ()))
     spec = DSModelSpec(**fields)
     meta_path = os.path.join(path, "ds_model_meta.json")
     meta = json.load(open(meta_path)) if os.path.exists(meta_path) else {"dtype": "bfloat16", "tp_size": 1}
@@ -124,7 +126,7 @@ def build_engine_from_ds_checkpoint(path, engine_config: RaggedInferenceEngineCo
             if s <= me < s + tp:
                 group = g
         rank = dist.get_rank(group)
-    model = DSInferenceModel(spec, group, tp, rank, to_dtype(meta["dtype"]), device)
+    model = model_class(spec)(spec, group, tp, rank, to_dtype(meta["dtype"]), device)
     sd = load_file(os.path.join(path, f"params_rank_{rank}.safetensors"), device=str(device))
     missing, unexpected = model.load_state_dict(sd, strict=False)
     if unexpected or any(not k.startswith(("rope_", "alibi")) for k in missing):

@@ -27,23 +27,37 @@ class InferenceEngineV2:
         self._model = model
         sm = self._config.state_manager
         bs = self._config.kv_cache.block_size
-        spec = model.spec
-        hk = max(spec.num_kv_heads // model.tp_size, 1)
+        from ..kv_cache import BlockedKVCache
+        slot_bytes = BlockedKVCache.slot_bytes(model.state_geometry())
+        num_slots = self._state_slots(sm, slot_bytes)
         if sm.memory_config.mode == AllocationMode.ALLOCATE:
             num_blocks = int(sm.memory_config.size)
         else:
-            from ..kv_cache import BlockedKVCache
             if model.device is not None and torch.device(model.device).type == "cuda":
                 free, _ = torch.cuda.mem_get_info(model.device)
-                avail = max(free - int(sm.memory_config.size), 0)
+                avail = max(free - int(sm.memory_config.size) - num_slots * slot_bytes, 0)
             else:
                 avail = 256 * 2**20  # host rehearsal: a small fixed pool
-            num_blocks = BlockedKVCache.blocks_for_memory(avail, spec.num_layers, hk, bs, spec.head_dim, model.dtype)
-        model.allocate_cache(num_blocks, bs)
-        self._state_manager = DSStateManager(sm, num_blocks, bs)
+            per_block = BlockedKVCache.block_bytes(model.kv_geometry(), bs, model.dtype)
+            # (a model without attention layers needs no blocks; keep the bookkeeping's pool non-trivial all the same)
+            num_blocks = max(avail // per_block, 1) if per_block else -(-sm.max_context // bs) * sm.max_tracked_sequences
+        model.allocate_cache(num_blocks, bs, num_slots)
+        self._state_manager = DSStateManager(sm, num_blocks, bs, num_slots)
         self._state_manager.attach_cache(getattr(model, "cache", None))
         self._device = model.device if model.device is not None else torch.device("cpu")
         self._batch = RaggedBatchWrapper(sm, bs, self._device)
+
+    def _state_slots(self, sm, slot_bytes):
+        """Slots for the state sequences carry through recurrent layers (0 for models without such layers)."""
+        if not slot_bytes:
+            return 0
+        if sm.state_slots:
+            return int(sm.state_slots)
+        if self._model.device is not None and torch.device(self._model.device).type == "cuda":
+            avail = torch.cuda.mem_get_info(self._model.device)[0] // 4
+        else:
+            avail = 256 * 2**20
+        return max(1, min(sm.max_tracked_sequences, avail // slot_bytes))
 
     # ------------------------------------------------------------------------------------------ properties
     @property
@@ -60,7 +74,10 @@ class InferenceEngineV2:
 
     # ------------------------------------------------------------------------------------------ forward
     @torch.no_grad()
-    def put(self, batch_uids: Iterable[int], batch_tokens: Iterable[torch.Tensor], do_checks=True) -> torch.Tensor:
+    def put(self, batch_uids: Iterable[int], batch_tokens: Iterable[torch.Tensor], do_checks=True,
+            logit_positions=None) -> torch.Tensor:
+        """One step. Returns one row of logits per sequence (its last new token), in the order given; with
+        `logit_positions` (per sequence, places among its new tokens) the rows of those places, in that order."""
         uids = list(batch_uids)
         toks = [t.reshape(-1) for t in batch_tokens]
         if do_checks:
@@ -76,9 +93,9 @@ class InferenceEngineV2:
             seq.pre_forward(t.numel())
             batch.insert_sequence(seq, t, do_checks=False)
             seqs.append(seq)
-        batch.finalize()
+        batch.finalize(logit_positions=logit_positions)
         logits = self._model.forward_ragged(batch.input_ids(), batch.meta)
-        out = batch.restore_order(logits)
+        out = batch.restore_order(logits) if logit_positions is None else logits
         for s in seqs:
             s.post_forward()
         return out
@@ -96,7 +113,8 @@ class InferenceEngineV2:
     def query(self, uid: int, max_request_tokens: int, max_request_blocks) -> Tuple[int, int]:
         seq = self._state_manager.get_sequence(uid)
         if seq is None:
-            if self._state_manager.n_tracked_sequences >= self._config.state_manager.max_tracked_sequences:
+            if self._state_manager.n_tracked_sequences >= self._config.state_manager.max_tracked_sequences \
+                    or self._state_manager.free_slots == 0:
                 return (0, 0)
             seq = PlaceholderSequenceDescriptor(self._state_manager.block_size)
         return self._kv_requirements(seq, max_request_tokens, int(max_request_blocks))
@@ -107,11 +125,15 @@ class InferenceEngineV2:
         if len(uids) > sm.max_ragged_sequence_count:
             return SchedulingResult.BatchSequenceLimitExceeded
         cur, free = self._state_manager.n_tracked_sequences, self._state_manager.free_blocks
-        total = 0
+        total, slots = 0, self._state_manager.free_slots
         for uid, n in zip(uids, lengths):
             seq = self._state_manager.get_sequence(uid)
             if seq is None:
                 cur += 1
+                if slots is not None:
+                    slots -= 1
+                    if slots < 0:
+                        return SchedulingResult.EngineSequenceLimitExceeded
                 seq = PlaceholderSequenceDescriptor(self._state_manager.block_size)
             if seq.seen_tokens + n > sm.max_context:
                 return SchedulingResult.SequenceTokenLimitExceeded

@@ -1,0 +1,70 @@
+"""Containers and policies of the hybrid decoders (`inference/model_implementations/hybrid.py`): checkpoints that are
+config.json + model.safetensors in this package's own layout, with the layers listed one by one in the config.
+
+A layer's container is assembled from the tensors its kind has: the mixer's, the feed-forward's if it has one, the
+norms and, for models with residual streams, the mixing matrices."""
+from ...model_implementations.hybrid import DSHybridModel
+from ...model_implementations.transformer import DSModelSpec
+from .inference_policy_base import ContainerMap, InferenceV2Policy, register
+from .layer_container_base import LayerContainer
+from .parameter_base import single
+
+_MIXER_TENSORS = {  # checkpoint name below `<layer>.mix.` -> canonical key
+    "attention": {"q": "q_w", "k": "k_w", "v": "v_w", "o": "o_w", "q.norm": "q_norm", "k.norm": "k_norm"},
+    "delta": {"q": "q_w", "k": "k_w", "v": "v_w", "g": "g_w", "b": "b_w", "a": "a_w", "o": "o_w", "q.conv": "q_conv",
+              "k.conv": "k_conv", "v.conv": "v_conv", "A_log": "a_log", "dt_bias": "dt_bias", "norm": "head_norm"},
+}
+_MLP_TENSORS = {"dense": {"gate": "gate_w", "up": "up_w", "down": "down_w"}}
+
+
+def container(name, tensors):
+    """A container class for {checkpoint tensor: canonical key}."""
+    return type(name, (LayerContainer, ), {"__annotations__": {key: single(key) for key in tensors.values()},
+                                           "PARAM_MAPPING": {src: f"{key}.params" for src, key in tensors.items()}})
+
+
+def layer_container(layer, streams):
+    """Container class of one entry of the config's layer list."""
+    if layer["type"] not in _MIXER_TENSORS:
+        raise NotImplementedError(f"no mixer {layer['type']!r}")
+    tensors = {f"mix.{n}": key for n, key in _MIXER_TENSORS[layer["type"]].items()}
+    if layer["mixer"].get("v_mix"):
+        tensors["mix.vmix"] = "vmix"
+    if layer.get("mlp"):
+        if layer["mlp"].get("kind") not in _MLP_TENSORS:
+            raise NotImplementedError(f"no feed-forward {layer['mlp'].get('kind')!r}")
+        tensors.update({f"mlp.{n}": key for n, key in _MLP_TENSORS[layer["mlp"]["kind"]].items()})
+    for q in (1, 2) if layer.get("mlp") else (1, ):
+        tensors[f"norm{q}"] = f"norm{q}_w"
+        if streams:
+            tensors.update({f"hc{q}.{n}": f"hc{q}_{n}" for n in ("in", "out", "mix")})
+    return container("HybridLayerContainer", tensors)
+
+
+TopContainer = container("HybridTopContainer", {"embed": "embed", "final.norm": "norm_w", "head": "lm_head"})
+
+
+@register
+class VopepelPolicy(InferenceV2Policy):
+    """Vopepel: gated-delta-rule and chunked softmax-attention layers over several residual streams."""
+    model_types = ("vopepel", )
+    model_class = DSHybridModel
+
+    def spec(self):
+        c = self._model_config
+        attn = [la["mixer"] for la in c.layers if la["type"] == "attention"]
+        first = (attn or [la["mixer"] for la in c.layers])[0]
+        return DSModelSpec(arch="vopepel", vocab_size=c.vocab, hidden_size=c.width, num_layers=len(c.layers),
+                           num_heads=first["heads"], num_kv_heads=first["kv_heads"], head_dim=first["dim"],
+                           intermediate_size=max([la["mlp"]["ff"] for la in c.layers if la.get("mlp")], default=0),
+                           norm="ln", norm_bias=False, norm_eps=float(c.norm["eps"]), pos="none",
+                           layer_specs=tuple(c.layers), streams=int(getattr(c, "streams", None) or 1),
+                           residual_mult=float(getattr(c, "residual_mult", 1.0)))
+
+    def build_container_map(self):
+        c = self._model_config
+        cmap = ContainerMap()
+        streams = bool(getattr(c, "streams", None))
+        cmap.set_transformer_params("l", [layer_container(la, streams)(self._view) for la in c.layers], sep="")
+        cmap.set_non_transformer_params(TopContainer(self._view))
+        return cmap

@@ -37,12 +37,13 @@ class ContainerMap:
     def non_transformer_params(self) -> LayerContainer:
         return self._non_transformer_params
 
-    def set_transformer_params(self, prefixes: Union[str, Iterable[str]], containers: List[LayerContainer]) -> None:
-        """`prefixes`: checkpoint prefix(es) of the layer list ("model.layers"): names `<prefix>.<i>.<rest>` go to
+    def set_transformer_params(self, prefixes: Union[str, Iterable[str]], containers: List[LayerContainer],
+                               sep=".") -> None:
+        """`prefixes`: checkpoint prefix(es) of the layer list ("model.layers"): names `<prefix><sep><i>.<rest>` go to
         containers[i] as `<rest>`."""
         prefixes = [prefixes] if isinstance(prefixes, str) else list(prefixes)
         self._transformer_params = containers
-        self._layer_rx = [re.compile("^" + re.escape(p) + r"\.(\d+)\.(.*)$") for p in prefixes]
+        self._layer_rx = [re.compile("^" + re.escape(p) + re.escape(sep) + r"(\d+)\.(.*)$") for p in prefixes]
 
     def set_non_transformer_params(self, container: LayerContainer) -> None:
         self._non_transformer_params = container
@@ -93,6 +94,7 @@ class _ModelView:
 class InferenceV2Policy(ABC):
     #: `model_type` values of HF configs this policy serves (registered into POLICIES by `register`)
     model_types = ()
+    model_class = DSInferenceModel
 
     def __init__(self, model_config, checkpoint_engine: Optional[CheckpointEngineBase] = None,
                  inf_checkpoint_path: Optional[str] = None) -> None:
@@ -119,7 +121,7 @@ class InferenceV2Policy(ABC):
         spec = self.spec()
         spec.max_positions = max(spec.max_positions, engine_config.state_manager.max_context)
         dtype = to_dtype(getattr(self, "dtype", None) or torch.bfloat16)
-        return DSInferenceModel(spec, mp_group, tp, rank, dtype, device)
+        return self.model_class(spec, mp_group, tp, rank, dtype, device)
 
     @abstractmethod
     def build_container_map(self) -> ContainerMap:

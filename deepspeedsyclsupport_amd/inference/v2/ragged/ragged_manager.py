@@ -7,10 +7,12 @@ from .sequence_descriptor import DSSequenceDescriptor
 
 class DSStateManager:
 
-    def __init__(self, config, num_blocks, block_size):
+    def __init__(self, config, num_blocks, block_size, num_slots=0):
+        """`num_slots`: state slots for models whose layers carry a state per sequence (0: the model has none)."""
         self.config = config
         self.block_size = block_size
         self.allocator = BlockedAllocator(num_blocks)
+        self.slot_allocator = BlockedAllocator(num_slots) if num_slots else None
         self._seqs = {}
         self._kv_cache = None
 
@@ -25,6 +27,11 @@ class DSStateManager:
     @property
     def free_blocks(self):
         return self.allocator.free_blocks
+
+    @property
+    def free_slots(self):
+        """State slots left for new sequences (None: the model keeps no such state)."""
+        return self.slot_allocator.free_blocks if self.slot_allocator is not None else None
 
     @property
     def kv_block_size(self):
@@ -57,7 +64,12 @@ class DSStateManager:
         if seq is None:
             if len(self._seqs) >= self.config.max_tracked_sequences:
                 raise RuntimeError("engine is tracking max_tracked_sequences sequences")
-            seq = self._seqs[uid] = DSSequenceDescriptor(uid, self.block_size)
+            slot = None
+            if self.slot_allocator is not None:
+                if not self.slot_allocator.free_blocks:
+                    raise RuntimeError("no free state slot for another sequence")
+                slot = self.slot_allocator.allocate(1)[0]
+            seq = self._seqs[uid] = DSSequenceDescriptor(uid, self.block_size, slot)
         return seq
 
     def allocate_blocks(self, seq, n_tokens):
@@ -70,6 +82,9 @@ class DSStateManager:
         if seq is not None:
             self.allocator.free(seq.blocks)
             seq.blocks = []
+            if seq.slot is not None:
+                self.slot_allocator.free([seq.slot])
+                seq.slot = None
 
     def block_table(self, seqs, device):
         width = max(len(s.blocks) for s in seqs)

@@ -58,9 +58,10 @@ class RaggedBatchWrapper:
         self._toks.append(tokens)
         self._n_tokens += tokens.numel()
 
-    def finalize(self, padding=False) -> None:
+    def finalize(self, padding=False, logit_positions=None) -> None:
         """Build and upload the index tables. `padding` is accepted for signature parity: the in-tree kernels take
-        exact counts, nothing is padded."""
+        exact counts, nothing is padded. `logit_positions`: per inserted sequence, the places among its new tokens
+        whose logits are wanted (default: the last one of each)."""
         if not self._seqs:
             raise RuntimeError("cannot finalize an empty ragged batch")
         n = [t.numel() for t in self._toks]
@@ -68,8 +69,16 @@ class RaggedBatchWrapper:
         self.order = sorted(range(len(n)), key=lambda i: 0 if is_decode[i] else 1)
         seqs = [self._seqs[i] for i in self.order]
         bs = self._block_size or seqs[0].block_size
+        rows = None
+        if logit_positions is not None:
+            first, at = {}, 0
+            for i in self.order:
+                first[i] = at
+                at += n[i]
+            rows = [first[i] + int(p) for i, want in enumerate(logit_positions) for p in want]
+        slots = [s.slot for s in seqs] if seqs[0].slot is not None else None
         self.meta = RaggedMeta.build([s.seen_tokens for s in seqs], [n[i] for i in self.order],
-                                     [s.blocks for s in seqs], sum(is_decode), bs, self._device)
+                                     [s.blocks for s in seqs], sum(is_decode), bs, self._device, slots, rows)
         ids = torch.cat([self._toks[i] for i in self.order])
         if self._device is not None:
             ids = ids.to(self._device, non_blocking=True)

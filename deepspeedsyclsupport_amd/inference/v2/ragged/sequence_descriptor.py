@@ -18,8 +18,9 @@ class BaseSequenceDescriptor:
 
 class DSSequenceDescriptor(BaseSequenceDescriptor):
 
-    def __init__(self, uid, block_size):
+    def __init__(self, uid, block_size, slot=None):
         self.uid = uid
+        self.slot = slot   # state slot, for models whose layers carry a state per sequence
         self._seen_tokens = 0
         self.in_flight_tokens = 0
         self.blocks = []

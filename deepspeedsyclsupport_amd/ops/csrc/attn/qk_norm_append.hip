@@ -1,0 +1,77 @@
+// QKV epilogue of attention layers with per-head query / key RMSNorm, CDNA4 (gfx950).
+//
+// One wave per (token, head): q and k heads are divided by their root mean square and scaled by a shared weight, v
+// heads are optionally mixed with the values of an earlier layer (v <- (1 - lambda) v + lambda v_first); q is written
+// out, k and v go straight into the paged cache, whose key and value rows may differ in width. No rotation.
+#include "ds_hip.h"
+
+namespace {
+
+template <typename T>
+__global__ void __launch_bounds__(256) qk_norm_append_kernel(
+    const T* __restrict__ qkv, const float* __restrict__ qw, const float* __restrict__ kw, float eps,
+    const T* __restrict__ vfirst, int64_t vf_stride, const float* __restrict__ lambda, const int* __restrict__ pos,
+    const int* __restrict__ seq_ids, const int* __restrict__ block_table, int max_blocks, T* __restrict__ q_out,
+    T* __restrict__ kc, T* __restrict__ vc, int tokens, int H, int G, int dk, int dv, int BS) {
+  const int slots = H + 2 * G, lane = threadIdx.x & 63;
+  const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= (int64_t)tokens * slots) return;
+  const int t = (int)(item / slots), h = (int)(item % slots);
+  const T* row = qkv + (int64_t)t * ((int64_t)(H + G) * dk + (int64_t)G * dv);
+  int64_t slot = 0;
+  if (h >= H) {
+    const int p = pos[t];
+    const int g = h < H + G ? h - H : h - H - G;
+    slot = ((int64_t)block_table[(int64_t)seq_ids[t] * max_blocks + p / BS] * G + g) * BS + p % BS;
+  }
+  if (h >= H + G) {
+    const int g = h - H - G;
+    const T* v = row + (int64_t)(H + G) * dk + (int64_t)g * dv;
+    const float lam = vfirst ? lambda[0] : 0.f;
+    for (int c = lane; c < dv; c += 64) {
+      float a = (float)v[c];
+      if (vfirst) a = (1.f - lam) * a + lam * (float)vfirst[(int64_t)t * vf_stride + (int64_t)g * dv + c];
+      vc[slot * dv + c] = (T)a;
+    }
+    return;
+  }
+  const T* src = row + (int64_t)h * dk;
+  float ss = 0.f;
+  for (int c = lane; c < dk; c += 64) {
+    const float a = (float)src[c];
+    ss = fmaf(a, a, ss);
+  }
+  const float rs = 1.f / sqrtf(wave_sum(ss) / (float)dk + eps);
+  T* dst = h < H ? q_out + ((int64_t)t * H + h) * dk : kc + slot * dk;
+  const float* w = h < H ? qw : kw;
+  for (int c = lane; c < dk; c += 64) dst[c] = (T)((float)src[c] * rs * w[c]);
+}
+
+template <typename T>
+int launch(const void* qkv, const float* qw, const float* kw, float eps, const void* vfirst, int64_t vf_stride,
+           const float* lambda, const int* pos, const int* seq_ids, const int* bt, int max_blocks, void* q, void* kc,
+           void* vc, int tokens, int H, int G, int dk, int dv, int BS, hipStream_t st) {
+  const int64_t items = (int64_t)tokens * (H + 2 * G);
+  hipLaunchKernelGGL((qk_norm_append_kernel<T>), dim3((unsigned)((items + 3) / 4)), dim3(256), 0, st, (const T*)qkv, qw,
+                     kw, eps, (const T*)vfirst, vf_stride, lambda, pos, seq_ids, bt, max_blocks, (T*)q, (T*)kc, (T*)vc,
+                     tokens, H, G, dk, dv, BS);
+  DS_CHECK_LAUNCH();
+  return 0;
+}
+
+}  // namespace
+
+extern "C" int ds_qk_norm_append(const void* qkv, const float* qw, const float* kw, float eps, const void* vfirst,
+                                 int64_t vf_stride, const float* lambda, const int* pos, const int* seq_ids,
+                                 const int* bt, int max_blocks, void* q, void* kc, void* vc, int tokens, int H, int G,
+                                 int dk, int dv, int BS, int dtype, hipStream_t st) {
+  if (tokens <= 0) return 0;
+  if (H <= 0 || G <= 0 || H % G || dk <= 0 || dv <= 0 || BS <= 0 || max_blocks <= 0 || (vfirst && !lambda))
+    return (int)hipErrorInvalidValue;
+#define GO(T) \
+  launch<T>(qkv, qw, kw, eps, vfirst, vf_stride, lambda, pos, seq_ids, bt, max_blocks, q, kc, vc, tokens, H, G, dk, dv, BS, st)
+  if (dtype == DS_F32) return GO(float);
+  if (dtype == DS_BF16) return GO(bf16);
+#undef GO
+  return (int)hipErrorInvalidValue;
+}

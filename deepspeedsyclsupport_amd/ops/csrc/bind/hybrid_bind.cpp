@@ -1,0 +1,236 @@
+// Module of the hybrid decoder's ops: multi-stream residual + norm, QKV epilogue with per-head norms, ragged paged
+// attention with chunked / windowed visibility and score capping, gated delta rule, clamped gated activation, and the
+// bf16 decode products they are used with. A shared object of its own, so that serving such a model compiles only this.
+#include <torch/extension.h>
+#include <ATen/hip/HIPContext.h>
+#include <hip/hip_runtime_api.h>
+
+#include <optional>
+
+extern "C" {
+int ds_stream_norm(float*, const void*, const int*, const void*, const int*, int, int, const float*, const float*, float,
+                   const float*, const float*, void*, int, float, int, hipStream_t);
+int ds_clamped_glu(const void*, void*, int64_t, int, float, float, float, int, hipStream_t);
+int ds_qk_norm_append(const void*, const float*, const float*, float, const void*, int64_t, const float*, const int*,
+                      const int*, const int*, int, void*, void*, void*, int, int, int, int, int, int, int, hipStream_t);
+int ds_paged_generic(const void*, const void*, const void*, void*, const int*, int, const int*, const int*, int, int, int,
+                     int, int, int, float, float, int, int, int, hipStream_t);
+int ds_delta_prepare(const void*, const float*, const void*, const float*, const float*, const int*, const int*,
+                     const int*, const int*, float*, void*, float*, int, int, int, int, int, int, int, hipStream_t);
+int ds_delta_recur(const float*, const void*, const float*, const void*, const float*, float, float*, void*, const int*,
+                   int, const int*, const int*, const int*, void*, int, int, int, int, int, int, hipStream_t);
+int ds_skinny_gemm(const void*, const void*, const void*, const void*, const void*, const void*, void*, void*, int, int,
+                   int, int, int, int, float, hipStream_t);
+int ds_skinny_mfma_ok(int, int, int);
+int ds_skinny_mfma(const void*, const void*, const void*, const void*, const void*, const void*, void*, void*, int, int,
+                   int, int, int, int, float, hipStream_t);
+}
+
+using torch::Tensor;
+using OptT = std::optional<Tensor>;
+
+namespace {
+hipStream_t stream() { return at::hip::getCurrentHIPStream().stream(); }
+void check(int rc, const char* what) { TORCH_CHECK(rc == 0, what, " failed: ", hipGetErrorString((hipError_t)rc)); }
+int dcode(const Tensor& t) {
+  if (t.scalar_type() == at::kFloat) return 0;
+  TORCH_CHECK(t.scalar_type() == at::kBFloat16, "fp32 or bf16 tensors");
+  return 1;
+}
+void need(const Tensor& t, const char* n) {
+  TORCH_CHECK(t.is_cuda() && t.is_contiguous(), n, " must be a contiguous device tensor");
+}
+const float* f32(const Tensor& t, int64_t n, const char* name) {
+  need(t, name);
+  TORCH_CHECK(t.scalar_type() == at::kFloat && t.numel() == n, name, ": fp32 with ", n, " elements");
+  return t.data_ptr<float>();
+}
+const int* i32(const Tensor& t, int64_t n, const char* name) {
+  need(t, name);
+  TORCH_CHECK(t.scalar_type() == at::kInt && t.numel() == n, name, ": int32 with ", n, " elements");
+  return t.data_ptr<int>();
+}
+bool has(const OptT& t) { return t.has_value() && t->defined(); }
+
+// x [T, S, W] fp32 (updated in place unless `rows`). Either y [T, W] with mix [S, S] / out [S] (finish a sublayer), or
+// ids [T] + embed [V, W] (start of the model). Returns the normed rows [R, W] in y's / embed's type.
+Tensor stream_norm(Tensor x, OptT y, OptT mix, OptT out, double m, OptT in, Tensor w, double eps, OptT ids, OptT embed,
+                   OptT rows) {
+  need(x, "x");
+  TORCH_CHECK(x.scalar_type() == at::kFloat && x.dim() == 3, "stream_norm: x [T, S, W] fp32");
+  const int64_t T = x.size(0), S = x.size(1), W = x.size(2);
+  TORCH_CHECK(S >= 1 && S <= 8, "stream_norm: 1 to 8 streams");
+  TORCH_CHECK(W <= 15360, "stream_norm: width up to 15360");
+  TORCH_CHECK(has(y) != has(embed), "stream_norm: y or embed");
+  const Tensor& src = has(y) ? *y : *embed;
+  need(src, "y / embed");
+  TORCH_CHECK(src.size(-1) == W, "stream_norm: width");
+  const float *mp = nullptr, *op = nullptr;
+  const int *ip = nullptr, *rp = nullptr;
+  if (has(y)) {
+    TORCH_CHECK(y->numel() == T * W, "stream_norm: y [T, W]");
+    mp = f32(*mix, S * S, "mix");
+    op = f32(*out, S, "out");
+  } else {
+    ip = i32(*ids, T, "ids");
+    TORCH_CHECK(!has(rows), "stream_norm: no row list at the start");
+  }
+  int64_t R = T;
+  if (has(rows)) {
+    R = rows->numel();
+    rp = i32(*rows, R, "rows");
+  }
+  auto normed = torch::empty({R, W}, src.options());
+  check(ds_stream_norm(x.data_ptr<float>(), has(y) ? y->data_ptr() : nullptr, ip, has(embed) ? embed->data_ptr() : nullptr,
+                       rp, (int)R, (int)S, mp, op, (float)m, has(in) ? f32(*in, S, "in") : nullptr,
+                       f32(w, W, "norm weight"), normed.data_ptr(), (int)W, (float)eps, dcode(src), stream()),
+        "stream_norm");
+  return normed;
+}
+
+Tensor clamped_glu(Tensor gu, double limit, double alpha, double shift) {
+  need(gu, "gate_up");
+  const int64_t F = gu.size(-1) / 2, rows = gu.numel() / gu.size(-1);
+  TORCH_CHECK(gu.size(-1) % 2 == 0, "clamped_glu: [.., 2F]");
+  auto sizes = gu.sizes().vec();
+  sizes.back() = F;
+  auto out = torch::empty(sizes, gu.options());
+  check(ds_clamped_glu(gu.data_ptr(), out.data_ptr(), rows, (int)F, (float)limit, (float)alpha, (float)shift, dcode(gu),
+                       stream()), "clamped_glu");
+  return out;
+}
+
+struct Cache {
+  int G, BS, dk, dv;
+};
+Cache cache_of(const Tensor& kc, const Tensor& vc) {
+  need(kc, "k cache"); need(vc, "v cache");
+  TORCH_CHECK(kc.dim() == 4 && vc.dim() == 4 && kc.size(0) == vc.size(0) && kc.size(1) == vc.size(1) &&
+              kc.size(2) == vc.size(2) && kc.scalar_type() == vc.scalar_type(), "caches [NB, G, BS, dk / dv]");
+  return {(int)kc.size(1), (int)kc.size(2), (int)kc.size(3), (int)vc.size(3)};
+}
+
+// qkv [T, (H + G) dk + G dv] -> q [T, H, dk]; k / v into the caches. vfirst: the same-shaped v columns [T, G dv] (row
+// stride free) of an earlier layer, mixed in with weight `lam` [1].
+Tensor qk_norm_append(Tensor qkv, Tensor qw, Tensor kw, double eps, OptT vfirst, OptT lam, Tensor pos, Tensor seq_ids,
+                      Tensor block_table, Tensor kc, Tensor vc, int64_t H) {
+  need(qkv, "qkv"); need(block_table, "block_table");
+  const Cache c = cache_of(kc, vc);
+  const int64_t N = (H + c.G) * c.dk + (int64_t)c.G * c.dv, T = qkv.numel() / N;
+  TORCH_CHECK(qkv.numel() == T * N && qkv.size(-1) == N, "qk_norm_append: qkv width");
+  TORCH_CHECK(qkv.scalar_type() == kc.scalar_type(), "qk_norm_append: projection and cache types differ");
+  TORCH_CHECK(block_table.dim() == 2 && block_table.scalar_type() == at::kInt, "block_table [S, M] int32");
+  const void* vf = nullptr;
+  int64_t vs = 0;
+  const float* lp = nullptr;
+  if (has(vfirst)) {
+    TORCH_CHECK(vfirst->is_cuda() && vfirst->dim() == 2 && vfirst->size(0) == T && vfirst->size(1) == (int64_t)c.G * c.dv &&
+                vfirst->stride(1) == 1 && vfirst->scalar_type() == qkv.scalar_type(), "vfirst [T, G dv]");
+    vf = vfirst->data_ptr();
+    vs = vfirst->stride(0);
+    lp = f32(*lam, 1, "lambda");
+  }
+  auto q = torch::empty({T, H, c.dk}, qkv.options());
+  check(ds_qk_norm_append(qkv.data_ptr(), f32(qw, c.dk, "q norm"), f32(kw, c.dk, "k norm"), (float)eps, vf, vs, lp,
+                          i32(pos, T, "pos"), i32(seq_ids, T, "seq_ids"), block_table.data_ptr<int>(),
+                          (int)block_table.size(1), q.data_ptr(), kc.data_ptr(), vc.data_ptr(), (int)T, (int)H, c.G, c.dk,
+                          c.dv, c.BS, dcode(qkv), stream()), "qk_norm_append");
+  return q;
+}
+
+// q [T, H, dk] at positions pos of sequences seq_ids -> o [T, H, dv]
+Tensor paged_generic(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor pos, Tensor seq_ids, double scale,
+                     double softcap, int64_t window, int64_t chunk) {
+  need(q, "q"); need(block_table, "block_table");
+  const Cache c = cache_of(kc, vc);
+  const int64_t T = q.size(0), H = q.size(1);
+  TORCH_CHECK(q.dim() == 3 && q.size(2) == c.dk && H % c.G == 0 && q.scalar_type() == kc.scalar_type(), "paged_generic: q");
+  TORCH_CHECK(block_table.dim() == 2 && block_table.scalar_type() == at::kInt, "block_table [S, M] int32");
+  TORCH_CHECK(c.dk <= 512 && c.dv <= 512, "paged_generic: head sizes up to 512");
+  auto o = torch::empty({T, H, c.dv}, q.options());
+  check(ds_paged_generic(q.data_ptr(), kc.data_ptr(), vc.data_ptr(), o.data_ptr(), block_table.data_ptr<int>(),
+                         (int)block_table.size(1), i32(pos, T, "pos"), i32(seq_ids, T, "seq_ids"), (int)T, (int)H, c.G,
+                         c.dk, c.dv, c.BS, (float)scale, (float)softcap, (int)window, (int)chunk, dcode(q), stream()),
+        "paged_generic");
+  return o;
+}
+
+void delta_dims_ok(int64_t Hk, int64_t H, int64_t dk, int64_t dv, int64_t taps) {
+  TORCH_CHECK(Hk > 0 && H % Hk == 0 && dk > 0 && dv > 0 && taps >= 1, "delta rule: head counts / sizes");
+  TORCH_CHECK(dk <= 256 && dv <= 256, "delta rule: head sizes up to 256");
+}
+
+// proj [T, 2 Hk dk + 2 H dv + 2 H] -> (qk fp32 [T, 2, Hk, dk], v [T, H, dv], gb fp32 [T, 2, H]: log decay, beta)
+std::vector<Tensor> delta_prepare(Tensor proj, Tensor conv_w, Tensor conv_state, Tensor a_log, Tensor dt_bias,
+                                  Tensor seq_ids, Tensor cu, Tensor start, Tensor slots, int64_t Hk, int64_t H, int64_t dk,
+                                  int64_t dv) {
+  need(proj, "proj"); need(conv_state, "conv_state");
+  const int64_t C = 2 * Hk * dk + H * dv, NP = C + H * dv + 2 * H, T = proj.numel() / NP, taps = conv_w.size(-1);
+  delta_dims_ok(Hk, H, dk, dv, taps);
+  TORCH_CHECK(proj.size(-1) == NP, "delta_prepare: projection width");
+  TORCH_CHECK(conv_state.dim() == 3 && conv_state.size(1) == taps - 1 && conv_state.size(2) == C &&
+              conv_state.scalar_type() == proj.scalar_type(), "delta_prepare: conv_state [slots, taps-1, C]");
+  const int64_t S = start.numel();
+  auto fo = proj.options().dtype(at::kFloat);
+  auto qk = torch::empty({T, 2, Hk, dk}, fo);
+  auto v = torch::empty({T, H, dv}, proj.options());
+  auto gb = torch::empty({T, 2, H}, fo);
+  check(ds_delta_prepare(proj.data_ptr(), f32(conv_w, C * taps, "conv_w"), conv_state.data_ptr(), f32(a_log, H, "A_log"),
+                         f32(dt_bias, H, "dt_bias"), i32(seq_ids, T, "seq_ids"), i32(cu, S + 1, "cu"),
+                         i32(start, S, "start"), i32(slots, S, "slots"), qk.data_ptr<float>(), v.data_ptr(),
+                         gb.data_ptr<float>(), (int)T, (int)Hk, (int)H, (int)dk, (int)dv, (int)taps, dcode(proj), stream()),
+        "delta_prepare");
+  return {qk, v, gb};
+}
+
+// Runs the sequences in `list`; writes their rows of out [T, H dv] and their state slots.
+void delta_recur(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, double eps, Tensor state, Tensor conv_state,
+                 Tensor list, Tensor cu, Tensor start, Tensor slots, Tensor out) {
+  need(proj, "proj"); need(v, "v"); need(state, "state"); need(conv_state, "conv_state"); need(out, "out");
+  const int64_t T = v.size(0), H = v.size(1), dv = v.size(2), Hk = qk.size(2), dk = qk.size(3), S = start.numel();
+  const int64_t taps = conv_state.size(1) + 1;
+  delta_dims_ok(Hk, H, dk, dv, taps);
+  TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == H && state.size(2) == dk &&
+              state.size(3) == dv && state.size(0) == conv_state.size(0), "delta: state [slots, H, dk, dv] fp32");
+  TORCH_CHECK(conv_state.size(2) == 2 * Hk * dk + H * dv, "delta: conv_state");
+  TORCH_CHECK(proj.numel() == T * (2 * Hk * dk + 2 * H * dv + 2 * H) && out.numel() == T * H * dv, "delta: proj / out");
+  TORCH_CHECK(v.scalar_type() == proj.scalar_type() && out.scalar_type() == proj.scalar_type() &&
+              conv_state.scalar_type() == proj.scalar_type(), "delta: types");
+  check(ds_delta_recur(f32(qk, T * 2 * Hk * dk, "qk"), v.data_ptr(), f32(gb, T * 2 * H, "gb"), proj.data_ptr(),
+                       f32(norm_w, dv, "norm"), (float)eps, state.data_ptr<float>(), conv_state.data_ptr(),
+                       i32(list, list.numel(), "list"), (int)list.numel(), i32(cu, S + 1, "cu"), i32(start, S, "start"),
+                       i32(slots, S, "slots"), out.data_ptr(), (int)Hk, (int)H, (int)dk, (int)dv, (int)taps, dcode(proj),
+                       stream()), "delta_recur");
+}
+
+bool decode_linear_ok(int64_t M, int64_t K) {
+  return M >= 1 && K % 8 == 0 && (M <= 8 || (M <= 16 && ds_skinny_mfma_ok((int)M, (int)K, 0)));
+}
+// x [M, K] . w [N, K]^T for M <= 16 bf16 rows: the vector kernel up to two rows (or where K does not tile), else MFMA
+Tensor decode_linear(Tensor x, Tensor w) {
+  need(x, "x"); need(w, "w");
+  const int64_t N = w.size(0), K = w.size(1), M = x.numel() / K;
+  TORCH_CHECK(x.scalar_type() == at::kBFloat16 && w.scalar_type() == at::kBFloat16 && x.size(-1) == K, "decode_linear");
+  TORCH_CHECK(decode_linear_ok(M, K), "decode_linear: up to 8 rows with K % 8 == 0 (16 with K % 256 == 0)");
+  auto sizes = x.sizes().vec();
+  sizes.back() = N;
+  auto y = torch::empty(sizes, x.options());
+  auto fn = M > 2 && ds_skinny_mfma_ok((int)M, (int)K, 0) ? ds_skinny_mfma : ds_skinny_gemm;
+  check(fn(w.data_ptr(), x.data_ptr(), nullptr, nullptr, nullptr, nullptr, y.data_ptr(), nullptr, (int)M, (int)N, (int)K,
+           0, 0, 0, 0.f, stream()), "decode_linear");
+  return y;
+}
+}  // namespace
+
+PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.def("stream_norm", &stream_norm, py::arg("x"), py::arg("y"), py::arg("mix"), py::arg("out"), py::arg("m"),
+        py::arg("in_"), py::arg("w"), py::arg("eps"), py::arg("ids") = py::none(), py::arg("embed") = py::none(),
+        py::arg("rows") = py::none());
+  m.def("clamped_glu", &clamped_glu);
+  m.def("qk_norm_append", &qk_norm_append);
+  m.def("paged_generic", &paged_generic);
+  m.def("delta_prepare", &delta_prepare);
+  m.def("delta_recur", &delta_recur);
+  m.def("decode_linear", &decode_linear);
+  m.def("decode_linear_ok", &decode_linear_ok);
+}

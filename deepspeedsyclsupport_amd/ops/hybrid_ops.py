@@ -1,0 +1,58 @@
+"""Ops of the hybrid decoder (`inference/model_implementations/hybrid.py`): multi-stream residual, attention with
+per-head norms and chunked visibility, gated delta rule, clamped gated activation.
+
+Device tensors run the gfx950 kernels of `ds_hybrid_ops` (fp32 or bf16 storage, fp32 arithmetic); host tensors the
+plain versions in `ops/reference.py`, as everywhere in `ops`."""
+import torch
+import torch.nn.functional as F
+
+from . import reference
+from .native import hybrid_ops, use_native
+
+DECODE_ROWS = 16
+
+
+def stream_norm(x, y, mix, out, m, in_, w, eps, ids=None, embed=None, rows=None):
+    """Finish a sublayer (y, mix, out) or embed (ids, embed) into the streams x [T, S, W] fp32, in place, and return
+    the layer norm of sum_s in_[s] x_s. `rows`: norm these rows only and leave x as it is (in_ None: plain sum)."""
+    f = hybrid_ops().stream_norm if use_native(x) else reference.stream_norm
+    return f(x, y, mix, out, m, in_, w, eps, ids, embed, rows)
+
+
+def clamped_glu(gu, limit, alpha=1.702, shift=1.0):
+    """[.., gate | up] -> g sigmoid(alpha g) (u + shift) with g = min(gate, limit), u = clamp(up, +-limit)."""
+    f = hybrid_ops().clamped_glu if use_native(gu) else reference.clamped_glu
+    return f(gu, limit, alpha, shift)
+
+
+def qk_norm_append(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H):
+    f = hybrid_ops().qk_norm_append if use_native(qkv) else reference.qk_norm_append
+    return f(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H)
+
+
+def ragged_attention(q, kc, vc, meta, scale, softcap=0.0, window=0, chunk=0):
+    """q [T, H, dk] of a ragged batch (`RaggedMeta`) over the paged cache, the new tokens already appended."""
+    args = (meta.block_tables, meta.pos_ids, meta.seq_ids, scale, softcap, window, chunk)
+    if not use_native(q):
+        return reference.paged_attention(q, kc, vc, *args)
+    return hybrid_ops().paged_generic(q, kc, vc, *args)
+
+
+def delta_rule(proj, conv_w, a_log, dt_bias, norm_w, eps, state, conv_state, meta, Hk, H, dk, dv):
+    """Fused projection rows [T, q | k | v | g | b | a] -> gated, normed read-out [T, H dv]; the state slots advance."""
+    out = proj.new_empty(proj.shape[0], H * dv)
+    ops = hybrid_ops() if use_native(proj) else reference
+    qk, v, gb = ops.delta_prepare(proj, conv_w, conv_state, a_log, dt_bias, meta.seq_ids, meta.cu_q, meta.start_pos,
+                                  meta.slots, Hk, H, dk, dv)
+    for seqs in (meta.seq_list, meta.chunk_seqs):
+        ops.delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, meta.cu_q, meta.start_pos, meta.slots, out)
+    return out
+
+
+def linear(x, w):
+    """x . w^T: a weight stream for decode-sized bf16 batches, else the library product."""
+    rows = x.numel() // x.shape[-1]
+    if x.is_cuda and x.dtype == torch.bfloat16 and 0 < rows <= DECODE_ROWS and \
+            hybrid_ops().decode_linear_ok(rows, x.shape[-1]):
+        return hybrid_ops().decode_linear(x, w)
+    return F.linear(x, w)

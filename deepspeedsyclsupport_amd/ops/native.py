@@ -19,6 +19,12 @@ def hip_ops():
 
 
 @functools.lru_cache(None)
+def hybrid_ops():
+    """The gfx950 ops of the hybrid decoder (a module of its own, see `op_builder.EXTENSIONS`)."""
+    return op_builder.load("ds_hybrid_ops")
+
+
+@functools.lru_cache(None)
 def cpu_ops():
     return op_builder.load("ds_cpu_ops")
 

@@ -58,6 +58,21 @@ EXTENSIONS = {
         "bindings": ["bind/ds_hip_ops.cpp", "bind/infer_bind.cpp", "bind/moe_bind.cpp", "bind/host_mem.cpp",
                      "bind/comm_bind.cpp", "bind/attn_small_bind.cpp"],
     },
+    # what serving a hybrid decoder (inference/model_implementations/hybrid.py) needs, and nothing else: in a fresh
+    # checkout such a model starts after compiling these sources only
+    "ds_hybrid_ops": {
+        "kind": "hip",
+        "kernels": [
+            "norm/stream_norm.hip",
+            "act/clamped_glu.hip",
+            "attn/qk_norm_append.hip",
+            "attn/paged_generic.hip",
+            "recur/delta_rule.hip",
+            "gemv/skinny_gemm.hip",
+            "gemv/skinny_mfma.hip",
+        ],
+        "bindings": ["bind/hybrid_bind.cpp"],
+    },
     # host ops: CPU Adam/Adagrad/Lion (ZeRO-Offload, Twin-Flow), async tensor I/O (ZeRO-Infinity), shm all-reduce
     "ds_cpu_ops": {
         "kind": "cpu",
@@ -131,13 +146,16 @@ def _write_ninja(names):
         "  command = $cxx $in -o $out $ldflags $libs",
         "  description = LINK $out",
     ]
+    kernel_objs = set()  # a kernel that several extensions link is compiled once
     for name in names:
         spec = EXTENSIONS[name]
         objs = []
         if spec["kind"] == "hip":
             for src in spec["kernels"]:
-                obj = os.path.join(BUILD_DIR, name, src.replace("/", "_") + ".o")
-                lines.append(f"build {obj}: hip {os.path.join(CSRC, src)}")
+                obj = os.path.join(BUILD_DIR, "kernels", src.replace("/", "_") + ".o")
+                if obj not in kernel_objs:
+                    lines.append(f"build {obj}: hip {os.path.join(CSRC, src)}")
+                    kernel_objs.add(obj)
                 objs.append(obj)
             for bsrc in spec["bindings"]:
                 bobj = os.path.join(BUILD_DIR, name, bsrc.replace("/", "_") + ".o")

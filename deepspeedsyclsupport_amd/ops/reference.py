@@ -126,3 +126,102 @@ def apply_rope_half(x, cos, sin, pos):
 def cross_entropy(logits, labels, ignore_index=-100, smoothing=0.0):
     return F.cross_entropy(logits.float(), labels, ignore_index=ignore_index, reduction="none",
                            label_smoothing=smoothing)
+
+
+# ------------------------------------------------------------------------------------------------ hybrid decoder
+def stream_norm(x, y, mix, out, m, in_, w, eps, ids=None, embed=None, rows=None):
+    """Multi-stream residual update (in place on x [T, S, W]) + layer norm of the streams' weighted sum."""
+    src = y if y is not None else embed
+    if y is not None:
+        xn = torch.einsum("st,nsw->ntw", mix, x) + m * out[None, :, None] * y.float().view(x.shape[0], 1, -1)
+    else:
+        xn = embed.float()[ids.long()][:, None].expand(-1, x.shape[1], -1)
+    if rows is not None:
+        xn = xn[rows.long()]
+    else:
+        x.copy_(xn)
+    u = (xn if in_ is None else xn * in_[None, :, None]).sum(1)
+    d = u - u.mean(-1, keepdim=True)
+    return (d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * w).to(src.dtype)
+
+
+def clamped_glu(gu, limit, alpha, shift):
+    g, u = gu.float().chunk(2, -1)
+    g = g.clamp(max=limit)
+    return (g * torch.sigmoid(alpha * g) * (u.clamp(-limit, limit) + shift)).to(gu.dtype)
+
+
+def qk_norm_append(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H):
+    G, BS, dk, dv = kc.shape[1], kc.shape[2], kc.shape[3], vc.shape[3]
+    T = qkv.shape[0]
+    q, k, v = qkv.float().split([H * dk, G * dk, G * dv], -1)
+    q, k, v = q.view(T, H, dk), k.view(T, G, dk), v.view(T, G, dv)
+    q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps) * qw
+    k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps) * kw
+    if vfirst is not None:
+        v = (1 - lam) * v + lam * vfirst.float().view(T, G, dv)
+    slot = pos.long()
+    blk = block_table.long()[seq_ids.long(), slot // BS]
+    kc[blk, :, slot % BS] = k.to(kc.dtype)
+    vc[blk, :, slot % BS] = v.to(vc.dtype)
+    return q.to(qkv.dtype)
+
+
+def paged_attention(q, kc, vc, block_table, pos, seq_ids, scale, softcap, window, chunk):
+    """q [T, H, dk] at absolute positions -> [T, H, dv]; visible keys [lo(pos), pos] (window / chunk start / 0)."""
+    G, BS = kc.shape[1], kc.shape[2]
+    out = q.new_empty(q.shape[0], q.shape[1], vc.shape[3])
+    for t in range(q.shape[0]):
+        p = int(pos[t])
+        lo = max(p // chunk * chunk if chunk else 0, p - window + 1 if window else 0)
+        j = torch.arange(lo, p + 1)
+        blk = block_table[int(seq_ids[t])].long()[j // BS]
+        k, v = kc[blk, :, j % BS].float(), vc[blk, :, j % BS].float()         # [n, G, d]
+        qq = q[t].float().view(G, q.shape[1] // G, -1)
+        s = torch.einsum("grd,ngd->grn", qq, k) * scale
+        if softcap:
+            s = softcap * torch.tanh(s / softcap)
+        out[t] = torch.einsum("grn,ngd->grd", s.softmax(-1), v).reshape(q.shape[1], -1).to(q.dtype)
+    return out
+
+
+def delta_prepare(proj, conv_w, conv_state, a_log, dt_bias, seq_ids, cu, start, slots, Hk, H, dk, dv):
+    T, taps = proj.shape[0], conv_w.shape[-1]
+    C = 2 * Hk * dk + H * dv
+    x = torch.empty(T, C)
+    for i in range(start.numel()):
+        a, b, slot = int(cu[i]), int(cu[i + 1]), int(slots[i])
+        old = conv_state[slot].float() if int(start[i]) else torch.zeros(taps - 1, C)
+        seq = torch.cat([old, proj[a:b, :C].float()])
+        x[a:b] = sum(seq[j:j + b - a] * conv_w[:, j] for j in range(taps))
+    x = F.silu(x)
+    q, k, v = x.split([Hk * dk, Hk * dk, H * dv], -1)
+    q, k = q.view(T, Hk, dk), k.view(T, Hk, dk)
+    q = q * torch.rsqrt(q.pow(2).sum(-1, keepdim=True) + 1e-6) * dk**-0.5
+    k = k * torch.rsqrt(k.pow(2).sum(-1, keepdim=True) + 1e-6)
+    b, a = proj[:, C + H * dv:].float().split(H, -1)
+    glog = -a_log.exp() * F.softplus(a + dt_bias)
+    return torch.stack([q, k], 1), v.view(T, H, dv).to(proj.dtype), torch.stack([glog, b.sigmoid()], 1)
+
+
+def delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, cu, start, slots, out):
+    T, H, dv = v.shape
+    Hk, dk = qk.shape[2], qk.shape[3]
+    C, taps = conv_state.shape[2], conv_state.shape[1] + 1
+    out = out.view(T, H, dv)
+    rep = H // Hk
+    for i in seqs.tolist():
+        a, b, slot = int(cu[i]), int(cu[i + 1]), int(slots[i])
+        S = state[slot].clone() if int(start[i]) else torch.zeros(H, dk, dv)
+        for t in range(a, b):
+            q, k = qk[t].repeat_interleave(rep, 1)
+            S = S * gb[t, 0].exp()[:, None, None]
+            u = gb[t, 1][:, None] * (v[t].float() - (S * k[:, :, None]).sum(1))
+            S = S + k[:, :, None] * u[:, None]
+            o = (S * q[:, :, None]).sum(1)
+            o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * norm_w
+            out[t] = (o * F.silu(proj[t, C:C + H * dv].float().view(H, dv))).to(out.dtype)
+        state[slot] = S
+        if taps > 1:
+            old = conv_state[slot] if int(start[i]) else torch.zeros_like(conv_state[slot])
+            conv_state[slot] = torch.cat([old, proj[a:b, :C]])[-(taps - 1):].clone()

@@ -44,7 +44,7 @@ setup(
     package_data={"deepspeedsyclsupport_amd": ["ops/csrc/**/*", "ops/lib/*.so"]},
     include_package_data=True,
     scripts=[os.path.join("bin", s) for s in ("deepspeed", "deepspeed.pt", "ds", "ds_report", "ds_ssh", "ds_bench",
-                                              "ds_elastic", "dsr")],
+                                              "ds_elastic", "dsr", "trace_run")],
     python_requires=">=3.8",
     install_requires=["torch", "numpy", "pydantic>=2", "psutil", "packaging", "tqdm", "ninja"],
     extras_require={"inf": ["transformers", "safetensors"], "sparse_attn": [], "autotuning": ["tabulate"]},
