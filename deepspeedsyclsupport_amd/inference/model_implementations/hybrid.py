@@ -207,6 +207,10 @@ class DSHybridLayer(ProjectionLayer):
 class DSHybridModel(DSInferenceModel):
     layer_class = DSHybridLayer
 
+    def __init__(self, spec, tp_group=None, tp_size=1, tp_rank=0, dtype=torch.bfloat16, device=None):
+        super().__init__(spec, tp_group, tp_size, tp_rank, dtype, device)
+        self.norm_w = _f32((spec.hidden_size, ), 1.0, device)  # norms read the fp32 streams
+
     # ------------------------------------------------------------------------------------------ cache
     def kv_geometry(self):
         return [(m.G, m.dk, m.dv) if m.kind == "attention" else None for m in (la.mixer for la in self.layers)]
