@@ -171,7 +171,8 @@ class RaggedMeta:
     block_size: int
     slots: Optional[torch.Tensor] = None     # [S] state slot of every sequence (models with recurrent layers)
     seq_list: Optional[torch.Tensor] = None  # sequences whose portion is short: recurrent layers go token by token
-    chunk_seqs: Optional[torch.Tensor] = None  # the others, which go by chunks of `STATE_CHUNK` tokens
+    chunk_seqs: Optional[torch.Tensor] = None  # [L, 2] the others, by chunks of `STATE_CHUNK` tokens: (sequence, first
+                                               # entry in chunk_work)
     chunk_work: Optional[torch.Tensor] = None  # [N, 2] (sequence, chunk) of those
 
     STATE_CHUNK = 64     # tokens per chunk of a recurrent layer's parallel form
@@ -200,14 +201,17 @@ class RaggedMeta:
         slots = [] if slots is None else list(slots)
         long = [i for i in range(S) if n_new[i] > RaggedMeta.STEP_TOKENS] if slots else []
         short = [i for i in range(S) if n_new[i] <= RaggedMeta.STEP_TOKENS] if slots else []
-        chunks = [(i, c) for i in long for c in range(-(-n_new[i] // RaggedMeta.STATE_CHUNK))]
-        flat = pos + sid + list(starts) + lens + cu + [x for w in work for x in w] + last + bt + slots + short + long + \
+        chunks, chunk_seqs = [], []
+        for i in long:
+            chunk_seqs += [i, len(chunks)]
+            chunks += [(i, c) for c in range(-(-n_new[i] // RaggedMeta.STATE_CHUNK))]
+        flat = pos + sid + list(starts) + lens + cu + [x for w in work for x in w] + last + bt + slots + short + chunk_seqs + \
             [x for w in chunks for x in w]
         buf = torch.tensor(flat, dtype=torch.int32)
         if device is not None and torch.device(device).type == "cuda":
             buf = buf.pin_memory().to(device, non_blocking=True)
         views, o = [], 0
-        for n in (T, T, S, S, S + 1, 2 * len(work), len(last), S * width, len(slots), len(short), len(long),
+        for n in (T, T, S, S, S + 1, 2 * len(work), len(last), S * width, len(slots), len(short), len(chunk_seqs),
                   2 * len(chunks)):
             views.append(buf[o:o + n])
             o += n
@@ -215,7 +219,7 @@ class RaggedMeta:
         return RaggedMeta(block_tables=bt_t.view(S, width), start_pos=st_t, seq_lens=len_t, pos_ids=pos_t,
                           seq_ids=sid_t, cu_q=cu_t, work=work_t.view(-1, 2), last_idx=last_t.long(),
                           n_decode=n_decode, cu_host=cu, start_host=list(starts), max_len=width * block_size,
-                          block_size=block_size, slots=slot_t, seq_list=short_t, chunk_seqs=long_t,
+                          block_size=block_size, slots=slot_t, seq_list=short_t, chunk_seqs=long_t.view(-1, 2),
                           chunk_work=chunk_t.view(-1, 2))
 
 

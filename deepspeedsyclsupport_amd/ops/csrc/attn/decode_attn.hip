@@ -12,7 +12,9 @@
 //  * scores for the slice live in LDS; softmax runs on LDS; P·V streams V rows with 16-B loads, 16 lanes per row;
 //  * partial (max, sum, unnormalised acc) per split are merged by a small combine kernel (log-sum-exp). (An in-kernel
 //    last-block merge was measured 2x slower: the device-scope fences it needs write back L2.)
-// Optional ALiBi slopes (BLOOM) and a sliding window (Mistral) are applied on the fly.
+// Optional ALiBi slopes (BLOOM) are applied on the fly. With a sliding window (Mistral) or chunked visibility only the
+// keys in sight are split and read. A second instantiation takes key and value widths of their own (multiples of 8), a
+// tanh score cap and GQA groups of any size.
 #include "../include/ds_hip.h"
 
 namespace {
@@ -21,35 +23,44 @@ constexpr int THREADS = 256;
 constexpr int MAXG = 8;          // query heads per kv head handled per workgroup (GQA group)
 constexpr int MAX_CHUNK = 1024;  // keys per split (LDS: MAXG * MAX_CHUNK * 4 B = 32 KiB)
 
-template <int D>
+// lanes per row of D elements, 8 each: D / 8 rounded up to a power of two
+constexpr int lanes_per_row(int d) { return d <= 64 ? 8 : (d <= 128 ? 16 : 32); }
+
+// DK, DV: the widths; 0: given at run time (dk, dv), LK / LV lanes per row
+template <int DK, int DV, int LK = lanes_per_row(DK), int LV = lanes_per_row(DV)>
 __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
-    const bf16* __restrict__ q,          // [B, Hq, D]
-    const bf16* __restrict__ kc,         // [NB, Hk, BS, D]
-    const bf16* __restrict__ vc,         // [NB, Hk, BS, D]
+    const bf16* __restrict__ q,          // [B, Hq, dk]
+    const bf16* __restrict__ kc,         // [NB, Hk, BS, dk]
+    const bf16* __restrict__ vc,         // [NB, Hk, BS, dv]
     const int* __restrict__ block_table, // [B, max_blocks]
     const int* __restrict__ seq_lens,    // [B]
     const float* __restrict__ alibi,     // [Hq] or null
-    float* __restrict__ part_acc,        // [B, Hq, S, D]  (only if S > 1)
+    float* __restrict__ part_acc,        // [B, Hq, S, dv]  (only if S > 1)
     float* __restrict__ part_ml,         // [B, Hq, S, 2]
-    bf16* __restrict__ out,              // [B, Hq, D]  (written directly when S == 1)
-    int Hq, int Hk, int BS, int max_blocks, int chunk, float scale, int window) {
-  static_assert(D % 16 == 0 && D >= 64 && D <= 256, "head dim");
+    bf16* __restrict__ out,              // [B, Hq, dv]  (written directly when S == 1)
+    int Hq, int Hk, int BS, int max_blocks, int chunk, float scale, int window, int mask_chunk, float softcap, int dk_rt,
+    int dv_rt) {
+  constexpr bool EXT = DK == 0;
+  static_assert(EXT || (DK % 16 == 0 && DK >= 64 && DK <= 256 && DK == DV), "head dim");
+  const int dk = EXT ? dk_rt : DK, dv = EXT ? dv_rt : DV;
   extern __shared__ __attribute__((aligned(16))) float sm[];  // scores [G][chunk] + reduction scratch
-  const int b = blockIdx.x, kh = blockIdx.y, split = blockIdx.z, S = gridDim.z;
-  const int G = Hq / Hk;
+  const int b = blockIdx.x, kh = EXT ? blockIdx.y % Hk : blockIdx.y, split = blockIdx.z, S = gridDim.z;
+  const int g0 = EXT ? blockIdx.y / Hk * MAXG : 0;              // first query head of the group this block serves
+  const int GA = Hq / Hk, G = EXT ? min(MAXG, GA - g0) : GA, h0 = kh * GA + g0;
   const int T = seq_lens[b];
-  const int t0 = split * chunk;
+  int tlo = window > 0 ? max(0, T - window) : 0;                // first key in sight
+  if (mask_chunk > 0) tlo = max(tlo, (T - 1) / mask_chunk * mask_chunk);
+  const int t0 = tlo + split * chunk;
   const int t1 = min(T, t0 + chunk);
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
-  const int tlo = window > 0 ? max(0, T - window) : 0;
   float* scores = sm;                       // [G][chunk]
   float* red = sm + MAXG * MAX_CHUNK;       // [THREADS/64 * MAXG * 2]
 
   // ---- q of the G heads of this GQA group; LPR lanes cover one row, 8 elements each. LPR is D/8 rounded up to a
   // power of two (head dims 80 and 96 use 16 lanes per row): the surplus lanes carry a zero query, re-read the row's
   // last chunk (a cache hit) and never write
-  constexpr int CPR = D / 8;                                   // 16-byte chunks per row
-  constexpr int LPR = CPR <= 8 ? 8 : (CPR <= 16 ? 16 : 32);    // lanes per key row (16 for D=128)
+  const int CPR = dk / 8;                                      // 16-byte chunks per row
+  constexpr int LPR = LK;                                      // lanes per key row (16 for D=128)
   constexpr int RPW = 64 / LPR;                                // rows per wave instruction
   const int sub = lane / LPR, li_raw = lane % LPR, li = li_raw < CPR ? li_raw : CPR - 1;
   const float lane_on = li_raw < CPR ? 1.f : 0.f;
@@ -58,7 +69,7 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
 #pragma unroll
   for (int g = 0; g < MAXG; ++g) {
     const int gc = g < G ? g : G - 1;
-    Vec8<bf16>::load(q + ((int64_t)b * Hq + kh * G + gc) * D + li * 8, qv[g]);
+    Vec8<bf16>::load(q + ((int64_t)b * Hq + h0 + gc) * dk + li * 8, qv[g]);
 #pragma unroll
     for (int j = 0; j < 8; ++j) qv[g][j] *= scale * lane_on;
   }
@@ -74,7 +85,7 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
 #pragma unroll
     for (int u = 0; u < UNR; ++u) {
       const int tc = min(tb + u * kstride, t1 - 1);
-      Vec8<bf16>::load(kc + (((int64_t)blk[u] * Hk + kh) * BS + tc % BS) * D + li * 8, kv[u]);
+      Vec8<bf16>::load(kc + (((int64_t)blk[u] * Hk + kh) * BS + tc % BS) * dk + li * 8, kv[u]);
     }
 #pragma unroll
     for (int u = 0; u < UNR; ++u) {
@@ -89,8 +100,8 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
 #pragma unroll
           for (int o = LPR / 2; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
           if (li_raw == 0) {
-            if (alibi) s += alibi[kh * G + g] * (float)(t - (T - 1));
-            if (t < tlo) s = -INFINITY;
+            if (alibi) s += alibi[h0 + g] * (float)(t - (T - 1));
+            if (EXT && softcap > 0.f) s = softcap * tanhf(s / softcap);
             scores[g * MAX_CHUNK + (t - t0)] = s;
           }
         }
@@ -98,12 +109,12 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
     }
   }
   // V rows do not depend on the scores: start the first P.V pass's loads before the softmax phases
-  constexpr int ROWS = THREADS / LPR;
-  const int r = tid / LPR, c_raw = tid % LPR, c = c_raw < CPR ? c_raw : CPR - 1;
+  constexpr int ROWS = THREADS / LV;
+  const int CPV = dv / 8, r = tid / LV, c_raw = tid % LV, c = c_raw < CPV ? c_raw : CPV - 1;
   float vpre[8];
   if (t0 + r < t1) {
     const int blk = bt[(t0 + r) / BS], off = (t0 + r) % BS;
-    Vec8<bf16>::load(vc + (((int64_t)blk * Hk + kh) * BS + off) * D + c * 8, vpre);
+    Vec8<bf16>::load(vc + (((int64_t)blk * Hk + kh) * BS + off) * dv + c * 8, vpre);
   }
   __syncthreads();
   // ---- phase 2: per-head max and sum over the split (one wave per head group, strided)
@@ -143,7 +154,7 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
 #pragma unroll
         for (int j = 0; j < 8; ++j) vv[u][j] = vpre[j];
       } else {
-        Vec8<bf16>::load(vc + (((int64_t)vblk[u] * Hk + kh) * BS + tc % BS) * D + c * 8, vv[u]);
+        Vec8<bf16>::load(vc + (((int64_t)vblk[u] * Hk + kh) * BS + tc % BS) * dv + c * 8, vv[u]);
       }
     }
 #pragma unroll
@@ -165,20 +176,20 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
 #pragma unroll
   for (int g = 0; g < MAXG; ++g) {
     if (g >= G) break;  // block-uniform
-    if (c_raw < CPR) {
+    if (c_raw < CPV) {
 #pragma unroll
-      for (int j = 0; j < 8; ++j) rb[r * D + c * 8 + j] = acc[g][j];
+      for (int j = 0; j < 8; ++j) rb[r * dv + c * 8 + j] = acc[g][j];
     }
     __syncthreads();
-    for (int idx = tid; idx < D; idx += THREADS) {
+    for (int idx = tid; idx < dv; idx += THREADS) {
       float s = 0.f;
-      for (int rr = 0; rr < ROWS; ++rr) s += rb[rr * D + idx];
-      const int hq = kh * G + g;
+      for (int rr = 0; rr < ROWS; ++rr) s += rb[rr * dv + idx];
+      const int hq = h0 + g;
       const float m = red[g * 2], l = red[g * 2 + 1];
       if (S == 1) {
-        out[((int64_t)b * Hq + hq) * D + idx] = (bf16)(l > 0.f ? s / l : 0.f);
+        out[((int64_t)b * Hq + hq) * dv + idx] = (bf16)(l > 0.f ? s / l : 0.f);
       } else {
-        part_acc[(((int64_t)b * Hq + hq) * S + split) * D + idx] = s;
+        part_acc[(((int64_t)b * Hq + hq) * S + split) * dv + idx] = s;
         if (idx == 0) {
           part_ml[(((int64_t)b * Hq + hq) * S + split) * 2] = m;
           part_ml[(((int64_t)b * Hq + hq) * S + split) * 2 + 1] = l;
@@ -189,10 +200,10 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
   }
 }
 
-template <int D>
-__global__ void __launch_bounds__(D) combine_kernel(const float* __restrict__ part_acc,
-                                                    const float* __restrict__ part_ml, bf16* __restrict__ out, int S) {
-  const int bh = blockIdx.x, d = threadIdx.x;
+// blockDim.x = D, the value width
+__global__ void __launch_bounds__(256) combine_kernel(const float* __restrict__ part_acc,
+                                                      const float* __restrict__ part_ml, bf16* __restrict__ out, int S) {
+  const int bh = blockIdx.x, d = threadIdx.x, D = blockDim.x;
   float M = -INFINITY;
   for (int s = 0; s < S; ++s) M = fmaxf(M, part_ml[((int64_t)bh * S + s) * 2]);
   float num = 0.f, den = 0.f;
@@ -316,17 +327,18 @@ extern "C" int ds_paged_decode(const void* q, const void* kc, const void* vc, co
                                int B, int Hq, int Hk, int D, int BS, int max_blocks, int max_len, int splits,
                                float scale, int window, hipStream_t s) {
   if (Hq % Hk || Hq / Hk > MAXG) return (int)hipErrorInvalidValue;
+  if (window > 0 && window < max_len) max_len = window;  // no more keys than that are in sight
   const int chunk = ((max_len + splits - 1) / splits + 63) / 64 * 64;
   if (chunk > MAX_CHUNK) return (int)hipErrorInvalidValue;
   const size_t lds = (size_t)(MAXG * MAX_CHUNK + 64) * sizeof(float);
   dim3 grid(B, Hk, splits);
 #define LAUNCH(DD)                                                                                                  \
-  hipLaunchKernelGGL((paged_decode_kernel<DD>), grid, dim3(THREADS), lds, s, (const bf16*)q, (const bf16*)kc,       \
+  hipLaunchKernelGGL((paged_decode_kernel<DD, DD>), grid, dim3(THREADS), lds, s, (const bf16*)q, (const bf16*)kc,       \
                      (const bf16*)vc, block_table, seq_lens, alibi, part_acc, part_ml, (bf16*)out, Hq, Hk, BS,       \
-                     max_blocks, chunk, scale, window);                                                             \
+                     max_blocks, chunk, scale, window, 0, 0.f, DD, DD);                                             \
   DS_CHECK_LAUNCH();                                                                                                \
   if (splits > 1) {                                                                                                 \
-    hipLaunchKernelGGL((combine_kernel<DD>), dim3(B * Hq), dim3(DD), 0, s, part_acc, part_ml, (bf16*)out, splits);  \
+    hipLaunchKernelGGL(combine_kernel, dim3(B * Hq), dim3(DD), 0, s, part_acc, part_ml, (bf16*)out, splits);  \
     DS_CHECK_LAUNCH();                                                                                              \
   }
   if (D == 64) { LAUNCH(64) }
@@ -336,6 +348,42 @@ extern "C" int ds_paged_decode(const void* q, const void* kc, const void* vc, co
   else if (D == 256) { LAUNCH(256) }
   else return (int)hipErrorInvalidValue;
 #undef LAUNCH
+  return 0;
+}
+
+// Key / value widths of their own (multiples of 8 up to 256), chunked and / or windowed visibility, score cap. `splits`
+// from ds_paged_decode_splits(B, Hk, span) with span = the most keys in sight.
+extern "C" int ds_paged_decode_ext(const void* q, const void* kc, const void* vc, const int* block_table,
+                                   const int* seq_lens, float* part_acc, float* part_ml, void* out, int B, int Hq, int Hk,
+                                   int dk, int dv, int BS, int max_blocks, int span, int splits, float scale,
+                                   float softcap, int window, int mask_chunk, hipStream_t s) {
+  if (Hk <= 0 || Hq % Hk || dk % 8 || dv % 8 || dk <= 0 || dv <= 0 || dk > 256 || dv > 256 || splits <= 0)
+    return (int)hipErrorInvalidValue;
+  const int chunk = ((span + splits - 1) / splits + 63) / 64 * 64;
+  if (chunk > MAX_CHUNK) return (int)hipErrorInvalidValue;
+  // scores [MAXG][MAX_CHUNK] + maxima / sums; the value reduction reuses it ([256 / lanes per row][dv] floats)
+  const size_t lds = (size_t)(MAXG * MAX_CHUNK + 64) * sizeof(float);
+  dim3 grid(B, Hk * ((Hq / Hk + MAXG - 1) / MAXG), splits);
+#define GO(LK, LV)                                                                                                  \
+  hipLaunchKernelGGL((paged_decode_kernel<0, 0, LK, LV>), grid, dim3(THREADS), lds, s, (const bf16*)q, (const bf16*)kc, \
+                     (const bf16*)vc, block_table, seq_lens, nullptr, part_acc, part_ml, (bf16*)out, Hq, Hk, BS,     \
+                     max_blocks, chunk, scale, window, mask_chunk, softcap, dk, dv)
+#define ROW(LK)                 \
+  {                             \
+    if (dv <= 64) GO(LK, 8);    \
+    else if (dv <= 128) GO(LK, 16); \
+    else GO(LK, 32);            \
+  }
+  if (dk <= 64) ROW(8)
+  else if (dk <= 128) ROW(16)
+  else ROW(32)
+#undef ROW
+#undef GO
+  DS_CHECK_LAUNCH();
+  if (splits > 1) {
+    hipLaunchKernelGGL(combine_kernel, dim3(B * Hq), dim3(dv), 0, s, part_acc, part_ml, (bf16*)out, splits);
+    DS_CHECK_LAUNCH();
+  }
   return 0;
 }
 

@@ -17,6 +17,9 @@
 //  * the compute core is flash_fwd.hip's: 4 waves x 32 rows, S^T = K.Q^T on v_mfma_f32_32x32x16_bf16 so each lane
 //    owns one query row's scores, P reused as the A operand of O += P.V, V by ds_read_b64_tr_b16 from the same
 //    XOR-swizzled LDS image, next tile's loads issued before the current tile's MFMAs;
+//  * a second instantiation (EXT) takes key and value widths of their own (any multiple of 8, tiled at the next of 32 /
+//    64 / 128 / 256), chunked visibility (key >= pos - pos % chunk) and a tanh score cap, with their sizes as run-time
+//    arguments. It keeps the softmax weights to 16 mantissa bits through the P.V product (two bf16 operands, high + low);
 //  * the head dim is a template parameter: D / 16 MFMA steps for the scores, ceil(D / 32) output column tiles (D = 80
 //    computes a third, half-used tile over zero-filled LDS columns), LDS rows pitched to 16 (D <= 128) or 32 (D = 256)
 //    16-byte chunks so one swizzle serves every size.
@@ -28,18 +31,19 @@ constexpr int BM = 128;
 constexpr int BN = 64;
 constexpr int NTHR = 256;
 
-template <int D>
+template <int DK, int DV>
 struct Cfg {
-  static_assert(D % 16 == 0 && D >= 64 && D <= 256, "head dim");
-  static constexpr int KC = D / 16;               // MFMA steps of the score product
-  static constexpr int DT = (D + 31) / 32;        // 32-column output tiles
-  static constexpr int CH = D / 8;                // 16-byte chunks holding data in one K / V row
-  static constexpr int PCH = D <= 128 ? 16 : 32;  // chunks per LDS row (pitch)
-  static constexpr int ROWB = PCH * 16;
-  static constexpr int TILE_BYTES = BN * ROWB;
-  static constexpr int NLD = BN * PCH / NTHR;     // chunks staged per thread per tile
-  static constexpr int LDS_BYTES = 4 * TILE_BYTES + 4 * 32 * 4;
-  static constexpr int OCC = D <= 128 ? 2 : 1;
+  static_assert(DK % 16 == 0 && DK >= 32 && DK <= 256 && DV % 16 == 0 && DV >= 32 && DV <= 256, "head dims");
+  static constexpr int KC = DK / 16;               // MFMA steps of the score product
+  static constexpr int DT = (DV + 31) / 32;        // 32-column output tiles
+  static constexpr int PK = DK <= 128 ? 16 : 32;   // 16-byte chunks per LDS row (pitch) of K, V
+  static constexpr int PV = DV <= 128 ? 16 : 32;
+  static constexpr int KBYTES = BN * PK * 16;
+  static constexpr int VBYTES = BN * PV * 16;
+  static constexpr int NLK = BN * PK / NTHR;       // chunks staged per thread per tile
+  static constexpr int NLV = BN * PV / NTHR;
+  static constexpr int LDS_BYTES = 2 * KBYTES + 2 * VBYTES + 4 * 32 * 4;
+  static constexpr int OCC = DK <= 128 && DV <= 128 ? 2 : 1;
 };
 
 typedef short s16x4_t __attribute__((ext_vector_type(4)));
@@ -65,13 +69,15 @@ struct PagedArgs {
   int Hq, Hk, BS, max_blocks, window;
   float c;                // softmax scale * log2(e)
   float inv_scale;        // 1 / softmax scale (ALiBi bias in score units)
+  int dk, dv, chunk;      // EXT: head widths, chunk of the visibility mask (0: none)
+  float cap_in, cap_out;  // EXT: capped score in log2 units = cap_out * tanh(score * cap_in); cap_out 0: no cap
 };
 
-template <int D>
-__global__ void __launch_bounds__(NTHR, Cfg<D>::OCC) paged_prefill_kernel(PagedArgs a) {
-  using C = Cfg<D>;
-  constexpr int KC = C::KC, DT = C::DT, CH = C::CH, PCH = C::PCH, ROWB = C::ROWB, TILE_BYTES = C::TILE_BYTES,
-                NLD = C::NLD;
+template <int DK, int DV, bool EXT>
+__global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel(PagedArgs a) {
+  using C = Cfg<DK, DV>;
+  constexpr int KC = C::KC, DT = C::DT, PK = C::PK, PV = C::PV, RK = PK * 16, RV = PV * 16, NLK = C::NLK, NLV = C::NLV;
+  const int dk = EXT ? a.dk : DK, dv = EXT ? a.dv : DV;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, h = lane >> 5, l32 = lane & 31;
   const int logical = xcd_remap(blockIdx.x, gridDim.x);
@@ -85,42 +91,78 @@ __global__ void __launch_bounds__(NTHR, Cfg<D>::OCC) paged_prefill_kernel(PagedA
   bf16x8_t qf[KC];
   {
     const int qr = min(q0w + l32, n - 1);
-    const bf16* qrow = a.q + ((int64_t)(t0 + qr) * a.Hq + hq) * D + 8 * h;
+    const bf16* qrow = a.q + ((int64_t)(t0 + qr) * a.Hq + hq) * dk + 8 * h;
 #pragma unroll
-    for (int kk = 0; kk < KC; ++kk) qf[kk] = *reinterpret_cast<const bf16x8_t*>(qrow + 16 * kk);
+    for (int kk = 0; kk < KC; ++kk) {
+      if (!EXT || 16 * kk + 8 * h < dk) {
+        qf[kk] = *reinterpret_cast<const bf16x8_t*>(qrow + 16 * kk);
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) qf[kk][e] = (bf16)0.f;
+      }
+    }
   }
   const int pos_lane = start + q0w + l32;                // this lane's query position
   const int pos_hi = start + min(q0 + BM, n) - 1;        // last query position of the block
   const int wpos_lo = start + q0w, wpos_hi = start + q0w + 31;
   int kt1 = min((Skv + BN - 1) / BN, pos_hi / BN + 1);
-  int kt0 = a.window > 0 ? max(0, (start + q0 - a.window + 1) / BN) : 0;
+  // first key a position sees (non-decreasing in the position)
+  auto first_key = [&](int p) {
+    int lo = EXT && a.chunk > 0 ? p / a.chunk * a.chunk : 0;
+    if (a.window > 0) lo = max(lo, p - a.window + 1);
+    return lo;
+  };
+  const int lo_lane = first_key(pos_lane), lo_whi = first_key(wpos_hi), lo_wlo = first_key(wpos_lo);
+  int kt0 = first_key(start + q0) / BN;
   if (kt0 > kt1) kt0 = kt1;
 
-  float* scratch = reinterpret_cast<float*>(smem + 4 * TILE_BYTES) + wid * 32;
-  u32x4_t kreg[NLD], vreg[NLD];
+  char* const ksm = smem;
+  char* const vsm = smem + 2 * C::KBYTES;
+  float* scratch = reinterpret_cast<float*>(smem + 2 * C::KBYTES + 2 * C::VBYTES) + wid * 32;
+  u32x4_t kreg[NLK], vreg[NLV];
+  auto slot_of = [&](int tile, int row) {
+    const int key = min(tile * BN + row, Skv - 1);
+    return ((int64_t)bt[key / a.BS] * a.Hk + hk) * a.BS + key % a.BS;
+  };
   auto stage_load = [&](int tile) {
+    if constexpr (!EXT) {  // one pitch, one width: the key and value chunk share their address
 #pragma unroll
-    for (int i = 0; i < NLD; ++i) {
-      const int cidx = tid + i * NTHR, row = cidx / PCH, ch = cidx % PCH;
-      if (ch < CH) {
-        const int key = min(tile * BN + row, Skv - 1);
-        const int64_t off = (((int64_t)bt[key / a.BS] * a.Hk + hk) * a.BS + key % a.BS) * D + ch * 8;
-        kreg[i] = *reinterpret_cast<const u32x4_t*>(a.kc + off);
-        vreg[i] = *reinterpret_cast<const u32x4_t*>(a.vc + off);
-      } else {  // pitch padding: zero columns (read by the last, partly used output tile of D = 80)
+      for (int i = 0; i < NLK; ++i) {
+        const int cidx = tid + i * NTHR, row = cidx / PK, ch = cidx % PK;
+        if (ch < DK / 8) {
+          const int64_t off = slot_of(tile, row) * DK + ch * 8;
+          kreg[i] = *reinterpret_cast<const u32x4_t*>(a.kc + off);
+          vreg[i] = *reinterpret_cast<const u32x4_t*>(a.vc + off);
+        } else {  // pitch padding: zero columns (read by the last, partly used output tile of D = 80)
+          kreg[i] = u32x4_t{0u, 0u, 0u, 0u};
+          vreg[i] = u32x4_t{0u, 0u, 0u, 0u};
+        }
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < NLK; ++i) {
+        const int cidx = tid + i * NTHR, row = cidx / PK, ch = cidx % PK;
         kreg[i] = u32x4_t{0u, 0u, 0u, 0u};
+        if (ch * 8 < dk) kreg[i] = *reinterpret_cast<const u32x4_t*>(a.kc + slot_of(tile, row) * dk + ch * 8);
+      }
+#pragma unroll
+      for (int i = 0; i < NLV; ++i) {
+        const int cidx = tid + i * NTHR, row = cidx / PV, ch = cidx % PV;
         vreg[i] = u32x4_t{0u, 0u, 0u, 0u};
+        if (ch * 8 < dv) vreg[i] = *reinterpret_cast<const u32x4_t*>(a.vc + slot_of(tile, row) * dv + ch * 8);
       }
     }
   };
   auto stage_store = [&](int buf) {
 #pragma unroll
-    for (int i = 0; i < NLD; ++i) {
-      const int cidx = tid + i * NTHR, row = cidx / PCH, ch = cidx % PCH;
-      if (ch < 4 * DT) {
-        *reinterpret_cast<u32x4_t*>(smem + buf * TILE_BYTES + lds_off<ROWB>(row, ch)) = kreg[i];
-        *reinterpret_cast<u32x4_t*>(smem + (2 + buf) * TILE_BYTES + lds_off<ROWB>(row, ch)) = vreg[i];
-      }
+    for (int i = 0; i < NLK; ++i) {
+      const int cidx = tid + i * NTHR, row = cidx / PK, ch = cidx % PK;
+      if (ch < DK / 8) *reinterpret_cast<u32x4_t*>(ksm + buf * C::KBYTES + lds_off<RK>(row, ch)) = kreg[i];
+    }
+#pragma unroll
+    for (int i = 0; i < NLV; ++i) {
+      const int cidx = tid + i * NTHR, row = cidx / PV, ch = cidx % PV;
+      if (ch < 4 * DT) *reinterpret_cast<u32x4_t*>(vsm + buf * C::VBYTES + lds_off<RV>(row, ch)) = vreg[i];
     }
   };
 
@@ -140,10 +182,10 @@ __global__ void __launch_bounds__(NTHR, Cfg<D>::OCC) paged_prefill_kernel(PagedA
     const int cur = (j - kt0) & 1;
     if (j + 1 < kt1) stage_load(j + 1);
     const int k0 = j * BN;
-    const bool active = q0w < n && k0 <= wpos_hi && (a.window <= 0 || k0 + BN - 1 > wpos_lo - a.window);
+    const bool active = q0w < n && k0 <= wpos_hi && k0 + BN - 1 >= lo_wlo;
     if (active) {
-      const char* Kt = smem + cur * TILE_BYTES;
-      const char* Vt = smem + (2 + cur) * TILE_BYTES;
+      const char* Kt = ksm + cur * C::KBYTES;
+      const char* Vt = vsm + cur * C::VBYTES;
       f32x16_t s[2];
 #pragma unroll
       for (int t = 0; t < 2; ++t) {
@@ -151,13 +193,21 @@ __global__ void __launch_bounds__(NTHR, Cfg<D>::OCC) paged_prefill_kernel(PagedA
         for (int r = 0; r < 16; ++r) s[t][r] = 0.f;
 #pragma unroll
         for (int kk = 0; kk < KC; ++kk) {
-          const bf16x8_t av = *reinterpret_cast<const bf16x8_t*>(Kt + lds_off<ROWB>(t * 32 + l32, 2 * kk + h));
+          const bf16x8_t av = *reinterpret_cast<const bf16x8_t*>(Kt + lds_off<RK>(t * 32 + l32, 2 * kk + h));
           s[t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(av, qf[kk], s[t], 0, 0, 0);
         }
       }
       // ALiBi bias, causal diagonal, window, key tail (lane = one query row, r = 32 keys of the 64)
-      const bool need_mask = k0 + BN - 1 > wpos_lo || k0 + BN > Skv ||
-                             (a.window > 0 && k0 <= wpos_hi - a.window);
+      const bool need_mask = k0 + BN - 1 > wpos_lo || k0 + BN > Skv || k0 < lo_whi;
+      if constexpr (EXT) {
+        if (a.cap_out > 0.f) {
+#pragma unroll
+          for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int r = 0; r < 16; ++r)  // tanh z = 1 - 2 / (e^2z + 1); cap_in carries the 2 log2(e)
+              s[t][r] = a.cap_out * (1.f - 2.f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s[t][r] * a.cap_in) + 1.f));
+        }
+      }
       if (a.alibi || need_mask) {
 #pragma unroll
         for (int t = 0; t < 2; ++t)
@@ -165,7 +215,7 @@ __global__ void __launch_bounds__(NTHR, Cfg<D>::OCC) paged_prefill_kernel(PagedA
           for (int r = 0; r < 16; ++r) {
             const int key = k0 + t * 32 + (r & 3) + 8 * (r >> 2) + 4 * h;
             float v = fmaf(slope, (float)(key - pos_lane), s[t][r]);
-            if (key >= Skv || key > pos_lane || (a.window > 0 && key <= pos_lane - a.window)) v = -INFINITY;
+            if (key >= Skv || key > pos_lane || key < lo_lane) v = -INFINITY;
             s[t][r] = v;
           }
       }
@@ -212,6 +262,15 @@ __global__ void __launch_bounds__(NTHR, Cfg<D>::OCC) paged_prefill_kernel(PagedA
         for (int ss = 0; ss < 2; ++ss)
 #pragma unroll
           for (int e = 0; e < 8; ++e) pa[t][ss][e] = (bf16)s[t][8 * ss + e];
+      bf16x8_t pl[2][2];  // what the bf16 weights leave out
+      if constexpr (EXT) {
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+          for (int ss = 0; ss < 2; ++ss)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) pl[t][ss][e] = (bf16)(s[t][8 * ss + e] - (float)pa[t][ss][e]);
+      }
       const int gq = (lane >> 2) & 3, gch = (lane >> 1) & 1, gb = 8 * (lane & 1), colhalf = (lane >> 4) & 1;
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) {
@@ -222,14 +281,17 @@ __global__ void __launch_bounds__(NTHR, Cfg<D>::OCC) paged_prefill_kernel(PagedA
           for (int ss = 0; ss < 2; ++ss) {
             const int rb = t * 32 + 16 * ss + 4 * h;
             const s16x4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                (__attribute__((address_space(3))) s16x4_t*)(Vt + lds_off<ROWB>(rb + gq, ch0) + gb));
+                (__attribute__((address_space(3))) s16x4_t*)(Vt + lds_off<RV>(rb + gq, ch0) + gb));
             const s16x4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                (__attribute__((address_space(3))) s16x4_t*)(Vt + lds_off<ROWB>(rb + 8 + gq, ch0) + gb));
+                (__attribute__((address_space(3))) s16x4_t*)(Vt + lds_off<RV>(rb + 8 + gq, ch0) + gb));
             s16x8 vv;
 #pragma unroll
             for (int e = 0; e < 4; ++e) { vv[e] = lo[e]; vv[4 + e] = hi[e]; }
             o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pa[t][ss], __builtin_bit_cast(bf16x8_t, vv), o[dt], 0,
                                                            0, 0);
+            if constexpr (EXT)
+              o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pl[t][ss], __builtin_bit_cast(bf16x8_t, vv), o[dt], 0, 0,
+                                                             0);
           }
       }
     }
@@ -253,23 +315,24 @@ __global__ void __launch_bounds__(NTHR, Cfg<D>::OCC) paged_prefill_kernel(PagedA
   for (int r = 0; r < 16; ++r) {
     const int qi = q0w + (r & 3) + 8 * (r >> 2) + 4 * h;
     if (qi < n) {
-      bf16* orow = a.o + ((int64_t)(t0 + qi) * a.Hq + hq) * D + l32;
+      bf16* orow = a.o + ((int64_t)(t0 + qi) * a.Hq + hq) * dv + l32;
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt)
-        if (D % 32 == 0 || dt * 32 + l32 < D) orow[dt * 32] = (bf16)(o[dt][r] * iv[r]);
+        if ((!EXT && DV % 32 == 0) || dt * 32 + l32 < dv) orow[dt * 32] = (bf16)(o[dt][r] * iv[r]);
     }
   }
 }
 
-template <int D>
+template <int DK, int DV, bool EXT>
 int launch(const PagedArgs& a, int nwork, hipStream_t st) {
+  constexpr int LDS = Cfg<DK, DV>::LDS_BYTES;
   static bool attr = false;
   if (!attr) {
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&paged_prefill_kernel<D>),
-                              hipFuncAttributeMaxDynamicSharedMemorySize, Cfg<D>::LDS_BYTES);
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&paged_prefill_kernel<DK, DV, EXT>),
+                              hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
     attr = true;
   }
-  hipLaunchKernelGGL((paged_prefill_kernel<D>), dim3(nwork * a.Hq), dim3(NTHR), Cfg<D>::LDS_BYTES, st, a);
+  hipLaunchKernelGGL((paged_prefill_kernel<DK, DV, EXT>), dim3(nwork * a.Hq), dim3(NTHR), LDS, st, a);
   DS_CHECK_LAUNCH();
   return 0;
 }
@@ -286,13 +349,43 @@ extern "C" int ds_paged_prefill(const void* q, const void* kc, const void* vc, v
   if (nwork <= 0) return 0;
   if (Hk <= 0 || Hq % Hk || BS <= 0 || max_blocks <= 0 || scale <= 0.f) return (int)hipErrorInvalidValue;
   PagedArgs a{(const bf16*)q, (const bf16*)kc, (const bf16*)vc, (bf16*)o, block_table, start, cu_q, work, alibi,
-              Hq, Hk, BS, max_blocks, window, scale * 1.4426950408889634f, 1.f / scale};
+              Hq, Hk, BS, max_blocks, window, scale * 1.4426950408889634f, 1.f / scale, D, D, 0, 0.f, 0.f};
   switch (D) {
-    case 64: return launch<64>(a, nwork, st);
-    case 80: return launch<80>(a, nwork, st);
-    case 96: return launch<96>(a, nwork, st);
-    case 128: return launch<128>(a, nwork, st);
-    case 256: return launch<256>(a, nwork, st);
+    case 64: return launch<64, 64, false>(a, nwork, st);
+    case 80: return launch<80, 80, false>(a, nwork, st);
+    case 96: return launch<96, 96, false>(a, nwork, st);
+    case 128: return launch<128, 128, false>(a, nwork, st);
+    case 256: return launch<256, 256, false>(a, nwork, st);
     default: return (int)hipErrorInvalidValue;
   }
+}
+
+// Key width dk and value width dv (multiples of 8 up to 256) of their own, chunked and / or windowed visibility,
+// optional score cap: score = softcap * tanh(scale * q.k / softcap).
+extern "C" int ds_paged_prefill_ext(const void* q, const void* kc, const void* vc, void* o, const int* block_table,
+                                    const int* start, const int* cu_q, const int* work, int nwork, int Hq, int Hk, int dk,
+                                    int dv, int BS, int max_blocks, int window, int chunk, float scale, float softcap,
+                                    hipStream_t st) {
+  if (nwork <= 0) return 0;
+  if (Hk <= 0 || Hq % Hk || BS <= 0 || max_blocks <= 0 || scale <= 0.f || dk % 8 || dv % 8 || dk <= 0 || dv <= 0)
+    return (int)hipErrorInvalidValue;
+  constexpr float LOG2E = 1.4426950408889634f;
+  const bool cap = softcap > 0.f;
+  // with a cap the scores leave the capping step in log2 units already
+  PagedArgs a{(const bf16*)q, (const bf16*)kc, (const bf16*)vc, (bf16*)o, block_table, start, cu_q, work, nullptr,
+              Hq, Hk, BS, max_blocks, window, cap ? 1.f : scale * LOG2E, 1.f / scale, dk, dv, chunk,
+              cap ? scale / softcap * 2.f * LOG2E : 0.f, cap ? softcap * LOG2E : 0.f};
+#define DS_ROW(K)                                              \
+  {                                                            \
+    if (dv <= 32) return launch<K, 32, true>(a, nwork, st);    \
+    if (dv <= 64) return launch<K, 64, true>(a, nwork, st);    \
+    if (dv <= 128) return launch<K, 128, true>(a, nwork, st);  \
+    if (dv <= 256) return launch<K, 256, true>(a, nwork, st);  \
+  }
+  if (dk <= 32) DS_ROW(32)
+  else if (dk <= 64) DS_ROW(64)
+  else if (dk <= 128) DS_ROW(128)
+  else if (dk <= 256) DS_ROW(256)
+#undef DS_ROW
+  return (int)hipErrorInvalidValue;
 }

@@ -19,6 +19,15 @@ int ds_delta_prepare(const void*, const float*, const void*, const float*, const
                      const int*, const int*, float*, void*, float*, int, int, int, int, int, int, int, hipStream_t);
 int ds_delta_recur(const float*, const void*, const float*, const void*, const float*, float, float*, void*, const int*,
                    int, const int*, const int*, const int*, void*, int, int, int, int, int, int, hipStream_t);
+int64_t ds_delta_chunk_ws(int, int, int, int);
+int ds_delta_chunk(const float*, const void*, const float*, const void*, const float*, float, float*, void*, const int*,
+                   int, const int*, int, const int*, const int*, const int*, float*, float*, void*, int, int, int, int,
+                   int, int, hipStream_t);
+int ds_paged_prefill_ext(const void*, const void*, const void*, void*, const int*, const int*, const int*, const int*, int,
+                         int, int, int, int, int, int, int, int, float, float, hipStream_t);
+int ds_paged_decode_splits(int, int, int);
+int ds_paged_decode_ext(const void*, const void*, const void*, const int*, const int*, float*, float*, void*, int, int,
+                        int, int, int, int, int, int, int, float, float, int, int, hipStream_t);
 int ds_skinny_gemm(const void*, const void*, const void*, const void*, const void*, const void*, void*, void*, int, int,
                    int, int, int, int, float, hipStream_t);
 int ds_skinny_mfma_ok(int, int, int);
@@ -155,6 +164,56 @@ Tensor paged_generic(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor 
   return o;
 }
 
+bool paged_tiled_ok(int64_t dk, int64_t dv) { return dk % 8 == 0 && dv % 8 == 0 && dk <= 256 && dv <= 256; }
+
+// Prompts and portions: q [T, H, dk] bf16 of every new token; work [n, 2] names (sequence, 128-row block) -> o [T, H, dv]
+// (rows of sequences the list leaves out are not written).
+Tensor paged_prefill(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor start, Tensor cu_q, Tensor work,
+                     double scale, double softcap, int64_t window, int64_t chunk) {
+  need(q, "q"); need(block_table, "block_table");
+  const Cache c = cache_of(kc, vc);
+  const int64_t T = q.size(0), H = q.size(1), S = start.numel();
+  TORCH_CHECK(q.dim() == 3 && q.size(2) == c.dk && H % c.G == 0 && q.scalar_type() == at::kBFloat16 &&
+              kc.scalar_type() == at::kBFloat16 && paged_tiled_ok(c.dk, c.dv), "paged_prefill: q / caches");
+  TORCH_CHECK(block_table.dim() == 2 && block_table.size(0) == S && block_table.scalar_type() == at::kInt, "block_table");
+  TORCH_CHECK(work.dim() == 2 && work.size(1) == 2 && scale > 0, "paged_prefill: work [n, 2], scale > 0");
+  auto o = torch::empty({T, H, c.dv}, q.options());
+  check(ds_paged_prefill_ext(q.data_ptr(), kc.data_ptr(), vc.data_ptr(), o.data_ptr(), block_table.data_ptr<int>(),
+                             i32(start, S, "start"), i32(cu_q, S + 1, "cu_q"), i32(work, work.numel(), "work"),
+                             (int)work.size(0), (int)H, c.G, c.dk, c.dv, c.BS, (int)block_table.size(1), (int)window,
+                             (int)chunk, (float)scale, (float)softcap, stream()), "paged_prefill");
+  return o;
+}
+
+// One new token per sequence: q [B, H, dk] bf16, the first B rows of the tables -> out[:B] of [.., H, dv]
+void paged_decode(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor seq_lens, int64_t max_len, double scale,
+                  double softcap, int64_t window, int64_t chunk, Tensor out) {
+  need(q, "q"); need(block_table, "block_table"); need(out, "out");
+  const Cache c = cache_of(kc, vc);
+  const int64_t B = q.size(0), H = q.size(1);
+  TORCH_CHECK(q.dim() == 3 && q.size(2) == c.dk && H % c.G == 0 && q.scalar_type() == at::kBFloat16 &&
+              kc.scalar_type() == at::kBFloat16 && paged_tiled_ok(c.dk, c.dv), "paged_decode: q / caches");
+  TORCH_CHECK(block_table.dim() == 2 && block_table.size(0) >= B && block_table.scalar_type() == at::kInt &&
+              block_table.size(1) * c.BS >= max_len, "block_table");
+  TORCH_CHECK(out.dim() == 3 && out.size(0) >= B && out.size(1) == H && out.size(2) == c.dv &&
+              out.scalar_type() == at::kBFloat16, "paged_decode: out");
+  int64_t span = max_len;
+  if (window > 0) span = std::min(span, window);
+  if (chunk > 0) span = std::min(span, chunk);
+  const int splits = ds_paged_decode_splits((int)B, c.G, (int)span);
+  Tensor acc, ml;
+  if (splits > 1) {
+    auto fo = q.options().dtype(at::kFloat);
+    acc = torch::empty({B, H, splits, c.dv}, fo);
+    ml = torch::empty({B, H, splits, 2}, fo);
+  }
+  check(ds_paged_decode_ext(q.data_ptr(), kc.data_ptr(), vc.data_ptr(), block_table.data_ptr<int>(),
+                            i32(seq_lens, seq_lens.numel(), "seq_lens"), splits > 1 ? acc.data_ptr<float>() : nullptr,
+                            splits > 1 ? ml.data_ptr<float>() : nullptr, out.data_ptr(), (int)B, (int)H, c.G, c.dk, c.dv,
+                            c.BS, (int)block_table.size(1), (int)span, splits, (float)scale, (float)softcap, (int)window,
+                            (int)chunk, stream()), "paged_decode");
+}
+
 void delta_dims_ok(int64_t Hk, int64_t H, int64_t dk, int64_t dv, int64_t taps) {
   TORCH_CHECK(Hk > 0 && H % Hk == 0 && dk > 0 && dv > 0 && taps >= 1, "delta rule: head counts / sizes");
   TORCH_CHECK(dk <= 256 && dv <= 256, "delta rule: head sizes up to 256");
@@ -203,6 +262,33 @@ void delta_recur(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, dou
                        stream()), "delta_recur");
 }
 
+// The same for long portions, by chunks of 64 tokens: seqs [n, 2] (sequence, its first entry in work), work [m, 2]
+// (sequence, chunk).
+void delta_chunk(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, double eps, Tensor state, Tensor conv_state,
+                 Tensor seqs, Tensor work, Tensor cu, Tensor start, Tensor slots, Tensor out) {
+  need(proj, "proj"); need(v, "v"); need(state, "state"); need(conv_state, "conv_state"); need(out, "out");
+  const int64_t T = v.size(0), H = v.size(1), dv = v.size(2), Hk = qk.size(2), dk = qk.size(3), S = start.numel();
+  const int64_t taps = conv_state.size(1) + 1;
+  delta_dims_ok(Hk, H, dk, dv, taps);
+  TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == H && state.size(2) == dk &&
+              state.size(3) == dv && state.size(0) == conv_state.size(0), "delta: state [slots, H, dk, dv] fp32");
+  TORCH_CHECK(conv_state.size(2) == 2 * Hk * dk + H * dv, "delta: conv_state");
+  TORCH_CHECK(proj.numel() == T * (2 * Hk * dk + 2 * H * dv + 2 * H) && out.numel() == T * H * dv, "delta: proj / out");
+  TORCH_CHECK(v.scalar_type() == proj.scalar_type() && out.scalar_type() == proj.scalar_type() &&
+              conv_state.scalar_type() == proj.scalar_type(), "delta: types");
+  TORCH_CHECK(seqs.dim() == 2 && seqs.size(1) == 2 && work.dim() == 2 && work.size(1) == 2, "delta_chunk: lists");
+  const int64_t nw = work.size(0);
+  auto fo = proj.options().dtype(at::kFloat);
+  auto ws = torch::empty({ds_delta_chunk_ws((int)nw, (int)H, (int)dk, (int)dv)}, fo);
+  auto o = torch::empty({T, H, dv}, fo);
+  check(ds_delta_chunk(f32(qk, T * 2 * Hk * dk, "qk"), v.data_ptr(), f32(gb, T * 2 * H, "gb"), proj.data_ptr(),
+                       f32(norm_w, dv, "norm"), (float)eps, state.data_ptr<float>(), conv_state.data_ptr(),
+                       i32(seqs, seqs.numel(), "seqs"), (int)seqs.size(0), i32(work, work.numel(), "work"), (int)nw,
+                       i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"), ws.data_ptr<float>(),
+                       o.data_ptr<float>(), out.data_ptr(), (int)Hk, (int)H, (int)dk, (int)dv, (int)taps, dcode(proj),
+                       stream()), "delta_chunk");
+}
+
 bool decode_linear_ok(int64_t M, int64_t K) {
   return M >= 1 && K % 8 == 0 && (M <= 8 || (M <= 16 && ds_skinny_mfma_ok((int)M, (int)K, 0)));
 }
@@ -231,6 +317,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("paged_generic", &paged_generic);
   m.def("delta_prepare", &delta_prepare);
   m.def("delta_recur", &delta_recur);
+  m.def("delta_chunk", &delta_chunk);
+  m.def("paged_tiled_ok", &paged_tiled_ok);
+  m.def("paged_prefill", &paged_prefill);
+  m.def("paged_decode", &paged_decode);
   m.def("decode_linear", &decode_linear);
   m.def("decode_linear_ok", &decode_linear_ok);
 }

@@ -80,7 +80,8 @@ Tensor paged_decode(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor s
   TORCH_CHECK(kc.size(3) == D, "head dim mismatch");
   const int max_blocks = (int)block_table.size(1);
   TORCH_CHECK((int64_t)max_blocks * BS >= max_len, "block table too small for max_len");
-  const int splits = ds_paged_decode_splits(B, Hk, (int)max_len);
+  const int64_t span = window > 0 && window < max_len ? window : max_len;  // keys in sight
+  const int splits = ds_paged_decode_splits(B, Hk, (int)span);
   auto out = torch::empty_like(q);
   auto fo = q.options().dtype(at::kFloat);
   Tensor pacc, pml;

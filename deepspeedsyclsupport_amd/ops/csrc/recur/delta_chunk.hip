@@ -1,0 +1,314 @@
+// Gated delta rule over long portions, by chunks of 64 tokens (CDNA4, gfx950). See delta_rule.hip for the recurrence.
+//
+// With the running log decay G_i of a chunk (its first token included) and the state S0 the chunk starts from, unrolling
+// the recurrence gives
+//     (I + A) U = diag(beta) (V - diag(e^G) K S0),        A_ij = beta_i e^{G_i - G_j} (k_i . k_j),  j < i
+//     o_i = e^{G_i} S0^T q_i + sum_{j <= i} P_ij u_j,      P_ij = e^{G_i - G_j} (q_i . k_j)
+//     S   = e^{G_C} S0 + sum_j e^{G_C - G_j} k_j u_j^T
+//  * chunk kernel: one workgroup per (chunk, head), all chunks of all sequences at once. K K^T and Q K^T on the fp32
+//    matrix cores, then W = (I + A)^-1 diag(beta e^G) K and X = (I + A)^-1 diag(beta) V by forward substitution, one
+//    column per thread with the 64 unknowns in registers. Writes W, X, P and the decays.
+//  * scan kernel: one workgroup per (sequence, head, 16 value columns) walks the chunks: U = X - W S0, the read-out and
+//    the next state are products of 16 x 16 tiles on the fp32 matrix cores; the state tile stays in LDS.
+//  * norm kernel: per-head RMS norm and gate of the read-out.
+// Everything is fp32: v_mfma_f32_16x16x4_f32 has the precision of the vector unit. The chunk borders are counted from
+// the portion's first token; where they fall changes rounding only. Log decays are summed in fp64: only differences
+// enter, and a strong decay early in a chunk must not cost the later ones their digits.
+#include "delta_rule.h"
+
+namespace {
+
+constexpr int C = 64;
+constexpr int NT = 256;
+
+__device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+}
+
+// 4 consecutive elements of a row of d, zero beyond its end
+__device__ __forceinline__ f32x4 load4(const float* row, int k, int d) {
+  if ((d & 3) == 0) return k < d ? *reinterpret_cast<const f32x4*>(row + k) : f32x4{0.f, 0.f, 0.f, 0.f};
+  f32x4 v;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) v[e] = k + e < d ? row[k + e] : 0.f;
+  return v;
+}
+
+template <typename T>
+__global__ void __launch_bounds__(NT) delta_chunk_kernel(
+    const float* __restrict__ qk, const T* __restrict__ v, const float* __restrict__ gb, const int* __restrict__ cu,
+    const int* __restrict__ work, float* __restrict__ Wo, float* __restrict__ Xo, float* __restrict__ Po,
+    float* __restrict__ dec, DeltaDims D) {
+  __shared__ __attribute__((aligned(16))) float A[C][C + 4];
+  __shared__ double G[C];
+  __shared__ float beta[C];
+  const int h = blockIdx.x % D.H, ci = blockIdx.x / D.H, hk = h / (D.H / D.Hk);
+  const int seq = work[2 * ci], c = work[2 * ci + 1];
+  const int t0 = cu[seq] + c * C, n = min(C, cu[seq + 1] - t0);
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, l16 = lane & 15, q4 = lane >> 4;
+  const int64_t base = (int64_t)ci * D.H + h;
+  if (w == 0) {
+    double g = lane < n ? (double)gb[((int64_t)(t0 + lane) * 2) * D.H + h] : 0.0;
+    for (int o = 1; o < 64; o <<= 1) {
+      const double p = __shfl_up(g, o, 64);
+      if (lane >= o) g += p;
+    }
+    G[lane] = g;
+    beta[lane] = lane < n ? gb[((int64_t)(t0 + lane) * 2 + 1) * D.H + h] : 0.f;
+    const double gc = __shfl(g, 63, 64);  // rows beyond n add nothing
+    dec[base * 2 * C + lane] = expf((float)g);
+    dec[base * 2 * C + C + lane] = expf((float)(gc - g));
+  }
+  __syncthreads();
+  // ---- K K^T and Q K^T, lower triangle of 16 x 16 tiles; wave w owns row tile w
+  const float* kbase = qk + (int64_t)D.Hk * D.dk + (int64_t)hk * D.dk;
+  const float* qbase = qk + (int64_t)hk * D.dk;
+  const int64_t rs = (int64_t)2 * D.Hk * D.dk;  // row stride of qk
+  const int64_t ri = (int64_t)(t0 + min(w * 16 + l16, n - 1)) * rs;
+  for (int jt = 0; jt < 4; ++jt) {
+    f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qq = {0.f, 0.f, 0.f, 0.f};
+    if (jt <= w) {
+      const int64_t rj = (int64_t)(t0 + min(jt * 16 + l16, n - 1)) * rs;
+      for (int k = 4 * q4; k < ((D.dk + 15) & ~15); k += 16) {
+        const f32x4 a = load4(kbase + ri, k, D.dk), q = load4(qbase + ri, k, D.dk), b = load4(kbase + rj, k, D.dk);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          kk = mfma4(a[e], b[e], kk);
+          qq = mfma4(q[e], b[e], qq);
+        }
+      }
+    }
+    float* prow = Po + base * C * C;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = w * 16 + 4 * q4 + r, j = jt * 16 + l16;
+      const float d = j <= i ? expf((float)(G[i] - G[j])) : 0.f;
+      A[i][j] = j < i && i < n ? beta[i] * d * kk[r] : 0.f;
+      prow[i * C + j] = j <= i && i < n ? d * qq[r] : 0.f;
+    }
+  }
+  __syncthreads();
+  // ---- forward substitution: column col of [W | X]
+  for (int col = tid; col < D.dk + D.dv; col += NT) {
+    const bool isw = col < D.dk;
+    float x[C];
+#pragma unroll
+    for (int i = 0; i < C; ++i) {
+      float r = 0.f;
+      if (i < n) {
+        const int64_t t = t0 + i;
+        if (isw) r = kbase[t * rs + col] * expf((float)G[i]);
+        else r = (float)v[(t * D.H + h) * D.dv + col - D.dk];
+        r *= beta[i];
+      }
+      x[i] = r;
+    }
+#pragma unroll
+    for (int i = 1; i < C; ++i) {
+      asm volatile("" ::: "memory");  // one row of A at a time: hoisting them all costs the registers x needs
+#pragma unroll
+      for (int j = 0; j < (i + 3) / 4; ++j) {  // entries at and right of the diagonal are zero
+        const f32x4 a = *reinterpret_cast<const f32x4*>(&A[i][4 * j]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (4 * j + e < i) x[i] = fmaf(-a[e], x[4 * j + e], x[i]);
+      }
+    }
+    float* dst = isw ? Wo + base * C * D.dk + col : Xo + base * C * D.dv + col - D.dk;
+    const int ld = isw ? D.dk : D.dv;
+#pragma unroll
+    for (int i = 0; i < C; ++i) dst[i * ld] = x[i];
+  }
+}
+
+// NK: 16-wide tiles of the key width (rounded up)
+template <typename T, int NK>
+__global__ void __launch_bounds__(NT) delta_scan_kernel(
+    const float* __restrict__ qk, const T* __restrict__ proj, const float* __restrict__ Wo, const float* __restrict__ Xo,
+    const float* __restrict__ Po, const float* __restrict__ dec, const int* __restrict__ seqs, const int* __restrict__ cu,
+    const int* __restrict__ start, const int* __restrict__ slots, float* __restrict__ state, T* __restrict__ conv_state,
+    float* __restrict__ o, DeltaDims D) {
+  __shared__ float S[NK * 16][17];
+  __shared__ float U[C][17];
+  const int vt = blockIdx.x, h = blockIdx.y, seq = seqs[2 * blockIdx.z], first = seqs[2 * blockIdx.z + 1];
+  const int hk = h / (D.H / D.Hk), tid = threadIdx.x, lane = tid & 63, w = tid >> 6, l16 = lane & 15, q4 = lane >> 4;
+  const int t0 = cu[seq], n = cu[seq + 1] - t0, nc = (n + C - 1) / C, v0 = vt * 16;
+  const bool fresh = start[seq] == 0;
+  float* st = state + ((int64_t)slots[seq] * D.H + h) * D.dk * D.dv;
+  for (int i = tid; i < NK * 256; i += NT) {
+    const int k = i / 16, j = i % 16;
+    S[k][j] = (!fresh && k < D.dk && v0 + j < D.dv) ? st[(int64_t)k * D.dv + v0 + j] : 0.f;
+  }
+  const int64_t rs = (int64_t)2 * D.Hk * D.dk;
+  const float* qbase = qk + (int64_t)hk * D.dk;
+  const float* kbase = qbase + (int64_t)D.Hk * D.dk;
+  constexpr int KT = (NK + 3) / 4;  // key tiles of the state per wave
+  f32x4 wf[NK], qf[NK], pf[4];
+  float kf[KT][16], xf[4], dq[4], du[4], dc = 0.f;
+  auto fetch = [&](int c) {
+    const int64_t base = (int64_t)(first + c) * D.H + h;
+    const int row = w * 16 + l16, last = t0 + n - 1, tc = t0 + c * C;
+    const float* wr = Wo + (base * C + row) * D.dk;
+    const float* qr = qbase + (int64_t)min(tc + row, last) * rs;
+#pragma unroll
+    for (int kk = 0; kk < NK; ++kk) {
+      wf[kk] = load4(wr, 16 * kk + 4 * q4, D.dk);
+      qf[kk] = load4(qr, 16 * kk + 4 * q4, D.dk);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = w * 16 + 4 * q4 + r;
+      xf[r] = v0 + l16 < D.dv ? Xo[(base * C + i) * D.dv + v0 + l16] : 0.f;
+      dq[r] = dec[base * 2 * C + i];
+      du[r] = dec[base * 2 * C + C + i];
+      pf[r] = *reinterpret_cast<const f32x4*>(Po + (base * C + row) * C + 16 * r + 4 * q4);
+    }
+    dc = dec[base * 2 * C + C - 1];
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) {
+      const int d = (w + 4 * kt) * 16 + l16;
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {  // k index of the product: token 16 (i / 4) + 4 q4 + i % 4
+        const int tok = min(tc + 16 * (i >> 2) + 4 * q4 + (i & 3), last);
+        kf[kt][i] = d < D.dk ? kbase[(int64_t)tok * rs + d] : 0.f;
+      }
+    }
+  };
+  fetch(0);
+  __syncthreads();
+  for (int c = 0; c < nc; ++c) {
+    f32x4 u = {0.f, 0.f, 0.f, 0.f}, oq = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int kk = 0; kk < NK; ++kk)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float s = S[16 * kk + 4 * q4 + e][l16];
+        u = mfma4(wf[kk][e], s, u);
+        oq = mfma4(qf[kk][e], s, oq);
+      }
+    f32x4 uu, acc;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      uu[r] = xf[r] - u[r];
+      acc[r] = dq[r] * oq[r];
+      U[w * 16 + 4 * q4 + r][l16] = uu[r];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int jt = 0; jt < 4; ++jt) {
+      if (jt > w) break;  // P is lower triangular
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc = mfma4(pf[jt][e], U[16 * jt + 4 * q4 + e][l16], acc);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = c * C + w * 16 + 4 * q4 + r;
+      if (i < n && v0 + l16 < D.dv) o[((int64_t)(t0 + i) * D.H + h) * D.dv + v0 + l16] = acc[r];
+    }
+    __syncthreads();
+    // U <- e^{G_C - G_i} U for the state update (every wave its own rows)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) U[w * 16 + 4 * q4 + r][l16] = uu[r] * du[r];
+    __syncthreads();
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) {
+      const int d0 = (w + 4 * kt) * 16;
+      if (w + 4 * kt < NK) {
+        f32x4 s;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s[r] = dc * S[d0 + 4 * q4 + r][l16];
+#pragma unroll
+        for (int i = 0; i < 16; ++i) s = mfma4(kf[kt][i], U[16 * (i >> 2) + 4 * q4 + (i & 3)][l16], s);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) S[d0 + 4 * q4 + r][l16] = s[r];
+      }
+    }
+    if (c + 1 < nc) fetch(c + 1);
+    __syncthreads();
+  }
+  for (int i = tid; i < D.dk * 16; i += NT) {
+    const int k = i / 16, j = i % 16;
+    if (v0 + j < D.dv) st[(int64_t)k * D.dv + v0 + j] = S[k][j];
+  }
+  if (vt == 0 && D.taps > 1)
+    advance_head(conv_state + (int64_t)slots[seq] * (D.taps - 1) * D.channels(), proj, t0, n, D, fresh, h);
+}
+
+// out = o / rms(o) * w * silu(gate), one wave per (token, head) of the long sequences' chunks
+template <typename T>
+__global__ void __launch_bounds__(NT) delta_norm_kernel(const float* __restrict__ o, const T* __restrict__ proj,
+                                                        const float* __restrict__ norm_w, float eps,
+                                                        const int* __restrict__ cu, const int* __restrict__ work,
+                                                        T* __restrict__ out, DeltaDims D) {
+  const int h = blockIdx.x % D.H, ci = blockIdx.x / D.H, lane = threadIdx.x & 63;
+  const int seq = work[2 * ci], t0 = cu[seq] + work[2 * ci + 1] * C, n = min(C, cu[seq + 1] - t0);
+  for (int i = threadIdx.x >> 6; i < n; i += NT / 64) {
+    const int64_t t = t0 + i, at = (t * D.H + h) * D.dv;
+    const T* gate = proj + t * D.row() + D.channels() + h * D.dv;
+    float x[4], ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const int c = k * 64 + lane;
+      x[k] = c < D.dv ? o[at + c] : 0.f;
+      ss = fmaf(x[k], x[k], ss);
+    }
+    const float rms = 1.f / sqrtf(wave_sum(ss) / (float)D.dv + eps);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const int c = k * 64 + lane;
+      if (c < D.dv) out[at + c] = (T)(x[k] * rms * norm_w[c] * silu((float)gate[c]));
+    }
+  }
+}
+
+template <typename T>
+int run(const float* qk, const void* v, const float* gb, const void* proj, const float* norm_w, float eps, float* state,
+        void* conv_state, const int* seqs, int nseq, const int* work, int nwork, const int* cu, const int* start,
+        const int* slots, float* ws, float* o, void* out, DeltaDims D, hipStream_t st) {
+  float* W = ws;
+  float* X = W + (int64_t)nwork * D.H * C * D.dk;
+  float* P = X + (int64_t)nwork * D.H * C * D.dv;
+  float* dec = P + (int64_t)nwork * D.H * C * C;
+  hipLaunchKernelGGL((delta_chunk_kernel<T>), dim3(nwork * D.H), dim3(NT), 0, st, qk, (const T*)v, gb, cu, work, W, X, P,
+                     dec, D);
+  DS_CHECK_LAUNCH();
+  const dim3 grid((D.dv + 15) / 16, D.H, nseq);
+#define GO(NK)                                                                                                       \
+  hipLaunchKernelGGL((delta_scan_kernel<T, NK>), grid, dim3(NT), 0, st, qk, (const T*)proj, W, X, P, dec, seqs, cu, start, \
+                     slots, state, (T*)conv_state, o, D)
+  if (D.dk <= 32) GO(2);
+  else if (D.dk <= 64) GO(4);
+  else if (D.dk <= 128) GO(8);
+  else GO(16);
+#undef GO
+  DS_CHECK_LAUNCH();
+  hipLaunchKernelGGL((delta_norm_kernel<T>), dim3(nwork * D.H), dim3(NT), 0, st, o, (const T*)proj, norm_w, eps, cu, work,
+                     (T*)out, D);
+  DS_CHECK_LAUNCH();
+  return 0;
+}
+
+}  // namespace
+
+// fp32 words of workspace a call needs
+extern "C" int64_t ds_delta_chunk_ws(int nwork, int H, int dk, int dv) {
+  return (int64_t)nwork * H * C * (dk + dv + C + 2);
+}
+
+// seqs [nseq, 2]: (sequence, index of its first entry in work); work [nwork, 2]: (sequence, chunk), a sequence's chunks
+// in order. o: fp32 [tokens, H, dv] scratch.
+extern "C" int ds_delta_chunk(const float* qk, const void* v, const float* gb, const void* proj, const float* norm_w,
+                              float eps, float* state, void* conv_state, const int* seqs, int nseq, const int* work,
+                              int nwork, const int* cu, const int* start, const int* slots, float* ws, float* o,
+                              void* out, int Hk, int H, int dk, int dv, int taps, int dtype, hipStream_t st) {
+  if (nseq <= 0 || nwork <= 0) return 0;
+  const DeltaDims D{Hk, H, dk, dv, taps};
+  if (!dims_ok(D) || H > 65535 || nseq > 65535) return (int)hipErrorInvalidValue;
+  if (dtype == DS_F32)
+    return run<float>(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, nseq, work, nwork, cu, start, slots, ws, o,
+                      out, D, st);
+  if (dtype == DS_BF16)
+    return run<bf16>(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, nseq, work, nwork, cu, start, slots, ws, o, out,
+                     D, st);
+  return (int)hipErrorInvalidValue;
+}

@@ -15,17 +15,9 @@
 //    while the portion's tokens pass one by one: decoding and short portions. It also moves the convolution's window
 //    on in the state slot (prepare, which reads the old one, has finished by then).
 // A sequence whose portion starts at position 0 starts from zero: slots need no clearing between owners.
-#include "ds_hip.h"
+#include "delta_rule.h"
 
 namespace {
-
-__device__ __forceinline__ float silu(float x) { return x / (1.f + expf(-x)); }
-
-struct DeltaDims {
-  int Hk, H, dk, dv, taps;
-  __host__ __device__ int channels() const { return 2 * Hk * dk + H * dv; }
-  __host__ __device__ int row() const { return channels() + H * dv + 2 * H; }
-};
 
 template <typename T>
 __global__ void __launch_bounds__(256) delta_prepare_kernel(
@@ -85,31 +77,6 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(
     const int c = i * 64 + lane;
     if (c < width) dst[c] = vals[i] * r;
   }
-}
-
-// Window of one channel: the last taps-1 inputs of [old window | the portion's inputs].
-template <typename T>
-__device__ __forceinline__ void advance_window(T* cs, const T* proj, int64_t t0, int n, int NP, int C, int taps, bool fresh,
-                                               int c) {
-  for (int j = 0; j < taps - 1; ++j) {
-    const int src = n + j;  // index in [old (taps-1) | new (n)]
-    T x = (T)0.f;
-    if (src >= taps - 1) x = proj[(t0 + src - (taps - 1)) * NP + c];
-    else if (!fresh) x = cs[(int64_t)src * C + c];
-    cs[(int64_t)j * C + c] = x;  // ascending: src > j, so nothing is overwritten before it is read
-  }
-}
-
-// Convolution windows of head h's own channels (its values, and the group's q / k if it is the group's first head).
-template <typename T>
-__device__ __forceinline__ void advance_head(T* cs, const T* proj, int64_t t0, int n, const DeltaDims& D, bool fresh, int h) {
-  const int NP = D.row(), C = D.channels(), rep = D.H / D.Hk;
-  for (int c = threadIdx.x; c < D.dv; c += blockDim.x)
-    advance_window(cs, proj, t0, n, NP, C, D.taps, fresh, 2 * D.Hk * D.dk + h * D.dv + c);
-  if (h % rep == 0)
-    for (int c = threadIdx.x; c < 2 * D.dk; c += blockDim.x)
-      advance_window(cs, proj, t0, n, NP, C, D.taps, fresh,
-                     (c < D.dk ? 0 : (D.Hk - 1) * D.dk) + (h / rep) * D.dk + c);
 }
 
 template <typename T, int E>
@@ -178,10 +145,6 @@ __global__ void __launch_bounds__(1024) delta_recur_kernel(
     }
   }
   if (D.taps > 1) advance_head(conv_state + (int64_t)slots[seq] * (D.taps - 1) * C, proj, t0, n, D, fresh, h);
-}
-
-bool dims_ok(const DeltaDims& D) {
-  return D.Hk > 0 && D.H > 0 && D.H % D.Hk == 0 && D.dk > 0 && D.dv > 0 && D.dk <= 256 && D.dv <= 256 && D.taps >= 1;
 }
 
 template <typename T>

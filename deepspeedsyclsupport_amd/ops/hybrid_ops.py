@@ -35,7 +35,19 @@ def ragged_attention(q, kc, vc, meta, scale, softcap=0.0, window=0, chunk=0):
     args = (meta.block_tables, meta.pos_ids, meta.seq_ids, scale, softcap, window, chunk)
     if not use_native(q):
         return reference.paged_attention(q, kc, vc, *args)
-    return hybrid_ops().paged_generic(q, kc, vc, *args)
+    ops = hybrid_ops()
+    if q.dtype != torch.bfloat16 or not ops.paged_tiled_ok(kc.shape[3], vc.shape[3]):
+        return ops.paged_generic(q, kc, vc, *args)
+    nd = meta.n_decode
+    if nd < len(meta.start_host):
+        o = ops.paged_prefill(q, kc, vc, meta.block_tables, meta.start_pos, meta.cu_q, meta.work, scale, softcap, window,
+                              chunk)
+    else:
+        o = q.new_empty(q.shape[0], q.shape[1], vc.shape[3])
+    if nd:
+        ops.paged_decode(q[:nd], kc, vc, meta.block_tables[:nd], meta.seq_lens[:nd], meta.max_len, scale, softcap, window,
+                         chunk, o)
+    return o
 
 
 def delta_rule(proj, conv_w, a_log, dt_bias, norm_w, eps, state, conv_state, meta, Hk, H, dk, dv):
@@ -44,8 +56,12 @@ def delta_rule(proj, conv_w, a_log, dt_bias, norm_w, eps, state, conv_state, met
     ops = hybrid_ops() if use_native(proj) else reference
     qk, v, gb = ops.delta_prepare(proj, conv_w, conv_state, a_log, dt_bias, meta.seq_ids, meta.cu_q, meta.start_pos,
                                   meta.slots, Hk, H, dk, dv)
-    for seqs in (meta.seq_list, meta.chunk_seqs):
-        ops.delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, meta.cu_q, meta.start_pos, meta.slots, out)
+    if meta.seq_list.numel():
+        ops.delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, meta.seq_list, meta.cu_q, meta.start_pos,
+                        meta.slots, out)
+    if meta.chunk_work.numel():
+        ops.delta_chunk(qk, v, gb, proj, norm_w, eps, state, conv_state, meta.chunk_seqs, meta.chunk_work, meta.cu_q,
+                        meta.start_pos, meta.slots, out)
     return out
 
 

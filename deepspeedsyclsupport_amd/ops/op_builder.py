@@ -67,7 +67,10 @@ EXTENSIONS = {
             "act/clamped_glu.hip",
             "attn/qk_norm_append.hip",
             "attn/paged_generic.hip",
+            "attn/paged_prefill.hip",
+            "attn/decode_attn.hip",
             "recur/delta_rule.hip",
+            "recur/delta_chunk.hip",
             "gemv/skinny_gemm.hip",
             "gemv/skinny_mfma.hip",
         ],

@@ -225,3 +225,8 @@ def delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, cu, start
         if taps > 1:
             old = conv_state[slot] if int(start[i]) else torch.zeros_like(conv_state[slot])
             conv_state[slot] = torch.cat([old, proj[a:b, :C]])[-(taps - 1):].clone()
+
+
+def delta_chunk(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, work, cu, start, slots, out):
+    """Long portions: the same recurrence (the device splits it into chunks)."""
+    delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs[:, 0], cu, start, slots, out)
