@@ -19,6 +19,7 @@ from ..utils.logging import log_dist
 from .config import DeepSpeedInferenceConfig
 from .model_implementations import convert
 from .model_implementations.transformer import BatchMeta, DSInferenceModel
+from .sampling import sample_tokens
 
 
 class GenerationOutput:
@@ -303,20 +304,7 @@ class InferenceEngine(torch.nn.Module):
 
     # ------------------------------------------------------------------------------------------ generate
     def _sample(self, logits, do_sample, temperature, top_k, top_p, generator):
-        if not do_sample:
-            return logits.argmax(-1)
-        logits = logits.float() / max(temperature, 1e-5)
-        if top_k and top_k > 0:
-            kth = torch.topk(logits, min(top_k, logits.shape[-1]), dim=-1).values[..., -1:]
-            logits = logits.masked_fill(logits < kth, float("-inf"))
-        if top_p is not None and top_p < 1.0:
-            srt, idx = torch.sort(logits, descending=True, dim=-1)
-            cum = srt.softmax(-1).cumsum(-1)
-            drop = cum - srt.softmax(-1) > top_p
-            srt = srt.masked_fill(drop, float("-inf"))
-            logits = torch.full_like(logits, float("-inf")).scatter(-1, idx, srt)
-        probs = logits.softmax(-1)
-        return torch.multinomial(probs, 1, generator=generator).squeeze(-1)
+        return sample_tokens(logits, do_sample, temperature, top_k, top_p, generator)
 
     def _moe_capturable(self, ids):
         """MoE layers capture only on the device routing path (the reference fallback reads counts on the host)."""

@@ -3,3 +3,4 @@ from .config_v2 import RaggedInferenceEngineConfig, DSStateManagerConfig, Memory
 from .engine_factory import build_engine_from_ds_checkpoint, build_hf_engine
 from .engine_v2 import InferenceEngineV2
 from .scheduling_utils import SchedulingError, SchedulingResult
+from .scheduler import RaggedScheduler

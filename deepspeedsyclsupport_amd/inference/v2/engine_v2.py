@@ -148,6 +148,20 @@ class InferenceEngineV2:
             return SchedulingResult.BatchTokenLimitExceeded
         return SchedulingResult.Success
 
+    @torch.no_grad()
+    def generate(self, prompts, max_new_tokens=64, eos_token_id=None, token_budget=None, do_sample=False,
+                 temperature=1.0, top_k=0, top_p=1.0, seed=None):
+        """Generate for a list of prompts (token id sequences) with continuous batching: returns the list of generated
+        ids per prompt. See `scheduler.RaggedScheduler` for adding and finishing requests as they come."""
+        from .scheduler import RaggedScheduler
+        sched = RaggedScheduler(self, token_budget, do_sample=do_sample, temperature=temperature, top_k=top_k,
+                                top_p=top_p, seed=seed)
+        for i, p in enumerate(prompts):
+            sched.add(i, p, max_new_tokens, eos_token_id)
+        while sched.pending:
+            sched.step()
+        return [sched.outputs[i] for i in range(len(prompts))]
+
     def flush(self, uid: int) -> None:
         self._state_manager.flush_sequence(uid)
 

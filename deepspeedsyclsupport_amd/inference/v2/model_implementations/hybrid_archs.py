@@ -17,13 +17,26 @@ _MIXER_TENSORS = {  # checkpoint name below `<layer>.mix.` -> canonical key
 _MLP_TENSORS = {"dense": {"gate": "gate_w", "up": "up_w", "down": "down_w"}}
 
 
-def container(name, tensors):
+class _HybridContainer(LayerContainer):
+    """A container that names every tensor it is made of: all must come, except those in `may_lack`."""
+    may_lack = ()
+
+    @property
+    def is_initialized(self):
+        return not self.missing()
+
+    def missing(self):
+        return [name for name, p in self._params.items() if not p.complete and name not in self.may_lack]
+
+
+def container(name, tensors, may_lack=()):
     """A container class for {checkpoint tensor: canonical key}."""
-    return type(name, (LayerContainer, ), {"__annotations__": {key: single(key) for key in tensors.values()},
-                                           "PARAM_MAPPING": {src: f"{key}.params" for src, key in tensors.items()}})
+    return type(name, (_HybridContainer, ), {"__annotations__": {key: single(key) for key in tensors.values()},
+                                             "PARAM_MAPPING": {src: f"{key}.params" for src, key in tensors.items()},
+                                             "may_lack": may_lack})
 
 
-def layer_container(layer, streams):
+def layer_container(layer, streams, may_lack=()):
     """Container class of one entry of the config's layer list."""
     if layer["type"] not in _MIXER_TENSORS:
         raise NotImplementedError(f"no mixer {layer['type']!r}")
@@ -38,7 +51,7 @@ def layer_container(layer, streams):
         tensors[f"norm{q}"] = f"norm{q}_w"
         if streams:
             tensors.update({f"hc{q}.{n}": f"hc{q}_{n}" for n in ("in", "out", "mix")})
-    return container("HybridLayerContainer", tensors)
+    return container("HybridLayerContainer", tensors, may_lack)
 
 
 TopContainer = container("HybridTopContainer", {"embed": "embed", "final.norm": "norm_w", "head": "lm_head"})
@@ -65,6 +78,9 @@ class VopepelPolicy(InferenceV2Policy):
         c = self._model_config
         cmap = ContainerMap()
         streams = bool(getattr(c, "streams", None))
-        cmap.set_transformer_params("l", [layer_container(la, streams)(self._view) for la in c.layers], sep="")
+        # the first value-mixing layer only lends its values: it has no use for a mixing weight
+        first = next((i for i, la in enumerate(c.layers) if la["mixer"].get("v_mix")), None)
+        cmap.set_transformer_params("l", [layer_container(la, streams, ("vmix", ) if i == first else ())(self._view)
+                                          for i, la in enumerate(c.layers)], sep="")
         cmap.set_non_transformer_params(TopContainer(self._view))
         return cmap
