@@ -40,6 +40,11 @@ def parse():
     ap.add_argument("--sp", type=int, default=1,
                     help="Ulysses sequence-parallel degree (BASELINE config: Llama-2 7B, seq 32k, sp over xGMI "
                          "all-to-all); dp = world / sp")
+    ap.add_argument("--workload", default="train", choices=["train", "hybrid"],
+                    help="train: the flagship training step (default); hybrid: serving throughput of a hybrid decoder "
+                         "beside the uniform one (benchmarks/hybrid_serving.py)")
+    ap.add_argument("--sizes", default="2048,4096", help="--workload hybrid: model widths")
+    ap.add_argument("--model-kind", default="both", choices=["hybrid", "uniform", "both"], help="--workload hybrid")
     ap.add_argument("--local_rank", type=int, default=0)
     ap.add_argument("--host-dryrun", action="store_true",
                     help="CPU/gloo rehearsal of the multi-rank control flow (tiny model; not a measurement)")
@@ -142,6 +147,9 @@ def forced_partition_loop(args, cfg, config, dev, batches, sync, steps=3, warmup
 
 def main():
     args = parse()
+    if args.workload == "hybrid":
+        from deepspeedsyclsupport_amd.benchmarks import hybrid_serving
+        return hybrid_serving.run([int(w) for w in args.sizes.split(",")], args.model_kind, iters=2 * args.steps, log=log)
     import deepspeedsyclsupport_amd as ds
     from deepspeedsyclsupport_amd import comm as dist
     from deepspeedsyclsupport_amd.models.llama import (LlamaConfig, LlamaForCausalLM, llama2_7b_config, llama2_13b_config,

@@ -1,0 +1,105 @@
+"""Serving throughput of a hybrid decoder (Vopepel layers: gated delta rule, chunked attention, residual streams) beside
+the uniform Llama-style decoder at equal width, feed-forward, head and layer counts, both through the ragged engine with
+random bf16 weights: whole-prompt prefill and batched decoding.
+
+    python bench.py --workload hybrid [--sizes 2048,4096] [--model-kind hybrid|uniform|both]
+"""
+import json
+import time
+
+import torch
+
+SIZES = {2048: dict(ff=5632, heads=16, kv=8), 4096: dict(ff=14336, heads=32, kv=8)}
+PATTERN = ("delta", "attention", "attention", "delta", "attention", "attention", "delta", "attention")
+HEAD, CHUNK, STREAMS, VOCAB = 128, 2048, 4, 32000
+
+
+def specs(width):
+    """(hybrid, uniform) model specs of one size."""
+    from ..inference.model_implementations.transformer import DSModelSpec
+    s = SIZES[width]
+    common = dict(vocab_size=VOCAB, hidden_size=width, num_layers=len(PATTERN), num_heads=s["heads"],
+                  num_kv_heads=s["kv"], intermediate_size=s["ff"], head_dim=HEAD)
+    mlp = {"kind": "dense", "ff": s["ff"], "limit": 7.0}
+    mixers = {"delta": {"heads": s["heads"], "kv_heads": s["kv"], "dim": HEAD, "vdim": HEAD, "conv": 4},
+              "attention": {"heads": s["heads"], "kv_heads": s["kv"], "dim": HEAD, "vdim": HEAD, "scale": HEAD**-0.5,
+                            "softcap": 30.0, "mask": {"size": CHUNK}, "v_mix": True}}
+    hybrid = DSModelSpec(arch="vopepel", norm="ln", norm_bias=False, pos="none", streams=STREAMS, residual_mult=0.7,
+                         layer_specs=tuple({"type": t, "mixer": mixers[t], "mlp": mlp} for t in PATTERN), **common)
+    uniform = DSModelSpec(arch="llama", norm="rms", pos="rope", max_positions=16384, **common)
+    return hybrid, uniform
+
+
+def build(spec, device, blocks):
+    from ..inference.model_implementations.hybrid import model_class
+    from ..inference.v2 import AllocationMode, InferenceEngineV2, RaggedInferenceEngineConfig
+    from ..inference.v2.engine_factory import _apply_decode_layout
+    torch.manual_seed(0)
+    model = model_class(spec)(spec, dtype=torch.bfloat16, device=device)
+    with torch.no_grad():
+        for p in model.parameters():
+            if p.dim() >= 2 and p.dtype == torch.bfloat16:
+                p.normal_(0, 0.02)
+            elif p.dim() == 2 and p.shape[0] == p.shape[1]:
+                p.copy_(torch.eye(p.shape[0]))      # stream mixing
+            elif p.dim() == 2:
+                p.normal_(0, 0.3)                   # convolution taps
+    _apply_decode_layout(model, "auto", 1, torch.device(device))
+    cfg = RaggedInferenceEngineConfig(
+        state_manager={"memory_config": {"mode": AllocationMode.ALLOCATE, "size": blocks}, "max_ragged_batch_size": 8192,
+                       "max_ragged_sequence_count": 64, "max_tracked_sequences": 64, "max_context": 16384},
+        kv_cache={"block_size": 64})
+    return InferenceEngineV2(model, cfg)
+
+
+def timed(fn, iters, warmup=2):
+    for _ in range(warmup):
+        fn()
+    torch.cuda.synchronize()
+    t = time.perf_counter()
+    for _ in range(iters):
+        fn()
+    torch.cuda.synchronize()
+    return (time.perf_counter() - t) / iters
+
+
+def measure(spec, device, prompts, batches, context, iters, log):
+    eng = build(spec, device, blocks=64 * (context // 64 + 2) + 256)
+    g = torch.Generator().manual_seed(0)
+    out = {"prefill_tok_s": {}, "decode_tok_s": {}, "decode_ms": {}}
+    for n, length in prompts:
+        toks = [torch.randint(0, spec.vocab_size, (length, ), generator=g) for _ in range(n)]
+
+        def prefill():
+            eng.put(list(range(n)), toks)
+            for u in range(n):
+                eng.flush(u)
+
+        t = timed(prefill, iters)
+        out["prefill_tok_s"][f"{n}x{length}"] = round(n * length / t, 1)
+        log(f"[bench] {spec.arch} w{spec.hidden_size} prefill {n}x{length}: {t * 1e3:.2f} ms")
+    for u in range(max(batches)):
+        eng.put([u], [torch.randint(0, spec.vocab_size, (context, ), generator=g)])
+    for b in batches:
+        one = [torch.tensor([u % spec.vocab_size]) for u in range(b)]
+        t = timed(lambda: eng.put(list(range(b)), one), iters * 2)
+        out["decode_tok_s"][str(b)] = round(b / t, 1)
+        out["decode_ms"][str(b)] = round(t * 1e3, 3)
+        log(f"[bench] {spec.arch} w{spec.hidden_size} decode b{b} ctx{context}: {t * 1e3:.3f} ms")
+    return out
+
+
+def run(sizes=(2048, 4096), kind="both", iters=10, prompts=((1, 8192), (4, 2048), (16, 128)), batches=(1, 16, 64),
+        context=1536, log=print):
+    device = torch.device("cuda", torch.cuda.current_device())
+    rows = []
+    for width in sizes:
+        row = {"width": width, "layers": len(PATTERN), **SIZES[width]}
+        for name, spec in zip(("hybrid", "uniform"), specs(width)):
+            if kind in (name, "both"):
+                row[name] = measure(spec, device, prompts, batches, context, iters, log)
+                torch.cuda.empty_cache()
+        rows.append(row)
+    print(json.dumps({"metric": "ragged-engine serving throughput, hybrid decoder beside the uniform one", "unit": "tokens/s",
+                      "dtype": "bf16", "data": "synthetic tokens, random-init weights", "context": context,
+                      "sizes": rows}), flush=True)
