@@ -216,7 +216,7 @@ class DSHybridModel(DSInferenceModel):
         return [(m.G, m.dk, m.dv) if m.kind == "attention" else None for m in (la.mixer for la in self.layers)]
 
     def state_geometry(self):
-        return [{"state": ((m.H, m.dk, m.dv), torch.float32), "conv": ((m.taps - 1, m.channels), self.dtype)}
+        return [{"state": ((m.H, m.dv, -(-m.dk // 4) * 4), torch.float32), "conv": ((m.taps - 1, m.channels), self.dtype)}
                 if m.kind == "delta" else None for m in (la.mixer for la in self.layers)]
 
     def shard_layer(self, idx, lw):

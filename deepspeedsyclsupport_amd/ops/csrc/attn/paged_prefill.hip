@@ -219,14 +219,20 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
             s[t][r] = v;
           }
       }
-      float mx = -INFINITY;
+      // a moderate cap bounds the scores: it serves as the maximum, and nothing is ever rescaled
+      const bool fixed = EXT && a.cap_out > 0.f && a.cap_out <= 48.f;
+      float alpha = 1.f, mc = a.cap_out;
+      if (!fixed) {
+        float mx = -INFINITY;
 #pragma unroll
-      for (int r = 0; r < 16; ++r) mx = fmaxf(mx, fmaxf(s[0][r], s[1][r]));
-      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      const float m_new = fmaxf(m_run, mx);
-      const float m_use = m_new == -INFINITY ? 0.f : m_new;
-      const float alpha = __builtin_amdgcn_exp2f((m_run - m_use) * a.c);
-      const float mc = m_use * a.c;
+        for (int r = 0; r < 16; ++r) mx = fmaxf(mx, fmaxf(s[0][r], s[1][r]));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        const float m_new = fmaxf(m_run, mx);
+        const float m_use = m_new == -INFINITY ? 0.f : m_new;
+        alpha = __builtin_amdgcn_exp2f((m_run - m_use) * a.c);
+        mc = m_use * a.c;
+        m_run = m_new;
+      }
       float psum = 0.f;
 #pragma unroll
       for (int t = 0; t < 2; ++t)
@@ -237,8 +243,7 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
           psum += p;
         }
       l_run = l_run * alpha + psum;
-      m_run = m_new;
-      if (!__all(alpha == 1.f)) {
+      if (!fixed && !__all(alpha == 1.f)) {
         if (lane < 32) scratch[lane] = alpha;
         __builtin_amdgcn_wave_barrier();
         __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");

@@ -249,8 +249,8 @@ void delta_recur(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, dou
   const int64_t T = v.size(0), H = v.size(1), dv = v.size(2), Hk = qk.size(2), dk = qk.size(3), S = start.numel();
   const int64_t taps = conv_state.size(1) + 1;
   delta_dims_ok(Hk, H, dk, dv, taps);
-  TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == H && state.size(2) == dk &&
-              state.size(3) == dv && state.size(0) == conv_state.size(0), "delta: state [slots, H, dk, dv] fp32");
+  TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == H && state.size(2) == dv &&
+              state.size(3) == (dk + 3) / 4 * 4 && state.size(0) == conv_state.size(0), "delta: state [slots, H, dv, dk padded to 4] fp32");
   TORCH_CHECK(conv_state.size(2) == 2 * Hk * dk + H * dv, "delta: conv_state");
   TORCH_CHECK(proj.numel() == T * (2 * Hk * dk + 2 * H * dv + 2 * H) && out.numel() == T * H * dv, "delta: proj / out");
   TORCH_CHECK(v.scalar_type() == proj.scalar_type() && out.scalar_type() == proj.scalar_type() &&
@@ -270,8 +270,8 @@ void delta_chunk(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, dou
   const int64_t T = v.size(0), H = v.size(1), dv = v.size(2), Hk = qk.size(2), dk = qk.size(3), S = start.numel();
   const int64_t taps = conv_state.size(1) + 1;
   delta_dims_ok(Hk, H, dk, dv, taps);
-  TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == H && state.size(2) == dk &&
-              state.size(3) == dv && state.size(0) == conv_state.size(0), "delta: state [slots, H, dk, dv] fp32");
+  TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == H && state.size(2) == dv &&
+              state.size(3) == (dk + 3) / 4 * 4 && state.size(0) == conv_state.size(0), "delta: state [slots, H, dv, dk padded to 4] fp32");
   TORCH_CHECK(conv_state.size(2) == 2 * Hk * dk + H * dv, "delta: conv_state");
   TORCH_CHECK(proj.numel() == T * (2 * Hk * dk + 2 * H * dv + 2 * H) && out.numel() == T * H * dv, "delta: proj / out");
   TORCH_CHECK(v.scalar_type() == proj.scalar_type() && out.scalar_type() == proj.scalar_type() &&

@@ -6,8 +6,8 @@
 //     o_i = e^{G_i} S0^T q_i + sum_{j <= i} P_ij u_j,      P_ij = e^{G_i - G_j} (q_i . k_j)
 //     S   = e^{G_C} S0 + sum_j e^{G_C - G_j} k_j u_j^T
 //  * chunk kernel: one workgroup per (chunk, head), all chunks of all sequences at once. K K^T and Q K^T on the fp32
-//    matrix cores, then W = (I + A)^-1 diag(beta e^G) K and X = (I + A)^-1 diag(beta) V by forward substitution, one
-//    column per thread with the 64 unknowns in registers. Writes W, X, P and the decays.
+//    matrix cores, then W = (I + A)^-1 diag(beta e^G) K and X = (I + A)^-1 diag(beta) V by forward substitution over
+//    16-row blocks (the diagonal blocks inverted first), again products of 16 x 16 tiles. Writes W, X, P and the decays.
 //  * scan kernel: one workgroup per (sequence, head, 16 value columns) walks the chunks: U = X - W S0, the read-out and
 //    the next state are products of 16 x 16 tiles on the fp32 matrix cores; the state tile stays in LDS.
 //  * norm kernel: per-head RMS norm and gate of the read-out.
@@ -41,7 +41,7 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
     float* __restrict__ dec, DeltaDims D) {
   __shared__ __attribute__((aligned(16))) float A[C][C + 4];
   __shared__ double G[C];
-  __shared__ float beta[C];
+  __shared__ float beta[C], eg[C];
   const int h = blockIdx.x % D.H, ci = blockIdx.x / D.H, hk = h / (D.H / D.Hk);
   const int seq = work[2 * ci], c = work[2 * ci + 1];
   const int t0 = cu[seq] + c * C, n = min(C, cu[seq + 1] - t0);
@@ -56,7 +56,8 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
     G[lane] = g;
     beta[lane] = lane < n ? gb[((int64_t)(t0 + lane) * 2 + 1) * D.H + h] : 0.f;
     const double gc = __shfl(g, 63, 64);  // rows beyond n add nothing
-    dec[base * 2 * C + lane] = expf((float)g);
+    eg[lane] = expf((float)g);
+    dec[base * 2 * C + lane] = eg[lane];
     dec[base * 2 * C + C + lane] = expf((float)(gc - g));
   }
   __syncthreads();
@@ -88,36 +89,62 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
     }
   }
   __syncthreads();
-  // ---- forward substitution: column col of [W | X]
-  for (int col = tid; col < D.dk + D.dv; col += NT) {
-    const bool isw = col < D.dk;
-    float x[C];
+  // ---- invert the unit lower-triangular diagonal blocks, wave w block w, a column per lane
+  if (lane < 16) {
+    float t[16];
 #pragma unroll
-    for (int i = 0; i < C; ++i) {
-      float r = 0.f;
-      if (i < n) {
-        const int64_t t = t0 + i;
-        if (isw) r = kbase[t * rs + col] * expf((float)G[i]);
-        else r = (float)v[(t * D.H + h) * D.dv + col - D.dk];
-        r *= beta[i];
-      }
-      x[i] = r;
+    for (int i = 0; i < 16; ++i) {
+      float r = i == lane ? 1.f : 0.f;
+#pragma unroll
+      for (int j = 0; j < i; ++j) r = fmaf(-A[w * 16 + i][w * 16 + j], t[j], r);
+      t[i] = r;
     }
+    __builtin_amdgcn_wave_barrier();
 #pragma unroll
-    for (int i = 1; i < C; ++i) {
-      asm volatile("" ::: "memory");  // one row of A at a time: hoisting them all costs the registers x needs
+    for (int i = 0; i < 16; ++i) A[w * 16 + i][w * 16 + lane] = t[i];
+  }
+  __syncthreads();
+  // ---- block forward substitution of [W | X], 16 columns per wave at a time: x_b = T_bb (r_b - sum_{c < b} A_bc x_c).
+  // A product's result layout (row 4 q4 + r of column l16) is the next one's right operand as it stands.
+  const int wt = (D.dk + 15) / 16, xt = (D.dv + 15) / 16;
+  for (int ct = w; ct < wt + xt; ct += 4) {
+    const bool isw = ct < wt;
+    const int col = (isw ? ct : ct - wt) * 16 + l16, width = isw ? D.dk : D.dv;
+    f32x4 x[4];
 #pragma unroll
-      for (int j = 0; j < (i + 3) / 4; ++j) {  // entries at and right of the diagonal are zero
-        const f32x4 a = *reinterpret_cast<const f32x4*>(&A[i][4 * j]);
+    for (int b = 0; b < 4; ++b)
 #pragma unroll
-        for (int e = 0; e < 4; ++e)
-          if (4 * j + e < i) x[i] = fmaf(-a[e], x[4 * j + e], x[i]);
+      for (int r = 0; r < 4; ++r) {
+        const int i = b * 16 + 4 * q4 + r;
+        float v0 = 0.f;
+        if (i < n && col < width) {
+          const int64_t t = t0 + i;
+          v0 = beta[i] * (isw ? kbase[t * rs + col] * eg[i] : (float)v[(t * D.H + h) * D.dv + col]);
+        }
+        x[b][r] = v0;
       }
-    }
-    float* dst = isw ? Wo + base * C * D.dk + col : Xo + base * C * D.dv + col - D.dk;
-    const int ld = isw ? D.dk : D.dv;
 #pragma unroll
-    for (int i = 0; i < C; ++i) dst[i * ld] = x[i];
+    for (int b = 0; b < 4; ++b) {
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int c2 = 0; c2 < b; ++c2) {
+        const f32x4 a = *reinterpret_cast<const f32x4*>(&A[b * 16 + l16][c2 * 16 + 4 * q4]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc = mfma4(a[e], x[c2][e], acc);
+      }
+      const f32x4 rhs = x[b] - acc, a = *reinterpret_cast<const f32x4*>(&A[b * 16 + l16][b * 16 + 4 * q4]);
+      f32x4 y = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y = mfma4(a[e], rhs[e], y);
+      x[b] = y;
+    }
+    if (col < width) {
+      float* dst = (isw ? Wo + base * C * D.dk : Xo + base * C * D.dv) + col;
+#pragma unroll
+      for (int b = 0; b < 4; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) dst[(b * 16 + 4 * q4 + r) * width] = x[b][r];
+    }
   }
 }
 
@@ -134,10 +161,10 @@ __global__ void __launch_bounds__(NT) delta_scan_kernel(
   const int hk = h / (D.H / D.Hk), tid = threadIdx.x, lane = tid & 63, w = tid >> 6, l16 = lane & 15, q4 = lane >> 4;
   const int t0 = cu[seq], n = cu[seq + 1] - t0, nc = (n + C - 1) / C, v0 = vt * 16;
   const bool fresh = start[seq] == 0;
-  float* st = state + ((int64_t)slots[seq] * D.H + h) * D.dk * D.dv;
+  float* st = state + ((int64_t)slots[seq] * D.H + h) * D.dks() * D.dv;
   for (int i = tid; i < NK * 256; i += NT) {
-    const int k = i / 16, j = i % 16;
-    S[k][j] = (!fresh && k < D.dk && v0 + j < D.dv) ? st[(int64_t)k * D.dv + v0 + j] : 0.f;
+    const int k = i % (NK * 16), j = i / (NK * 16);
+    S[k][j] = (!fresh && k < D.dk && v0 + j < D.dv) ? st[(int64_t)(v0 + j) * D.dks() + k] : 0.f;
   }
   const int64_t rs = (int64_t)2 * D.Hk * D.dk;
   const float* qbase = qk + (int64_t)hk * D.dk;
@@ -226,9 +253,9 @@ __global__ void __launch_bounds__(NT) delta_scan_kernel(
     if (c + 1 < nc) fetch(c + 1);
     __syncthreads();
   }
-  for (int i = tid; i < D.dk * 16; i += NT) {
-    const int k = i / 16, j = i % 16;
-    if (v0 + j < D.dv) st[(int64_t)k * D.dv + v0 + j] = S[k][j];
+  for (int i = tid; i < NK * 256; i += NT) {
+    const int k = i % (NK * 16), j = i / (NK * 16);
+    if (k < D.dk && v0 + j < D.dv) st[(int64_t)(v0 + j) * D.dks() + k] = S[k][j];
   }
   if (vt == 0 && D.taps > 1)
     advance_head(conv_state + (int64_t)slots[seq] * (D.taps - 1) * D.channels(), proj, t0, n, D, fresh, h);
@@ -245,18 +272,23 @@ __global__ void __launch_bounds__(NT) delta_norm_kernel(const float* __restrict_
   for (int i = threadIdx.x >> 6; i < n; i += NT / 64) {
     const int64_t t = t0 + i, at = (t * D.H + h) * D.dv;
     const T* gate = proj + t * D.row() + D.channels() + h * D.dv;
-    float x[4], ss = 0.f;
+    float x[2][2], ss = 0.f;
 #pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      const int c = k * 64 + lane;
-      x[k] = c < D.dv ? o[at + c] : 0.f;
-      ss = fmaf(x[k], x[k], ss);
+    for (int k = 0; k < 2; ++k) {
+      const int c = k * 128 + 2 * lane;
+      load2(o + at + c, D.dv - c, x[k]);
+      ss = fmaf(x[k][0], x[k][0], fmaf(x[k][1], x[k][1], ss));
     }
     const float rms = 1.f / sqrtf(wave_sum(ss) / (float)D.dv + eps);
 #pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      const int c = k * 64 + lane;
-      if (c < D.dv) out[at + c] = (T)(x[k] * rms * norm_w[c] * silu((float)gate[c]));
+    for (int k = 0; k < 2; ++k) {
+      const int c = k * 128 + 2 * lane;
+      float g[2], nw[2];
+      load2(gate + c, D.dv - c, g);
+      load2(norm_w + c, D.dv - c, nw);
+#pragma unroll
+      for (int e = 0; e < 2; ++e) g[e] = x[k][e] * rms * nw[e] * silu(g[e]);
+      store2(out + at + c, D.dv - c, g);
     }
   }
 }

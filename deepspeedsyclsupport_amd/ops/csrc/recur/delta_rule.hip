@@ -8,10 +8,10 @@
 //
 // The fused projection row of a token is [q (Hk dk) | k (Hk dk) | v (H dv) | g (H dv) | b (H) | a (H)].
 //
-//  * prepare: one wave per (token, head part): convolution + silu + unit norm / decays, reading earlier tokens of the
+//  * prepare: one wave per (few consecutive tokens, head part): convolution + silu + unit norm / decays, reading earlier tokens of the
 //    same portion from the projection itself and the ones before it from the sequence's state slot. Everything that
 //    enters the recurrence leaves it in fp32 (v in the storage type: it is a convolution output).
-//  * recur: one workgroup per (sequence, head); the state sits in registers (LPC lanes per value column, E rows each)
+//  * recur: one workgroup per (sequence, head); the state, kept as [dv, dk] (dk padded to 4), sits in registers
 //    while the portion's tokens pass one by one: decoding and short portions. It also moves the convolution's window
 //    on in the state slot (prepare, which reads the old one, has finished by then).
 // A sequence whose portion starts at position 0 starts from zero: slots need no clearing between owners.
@@ -19,96 +19,157 @@
 
 namespace {
 
-template <typename T>
+constexpr int TILE = 8;  // consecutive tokens a prepare wave walks
+
+// TAPS: filter length held in registers (the window slides from token to token); 0: any length, read afresh per token
+template <typename T, int TAPS>
 __global__ void __launch_bounds__(256) delta_prepare_kernel(
     const T* __restrict__ proj, const float* __restrict__ conv_w, const T* __restrict__ conv_state,
     const float* __restrict__ a_log, const float* __restrict__ dt_bias, const int* __restrict__ seq_ids,
     const int* __restrict__ cu, const int* __restrict__ start, const int* __restrict__ slots, float* __restrict__ qk,
-    T* __restrict__ v_out, float* __restrict__ gb, int tokens, DeltaDims D) {
+    T* __restrict__ v_out, float* __restrict__ gb, int tokens, int tile, DeltaDims D) {
   const int parts = 2 * D.Hk + D.H + 1, lane = threadIdx.x & 63;
   const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (item >= (int64_t)tokens * parts) return;
-  const int t = (int)(item / parts), part = (int)(item % parts);
-  const int NP = D.row(), C = D.channels();
+  const int t_lo = (int)(item / parts) * tile, part = (int)(item % parts), t_hi = min(t_lo + tile, tokens);
+  const int NP = D.row(), CH = D.channels(), taps = TAPS ? TAPS : D.taps;
   if (part == parts - 1) {  // decays (as logarithms) and write strengths
-    const T* b = proj + (int64_t)t * NP + C + D.H * D.dv;
-    for (int h = lane; h < D.H; h += 64) {
-      const float z = (float)b[D.H + h] + dt_bias[h];
-      const float sp = z > 20.f ? z : log1pf(expf(z));
-      gb[((int64_t)t * 2) * D.H + h] = -expf(a_log[h]) * sp;
-      gb[((int64_t)t * 2 + 1) * D.H + h] = 1.f / (1.f + expf(-(float)b[h]));
+    for (int t = t_lo; t < t_hi; ++t) {
+      const T* b = proj + (int64_t)t * NP + CH + D.H * D.dv;
+      for (int h = lane; h < D.H; h += 64) {
+        const float z = (float)b[D.H + h] + dt_bias[h];
+        const float sp = z > 20.f ? z : log1pf(expf(z));
+        gb[((int64_t)t * 2) * D.H + h] = -expf(a_log[h]) * sp;
+        gb[((int64_t)t * 2 + 1) * D.H + h] = 1.f / (1.f + expf(-(float)b[h]));
+      }
     }
     return;
   }
   const bool is_v = part >= 2 * D.Hk;
   const int width = is_v ? D.dv : D.dk;
   const int c0 = is_v ? 2 * D.Hk * D.dk + (part - 2 * D.Hk) * D.dv : part * D.dk;
-  const int seq = seq_ids[t], j = t - cu[seq];  // index of the token in its portion
-  const bool fresh = start[seq] == 0;
-  const T* cs = conv_state + (int64_t)slots[seq] * (D.taps - 1) * C;
-  auto conv = [&](int c) {
-    float a = 0.f;
-    for (int i = 0; i < D.taps; ++i) {
-      const int src = j - (D.taps - 1) + i;  // relative to the portion's first token
-      float x = 0.f;
-      if (src >= 0) x = (float)proj[(int64_t)(t - j + src) * NP + c];
-      else if (!fresh) x = (float)cs[(int64_t)(src + D.taps - 1) * C + c];
-      a = fmaf(conv_w[(int64_t)c * D.taps + i], x, a);
-    }
-    return silu(a);
+  // a lane's channels: 2 lane, 2 lane + 1, and the same 128 further on
+  float cw[2][2][TAPS ? TAPS : 1], win[2][2][TAPS ? TAPS : 1];
+  if constexpr (TAPS != 0) {
+#pragma unroll
+    for (int k = 0; k < 2; ++k)
+#pragma unroll
+      for (int e = 0; e < 2; ++e) {
+        const int c = k * 128 + 2 * lane + e;
+#pragma unroll
+        for (int i = 0; i < TAPS; ++i) cw[k][e][i] = c < width ? conv_w[(int64_t)(c0 + c) * TAPS + i] : 0.f;
+      }
+  }
+  int seq = -1, first = 0;
+  const T* cs = nullptr;
+  // input of the convolution at place j of the portion (negative: before it)
+  auto input = [&](int j, int k, float (&x)[2]) {
+    const int c = k * 128 + 2 * lane;
+    x[0] = x[1] = 0.f;
+    if (c >= width) return;
+    if (j >= 0) load2(proj + (int64_t)(first + j) * NP + c0 + c, width - c, x);
+    else if (cs) load2(cs + (int64_t)(j + taps - 1) * CH + c0 + c, width - c, x);
   };
-  if (is_v) {
-    T* dst = v_out + (int64_t)t * D.H * D.dv + (part - 2 * D.Hk) * D.dv;
-    for (int c = lane; c < width; c += 64) dst[c] = (T)conv(c0 + c);
-    return;
-  }
-  float vals[4], ss = 0.f;  // dk <= 256
+  for (int t = t_lo; t < t_hi; ++t) {
+    const bool fill = t == t_lo || seq_ids[t] != seq;
+    if (fill) {
+      seq = seq_ids[t];
+      first = cu[seq];
+      cs = start[seq] == 0 ? nullptr : conv_state + (int64_t)slots[seq] * (taps - 1) * CH;
+    }
+    const int j = t - first;
+    float y[2][2];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int c = i * 64 + lane;
-    vals[i] = c < width ? conv(c0 + c) : 0.f;
-    ss = fmaf(vals[i], vals[i], ss);
-  }
-  float r = 1.f / sqrtf(wave_sum(ss) + 1e-6f);
-  if (part < D.Hk) r *= 1.f / sqrtf((float)D.dk);
-  float* dst = qk + (int64_t)t * 2 * D.Hk * D.dk + (int64_t)part * D.dk;
+    for (int k = 0; k < 2; ++k) {
+      float acc[2] = {0.f, 0.f};
+      if (k * 128 < width) {
+        float x[2];
+        if constexpr (TAPS != 0) {
+          if (fill) {
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int c = i * 64 + lane;
-    if (c < width) dst[c] = vals[i] * r;
+            for (int i = 1; i < TAPS; ++i) {
+              input(j - TAPS + i, k, x);
+              win[k][0][i] = x[0];
+              win[k][1][i] = x[1];
+            }
+          }
+          input(j, k, x);
+#pragma unroll
+          for (int e = 0; e < 2; ++e) {
+#pragma unroll
+            for (int i = 0; i + 1 < TAPS; ++i) win[k][e][i] = win[k][e][i + 1];
+            win[k][e][TAPS - 1] = x[e];
+#pragma unroll
+            for (int i = 0; i < TAPS; ++i) acc[e] = fmaf(cw[k][e][i], win[k][e][i], acc[e]);
+          }
+        } else {
+          for (int i = 0; i < taps; ++i) {
+            input(j - (taps - 1) + i, k, x);
+#pragma unroll
+            for (int e = 0; e < 2; ++e) {
+              const int c = k * 128 + 2 * lane + e;
+              if (c < width) acc[e] = fmaf(conv_w[(int64_t)(c0 + c) * taps + i], x[e], acc[e]);
+            }
+          }
+        }
+      }
+      y[k][0] = silu(acc[0]);
+      y[k][1] = silu(acc[1]);
+    }
+    if (is_v) {
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        const int c = k * 128 + 2 * lane;
+        store2(v_out + ((int64_t)t * D.H + part - 2 * D.Hk) * D.dv + c, width - c, y[k]);
+      }
+      continue;
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < 2; ++k) ss = fmaf(y[k][0], y[k][0], fmaf(y[k][1], y[k][1], ss));  // silu(0) = 0 in the padding
+    float r = 1.f / sqrtf(wave_sum(ss) + 1e-6f);
+    if (part < D.Hk) r *= 1.f / sqrtf((float)D.dk);
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const int c = k * 128 + 2 * lane;
+      y[k][0] *= r;
+      y[k][1] *= r;
+      store2(qk + ((int64_t)t * 2 * D.Hk + part) * D.dk + c, width - c, y[k]);
+    }
   }
 }
 
-template <typename T, int E>
+// LPC lanes per value column, each with 4 NV key rows in quads: row 4 (p + LPC i) + e. The state is stored with the key
+// index innermost, [dv, dk], so a column's lanes read consecutive 16-byte pieces.
+template <typename T, int NV, int LPC>
 __global__ void __launch_bounds__(1024) delta_recur_kernel(
     const float* __restrict__ qk, const T* __restrict__ v, const float* __restrict__ gb, const T* __restrict__ proj,
     const float* __restrict__ norm_w, float eps, float* __restrict__ state, T* __restrict__ conv_state,
     const int* __restrict__ list, const int* __restrict__ cu, const int* __restrict__ start,
-    const int* __restrict__ slots, T* __restrict__ out, DeltaDims D, int lpc) {
-  extern __shared__ __attribute__((aligned(16))) float sm[];
+    const int* __restrict__ slots, T* __restrict__ out, DeltaDims D) {
+  constexpr int KP = 4 * NV * LPC;  // padded key width
+  __shared__ __attribute__((aligned(16))) float qs[KP];
+  __shared__ __attribute__((aligned(16))) float ks[KP];
+  __shared__ float red[16];
   const int seq = list[blockIdx.x], h = blockIdx.y, hk = h / (D.H / D.Hk), tid = threadIdx.x;
-  const int kp = lpc * E;  // padded key width
-  float* qs = sm;
-  float* ks = sm + kp;
-  float* red = sm + 2 * kp;
   const int64_t t0 = cu[seq];
   const int n = cu[seq + 1] - (int)t0;
   const bool fresh = start[seq] == 0;
-  const int NP = D.row(), C = D.channels(), col = tid / lpc, p = tid % lpc;
+  const int NP = D.row(), C = D.channels(), col = tid / LPC, p = tid % LPC;
   const bool on = col < D.dv;
-  float* st = state + ((int64_t)slots[seq] * D.H + h) * D.dk * D.dv;
-  float S[E];
+  float* st = state + (((int64_t)slots[seq] * D.H + h) * D.dv + col) * D.dks();
+  f32x4 S[NV];
 #pragma unroll
-  for (int i = 0; i < E; ++i) {
-    const int k = p + lpc * i;
-    S[i] = (on && !fresh && k < D.dk) ? st[(int64_t)k * D.dv + col] : 0.f;
+  for (int i = 0; i < NV; ++i) {
+    const int k = 4 * (p + LPC * i);
+    S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (on && !fresh && k < D.dk) S[i] = *reinterpret_cast<const f32x4*>(st + k);
   }
   for (int t = 0; t < n; ++t) {
     const int64_t tok = t0 + t;
     const float* qr = qk + (tok * 2 * D.Hk + hk) * D.dk;
     const float* kr = qr + (int64_t)D.Hk * D.dk;
     __syncthreads();
-    for (int c = tid; c < kp; c += blockDim.x) {
+    for (int c = tid; c < KP; c += blockDim.x) {
       qs[c] = c < D.dk ? qr[c] : 0.f;
       ks[c] = c < D.dk ? kr[c] : 0.f;
     }
@@ -117,19 +178,31 @@ __global__ void __launch_bounds__(1024) delta_recur_kernel(
     __syncthreads();
     float a = 0.f;
 #pragma unroll
-    for (int i = 0; i < E; ++i) {
-      S[i] *= g;
-      a = fmaf(S[i], ks[p + lpc * i], a);
+    for (int i = 0; i < NV; ++i) {
+      const f32x4 k4 = *reinterpret_cast<const f32x4*>(ks + 4 * (p + LPC * i));
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        S[i][e] *= g;
+        a = fmaf(S[i][e], k4[e], a);
+      }
     }
-    for (int o = 1; o < lpc; o <<= 1) a += __shfl_xor(a, o, 64);
+#pragma unroll
+    for (int o = 1; o < LPC; o <<= 1) a += __shfl_xor(a, o, 64);
     const float u = beta * (vv - a);
     float ov = 0.f;
+    asm volatile("" ::: "memory");  // keys come from LDS again: holding them costs the occupancy
 #pragma unroll
-    for (int i = 0; i < E; ++i) {
-      S[i] = fmaf(ks[p + lpc * i], u, S[i]);
-      ov = fmaf(S[i], qs[p + lpc * i], ov);
+    for (int i = 0; i < NV; ++i) {
+      const f32x4 k4 = *reinterpret_cast<const f32x4*>(ks + 4 * (p + LPC * i));
+      const f32x4 q4 = *reinterpret_cast<const f32x4*>(qs + 4 * (p + LPC * i));
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        S[i][e] = fmaf(k4[e], u, S[i][e]);
+        ov = fmaf(S[i][e], q4[e], ov);
+      }
     }
-    for (int o = 1; o < lpc; o <<= 1) ov += __shfl_xor(ov, o, 64);
+#pragma unroll
+    for (int o = 1; o < LPC; o <<= 1) ov += __shfl_xor(ov, o, 64);
     const float ss = block_sum(on && p == 0 ? ov * ov : 0.f, red);
     const float rs = 1.f / sqrtf(ss / (float)D.dv + eps);
     if (on && p == 0) {
@@ -139,9 +212,9 @@ __global__ void __launch_bounds__(1024) delta_recur_kernel(
   }
   if (on) {
 #pragma unroll
-    for (int i = 0; i < E; ++i) {
-      const int k = p + lpc * i;
-      if (k < D.dk) st[(int64_t)k * D.dv + col] = S[i];
+    for (int i = 0; i < NV; ++i) {
+      const int k = 4 * (p + LPC * i);
+      if (k < D.dk) *reinterpret_cast<f32x4*>(st + k) = S[i];
     }
   }
   if (D.taps > 1) advance_head(conv_state + (int64_t)slots[seq] * (D.taps - 1) * C, proj, t0, n, D, fresh, h);
@@ -151,19 +224,22 @@ template <typename T>
 int recur(const float* qk, const void* v, const float* gb, const void* proj, const float* norm_w, float eps, float* state,
           void* conv_state, const int* list, int nlist, const int* cu, const int* start, const int* slots, void* out,
           DeltaDims D, hipStream_t st) {
-  int lpc = 1;
-  while (lpc < 16 && ((D.dk + lpc - 1) / lpc > 32 || lpc * D.dv < 128) && lpc * 2 * D.dv <= 1024) lpc *= 2;
-  const int e = (D.dk + lpc - 1) / lpc, nt = (lpc * D.dv + 63) / 64 * 64;
-#define GO(E)                                                                                                       \
-  hipLaunchKernelGGL((delta_recur_kernel<T, E>), dim3(nlist, D.H), dim3(nt), (size_t)(2 * lpc * E + 16) * 4, st, qk,  \
-                     (const T*)v, gb, (const T*)proj, norm_w, eps, state, (T*)conv_state, list, cu, start, slots,     \
-                     (T*)out, D, lpc)
-  if (e <= 4) GO(4);
-  else if (e <= 8) GO(8);
-  else if (e <= 16) GO(16);
-  else if (e <= 32) GO(32);
-  else if (e <= 64) GO(64);
-  else return (int)hipErrorInvalidValue;
+  // 8 lanes per column where the workgroup allows it (128-byte pieces of the state per column), fewer for wide heads
+  const int q = (D.dk + 3) / 4, lpc = D.dv <= 128 ? 8 : 4, nt = (lpc * D.dv + 63) / 64 * 64, nv = (q + lpc - 1) / lpc;
+#define GO(NV, LPC)                                                                                                  \
+  hipLaunchKernelGGL((delta_recur_kernel<T, NV, LPC>), dim3(nlist, D.H), dim3(nt), 0, st, qk, (const T*)v, gb,         \
+                     (const T*)proj, norm_w, eps, state, (T*)conv_state, list, cu, start, slots, (T*)out, D)
+#define ROW(LPC)             \
+  {                          \
+    if (nv <= 1) GO(1, LPC); \
+    else if (nv <= 2) GO(2, LPC); \
+    else if (nv <= 4) GO(4, LPC); \
+    else if (nv <= 8) GO(8, LPC); \
+    else GO(16, LPC);        \
+  }
+  if (lpc == 8) ROW(8)
+  else ROW(4)
+#undef ROW
 #undef GO
   DS_CHECK_LAUNCH();
   return 0;
@@ -178,14 +254,24 @@ extern "C" int ds_delta_prepare(const void* proj, const float* conv_w, const voi
   if (tokens <= 0) return 0;
   const DeltaDims D{Hk, H, dk, dv, taps};
   if (!dims_ok(D)) return (int)hipErrorInvalidValue;
-  const int64_t items = (int64_t)tokens * (2 * Hk + H + 1);
-#define GO(T)                                                                                                       \
-  hipLaunchKernelGGL((delta_prepare_kernel<T>), dim3((unsigned)((items + 3) / 4)), dim3(256), 0, st, (const T*)proj,  \
-                     conv_w, (const T*)conv_state, a_log, dt_bias, seq_ids, cu, start, slots, qk, (T*)v, gb, tokens, D)
-  if (dtype == DS_F32) GO(float);
-  else if (dtype == DS_BF16) GO(bf16);
+  const int tile = tokens >= 512 ? TILE : 1;  // few tokens: as many waves as there are
+  const int64_t items = (int64_t)((tokens + tile - 1) / tile) * (2 * Hk + H + 1);
+#define LAUNCH(T, TAPS)                                                                                             \
+  hipLaunchKernelGGL((delta_prepare_kernel<T, TAPS>), dim3((unsigned)((items + 3) / 4)), dim3(256), 0, st,            \
+                     (const T*)proj, conv_w, (const T*)conv_state, a_log, dt_bias, seq_ids, cu, start, slots, qk, (T*)v, gb, \
+                     tokens, tile, D)
+#define GO(T)                     \
+  {                               \
+    if (taps == 4) LAUNCH(T, 4);  \
+    else if (taps == 3) LAUNCH(T, 3); \
+    else if (taps == 2) LAUNCH(T, 2); \
+    else LAUNCH(T, 0);            \
+  }
+  if (dtype == DS_F32) GO(float)
+  else if (dtype == DS_BF16) GO(bf16)
   else return (int)hipErrorInvalidValue;
 #undef GO
+#undef LAUNCH
   DS_CHECK_LAUNCH();
   return 0;
 }

@@ -212,7 +212,7 @@ def delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, cu, start
     rep = H // Hk
     for i in seqs.tolist():
         a, b, slot = int(cu[i]), int(cu[i + 1]), int(slots[i])
-        S = state[slot].clone() if int(start[i]) else torch.zeros(H, dk, dv)
+        S = state[slot, ..., :dk].transpose(1, 2).clone() if int(start[i]) else torch.zeros(H, dk, dv)
         for t in range(a, b):
             q, k = qk[t].repeat_interleave(rep, 1)
             S = S * gb[t, 0].exp()[:, None, None]
@@ -221,7 +221,7 @@ def delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, cu, start
             o = (S * q[:, :, None]).sum(1)
             o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * norm_w
             out[t] = (o * F.silu(proj[t, C:C + H * dv].float().view(H, dv))).to(out.dtype)
-        state[slot] = S
+        state[slot, ..., :dk] = S.transpose(1, 2)
         if taps > 1:
             old = conv_state[slot] if int(start[i]) else torch.zeros_like(conv_state[slot])
             conv_state[slot] = torch.cat([old, proj[a:b, :C]])[-(taps - 1):].clone()

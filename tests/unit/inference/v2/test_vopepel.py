@@ -253,7 +253,7 @@ def test_geometry_and_pools(tmp_path):
     c = eng.model.cache
     assert c.k[0] is None and c.state[1] is None
     assert tuple(c.k[1].shape[1:]) == (2, 16, 32) and tuple(c.v[1].shape[1:]) == (2, 16, 16)
-    assert tuple(c.state[0]["state"].shape) == (4, 6, 16, 24) and c.state[0]["state"].dtype == torch.float32
+    assert tuple(c.state[0]["state"].shape) == (4, 6, 24, 16) and c.state[0]["state"].dtype == torch.float32
     per_block = BlockedKVCache.block_bytes(eng.model.kv_geometry(), 16, torch.float32)
     per_slot = BlockedKVCache.slot_bytes(eng.model.state_geometry())
     assert c.bytes() == 64 * per_block + 4 * per_slot
