@@ -219,7 +219,7 @@ void delta_dims_ok(int64_t Hk, int64_t H, int64_t dk, int64_t dv, int64_t taps) 
   TORCH_CHECK(dk <= 256 && dv <= 256, "delta rule: head sizes up to 256");
 }
 
-// proj [T, 2 Hk dk + 2 H dv + 2 H] -> (qk fp32 [T, 2, Hk, dk], v [T, H, dv], gb fp32 [T, 2, H]: log decay, beta)
+// proj [T, 2 Hk dk + 2 H dv + 2 H] -> (qk fp32 [T, 2, Hk, dk padded to 4], v [T, H, dv], gb fp32 [T, 2, H]: log decay, beta)
 std::vector<Tensor> delta_prepare(Tensor proj, Tensor conv_w, Tensor conv_state, Tensor a_log, Tensor dt_bias,
                                   Tensor seq_ids, Tensor cu, Tensor start, Tensor slots, int64_t Hk, int64_t H, int64_t dk,
                                   int64_t dv) {
@@ -231,7 +231,7 @@ std::vector<Tensor> delta_prepare(Tensor proj, Tensor conv_w, Tensor conv_state,
               conv_state.scalar_type() == proj.scalar_type(), "delta_prepare: conv_state [slots, taps-1, C]");
   const int64_t S = start.numel();
   auto fo = proj.options().dtype(at::kFloat);
-  auto qk = torch::empty({T, 2, Hk, dk}, fo);
+  auto qk = torch::empty({T, 2, Hk, (dk + 3) / 4 * 4}, fo);  // zero padded rows
   auto v = torch::empty({T, H, dv}, proj.options());
   auto gb = torch::empty({T, 2, H}, fo);
   check(ds_delta_prepare(proj.data_ptr(), f32(conv_w, C * taps, "conv_w"), conv_state.data_ptr(), f32(a_log, H, "A_log"),
@@ -244,9 +244,9 @@ std::vector<Tensor> delta_prepare(Tensor proj, Tensor conv_w, Tensor conv_state,
 
 // Runs the sequences in `list`; writes their rows of out [T, H dv] and their state slots.
 void delta_recur(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, double eps, Tensor state, Tensor conv_state,
-                 Tensor list, Tensor cu, Tensor start, Tensor slots, Tensor out) {
+                 Tensor list, Tensor cu, Tensor start, Tensor slots, Tensor out, int64_t dk) {
   need(proj, "proj"); need(v, "v"); need(state, "state"); need(conv_state, "conv_state"); need(out, "out");
-  const int64_t T = v.size(0), H = v.size(1), dv = v.size(2), Hk = qk.size(2), dk = qk.size(3), S = start.numel();
+  const int64_t T = v.size(0), H = v.size(1), dv = v.size(2), Hk = qk.size(2), S = start.numel();
   const int64_t taps = conv_state.size(1) + 1;
   delta_dims_ok(Hk, H, dk, dv, taps);
   TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == H && state.size(2) == dv &&
@@ -255,7 +255,7 @@ void delta_recur(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, dou
   TORCH_CHECK(proj.numel() == T * (2 * Hk * dk + 2 * H * dv + 2 * H) && out.numel() == T * H * dv, "delta: proj / out");
   TORCH_CHECK(v.scalar_type() == proj.scalar_type() && out.scalar_type() == proj.scalar_type() &&
               conv_state.scalar_type() == proj.scalar_type(), "delta: types");
-  check(ds_delta_recur(f32(qk, T * 2 * Hk * dk, "qk"), v.data_ptr(), f32(gb, T * 2 * H, "gb"), proj.data_ptr(),
+  check(ds_delta_recur(f32(qk, T * 2 * Hk * ((dk + 3) / 4 * 4), "qk"), v.data_ptr(), f32(gb, T * 2 * H, "gb"), proj.data_ptr(),
                        f32(norm_w, dv, "norm"), (float)eps, state.data_ptr<float>(), conv_state.data_ptr(),
                        i32(list, list.numel(), "list"), (int)list.numel(), i32(cu, S + 1, "cu"), i32(start, S, "start"),
                        i32(slots, S, "slots"), out.data_ptr(), (int)Hk, (int)H, (int)dk, (int)dv, (int)taps, dcode(proj),
@@ -265,9 +265,9 @@ void delta_recur(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, dou
 // The same for long portions, by chunks of 64 tokens: seqs [n, 2] (sequence, its first entry in work), work [m, 2]
 // (sequence, chunk).
 void delta_chunk(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, double eps, Tensor state, Tensor conv_state,
-                 Tensor seqs, Tensor work, Tensor cu, Tensor start, Tensor slots, Tensor out) {
+                 Tensor seqs, Tensor work, Tensor cu, Tensor start, Tensor slots, Tensor out, int64_t dk) {
   need(proj, "proj"); need(v, "v"); need(state, "state"); need(conv_state, "conv_state"); need(out, "out");
-  const int64_t T = v.size(0), H = v.size(1), dv = v.size(2), Hk = qk.size(2), dk = qk.size(3), S = start.numel();
+  const int64_t T = v.size(0), H = v.size(1), dv = v.size(2), Hk = qk.size(2), S = start.numel();
   const int64_t taps = conv_state.size(1) + 1;
   delta_dims_ok(Hk, H, dk, dv, taps);
   TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == H && state.size(2) == dv &&
@@ -281,7 +281,7 @@ void delta_chunk(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, dou
   auto fo = proj.options().dtype(at::kFloat);
   auto ws = torch::empty({ds_delta_chunk_ws((int)nw, (int)H, (int)dk, (int)dv)}, fo);
   auto o = torch::empty({T, H, dv}, fo);
-  check(ds_delta_chunk(f32(qk, T * 2 * Hk * dk, "qk"), v.data_ptr(), f32(gb, T * 2 * H, "gb"), proj.data_ptr(),
+  check(ds_delta_chunk(f32(qk, T * 2 * Hk * ((dk + 3) / 4 * 4), "qk"), v.data_ptr(), f32(gb, T * 2 * H, "gb"), proj.data_ptr(),
                        f32(norm_w, dv, "norm"), (float)eps, state.data_ptr<float>(), conv_state.data_ptr(),
                        i32(seqs, seqs.numel(), "seqs"), (int)seqs.size(0), i32(work, work.numel(), "work"), (int)nw,
                        i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"), ws.data_ptr<float>(),

@@ -14,8 +14,6 @@
 
 namespace {
 
-constexpr int NT = 256;
-
 template <typename T, int V>
 __device__ __forceinline__ void ldv(const T* p, float (&v)[V]) {
   if constexpr (V == 1) {
@@ -47,7 +45,8 @@ __device__ __forceinline__ void stv(T* p, const float (&v)[V]) {
   }
 }
 
-template <typename T, int S, int V>
+// NT threads per token: 256, or 1024 when there are too few tokens to fill the chip (latency counts then)
+template <typename T, int S, int V, int NT>
 __global__ void __launch_bounds__(NT) stream_norm_kernel(
     float* __restrict__ x, const T* __restrict__ y, const int* __restrict__ ids, const T* __restrict__ embed,
     const int* __restrict__ rows, const float* __restrict__ mix, const float* __restrict__ out, float m,
@@ -134,12 +133,14 @@ __global__ void __launch_bounds__(NT) stream_norm_kernel(
 template <typename T, int S>
 int launch(float* x, const void* y, const int* ids, const void* embed, const int* rows, int nrows, const float* mix,
            const float* out, float m, const float* in, const float* w, void* normed, int W, float eps, hipStream_t st) {
-  const size_t lds = (size_t)(((W + 3) & ~3) + 8) * sizeof(float);
-#define GO(V)                                                                                                       \
-  hipLaunchKernelGGL((stream_norm_kernel<T, S, V>), dim3(nrows), dim3(NT), lds, st, x, (const T*)y, ids,            \
+  const size_t lds = (size_t)(((W + 3) & ~3) + 16) * sizeof(float);
+#define GO(V, NT)                                                                                                   \
+  hipLaunchKernelGGL((stream_norm_kernel<T, S, V, NT>), dim3(nrows), dim3(NT), lds, st, x, (const T*)y, ids,            \
                      (const T*)embed, rows, mix, out, m, in, w, (T*)normed, W, eps)
-  if (W % 4 == 0) GO(4);
-  else GO(1);
+  const bool wide = nrows <= 512 && W >= 2048;
+  if (W % 4 == 0 && wide) GO(4, 1024);
+  else if (W % 4 == 0) GO(4, 256);
+  else GO(1, 256);
 #undef GO
   DS_CHECK_LAUNCH();
   return 0;

@@ -25,16 +25,15 @@ __device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
 }
 
-// 4 consecutive elements of a row of d, zero beyond its end
+// 4 consecutive elements of a row padded to d (a multiple of 4), zero beyond its end; one unconditional access
 __device__ __forceinline__ f32x4 load4(const float* row, int k, int d) {
-  if ((d & 3) == 0) return k < d ? *reinterpret_cast<const f32x4*>(row + k) : f32x4{0.f, 0.f, 0.f, 0.f};
-  f32x4 v;
-#pragma unroll
-  for (int e = 0; e < 4; ++e) v[e] = k + e < d ? row[k + e] : 0.f;
-  return v;
+  const f32x4 v = *reinterpret_cast<const f32x4*>(row + min(k, d - 4));
+  const float z = k < d ? 1.f : 0.f;
+  return v * z;
 }
 
-template <typename T>
+// NK: 16-wide tiles of the key width (rounded up)
+template <typename T, int NK>
 __global__ void __launch_bounds__(NT) delta_chunk_kernel(
     const float* __restrict__ qk, const T* __restrict__ v, const float* __restrict__ gb, const int* __restrict__ cu,
     const int* __restrict__ work, float* __restrict__ Wo, float* __restrict__ Xo, float* __restrict__ Po,
@@ -62,22 +61,31 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
   }
   __syncthreads();
   // ---- K K^T and Q K^T, lower triangle of 16 x 16 tiles; wave w owns row tile w
-  const float* kbase = qk + (int64_t)D.Hk * D.dk + (int64_t)hk * D.dk;
-  const float* qbase = qk + (int64_t)hk * D.dk;
-  const int64_t rs = (int64_t)2 * D.Hk * D.dk;  // row stride of qk
+  const int dks = D.dks();
+  const float* kbase = qk + (int64_t)D.Hk * dks + (int64_t)hk * dks;
+  const float* qbase = qk + (int64_t)hk * dks;
+  const int64_t rs = (int64_t)2 * D.Hk * dks;  // row stride of qk
   const int64_t ri = (int64_t)(t0 + min(w * 16 + l16, n - 1)) * rs;
+  f32x4 ka[NK], qa[NK];
+#pragma unroll
+  for (int t = 0; t < NK; ++t) {
+    ka[t] = load4(kbase + ri, 16 * t + 4 * q4, dks);
+    qa[t] = load4(qbase + ri, 16 * t + 4 * q4, dks);
+  }
   for (int jt = 0; jt < 4; ++jt) {
     f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qq = {0.f, 0.f, 0.f, 0.f};
     if (jt <= w) {
       const int64_t rj = (int64_t)(t0 + min(jt * 16 + l16, n - 1)) * rs;
-      for (int k = 4 * q4; k < ((D.dk + 15) & ~15); k += 16) {
-        const f32x4 a = load4(kbase + ri, k, D.dk), q = load4(qbase + ri, k, D.dk), b = load4(kbase + rj, k, D.dk);
+      f32x4 kb[NK];
+#pragma unroll
+      for (int t = 0; t < NK; ++t) kb[t] = load4(kbase + rj, 16 * t + 4 * q4, dks);
+#pragma unroll
+      for (int t = 0; t < NK; ++t)
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          kk = mfma4(a[e], b[e], kk);
-          qq = mfma4(q[e], b[e], qq);
+          kk = mfma4(ka[t][e], kb[t][e], kk);
+          qq = mfma4(qa[t][e], kb[t][e], qq);
         }
-      }
     }
     float* prow = Po + base * C * C;
 #pragma unroll
@@ -106,22 +114,21 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
   __syncthreads();
   // ---- block forward substitution of [W | X], 16 columns per wave at a time: x_b = T_bb (r_b - sum_{c < b} A_bc x_c).
   // A product's result layout (row 4 q4 + r of column l16) is the next one's right operand as it stands.
-  const int wt = (D.dk + 15) / 16, xt = (D.dv + 15) / 16;
+  const int wt = (dks + 15) / 16, xt = (D.dv + 15) / 16;
   for (int ct = w; ct < wt + xt; ct += 4) {
     const bool isw = ct < wt;
-    const int col = (isw ? ct : ct - wt) * 16 + l16, width = isw ? D.dk : D.dv;
+    const int col = (isw ? ct : ct - wt) * 16 + l16, width = isw ? dks : D.dv;
+    const int cc = min(col, width - 1);
     f32x4 x[4];
 #pragma unroll
     for (int b = 0; b < 4; ++b)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int i = b * 16 + 4 * q4 + r;
-        float v0 = 0.f;
-        if (i < n && col < width) {
-          const int64_t t = t0 + i;
-          v0 = beta[i] * (isw ? kbase[t * rs + col] * eg[i] : (float)v[(t * D.H + h) * D.dv + col]);
-        }
-        x[b][r] = v0;
+        const int64_t t = t0 + min(i, n - 1);
+        // (rows past the end have beta 0, columns past it are not stored)
+        if (isw) x[b][r] = kbase[t * rs + cc] * (beta[i] * eg[i]);
+        else x[b][r] = (float)v[(t * D.H + h) * D.dv + cc] * beta[i];
       }
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
@@ -139,7 +146,7 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
       x[b] = y;
     }
     if (col < width) {
-      float* dst = (isw ? Wo + base * C * D.dk : Xo + base * C * D.dv) + col;
+      float* dst = (isw ? Wo + base * C * dks : Xo + base * C * D.dv) + col;
 #pragma unroll
       for (int b = 0; b < 4; ++b)
 #pragma unroll
@@ -148,7 +155,6 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
   }
 }
 
-// NK: 16-wide tiles of the key width (rounded up)
 template <typename T, int NK>
 __global__ void __launch_bounds__(NT) delta_scan_kernel(
     const float* __restrict__ qk, const T* __restrict__ proj, const float* __restrict__ Wo, const float* __restrict__ Xo,
@@ -166,26 +172,28 @@ __global__ void __launch_bounds__(NT) delta_scan_kernel(
     const int k = i % (NK * 16), j = i / (NK * 16);
     S[k][j] = (!fresh && k < D.dk && v0 + j < D.dv) ? st[(int64_t)(v0 + j) * D.dks() + k] : 0.f;
   }
-  const int64_t rs = (int64_t)2 * D.Hk * D.dk;
-  const float* qbase = qk + (int64_t)hk * D.dk;
-  const float* kbase = qbase + (int64_t)D.Hk * D.dk;
+  const int dks = D.dks();
+  const int64_t rs = (int64_t)2 * D.Hk * dks;
+  const float* qbase = qk + (int64_t)hk * dks;
+  const float* kbase = qbase + (int64_t)D.Hk * dks;
+  const int vc = min(v0 + l16, D.dv - 1);  // columns past the end compute what nobody stores
   constexpr int KT = (NK + 3) / 4;  // key tiles of the state per wave
   f32x4 wf[NK], qf[NK], pf[4];
   float kf[KT][16], xf[4], dq[4], du[4], dc = 0.f;
   auto fetch = [&](int c) {
     const int64_t base = (int64_t)(first + c) * D.H + h;
     const int row = w * 16 + l16, last = t0 + n - 1, tc = t0 + c * C;
-    const float* wr = Wo + (base * C + row) * D.dk;
+    const float* wr = Wo + (base * C + row) * dks;
     const float* qr = qbase + (int64_t)min(tc + row, last) * rs;
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk) {
-      wf[kk] = load4(wr, 16 * kk + 4 * q4, D.dk);
-      qf[kk] = load4(qr, 16 * kk + 4 * q4, D.dk);
+      wf[kk] = load4(wr, 16 * kk + 4 * q4, dks);
+      qf[kk] = load4(qr, 16 * kk + 4 * q4, dks);
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int i = w * 16 + 4 * q4 + r;
-      xf[r] = v0 + l16 < D.dv ? Xo[(base * C + i) * D.dv + v0 + l16] : 0.f;
+      xf[r] = Xo[(base * C + i) * D.dv + vc];
       dq[r] = dec[base * 2 * C + i];
       du[r] = dec[base * 2 * C + C + i];
       pf[r] = *reinterpret_cast<const f32x4*>(Po + (base * C + row) * C + 16 * r + 4 * q4);
@@ -197,7 +205,7 @@ __global__ void __launch_bounds__(NT) delta_scan_kernel(
 #pragma unroll
       for (int i = 0; i < 16; ++i) {  // k index of the product: token 16 (i / 4) + 4 q4 + i % 4
         const int tok = min(tc + 16 * (i >> 2) + 4 * q4 + (i & 3), last);
-        kf[kt][i] = d < D.dk ? kbase[(int64_t)tok * rs + d] : 0.f;
+        kf[kt][i] = kbase[(int64_t)tok * rs + min(d, dks - 1)] * (d < dks ? 1.f : 0.f);
       }
     }
   };
@@ -262,33 +270,48 @@ __global__ void __launch_bounds__(NT) delta_scan_kernel(
 }
 
 // out = o / rms(o) * w * silu(gate), one wave per (token, head) of the long sequences' chunks
-template <typename T>
+template <typename T, bool PAIR>
 __global__ void __launch_bounds__(NT) delta_norm_kernel(const float* __restrict__ o, const T* __restrict__ proj,
                                                         const float* __restrict__ norm_w, float eps,
                                                         const int* __restrict__ cu, const int* __restrict__ work,
                                                         T* __restrict__ out, DeltaDims D) {
   const int h = blockIdx.x % D.H, ci = blockIdx.x / D.H, lane = threadIdx.x & 63;
   const int seq = work[2 * ci], t0 = cu[seq] + work[2 * ci + 1] * C, n = min(C, cu[seq + 1] - t0);
-  for (int i = threadIdx.x >> 6; i < n; i += NT / 64) {
-    const int64_t t = t0 + i, at = (t * D.H + h) * D.dv;
-    const T* gate = proj + t * D.row() + D.channels() + h * D.dv;
-    float x[2][2], ss = 0.f;
+  float nw[2][2];
 #pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      const int c = k * 128 + 2 * lane;
-      load2(o + at + c, D.dv - c, x[k]);
-      ss = fmaf(x[k][0], x[k][0], fmaf(x[k][1], x[k][1], ss));
+  for (int k = 0; k < 2; ++k) load2<PAIR>(norm_w, k * 128 + 2 * lane, D.dv, nw[k]);
+  constexpr int UNR = 4;
+  for (int i0 = threadIdx.x >> 6; i0 < n; i0 += UNR * NT / 64) {
+    float x[UNR][2][2], g[UNR][2][2];
+#pragma unroll
+    for (int u = 0; u < UNR; ++u) {
+      const int64_t t = t0 + min(i0 + u * (NT / 64), n - 1);
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        x[u][k][0] = x[u][k][1] = 0.f;
+        if (k * 128 >= D.dv) continue;
+        const int c = k * 128 + 2 * lane;
+        load2<PAIR>(o + (t * D.H + h) * D.dv, c, D.dv, x[u][k]);
+        load2<PAIR>(proj + t * D.row() + D.channels() + h * D.dv, c, D.dv, g[u][k]);
+        x[u][k][0] *= c < D.dv ? 1.f : 0.f;
+        x[u][k][1] *= c + 1 < D.dv ? 1.f : 0.f;
+      }
     }
-    const float rms = 1.f / sqrtf(wave_sum(ss) / (float)D.dv + eps);
 #pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      const int c = k * 128 + 2 * lane;
-      float g[2], nw[2];
-      load2(gate + c, D.dv - c, g);
-      load2(norm_w + c, D.dv - c, nw);
+    for (int u = 0; u < UNR; ++u) {
+      const int i = i0 + u * (NT / 64);
+      if (i >= n) break;
+      float ss = 0.f;
 #pragma unroll
-      for (int e = 0; e < 2; ++e) g[e] = x[k][e] * rms * nw[e] * silu(g[e]);
-      store2(out + at + c, D.dv - c, g);
+      for (int k = 0; k < 2; ++k) ss = fmaf(x[u][k][0], x[u][k][0], fmaf(x[u][k][1], x[u][k][1], ss));
+      const float rms = 1.f / sqrtf(wave_sum(ss) / (float)D.dv + eps);
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        if (k * 128 >= D.dv) continue;
+#pragma unroll
+        for (int e = 0; e < 2; ++e) g[u][k][e] = x[u][k][e] * rms * nw[k][e] * silu(g[u][k][e]);
+        store2<PAIR>(out + ((int64_t)(t0 + i) * D.H + h) * D.dv, k * 128 + 2 * lane, D.dv, g[u][k]);
+      }
     }
   }
 }
@@ -298,24 +321,30 @@ int run(const float* qk, const void* v, const float* gb, const void* proj, const
         void* conv_state, const int* seqs, int nseq, const int* work, int nwork, const int* cu, const int* start,
         const int* slots, float* ws, float* o, void* out, DeltaDims D, hipStream_t st) {
   float* W = ws;
-  float* X = W + (int64_t)nwork * D.H * C * D.dk;
+  float* X = W + (int64_t)nwork * D.H * C * D.dks();
   float* P = X + (int64_t)nwork * D.H * C * D.dv;
   float* dec = P + (int64_t)nwork * D.H * C * C;
-  hipLaunchKernelGGL((delta_chunk_kernel<T>), dim3(nwork * D.H), dim3(NT), 0, st, qk, (const T*)v, gb, cu, work, W, X, P,
-                     dec, D);
-  DS_CHECK_LAUNCH();
   const dim3 grid((D.dv + 15) / 16, D.H, nseq);
 #define GO(NK)                                                                                                       \
-  hipLaunchKernelGGL((delta_scan_kernel<T, NK>), grid, dim3(NT), 0, st, qk, (const T*)proj, W, X, P, dec, seqs, cu, start, \
-                     slots, state, (T*)conv_state, o, D)
-  if (D.dk <= 32) GO(2);
-  else if (D.dk <= 64) GO(4);
-  else if (D.dk <= 128) GO(8);
-  else GO(16);
+  {                                                                                                                  \
+    hipLaunchKernelGGL((delta_chunk_kernel<T, NK>), dim3(nwork * D.H), dim3(NT), 0, st, qk, (const T*)v, gb, cu, work, \
+                       W, X, P, dec, D);                                                                             \
+    DS_CHECK_LAUNCH();                                                                                               \
+    hipLaunchKernelGGL((delta_scan_kernel<T, NK>), grid, dim3(NT), 0, st, qk, (const T*)proj, W, X, P, dec, seqs, cu,  \
+                       start, slots, state, (T*)conv_state, o, D);                                                   \
+  }
+  if (D.dk <= 32) GO(2)
+  else if (D.dk <= 64) GO(4)
+  else if (D.dk <= 128) GO(8)
+  else GO(16)
 #undef GO
   DS_CHECK_LAUNCH();
-  hipLaunchKernelGGL((delta_norm_kernel<T>), dim3(nwork * D.H), dim3(NT), 0, st, o, (const T*)proj, norm_w, eps, cu, work,
-                     (T*)out, D);
+#define NORM(PAIR)                                                                                                   \
+  hipLaunchKernelGGL((delta_norm_kernel<T, PAIR>), dim3(nwork * D.H), dim3(NT), 0, st, o, (const T*)proj, norm_w, eps, \
+                     cu, work, (T*)out, D)
+  if (D.dv % 2 == 0 && D.dk % 2 == 0) NORM(true);
+  else NORM(false);
+#undef NORM
   DS_CHECK_LAUNCH();
   return 0;
 }
@@ -324,7 +353,7 @@ int run(const float* qk, const void* v, const float* gb, const void* proj, const
 
 // fp32 words of workspace a call needs
 extern "C" int64_t ds_delta_chunk_ws(int nwork, int H, int dk, int dv) {
-  return (int64_t)nwork * H * C * (dk + dv + C + 2);
+  return (int64_t)nwork * H * C * ((dk + 3) / 4 * 4 + dv + C + 2);
 }
 
 // seqs [nseq, 2]: (sequence, index of its first entry in work); work [nwork, 2]: (sequence, chunk), a sequence's chunks

@@ -6,38 +6,38 @@ namespace {
 
 __device__ __forceinline__ float silu(float x) { return x / (1.f + expf(-x)); }
 
-// Two adjacent elements (zero / nothing beyond `left` of them); one access when the address allows.
-template <typename T>
-__device__ __forceinline__ void load2(const T* p, int left, float (&v)[2]) {
+// Elements c, c + 1 of a row of `width` (c even); where c lies beyond the row, some element of it (the caller drops it).
+// PAIR: rows are even and pair-aligned, so this is one unconditional access.
+template <bool PAIR, typename T>
+__device__ __forceinline__ void load2(const T* row, int c, int width, float (&v)[2]) {
   typedef T T2 __attribute__((ext_vector_type(2)));
-  v[0] = v[1] = 0.f;
-  if (left >= 2 && (reinterpret_cast<uintptr_t>(p) & (2 * sizeof(T) - 1)) == 0) {
-    const T2 a = *reinterpret_cast<const T2*>(p);
+  if constexpr (PAIR) {
+    const T2 a = *reinterpret_cast<const T2*>(row + min(c, width - 2));
     v[0] = (float)a[0];
     v[1] = (float)a[1];
-  } else if (left > 0) {
-    v[0] = (float)p[0];
-    if (left > 1) v[1] = (float)p[1];
+  } else {
+    v[0] = (float)row[min(c, width - 1)];
+    v[1] = (float)row[min(c + 1, width - 1)];
   }
 }
-template <typename T>
-__device__ __forceinline__ void store2(T* p, int left, const float (&v)[2]) {
+template <bool PAIR, typename T>
+__device__ __forceinline__ void store2(T* row, int c, int width, const float (&v)[2]) {
   typedef T T2 __attribute__((ext_vector_type(2)));
-  if (left >= 2 && (reinterpret_cast<uintptr_t>(p) & (2 * sizeof(T) - 1)) == 0) {
+  if constexpr (PAIR) {
     T2 a;
     a[0] = (T)v[0];
     a[1] = (T)v[1];
-    *reinterpret_cast<T2*>(p) = a;
-  } else if (left > 0) {
-    p[0] = (T)v[0];
-    if (left > 1) p[1] = (T)v[1];
+    if (c < width) *reinterpret_cast<T2*>(row + c) = a;
+  } else {
+    if (c < width) row[c] = (T)v[0];
+    if (c + 1 < width) row[c + 1] = (T)v[1];
   }
 }
 
 struct DeltaDims {
   int Hk, H, dk, dv, taps;
   __host__ __device__ int channels() const { return 2 * Hk * dk + H * dv; }
-  __host__ __device__ int dks() const { return (dk + 3) & ~3; }  // key width as the state is stored (padded with zeros)
+  __host__ __device__ int dks() const { return (dk + 3) & ~3; }  // key width as q, k and the state are stored (zero padded)
   __host__ __device__ int row() const { return channels() + H * dv + 2 * H; }
 };
 

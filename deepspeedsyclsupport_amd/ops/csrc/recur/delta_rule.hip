@@ -21,8 +21,8 @@ namespace {
 
 constexpr int TILE = 8;  // consecutive tokens a prepare wave walks
 
-// TAPS: filter length held in registers (the window slides from token to token); 0: any length, read afresh per token
-template <typename T, int TAPS>
+// TAPS: filter length, the tile's inputs in registers; 0: any length, inputs read per tap. PAIR: even head sizes.
+template <typename T, int TAPS, bool PAIR>
 __global__ void __launch_bounds__(256) delta_prepare_kernel(
     const T* __restrict__ proj, const float* __restrict__ conv_w, const T* __restrict__ conv_state,
     const float* __restrict__ a_log, const float* __restrict__ dt_bias, const int* __restrict__ seq_ids,
@@ -31,6 +31,7 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(
   const int parts = 2 * D.Hk + D.H + 1, lane = threadIdx.x & 63;
   const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   const int t_lo = (int)(item / parts) * tile, part = (int)(item % parts), t_hi = min(t_lo + tile, tokens);
+  if (t_lo >= tokens) return;
   const int NP = D.row(), CH = D.channels(), taps = TAPS ? TAPS : D.taps;
   if (part == parts - 1) {  // decays (as logarithms) and write strengths
     for (int t = t_lo; t < t_hi; ++t) {
@@ -47,94 +48,91 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(
   const bool is_v = part >= 2 * D.Hk;
   const int width = is_v ? D.dv : D.dk;
   const int c0 = is_v ? 2 * D.Hk * D.dk + (part - 2 * D.Hk) * D.dv : part * D.dk;
-  // a lane's channels: 2 lane, 2 lane + 1, and the same 128 further on
-  float cw[2][2][TAPS ? TAPS : 1], win[2][2][TAPS ? TAPS : 1];
-  if constexpr (TAPS != 0) {
+  for (int ta = t_lo; ta < t_hi;) {  // runs of tokens of one sequence
+    const int seq = seq_ids[ta], first = cu[seq], tb = min(t_hi, cu[seq + 1]), n = tb - ta, j0 = ta - first;
+    const T* cs = start[seq] == 0 ? nullptr : conv_state + (int64_t)slots[seq] * (taps - 1) * CH;
+    // the convolution's input row at place j of the portion (negative: before it); zero tells that there is none
+    auto row = [&](int j, float& zero) {
+      zero = j >= 0 || cs ? 1.f : 0.f;
+      return j >= 0 || !cs ? proj + (int64_t)(first + max(j, 0)) * NP + c0 : cs + (int64_t)(j + taps - 1) * CH + c0;
+    };
+    float y[TILE][2][2];
 #pragma unroll
-    for (int k = 0; k < 2; ++k)
+    for (int k = 0; k < 2; ++k) {  // a lane's channels: 2 lane, 2 lane + 1, and the same 128 further on
+      const int c = k * 128 + 2 * lane;
+      if (k * 128 >= width) {
 #pragma unroll
-      for (int e = 0; e < 2; ++e) {
-        const int c = k * 128 + 2 * lane + e;
+        for (int t = 0; t < TILE; ++t) y[t][k][0] = y[t][k][1] = 0.f;
+      } else if constexpr (TAPS != 0) {
+        float x[TILE + TAPS - 1][2], cw[2][TAPS];
 #pragma unroll
-        for (int i = 0; i < TAPS; ++i) cw[k][e][i] = c < width ? conv_w[(int64_t)(c0 + c) * TAPS + i] : 0.f;
-      }
-  }
-  int seq = -1, first = 0;
-  const T* cs = nullptr;
-  // input of the convolution at place j of the portion (negative: before it)
-  auto input = [&](int j, int k, float (&x)[2]) {
-    const int c = k * 128 + 2 * lane;
-    x[0] = x[1] = 0.f;
-    if (c >= width) return;
-    if (j >= 0) load2(proj + (int64_t)(first + j) * NP + c0 + c, width - c, x);
-    else if (cs) load2(cs + (int64_t)(j + taps - 1) * CH + c0 + c, width - c, x);
-  };
-  for (int t = t_lo; t < t_hi; ++t) {
-    const bool fill = t == t_lo || seq_ids[t] != seq;
-    if (fill) {
-      seq = seq_ids[t];
-      first = cu[seq];
-      cs = start[seq] == 0 ? nullptr : conv_state + (int64_t)slots[seq] * (taps - 1) * CH;
-    }
-    const int j = t - first;
-    float y[2][2];
+        for (int i = 0; i < TILE + TAPS - 1; ++i) {
+          float zero;
+          const T* r = row(j0 + min(i, n + TAPS - 2) - (TAPS - 1), zero);
+          load2<PAIR>(r, c, width, x[i]);
+          x[i][0] *= zero;
+          x[i][1] *= zero;
+        }
 #pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      float acc[2] = {0.f, 0.f};
-      if (k * 128 < width) {
-        float x[2];
-        if constexpr (TAPS != 0) {
-          if (fill) {
+        for (int e = 0; e < 2; ++e)
 #pragma unroll
-            for (int i = 1; i < TAPS; ++i) {
-              input(j - TAPS + i, k, x);
-              win[k][0][i] = x[0];
-              win[k][1][i] = x[1];
-            }
-          }
-          input(j, k, x);
+          for (int i = 0; i < TAPS; ++i)
+            cw[e][i] = conv_w[(int64_t)(c0 + min(c + e, width - 1)) * TAPS + i] * (c + e < width ? 1.f : 0.f);
+#pragma unroll
+        for (int t = 0; t < TILE; ++t)
 #pragma unroll
           for (int e = 0; e < 2; ++e) {
+            float acc = 0.f;
 #pragma unroll
-            for (int i = 0; i + 1 < TAPS; ++i) win[k][e][i] = win[k][e][i + 1];
-            win[k][e][TAPS - 1] = x[e];
-#pragma unroll
-            for (int i = 0; i < TAPS; ++i) acc[e] = fmaf(cw[k][e][i], win[k][e][i], acc[e]);
+            for (int i = 0; i < TAPS; ++i) acc = fmaf(cw[e][i], x[t + i][e], acc);
+            y[t][k][e] = silu(acc);  // 0 beyond the width
           }
-        } else {
-          for (int i = 0; i < taps; ++i) {
-            input(j - (taps - 1) + i, k, x);
+      } else {
+        float acc[TILE][2];
 #pragma unroll
-            for (int e = 0; e < 2; ++e) {
-              const int c = k * 128 + 2 * lane + e;
-              if (c < width) acc[e] = fmaf(conv_w[(int64_t)(c0 + c) * taps + i], x[e], acc[e]);
-            }
+        for (int t = 0; t < TILE; ++t) acc[t][0] = acc[t][1] = 0.f;
+        for (int i = 0; i < taps; ++i) {
+          const float w0 = c < width ? conv_w[(int64_t)(c0 + c) * taps + i] : 0.f;
+          const float w1 = c + 1 < width ? conv_w[(int64_t)(c0 + c + 1) * taps + i] : 0.f;
+#pragma unroll
+          for (int t = 0; t < TILE; ++t) {
+            float zero, x[2];
+            const T* r = row(j0 + min(t, n - 1) - (taps - 1) + i, zero);
+            load2<PAIR>(r, c, width, x);
+            acc[t][0] = fmaf(w0, x[0] * zero, acc[t][0]);
+            acc[t][1] = fmaf(w1, x[1] * zero, acc[t][1]);
           }
         }
+#pragma unroll
+        for (int t = 0; t < TILE; ++t) {
+          y[t][k][0] = silu(acc[t][0]);
+          y[t][k][1] = silu(acc[t][1]);
+        }
       }
-      y[k][0] = silu(acc[0]);
-      y[k][1] = silu(acc[1]);
     }
-    if (is_v) {
+#pragma unroll
+    for (int t = 0; t < TILE; ++t) {
+      if (t >= n) break;
+      const int64_t tok = ta + t;
+      if (is_v) {
+#pragma unroll
+        for (int k = 0; k < 2; ++k)
+          store2<PAIR>(v_out + (tok * D.H + part - 2 * D.Hk) * D.dv, k * 128 + 2 * lane, width, y[t][k]);
+        continue;
+      }
+      float ss = 0.f;
+#pragma unroll
+      for (int k = 0; k < 2; ++k) ss = fmaf(y[t][k][0], y[t][k][0], fmaf(y[t][k][1], y[t][k][1], ss));
+      float r = 1.f / sqrtf(wave_sum(ss) + 1e-6f);
+      if (part < D.Hk) r *= 1.f / sqrtf((float)D.dk);
 #pragma unroll
       for (int k = 0; k < 2; ++k) {
-        const int c = k * 128 + 2 * lane;
-        store2(v_out + ((int64_t)t * D.H + part - 2 * D.Hk) * D.dv + c, width - c, y[k]);
+        y[t][k][0] *= r;
+        y[t][k][1] *= r;
+        store2<true>(qk + (tok * 2 * D.Hk + part) * D.dks(), k * 128 + 2 * lane, D.dks(), y[t][k]);
       }
-      continue;
     }
-    float ss = 0.f;
-#pragma unroll
-    for (int k = 0; k < 2; ++k) ss = fmaf(y[k][0], y[k][0], fmaf(y[k][1], y[k][1], ss));  // silu(0) = 0 in the padding
-    float r = 1.f / sqrtf(wave_sum(ss) + 1e-6f);
-    if (part < D.Hk) r *= 1.f / sqrtf((float)D.dk);
-#pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      const int c = k * 128 + 2 * lane;
-      y[k][0] *= r;
-      y[k][1] *= r;
-      store2(qk + ((int64_t)t * 2 * D.Hk + part) * D.dk + c, width - c, y[k]);
-    }
+    ta = tb;
   }
 }
 
@@ -166,8 +164,8 @@ __global__ void __launch_bounds__(1024) delta_recur_kernel(
   }
   for (int t = 0; t < n; ++t) {
     const int64_t tok = t0 + t;
-    const float* qr = qk + (tok * 2 * D.Hk + hk) * D.dk;
-    const float* kr = qr + (int64_t)D.Hk * D.dk;
+    const float* qr = qk + (tok * 2 * D.Hk + hk) * D.dks();
+    const float* kr = qr + (int64_t)D.Hk * D.dks();
     __syncthreads();
     for (int c = tid; c < KP; c += blockDim.x) {
       qs[c] = c < D.dk ? qr[c] : 0.f;
@@ -256,16 +254,18 @@ extern "C" int ds_delta_prepare(const void* proj, const float* conv_w, const voi
   if (!dims_ok(D)) return (int)hipErrorInvalidValue;
   const int tile = tokens >= 512 ? TILE : 1;  // few tokens: as many waves as there are
   const int64_t items = (int64_t)((tokens + tile - 1) / tile) * (2 * Hk + H + 1);
-#define LAUNCH(T, TAPS)                                                                                             \
-  hipLaunchKernelGGL((delta_prepare_kernel<T, TAPS>), dim3((unsigned)((items + 3) / 4)), dim3(256), 0, st,            \
+  const bool pair = dk % 2 == 0 && dv % 2 == 0;
+#define LAUNCH(T, TAPS, PAIR)                                                                                       \
+  hipLaunchKernelGGL((delta_prepare_kernel<T, TAPS, PAIR>), dim3((unsigned)((items + 3) / 4)), dim3(256), 0, st,      \
                      (const T*)proj, conv_w, (const T*)conv_state, a_log, dt_bias, seq_ids, cu, start, slots, qk, (T*)v, gb, \
                      tokens, tile, D)
-#define GO(T)                     \
-  {                               \
-    if (taps == 4) LAUNCH(T, 4);  \
-    else if (taps == 3) LAUNCH(T, 3); \
-    else if (taps == 2) LAUNCH(T, 2); \
-    else LAUNCH(T, 0);            \
+#define GO(T)                                  \
+  {                                            \
+    if (!pair) LAUNCH(T, 0, false);            \
+    else if (taps == 4) LAUNCH(T, 4, true);    \
+    else if (taps == 3) LAUNCH(T, 3, true);    \
+    else if (taps == 2) LAUNCH(T, 2, true);    \
+    else LAUNCH(T, 0, true);                   \
   }
   if (dtype == DS_F32) GO(float)
   else if (dtype == DS_BF16) GO(bf16)

@@ -58,10 +58,10 @@ def delta_rule(proj, conv_w, a_log, dt_bias, norm_w, eps, state, conv_state, met
                                   meta.slots, Hk, H, dk, dv)
     if meta.seq_list.numel():
         ops.delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, meta.seq_list, meta.cu_q, meta.start_pos,
-                        meta.slots, out)
+                        meta.slots, out, dk)
     if meta.chunk_work.numel():
         ops.delta_chunk(qk, v, gb, proj, norm_w, eps, state, conv_state, meta.chunk_seqs, meta.chunk_work, meta.cu_q,
-                        meta.start_pos, meta.slots, out)
+                        meta.start_pos, meta.slots, out, dk)
     return out
 
 

@@ -204,9 +204,9 @@ def delta_prepare(proj, conv_w, conv_state, a_log, dt_bias, seq_ids, cu, start, 
     return torch.stack([q, k], 1), v.view(T, H, dv).to(proj.dtype), torch.stack([glog, b.sigmoid()], 1)
 
 
-def delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, cu, start, slots, out):
+def delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, cu, start, slots, out, dk):
     T, H, dv = v.shape
-    Hk, dk = qk.shape[2], qk.shape[3]
+    Hk = qk.shape[2]
     C, taps = conv_state.shape[2], conv_state.shape[1] + 1
     out = out.view(T, H, dv)
     rep = H // Hk
@@ -227,6 +227,6 @@ def delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, cu, start
             conv_state[slot] = torch.cat([old, proj[a:b, :C]])[-(taps - 1):].clone()
 
 
-def delta_chunk(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, work, cu, start, slots, out):
+def delta_chunk(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, work, cu, start, slots, out, dk):
     """Long portions: the same recurrence (the device splits it into chunks)."""
-    delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs[:, 0], cu, start, slots, out)
+    delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs[:, 0], cu, start, slots, out, dk)
