@@ -47,11 +47,72 @@ __global__ void __launch_bounds__(256) qk_norm_append_kernel(
   for (int c = lane; c < dk; c += 64) dst[c] = (T)((float)src[c] * rs * w[c]);
 }
 
+// The same for head widths that are multiples of 8: LPH lanes per head with 8 elements each, 64 / LPH heads per wave
+template <typename T, int LPH>
+__global__ void __launch_bounds__(256) qk_norm_append_vec_kernel(
+    const T* __restrict__ qkv, const float* __restrict__ qw, const float* __restrict__ kw, float eps,
+    const T* __restrict__ vfirst, int64_t vf_stride, const float* __restrict__ lambda, const int* __restrict__ pos,
+    const int* __restrict__ seq_ids, const int* __restrict__ block_table, int max_blocks, T* __restrict__ q_out,
+    T* __restrict__ kc, T* __restrict__ vc, int tokens, int H, int G, int dk, int dv, int BS) {
+  constexpr int HPB = 256 / LPH;
+  const int slots = H + 2 * G, li = threadIdx.x % LPH, c = li * 8;
+  const int64_t item = (int64_t)blockIdx.x * HPB + threadIdx.x / LPH;
+  if (item >= (int64_t)tokens * slots) return;  // whole lane groups
+  const int t = (int)(item / slots), h = (int)(item % slots);
+  const T* row = qkv + (int64_t)t * ((int64_t)(H + G) * dk + (int64_t)G * dv);
+  const bool is_v = h >= H + G;
+  const int width = is_v ? dv : dk;
+  const T* src = row + (is_v ? (int64_t)(H + G) * dk + (int64_t)(h - H - G) * dv : (int64_t)h * dk);
+  int64_t slot = 0;
+  if (h >= H) {
+    const int p = pos[t], g = is_v ? h - H - G : h - H;
+    slot = ((int64_t)block_table[(int64_t)seq_ids[t] * max_blocks + p / BS] * G + g) * BS + p % BS;
+  }
+  const bool on = c < width;
+  float x[8];
+  Vec8<T>::load(src + (on ? c : 0), x);
+  if (is_v) {
+    if (vfirst) {
+      const float lam = lambda[0];
+      const T* vf = vfirst + (int64_t)t * vf_stride + (int64_t)(h - H - G) * dv + (on ? c : 0);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] = (1.f - lam) * x[j] + lam * (float)vf[j];
+    }
+    if (on) Vec8<T>::store(vc + slot * dv + c, x);
+    return;
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) ss = fmaf(x[j], x[j], ss);
+  if (!on) ss = 0.f;
+#pragma unroll
+  for (int o = LPH / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+  const float rs = 1.f / sqrtf(ss / (float)dk + eps);
+  if (!on) return;
+  float w[8];
+  Vec8<float>::load((h < H ? qw : kw) + c, w);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) x[j] *= rs * w[j];
+  Vec8<T>::store((h < H ? q_out + ((int64_t)t * H + h) * dk : kc + slot * dk) + c, x);
+}
+
 template <typename T>
 int launch(const void* qkv, const float* qw, const float* kw, float eps, const void* vfirst, int64_t vf_stride,
            const float* lambda, const int* pos, const int* seq_ids, const int* bt, int max_blocks, void* q, void* kc,
            void* vc, int tokens, int H, int G, int dk, int dv, int BS, hipStream_t st) {
   const int64_t items = (int64_t)tokens * (H + 2 * G);
+  if (dk % 8 == 0 && dv % 8 == 0 && dk <= 256 && dv <= 256) {
+#define VEC(LPH)                                                                                                    \
+  hipLaunchKernelGGL((qk_norm_append_vec_kernel<T, LPH>), dim3((unsigned)((items * LPH + 255) / 256)), dim3(256), 0, st, \
+                     (const T*)qkv, qw, kw, eps, (const T*)vfirst, vf_stride, lambda, pos, seq_ids, bt, max_blocks, (T*)q, \
+                     (T*)kc, (T*)vc, tokens, H, G, dk, dv, BS)
+    if (dk <= 64 && dv <= 64) VEC(8);
+    else if (dk <= 128 && dv <= 128) VEC(16);
+    else VEC(32);
+#undef VEC
+    DS_CHECK_LAUNCH();
+    return 0;
+  }
   hipLaunchKernelGGL((qk_norm_append_kernel<T>), dim3((unsigned)((items + 3) / 4)), dim3(256), 0, st, (const T*)qkv, qw,
                      kw, eps, (const T*)vfirst, vf_stride, lambda, pos, seq_ids, bt, max_blocks, (T*)q, (T*)kc, (T*)vc,
                      tokens, H, G, dk, dv, BS);

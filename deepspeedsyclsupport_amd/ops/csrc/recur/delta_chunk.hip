@@ -41,7 +41,8 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
   __shared__ __attribute__((aligned(16))) float A[C][C + 4];
   __shared__ double G[C];
   __shared__ float beta[C], eg[C];
-  const int h = blockIdx.x % D.H, ci = blockIdx.x / D.H, hk = h / (D.H / D.Hk);
+  const int bid = xcd_remap(blockIdx.x, gridDim.x);  // the heads of a key group share its rows in one L2
+  const int h = bid % D.H, ci = bid / D.H, hk = h / (D.H / D.Hk);
   const int seq = work[2 * ci], c = work[2 * ci + 1];
   const int t0 = cu[seq] + c * C, n = min(C, cu[seq + 1] - t0);
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, l16 = lane & 15, q4 = lane >> 4;
@@ -163,7 +164,9 @@ __global__ void __launch_bounds__(NT) delta_scan_kernel(
     float* __restrict__ o, DeltaDims D) {
   __shared__ float S[NK * 16][17];
   __shared__ float U[C][17];
-  const int vt = blockIdx.x, h = blockIdx.y, seq = seqs[2 * blockIdx.z], first = seqs[2 * blockIdx.z + 1];
+  // the value tiles of a head walk the same W, P, q and k: neighbours in one XCD's L2
+  const int bid = xcd_remap(blockIdx.x, gridDim.x), vts = (D.dv + 15) / 16;
+  const int vt = bid % vts, h = bid / vts % D.H, sq = bid / (vts * D.H), seq = seqs[2 * sq], first = seqs[2 * sq + 1];
   const int hk = h / (D.H / D.Hk), tid = threadIdx.x, lane = tid & 63, w = tid >> 6, l16 = lane & 15, q4 = lane >> 4;
   const int t0 = cu[seq], n = cu[seq + 1] - t0, nc = (n + C - 1) / C, v0 = vt * 16;
   const bool fresh = start[seq] == 0;
@@ -324,7 +327,7 @@ int run(const float* qk, const void* v, const float* gb, const void* proj, const
   float* X = W + (int64_t)nwork * D.H * C * D.dks();
   float* P = X + (int64_t)nwork * D.H * C * D.dv;
   float* dec = P + (int64_t)nwork * D.H * C * C;
-  const dim3 grid((D.dv + 15) / 16, D.H, nseq);
+  const dim3 grid((unsigned)((D.dv + 15) / 16 * D.H * nseq));
 #define GO(NK)                                                                                                       \
   {                                                                                                                  \
     hipLaunchKernelGGL((delta_chunk_kernel<T, NK>), dim3(nwork * D.H), dim3(NT), 0, st, qk, (const T*)v, gb, cu, work, \
@@ -364,7 +367,7 @@ extern "C" int ds_delta_chunk(const float* qk, const void* v, const float* gb, c
                               void* out, int Hk, int H, int dk, int dv, int taps, int dtype, hipStream_t st) {
   if (nseq <= 0 || nwork <= 0) return 0;
   const DeltaDims D{Hk, H, dk, dv, taps};
-  if (!dims_ok(D) || H > 65535 || nseq > 65535) return (int)hipErrorInvalidValue;
+  if (!dims_ok(D) || (int64_t)nwork * H * 16 > INT32_MAX) return (int)hipErrorInvalidValue;
   if (dtype == DS_F32)
     return run<float>(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, nseq, work, nwork, cu, start, slots, ws, o,
                       out, D, st);
