@@ -18,11 +18,11 @@ int ds_paged_generic(const void*, const void*, const void*, void*, const int*, i
 int ds_delta_prepare(const void*, const float*, const void*, const float*, const float*, const int*, const int*,
                      const int*, const int*, float*, void*, float*, int, int, int, int, int, int, int, hipStream_t);
 int ds_delta_recur(const float*, const void*, const float*, const void*, const float*, float, float*, void*, const int*,
-                   int, const int*, const int*, const int*, void*, int, int, int, int, int, int, hipStream_t);
+                   int, const int*, const int*, const int*, void*, int, int, int, int, int, int, int, hipStream_t);
 int64_t ds_delta_chunk_ws(int, int, int, int);
 int ds_delta_chunk(const float*, const void*, const float*, const void*, const float*, float, float*, void*, const int*,
                    int, const int*, int, const int*, const int*, const int*, float*, float*, void*, int, int, int, int,
-                   int, int, hipStream_t);
+                   int, int, int, hipStream_t);
 int ds_paged_prefill_ext(const void*, const void*, const void*, void*, const int*, const int*, const int*, const int*, int,
                          int, int, int, int, int, int, int, int, float, float, hipStream_t);
 int ds_paged_decode_splits(int, int, int);
@@ -219,7 +219,7 @@ void delta_dims_ok(int64_t Hk, int64_t H, int64_t dk, int64_t dv, int64_t taps) 
   TORCH_CHECK(dk <= 256 && dv <= 256, "delta rule: head sizes up to 256");
 }
 
-// proj [T, 2 Hk dk + 2 H dv + 2 H] -> (qk fp32 [T, 2, Hk, dk padded to 4], v [T, H, dv], gb fp32 [T, 2, H]: log decay, beta)
+// proj [T, 2 Hk dk + 2 H dv + 2 H] -> (qk fp32 [2, Hk, T, dk padded to 4], v [H, T, dv], gb fp32 [T, 2, H]: log decay, beta)
 std::vector<Tensor> delta_prepare(Tensor proj, Tensor conv_w, Tensor conv_state, Tensor a_log, Tensor dt_bias,
                                   Tensor seq_ids, Tensor cu, Tensor start, Tensor slots, int64_t Hk, int64_t H, int64_t dk,
                                   int64_t dv) {
@@ -231,8 +231,8 @@ std::vector<Tensor> delta_prepare(Tensor proj, Tensor conv_w, Tensor conv_state,
               conv_state.scalar_type() == proj.scalar_type(), "delta_prepare: conv_state [slots, taps-1, C]");
   const int64_t S = start.numel();
   auto fo = proj.options().dtype(at::kFloat);
-  auto qk = torch::empty({T, 2, Hk, (dk + 3) / 4 * 4}, fo);  // zero padded rows
-  auto v = torch::empty({T, H, dv}, proj.options());
+  auto qk = torch::empty({2, Hk, T, (dk + 3) / 4 * 4}, fo);  // zero padded rows
+  auto v = torch::empty({H, T, dv}, proj.options());
   auto gb = torch::empty({T, 2, H}, fo);
   check(ds_delta_prepare(proj.data_ptr(), f32(conv_w, C * taps, "conv_w"), conv_state.data_ptr(), f32(a_log, H, "A_log"),
                          f32(dt_bias, H, "dt_bias"), i32(seq_ids, T, "seq_ids"), i32(cu, S + 1, "cu"),
@@ -246,7 +246,7 @@ std::vector<Tensor> delta_prepare(Tensor proj, Tensor conv_w, Tensor conv_state,
 void delta_recur(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, double eps, Tensor state, Tensor conv_state,
                  Tensor list, Tensor cu, Tensor start, Tensor slots, Tensor out, int64_t dk) {
   need(proj, "proj"); need(v, "v"); need(state, "state"); need(conv_state, "conv_state"); need(out, "out");
-  const int64_t T = v.size(0), H = v.size(1), dv = v.size(2), Hk = qk.size(2), S = start.numel();
+  const int64_t T = v.size(1), H = v.size(0), dv = v.size(2), Hk = qk.size(1), S = start.numel();
   const int64_t taps = conv_state.size(1) + 1;
   delta_dims_ok(Hk, H, dk, dv, taps);
   TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == H && state.size(2) == dv &&
@@ -258,8 +258,8 @@ void delta_recur(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, dou
   check(ds_delta_recur(f32(qk, T * 2 * Hk * ((dk + 3) / 4 * 4), "qk"), v.data_ptr(), f32(gb, T * 2 * H, "gb"), proj.data_ptr(),
                        f32(norm_w, dv, "norm"), (float)eps, state.data_ptr<float>(), conv_state.data_ptr(),
                        i32(list, list.numel(), "list"), (int)list.numel(), i32(cu, S + 1, "cu"), i32(start, S, "start"),
-                       i32(slots, S, "slots"), out.data_ptr(), (int)Hk, (int)H, (int)dk, (int)dv, (int)taps, dcode(proj),
-                       stream()), "delta_recur");
+                       i32(slots, S, "slots"), out.data_ptr(), (int)T, (int)Hk, (int)H, (int)dk, (int)dv, (int)taps,
+                       dcode(proj), stream()), "delta_recur");
 }
 
 // The same for long portions, by chunks of 64 tokens: seqs [n, 2] (sequence, its first entry in work), work [m, 2]
@@ -267,7 +267,7 @@ void delta_recur(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, dou
 void delta_chunk(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, double eps, Tensor state, Tensor conv_state,
                  Tensor seqs, Tensor work, Tensor cu, Tensor start, Tensor slots, Tensor out, int64_t dk) {
   need(proj, "proj"); need(v, "v"); need(state, "state"); need(conv_state, "conv_state"); need(out, "out");
-  const int64_t T = v.size(0), H = v.size(1), dv = v.size(2), Hk = qk.size(2), S = start.numel();
+  const int64_t T = v.size(1), H = v.size(0), dv = v.size(2), Hk = qk.size(1), S = start.numel();
   const int64_t taps = conv_state.size(1) + 1;
   delta_dims_ok(Hk, H, dk, dv, taps);
   TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == H && state.size(2) == dv &&
@@ -280,12 +280,12 @@ void delta_chunk(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, dou
   const int64_t nw = work.size(0);
   auto fo = proj.options().dtype(at::kFloat);
   auto ws = torch::empty({ds_delta_chunk_ws((int)nw, (int)H, (int)dk, (int)dv)}, fo);
-  auto o = torch::empty({T, H, dv}, fo);
+  auto o = torch::empty({H, T, dv}, fo);
   check(ds_delta_chunk(f32(qk, T * 2 * Hk * ((dk + 3) / 4 * 4), "qk"), v.data_ptr(), f32(gb, T * 2 * H, "gb"), proj.data_ptr(),
                        f32(norm_w, dv, "norm"), (float)eps, state.data_ptr<float>(), conv_state.data_ptr(),
                        i32(seqs, seqs.numel(), "seqs"), (int)seqs.size(0), i32(work, work.numel(), "work"), (int)nw,
                        i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"), ws.data_ptr<float>(),
-                       o.data_ptr<float>(), out.data_ptr(), (int)Hk, (int)H, (int)dk, (int)dv, (int)taps, dcode(proj),
+                       o.data_ptr<float>(), out.data_ptr(), (int)T, (int)Hk, (int)H, (int)dk, (int)dv, (int)taps, dcode(proj),
                        stream()), "delta_chunk");
 }
 

@@ -25,11 +25,18 @@ __device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
 }
 
+// Workgroup barrier for LDS: earlier LDS accesses have completed, global loads may still be under way
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
 // 4 consecutive elements of a row padded to d (a multiple of 4), zero beyond its end; one unconditional access
 __device__ __forceinline__ f32x4 load4(const float* row, int k, int d) {
   const f32x4 v = *reinterpret_cast<const f32x4*>(row + min(k, d - 4));
   const float z = k < d ? 1.f : 0.f;
   return v * z;
+}
+// the same without the zeros, for products whose other operand has them: the value is not touched before its use
+__device__ __forceinline__ f32x4 load4_raw(const float* row, int k, int d) {
+  return *reinterpret_cast<const f32x4*>(row + min(k, d - 4));
 }
 
 // NK: 16-wide tiles of the key width (rounded up)
@@ -63,9 +70,9 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
   __syncthreads();
   // ---- K K^T and Q K^T, lower triangle of 16 x 16 tiles; wave w owns row tile w
   const int dks = D.dks();
-  const float* kbase = qk + (int64_t)D.Hk * dks + (int64_t)hk * dks;
-  const float* qbase = qk + (int64_t)hk * dks;
-  const int64_t rs = (int64_t)2 * D.Hk * dks;  // row stride of qk
+  const float* kbase = qk + D.k_at(hk, 0);
+  const float* qbase = qk + D.q_at(hk, 0);
+  const int64_t rs = dks;
   const int64_t ri = (int64_t)(t0 + min(w * 16 + l16, n - 1)) * rs;
   f32x4 ka[NK], qa[NK];
 #pragma unroll
@@ -129,7 +136,7 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
         const int64_t t = t0 + min(i, n - 1);
         // (rows past the end have beta 0, columns past it are not stored)
         if (isw) x[b][r] = kbase[t * rs + cc] * (beta[i] * eg[i]);
-        else x[b][r] = (float)v[(t * D.H + h) * D.dv + cc] * beta[i];
+        else x[b][r] = (float)v[D.v_at(h, t) + cc] * beta[i];
       }
 #pragma unroll
     for (int b = 0; b < 4; ++b) {
@@ -157,13 +164,14 @@ __global__ void __launch_bounds__(NT) delta_chunk_kernel(
 }
 
 template <typename T, int NK>
-__global__ void __launch_bounds__(NT) delta_scan_kernel(
+__global__ void __launch_bounds__(NT, (NK <= 8 ? 2 : 1)) delta_scan_kernel(
     const float* __restrict__ qk, const T* __restrict__ proj, const float* __restrict__ Wo, const float* __restrict__ Xo,
     const float* __restrict__ Po, const float* __restrict__ dec, const int* __restrict__ seqs, const int* __restrict__ cu,
     const int* __restrict__ start, const int* __restrict__ slots, float* __restrict__ state, T* __restrict__ conv_state,
     float* __restrict__ o, DeltaDims D) {
-  __shared__ float S[NK * 16][17];
-  __shared__ float U[C][17];
+  constexpr int LD = 20;  // the four row groups of an operand read (4 rows apart) fall on different banks
+  __shared__ float S[NK * 16][LD];
+  __shared__ float U[C][LD];
   // the value tiles of a head walk the same W, P, q and k: neighbours in one XCD's L2
   const int bid = xcd_remap(blockIdx.x, gridDim.x), vts = (D.dv + 15) / 16;
   const int vt = bid % vts, h = bid / vts % D.H, sq = bid / (vts * D.H), seq = seqs[2 * sq], first = seqs[2 * sq + 1];
@@ -176,45 +184,59 @@ __global__ void __launch_bounds__(NT) delta_scan_kernel(
     S[k][j] = (!fresh && k < D.dk && v0 + j < D.dv) ? st[(int64_t)(v0 + j) * D.dks() + k] : 0.f;
   }
   const int dks = D.dks();
-  const int64_t rs = (int64_t)2 * D.Hk * dks;
-  const float* qbase = qk + (int64_t)hk * dks;
-  const float* kbase = qbase + (int64_t)D.Hk * dks;
+  const int64_t rs = dks;
+  const float* qbase = qk + D.q_at(hk, 0);
+  const float* kbase = qk + D.k_at(hk, 0);
   const int vc = min(v0 + l16, D.dv - 1);  // columns past the end compute what nobody stores
   constexpr int KT = (NK + 3) / 4;  // key tiles of the state per wave
   f32x4 wf[NK], qf[NK], pf[4];
   float kf[KT][16], xf[4], dq[4], du[4], dc = 0.f;
-  auto fetch = [&](int c) {
+  // The next chunk's operands are requested as soon as this chunk's are used up; the barriers below order LDS only, so
+  // the requests stay in flight across them.
+  const int row = w * 16 + l16, last = t0 + n - 1;
+  auto fetch_rows = [&](int c) {
     const int64_t base = (int64_t)(first + c) * D.H + h;
-    const int row = w * 16 + l16, last = t0 + n - 1, tc = t0 + c * C;
     const float* wr = Wo + (base * C + row) * dks;
-    const float* qr = qbase + (int64_t)min(tc + row, last) * rs;
+    const float* qr = qbase + (int64_t)min(t0 + c * C + row, last) * rs;
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk) {
-      wf[kk] = load4(wr, 16 * kk + 4 * q4, dks);
-      qf[kk] = load4(qr, 16 * kk + 4 * q4, dks);
+      wf[kk] = load4_raw(wr, 16 * kk + 4 * q4, dks);  // rows of S past the key width stay zero
+      qf[kk] = load4_raw(qr, 16 * kk + 4 * q4, dks);
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int i = w * 16 + 4 * q4 + r;
       xf[r] = Xo[(base * C + i) * D.dv + vc];
       dq[r] = dec[base * 2 * C + i];
-      du[r] = dec[base * 2 * C + C + i];
+    }
+  };
+  auto fetch_p = [&](int c) {
+    const int64_t base = (int64_t)(first + c) * D.H + h;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      du[r] = dec[base * 2 * C + C + w * 16 + 4 * q4 + r];
       pf[r] = *reinterpret_cast<const f32x4*>(Po + (base * C + row) * C + 16 * r + 4 * q4);
     }
-    dc = dec[base * 2 * C + C - 1];
+  };
+  auto fetch_keys = [&](int c) {
+    const int tc = t0 + c * C;
+    dc = dec[((int64_t)(first + c) * D.H + h) * 2 * C + C - 1];
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt) {
       const int d = (w + 4 * kt) * 16 + l16;
 #pragma unroll
       for (int i = 0; i < 16; ++i) {  // k index of the product: token 16 (i / 4) + 4 q4 + i % 4
         const int tok = min(tc + 16 * (i >> 2) + 4 * q4 + (i & 3), last);
-        kf[kt][i] = kbase[(int64_t)tok * rs + min(d, dks - 1)] * (d < dks ? 1.f : 0.f);
+        kf[kt][i] = kbase[(int64_t)tok * rs + min(d, dks - 1)];
       }
     }
   };
-  fetch(0);
-  __syncthreads();
+  fetch_rows(0);
+  fetch_p(0);
+  fetch_keys(0);
+  lds_barrier();
   for (int c = 0; c < nc; ++c) {
+    const int cn = min(c + 1, nc - 1);
     f32x4 u = {0.f, 0.f, 0.f, 0.f}, oq = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk)
@@ -231,7 +253,8 @@ __global__ void __launch_bounds__(NT) delta_scan_kernel(
       acc[r] = dq[r] * oq[r];
       U[w * 16 + 4 * q4 + r][l16] = uu[r];
     }
-    __syncthreads();
+    fetch_rows(cn);
+    lds_barrier();
 #pragma unroll
     for (int jt = 0; jt < 4; ++jt) {
       if (jt > w) break;  // P is lower triangular
@@ -241,13 +264,14 @@ __global__ void __launch_bounds__(NT) delta_scan_kernel(
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int i = c * C + w * 16 + 4 * q4 + r;
-      if (i < n && v0 + l16 < D.dv) o[((int64_t)(t0 + i) * D.H + h) * D.dv + v0 + l16] = acc[r];
+      if (i < n && v0 + l16 < D.dv) o[D.v_at(h, t0 + i) + v0 + l16] = acc[r];
     }
-    __syncthreads();
+    lds_barrier();
     // U <- e^{G_C - G_i} U for the state update (every wave its own rows)
 #pragma unroll
     for (int r = 0; r < 4; ++r) U[w * 16 + 4 * q4 + r][l16] = uu[r] * du[r];
-    __syncthreads();
+    fetch_p(cn);
+    lds_barrier();
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt) {
       const int d0 = (w + 4 * kt) * 16;
@@ -258,11 +282,12 @@ __global__ void __launch_bounds__(NT) delta_scan_kernel(
 #pragma unroll
         for (int i = 0; i < 16; ++i) s = mfma4(kf[kt][i], U[16 * (i >> 2) + 4 * q4 + (i & 3)][l16], s);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) S[d0 + 4 * q4 + r][l16] = s[r];
+        for (int r = 0; r < 4; ++r)
+          if (d0 + 4 * q4 < dks) S[d0 + 4 * q4 + r][l16] = s[r];
       }
     }
-    if (c + 1 < nc) fetch(c + 1);
-    __syncthreads();
+    fetch_keys(cn);
+    lds_barrier();
   }
   for (int i = tid; i < NK * 256; i += NT) {
     const int k = i % (NK * 16), j = i / (NK * 16);
@@ -294,7 +319,7 @@ __global__ void __launch_bounds__(NT) delta_norm_kernel(const float* __restrict_
         x[u][k][0] = x[u][k][1] = 0.f;
         if (k * 128 >= D.dv) continue;
         const int c = k * 128 + 2 * lane;
-        load2<PAIR>(o + (t * D.H + h) * D.dv, c, D.dv, x[u][k]);
+        load2<PAIR>(o + D.v_at(h, t), c, D.dv, x[u][k]);
         load2<PAIR>(proj + t * D.row() + D.channels() + h * D.dv, c, D.dv, g[u][k]);
         x[u][k][0] *= c < D.dv ? 1.f : 0.f;
         x[u][k][1] *= c + 1 < D.dv ? 1.f : 0.f;
@@ -360,13 +385,14 @@ extern "C" int64_t ds_delta_chunk_ws(int nwork, int H, int dk, int dv) {
 }
 
 // seqs [nseq, 2]: (sequence, index of its first entry in work); work [nwork, 2]: (sequence, chunk), a sequence's chunks
-// in order. o: fp32 [tokens, H, dv] scratch.
+// in order. o: fp32 [H, tokens, dv] scratch.
 extern "C" int ds_delta_chunk(const float* qk, const void* v, const float* gb, const void* proj, const float* norm_w,
                               float eps, float* state, void* conv_state, const int* seqs, int nseq, const int* work,
                               int nwork, const int* cu, const int* start, const int* slots, float* ws, float* o,
-                              void* out, int Hk, int H, int dk, int dv, int taps, int dtype, hipStream_t st) {
+                              void* out, int tokens, int Hk, int H, int dk, int dv, int taps, int dtype,
+                              hipStream_t st) {
   if (nseq <= 0 || nwork <= 0) return 0;
-  const DeltaDims D{Hk, H, dk, dv, taps};
+  const DeltaDims D{Hk, H, dk, dv, taps, tokens};
   if (!dims_ok(D) || (int64_t)nwork * H * 16 > INT32_MAX) return (int)hipErrorInvalidValue;
   if (dtype == DS_F32)
     return run<float>(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, nseq, work, nwork, cu, start, slots, ws, o,

@@ -36,8 +36,14 @@ __device__ __forceinline__ void store2(T* row, int c, int width, const float (&v
 
 struct DeltaDims {
   int Hk, H, dk, dv, taps;
+  int64_t T;  // tokens of the batch
   __host__ __device__ int channels() const { return 2 * Hk * dk + H * dv; }
   __host__ __device__ int dks() const { return (dk + 3) & ~3; }  // key width as q, k and the state are stored (zero padded)
+  // q, k (and v, the read-out) are kept head by head, [heads, T, width]: a head's rows are contiguous, and tiles of them
+  // spread over the memory channels whatever the head count
+  __host__ __device__ int64_t q_at(int hk, int64_t t) const { return ((int64_t)hk * T + t) * dks(); }
+  __host__ __device__ int64_t k_at(int hk, int64_t t) const { return ((int64_t)(Hk + hk) * T + t) * dks(); }
+  __host__ __device__ int64_t v_at(int h, int64_t t) const { return ((int64_t)h * T + t) * dv; }
   __host__ __device__ int row() const { return channels() + H * dv + 2 * H; }
 };
 

@@ -117,7 +117,7 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(
       if (is_v) {
 #pragma unroll
         for (int k = 0; k < 2; ++k)
-          store2<PAIR>(v_out + (tok * D.H + part - 2 * D.Hk) * D.dv, k * 128 + 2 * lane, width, y[t][k]);
+          store2<PAIR>(v_out + D.v_at(part - 2 * D.Hk, tok), k * 128 + 2 * lane, width, y[t][k]);
         continue;
       }
       float ss = 0.f;
@@ -129,7 +129,7 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(
       for (int k = 0; k < 2; ++k) {
         y[t][k][0] *= r;
         y[t][k][1] *= r;
-        store2<true>(qk + (tok * 2 * D.Hk + part) * D.dks(), k * 128 + 2 * lane, D.dks(), y[t][k]);
+        store2<true>(qk + D.q_at(part, tok), k * 128 + 2 * lane, D.dks(), y[t][k]);
       }
     }
     ta = tb;
@@ -164,15 +164,15 @@ __global__ void __launch_bounds__(1024) delta_recur_kernel(
   }
   for (int t = 0; t < n; ++t) {
     const int64_t tok = t0 + t;
-    const float* qr = qk + (tok * 2 * D.Hk + hk) * D.dks();
-    const float* kr = qr + (int64_t)D.Hk * D.dks();
+    const float* qr = qk + D.q_at(hk, tok);
+    const float* kr = qk + D.k_at(hk, tok);
     __syncthreads();
     for (int c = tid; c < KP; c += blockDim.x) {
       qs[c] = c < D.dk ? qr[c] : 0.f;
       ks[c] = c < D.dk ? kr[c] : 0.f;
     }
     const float g = expf(gb[tok * 2 * D.H + h]), beta = gb[(tok * 2 + 1) * D.H + h];
-    const float vv = on ? (float)v[(tok * D.H + h) * D.dv + col] : 0.f;
+    const float vv = on ? (float)v[D.v_at(h, tok) + col] : 0.f;
     __syncthreads();
     float a = 0.f;
 #pragma unroll
@@ -250,7 +250,7 @@ extern "C" int ds_delta_prepare(const void* proj, const float* conv_w, const voi
                                 const int* slots, float* qk, void* v, float* gb, int tokens, int Hk, int H, int dk,
                                 int dv, int taps, int dtype, hipStream_t st) {
   if (tokens <= 0) return 0;
-  const DeltaDims D{Hk, H, dk, dv, taps};
+  const DeltaDims D{Hk, H, dk, dv, taps, tokens};
   if (!dims_ok(D)) return (int)hipErrorInvalidValue;
   const int tile = tokens >= 512 ? TILE : 1;  // few tokens: as many waves as there are
   const int64_t items = (int64_t)((tokens + tile - 1) / tile) * (2 * Hk + H + 1);
@@ -279,10 +279,10 @@ extern "C" int ds_delta_prepare(const void* proj, const float* conv_w, const voi
 // list: the sequences (indices into cu / start / slots) to run
 extern "C" int ds_delta_recur(const float* qk, const void* v, const float* gb, const void* proj, const float* norm_w,
                               float eps, float* state, void* conv_state, const int* list, int nlist, const int* cu,
-                              const int* start, const int* slots, void* out, int Hk, int H, int dk, int dv, int taps,
-                              int dtype, hipStream_t st) {
+                              const int* start, const int* slots, void* out, int tokens, int Hk, int H, int dk, int dv,
+                              int taps, int dtype, hipStream_t st) {
   if (nlist <= 0) return 0;
-  const DeltaDims D{Hk, H, dk, dv, taps};
+  const DeltaDims D{Hk, H, dk, dv, taps, tokens};
   if (!dims_ok(D)) return (int)hipErrorInvalidValue;
   if (dtype == DS_F32)
     return recur<float>(qk, v, gb, proj, norm_w, eps, state, conv_state, list, nlist, cu, start, slots, out, D, st);
