@@ -172,7 +172,16 @@ class DSHybridLayer(ProjectionLayer):
     def _linear(self, x, name, bias=None):
         if name in self.quant:
             return super()._linear(x, name, bias)
-        return ops.linear(x, getattr(self, name))
+        return ops.linear(x, getattr(self, name), self.sh.get(name))
+
+    def add_decode_layout(self):
+        """Shuffled copies of the projections whose shape allows one (see the base class)."""
+        from ...ops.bf16_gemv import Bf16Weight
+        if self.quant:
+            return False
+        self.sh = {n: Bf16Weight(w.data) for n, w in ((n, getattr(self, n)) for n in self.projection_names())
+                   if w.is_cuda and Bf16Weight.supported(w.data)}
+        return bool(self.sh)
 
     def shard(self, lw, r, tp):
         """Canonical full weights -> {attribute path: this rank's tensor}."""
@@ -222,9 +231,6 @@ class DSHybridModel(DSInferenceModel):
     def shard_layer(self, idx, lw):
         return self.layers[idx].shard(lw, self.tp_rank, self.tp_size)
 
-    def add_decode_layout(self):
-        return 0  # decode-sized products stream the row-major weights
-
     # ------------------------------------------------------------------------------------------ forward
     def forward(self, input_ids, meta, all_logits=False):
         raise NotImplementedError("hybrid decoders are served by the ragged engine (inference v2)")
@@ -253,7 +259,7 @@ class DSHybridModel(DSInferenceModel):
         return self._logits(h)
 
     def _logits(self, h):
-        return self._gather_vocab(ops.linear(h, self.lm_head))
+        return self._gather_vocab(ops.linear(h, self.lm_head, getattr(self, "lm_head_sh", None)))
 
 
 def model_class(spec):

@@ -5,7 +5,9 @@
 #include <ATen/hip/HIPContext.h>
 #include <hip/hip_runtime_api.h>
 
+#include <map>
 #include <optional>
+#include <utility>
 
 extern "C" {
 int ds_stream_norm(float*, const void*, const int*, const void*, const int*, int, int, const float*, const float*, float,
@@ -30,6 +32,8 @@ int ds_paged_decode_ext(const void*, const void*, const void*, const int*, const
                         int, int, int, int, int, int, int, float, float, int, int, hipStream_t);
 int ds_skinny_gemm(const void*, const void*, const void*, const void*, const void*, const void*, void*, void*, int, int,
                    int, int, int, int, float, hipStream_t);
+int ds_skinny_b16_mfma_ok(int, int);
+int ds_skinny_b16_mfma(const void*, const void*, const void*, void*, float*, int, int, int, hipStream_t);
 int ds_skinny_mfma_ok(int, int, int);
 int ds_skinny_mfma(const void*, const void*, const void*, const void*, const void*, const void*, void*, void*, int, int,
                    int, int, int, int, float, hipStream_t);
@@ -306,6 +310,26 @@ Tensor decode_linear(Tensor x, Tensor w) {
            0, 0, 0, 0.f, stream()), "decode_linear");
   return y;
 }
+
+// x [M, K] . w^T (M <= 16) over a weight in the shuffled decode layout (ops/bf16_gemv.py: preshuffle16), w [N, K]
+Tensor decode_linear_sh(Tensor x, Tensor wsh, int64_t N) {
+  need(x, "x"); need(wsh, "wsh");
+  const int64_t K = x.size(-1), M = x.numel() / K, NB = (N + 15) / 16;
+  TORCH_CHECK(x.scalar_type() == at::kBFloat16 && wsh.scalar_type() == at::kBFloat16 && wsh.numel() == NB * 16 * K &&
+              ds_skinny_b16_mfma_ok((int)M, (int)K), "decode_linear_sh: up to 16 bf16 rows, K % 64 == 0");
+  TORCH_CHECK(NB * K < ((int64_t)1 << 40) && N < ((int64_t)1 << 31) / 16, "decode_linear_sh: matrix too large");
+  // fp32 split-K sums, zero between calls (the kernels leave it so); one per device and stream, grown on demand
+  static std::map<std::pair<int, hipStream_t>, Tensor> workspaces;
+  Tensor& ws = workspaces[{x.get_device(), stream()}];
+  const int64_t nf = 16 * ((NB + 3) / 4) * 64;
+  if (!ws.defined() || ws.numel() < nf) ws = torch::zeros({nf}, x.options().dtype(at::kFloat));
+  auto sizes = x.sizes().vec();
+  sizes.back() = N;
+  auto y = torch::empty(sizes, x.options());
+  check(ds_skinny_b16_mfma(x.data_ptr(), wsh.data_ptr(), nullptr, y.data_ptr(), ws.data_ptr<float>(), (int)M, (int)N, (int)K,
+                           stream()), "decode_linear_sh");
+  return y;
+}
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -323,4 +347,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("paged_decode", &paged_decode);
   m.def("decode_linear", &decode_linear);
   m.def("decode_linear_ok", &decode_linear_ok);
+  m.def("decode_linear_sh", &decode_linear_sh);
 }

@@ -65,9 +65,12 @@ def delta_rule(proj, conv_w, a_log, dt_bias, norm_w, eps, state, conv_state, met
     return out
 
 
-def linear(x, w):
-    """x . w^T: a weight stream for decode-sized bf16 batches, else the library product."""
+def linear(x, w, sh=None):
+    """x . w^T: a weight stream for decode-sized bf16 batches (over the shuffled copy `sh`, a `Bf16Weight`, from two
+    rows up), else the library product."""
     rows = x.numel() // x.shape[-1]
+    if sh is not None and x.is_cuda and 2 <= rows <= DECODE_ROWS:
+        return hybrid_ops().decode_linear_sh(x, sh.wsh, sh.shape[0])
     if x.is_cuda and x.dtype == torch.bfloat16 and 0 < rows <= DECODE_ROWS and \
             hybrid_ops().decode_linear_ok(rows, x.shape[-1]):
         return hybrid_ops().decode_linear(x, w)

@@ -73,6 +73,8 @@ EXTENSIONS = {
             "recur/delta_chunk.hip",
             "gemv/skinny_gemm.hip",
             "gemv/skinny_mfma.hip",
+            "gemv/skinny_bf16_sh.hip",
+            "gemv/skinny_finalize.hip",
         ],
         "bindings": ["bind/hybrid_bind.cpp"],
     },
