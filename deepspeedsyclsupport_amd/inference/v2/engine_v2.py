@@ -84,6 +84,12 @@ class InferenceEngineV2:
             res = self.can_schedule(uids, [t.numel() for t in toks])
             if res != SchedulingResult.Success:
                 raise SchedulingError(res)
+            host = [t for t in toks if not t.is_cuda and t.numel()]
+            if host:  # an id the embedding does not have must not reach the device
+                lo, hi = torch.aminmax(torch.cat(host))
+                if int(lo) < 0 or int(hi) >= self._model.spec.vocab_size:
+                    raise ValueError(f"token ids {int(lo)} to {int(hi)} outside the vocabulary of "
+                                     f"{self._model.spec.vocab_size}")
         batch = self._batch
         batch.clear()
         seqs = []

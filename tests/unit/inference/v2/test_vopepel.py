@@ -5,6 +5,7 @@ import json
 import pytest
 import torch
 
+from ...common import run_distributed
 from . import vopepel_oracle as O
 
 GPU = pytest.mark.gpu
@@ -174,6 +175,24 @@ def test_far_key_and_score_cap(tmp_path, dtype, tol):
 
 
 @pytest.mark.parametrize("dtype,tol", PRECISION)
+@pytest.mark.parametrize("softcap", [None, 1.5, 33.0, 34.0, 90.0])
+def test_score_caps(tmp_path, dtype, tol, softcap):
+    """No cap, one that bends most scores, and ones on both sides of where the prefill kernel stops taking the cap for
+    the maximum; no chunks; values not mixed; sharp scores."""
+    cfg = O.config([O.attention_layer(heads=4, kv_heads=1, dim=48, vdim=72, size=10**6, scale=0.5, softcap=softcap,
+                                      v_mix=False, ff=0)], streams=2)
+    del cfg["layers"][0]["mixer"]["v_mix"]
+    if softcap is None:
+        del cfg["layers"][0]["mixer"]["softcap"], cfg["layers"][0]["mixer"]["mask"]
+    w = O.random_model(cfg, 14, peak=1.6)
+    eng = engine(tmp_path, cfg, w, dtype)
+    ids = tokens(cfg, 150)
+    want = O.forward(cfg, w, ids)
+    assert err(feed(eng, 0, ids, [150]), want) < tol
+    assert err(feed(eng, 1, ids, [120, 1]), want) < tol
+
+
+@pytest.mark.parametrize("dtype,tol", PRECISION)
 def test_long_state(tmp_path, dtype, tol):
     """Slow decays: tokens far back stay in the state; long decoding after a long prompt."""
     cfg = O.config([O.delta_layer(heads=4, kv_heads=2, dim=24, vdim=40, conv=4, ff=0),
@@ -239,6 +258,8 @@ def test_scheduling_slots(tmp_path):
     assert eng._state_manager.free_slots == 2
     assert eng.can_schedule([1, 2], [4, 4]) == SchedulingResult.Success
     assert eng.can_schedule([1, 2, 3], [4, 4, 4]) == SchedulingResult.EngineSequenceLimitExceeded
+    with pytest.raises(ValueError, match="outside the vocabulary"):
+        eng.put([1], [torch.tensor([3, cfg["vocab"]])])
     eng.put([1, 2], [tokens(cfg, 4), tokens(cfg, 3)])
     assert eng.query(3, 8, 4) == (0, 0)
     eng.flush(1)
@@ -303,6 +324,31 @@ def test_weight_only_int8(tmp_path):
     want = O.forward(cfg, w, ids)
     eng.model.quantize_weights(8)
     assert err(feed(eng, 0, ids, [30, 1]), want) < 0.12
+
+
+def _tp_run(path, ids, want):
+    from deepspeedsyclsupport_amd.inference.v2 import (AllocationMode, RaggedInferenceEngineConfig, build_hf_engine)
+    torch.set_num_threads(1)
+    conf = RaggedInferenceEngineConfig(
+        state_manager={"memory_config": {"mode": AllocationMode.ALLOCATE, "size": 16}, "max_tracked_sequences": 2,
+                       "max_ragged_sequence_count": 2, "max_context": 256}, kv_cache={"block_size": 16},
+        tensor_parallel={"tp_size": 2})
+    eng = build_hf_engine(path, conf, dtype=torch.float32)
+    assert eng.model.layers[0].mixer.H == 3
+    got = torch.cat([eng.put([0], [ids[:40]], logit_positions=[range(40)]),
+                     eng.put([0], [ids[40:]], logit_positions=[range(10)])])
+    assert err(got, want) < 2e-5
+
+
+@pytest.mark.skipif(torch.cuda.is_available(), reason="ranks exchange host tensors")
+def test_tensor_parallel(tmp_path):
+    """Heads, states, convolution windows, feed-forward and vocabulary over two ranks."""
+    cfg = O.config([O.delta_layer(heads=6, kv_heads=2, dim=16, vdim=24, conv=3),
+                    O.attention_layer(heads=6, kv_heads=2, dim=32, vdim=16, size=24),
+                    O.attention_layer(heads=4, kv_heads=2, dim=24, vdim=16, size=70, ff=0)])
+    w = O.random_model(cfg, 15)
+    ids = tokens(cfg, 50)
+    run_distributed(_tp_run, 2, save(tmp_path / "m", cfg, w), ids, O.forward(cfg, w, ids))
 
 
 # ------------------------------------------------------------------------------------------------ trace replay
