@@ -208,6 +208,22 @@ def test_long_state(tmp_path, dtype, tol):
     assert err(feed(eng, 2, ids, [100, 17, 16, 2]), want) < tol
 
 
+@pytest.mark.parametrize("dtype,tol", PRECISION)
+@pytest.mark.parametrize("width,vocab,streams", [(200, 131, 2), (132, 61, 8), (37, 50, 5)])
+def test_model_widths(tmp_path, dtype, tol, width, vocab, streams):
+    """Widths no vector or matrix tile divides, other stream counts, a feed-forward of 1-wide remainder."""
+    cfg = O.config([O.attention_layer(heads=3, kv_heads=1, dim=20, vdim=12, size=31, ff=45),
+                    O.delta_layer(heads=3, kv_heads=3, dim=18, vdim=10, conv=2, ff=24),
+                    O.attention_layer(heads=2, kv_heads=1, dim=16, vdim=12, size=20, ff=0)], width=width, vocab=vocab,
+                   streams=streams, residual_mult=1.0, eps=1e-3)
+    w = O.random_model(cfg, 16)
+    eng = engine(tmp_path, cfg, w, dtype)
+    ids = tokens(cfg, 90)
+    want = O.forward(cfg, w, ids)
+    for u, cuts in enumerate(([90], [40, 2], [60, 1])):
+        assert err(feed(eng, u, ids, cuts), want) < 2 * tol, cuts
+
+
 @GPU
 @pytest.mark.parametrize("dims", [(8, 4, 128, 128, 128, 128), (4, 2, 256, 256, 256, 192), (4, 4, 64, 96, 80, 64),
                                   (12, 1, 48, 20, 72, 200), (2, 1, 20, 33, 36, 28)])
