@@ -136,7 +136,11 @@ class ClampedMLP:
                 "fc2_w": _shard(lw["down_w"], r, tp, 1)}
 
     def run(self, layer, h):
-        return layer._linear(ops.clamped_glu(layer._linear(h, "fc1_w"), self.limit), "fc2_w")
+        if "fc1_w" in layer.quant:
+            mid = ops.clamped_glu(layer._linear(h, "fc1_w"), self.limit)
+        else:
+            mid = ops.glu_linear(h, layer.fc1_w, layer.sh.get("fc1_w"), self.limit)
+        return layer._linear(mid, "fc2_w")
 
 
 MLPS = {m.kind: m for m in (ClampedMLP, )}

@@ -5,12 +5,6 @@
 
 namespace {
 
-__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha, float shift) {
-  g = fminf(g, limit);
-  u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.f + expf(-alpha * g)) * (u + shift);
-}
-
 template <typename T, bool VEC>
 __global__ void __launch_bounds__(256) clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ out, int64_t rows,
                                                           int F, float limit, float alpha, float shift) {
@@ -25,10 +19,10 @@ __global__ void __launch_bounds__(256) clamped_glu_kernel(const T* __restrict__ 
       Vec8<T>::load(g, a);
       Vec8<T>::load(g + F, b);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) a[j] = clamped_glu(a[j], b[j], limit, alpha, shift);
+      for (int j = 0; j < 8; ++j) a[j] = clamped_glu_f(a[j], b[j], limit, alpha, shift);
       Vec8<T>::store(out + r * F + c, a);
     } else {
-      out[r * F + c] = (T)clamped_glu((float)g[0], (float)g[F], limit, alpha, shift);
+      out[r * F + c] = (T)clamped_glu_f((float)g[0], (float)g[F], limit, alpha, shift);
     }
   }
 }

@@ -45,7 +45,7 @@ int64_t ds_skinny_i4_mfma_ws_floats(int);
 void ds_skinny_i4_tune(int, int, int);
 int ds_dequant_sh4(const int8_t*, const float*, void*, int, int, int, hipStream_t);
 int ds_skinny_finalize_rms(float*, const void*, const void*, const void*, void*, void*, int, int, int, float, hipStream_t);
-int ds_skinny_finalize_gated(float*, const void*, void*, int, int, int, int, hipStream_t);
+int ds_skinny_finalize_gated(float*, const void*, void*, int, int, int, int, float, hipStream_t);
 int ds_skinny_finalize_plain(float*, const void*, void*, int, int, int, hipStream_t);
 int ds_quantize(const void*, int8_t*, float*, float*, int64_t, int, int, int, int, unsigned, int, hipStream_t);
 int ds_dequantize(const int8_t*, const float*, const float*, void*, int64_t, int, int, int, int, hipStream_t);
@@ -482,7 +482,7 @@ Tensor skinny_finalize_gated(Tensor acc, int64_t M, int64_t N, OptT bias, int64_
   const void* bp = opt_bf16(bias, N, "bias");
   auto out = torch::empty({M, N / 2}, acc.options().dtype(at::kBFloat16));
   check(ds_skinny_finalize_gated(acc.data_ptr<float>(), bp, out.data_ptr(), (int)M, (int)N, (int)acc.size(1), (int)act,
-                                 stream()), "skinny_finalize_gated");
+                                 0.f, stream()), "skinny_finalize_gated");
   return out;
 }
 

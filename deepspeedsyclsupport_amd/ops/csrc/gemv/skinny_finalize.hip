@@ -71,7 +71,8 @@ __global__ void __launch_bounds__(1024) finalize_rms_kernel(float* __restrict__ 
 
 // out[t, i] = act(acc[t, i] + b[i]) * (acc[t, I + i] + b[I + i]),  N = 2 I
 __global__ void __launch_bounds__(256) finalize_gated_kernel(float* __restrict__ acc, const bf16* __restrict__ bias,
-                                                             bf16* __restrict__ out, int M, int I, int NP, int act) {
+                                                             bf16* __restrict__ out, int M, int I, int NP, int act,
+                                                             float limit) {
   const int64_t e = (int64_t)blockIdx.x * 256 + threadIdx.x;
   const int half = NP - I;  // columns [I, NP) hold the up half and the padding
   if (e >= (int64_t)M * half) return;
@@ -83,7 +84,8 @@ __global__ void __launch_bounds__(256) finalize_gated_kernel(float* __restrict__
     const float g = arow[j];
     arow[j] = 0.f;
     const float gb = bias ? (float)bias[j] : 0.f, ub = bias ? (float)bias[I + j] : 0.f;
-    out[(int64_t)t * I + j] = (bf16)(act_any(act, g + gb) * (u + ub));
+    out[(int64_t)t * I + j] = (bf16)(act == DS_ACT_CLAMPED_GLU ? clamped_glu_f(g + gb, u + ub, limit)
+                                                                  : act_any(act, g + gb) * (u + ub));
   }
 }
 
@@ -117,12 +119,12 @@ extern "C" int ds_skinny_finalize_rms(float* ws, const void* bias, const void* r
 }
 
 extern "C" int ds_skinny_finalize_gated(float* ws, const void* bias, void* out, int M, int N, int NP, int act,
-                                        hipStream_t st) {
+                                        float limit, hipStream_t st) {
   if (M < 1 || M > 16 || N < 2 || N % 2 || NP < N) return (int)hipErrorInvalidValue;
   const int I = N / 2;
   const int64_t total = (int64_t)M * (NP - I);
   hipLaunchKernelGGL(finalize_gated_kernel, dim3((int)((total + 255) / 256)), dim3(256), 0, st, ws, (const bf16*)bias,
-                     (bf16*)out, M, I, NP, act);
+                     (bf16*)out, M, I, NP, act, limit);
   DS_CHECK_LAUNCH();
   return 0;
 }

@@ -30,6 +30,11 @@ __device__ __forceinline__ float act_f(float g, int act) {
     default: return g;
   }
 }
+// gated epilogue; for the clamped activation `limit` is the clamp (it travels in the kernel's eps argument, which only
+// the norm-fused input mode uses)
+__device__ __forceinline__ float gated_f(float g, float u, int act, float limit) {
+  return act == DS_ACT_CLAMPED_GLU ? clamped_glu_f(g, u, limit) : act_f(g, act) * u;
+}
 
 __device__ __forceinline__ bf16x8 ld_stream(const bf16* p) {
   return __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(p));
@@ -230,7 +235,7 @@ __global__ void __launch_bounds__(WAVES * 64) skinny_kernel(
         if (GATED) {
           const float g = (float)(bf16)o0, u = (float)(bf16)o1;  // HF rounds the projections to bf16 first
           const int Nh = N / 2;
-          y[(int64_t)m * Nh + p] = (bf16)(act_f(g, act) * u + (add ? (float)add[(int64_t)m * Nh + p] : 0.f));
+          y[(int64_t)m * Nh + p] = (bf16)(gated_f(g, u, act, eps) + (add ? (float)add[(int64_t)m * Nh + p] : 0.f));
         } else {
           if (add) o0 += (float)add[(int64_t)m * N + n0];
           y[(int64_t)m * N + n0] = (bf16)o0;
@@ -309,6 +314,7 @@ extern "C" int ds_skinny_gemm(const void* W, const void* x, const void* r, const
   if (M < 1 || M > 8 || K % 8 != 0 || in_mode < 0 || in_mode > 1) return (int)hipErrorInvalidValue;
   if (in_mode == 1 && !nw) return (int)hipErrorInvalidValue;
   if (gated && (N % 2)) return (int)hipErrorInvalidValue;
+  if (gated && act == DS_ACT_CLAMPED_GLU && in_mode != 0) return (int)hipErrorInvalidValue;
   const bool xlds = ds_skinny_fits_lds(M, K);
   auto W_ = (const bf16*)W;
   auto x_ = (const bf16*)x;

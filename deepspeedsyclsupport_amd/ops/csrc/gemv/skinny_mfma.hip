@@ -29,6 +29,11 @@ __device__ __forceinline__ float act_f(float g, int act) {
     default: return g;
   }
 }
+// gated epilogue; for the clamped activation `limit` is the clamp (it travels in the kernel's eps argument, which only
+// the norm-fused input mode uses)
+__device__ __forceinline__ float gated_f(float g, float u, int act, float limit) {
+  return act == DS_ACT_CLAMPED_GLU ? clamped_glu_f(g, u, limit) : act_f(g, act) * u;
+}
 
 // k offset (within a K-slice) of MFMA step s for lane-group q = lane >> 4: steps come in pairs sharing one 32-byte
 // contiguous run per lane (pair i covers k in [64 i, 64 i + 64), group q owns [64 i + 16 q, 64 i + 16 q + 16)).
@@ -158,7 +163,7 @@ __global__ void __launch_bounds__(NW * 64) skinny_mfma_kernel(
     if (GATED) {
       const float g = (float)(bf16)(v[0] + (bias ? (float)bias[n] : 0.f));
       const float u = (float)(bf16)(v[1] + (bias ? (float)bias[Nout + n] : 0.f));
-      o = act_f(g, act) * u;
+      o = gated_f(g, u, act, eps);
     } else {
       o = v[0] + (bias ? (float)bias[n] : 0.f);
     }
@@ -198,6 +203,7 @@ extern "C" int ds_skinny_mfma(const void* W, const void* x, const void* r, const
                               const void* add, void* y, void* res_out, int M, int N, int K, int in_mode, int gated,
                               int act, float eps, hipStream_t s) {
   if (!ds_skinny_mfma_ok(M, K, in_mode) || (gated && N % 2)) return (int)hipErrorInvalidValue;
+  if (gated && act == DS_ACT_CLAMPED_GLU && in_mode != 0) return (int)hipErrorInvalidValue;
   auto W_ = (const bf16*)W;
   auto x_ = (const bf16*)x;
   auto r_ = (const bf16*)r;

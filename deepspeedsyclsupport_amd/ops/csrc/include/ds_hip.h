@@ -75,6 +75,16 @@ template <> struct Vec8<fp16> {
 template <typename T> __device__ __forceinline__ float to_f32(T x) { return (float)x; }
 template <typename T> __device__ __forceinline__ T from_f32(float x) { return (T)x; }
 
+// ---------------------------------------------------------------- clamped gated activation
+// g sigmoid(alpha g) (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit). As the epilogue of a gated
+// decode product it is activation code DS_ACT_CLAMPED_GLU with alpha 1.702 and shift 1.
+#define DS_ACT_CLAMPED_GLU 5
+__device__ __forceinline__ float clamped_glu_f(float g, float u, float limit, float alpha = 1.702f, float shift = 1.f) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.f + expf(-alpha * g)) * (u + shift);
+}
+
 // ---------------------------------------------------------------- wave64 / block reductions
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

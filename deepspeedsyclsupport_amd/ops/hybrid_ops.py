@@ -75,3 +75,14 @@ def linear(x, w, sh=None):
             hybrid_ops().decode_linear_ok(rows, x.shape[-1]):
         return hybrid_ops().decode_linear(x, w)
     return F.linear(x, w)
+
+
+def glu_linear(x, w, sh, limit):
+    """Clamped gated activation of x . [gate | up]^T: the epilogue of the weight stream for decode-sized bf16 batches."""
+    rows = x.numel() // x.shape[-1]
+    if x.is_cuda and x.dtype == torch.bfloat16 and 0 < rows <= DECODE_ROWS:
+        if sh is not None and rows >= 2:
+            return hybrid_ops().decode_linear_sh(x, sh.wsh, sh.shape[0], limit)
+        if hybrid_ops().decode_linear_ok(rows, x.shape[-1]):
+            return hybrid_ops().decode_linear(x, w, limit)
+    return clamped_glu(F.linear(x, w), limit)

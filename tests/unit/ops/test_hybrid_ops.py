@@ -179,10 +179,15 @@ def test_delta_rule(device, dtype, tol, Hk, rep, dk, dv, taps):
 
 @GPU
 @pytest.mark.parametrize("rows", [1, 2, 5, 16])
-@pytest.mark.parametrize("N,K", [(96, 64), (513, 320), (1024, 2048)])
+@pytest.mark.parametrize("N,K", [(96, 64), (513, 320), (90, 256), (1024, 2048)])
 def test_decode_products(rows, N, K):
     from deepspeedsyclsupport_amd.ops.bf16_gemv import Bf16Weight
     x, w = rnd(rows, K).bfloat16().cuda(), rnd(N, K, seed=1, scale=K**-0.5).bfloat16().cuda()
     want = x.double().cpu() @ w.double().cpu().t()
     close(ops.linear(x, w), want, 1e-2)
     close(ops.linear(x, w, Bf16Weight(w)), want, 1e-2)
+    if N % 2 == 0:
+        glu = O.clamped_glu(want[:, :N // 2], want[:, N // 2:], 0.7)
+        close(ops.glu_linear(x, w, None, 0.7), glu, 1e-2)
+        close(ops.glu_linear(x, w, Bf16Weight(w), 0.7), glu, 1e-2)
+        close(ops.linear(x, w, Bf16Weight(w)), want, 1e-2)   # the gated finalize leaves the sums cleared
