@@ -81,6 +81,24 @@ def test_ragged_matches_hf(chunk):
     assert eng._state_manager.free_blocks > free0 and eng._state_manager.get_sequence(10) is None
 
 
+def test_generate_matches_hf():
+    """Continuous batching: prompts split by the token budget, more requests than fit at once, all equal to HF greedy."""
+    m = _model()
+    eng = _engine(m, blocks=12, bs=8)
+    g = torch.Generator().manual_seed(3)
+    prompts = [torch.randint(0, 128, (n, ), generator=g) for n in (7, 30, 3, 19, 12)]
+    outs = eng.generate(prompts, max_new_tokens=6, token_budget=16)
+    for p, o in zip(prompts, outs):
+        assert o == _ref(m, p, 6)
+    assert eng._state_manager.free_blocks == 12
+    with pytest.raises(ValueError, match="does not fit"):
+        eng.generate([torch.arange(100)], max_new_tokens=20)
+    rows = eng.put([5], [prompts[1]], logit_positions=[[3, 29]])
+    assert torch.allclose(rows[1], eng.put([6], [prompts[1]])[0], atol=1e-5)
+    with torch.no_grad():
+        assert torch.allclose(rows, m(prompts[1][None]).logits[0, [3, 29]], atol=1e-4)
+
+
 def test_scheduling_limits():
     from deepspeedsyclsupport_amd.inference.v2 import SchedulingError, SchedulingResult
     eng = _engine(_model(), blocks=4, bs=8)   # 32 tokens of cache
