@@ -591,6 +591,12 @@ def load_top(model: DSInferenceModel, top):
     if spec.embed_norm:
         _put(model.embed_ln_w, top["embed_ln_w"])
         _put(model.embed_ln_b, top["embed_ln_b"])
+    if hasattr(model, "shard_top"):
+        for path, t in model.shard_top(top).items():
+            p = model.get_parameter(path)
+            if p.shape != t.shape:
+                raise ValueError(f"{path} is {tuple(t.shape)} in the checkpoint, {tuple(p.shape)} by the configuration")
+            _put(p, t)
     _put(model.norm_w, top["norm_w"])
     _put(model.norm_b, top.get("norm_b"))
     V, vl = spec.vocab_size, model.vocab_local

@@ -66,6 +66,9 @@ class DSModelSpec:
     layer_specs: tuple = ()
     streams: int = 1                 # residual streams (hyper-connections)
     residual_mult: float = 1.0       # factor of every sublayer's output
+    residual: str = "streams"        # "streams" (pre-norm over the streams) | "post_norm" (norms on sublayer outputs)
+    token_side: int = 0              # width of a side embedding per layer and token (0: none)
+    logit_scale: float = 1.0
 
     def __post_init__(self):
         if not self.head_dim:
@@ -154,7 +157,7 @@ class BatchMeta:
 @dataclass
 class RaggedMeta:
     """One ragged batch (inference v2 `put()`): the new tokens of every sequence concatenated, decode sequences (one
-    token each) first, then prompt / chunk sequences. Device tensors come from ONE packed host->device copy
+    token each) first, then short portions (up to `SHORT_TOKENS`), then longer prompts and portions. Device tensors come from ONE packed host->device copy
     (`RaggedMeta.build`); the host lists are kept so no step needs a device->host sync."""
     block_tables: torch.Tensor       # [S, max_blocks] int32
     start_pos: torch.Tensor          # [S] tokens cached before this step
@@ -174,7 +177,11 @@ class RaggedMeta:
     chunk_seqs: Optional[torch.Tensor] = None  # [L, 2] the others, by chunks of `STATE_CHUNK` tokens: (sequence, first
                                                # entry in chunk_work)
     chunk_work: Optional[torch.Tensor] = None  # [N, 2] (sequence, chunk) of those
+    n_short: int = 0                 # sequences [0, n_short) are decodes or short portions
+    kv_offs: Optional[torch.Tensor] = None   # [S - n_short + 1] offsets of the other sequences' contexts laid end to end
+    kv_total: int = 0                # ... and their end
 
+    SHORT_TOKENS = 64    # portions up to this long count as short
     STATE_CHUNK = 64     # tokens per chunk of a recurrent layer's parallel form
     STEP_TOKENS = 16     # portions up to this long pass a recurrent layer token by token
 
@@ -205,22 +212,27 @@ class RaggedMeta:
         for i in long:
             chunk_seqs += [i, len(chunks)]
             chunks += [(i, c) for c in range(-(-n_new[i] // RaggedMeta.STATE_CHUNK))]
+        # (a sequence is only counted as short if everything before it in the batch is)
+        n_short = next((i for i in range(n_decode, S) if n_new[i] > RaggedMeta.SHORT_TOKENS), S)
+        kv = [0]
+        for i in range(n_short, S):
+            kv.append(kv[-1] + lens[i])
         flat = pos + sid + list(starts) + lens + cu + [x for w in work for x in w] + last + bt + slots + short + chunk_seqs + \
-            [x for w in chunks for x in w]
+            [x for w in chunks for x in w] + kv
         buf = torch.tensor(flat, dtype=torch.int32)
         if device is not None and torch.device(device).type == "cuda":
             buf = buf.pin_memory().to(device, non_blocking=True)
         views, o = [], 0
         for n in (T, T, S, S, S + 1, 2 * len(work), len(last), S * width, len(slots), len(short), len(chunk_seqs),
-                  2 * len(chunks)):
+                  2 * len(chunks), len(kv)):
             views.append(buf[o:o + n])
             o += n
-        pos_t, sid_t, st_t, len_t, cu_t, work_t, last_t, bt_t, slot_t, short_t, long_t, chunk_t = views
+        pos_t, sid_t, st_t, len_t, cu_t, work_t, last_t, bt_t, slot_t, short_t, long_t, chunk_t, kv_t = views
         return RaggedMeta(block_tables=bt_t.view(S, width), start_pos=st_t, seq_lens=len_t, pos_ids=pos_t,
                           seq_ids=sid_t, cu_q=cu_t, work=work_t.view(-1, 2), last_idx=last_t.long(),
                           n_decode=n_decode, cu_host=cu, start_host=list(starts), max_len=width * block_size,
                           block_size=block_size, slots=slot_t, seq_list=short_t, chunk_seqs=long_t.view(-1, 2),
-                          chunk_work=chunk_t.view(-1, 2))
+                          chunk_work=chunk_t.view(-1, 2), n_short=n_short, kv_offs=kv_t, kv_total=kv[-1])
 
 
 class ProjectionLayer(nn.Module):

@@ -13,8 +13,14 @@ _MIXER_TENSORS = {  # checkpoint name below `<layer>.mix.` -> canonical key
     "attention": {"q": "q_w", "k": "k_w", "v": "v_w", "o": "o_w", "q.norm": "q_norm", "k.norm": "k_norm"},
     "delta": {"q": "q_w", "k": "k_w", "v": "v_w", "g": "g_w", "b": "b_w", "a": "a_w", "o": "o_w", "q.conv": "q_conv",
               "k.conv": "k_conv", "v.conv": "v_conv", "A_log": "a_log", "dt_bias": "dt_bias", "norm": "head_norm"},
+    "latent_attention": {"dq": "dq_w", "dq.norm": "q_norm", "uq": "uq_w", "dkv": "dkv_w", "dkv.norm": "kv_norm",
+                         "uk": "uk_w", "uv": "uv_w", "sink": "sink", "o": "o_w"},
+    "mamba2": {"in": "in_w", "conv": "conv_w", "conv.b": "conv_b", "dt_bias": "dt_bias", "A_log": "a_log", "D": "skip",
+               "norm": "head_norm", "o": "o_w"},
+    "lightning": {"q": "q_w", "k": "k_w", "v": "v_w", "g": "g_w", "o": "o_w", "norm": "head_norm"},
 }
-_MLP_TENSORS = {"dense": {"gate": "gate_w", "up": "up_w", "down": "down_w"}}
+_MLP_TENSORS = {"dense": {"gate": "gate_w", "up": "up_w", "down": "down_w"}, "gelu": {"up": "up_w", "down": "down_w"}}
+_SIDE_TENSORS = {"side.gate": "side_gate_w", "side.proj": "side_proj_w", "side.norm": "side_norm_w"}
 
 
 class _HybridContainer(LayerContainer):
@@ -36,8 +42,8 @@ def container(name, tensors, may_lack=()):
                                              "may_lack": may_lack})
 
 
-def layer_container(layer, streams, may_lack=()):
-    """Container class of one entry of the config's layer list."""
+def layer_container(layer, streams=False, may_lack=(), side=False):
+    """Container class of one entry of the spec's layer list."""
     if layer["type"] not in _MIXER_TENSORS:
         raise NotImplementedError(f"no mixer {layer['type']!r}")
     tensors = {f"mix.{n}": key for n, key in _MIXER_TENSORS[layer["type"]].items()}
@@ -51,10 +57,14 @@ def layer_container(layer, streams, may_lack=()):
         tensors[f"norm{q}"] = f"norm{q}_w"
         if streams:
             tensors.update({f"hc{q}.{n}": f"hc{q}_{n}" for n in ("in", "out", "mix")})
+    if side:
+        tensors.update(_SIDE_TENSORS)
     return container("HybridLayerContainer", tensors, may_lack)
 
 
-TopContainer = container("HybridTopContainer", {"embed": "embed", "final.norm": "norm_w", "head": "lm_head"})
+_TOP_TENSORS = {"embed": "embed", "final.norm": "norm_w", "head": "lm_head"}
+TopContainer = container("HybridTopContainer", _TOP_TENSORS)
+SideTopContainer = container("HybridSideTopContainer", {**_TOP_TENSORS, "side.embed": "side_embed"})
 
 
 @register
@@ -83,4 +93,32 @@ class VopepelPolicy(InferenceV2Policy):
         cmap.set_transformer_params("l", [layer_container(la, streams, ("vmix", ) if i == first else ())(self._view)
                                           for i, la in enumerate(c.layers)], sep="")
         cmap.set_non_transformer_params(TopContainer(self._view))
+        return cmap
+
+
+@register
+class PerelornPolicy(InferenceV2Policy):
+    """Perelorn: state-space, linear-attention and latent-attention layers under norms on the sublayers' outputs, with a
+    token-side input in every layer."""
+    model_types = ("perelorn", )
+    model_class = DSHybridModel
+
+    def layers(self):
+        """The config's layers in the spec's terms: its "dense" feed-forward is the ungated gelu one."""
+        return [{**la, "mlp": {**la["mlp"], "kind": {"dense": "gelu"}.get(la["mlp"].get("kind"), la["mlp"].get("kind"))}
+                 if la.get("mlp") else None} for la in self._model_config.layers]
+
+    def spec(self):
+        c = self._model_config
+        first = next((la["mixer"] for la in c.layers if la["type"] == "latent_attention"), c.layers[0]["mixer"])
+        return DSModelSpec(arch="perelorn", vocab_size=c.vocab, hidden_size=c.width, num_layers=len(c.layers),
+                           num_heads=first["heads"], num_kv_heads=first["heads"], head_dim=first["vdim"],
+                           intermediate_size=max([la["mlp"]["ff"] for la in c.layers if la.get("mlp")], default=0),
+                           norm="rms", norm_eps=float(c.norm["eps"]), pos="none", layer_specs=tuple(self.layers()),
+                           residual="post_norm", token_side=int(c.token_side["dim"]), logit_scale=float(c.logit_scale))
+
+    def build_container_map(self):
+        cmap = ContainerMap()
+        cmap.set_transformer_params("l", [layer_container(la, side=True)(self._view) for la in self.layers()], sep="")
+        cmap.set_non_transformer_params(SideTopContainer(self._view))
         return cmap

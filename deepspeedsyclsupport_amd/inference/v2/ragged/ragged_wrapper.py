@@ -1,7 +1,7 @@
 """Host-side assembly of one ragged batch (reference `inference/v2/ragged/ragged_wrapper.py:31-193`).
 
 Sequences are inserted one by one with their new tokens; `finalize()` orders them (single-token decodes of known
-sequences first: the paged decode kernel takes a leading slice; prompts and prompt chunks after), builds every index
+sequences first: the paged decode kernel takes a leading slice; then short portions, then prompts and long portions), builds every index
 table the kernels need and ships them to the device in ONE packed pinned copy (`RaggedMeta.build`). The kernels of
 `inference/v2/kernels/ragged_ops.py` and `DSInferenceModel.forward_ragged` read the tables from `.meta`.
 """
@@ -66,7 +66,7 @@ class RaggedBatchWrapper:
             raise RuntimeError("cannot finalize an empty ragged batch")
         n = [t.numel() for t in self._toks]
         is_decode = [n[i] == 1 and self._seqs[i].seen_tokens > 0 for i in range(len(n))]
-        self.order = sorted(range(len(n)), key=lambda i: 0 if is_decode[i] else 1)
+        self.order = sorted(range(len(n)), key=lambda i: 0 if is_decode[i] else 1 if n[i] <= RaggedMeta.SHORT_TOKENS else 2)
         seqs = [self._seqs[i] for i in self.order]
         bs = self._block_size or seqs[0].block_size
         rows = None

@@ -6,10 +6,11 @@ plain versions in `ops/reference.py`, as everywhere in `ops`."""
 import torch
 import torch.nn.functional as F
 
-from . import reference
-from .native import hybrid_ops, use_native
+from . import mixer_ops, reference
+from .native import gemv_ops, hybrid_ops, use_native
 
 DECODE_ROWS = 16
+ACTS = {"gelu": 2}  # epilogue codes of the decode products (csrc/gemv/skinny_*.hip)
 
 
 def stream_norm(x, y, mix, out, m, in_, w, eps, ids=None, embed=None, rows=None):
@@ -65,16 +66,18 @@ def delta_rule(proj, conv_w, a_log, dt_bias, norm_w, eps, state, conv_state, met
     return out
 
 
-def linear(x, w, sh=None):
+def linear(x, w, sh=None, act=None):
     """x . w^T: a weight stream for decode-sized bf16 batches (over the shuffled copy `sh`, a `Bf16Weight`, from two
-    rows up), else the library product."""
+    rows up), else the library product. act "gelu": the exact gelu of it (the stream's epilogue, else a pass of its own)."""
     rows = x.numel() // x.shape[-1]
+    code = None if act is None else ACTS[act]
     if sh is not None and x.is_cuda and 2 <= rows <= DECODE_ROWS:
-        return hybrid_ops().decode_linear_sh(x, sh.wsh, sh.shape[0])
+        return gemv_ops().decode_linear_sh(x, sh.wsh, sh.shape[0], act=code)
     if x.is_cuda and x.dtype == torch.bfloat16 and 0 < rows <= DECODE_ROWS and \
-            hybrid_ops().decode_linear_ok(rows, x.shape[-1]):
-        return hybrid_ops().decode_linear(x, w)
-    return F.linear(x, w)
+            gemv_ops().decode_linear_ok(rows, x.shape[-1]):
+        return gemv_ops().decode_linear(x, w, act=code)
+    y = F.linear(x, w)
+    return y if act is None else mixer_ops.gelu(y)
 
 
 def glu_linear(x, w, sh, limit):
@@ -82,7 +85,7 @@ def glu_linear(x, w, sh, limit):
     rows = x.numel() // x.shape[-1]
     if x.is_cuda and x.dtype == torch.bfloat16 and 0 < rows <= DECODE_ROWS:
         if sh is not None and rows >= 2:
-            return hybrid_ops().decode_linear_sh(x, sh.wsh, sh.shape[0], limit)
-        if hybrid_ops().decode_linear_ok(rows, x.shape[-1]):
-            return hybrid_ops().decode_linear(x, w, limit)
+            return gemv_ops().decode_linear_sh(x, sh.wsh, sh.shape[0], limit)
+        if gemv_ops().decode_linear_ok(rows, x.shape[-1]):
+            return gemv_ops().decode_linear(x, w, limit)
     return clamped_glu(F.linear(x, w), limit)

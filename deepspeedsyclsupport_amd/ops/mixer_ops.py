@@ -1,0 +1,124 @@
+"""Ops of hybrid decoders without residual streams (`inference/model_implementations/hybrid.py`): norms on sublayer
+outputs, latent attention, recurrences with a scalar decay per head, gated norms, token-side inputs.
+
+Device tensors run the gfx950 kernels of `ds_mixer_ops` (fp32 or bf16 storage); host tensors the plain versions in
+`ops/reference.py`, as everywhere in `ops`. Residual, norms, angles, scores, softmax, decays and the recurrent state are
+fp32 whatever the storage type."""
+from dataclasses import dataclass
+
+import torch
+import torch.nn.functional as F
+
+from . import reference
+from .native import mixer_ops, use_native
+
+
+def post_norm(x, y, w, eps, ids=None, embed=None, rows=None, final_w=None, mult=1.0):
+    """Residual x [T, W] fp32, in place: x += y / rms(y) * w, or x = embed[ids]. Returns x in y's (embed's) type, the
+    next sublayer's input. With `rows`: x stays, and those rows of the sum come back RMS-normed by `final_w`, times
+    `mult`."""
+    f = mixer_ops().post_norm if use_native(x) else reference.post_norm
+    return f(x, y, w, eps, ids, embed, rows, final_w, mult)
+
+
+def gelu(x):
+    """Exact gelu."""
+    return mixer_ops().gelu(x) if use_native(x) else reference.gelu_erf(x)
+
+
+def token_gate(g, ids, table, first):
+    """gelu_tanh(g) * table[ids, first:first + width]."""
+    f = mixer_ops().token_gate if use_native(g) else reference.token_gate
+    return f(g, ids, table, first)
+
+
+def gated_norm(y, proj, gate, w, parts, eps, mode):
+    """y [T, C] with the gate columns proj[:, gate:gate + C]. "silu_before": y silu(gate), then every one of `parts` equal
+    parts of a row by its own rms, times w. "sigmoid_after": the parts of y by their rms, times w sigmoid(gate)."""
+    before = {"silu_before": True, "sigmoid_after": False}[mode]
+    f = mixer_ops().gated_norm if use_native(y) else reference.gated_norm
+    return f(y, proj, gate, w, parts, eps, before)
+
+
+# ------------------------------------------------------------------------------------------------ latent attention
+def latent_prepare(down, qw, kvw, eps, freq, meta, lat, q_rank):
+    """Projection rows [q latent | kv latent | rotated part] -> normed query latent [T, q_rank]; the normed latent and the
+    rotated part of every token go into the paged cache lat [blocks, 1, block, kv_rank + rot]."""
+    f = mixer_ops().latent_prepare if use_native(down) else reference.latent_prepare
+    return f(down, qw, kvw, eps, freq, meta.pos_ids, meta.seq_ids, meta.block_tables, lat, q_rank)
+
+
+def latent_attention(q, lat, ukv, ukt, freq, sink, meta, scale, d, e):
+    """q [T, H, d + rot] (not rotated yet) of a ragged batch over the paged latents -> [T, H, e].
+
+    Decodes and short portions fold the key map into the query and attend to the latents themselves (every cached byte is
+    read once for all heads); longer portions expand keys and values of their context with one product and run tiled
+    attention per head. ukv [H (d + e), kv_rank]: key rows, then value rows; ukt [H, kv_rank, d]: the key map per head."""
+    T, H, R = q.shape[0], q.shape[1], ukt.shape[1]
+    if not use_native(q):
+        return reference.latent_attention(q, lat, ukv, freq, sink, meta.block_tables, meta.pos_ids, meta.seq_ids, scale, d, e)
+    ops = mixer_ops()
+    tiled = q.dtype == torch.bfloat16 and ops.latent_tiled_ok(d, q.shape[2] - d, e, R)
+    short = meta.cu_host[meta.n_short] if tiled else T
+    o = q.new_empty(T, H, e)
+    if short:
+        ql = ops.head_linear(q[:short], ukt, freq, meta.pos_ids[:short])
+        if tiled:
+            ol = ops.latent_decode(ql, lat, meta.block_tables, meta.cu_q, meta.start_pos, meta.n_short, meta.n_decode,
+                                   meta.max_len, R, scale, sink)
+        else:
+            ol = ops.latent_generic(ql, lat, meta.block_tables, meta.pos_ids, meta.seq_ids, R, scale, sink)
+        ops.head_linear(ol, ukv[H * d:].view(H, e, R), out=o[:short])
+    if short < T:
+        ctx = ops.latent_gather(lat, meta.block_tables, meta.kv_offs, meta.n_short, meta.kv_total)
+        kv = F.linear(ctx[:, :R], ukv)
+        ops.rotate_tail(q[short:], freq, meta.pos_ids[short:])
+        ops.latent_prefill(q, kv, ctx, meta.start_pos, meta.cu_q, meta.work[meta.n_short - meta.n_decode:], meta.kv_offs,
+                           meta.n_short, d, e, scale, sink, o)
+    return o
+
+
+# ------------------------------------------------------------------------------------------------ recurrences
+@dataclass(frozen=True)
+class ScanLayout:
+    """Where a fused projection row [rows] holds what. q, k [Hk heads of dk], v [H heads of dv] and the output gate start
+    at the given columns. With taps > 1, columns conv .. conv + channels (they hold q, k and v) pass a causal convolution
+    with bias; q, k and v pass silu either way. dt: first of H step-size columns, or -1 (constant decays, step 1)."""
+    rows: int
+    q: int
+    k: int
+    v: int
+    gate: int
+    Hk: int
+    H: int
+    dk: int
+    dv: int
+    taps: int = 1
+    conv: int = 0
+    channels: int = 0
+    dt: int = -1
+
+    @property
+    def dks(self):
+        """Key width as the state is stored."""
+        return -(-self.dk // 8) * 8
+
+
+def decayed_scan(proj, lay, state, meta, conv_w=None, conv_b=None, conv_state=None, a_log=None, dt_bias=None, skip=None,
+                 log_decay=None):
+    """S_t = a_t S_(t-1) + b_t k_t v_t^T, o_t = S_t^T q_t + skip v_t for every head -> [T, H dv]; state slots
+    [slots, H, dv, dks] fp32 (and the convolution's windows) advance. Step sizes b = softplus(dt + dt_bias) with
+    a = exp(-exp(a_log) b), or b = 1 with a = exp(log_decay).
+
+    Portions up to `RaggedMeta.STEP_TOKENS` go token by token, longer ones by chunks."""
+    ops = mixer_ops() if use_native(proj) else reference
+    dims = (lay.rows, lay.q, lay.k, lay.v, lay.Hk, lay.H, lay.dk, lay.dv, lay.taps, lay.conv, lay.channels, lay.dt)
+    qk, v, gb = ops.scan_prepare(proj, dims, conv_w, conv_b, conv_state, a_log, dt_bias, meta.seq_ids, meta.cu_q,
+                                 meta.start_pos, meta.slots)
+    out = proj.new_empty(proj.shape[0], lay.H * lay.dv)
+    args = (qk, v, gb, log_decay, skip, proj, dims, state, conv_state)
+    if meta.seq_list.numel():
+        ops.scan_recur(*args, meta.seq_list, meta.cu_q, meta.start_pos, meta.slots, out)
+    if meta.chunk_seqs.numel():
+        ops.scan_chunk(*args, meta.chunk_seqs, meta.cu_q, meta.start_pos, meta.slots, out)
+    return out

@@ -20,8 +20,20 @@ def hip_ops():
 
 @functools.lru_cache(None)
 def hybrid_ops():
-    """The gfx950 ops of the hybrid decoder (a module of its own, see `op_builder.EXTENSIONS`)."""
+    """The gfx950 ops of hybrid decoders with residual streams (a module of its own, see `op_builder.EXTENSIONS`)."""
     return op_builder.load("ds_hybrid_ops")
+
+
+@functools.lru_cache(None)
+def mixer_ops():
+    """The gfx950 ops of `ops/mixer_ops.py`."""
+    return op_builder.load("ds_mixer_ops")
+
+
+@functools.lru_cache(None)
+def gemv_ops():
+    """bf16 decode products, shared by the hybrid decoders."""
+    return op_builder.load("ds_gemv_ops")
 
 
 @functools.lru_cache(None)

@@ -230,3 +230,122 @@ def delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, cu, start
 def delta_chunk(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs, work, cu, start, slots, out, dk):
     """Long portions: the same recurrence (the device splits it into chunks)."""
     delta_recur(qk, v, gb, proj, norm_w, eps, state, conv_state, seqs[:, 0], cu, start, slots, out, dk)
+
+
+# ---------------------------------------------------------------- latent attention, decayed scans, post-norm residual
+def _rms(x, eps):
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def post_norm(x, y, w, eps, ids, embed, rows, final_w, mult):
+    if y is None:
+        x.copy_(embed.float()[ids.long()])
+        return x.to(embed.dtype)
+    s = x + _rms(y.float().view(x.shape), eps) * w
+    if rows is not None:
+        return (_rms(s[rows.long()], eps) * final_w * mult).to(y.dtype)
+    x.copy_(s)
+    return x.to(y.dtype)
+
+
+def gelu_erf(x):
+    return F.gelu(x.float()).to(x.dtype)
+
+
+def token_gate(g, ids, table, first):
+    e = table[ids.long(), first:first + g.shape[-1]].float()
+    return (F.gelu(g.float(), approximate="tanh") * e).to(g.dtype)
+
+
+def gated_norm(y, proj, gate, w, parts, eps, before):
+    T, C = y.shape
+    g, v = proj[:, gate:gate + C].float(), y.float()
+    if before:
+        v = v * F.silu(g)
+    v = _rms(v.view(T, parts, C // parts), eps).view(T, C) * w
+    return (v if before else v * torch.sigmoid(g)).to(y.dtype)
+
+
+def _turn(x, freq, pos):
+    """Rotate-half on the first 2 len(freq) columns of x [T, .., r] at positions pos [T]."""
+    h = freq.numel()
+    a = (pos.double()[:, None] * freq.double()).view(-1, *[1] * (x.dim() - 2), h)
+    c, s = a.cos().float(), a.sin().float()
+    u, v = x[..., :h], x[..., h:2 * h]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * h:]], -1)
+
+
+def latent_prepare(down, qw, kvw, eps, freq, pos, seq_ids, block_table, lat, q_rank):
+    R, BS = kvw.numel(), lat.shape[2]
+    d = down.float()
+    rows = torch.cat([_rms(d[:, q_rank:q_rank + R], eps) * kvw, _turn(d[:, q_rank + R:], freq, pos)], -1)
+    slot = pos.long()
+    lat[block_table.long()[seq_ids.long(), slot // BS], 0, slot % BS] = rows.to(lat.dtype)
+    return (_rms(d[:, :q_rank], eps) * qw).to(down.dtype)
+
+
+def latent_attention(q, lat, ukv, freq, sink, block_table, pos, seq_ids, scale, d, e):
+    T, H = q.shape[:2]
+    R, BS = ukv.shape[1], lat.shape[2]
+    uk, uv = ukv.float().split([H * d, H * e])
+    q = torch.cat([q[..., :d].float(), _turn(q[..., d:].float(), freq, pos)], -1)
+    out = q.new_empty(T, H, e, dtype=ukv.dtype)
+    for s in seq_ids.unique().tolist():
+        rows = (seq_ids == s).nonzero().view(-1)
+        j = torch.arange(int(pos[rows].max()) + 1)
+        c = lat[block_table[s].long()[j // BS], 0, j % BS].float()
+        k = torch.cat([(c[:, :R] @ uk.t()).view(-1, H, d), c[:, None, R:].expand(-1, H, -1)], -1)
+        v = (c[:, :R] @ uv.t()).view(-1, H, e)
+        sc = torch.einsum("thd,jhd->htj", q[rows], k) * scale
+        sc = sc.masked_fill(j > pos[rows][:, None], float("-inf"))
+        p = torch.cat([sc, sink[:, None, None].expand(-1, rows.numel(), 1)], -1).softmax(-1)[..., :-1]
+        out[rows] = torch.einsum("htj,jhe->the", p, v).to(out.dtype)
+    return out
+
+
+def _scan_dims(dims):
+    return dict(zip(("rows", "q", "k", "v", "Hk", "H", "dk", "dv", "taps", "conv", "channels", "dt"), dims))
+
+
+def scan_prepare(proj, dims, conv_w, conv_b, conv_state, a_log, dt_bias, seq_ids, cu, start, slots):
+    D = _scan_dims(dims)
+    T, x = proj.shape[0], proj.float().clone()
+    if conv_w is not None:
+        c0, C, taps = D["conv"], D["channels"], D["taps"]
+        for i in range(start.numel()):
+            a, b = int(cu[i]), int(cu[i + 1])
+            old = conv_state[int(slots[i])].float() if int(start[i]) and taps > 1 else torch.zeros(taps - 1, C)
+            seq = torch.cat([old, proj[a:b, c0:c0 + C].float()])
+            x[a:b, c0:c0 + C] = sum(seq[j:j + b - a] * conv_w[:, j] for j in range(taps)) + conv_b
+    part = lambda at, n, w: F.silu(x[:, at:at + n * w]).view(T, n, w).to(proj.dtype)
+    qk = torch.stack([part(D["q"], D["Hk"], D["dk"]), part(D["k"], D["Hk"], D["dk"])], 1)
+    gb = None
+    if D["dt"] >= 0:
+        b = F.softplus(proj[:, D["dt"]:D["dt"] + D["H"]].float() + dt_bias)
+        gb = torch.stack([-a_log.exp() * b, b], 1)
+    return qk, part(D["v"], D["H"], D["dv"]), gb
+
+
+def scan_recur(qk, v, gb, log_decay, skip, proj, dims, state, conv_state, seqs, cu, start, slots, out):
+    D = _scan_dims(dims)
+    T, H, dk = proj.shape[0], D["H"], D["dk"]
+    rep, out = H // D["Hk"], out.view(T, H, D["dv"])
+    for i in seqs.tolist():
+        a, b, slot = int(cu[i]), int(cu[i + 1]), int(slots[i])
+        S = state[slot, ..., :dk].transpose(1, 2).clone() if int(start[i]) else torch.zeros(H, dk, D["dv"])
+        for t in range(a, b):
+            q, k = qk[t].float().repeat_interleave(rep, 1)
+            g, step = (gb[t, 0], gb[t, 1]) if gb is not None else (log_decay, torch.ones(H))
+            S = S * g.exp()[:, None, None] + (k * step[:, None])[:, :, None] * v[t].float()[:, None]
+            o = (S * q[:, :, None]).sum(1)
+            out[t] = (o if skip is None else o + skip[:, None] * v[t].float()).to(out.dtype)
+        state[slot, ..., :dk] = S.transpose(1, 2)
+        if conv_state is not None and conv_state.shape[1]:
+            old = conv_state[slot] if int(start[i]) else torch.zeros_like(conv_state[slot])
+            new = proj[a:b, D["conv"]:D["conv"] + D["channels"]]
+            conv_state[slot] = torch.cat([old, new])[-(D["taps"] - 1):].clone()
+
+
+def scan_chunk(qk, v, gb, log_decay, skip, proj, dims, state, conv_state, seqs, cu, start, slots, out):
+    """Long portions: the same recurrence (the device splits it into chunks)."""
+    scan_recur(qk, v, gb, log_decay, skip, proj, dims, state, conv_state, seqs[:, 0], cu, start, slots, out)
