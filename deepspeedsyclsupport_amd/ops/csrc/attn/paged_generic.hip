@@ -3,18 +3,21 @@
 //
 // One wave per (token, query head): 64 keys at a time, a lane per key for the scores, then a lane per value column
 // for the weighted sum. Scores, softmax and sums are fp32. A key j is visible to position i if lo(i) <= j <= i, where
-// lo is i - window + 1 (sliding window), the start of i's chunk (chunked attention), or 0. Optional tanh soft cap.
+// lo is i - window + 1 (sliding window), the start of i's chunk (chunked attention), or 0. Optional tanh soft cap;
+// optional sink: exp(sink of the head) joins the softmax's denominator. Value rows may lie further apart than their
+// width: latent attention's values are the first columns of its keys.
 #include "ds_hip.h"
 
 namespace {
 
-constexpr int MAXD = 512;  // query / key width (LDS) and value width (8 columns per lane)
+constexpr int MAXD = 1024;  // query / key width (LDS) and value width (16 columns per lane)
 
 template <typename T>
 __global__ void __launch_bounds__(64) paged_generic_kernel(
     const T* __restrict__ q, const T* __restrict__ kc, const T* __restrict__ vc, T* __restrict__ o,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ pos, const int* __restrict__ seq_ids,
-    int H, int G, int dk, int dv, int BS, float scale, float softcap, int window, int chunk) {
+    int H, int G, int dk, int dv, int vrow, int BS, float scale, float softcap, int window, int chunk,
+    const float* __restrict__ sink) {
   __shared__ float qs[MAXD];
   __shared__ float ps[64];
   __shared__ int64_t slot_s[64];
@@ -53,10 +56,16 @@ __global__ void __launch_bounds__(64) paged_generic_kernel(
       if (i * 64 >= dv) break;
       float a = acc[i] * alpha;
       if (c < dv)
-        for (int j = 0; j < nk; ++j) a = fmaf(ps[j], (float)vc[slot_s[j] * dv + c], a);
+        for (int j = 0; j < nk; ++j) a = fmaf(ps[j], (float)vc[slot_s[j] * vrow + c], a);
       acc[i] = a;
     }
     __syncthreads();
+  }
+  if (sink) {  // (in the frame of the maximum; a sink far above every score takes all the weight)
+    const float mn = fmaxf(m, sink[h]), alpha = expf(m - mn);
+    l = l * alpha + expf(sink[h] - mn);
+#pragma unroll
+    for (int i = 0; i < MAXD / 64; ++i) acc[i] *= alpha;
   }
   T* orow = o + ((int64_t)t * H + h) * dv;
 #pragma unroll
@@ -69,14 +78,16 @@ __global__ void __launch_bounds__(64) paged_generic_kernel(
 }  // namespace
 
 extern "C" int ds_paged_generic(const void* q, const void* kc, const void* vc, void* o, const int* bt, int max_blocks,
-                                const int* pos, const int* seq_ids, int tokens, int H, int G, int dk, int dv, int BS,
-                                float scale, float softcap, int window, int chunk, int dtype, hipStream_t st) {
+                                const int* pos, const int* seq_ids, int tokens, int H, int G, int dk, int dv, int vrow,
+                                int BS, float scale, float softcap, int window, int chunk, const float* sink, int dtype,
+                                hipStream_t st) {
   if (tokens <= 0) return 0;
-  if (G <= 0 || H % G || dk <= 0 || dv <= 0 || dk > MAXD || dv > MAXD || BS <= 0 || H > 65535)
+  if (G <= 0 || H % G || dk <= 0 || dv <= 0 || vrow < dv || dk > MAXD || dv > MAXD || BS <= 0 || H > 65535)
     return (int)hipErrorInvalidValue;
 #define GO(T)                                                                                                        \
   hipLaunchKernelGGL((paged_generic_kernel<T>), dim3(tokens, H), dim3(64), 0, st, (const T*)q, (const T*)kc,         \
-                     (const T*)vc, (T*)o, bt, max_blocks, pos, seq_ids, H, G, dk, dv, BS, scale, softcap, window, chunk)
+                     (const T*)vc, (T*)o, bt, max_blocks, pos, seq_ids, H, G, dk, dv, vrow, BS, scale, softcap, window, chunk, \
+                     sink)
   if (dtype == DS_F32) GO(float);
   else if (dtype == DS_BF16) GO(bf16);
   else return (int)hipErrorInvalidValue;

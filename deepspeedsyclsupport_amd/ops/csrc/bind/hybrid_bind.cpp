@@ -1,13 +1,7 @@
 // Module of the hybrid decoder's ops: multi-stream residual + norm, QKV epilogue with per-head norms, ragged paged
-// attention with chunked / windowed visibility and score capping, gated delta rule, clamped gated activation, and the
-// bf16 decode products they are used with. A shared object of its own, so that serving such a model compiles only this.
-#include <torch/extension.h>
-#include <ATen/hip/HIPContext.h>
-#include <hip/hip_runtime_api.h>
-
-#include <map>
-#include <optional>
-#include <utility>
+// attention with chunked / windowed visibility and score capping, gated delta rule, clamped gated activation. A shared
+// object of its own, so that serving such a model compiles only this and the decode products (gemv_bind.cpp).
+#include "bind_util.h"
 
 extern "C" {
 int ds_stream_norm(float*, const void*, const int*, const void*, const int*, int, int, const float*, const float*, float,
@@ -16,7 +10,7 @@ int ds_clamped_glu(const void*, void*, int64_t, int, float, float, float, int, h
 int ds_qk_norm_append(const void*, const float*, const float*, float, const void*, int64_t, const float*, const int*,
                       const int*, const int*, int, void*, void*, void*, int, int, int, int, int, int, int, hipStream_t);
 int ds_paged_generic(const void*, const void*, const void*, void*, const int*, int, const int*, const int*, int, int, int,
-                     int, int, int, float, float, int, int, int, hipStream_t);
+                     int, int, int, int, float, float, int, int, const float*, int, hipStream_t);
 int ds_delta_prepare(const void*, const float*, const void*, const float*, const float*, const int*, const int*,
                      const int*, const int*, float*, void*, float*, int, int, int, int, int, int, int, hipStream_t);
 int ds_delta_recur(const float*, const void*, const float*, const void*, const float*, float, float*, void*, const int*,
@@ -30,42 +24,9 @@ int ds_paged_prefill_ext(const void*, const void*, const void*, void*, const int
 int ds_paged_decode_splits(int, int, int);
 int ds_paged_decode_ext(const void*, const void*, const void*, const int*, const int*, float*, float*, void*, int, int,
                         int, int, int, int, int, int, int, float, float, int, int, hipStream_t);
-int ds_skinny_gemm(const void*, const void*, const void*, const void*, const void*, const void*, void*, void*, int, int,
-                   int, int, int, int, float, hipStream_t);
-int ds_skinny_b16_mfma_ok(int, int);
-int ds_skinny_b16_mfma(const void*, const void*, const void*, void*, float*, int, int, int, hipStream_t);
-int ds_skinny_finalize_gated(float*, const void*, void*, int, int, int, int, float, hipStream_t);
-int ds_skinny_mfma_ok(int, int, int);
-int ds_skinny_mfma(const void*, const void*, const void*, const void*, const void*, const void*, void*, void*, int, int,
-                   int, int, int, int, float, hipStream_t);
 }
-
-using torch::Tensor;
-using OptT = std::optional<Tensor>;
 
 namespace {
-hipStream_t stream() { return at::hip::getCurrentHIPStream().stream(); }
-void check(int rc, const char* what) { TORCH_CHECK(rc == 0, what, " failed: ", hipGetErrorString((hipError_t)rc)); }
-int dcode(const Tensor& t) {
-  if (t.scalar_type() == at::kFloat) return 0;
-  TORCH_CHECK(t.scalar_type() == at::kBFloat16, "fp32 or bf16 tensors");
-  return 1;
-}
-void need(const Tensor& t, const char* n) {
-  TORCH_CHECK(t.is_cuda() && t.is_contiguous(), n, " must be a contiguous device tensor");
-}
-const float* f32(const Tensor& t, int64_t n, const char* name) {
-  need(t, name);
-  TORCH_CHECK(t.scalar_type() == at::kFloat && t.numel() == n, name, ": fp32 with ", n, " elements");
-  return t.data_ptr<float>();
-}
-const int* i32(const Tensor& t, int64_t n, const char* name) {
-  need(t, name);
-  TORCH_CHECK(t.scalar_type() == at::kInt && t.numel() == n, name, ": int32 with ", n, " elements");
-  return t.data_ptr<int>();
-}
-bool has(const OptT& t) { return t.has_value() && t->defined(); }
-
 // x [T, S, W] fp32 (updated in place unless `rows`). Either y [T, W] with mix [S, S] / out [S] (finish a sublayer), or
 // ids [T] + embed [V, W] (start of the model). Returns the normed rows [R, W] in y's / embed's type.
 Tensor stream_norm(Tensor x, OptT y, OptT mix, OptT out, double m, OptT in, Tensor w, double eps, OptT ids, OptT embed,
@@ -160,12 +121,12 @@ Tensor paged_generic(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor 
   const int64_t T = q.size(0), H = q.size(1);
   TORCH_CHECK(q.dim() == 3 && q.size(2) == c.dk && H % c.G == 0 && q.scalar_type() == kc.scalar_type(), "paged_generic: q");
   TORCH_CHECK(block_table.dim() == 2 && block_table.scalar_type() == at::kInt, "block_table [S, M] int32");
-  TORCH_CHECK(c.dk <= 512 && c.dv <= 512, "paged_generic: head sizes up to 512");
+  TORCH_CHECK(c.dk <= 1024 && c.dv <= 1024, "paged_generic: head sizes up to 1024");
   auto o = torch::empty({T, H, c.dv}, q.options());
   check(ds_paged_generic(q.data_ptr(), kc.data_ptr(), vc.data_ptr(), o.data_ptr(), block_table.data_ptr<int>(),
                          (int)block_table.size(1), i32(pos, T, "pos"), i32(seq_ids, T, "seq_ids"), (int)T, (int)H, c.G,
-                         c.dk, c.dv, c.BS, (float)scale, (float)softcap, (int)window, (int)chunk, dcode(q), stream()),
-        "paged_generic");
+                         c.dk, c.dv, c.dv, c.BS, (float)scale, (float)softcap, (int)window, (int)chunk, nullptr, dcode(q),
+                         stream()), "paged_generic");
   return o;
 }
 
@@ -293,54 +254,6 @@ void delta_chunk(Tensor qk, Tensor v, Tensor gb, Tensor proj, Tensor norm_w, dou
                        o.data_ptr<float>(), out.data_ptr(), (int)T, (int)Hk, (int)H, (int)dk, (int)dv, (int)taps, dcode(proj),
                        stream()), "delta_chunk");
 }
-
-bool decode_linear_ok(int64_t M, int64_t K) {
-  return M >= 1 && K % 8 == 0 && (M <= 8 || (M <= 16 && ds_skinny_mfma_ok((int)M, (int)K, 0)));
-}
-constexpr int CLAMPED_GLU = 5;  // DS_ACT_CLAMPED_GLU
-
-// x [M, K] . w [N, K]^T for M <= 16 bf16 rows: the vector kernel up to two rows (or where K does not tile), else MFMA.
-// With a limit, w is a fused [gate | up] weight and the result its clamped gated activation [M, N / 2].
-Tensor decode_linear(Tensor x, Tensor w, std::optional<double> glu_limit) {
-  need(x, "x"); need(w, "w");
-  const int64_t N = w.size(0), K = w.size(1), M = x.numel() / K;
-  const bool glu = glu_limit.has_value();
-  TORCH_CHECK(x.scalar_type() == at::kBFloat16 && w.scalar_type() == at::kBFloat16 && x.size(-1) == K, "decode_linear");
-  TORCH_CHECK(decode_linear_ok(M, K), "decode_linear: up to 8 rows with K % 8 == 0 (16 with K % 256 == 0)");
-  TORCH_CHECK(!glu || N % 2 == 0, "decode_linear: [gate | up] rows");
-  auto sizes = x.sizes().vec();
-  sizes.back() = glu ? N / 2 : N;
-  auto y = torch::empty(sizes, x.options());
-  auto fn = M > 2 && ds_skinny_mfma_ok((int)M, (int)K, 0) ? ds_skinny_mfma : ds_skinny_gemm;
-  check(fn(w.data_ptr(), x.data_ptr(), nullptr, nullptr, nullptr, nullptr, y.data_ptr(), nullptr, (int)M, (int)N, (int)K,
-           0, glu ? 1 : 0, glu ? CLAMPED_GLU : 0, glu ? (float)*glu_limit : 0.f, stream()), "decode_linear");
-  return y;
-}
-
-// The same over a weight in the shuffled decode layout (ops/bf16_gemv.py: preshuffle16), w [N, K], K % 64 == 0
-Tensor decode_linear_sh(Tensor x, Tensor wsh, int64_t N, std::optional<double> glu_limit) {
-  need(x, "x"); need(wsh, "wsh");
-  const int64_t K = x.size(-1), M = x.numel() / K, NB = (N + 15) / 16;
-  const bool glu = glu_limit.has_value();
-  TORCH_CHECK(x.scalar_type() == at::kBFloat16 && wsh.scalar_type() == at::kBFloat16 && wsh.numel() == NB * 16 * K &&
-              ds_skinny_b16_mfma_ok((int)M, (int)K), "decode_linear_sh: up to 16 bf16 rows, K % 64 == 0");
-  TORCH_CHECK(NB * K < ((int64_t)1 << 40) && N < ((int64_t)1 << 31) / 16, "decode_linear_sh: matrix too large");
-  TORCH_CHECK(!glu || N % 2 == 0, "decode_linear_sh: [gate | up] rows");
-  // fp32 split-K sums, zero between calls (the kernels leave it so); one per device and stream, grown on demand
-  static std::map<std::pair<int, hipStream_t>, Tensor> workspaces;
-  Tensor& ws = workspaces[{x.get_device(), stream()}];
-  const int64_t NP = (NB + 3) / 4 * 64;  // row length of the sums
-  if (!ws.defined() || ws.numel() < 16 * NP) ws = torch::zeros({16 * NP}, x.options().dtype(at::kFloat));
-  auto sizes = x.sizes().vec();
-  sizes.back() = glu ? N / 2 : N;
-  auto y = torch::empty(sizes, x.options());
-  check(ds_skinny_b16_mfma(x.data_ptr(), wsh.data_ptr(), nullptr, glu ? nullptr : y.data_ptr(), ws.data_ptr<float>(),
-                           (int)M, (int)N, (int)K, stream()), "decode_linear_sh");
-  if (glu)
-    check(ds_skinny_finalize_gated(ws.data_ptr<float>(), nullptr, y.data_ptr(), (int)M, (int)N, (int)NP, CLAMPED_GLU,
-                                   (float)*glu_limit, stream()), "decode_linear_sh (gated)");
-  return y;
-}
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -356,8 +269,4 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("paged_tiled_ok", &paged_tiled_ok);
   m.def("paged_prefill", &paged_prefill);
   m.def("paged_decode", &paged_decode);
-  m.def("decode_linear", &decode_linear, py::arg("x"), py::arg("w"), py::arg("glu_limit") = py::none());
-  m.def("decode_linear_ok", &decode_linear_ok);
-  m.def("decode_linear_sh", &decode_linear_sh, py::arg("x"), py::arg("wsh"), py::arg("N"),
-        py::arg("glu_limit") = py::none());
 }

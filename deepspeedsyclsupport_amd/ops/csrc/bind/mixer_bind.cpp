@@ -1,0 +1,350 @@
+// Module of the ops of hybrid decoders without residual streams: norms on sublayer outputs, gated norms, token-side gates,
+// latent attention, recurrences with a scalar decay per head. A shared object of its own, so that serving such a model
+// compiles only this and the decode products (gemv_bind.cpp).
+#include "bind_util.h"
+
+extern "C" {
+int ds_post_norm(float*, const void*, const float*, const int*, const void*, const int*, int, const float*, float, void*, int,
+                 float, int, hipStream_t);
+int ds_gated_norm(const void*, const void*, int64_t, const float*, void*, int64_t, int, int, float, int, int, hipStream_t);
+int ds_gelu(const void*, void*, int64_t, int, hipStream_t);
+int ds_token_gate(const void*, const int*, const void*, int64_t, void*, int64_t, int, int, hipStream_t);
+int ds_latent_prepare(const void*, const float*, const float*, float, const double*, int, const int*, const int*, const int*,
+                      int, void*, void*, int, int, int, int, int, int, hipStream_t);
+int ds_rotate_tail(void*, int, int, int, int, const double*, int, const int*, int, hipStream_t);
+int ds_head_linear(const void*, const void*, void*, int, int, int, int, int, int, int, int, const double*, const int*, int,
+                   hipStream_t);
+int ds_latent_gather(const void*, const int*, int, const int*, int, int, void*, int64_t, int, int, hipStream_t);
+int ds_paged_generic(const void*, const void*, const void*, void*, const int*, int, const int*, const int*, int, int, int,
+                     int, int, int, int, float, float, int, int, const float*, int, hipStream_t);
+int ds_latent_decode_ok(int, int);
+void ds_latent_decode_plan(int, int, int, int, int, int*, int*);
+int ds_latent_decode(const void*, const void*, void*, float*, float*, const int*, int, const int*, const int*, int, int, int,
+                     int, int, int, int, int, int, int, int, const float*, float, hipStream_t);
+int ds_latent_prefill_ok(int, int, int);
+int ds_latent_prefill(const void*, const void*, const void*, void*, const int*, const int*, const int*, int, const int*, int,
+                      int, int, int, int, int, int, const float*, float, hipStream_t);
+int ds_scan_prepare(const void*, const float*, const float*, const void*, const float*, const float*, const int*, const int*,
+                    const int*, const int*, void*, void*, float*, const int*, int, int, hipStream_t);
+int ds_scan_recur(const void*, const void*, const float*, const float*, const float*, const void*, float*, void*, const int*,
+                  int, int, const int*, const int*, const int*, void*, const int*, int, int, hipStream_t);
+int ds_scan_chunk_ok(int);
+int ds_scan_chunk(const void*, const void*, const float*, const float*, const float*, const void*, float*, void*, const int*,
+                  int, const int*, const int*, const int*, void*, const int*, int, hipStream_t);
+}
+
+namespace {
+const float* opt_f32(const OptT& t, int64_t n, const char* name) { return has(t) ? f32(*t, n, name) : nullptr; }
+const double* f64(const Tensor& t, const char* name) {
+  need(t, name);
+  TORCH_CHECK(t.scalar_type() == at::kDouble, name, ": fp64");
+  return t.data_ptr<double>();
+}
+void table(const Tensor& bt, int64_t seqs) {
+  need(bt, "block_table");
+  TORCH_CHECK(bt.dim() == 2 && bt.scalar_type() == at::kInt && bt.size(0) >= seqs, "block_table [S, M] int32");
+}
+
+// x [T, W] fp32, in place. y [T, W] + w: x += y / rms(y) w; ids + embed: x = embed[ids]. -> x in y's / embed's type; with
+// rows: those rows of the sum, normed by final_w, times mult (x stays)
+Tensor post_norm(Tensor x, OptT y, OptT w, double eps, OptT ids, OptT embed, OptT rows, OptT final_w, double mult) {
+  need(x, "x");
+  TORCH_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2, "post_norm: x [T, W] fp32");
+  const int64_t T = x.size(0), W = x.size(1);
+  TORCH_CHECK(has(y) != has(embed), "post_norm: y or embed");
+  const Tensor& src = has(y) ? *y : *embed;
+  need(src, "y / embed");
+  TORCH_CHECK(src.size(-1) == W && (has(embed) || src.numel() == T * W), "post_norm: width");
+  TORCH_CHECK(!has(rows) || has(y), "post_norm: no row list at the start");
+  const int64_t R = has(rows) ? rows->numel() : T;
+  auto out = torch::empty({R, W}, src.options());
+  check(ds_post_norm(x.data_ptr<float>(), has(y) ? y->data_ptr() : nullptr, has(y) ? f32(*w, W, "norm weight") : nullptr,
+                     has(embed) ? i32(*ids, T, "ids") : nullptr, has(embed) ? embed->data_ptr() : nullptr,
+                     has(rows) ? i32(*rows, R, "rows") : nullptr, (int)R, has(rows) ? f32(*final_w, W, "final norm") : nullptr,
+                     (float)mult, out.data_ptr(), (int)W, (float)eps, dcode(src), stream()), "post_norm");
+  return out;
+}
+
+Tensor gated_norm(Tensor y, Tensor proj, int64_t gate, Tensor w, int64_t parts, double eps, bool before) {
+  need(y, "y"); need(proj, "proj");
+  const int64_t T = y.size(0), C = y.size(1);
+  TORCH_CHECK(y.dim() == 2 && proj.dim() == 2 && proj.size(0) == T && gate >= 0 && gate + C <= proj.size(1) &&
+              proj.scalar_type() == y.scalar_type() && parts > 0 && C % parts == 0, "gated_norm: y [T, C], gate columns of proj");
+  auto out = torch::empty_like(y);
+  check(ds_gated_norm(y.data_ptr(), (const char*)proj.data_ptr() + gate * proj.element_size(), proj.size(1), f32(w, C, "norm"),
+                      out.data_ptr(), T, (int)C, (int)parts, (float)eps, before, dcode(y), stream()), "gated_norm");
+  return out;
+}
+
+Tensor gelu(Tensor x) {
+  need(x, "x");
+  auto out = torch::empty_like(x);
+  check(ds_gelu(x.data_ptr(), out.data_ptr(), x.numel(), dcode(x), stream()), "gelu");
+  return out;
+}
+
+Tensor token_gate(Tensor g, Tensor ids, Tensor table_, int64_t first) {
+  need(g, "g"); need(table_, "table");
+  const int64_t D = g.size(-1), T = g.numel() / D;
+  TORCH_CHECK(table_.dim() == 2 && table_.scalar_type() == g.scalar_type() && first >= 0 && first + D <= table_.size(1),
+              "token_gate: table");
+  auto out = torch::empty_like(g);
+  check(ds_token_gate(g.data_ptr(), i32(ids, T, "ids"), (const char*)table_.data_ptr() + first * table_.element_size(),
+                      table_.size(1), out.data_ptr(), T, (int)D, dcode(g), stream()), "token_gate");
+  return out;
+}
+
+// ---------------------------------------------------------------------------------------------- latent attention
+struct Lat {
+  int BS, W;
+};
+Lat lat_of(const Tensor& lat) {
+  need(lat, "latents");
+  TORCH_CHECK(lat.dim() == 4 && lat.size(1) == 1, "latents [blocks, 1, block, width]");
+  return {(int)lat.size(2), (int)lat.size(3)};
+}
+
+// down [T, Q + R + r] -> normed query latent [T, Q]; the cached rows [R + r] of every token are written
+Tensor latent_prepare(Tensor down, Tensor qw, Tensor kvw, double eps, Tensor freq, Tensor pos, Tensor seq_ids, Tensor bt,
+                      Tensor lat, int64_t Q) {
+  need(down, "down"); table(bt, 1);
+  const Lat c = lat_of(lat);
+  const int64_t R = kvw.numel(), r = c.W - R, T = down.size(0), half = freq.numel();
+  TORCH_CHECK(down.dim() == 2 && down.size(1) == Q + c.W && r >= 0 && 2 * half <= r && down.scalar_type() == lat.scalar_type(),
+              "latent_prepare: widths / types");
+  auto cq = torch::empty({T, Q}, down.options());
+  check(ds_latent_prepare(down.data_ptr(), f32(qw, Q, "q norm"), f32(kvw, R, "kv norm"), (float)eps, f64(freq, "freq"),
+                          (int)half, i32(pos, T, "pos"), i32(seq_ids, T, "seq_ids"), bt.data_ptr<int>(), (int)bt.size(1),
+                          lat.data_ptr(), cq.data_ptr(), (int)T, (int)Q, (int)R, (int)r, c.BS, dcode(down), stream()),
+        "latent_prepare");
+  return cq;
+}
+
+// Last columns of every head of q [T, H, row] (the ones behind row - r), rotated in place. q may be rows of a larger batch.
+void rotate_tail(Tensor q, Tensor freq, Tensor pos, int64_t r) {
+  need(q, "q");
+  TORCH_CHECK(q.dim() == 3 && r <= q.size(2) && 2 * freq.numel() <= r, "rotate_tail: q [T, H, row]");
+  check(ds_rotate_tail(q.data_ptr(), (int)q.size(0), (int)q.size(1), (int)q.size(2), (int)r, f64(freq, "freq"),
+                       (int)freq.numel(), i32(pos, q.size(0), "pos"), dcode(q), stream()), "rotate_tail");
+}
+
+// y[t, h] = w[h] x[t, h, :K]: x [T, H, xrow], w [H, N, K]. With freq and pos the columns of x behind K are rotated and put
+// behind the N of y. `out`: [T, H, N] to write into.
+Tensor head_linear(Tensor x, Tensor w, OptT freq, OptT pos, OptT out) {
+  need(x, "x"); need(w, "w");
+  TORCH_CHECK(x.dim() == 3 && w.dim() == 3 && w.size(0) == x.size(1) && w.size(2) <= x.size(2) &&
+              x.scalar_type() == w.scalar_type(), "head_linear: x [T, H, >= K], w [H, N, K]");
+  const int64_t T = x.size(0), H = x.size(1), N = w.size(1), K = w.size(2), r = has(freq) ? x.size(2) - K : 0;
+  const int64_t half = has(freq) ? freq->numel() : 0;
+  TORCH_CHECK(2 * half <= r || !has(freq), "head_linear: rotated columns");
+  Tensor y = has(out) ? *out : torch::empty({T, H, N + r}, x.options());
+  need(y, "out");
+  TORCH_CHECK(y.dim() == 3 && y.size(0) == T && y.size(1) == H && y.size(2) == N + r && y.scalar_type() == x.scalar_type(),
+              "head_linear: out");
+  check(ds_head_linear(x.data_ptr(), w.data_ptr(), y.data_ptr(), (int)T, (int)H, (int)N, (int)K, (int)x.size(2), (int)y.size(2),
+                       (int)r, (int)half, has(freq) ? f64(*freq, "freq") : nullptr, r ? i32(*pos, T, "pos") : nullptr, dcode(x),
+                       stream()), "head_linear");
+  return y;
+}
+
+Tensor latent_generic(Tensor q, Tensor lat, Tensor bt, Tensor pos, Tensor seq_ids, int64_t R, double scale, Tensor sink) {
+  need(q, "q"); table(bt, 1);
+  const Lat c = lat_of(lat);
+  const int64_t T = q.size(0), H = q.size(1);
+  TORCH_CHECK(q.dim() == 3 && q.size(2) == c.W && q.scalar_type() == lat.scalar_type() && R > 0 && R <= c.W, "latent_generic: q");
+  TORCH_CHECK(c.W <= 1024, "latent_generic: rows up to 1024");
+  auto o = torch::empty({T, H, R}, q.options());
+  check(ds_paged_generic(q.data_ptr(), lat.data_ptr(), lat.data_ptr(), o.data_ptr(), bt.data_ptr<int>(), (int)bt.size(1),
+                         i32(pos, T, "pos"), i32(seq_ids, T, "seq_ids"), (int)T, (int)H, 1, c.W, (int)R, c.W, c.BS, (float)scale,
+                         0.f, 0, 0, f32(sink, H, "sink"), dcode(q), stream()), "latent_generic");
+  return o;
+}
+
+bool latent_tiled_ok(int64_t d, int64_t r, int64_t e, int64_t R) {
+  return ds_latent_decode_ok((int)R, (int)r) && ds_latent_prefill_ok((int)d, (int)r, (int)e);
+}
+
+// Tokens tok0 .. tok1 of the batch, those of sequences first .. first + nseq with up to max_new tokens each:
+// q [.., H, R + r] -> out [.., H, R], rows tok0 .. tok1 of both
+void latent_decode(Tensor q, Tensor lat, Tensor bt, Tensor cu, Tensor start, int64_t first, int64_t nseq, int64_t max_new,
+                   int64_t tok0, int64_t tok1, int64_t max_len, int64_t R, double scale, Tensor sink, Tensor out) {
+  need(q, "q"); need(out, "out"); table(bt, first + nseq);
+  const Lat c = lat_of(lat);
+  const int64_t H = q.size(1), n = tok1 - tok0, S = start.numel();
+  TORCH_CHECK(q.dim() == 3 && q.size(2) == c.W && q.scalar_type() == at::kBFloat16 && lat.scalar_type() == at::kBFloat16 &&
+              tok0 >= 0 && n >= 0 && tok1 <= q.size(0) && first >= 0 && first + nseq <= S && max_new > 0 &&
+              bt.size(1) * c.BS >= max_len && ds_latent_decode_ok((int)R, (int)(c.W - R)), "latent_decode: q / latents / tables");
+  TORCH_CHECK(out.dim() == 3 && out.size(0) >= tok1 && out.size(1) == H && out.size(2) == R && out.scalar_type() == q.scalar_type(),
+              "latent_decode: out");
+  int range = 0, splits = 1;
+  ds_latent_decode_plan((int)nseq, (int)max_new, (int)H, c.W, (int)max_len, &range, &splits);
+  Tensor acc, ml;
+  if (splits > 1) {
+    auto fo = q.options().dtype(at::kFloat);
+    acc = torch::empty({splits, n * H, R}, fo);
+    ml = torch::empty({splits, n * H, 2}, fo);
+  }
+  check(ds_latent_decode((const char*)q.data_ptr() + tok0 * H * c.W * 2, lat.data_ptr(), (char*)out.data_ptr() + tok0 * H * R * 2,
+                         splits > 1 ? acc.data_ptr<float>() : nullptr, splits > 1 ? ml.data_ptr<float>() : nullptr,
+                         bt.data_ptr<int>(), (int)bt.size(1), i32(cu, S + 1, "cu"), i32(start, S, "start"), (int)first, (int)nseq,
+                         (int)max_new, (int)tok0, (int)n, (int)H, (int)R, (int)(c.W - R), c.BS, range, splits,
+                         f32(sink, H, "sink"), (float)scale, stream()), "latent_decode");
+}
+
+// cached rows of the contexts of sequences first .. first + nseq, end to end
+Tensor latent_gather(Tensor lat, Tensor bt, Tensor offs, int64_t first, int64_t total) {
+  const Lat c = lat_of(lat);
+  const int64_t nseq = offs.numel() - 1;
+  table(bt, first + nseq);
+  TORCH_CHECK(lat.scalar_type() == at::kBFloat16 && c.W % 8 == 0 && nseq > 0, "latent_gather: bf16 rows of 16-byte pieces");
+  auto ctx = torch::empty({total, c.W}, lat.options());
+  check(ds_latent_gather(lat.data_ptr(), bt.data_ptr<int>(), (int)bt.size(1), i32(offs, nseq + 1, "offs"), (int)first, (int)nseq,
+                         ctx.data_ptr(), total, c.W, c.BS, stream()), "latent_gather");
+  return ctx;
+}
+
+// q [T, H, d + r] rotated; kv [rows, H (d + e)], ctx [rows, R + r] -> rows of o [T, H, e] of the sequences in work
+void latent_prefill(Tensor q, Tensor kv, Tensor ctx, Tensor start, Tensor cu_q, Tensor work, Tensor offs, int64_t first,
+                    int64_t d, int64_t e, double scale, Tensor sink, Tensor o) {
+  need(q, "q"); need(kv, "kv"); need(ctx, "ctx"); need(o, "o");
+  const int64_t T = q.size(0), H = q.size(1), r = q.size(2) - d, S = start.numel();
+  TORCH_CHECK(q.dim() == 3 && q.scalar_type() == at::kBFloat16 && kv.scalar_type() == at::kBFloat16 &&
+              ctx.scalar_type() == at::kBFloat16 && kv.dim() == 2 && kv.size(1) == H * (d + e) && ctx.dim() == 2 &&
+              ctx.size(0) == kv.size(0) && ctx.size(1) >= r && ds_latent_prefill_ok((int)d, (int)r, (int)e), "latent_prefill");
+  TORCH_CHECK(o.dim() == 3 && o.size(0) == T && o.size(1) == H && o.size(2) == e && o.scalar_type() == q.scalar_type() &&
+              work.dim() == 2 && work.size(1) == 2 && offs.numel() == S - first + 1 && scale > 0, "latent_prefill: o / tables");
+  check(ds_latent_prefill(q.data_ptr(), kv.data_ptr(), ctx.data_ptr(), o.data_ptr(), i32(start, S, "start"),
+                          i32(cu_q, S + 1, "cu_q"), i32(work, work.numel(), "work"), (int)work.size(0),
+                          i32(offs, offs.numel(), "offs"), (int)first, (int)H, (int)d, (int)r, (int)e, (int)ctx.size(1),
+                          (int)(ctx.size(1) - r), f32(sink, H, "sink"), (float)scale, stream()), "latent_prefill");
+}
+
+// ---------------------------------------------------------------------------------------------- recurrences
+struct Dims {  // ops/mixer_ops.py: ScanLayout
+  int v[12];
+  int rows() const { return v[0]; }
+  int Hk() const { return v[4]; }
+  int H() const { return v[5]; }
+  int dk() const { return v[6]; }
+  int dv() const { return v[7]; }
+  int taps() const { return v[8]; }
+  int conv() const { return v[9]; }
+  int channels() const { return v[10]; }
+  int dt() const { return v[11]; }
+  int dks() const { return (dk() + 7) / 8 * 8; }
+  int dvs() const { return (dv() + 7) / 8 * 8; }
+};
+Dims dims_of(const std::vector<int64_t>& d) {
+  TORCH_CHECK(d.size() == 12, "scan: 12 dimensions");
+  Dims D;
+  for (int i = 0; i < 12; ++i) D.v[i] = (int)d[i];
+  TORCH_CHECK(D.Hk() > 0 && D.H() > 0 && D.H() % D.Hk() == 0 && D.dk() > 0 && D.dk() <= 512 && D.dv() > 0 && D.taps() >= 1,
+              "scan: head counts / sizes (keys up to 512)");
+  auto inside = [&](int64_t at, int64_t n, int64_t lo, int64_t hi) { return at >= lo && at + n <= hi; };
+  const int64_t nk = (int64_t)D.Hk() * D.dk(), nv = (int64_t)D.H() * D.dv(), lo = D.channels() ? D.conv() : 0,
+                hi = D.channels() ? D.conv() + D.channels() : D.rows();
+  TORCH_CHECK(inside(D.conv(), D.channels(), 0, D.rows()) && inside(D.v[1], nk, lo, hi) && inside(D.v[2], nk, lo, hi) &&
+              inside(D.v[3], nv, lo, hi) && (D.dt() < 0 || inside(D.dt(), D.H(), 0, D.rows())) &&
+              (D.taps() == 1 || D.channels() > 0), "scan: columns outside the projection");
+  return D;
+}
+void conv_ok(const Dims& D, const OptT& cs, const Tensor& proj) {
+  TORCH_CHECK(D.taps() == 1 || (has(cs) && cs->is_cuda() && cs->is_contiguous() && cs->dim() == 3 && cs->size(1) == D.taps() - 1 &&
+              cs->size(2) == D.channels() && cs->scalar_type() == proj.scalar_type()), "scan: conv_state [slots, taps-1, channels]");
+}
+
+// proj [T, rows] -> qk [2, Hk, T, dks], v [H, T, dvs] (storage type), gb [T, 2, H] fp32 or None
+std::tuple<Tensor, Tensor, OptT> scan_prepare(Tensor proj, std::vector<int64_t> dims, OptT conv_w, OptT conv_b, OptT conv_state,
+                                              OptT a_log, OptT dt_bias, Tensor seq_ids, Tensor cu, Tensor start, Tensor slots) {
+  need(proj, "proj");
+  const Dims D = dims_of(dims);
+  const int64_t T = proj.size(0), S = start.numel();
+  TORCH_CHECK(proj.dim() == 2 && proj.size(1) == D.rows(), "scan_prepare: proj [T, rows]");
+  TORCH_CHECK(has(conv_w) == (D.channels() > 0) && has(conv_b) == has(conv_w), "scan_prepare: convolution weights");
+  conv_ok(D, conv_state, proj);
+  // (rows are padded to 16-byte pieces with zeros)
+  auto make = [&](at::IntArrayRef s, bool pad) { return pad ? torch::zeros(s, proj.options()) : torch::empty(s, proj.options()); };
+  Tensor qk = make({2, D.Hk(), T, D.dks()}, D.dks() != D.dk()), v = make({D.H(), T, D.dvs()}, D.dvs() != D.dv());
+  OptT gb;
+  if (D.dt() >= 0) gb = torch::empty({T, 2, D.H()}, proj.options().dtype(at::kFloat));
+  check(ds_scan_prepare(proj.data_ptr(), opt_f32(conv_w, (int64_t)D.channels() * D.taps(), "conv_w"),
+                        opt_f32(conv_b, D.channels(), "conv_b"), D.taps() > 1 ? conv_state->data_ptr() : nullptr,
+                        D.dt() >= 0 ? f32(*a_log, D.H(), "a_log") : nullptr, D.dt() >= 0 ? f32(*dt_bias, D.H(), "dt_bias") : nullptr,
+                        i32(seq_ids, T, "seq_ids"), i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"),
+                        qk.data_ptr(), v.data_ptr(), gb ? gb->data_ptr<float>() : nullptr, D.v, (int)T, dcode(proj), stream()),
+        "scan_prepare");
+  return {qk, v, gb};
+}
+
+struct ScanCheck {
+  ScanCheck(const Dims& D, const Tensor& qk, const Tensor& v, const OptT& gb, const OptT& ld, const Tensor& proj,
+            const Tensor& state, const OptT& conv_state, const Tensor& out) {
+    need(qk, "qk"); need(v, "v"); need(proj, "proj"); need(state, "state"); need(out, "out");
+    const int64_t T = proj.size(0);
+    TORCH_CHECK(proj.size(1) == D.rows() && qk.numel() == 2 * D.Hk() * T * D.dks() && v.numel() == D.H() * T * D.dvs() &&
+                qk.scalar_type() == proj.scalar_type() && v.scalar_type() == proj.scalar_type(), "scan: qk / v");
+    TORCH_CHECK(has(gb) != has(ld), "scan: decays per token or per head");
+    TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == D.H() && state.size(2) == D.dv() &&
+                state.size(3) == D.dks(), "scan: state [slots, H, dv, dks] fp32");
+    TORCH_CHECK(out.numel() == T * D.H() * D.dv() && out.scalar_type() == proj.scalar_type(), "scan: out [T, H dv]");
+    conv_ok(D, conv_state, proj);
+    TORCH_CHECK(D.taps() == 1 || conv_state->size(0) == state.size(0), "scan: slots");
+  }
+};
+
+// Runs the sequences in `list` token by token; writes their rows of out and their state slots
+void recur_list(Tensor qk, Tensor v, OptT gb, OptT log_decay, OptT skip, Tensor proj, const Dims& D, Tensor state,
+                OptT conv_state, Tensor list, int stride, Tensor cu, Tensor start, Tensor slots, Tensor out) {
+  const int64_t T = proj.size(0), S = start.numel();
+  check(ds_scan_recur(qk.data_ptr(), v.data_ptr(), opt_f32(gb, T * 2 * D.H(), "gb"), opt_f32(log_decay, D.H(), "log_decay"),
+                      opt_f32(skip, D.H(), "skip"), proj.data_ptr(), state.data_ptr<float>(),
+                      D.taps() > 1 ? conv_state->data_ptr() : nullptr, i32(list, list.numel(), "list"),
+                      (int)(list.numel() / stride), stride, i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"),
+                      out.data_ptr(), D.v, (int)T, dcode(proj), stream()), "scan_recur");
+}
+
+void scan_recur(Tensor qk, Tensor v, OptT gb, OptT log_decay, OptT skip, Tensor proj, std::vector<int64_t> dims, Tensor state,
+                OptT conv_state, Tensor list, Tensor cu, Tensor start, Tensor slots, Tensor out) {
+  const Dims D = dims_of(dims);
+  ScanCheck(D, qk, v, gb, log_decay, proj, state, conv_state, out);
+  recur_list(qk, v, gb, log_decay, skip, proj, D, state, conv_state, list, 1, cu, start, slots, out);
+}
+
+// The same for long portions, seqs [n, 2]: bf16 by chunks of 64 tokens on the matrix cores; fp32 (and key widths above 256)
+// token by token
+void scan_chunk(Tensor qk, Tensor v, OptT gb, OptT log_decay, OptT skip, Tensor proj, std::vector<int64_t> dims, Tensor state,
+                OptT conv_state, Tensor seqs, Tensor cu, Tensor start, Tensor slots, Tensor out) {
+  const Dims D = dims_of(dims);
+  ScanCheck(D, qk, v, gb, log_decay, proj, state, conv_state, out);
+  TORCH_CHECK(seqs.dim() == 2 && seqs.size(1) == 2, "scan_chunk: seqs [n, 2]");
+  if (proj.scalar_type() != at::kBFloat16 || !ds_scan_chunk_ok(D.dk())) {
+    recur_list(qk, v, gb, log_decay, skip, proj, D, state, conv_state, seqs, 2, cu, start, slots, out);
+    return;
+  }
+  const int64_t T = proj.size(0), S = start.numel();
+  check(ds_scan_chunk(qk.data_ptr(), v.data_ptr(), opt_f32(gb, T * 2 * D.H(), "gb"), opt_f32(log_decay, D.H(), "log_decay"),
+                      opt_f32(skip, D.H(), "skip"), proj.data_ptr(), state.data_ptr<float>(),
+                      D.taps() > 1 ? conv_state->data_ptr() : nullptr, i32(seqs, seqs.numel(), "seqs"), (int)seqs.size(0),
+                      i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"), out.data_ptr(), D.v, (int)T, stream()),
+        "scan_chunk");
+}
+}  // namespace
+
+PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.def("post_norm", &post_norm);
+  m.def("gated_norm", &gated_norm);
+  m.def("gelu", &gelu);
+  m.def("token_gate", &token_gate);
+  m.def("latent_prepare", &latent_prepare);
+  m.def("rotate_tail", &rotate_tail);
+  m.def("head_linear", &head_linear, py::arg("x"), py::arg("w"), py::arg("freq") = py::none(), py::arg("pos") = py::none(),
+        py::arg("out") = py::none());
+  m.def("latent_generic", &latent_generic);
+  m.def("latent_tiled_ok", &latent_tiled_ok);
+  m.def("latent_decode", &latent_decode);
+  m.def("latent_gather", &latent_gather);
+  m.def("latent_prefill", &latent_prefill);
+  m.def("scan_prepare", &scan_prepare);
+  m.def("scan_recur", &scan_recur);
+  m.def("scan_chunk", &scan_chunk);
+}

@@ -100,6 +100,17 @@ __global__ void __launch_bounds__(256) finalize_plain_kernel(float* __restrict__
   if (n < N) y[(int64_t)t * N + n] = (bf16)(v + (bias ? (float)bias[n] : 0.f));
 }
 
+// y = bf16(act(acc)), workspace re-zeroed
+__global__ void __launch_bounds__(256) finalize_act_kernel(float* __restrict__ acc, bf16* __restrict__ y, int M, int N, int NP,
+                                                           int act) {
+  const int64_t e = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (e >= (int64_t)M * NP) return;
+  const int t = (int)(e / NP), n = (int)(e % NP);
+  const float v = acc[e];
+  acc[e] = 0.f;
+  if (n < N) y[(int64_t)t * N + n] = (bf16)act_any(act, v);
+}
+
 }  // namespace
 
 extern "C" int ds_skinny_finalize_rms(float* ws, const void* bias, const void* residual, const void* w, void* y,
@@ -133,6 +144,14 @@ extern "C" int ds_skinny_finalize_plain(float* ws, const void* bias, void* y, in
   if (M < 1 || M > 16 || N < 1 || NP < N) return (int)hipErrorInvalidValue;
   hipLaunchKernelGGL(finalize_plain_kernel, dim3((int)(((int64_t)M * NP + 255) / 256)), dim3(256), 0, st, ws,
                      (const bf16*)bias, (bf16*)y, M, N, NP);
+  DS_CHECK_LAUNCH();
+  return 0;
+}
+
+extern "C" int ds_skinny_finalize_act(float* ws, void* y, int M, int N, int NP, int act, hipStream_t st) {
+  if (M < 1 || M > 16 || N < 1 || NP < N) return (int)hipErrorInvalidValue;
+  hipLaunchKernelGGL(finalize_act_kernel, dim3((int)(((int64_t)M * NP + 255) / 256)), dim3(256), 0, st, ws, (bf16*)y, M, N,
+                     NP, act);
   DS_CHECK_LAUNCH();
   return 0;
 }

@@ -237,6 +237,10 @@ __global__ void __launch_bounds__(WAVES * 64) skinny_kernel(
           const int Nh = N / 2;
           y[(int64_t)m * Nh + p] = (bf16)(gated_f(g, u, act, eps) + (add ? (float)add[(int64_t)m * Nh + p] : 0.f));
         } else {
+          if (act >= DS_ACT_UNARY) {
+            o0 = act_f(o0, act - DS_ACT_UNARY);
+            o1 = act_f(o1, act - DS_ACT_UNARY);
+          }
           if (add) o0 += (float)add[(int64_t)m * N + n0];
           y[(int64_t)m * N + n0] = (bf16)o0;
           if (n1 != n0) {

@@ -166,6 +166,7 @@ __global__ void __launch_bounds__(NW * 64) skinny_mfma_kernel(
       o = gated_f(g, u, act, eps);
     } else {
       o = v[0] + (bias ? (float)bias[n] : 0.f);
+      if (act >= DS_ACT_UNARY) o = act_f(o, act - DS_ACT_UNARY);
     }
     if (add) o += (float)add[(int64_t)m * Nout + n];
     y[(int64_t)m * Nout + n] = (bf16)o;

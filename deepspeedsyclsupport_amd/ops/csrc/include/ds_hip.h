@@ -79,6 +79,8 @@ template <typename T> __device__ __forceinline__ T from_f32(float x) { return (T
 // g sigmoid(alpha g) (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit). As the epilogue of a gated
 // decode product it is activation code DS_ACT_CLAMPED_GLU with alpha 1.702 and shift 1.
 #define DS_ACT_CLAMPED_GLU 5
+// activation codes from here on: code - DS_ACT_UNARY applied to the result of an ungated decode product
+#define DS_ACT_UNARY 16
 __device__ __forceinline__ float clamped_glu_f(float g, float u, float limit, float alpha = 1.702f, float shift = 1.f) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);

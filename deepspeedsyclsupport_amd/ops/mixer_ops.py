@@ -62,17 +62,22 @@ def latent_attention(q, lat, ukv, ukt, freq, sink, meta, scale, d, e):
     short = meta.cu_host[meta.n_short] if tiled else T
     o = q.new_empty(T, H, e)
     if short:
-        ql = ops.head_linear(q[:short], ukt, freq, meta.pos_ids[:short])
+        ql = ops.head_linear(q[:short], ukt, freq, meta.pos_ids[:short])  # [short, H, R + rot]
         if tiled:
-            ol = ops.latent_decode(ql, lat, meta.block_tables, meta.cu_q, meta.start_pos, meta.n_short, meta.n_decode,
-                                   meta.max_len, R, scale, sink)
+            ol = q.new_empty(short, H, R)
+            for a, b in ((0, meta.n_decode), (meta.n_decode, meta.n_short)):  # decodes; short portions
+                if a < b:
+                    cu = meta.cu_host
+                    ops.latent_decode(ql, lat, meta.block_tables, meta.cu_q, meta.start_pos, a, b - a,
+                                      max(cu[i + 1] - cu[i] for i in range(a, b)), cu[a], cu[b], meta.max_len, R, scale, sink,
+                                      ol)
         else:
             ol = ops.latent_generic(ql, lat, meta.block_tables, meta.pos_ids, meta.seq_ids, R, scale, sink)
         ops.head_linear(ol, ukv[H * d:].view(H, e, R), out=o[:short])
     if short < T:
         ctx = ops.latent_gather(lat, meta.block_tables, meta.kv_offs, meta.n_short, meta.kv_total)
         kv = F.linear(ctx[:, :R], ukv)
-        ops.rotate_tail(q[short:], freq, meta.pos_ids[short:])
+        ops.rotate_tail(q[short:], freq, meta.pos_ids[short:], q.shape[2] - d)
         ops.latent_prefill(q, kv, ctx, meta.start_pos, meta.cu_q, meta.work[meta.n_short - meta.n_decode:], meta.kv_offs,
                            meta.n_short, d, e, scale, sink, o)
     return o

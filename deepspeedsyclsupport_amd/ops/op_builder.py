@@ -58,8 +58,34 @@ EXTENSIONS = {
         "bindings": ["bind/ds_hip_ops.cpp", "bind/infer_bind.cpp", "bind/moe_bind.cpp", "bind/host_mem.cpp",
                      "bind/comm_bind.cpp", "bind/attn_small_bind.cpp"],
     },
-    # what serving a hybrid decoder (inference/model_implementations/hybrid.py) needs, and nothing else: in a fresh
-    # checkout such a model starts after compiling these sources only
+    # what serving the hybrid decoders (inference/model_implementations/hybrid.py) needs, and nothing else: in a fresh
+    # checkout such a model starts after compiling the decode products and its own mixers' sources only
+    "ds_gemv_ops": {
+        "kind": "hip",
+        "kernels": [
+            "gemv/skinny_gemm.hip",
+            "gemv/skinny_mfma.hip",
+            "gemv/skinny_bf16_sh.hip",
+            "gemv/skinny_finalize.hip",
+        ],
+        "bindings": ["bind/gemv_bind.cpp"],
+    },
+    # norms on sublayer outputs, latent attention, recurrences with a scalar decay per head
+    "ds_mixer_ops": {
+        "kind": "hip",
+        "kernels": [
+            "norm/post_norm.hip",
+            "act/token_gate.hip",
+            "attn/latent_ops.hip",
+            "attn/latent_decode.hip",
+            "attn/latent_prefill.hip",
+            "attn/paged_generic.hip",
+            "recur/decayed_scan.hip",
+            "recur/decayed_chunk.hip",
+        ],
+        "bindings": ["bind/mixer_bind.cpp"],
+    },
+    # residual streams, attention with head norms, gated delta rule
     "ds_hybrid_ops": {
         "kind": "hip",
         "kernels": [
@@ -71,10 +97,6 @@ EXTENSIONS = {
             "attn/decode_attn.hip",
             "recur/delta_rule.hip",
             "recur/delta_chunk.hip",
-            "gemv/skinny_gemm.hip",
-            "gemv/skinny_mfma.hip",
-            "gemv/skinny_bf16_sh.hip",
-            "gemv/skinny_finalize.hip",
         ],
         "bindings": ["bind/hybrid_bind.cpp"],
     },
