@@ -41,10 +41,11 @@ def parse():
                     help="Ulysses sequence-parallel degree (BASELINE config: Llama-2 7B, seq 32k, sp over xGMI "
                          "all-to-all); dp = world / sp")
     ap.add_argument("--workload", default="train", choices=["train", "hybrid"],
-                    help="train: the flagship training step (default); hybrid: serving throughput of a hybrid decoder "
+                    help="train: the flagship training step (default); hybrid: serving throughput of hybrid decoders "
                          "beside the uniform one (benchmarks/hybrid_serving.py)")
     ap.add_argument("--sizes", default="2048,4096", help="--workload hybrid: model widths")
-    ap.add_argument("--model-kind", default="both", choices=["hybrid", "uniform", "both"], help="--workload hybrid")
+    ap.add_argument("--model-kind", default="both", choices=["hybrid", "perelorn", "uniform", "both", "all"],
+                    help="--workload hybrid")
     ap.add_argument("--local_rank", type=int, default=0)
     ap.add_argument("--host-dryrun", action="store_true",
                     help="CPU/gloo rehearsal of the multi-rank control flow (tiny model; not a measurement)")

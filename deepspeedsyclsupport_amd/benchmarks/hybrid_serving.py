@@ -1,21 +1,30 @@
-"""Serving throughput of a hybrid decoder (Vopepel layers: gated delta rule, chunked attention, residual streams) beside
-the uniform Llama-style decoder at equal width, feed-forward, head and layer counts, both through the ragged engine with
-random bf16 weights: whole-prompt prefill and batched decoding.
+"""Serving throughput of hybrid decoders beside the uniform Llama-style decoder at equal width, feed-forward, head and layer
+counts, all through the ragged engine with random bf16 weights: whole-prompt prefill and batched decoding.
 
-    python bench.py --workload hybrid [--sizes 2048,4096] [--model-kind hybrid|uniform|both]
+* hybrid: Vopepel layers (gated delta rule, chunked attention, residual streams)
+* perelorn: Perelorn layers (Mamba-2, latent attention, lightning attention, norms on sublayer outputs, token-side input)
+
+    python bench.py --workload hybrid [--sizes 2048,4096] [--model-kind hybrid|perelorn|uniform|both|all]
 """
 import json
+import math
 import time
 
 import torch
 
 SIZES = {2048: dict(ff=5632, heads=16, kv=8), 4096: dict(ff=14336, heads=32, kv=8)}
 PATTERN = ("delta", "attention", "attention", "delta", "attention", "attention", "delta", "attention")
-HEAD, CHUNK, STREAMS, VOCAB = 128, 2048, 4, 32000
+HEAD, CHUNK, STREAMS, VOCAB, SIDE = 128, 2048, 4, 32000, 256
+
+
+# Perelorn: the delta layers' places go to Mamba-2 and lightning, attention to latent attention; every layer keeps its
+# feed-forward, so that the projections are of one size
+PERELORN = ("mamba2", "latent_attention", "lightning", "mamba2", "latent_attention", "lightning", "mamba2", "latent_attention")
+KINDS = {"both": ("hybrid", "uniform"), "all": ("hybrid", "perelorn", "uniform")}
 
 
 def specs(width):
-    """(hybrid, uniform) model specs of one size."""
+    """{kind: model spec} of one size."""
     from ..inference.model_implementations.transformer import DSModelSpec
     s = SIZES[width]
     common = dict(vocab_size=VOCAB, hidden_size=width, num_layers=len(PATTERN), num_heads=s["heads"],
@@ -27,7 +36,15 @@ def specs(width):
     hybrid = DSModelSpec(arch="vopepel", norm="ln", norm_bias=False, pos="none", streams=STREAMS, residual_mult=0.7,
                          layer_specs=tuple({"type": t, "mixer": mixers[t], "mlp": mlp} for t in PATTERN), **common)
     uniform = DSModelSpec(arch="llama", norm="rms", pos="rope", max_positions=16384, **common)
-    return hybrid, uniform
+    h = s["heads"]
+    mixers = {"mamba2": {"heads": 2 * h, "groups": 1, "state": HEAD, "vdim": HEAD // 2, "conv": 4, "norm_groups": 1},
+              "lightning": {"heads": h, "dim": HEAD, "vdim": HEAD, "decay": [math.exp(-2**(-8 * (i + 1) / h)) for i in range(h)]},
+              "latent_attention": {"heads": h, "dim": HEAD, "rot_dim": 64, "vdim": HEAD, "kv_rank": 512, "q_rank": 1536,
+                                   "rot": {"base": 10000.0, "dims": 64}, "scale": (HEAD + 64)**-0.5}}
+    perelorn = DSModelSpec(arch="perelorn", norm="rms", pos="none", residual="post_norm", token_side=SIDE, logit_scale=1.0,
+                           layer_specs=tuple({"type": t, "mixer": mixers[t], "mlp": {"kind": "gelu", "ff": s["ff"]}}
+                                             for t in PERELORN), **common)
+    return {"hybrid": hybrid, "perelorn": perelorn, "uniform": uniform}
 
 
 def build(spec, device, blocks):
@@ -95,11 +112,11 @@ def run(sizes=(2048, 4096), kind="both", iters=10, prompts=((1, 8192), (4, 2048)
     rows = []
     for width in sizes:
         row = {"width": width, "layers": len(PATTERN), **SIZES[width]}
-        for name, spec in zip(("hybrid", "uniform"), specs(width)):
-            if kind in (name, "both"):
+        for name, spec in specs(width).items():
+            if name in KINDS.get(kind, (kind, )):
                 row[name] = measure(spec, device, prompts, batches, context, iters, log)
                 torch.cuda.empty_cache()
         rows.append(row)
-    print(json.dumps({"metric": "ragged-engine serving throughput, hybrid decoder beside the uniform one", "unit": "tokens/s",
+    print(json.dumps({"metric": "ragged-engine serving throughput, hybrid decoders beside the uniform one", "unit": "tokens/s",
                       "dtype": "bf16", "data": "synthetic tokens, random-init weights", "context": context,
                       "sizes": rows}), flush=True)

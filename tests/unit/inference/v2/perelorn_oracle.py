@@ -2,10 +2,29 @@
 mechanism, written straight from the model's equations in PyTorch on the CPU. It shares no code with the package.
 
 Weights come as a dict of tensors under the checkpoint's names; arithmetic runs in the dtype of `cast` (float64 by
-default). Nothing here is cached, paged, batched, absorbed, chunked or fused."""
+default). Nothing here is cached, paged, batched, absorbed, chunked or fused. Under `Rounded()` the operands and results of
+the projections are rounded to bf16: what a model in 16 bits cannot do better than."""
 import math
 
 import torch
+
+
+class Rounded:
+    """Context in which `project` works on bf16 operands and results."""
+    on = False
+
+    def __enter__(self):
+        Rounded.on = True
+
+    def __exit__(self, *exc):
+        Rounded.on = False
+
+
+def project(x, w):
+    """W x for every row."""
+    if not Rounded.on:
+        return x @ w.t()
+    return (x.bfloat16().to(w.dtype) @ w.t()).bfloat16().to(w.dtype)
 
 
 # ------------------------------------------------------------------------------------------------ mechanisms
@@ -91,7 +110,7 @@ def grouped_rms(x, parts, eps):
 def mamba2_mixer(w, p, mx, h, eps):
     n, H, e, N, G = h.shape[0], mx["heads"], mx["vdim"], mx["state"], mx["groups"]
     inner = H * e
-    z, x, B, C, dt = torch.split(h @ w[p + "in"].t(), [inner, inner, G * N, G * N, H], -1)
+    z, x, B, C, dt = torch.split(project(h, w[p + "in"]), [inner, inner, G * N, G * N, H], -1)
     xbc = silu(causal_conv(torch.cat([x, B, C], -1), w[p + "conv"], w[p + "conv.b"]))
     x, B, C = torch.split(xbc, [inner, G * N, G * N], -1)
     x, B, C = x.view(n, H, e), B.view(n, G, N), C.view(n, G, N)
@@ -103,33 +122,33 @@ def mamba2_mixer(w, p, mx, h, eps):
         o, _ = decayed_scan(C[:, g], B[:, g], x[:, i], decay[:, i], dt[:, i])
         y.append(o + w[p + "D"][i] * x[:, i])
     y = torch.stack(y, 1).reshape(n, inner) * silu(z)
-    return (grouped_rms(y, mx["norm_groups"], eps) * w[p + "norm"]) @ w[p + "o"].t()
+    return project(grouped_rms(y, mx["norm_groups"], eps) * w[p + "norm"], w[p + "o"])
 
 
 def lightning_mixer(w, p, mx, h, eps):
     n, H, d, e = h.shape[0], mx["heads"], mx["dim"], mx["vdim"]
-    q = silu(h @ w[p + "q"].t()).view(n, H, d)
-    k = silu(h @ w[p + "k"].t()).view(n, H, d)
-    v = silu(h @ w[p + "v"].t()).view(n, H, e)
+    q = silu(project(h, w[p + "q"])).view(n, H, d)
+    k = silu(project(h, w[p + "k"])).view(n, H, d)
+    v = silu(project(h, w[p + "v"])).view(n, H, e)
     one = torch.ones(n, dtype=h.dtype)
     o = torch.stack([decayed_scan(q[:, i], k[:, i], v[:, i], mx["decay"][i] * one, one)[0] for i in range(H)], 1)
-    o = rms_norm(o.reshape(n, H * e), w[p + "norm"], eps) * sigmoid(h @ w[p + "g"].t())
-    return o @ w[p + "o"].t()
+    o = rms_norm(o.reshape(n, H * e), w[p + "norm"], eps) * sigmoid(project(h, w[p + "g"]))
+    return project(o, w[p + "o"])
 
 
 def latent_mixer(w, p, mx, h, eps):
     n, H, d, r, e, R = h.shape[0], mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"], mx["kv_rank"]
-    q = (rms_norm(h @ w[p + "dq"].t(), w[p + "dq.norm"], eps) @ w[p + "uq"].t()).view(n, H, d + r)
-    down = h @ w[p + "dkv"].t()
+    q = project(rms_norm(project(h, w[p + "dq"]), w[p + "dq.norm"], eps), w[p + "uq"]).view(n, H, d + r)
+    down = project(h, w[p + "dkv"])
     c = rms_norm(down[:, :R], w[p + "dkv.norm"], eps)
     kr = rotate(down[:, R:], mx["rot"]["dims"], mx["rot"]["base"])
-    k, v = (c @ w[p + "uk"].t()).view(n, H, d), (c @ w[p + "uv"].t()).view(n, H, e)
+    k, v = project(c, w[p + "uk"]).view(n, H, d), project(c, w[p + "uv"]).view(n, H, e)
     out = []
     for i in range(H):
         qr = rotate(q[:, i, d:], mx["rot"]["dims"], mx["rot"]["base"])
         out.append(sink_attention(torch.cat([q[:, i, :d], qr], -1), torch.cat([k[:, i], kr], -1), v[:, i], mx["scale"],
                                   w[p + "sink"][i]))
-    return torch.stack(out, 1).reshape(n, H * e) @ w[p + "o"].t()
+    return project(torch.stack(out, 1).reshape(n, H * e), w[p + "o"])
 
 
 MIXERS = {"mamba2": mamba2_mixer, "lightning": lightning_mixer, "latent_attention": latent_mixer}
@@ -138,8 +157,8 @@ MIXERS = {"mamba2": mamba2_mixer, "lightning": lightning_mixer, "latent_attentio
 def token_side(w, p, dim, i, x, tokens, eps):
     """The layer's own embedding of each token, gated by the residual and added to it."""
     e = w["side.embed"][tokens][:, i * dim:(i + 1) * dim]
-    g = gelu_tanh(x @ w[p + "side.gate"].t()) * e
-    return rms_norm(g @ w[p + "side.proj"].t(), w[p + "side.norm"], eps)
+    g = gelu_tanh(project(x, w[p + "side.gate"])) * e
+    return rms_norm(project(g, w[p + "side.proj"]), w[p + "side.norm"], eps)
 
 
 def forward(cfg, weights, tokens, cast=torch.float64, trace=None):
@@ -151,12 +170,12 @@ def forward(cfg, weights, tokens, cast=torch.float64, trace=None):
         p = f"l{i}."
         x = x + rms_norm(MIXERS[layer["type"]](w, p + "mix.", layer["mixer"], x, eps), w[p + "norm1"], eps)
         if layer.get("mlp"):
-            y = gelu_erf(x @ w[p + "mlp.up"].t()) @ w[p + "mlp.down"].t()
+            y = project(gelu_erf(project(x, w[p + "mlp.up"])), w[p + "mlp.down"])
             x = x + rms_norm(y, w[p + "norm2"], eps)
         x = x + token_side(w, p, cfg["token_side"]["dim"], i, x, ids, eps)
         if trace is not None:
             trace.append(x)
-    return rms_norm(x, w["final.norm"], eps) @ w["head"].t() * cfg["logit_scale"]
+    return project(rms_norm(x, w["final.norm"], eps), w["head"]) * cfg["logit_scale"]
 
 
 # ------------------------------------------------------------------------------------------------ test models
