@@ -240,26 +240,35 @@ __global__ void __launch_bounds__(NT) latent_decode_kernel(LatArgs a) {
   }
 }
 
-// one workgroup per row
+// one workgroup per row; up to MAX_SPLITS ranges
+constexpr int MAX_SPLITS = 1024;
 __global__ void __launch_bounds__(128) latent_combine_kernel(const float* __restrict__ acc, const float* __restrict__ ml,
                                                              const float* __restrict__ sink, bf16* __restrict__ out,
                                                              int64_t rows, int H, int R, int splits) {
+  __shared__ float wt[MAX_SPLITS];
+  __shared__ float red[2];
   const int64_t r = blockIdx.x;
-  float M = -INFINITY;
-  for (int s = 0; s < splits; ++s) M = fmaxf(M, ml[(s * rows + r) * 2]);
-  float den = 0.f;
-  if (sink) {
-    const float sk = sink[r % H] * LOG2E;
-    M = fmaxf(M, sk);
-    den = exp2f(sk - M);
+  const float sk = sink ? sink[r % H] * LOG2E : -INFINITY;
+  float M = sk, den = 0.f;
+  for (int s = threadIdx.x; s < splits; s += 128) {
+    wt[s] = ml[(s * rows + r) * 2];
+    M = fmaxf(M, wt[s]);
   }
-  for (int s = 0; s < splits; ++s) den = fmaf(exp2f(ml[(s * rows + r) * 2] - M), ml[(s * rows + r) * 2 + 1], den);
+  M = block_max(M, red);
+  for (int s = threadIdx.x; s < splits; s += 128) {
+    wt[s] = exp2f(wt[s] - M);  // 0 for ranges that had nothing to add, and wrote nothing
+    den = fmaf(wt[s], ml[(s * rows + r) * 2 + 1], den);
+  }
+  den = block_sum(den, red) + exp2f(sk - M);  // (its barriers publish the weights)
   for (int c = threadIdx.x * 4; c < R; c += 512) {
+    const float* a = acc + r * R + c;
     f32x4 v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
     for (int s = 0; s < splits; ++s) {
-      const float m = ml[(s * rows + r) * 2];
-      if (m == -INFINITY) continue;  // that range had nothing to add, and wrote nothing
-      v += *reinterpret_cast<const f32x4*>(acc + (s * rows + r) * R + c) * exp2f(m - M);
+      const f32x4 x = *reinterpret_cast<const f32x4*>(a + s * rows * R);
+      const float w = wt[s];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = w > 0.f ? fmaf(x[j], w, v[j]) : v[j];
     }
     bf16x4 o;
 #pragma unroll
@@ -302,7 +311,9 @@ extern "C" int ds_latent_decode_ok(int R, int r) {
 extern "C" void ds_latent_decode_plan(int nseq, int max_new, int H, int W, int max_len, int* range, int* splits) {
   const int rows = max_new * H, per = 16 * row_tiles(rows, W), blocks = (rows + per - 1) / per;
   const int tiles = (max_len + BN - 1) / BN;
-  int want = (512 + nseq * blocks - 1) / (nseq * blocks);
+  // as many workgroups as the chip's LDS holds at once: a second, partly filled round would cost as much as the first
+  const int resident = 256 * (int)(LDS_MAX / lds_bytes(row_tiles(rows, W), W));
+  int want = (resident < 1024 ? resident : 1024) / (nseq * blocks);
   if (want > tiles) want = tiles;
   if (want < 1) want = 1;
   const int per_range = (tiles + want - 1) / want;
@@ -317,7 +328,7 @@ extern "C" int ds_latent_decode(const void* q, const void* lat, void* out, float
                                 int r, int BS, int range, int splits, const float* sink, float scale, hipStream_t st) {
   if (nseq <= 0) return 0;
   if (!ds_latent_decode_ok(R, r) || H <= 0 || BS <= 0 || max_blocks <= 0 || range <= 0 || range % BN || splits <= 0 ||
-      splits > 65535 || max_new <= 0 || tokens <= 0 || (splits > 1 && (!acc || !ml)))
+      splits > MAX_SPLITS || max_new <= 0 || tokens <= 0 || (splits > 1 && (!acc || !ml)))
     return (int)hipErrorInvalidValue;
   const LatArgs a{(const bf16*)q, (const bf16*)lat, (bf16*)out, acc, ml, bt, cu, start, sink, first, tok_base, H, R, r, BS,
                   max_blocks, range, splits, (int64_t)tokens * H, scale * LOG2E};

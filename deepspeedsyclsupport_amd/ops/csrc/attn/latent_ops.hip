@@ -68,25 +68,27 @@ __global__ void __launch_bounds__(256) latent_prepare_kernel(
   for (int i = 2 * half + lane; i < r; i += 64) dst[R + i] = src[R + i];
 }
 
-// The columns behind the map's, one token's heads per workgroup
+// Item j of the columns behind the map's: pair (j, half + j) turned, or a single column carried over
+template <typename T>
+__device__ __forceinline__ void rotate_one(const T* s, T* d, int j, int half, int p, const double* freq) {
+  if (j < half) {
+    float co, si;
+    turn_of(p, freq[j], co, si);
+    const float u = (float)s[j], v = (float)s[half + j];
+    d[j] = (T)(u * co - v * si);
+    d[half + j] = (T)(v * co + u * si);
+  } else {
+    d[half + j] = s[half + j];
+  }
+}
+
+// ... of all heads of a token, by a workgroup
 template <typename T>
 __device__ __forceinline__ void rotate_heads(const T* src, int64_t sh, T* dst, int64_t dh, int H, int r, int half, int p,
                                              const double* freq) {
-  const int rest = r - 2 * half, per = half + rest;
-  for (int i = threadIdx.x; i < H * per; i += blockDim.x) {
-    const int h = i / per, j = i % per;
-    const T* s = src + h * sh;
-    T* d = dst + h * dh;
-    if (j < half) {
-      float co, si;
-      turn_of(p, freq[j], co, si);
-      const float u = (float)s[j], v = (float)s[half + j];
-      d[j] = (T)(u * co - v * si);
-      d[half + j] = (T)(v * co + u * si);
-    } else {
-      d[half + j] = s[half + j];
-    }
-  }
+  const int per = r - half;
+  for (int i = threadIdx.x; i < H * per; i += blockDim.x)
+    rotate_one(src + i / per * sh, dst + i / per * dh, i % per, half, p, freq);
 }
 
 template <typename T>
@@ -127,9 +129,12 @@ __global__ void __launch_bounds__(256) head_linear_mfma_kernel(HeadArgs a) {
   const int h = blockIdx.y, lane = threadIdx.x & 63, wid = threadIdx.x >> 6, l16 = lane & 15, q4 = lane >> 4;
   const int t0 = blockIdx.z * 16 * TT, ntiles = (a.N + 63) / 64;
   if ((int)blockIdx.x >= ntiles) {
-    for (int t = t0; t < min(t0 + 16 * TT, a.T); ++t)
-      rotate_heads((const bf16*)a.x + ((int64_t)t * a.H + h) * a.xrow + a.K, 0,
-                   (bf16*)a.y + ((int64_t)t * a.H + h) * a.yrow + a.N, 0, 1, a.r, a.half, a.pos[t], a.freq);
+    const int per = a.r - a.half, nt = min(16 * TT, a.T - t0);  // pairs and single columns of a token
+    for (int i = threadIdx.x; i < nt * per; i += 256) {
+      const int t = t0 + i / per;
+      rotate_one((const bf16*)a.x + ((int64_t)t * a.H + h) * a.xrow + a.K, (bf16*)a.y + ((int64_t)t * a.H + h) * a.yrow + a.N,
+                 i % per, a.half, a.pos[t], a.freq);
+    }
     return;
   }
   const int n0 = blockIdx.x * 64 + wid * 16;

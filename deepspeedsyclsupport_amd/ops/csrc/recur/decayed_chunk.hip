@@ -4,10 +4,10 @@
 // With the running log decay G_i of a chunk (its first token included) and the state S0 the chunk starts from:
 //     o_i = e^{G_i} S0^T q_i + sum_{j <= i} P_ij v_j + D v_i,    P_ij = e^{G_i - G_j} b_j (q_i . k_j)
 //     S   = e^{G_C} S0 + sum_j e^{G_C - G_j} b_j k_j v_j^T
-// One workgroup per (sequence, head, 64 value columns) walks the chunks. Each of its four waves owns 16 value columns and
-// keeps their state [dk, 16] in registers, in the result layout of the matrix instructions: the next state accumulates
-// into it, and the same registers are the left operand of the read-out (a product's k order is free as long as both sides
-// agree on it). The 64 x 64 weights P are computed once per workgroup and shared through LDS.
+// One workgroup per (sequence, head, 16 WC value columns) walks the chunks. Two of its 2 WC waves share 16 value columns: each
+// keeps half of the key rows of their state in registers, in the result layout of the matrix instructions. The next state
+// accumulates into it, and the same registers are the left operand of the read-out (a product's k order is free as long as
+// both sides agree on it). The two halves of the read-out meet in LDS, where the 64 x 64 weights P are shared too.
 //
 // Precision: q, k and v are bf16 activations; everything else is fp32. The bf16 matrix instructions take an fp32 operand
 // as three bf16 terms (8 + 8 + 8 mantissa bits, nothing is lost) with fp32 accumulation, so state, weights and decays
@@ -19,12 +19,11 @@
 namespace {
 
 constexpr int C = 64;
-constexpr int NT = 256;
-constexpr int VT = 64;       // value columns per workgroup
-constexpr int VP = VT + 8;   // LDS row lengths (elements)
-constexpr int PP = C + 8;
+constexpr int PP = C + 8;  // LDS row length (elements) of the weights
+constexpr double LOG2E = 1.4426950408889634073599246810019;
 
 typedef short s16x4_t __attribute__((ext_vector_type(4)));
+typedef unsigned u32x4_t __attribute__((ext_vector_type(4)));
 
 __device__ __forceinline__ f32x4 mfma(bf16x8 a, bf16x8 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
@@ -32,12 +31,40 @@ __device__ __forceinline__ f32x4 mfma(bf16x8 a, bf16x8 b, f32x4 c) {
 // Workgroup barrier for LDS: earlier LDS accesses have completed, global loads may still be under way
 __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
-// x as three bf16 terms
-__device__ __forceinline__ void split3(float x, bf16& a, bf16& b, bf16& c) {
-  a = (bf16)x;
-  const float r = x - (float)a;
-  b = (bf16)r;
-  c = (bf16)(r - (float)b);
+// Upper halves of two words side by side: two fp32 numbers cut to bf16
+__device__ __forceinline__ unsigned pack_hi(unsigned lo, unsigned hi) { return __builtin_amdgcn_perm(hi, lo, 0x07060302u); }
+
+// Pairs of fp32 numbers as the sums of three bf16 numbers each: the leading 8 mantissa bits, the next 8, the rest (exact)
+__device__ __forceinline__ void split3(float x, float y, unsigned& a, unsigned& b, unsigned& c) {
+  const unsigned xi = __float_as_uint(x), yi = __float_as_uint(y);
+  const float xr = x - __uint_as_float(xi & 0xffff0000u), yr = y - __uint_as_float(yi & 0xffff0000u);
+  const unsigned xj = __float_as_uint(xr), yj = __float_as_uint(yr);
+  a = pack_hi(xi, yi);
+  b = pack_hi(xj, yj);
+  c = pack_hi(__float_as_uint(xr - __uint_as_float(xj & 0xffff0000u)), __float_as_uint(yr - __uint_as_float(yj & 0xffff0000u)));
+}
+// The same for the 8 elements of an operand
+__device__ __forceinline__ void split3(const float (&x)[8], bf16x8& a, bf16x8& b, bf16x8& c) {
+  u32x4_t u, v, w;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    unsigned p, q, r;
+    split3(x[2 * i], x[2 * i + 1], p, q, r);
+    u[i] = p;
+    v[i] = q;
+    w[i] = r;
+  }
+  a = __builtin_bit_cast(bf16x8, u);
+  b = __builtin_bit_cast(bf16x8, v);
+  c = __builtin_bit_cast(bf16x8, w);
+}
+
+// by value: a choice between array elements must not become one between addresses
+__device__ __forceinline__ f32x4 pick(bool c, f32x4 a, f32x4 b) {
+  f32x4 r;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) r[i] = c ? a[i] : b[i];
+  return r;
 }
 
 // Operand whose lane wants one column of 8 rows: rows r .. r + 3 and r2 .. r2 + 3 of 16 columns from `col` on, transposed
@@ -57,237 +84,267 @@ __device__ __forceinline__ bf16x8 read_tr(const bf16* base, int pitch, int r, in
   return __builtin_bit_cast(bf16x8, v);
 }
 
-// NK: 32-wide steps of the key width (rounded up)
-template <int NK>
-__global__ void __launch_bounds__(NT, (NK <= 4 ? 2 : 1)) decayed_chunk_kernel(
+// NK: 32-wide steps of the key width (rounded up), even unless the waves of a pair cannot share (NK 1: the second one has
+// no rows); WC: groups of 16 value columns
+template <int NK, int WC>
+__global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decayed_chunk_kernel(
     const bf16* __restrict__ qk, const bf16* __restrict__ v, const float* __restrict__ gb,
     const float* __restrict__ log_decay, const float* __restrict__ skip, const bf16* __restrict__ proj,
     float* __restrict__ state, bf16* __restrict__ conv_state, const int* __restrict__ seqs, const int* __restrict__ cu,
     const int* __restrict__ start, const int* __restrict__ slots, bf16* __restrict__ out, ScanDims D) {
-  constexpr int KP = 32 * NK + 8;  // LDS row length of q and k
+  constexpr int NT = 128 * WC, NW = 2 * WC, VT = 16 * WC;
+  constexpr int KP = 32 * NK + 8, VP = VT + 8;      // LDS row lengths of q and k, of v
+  constexpr int KH = (NK + 1) / 2;                  // steps of a wave's half of the key rows
+  constexpr int PQ = C * 4 * NK / NT, PV = (C * VT / 8 + NT - 1) / NT;  // 16-byte pieces per thread of q or k, of v
+  static_assert(C * 4 * NK % NT == 0 || NK == 1, "pieces");
+  constexpr int PQN = PQ > 0 ? PQ : 1;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   bf16* const Qs = reinterpret_cast<bf16*>(smem);
   bf16* const Ks = Qs + C * KP;
   bf16* const Vs = Ks + C * KP;
   bf16* const Ps = Vs + C * VP;                                   // [3][C][PP]
-  double* const Gs = reinterpret_cast<double*>(Ps + 3 * C * PP);  // [2][C]
-  float* const bs = reinterpret_cast<float*>(Gs + 2 * C);         // [2][C] step sizes
-  float* const eg = bs + 2 * C;                                   // [2][C] e^{G_i}
-  float* const ws = eg + 2 * C;                                   // [2][C] e^{G_C - G_j} b_j
+  f32x4* const Ys = reinterpret_cast<f32x4*>(Ps + 3 * C * PP);    // [NW][2][64]: halves of the read-out on their way
+  double* const Gs = reinterpret_cast<double*>(Ys + NW * 2 * 64); // [2 NW][C] running log2 decay
+  float* const bs = reinterpret_cast<float*>(Gs + 2 * NW * C);    // [2 NW][C] step sizes
+  float* const eg = bs + 2 * NW * C;                              // [2 NW][C] e^{G_i}
+  float* const ws = eg + 2 * NW * C;                              // [2 NW][C] e^{G_C - G_j} b_j
 
   const int vts = (D.dv + VT - 1) / VT, bid = xcd_remap(blockIdx.x, gridDim.x);
   const int vt = bid % vts, h = bid / vts % D.H, seq = seqs[2 * (bid / (vts * D.H))];
-  const int g = h / (D.H / D.Hk), tid = threadIdx.x, lane = tid & 63, w = tid >> 6, l16 = lane & 15, q4 = lane >> 4;
+  const int g = h / (D.H / D.Hk), tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, q4 = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6), wc = w >> 1, half = w & 1;
   const int t0 = cu[seq], n = cu[seq + 1] - t0, nc = (n + C - 1) / C, v0 = vt * VT, dks = D.dks(), dvs = D.dvs();
   const bool fresh = start[seq] == 0;
-  const int col = v0 + 16 * w + l16;  // this lane's column of the state
+  const int col = v0 + 16 * wc + l16;  // this lane's column of the state
+  const int k_first = half * KH * 32;  // first key row of the wave's half (NK 1: rows 32 .. 63 do not exist)
+  const bool rows_ok = half * KH < NK;
   float* st = state + (((int64_t)slots[seq] * D.H + h) * D.dv + min(col, D.dv - 1)) * dks;
 
-  f32x4 S[2 * NK];  // rows 16 t + 4 q4 + 0..3
+  f32x4 S[2 * KH];  // rows k_first + 16 t + 4 q4 + 0..3
 #pragma unroll
-  for (int t = 0; t < 2 * NK; ++t) {
-    const int k = 16 * t + 4 * q4;
+  for (int t = 0; t < 2 * KH; ++t) {
+    const int k = k_first + 16 * t + 4 * q4;
     S[t] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (!fresh && col < D.dv && k < dks) S[t] = *reinterpret_cast<const f32x4*>(st + k);
   }
   const float sk = skip ? skip[h] : 0.f, ld = log_decay ? log_decay[h] : 0.f;
   const bf16* qbase = qk + D.q_at(g, t0);
   const bf16* kbase = qk + D.k_at(g, t0);
-  const bf16* vbase = v + D.v_at(h, t0);
+  const bf16* vbase = v + D.v_at(h, t0) + v0;
+  const int vw = min(dvs - v0, VT);    // v columns of this workgroup that exist
+  const bool k_full = dks == 32 * NK, v_full = vw == VT;
 
-  // ---- a chunk's rows on their way to LDS: 4 NK (q, k) and 8 (v) 16-byte pieces per row
-  bf16x8 rq[NK], rk[NK], rv[2];
+  // ---- a chunk's rows on their way to LDS: 4 NK (q, k) and VT / 8 (v) 16-byte pieces per row
+  bf16x8 rq[PQN], rk[PQN], rv[PV];
   auto fetch = [&](int c) {
+    const bool whole = (c + 1) * C <= n;
+    const int64_t base = (int64_t)c * C * dks, vb = (int64_t)c * C * dvs;
+    const int last = n - 1 - c * C;
 #pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int p = tid + i * NT, row = p / (4 * NK), ch = p % (4 * NK) * 8;
-      const int64_t off = (int64_t)min(c * C + row, n - 1) * dks + min(ch, dks - 8);
-      rq[i] = *reinterpret_cast<const bf16x8*>(qbase + off);
-      rk[i] = *reinterpret_cast<const bf16x8*>(kbase + off);
+    for (int i = 0; i < PQN; ++i) {
+      const int p = tid + i * NT;
+      int row = p / (4 * NK), ch = p % (4 * NK) * 8;
+      if (!whole) row = min(row, last);
+      if (!k_full) ch = min(ch, dks - 8);
+      if (PQ > 0 || p < C * 4 * NK) {
+        rq[i] = *reinterpret_cast<const bf16x8*>(qbase + base + row * dks + ch);
+        rk[i] = *reinterpret_cast<const bf16x8*>(kbase + base + row * dks + ch);
+      }
     }
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const int p = tid + i * NT, row = p / 8, ch = v0 + p % 8 * 8;
-      rv[i] = *reinterpret_cast<const bf16x8*>(vbase + (int64_t)min(c * C + row, n - 1) * dvs + min(ch, dvs - 8));
+    for (int i = 0; i < PV; ++i) {
+      const int p = tid + i * NT;
+      int row = p / (VT / 8), ch = p % (VT / 8) * 8;
+      if (!whole) row = min(row, last);
+      if (!v_full) ch = min(ch, vw - 8);
+      if (p < C * VT / 8) rv[i] = *reinterpret_cast<const bf16x8*>(vbase + vb + row * dvs + ch);
     }
   };
   auto stage = [&](int c) {  // rows past the portion's end and columns past the widths become zero
+    const bool whole = (c + 1) * C <= n;
     bf16x8 z;
 #pragma unroll
     for (int e = 0; e < 8; ++e) z[e] = (bf16)0.f;
+    if (!whole || !k_full || !v_full) {
 #pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int p = tid + i * NT, row = p / (4 * NK), ch = p % (4 * NK) * 8;
-      const bool ok = c * C + row < n && ch < dks;
-      *reinterpret_cast<bf16x8*>(Qs + row * KP + ch) = ok ? rq[i] : z;
-      *reinterpret_cast<bf16x8*>(Ks + row * KP + ch) = ok ? rk[i] : z;
+      for (int i = 0; i < PQN; ++i) {
+        const int p = tid + i * NT;
+        if (c * C + p / (4 * NK) >= n || p % (4 * NK) * 8 >= dks) rq[i] = rk[i] = z;
+      }
+#pragma unroll
+      for (int i = 0; i < PV; ++i) {
+        const int p = tid + i * NT;
+        if (c * C + p / (VT / 8) >= n || p % (VT / 8) * 8 >= vw) rv[i] = z;
+      }
     }
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const int p = tid + i * NT, row = p / 8, ch = p % 8 * 8;
-      *reinterpret_cast<bf16x8*>(Vs + row * VP + ch) = c * C + row < n && v0 + ch < dvs ? rv[i] : z;
+    for (int i = 0; i < PQN; ++i) {
+      const int p = tid + i * NT, row = p / (4 * NK), ch = p % (4 * NK) * 8;
+      if (PQ > 0 || p < C * 4 * NK) {
+        *reinterpret_cast<bf16x8*>(Qs + row * KP + ch) = rq[i];
+        *reinterpret_cast<bf16x8*>(Ks + row * KP + ch) = rk[i];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < PV; ++i) {
+      const int p = tid + i * NT;
+      if (p < C * VT / 8) *reinterpret_cast<bf16x8*>(Vs + p / (VT / 8) * VP + p % (VT / 8) * 8) = rv[i];
     }
   };
-  // ---- a chunk's decays and step sizes, a lane per token (one wave does it)
+  // ---- decays and step sizes of a chunk, a lane per token: every NW chunks each wave prepares one of the next NW
   float lg = 0.f, lb = 0.f;
   auto fetch_gb = [&](int c) {
-    const int i = c * C + lane;
-    const int64_t t = t0 + min(i, n - 1);
+    const int64_t t = t0 + min(c * C + lane, n - 1);
     lg = gb ? gb[t * 2 * D.H + h] : ld;
     lb = gb ? gb[(t * 2 + 1) * D.H + h] : 1.f;
-    if (i >= n) lg = lb = 0.f;  // rows past the end neither decay nor add anything
   };
   auto scan_gb = [&](int c) {
-    double G = (double)lg;
+    const bool ok = c * C + lane < n;  // rows past the end neither decay nor add anything
+    const float b0 = ok ? lb : 0.f;
+    double G = ok ? (double)lg * LOG2E : 0.0;
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
       const double p = __shfl_up(G, o, 64);
       if (lane >= o) G += p;
     }
     const double GC = __shfl(G, 63, 64);
-    const int b = (c & 1) * C + lane;
+    const int b = c % (2 * NW) * C + lane;
     Gs[b] = G;
-    bs[b] = lb;
-    eg[b] = expf((float)G);
-    ws[b] = expf((float)(GC - G)) * lb;
+    bs[b] = b0;
+    eg[b] = __builtin_amdgcn_exp2f((float)G);
+    ws[b] = __builtin_amdgcn_exp2f((float)(GC - G)) * b0;
   };
   fetch(0);
-  if (w == 0) {
-    fetch_gb(0);
-    scan_gb(0);
-  }
+  fetch_gb(w);
+  scan_gb(w);
   for (int c = 0; c < nc; ++c) {
-    const int cb = (c & 1) * C;
+    const int cb = c % (2 * NW) * C;
+    const bool ahead = c % NW == 0 && c + NW < nc;
     stage(c);
-    if (c + 1 < nc) {
-      fetch(c + 1);
-      if (w == (c & 3)) fetch_gb(c + 1);
-    }
+    if (c + 1 < nc) fetch(c + 1);
+    if (ahead) fetch_gb(c + NW + w);
     lds_barrier();
-    // ---- P, row tile w
-    {
-      bf16x8 qa[NK];
+    // ---- P. The read-out takes pairs of 16 x 16 tiles of a row: 10 tiles up to the diagonal, and 2 behind it that are zero
 #pragma unroll
-      for (int kk = 0; kk < NK; ++kk) qa[kk] = *reinterpret_cast<const bf16x8*>(Qs + (16 * w + l16) * KP + 32 * kk + 8 * q4);
-      double gi[4];
+    for (int u = 0; u < (12 + NW - 1) / NW; ++u) {
+      const int tl = w + u * NW;
+      if (tl >= 12) break;
+      const int it = tl < 4 ? tl >> 1 : 2 + ((tl - 4) >> 2), jt = tl < 4 ? tl & 1 : (tl - 4) & 3;
+      f32x4 s = {0.f, 0.f, 0.f, 0.f};
+      if (jt <= it) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) gi[r] = Gs[cb + 16 * w + 4 * q4 + r];
+        for (int kk = 0; kk < NK; ++kk)
+          s = mfma(*reinterpret_cast<const bf16x8*>(Ks + (16 * jt + l16) * KP + 32 * kk + 8 * q4),
+                   *reinterpret_cast<const bf16x8*>(Qs + (16 * it + l16) * KP + 32 * kk + 8 * q4), s);
+        // lane: row i of P, columns j .. j + 3
+        const int i = 16 * it + l16, j = 16 * jt + 4 * q4;
+        const double gi = Gs[cb + i];
 #pragma unroll
-      for (int jt = 0; jt < 4; ++jt) {
-        if (jt > (w | 1)) break;  // read-out takes pairs of tiles: above the diagonal only the pair's second one is read
-        f32x4 s = {0.f, 0.f, 0.f, 0.f};
-        if (jt <= w) {
-#pragma unroll
-          for (int kk = 0; kk < NK; ++kk)
-            s = mfma(qa[kk], *reinterpret_cast<const bf16x8*>(Ks + (16 * jt + l16) * KP + 32 * kk + 8 * q4), s);
-        }
-        const int j = 16 * jt + l16;
-        const double gj = Gs[cb + j];
-        const float bj = bs[cb + j];
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int i = 16 * w + 4 * q4 + r;
-          const float x = j <= i ? s[r] * expf((float)(gi[r] - gj)) * bj : 0.f;
-          bf16 a, b, d;
-          split3(x, a, b, d);
-          Ps[i * PP + j] = a;
-          Ps[(C + i) * PP + j] = b;
-          Ps[(2 * C + i) * PP + j] = d;
+        for (int r = 0; r < 4; ++r)
+        {  // (no branch: behind the diagonal the factor is some number, or infinite)
+          const float f = s[r] * (__builtin_amdgcn_exp2f((float)(gi - Gs[cb + j + r])) * bs[cb + j + r]);
+          s[r] = j + r <= i ? f : 0.f;
         }
       }
+      unsigned a[2], b[2], d[2];
+      split3(s[0], s[1], a[0], b[0], d[0]);
+      split3(s[2], s[3], a[1], b[1], d[1]);
+      bf16* p = Ps + (16 * it + l16) * PP + 16 * jt + 4 * q4;
+      *reinterpret_cast<uint2*>(p) = uint2{a[0], a[1]};
+      *reinterpret_cast<uint2*>(p + C * PP) = uint2{b[0], b[1]};
+      *reinterpret_cast<uint2*>(p + 2 * C * PP) = uint2{d[0], d[1]};
     }
-    // ---- read-out of the state the chunk starts from: y^T [16 columns, 64 tokens] = S^T q^T
+    // ---- read-out of the state the chunk starts from, this half of the key rows: y^T [16 columns, 64 tokens] = S^T q^T
     f32x4 y[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) y[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (rows_ok) {
 #pragma unroll
-    for (int kk = 0; kk < NK; ++kk) {
-      bf16x8 s0, s1, s2;  // k slot 8 q4 + e is key row 32 kk + 16 (e / 4) + 4 q4 + e % 4
+      for (int kk = 0; kk < KH; ++kk) {
+        bf16x8 s0, s1, s2;  // k slot 8 q4 + e is key row k_first + 32 kk + 16 (e / 4) + 4 q4 + e % 4
+        float x[8];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        bf16 a, b, d;
-        split3(S[2 * kk + (e >> 2)][e & 3], a, b, d);
-        s0[e] = a;
-        s1[e] = b;
-        s2[e] = d;
-      }
+        for (int e = 0; e < 8; ++e) x[e] = S[2 * kk + (e >> 2)][e & 3];
+        split3(x, s0, s1, s2);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const bf16* qr = Qs + (16 * i + l16) * KP + 32 * kk + 4 * q4;
-        const bf16x4 lo = *reinterpret_cast<const bf16x4*>(qr), hi = *reinterpret_cast<const bf16x4*>(qr + 16);
-        bf16x8 qb;
+        for (int i = 0; i < 4; ++i) {
+          const bf16* qr = Qs + (16 * i + l16) * KP + k_first + 32 * kk + 4 * q4;
+          const bf16x4 lo = *reinterpret_cast<const bf16x4*>(qr), hi = *reinterpret_cast<const bf16x4*>(qr + 16);
+          bf16x8 qb;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          qb[e] = lo[e];
-          qb[4 + e] = hi[e];
+          for (int e = 0; e < 4; ++e) {
+            qb[e] = lo[e];
+            qb[4 + e] = hi[e];
+          }
+          y[i] = mfma(s2, qb, y[i]);
+          y[i] = mfma(s1, qb, y[i]);
+          y[i] = mfma(s0, qb, y[i]);
         }
-        y[i] = mfma(s2, qb, y[i]);
-        y[i] = mfma(s1, qb, y[i]);
-        y[i] = mfma(s0, qb, y[i]);
       }
     }
+    // each wave of a pair finishes two token tiles: the other two go to its partner
 #pragma unroll
-    for (int i = 0; i < 4; ++i) y[i] *= eg[cb + 16 * i + l16];
-    // this wave's columns of v: lane l16 a column, tokens 32 s + 8 q4 + e
+    for (int i = 0; i < 2; ++i) Ys[(w * 2 + i) * 64 + lane] = pick(half, y[i], y[2 + i]);
+    // this pair's columns of v: lane l16 a column, tokens 32 s + 8 q4 + e
     bf16x8 vf[2];
 #pragma unroll
-    for (int s = 0; s < 2; ++s) vf[s] = read_tr(Vs, VP, 32 * s + 8 * q4, 32 * s + 8 * q4 + 4, 16 * w, l16);
+    for (int s = 0; s < 2; ++s) vf[s] = read_tr(Vs, VP, 32 * s + 8 * q4, 32 * s + 8 * q4 + 4, 16 * wc, l16);
     // ---- next state
-    const float dc = eg[cb + C - 1];
+    if (rows_ok) {
+      const float dc = eg[cb + C - 1];
 #pragma unroll
-    for (int s = 0; s < 2; ++s) {
-      bf16x8 u0, u1, u2;
+      for (int s = 0; s < 2; ++s) {
+        bf16x8 u0, u1, u2;
+        float x[8];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        bf16 a, b, d;
-        split3((float)vf[s][e] * ws[cb + 32 * s + 8 * q4 + e], a, b, d);
-        u0[e] = a;
-        u1[e] = b;
-        u2[e] = d;
-      }
+        for (int e = 0; e < 8; ++e) x[e] = (float)vf[s][e] * ws[cb + 32 * s + 8 * q4 + e];
+        split3(x, u0, u1, u2);
 #pragma unroll
-      for (int t = 0; t < 2 * NK; ++t) {
-        const bf16x8 kf = read_tr(Ks, KP, 32 * s + 8 * q4, 32 * s + 8 * q4 + 4, 16 * t, l16);
-        if (s == 0) S[t] *= dc;
-        S[t] = mfma(kf, u2, S[t]);
-        S[t] = mfma(kf, u1, S[t]);
-        S[t] = mfma(kf, u0, S[t]);
-      }
-    }
-    lds_barrier();  // P is complete
-    // ---- within the chunk
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-#pragma unroll
-      for (int s = 0; s <= (i >> 1); ++s) {
-        const bf16* pr = Ps + (16 * i + l16) * PP + 32 * s + 8 * q4;
-        y[i] = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr + 2 * C * PP), y[i]);
-        y[i] = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr + C * PP), y[i]);
-        y[i] = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr), y[i]);
-      }
-      const int t = c * C + 16 * i + l16, cv = v0 + 16 * w + 4 * q4;
-      const bf16x4 vv = *reinterpret_cast<const bf16x4*>(Vs + (16 * i + l16) * VP + 16 * w + 4 * q4);
-      bf16x4 o;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) o[r] = (bf16)fmaf(sk, (float)vv[r], y[i][r]);
-      if (t < n) {
-        bf16* dst = out + ((int64_t)(t0 + t) * D.H + h) * D.dv + cv;
-        if (cv + 3 < D.dv && D.dv % 4 == 0) {
-          *reinterpret_cast<bf16x4*>(dst) = o;
-        } else {
-#pragma unroll
-          for (int r = 0; r < 4; ++r)
-            if (cv + r < D.dv) dst[r] = o[r];
+        for (int t = 0; t < 2 * KH; ++t) {
+          const bf16x8 kf = read_tr(Ks, KP, 32 * s + 8 * q4, 32 * s + 8 * q4 + 4, k_first + 16 * t, l16);
+          if (s == 0) S[t] *= dc;
+          S[t] = mfma(kf, u2, S[t]);
+          S[t] = mfma(kf, u1, S[t]);
+          S[t] = mfma(kf, u0, S[t]);
         }
       }
     }
-    if (c + 1 < nc && w == (c & 3)) scan_gb(c + 1);
+    lds_barrier();  // P and the partner's half are complete
+    // ---- within the chunk, token tiles 2 half and 2 half + 1
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const int i = 2 * half + k;
+      f32x4 acc = pick(half, y[2 + k], y[k]);
+      acc = (acc + Ys[((w ^ 1) * 2 + k) * 64 + lane]) * eg[cb + 16 * i + l16];
+#pragma unroll
+      for (int s = 0; s < 2; ++s) {
+        if (s > half) break;
+        const bf16* pr = Ps + (16 * i + l16) * PP + 32 * s + 8 * q4;
+        acc = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr + 2 * C * PP), acc);
+        acc = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr + C * PP), acc);
+        acc = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr), acc);
+      }
+      const int t = c * C + 16 * i + l16, cv = v0 + 16 * wc + 4 * q4;
+      const bf16x4 vv = *reinterpret_cast<const bf16x4*>(Vs + (16 * i + l16) * VP + 16 * wc + 4 * q4);
+      bf16x4 o;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[r] = (bf16)fmaf(sk, (float)vv[r], acc[r]);
+      bf16* dst = out + ((int64_t)(t0 + t) * D.H + h) * D.dv + cv;
+      if (D.dv % 4 == 0) {
+        if (t < n && cv < D.dv) *reinterpret_cast<bf16x4*>(dst) = o;
+      } else if (t < n) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (cv + r < D.dv) dst[r] = o[r];
+      }
+    }
+    if (ahead) scan_gb(c + NW + w);
     lds_barrier();
   }
   if (col < D.dv) {
 #pragma unroll
-    for (int t = 0; t < 2 * NK; ++t) {
-      const int k = 16 * t + 4 * q4;
+    for (int t = 0; t < 2 * KH; ++t) {
+      const int k = k_first + 16 * t + 4 * q4;
       if (k < dks) *reinterpret_cast<f32x4*>(st + k) = S[t];
     }
   }
@@ -295,20 +352,21 @@ __global__ void __launch_bounds__(NT, (NK <= 4 ? 2 : 1)) decayed_chunk_kernel(
     advance_windows(conv_state + (int64_t)slots[seq] * (D.taps - 1) * D.channels, proj, t0, n, D, fresh, h);
 }
 
-template <int NK>
+template <int NK, int WC>
 int launch(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip, const void* proj,
            float* state, void* conv_state, const int* seqs, int nseq, const int* cu, const int* start, const int* slots,
            void* out, const ScanDims& D, hipStream_t st) {
-  constexpr int LDS = (2 * C * (32 * NK + 8) + C * VP + 3 * C * PP) * 2 + 2 * C * 8 + 6 * C * 4;
+  constexpr int VT = 16 * WC;
+  constexpr int LDS = (2 * C * (32 * NK + 8) + C * (VT + 8) + 3 * C * PP) * 2 + 2 * WC * 2 * 64 * 16 + 4 * WC * C * 20;
   static bool attr = false;
   if (!attr) {
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<NK>),
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<NK, WC>),
                               hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
     attr = true;
   }
-  hipLaunchKernelGGL((decayed_chunk_kernel<NK>), dim3((unsigned)((D.dv + VT - 1) / VT * D.H * nseq)), dim3(NT), LDS, st,
-                     (const bf16*)qk, (const bf16*)v, gb, log_decay, skip, (const bf16*)proj, state, (bf16*)conv_state, seqs,
-                     cu, start, slots, (bf16*)out, D);
+  hipLaunchKernelGGL((decayed_chunk_kernel<NK, WC>), dim3((unsigned)((D.dv + VT - 1) / VT * D.H * nseq)), dim3(128 * WC), LDS,
+                     st, (const bf16*)qk, (const bf16*)v, gb, log_decay, skip, (const bf16*)proj, state, (bf16*)conv_state,
+                     seqs, cu, start, slots, (bf16*)out, D);
   DS_CHECK_LAUNCH();
   return 0;
 }
@@ -325,10 +383,13 @@ extern "C" int ds_scan_chunk(const void* qk, const void* v, const float* gb, con
   const ScanDims D{dims[0], dims[1], dims[2], dims[3], dims[4], dims[5], dims[6], dims[7], dims[8], dims[9], dims[10], dims[11],
                    tokens};
   if (!scan_dims_ok(D) || !ds_scan_chunk_ok(D.dk) || (!gb == !log_decay) || (D.taps > 1 && !conv_state) ||
-      (int64_t)nseq * D.H * ((D.dv + VT - 1) / VT) > INT32_MAX)
+      (int64_t)nseq * D.H * ((D.dv + 31) / 32) > INT32_MAX)
     return (int)hipErrorInvalidValue;
-#define GO(NK)                                                                                                      \
-  return launch<NK>(qk, v, gb, log_decay, skip, proj, state, conv_state, seqs, nseq, cu, start, slots, out, D, st)
+  // wide workgroups share q, k and P among more columns; narrow ones where there are too few to fill the chip
+  const bool wide = D.dv > 32 && (int64_t)nseq * D.H * ((D.dv + 63) / 64) >= 192;
+#define GO(NK)                                                                                                         \
+  return wide ? launch<NK, 4>(qk, v, gb, log_decay, skip, proj, state, conv_state, seqs, nseq, cu, start, slots, out, D, st) \
+              : launch<NK, 2>(qk, v, gb, log_decay, skip, proj, state, conv_state, seqs, nseq, cu, start, slots, out, D, st)
   if (D.dk <= 32) GO(1);
   if (D.dk <= 64) GO(2);
   if (D.dk <= 128) GO(4);
