@@ -202,10 +202,19 @@ __global__ void __launch_bounds__(256) head_linear_any_kernel(HeadArgs a) {
 // one wave per context row of 16-byte pieces
 __global__ void __launch_bounds__(256) latent_gather_kernel(const bf16* __restrict__ lat, const int* __restrict__ bt,
                                                             int max_blocks, const int* __restrict__ offs, int first,
-                                                            int nseq, bf16* __restrict__ ctx, int64_t total, int row,
-                                                            int BS) {
+                                                            int nseq, bf16* __restrict__ ctx, int64_t total, int pad,
+                                                            int row, int BS) {
   const int64_t i = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (i >= total) return;
+  if (i >= total + pad) return;
+  if (i >= total) {
+    for (int c = (threadIdx.x & 63) * 8; c < row; c += 512) {
+      bf16x8 z;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) z[j] = (bf16)0.f;
+      *reinterpret_cast<bf16x8*>(ctx + i * row + c) = z;
+    }
+    return;
+  }
   int s = 0;
   while (s + 1 < nseq && i >= offs[s + 1]) ++s;
   const int p = (int)(i - offs[s]);
@@ -273,13 +282,14 @@ extern "C" int ds_head_linear(const void* x, const void* w, void* y, int T, int 
   return 0;
 }
 
-// contexts of sequences first .. first + nseq, offs [nseq + 1] their places in ctx [total, row] (bf16)
+// contexts of sequences first .. first + nseq, offs [nseq + 1] their places in ctx [total + pad, row] (bf16), whose
+// last `pad` rows become zero
 extern "C" int ds_latent_gather(const void* lat, const int* bt, int max_blocks, const int* offs, int first, int nseq, void* ctx,
-                                int64_t total, int row, int BS, hipStream_t st) {
+                                int64_t total, int pad, int row, int BS, hipStream_t st) {
   if (total <= 0) return 0;
   if (row <= 0 || row % 8 || BS <= 0 || max_blocks <= 0 || nseq <= 0) return (int)hipErrorInvalidValue;
-  hipLaunchKernelGGL(latent_gather_kernel, dim3((unsigned)((total + 3) / 4)), dim3(256), 0, st, (const bf16*)lat, bt, max_blocks,
-                     offs, first, nseq, (bf16*)ctx, total, row, BS);
+  hipLaunchKernelGGL(latent_gather_kernel, dim3((unsigned)((total + pad + 3) / 4)), dim3(256), 0, st, (const bf16*)lat, bt,
+                     max_blocks, offs, first, nseq, (bf16*)ctx, total, pad, row, BS);
   DS_CHECK_LAUNCH();
   return 0;
 }

@@ -4,7 +4,8 @@
 
 // q / o [T, H, dn + r] / [T, H, dv] bf16, rotated; kv [rows, H (dn + dv)]: expanded context rows, keys of all heads, then
 // values; ctx [rows, ldr]: the latents' rows, whose columns rot0 .. rot0 + r are the rotated key part. kv_offs: place of the
-// contexts of sequences first, first + 1, ...; work [nwork, 2] (sequence, 128-row query block).
+// contexts of sequences first, first + 1, ...; work [nwork, 2] (sequence, 128-row query block). Tiles of 64 keys are
+// read whole: 64 (finite) rows must exist behind the last context in kv and ctx.
 extern "C" int ds_latent_prefill(const void* q, const void* kv, const void* ctx, void* o, const int* start, const int* cu_q,
                                  const int* work, int nwork, const int* kv_offs, int first, int H, int dn, int r, int dv,
                                  int ldr, int rot0, const float* sink, float scale, hipStream_t st) {

@@ -123,6 +123,7 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
   int kt1 = min((Skv + BN - 1) / BN, pos_hi / BN + 1);
   // first key a position sees (non-decreasing in the position)
   auto first_key = [&](int p) {
+    if (LAT) return 0;
     int lo = EXT && a.chunk > 0 ? p / a.chunk * a.chunk : 0;
     if (a.window > 0) lo = max(lo, p - a.window + 1);
     return lo;
@@ -134,7 +135,30 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
   char* const ksm = smem;
   char* const vsm = smem + 2 * C::KBYTES;
   float* scratch = reinterpret_cast<float*>(smem + 2 * C::KBYTES + 2 * C::VBYTES) + wid * 32;
-  u32x4_t kreg[NLK], vreg[NLV];
+  constexpr int CK = LAT ? DK / 8 : PK, CV = LAT ? DV / 8 : PV;    // pieces of a row that are staged
+  constexpr int NK_ = LAT ? BN * CK / NTHR : NLK, NV_ = LAT ? BN * CV / NTHR : NLV;
+  u32x4_t kreg[NK_], vreg[NV_];
+  // LATENT: rows lie end to end, so every piece has a place of its own that moves on by the same step with every tile. Pieces
+  // past the widths repeat the last one: there the queries are zero, or nothing is stored. (Rows past the context's end are
+  // masked; 64 of them exist behind the last context.)
+  const bf16* kp_[NK_];
+  const bf16* vp_[NV_];
+  int kstep[NK_];
+  if constexpr (LAT) {
+#pragma unroll
+    for (int i = 0; i < NK_; ++i) {
+      const int row = (tid + i * NTHR) / CK, c = min((tid + i * NTHR) % CK * 8, dk - 8);
+      const bool up = c < a.dn;
+      const int64_t r_ = ctx0 + (int64_t)kt0 * BN + row;
+      kp_[i] = up ? a.kc + r_ * a.ldk + hq * a.dn + c : a.vc + r_ * a.ldr + a.rot0 + c - a.dn;
+      kstep[i] = BN * (up ? a.ldk : a.ldr);
+    }
+#pragma unroll
+    for (int i = 0; i < NV_; ++i) {
+      const int row = (tid + i * NTHR) / CV, c = min((tid + i * NTHR) % CV * 8, dv - 8);
+      vp_[i] = a.kc + (ctx0 + (int64_t)kt0 * BN + row) * a.ldk + a.Hq * a.dn + hq * dv + c;
+    }
+  }
   auto slot_of = [&](int tile, int row) {
     const int key = min(tile * BN + row, Skv - 1);
     return ((int64_t)bt[key / a.BS] * a.Hk + hk) * a.BS + key % a.BS;
@@ -153,40 +177,42 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
           vreg[i] = u32x4_t{0u, 0u, 0u, 0u};
         }
       }
+    } else if constexpr (LAT) {  // tiles are asked for in order
+#pragma unroll
+      for (int i = 0; i < NK_; ++i) {
+        kreg[i] = *reinterpret_cast<const u32x4_t*>(kp_[i]);
+        kp_[i] += kstep[i];
+      }
+#pragma unroll
+      for (int i = 0; i < NV_; ++i) {
+        vreg[i] = *reinterpret_cast<const u32x4_t*>(vp_[i]);
+        vp_[i] += BN * a.ldk;
+      }
     } else {
 #pragma unroll
       for (int i = 0; i < NLK; ++i) {
         const int cidx = tid + i * NTHR, row = cidx / PK, ch = cidx % PK;
         kreg[i] = u32x4_t{0u, 0u, 0u, 0u};
-        if constexpr (LAT) {
-          const int64_t row_ = ctx0 + min(tile * BN + row, Skv - 1);
-          if (ch * 8 < dk)
-            kreg[i] = *reinterpret_cast<const u32x4_t*>(ch * 8 < a.dn ? a.kc + row_ * a.ldk + hq * a.dn + ch * 8
-                                                                     : a.vc + row_ * a.ldr + a.rot0 + ch * 8 - a.dn);
-        } else if (ch * 8 < dk) kreg[i] = *reinterpret_cast<const u32x4_t*>(a.kc + slot_of(tile, row) * dk + ch * 8);
+        if (ch * 8 < dk) kreg[i] = *reinterpret_cast<const u32x4_t*>(a.kc + slot_of(tile, row) * dk + ch * 8);
       }
 #pragma unroll
       for (int i = 0; i < NLV; ++i) {
         const int cidx = tid + i * NTHR, row = cidx / PV, ch = cidx % PV;
         vreg[i] = u32x4_t{0u, 0u, 0u, 0u};
-        if constexpr (LAT) {
-          const int64_t row_ = ctx0 + min(tile * BN + row, Skv - 1);
-          if (ch * 8 < dv)
-            vreg[i] = *reinterpret_cast<const u32x4_t*>(a.kc + row_ * a.ldk + a.Hq * a.dn + hq * dv + ch * 8);
-        } else if (ch * 8 < dv) vreg[i] = *reinterpret_cast<const u32x4_t*>(a.vc + slot_of(tile, row) * dv + ch * 8);
+        if (ch * 8 < dv) vreg[i] = *reinterpret_cast<const u32x4_t*>(a.vc + slot_of(tile, row) * dv + ch * 8);
       }
     }
   };
   auto stage_store = [&](int buf) {
 #pragma unroll
-    for (int i = 0; i < NLK; ++i) {
-      const int cidx = tid + i * NTHR, row = cidx / PK, ch = cidx % PK;
-      if (ch < DK / 8) *reinterpret_cast<u32x4_t*>(ksm + buf * C::KBYTES + lds_off<RK>(row, ch)) = kreg[i];
+    for (int i = 0; i < NK_; ++i) {
+      const int cidx = tid + i * NTHR, row = cidx / CK, ch = cidx % CK;
+      if (LAT || ch < DK / 8) *reinterpret_cast<u32x4_t*>(ksm + buf * C::KBYTES + lds_off<RK>(row, ch)) = kreg[i];
     }
 #pragma unroll
-    for (int i = 0; i < NLV; ++i) {
-      const int cidx = tid + i * NTHR, row = cidx / PV, ch = cidx % PV;
-      if (ch < 4 * DT) *reinterpret_cast<u32x4_t*>(vsm + buf * C::VBYTES + lds_off<RV>(row, ch)) = vreg[i];
+    for (int i = 0; i < NV_; ++i) {
+      const int cidx = tid + i * NTHR, row = cidx / CV, ch = cidx % CV;
+      if (LAT || ch < 4 * DT) *reinterpret_cast<u32x4_t*>(vsm + buf * C::VBYTES + lds_off<RV>(row, ch)) = vreg[i];
     }
   };
 
@@ -222,8 +248,8 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
         }
       }
       // ALiBi bias, causal diagonal, window, key tail (lane = one query row, r = 32 keys of the 64)
-      const bool need_mask = k0 + BN - 1 > wpos_lo || k0 + BN > Skv || k0 < lo_whi;
-      if constexpr (EXT) {
+      const bool need_mask = k0 + BN - 1 > wpos_lo || (!LAT && (k0 + BN > Skv || k0 < lo_whi));
+      if constexpr (MODE == EXT_) {
         if (a.cap_out > 0.f) {
 #pragma unroll
           for (int t = 0; t < 2; ++t)
@@ -232,19 +258,19 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
               s[t][r] = a.cap_out * (1.f - 2.f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s[t][r] * a.cap_in) + 1.f));
         }
       }
-      if (a.alibi || need_mask) {
+      if ((!LAT && a.alibi) || need_mask) {
 #pragma unroll
         for (int t = 0; t < 2; ++t)
 #pragma unroll
           for (int r = 0; r < 16; ++r) {
             const int key = k0 + t * 32 + (r & 3) + 8 * (r >> 2) + 4 * h;
-            float v = fmaf(slope, (float)(key - pos_lane), s[t][r]);
-            if (key >= Skv || key > pos_lane || key < lo_lane) v = -INFINITY;
+            float v = LAT ? s[t][r] : fmaf(slope, (float)(key - pos_lane), s[t][r]);
+            if (LAT ? key > pos_lane : key >= Skv || key > pos_lane || key < lo_lane) v = -INFINITY;
             s[t][r] = v;
           }
       }
       // a moderate cap bounds the scores: it serves as the maximum, and nothing is ever rescaled
-      const bool fixed = EXT && a.cap_out > 0.f && a.cap_out <= 48.f;
+      const bool fixed = MODE == EXT_ && a.cap_out > 0.f && a.cap_out <= 48.f;
       float alpha = 1.f, mc = a.cap_out;
       if (!fixed) {
         float mx = -INFINITY;
@@ -284,44 +310,51 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
           for (int r = 0; r < 16; ++r) o[dt][r] *= a4[r];
         __builtin_amdgcn_wave_barrier();
       }
-      bf16x8_t pa[2][2];
+      const int gq = (lane >> 2) & 3, gch = (lane >> 1) & 1, gb = 8 * (lane & 1), colhalf = (lane >> 4) & 1;
+      auto v_of = [&](int t, int ss, int dt) {  // 16 keys of 32 value columns, transposed on the way out of LDS
+        const int ch0 = dt * 4 + colhalf * 2 + gch, rb = t * 32 + 16 * ss + 4 * h;
+        const s16x4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (__attribute__((address_space(3))) s16x4_t*)(Vt + lds_off<RV>(rb + gq, ch0) + gb));
+        const s16x4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (__attribute__((address_space(3))) s16x4_t*)(Vt + lds_off<RV>(rb + 8 + gq, ch0) + gb));
+        s16x8 vv;
 #pragma unroll
-      for (int t = 0; t < 2; ++t)
+        for (int e = 0; e < 4; ++e) { vv[e] = lo[e]; vv[4 + e] = hi[e]; }
+        return __builtin_bit_cast(bf16x8_t, vv);
+      };
+      if constexpr (EXT) {  // 16 keys at a time: weights as two bf16 terms, the second what the first leaves out
 #pragma unroll
-        for (int ss = 0; ss < 2; ++ss)
+        for (int t = 0; t < 2; ++t)
 #pragma unroll
-          for (int e = 0; e < 8; ++e) pa[t][ss][e] = (bf16)s[t][8 * ss + e];
-      bf16x8_t pl[2][2];  // what the bf16 weights leave out
-      if constexpr (EXT) {
+          for (int ss = 0; ss < 2; ++ss) {
+            bf16x8_t pa, pl;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+              pa[e] = (bf16)s[t][8 * ss + e];
+              pl[e] = (bf16)(s[t][8 * ss + e] - (float)pa[e]);
+            }
+#pragma unroll
+            for (int dt = 0; dt < DT; ++dt) {
+              const bf16x8_t vv = v_of(t, ss, dt);
+              o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pa, vv, o[dt], 0, 0, 0);
+              o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pl, vv, o[dt], 0, 0, 0);
+            }
+          }
+      } else {
+        bf16x8_t pa[2][2];
 #pragma unroll
         for (int t = 0; t < 2; ++t)
 #pragma unroll
           for (int ss = 0; ss < 2; ++ss)
 #pragma unroll
-            for (int e = 0; e < 8; ++e) pl[t][ss][e] = (bf16)(s[t][8 * ss + e] - (float)pa[t][ss][e]);
-      }
-      const int gq = (lane >> 2) & 3, gch = (lane >> 1) & 1, gb = 8 * (lane & 1), colhalf = (lane >> 4) & 1;
+            for (int e = 0; e < 8; ++e) pa[t][ss][e] = (bf16)s[t][8 * ss + e];
 #pragma unroll
-      for (int dt = 0; dt < DT; ++dt) {
-        const int ch0 = dt * 4 + colhalf * 2 + gch;
+        for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
-        for (int t = 0; t < 2; ++t)
+          for (int t = 0; t < 2; ++t)
 #pragma unroll
-          for (int ss = 0; ss < 2; ++ss) {
-            const int rb = t * 32 + 16 * ss + 4 * h;
-            const s16x4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                (__attribute__((address_space(3))) s16x4_t*)(Vt + lds_off<RV>(rb + gq, ch0) + gb));
-            const s16x4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                (__attribute__((address_space(3))) s16x4_t*)(Vt + lds_off<RV>(rb + 8 + gq, ch0) + gb));
-            s16x8 vv;
-#pragma unroll
-            for (int e = 0; e < 4; ++e) { vv[e] = lo[e]; vv[4 + e] = hi[e]; }
-            o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pa[t][ss], __builtin_bit_cast(bf16x8_t, vv), o[dt], 0,
-                                                           0, 0);
-            if constexpr (EXT)
-              o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pl[t][ss], __builtin_bit_cast(bf16x8_t, vv), o[dt], 0, 0,
-                                                             0);
-          }
+            for (int ss = 0; ss < 2; ++ss)
+              o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pa[t][ss], v_of(t, ss, dt), o[dt], 0, 0, 0);
       }
     }
     if (j + 1 < kt1) stage_store(cur ^ 1);
@@ -332,7 +365,7 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
   float inv = l_tot > 0.f ? 1.f / l_tot : 0.f;
   if constexpr (EXT) {
     if (a.sink) {  // in the frame of the maximum the weights were taken in
-      const float sk = a.sink[hq] * 1.4426950408889634f, m = a.cap_out > 0.f && a.cap_out <= 48.f ? a.cap_out : m_run * a.c;
+      const float sk = a.sink[hq] * 1.4426950408889634f, m = MODE == EXT_ && a.cap_out > 0.f && a.cap_out <= 48.f ? a.cap_out : m_run * a.c;
       const float mn = fmaxf(m, sk), f = __builtin_amdgcn_exp2f(m - mn);
       inv = f / fmaf(l_tot, f, __builtin_amdgcn_exp2f(sk - mn));
     }

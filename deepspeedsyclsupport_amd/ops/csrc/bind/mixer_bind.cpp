@@ -14,7 +14,7 @@ int ds_latent_prepare(const void*, const float*, const float*, float, const doub
 int ds_rotate_tail(void*, int, int, int, int, const double*, int, const int*, int, hipStream_t);
 int ds_head_linear(const void*, const void*, void*, int, int, int, int, int, int, int, int, const double*, const int*, int,
                    hipStream_t);
-int ds_latent_gather(const void*, const int*, int, const int*, int, int, void*, int64_t, int, int, hipStream_t);
+int ds_latent_gather(const void*, const int*, int, const int*, int, int, void*, int64_t, int, int, int, hipStream_t);
 int ds_paged_generic(const void*, const void*, const void*, void*, const int*, int, const int*, const int*, int, int, int,
                      int, int, int, int, float, float, int, int, const float*, int, hipStream_t);
 int ds_latent_decode_ok(int, int);
@@ -191,26 +191,28 @@ void latent_decode(Tensor q, Tensor lat, Tensor bt, Tensor cu, Tensor start, int
                          f32(sink, H, "sink"), (float)scale, stream()), "latent_decode");
 }
 
-// cached rows of the contexts of sequences first .. first + nseq, end to end
+// cached rows of the contexts of sequences first .. first + nseq, end to end, and PAD_ROWS rows of zeros: latent_prefill
+// reads whole tiles of keys
+constexpr int PAD_ROWS = 64;
 Tensor latent_gather(Tensor lat, Tensor bt, Tensor offs, int64_t first, int64_t total) {
   const Lat c = lat_of(lat);
   const int64_t nseq = offs.numel() - 1;
   table(bt, first + nseq);
   TORCH_CHECK(lat.scalar_type() == at::kBFloat16 && c.W % 8 == 0 && nseq > 0, "latent_gather: bf16 rows of 16-byte pieces");
-  auto ctx = torch::empty({total, c.W}, lat.options());
+  auto ctx = torch::empty({total + PAD_ROWS, c.W}, lat.options());
   check(ds_latent_gather(lat.data_ptr(), bt.data_ptr<int>(), (int)bt.size(1), i32(offs, nseq + 1, "offs"), (int)first, (int)nseq,
-                         ctx.data_ptr(), total, c.W, c.BS, stream()), "latent_gather");
+                         ctx.data_ptr(), total, PAD_ROWS, c.W, c.BS, stream()), "latent_gather");
   return ctx;
 }
 
-// q [T, H, d + r] rotated; kv [rows, H (d + e)], ctx [rows, R + r] -> rows of o [T, H, e] of the sequences in work
+// q [T, H, d + r] rotated; kv [total + PAD_ROWS, H (d + e)], ctx [total + PAD_ROWS, R + r] -> rows of o [T, H, e] of the sequences in work
 void latent_prefill(Tensor q, Tensor kv, Tensor ctx, Tensor start, Tensor cu_q, Tensor work, Tensor offs, int64_t first,
-                    int64_t d, int64_t e, double scale, Tensor sink, Tensor o) {
+                    int64_t total, int64_t d, int64_t e, double scale, Tensor sink, Tensor o) {
   need(q, "q"); need(kv, "kv"); need(ctx, "ctx"); need(o, "o");
   const int64_t T = q.size(0), H = q.size(1), r = q.size(2) - d, S = start.numel();
   TORCH_CHECK(q.dim() == 3 && q.scalar_type() == at::kBFloat16 && kv.scalar_type() == at::kBFloat16 &&
               ctx.scalar_type() == at::kBFloat16 && kv.dim() == 2 && kv.size(1) == H * (d + e) && ctx.dim() == 2 &&
-              ctx.size(0) == kv.size(0) && ctx.size(1) >= r && ds_latent_prefill_ok((int)d, (int)r, (int)e), "latent_prefill");
+              ctx.size(0) == kv.size(0) && ctx.size(0) == total + PAD_ROWS && ctx.size(1) >= r && ds_latent_prefill_ok((int)d, (int)r, (int)e), "latent_prefill");
   TORCH_CHECK(o.dim() == 3 && o.size(0) == T && o.size(1) == H && o.size(2) == e && o.scalar_type() == q.scalar_type() &&
               work.dim() == 2 && work.size(1) == 2 && offs.numel() == S - first + 1 && scale > 0, "latent_prefill: o / tables");
   check(ds_latent_prefill(q.data_ptr(), kv.data_ptr(), ctx.data_ptr(), o.data_ptr(), i32(start, S, "start"),

@@ -79,7 +79,7 @@ def latent_attention(q, lat, ukv, ukt, freq, sink, meta, scale, d, e):
         kv = F.linear(ctx[:, :R], ukv)
         ops.rotate_tail(q[short:], freq, meta.pos_ids[short:], q.shape[2] - d)
         ops.latent_prefill(q, kv, ctx, meta.start_pos, meta.cu_q, meta.work[meta.n_short - meta.n_decode:], meta.kv_offs,
-                           meta.n_short, d, e, scale, sink, o)
+                           meta.n_short, meta.kv_total, d, e, scale, sink, o)
     return o
 
 
