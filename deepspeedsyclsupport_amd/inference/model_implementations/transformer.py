@@ -12,7 +12,9 @@ all-reduce each (bias added once after it), vocab-parallel LM head with an all-g
 Weight-only int8/int4 quantisation keeps group-quantised weights and dequantises into a per-layer workspace.
 """
 import math
+from array import array
 from dataclasses import dataclass, field
+from itertools import accumulate, repeat
 from typing import List, Optional
 
 import torch
@@ -190,43 +192,56 @@ class RaggedMeta:
         """`slots`: state slots of the sequences; `logit_rows`: rows (of the concatenated tokens) whose logits are
         wanted instead of every sequence's last."""
         S = len(starts)
-        cu = [0]
-        for n in n_new:
-            cu.append(cu[-1] + n)
+        cu = list(accumulate(n_new, initial=0))
         T = cu[-1]
         width = max(1, max(len(b) for b in block_lists))
-        pos, sid = [], []
-        for i, (st, n) in enumerate(zip(starts, n_new)):
-            pos.extend(range(st, st + n))
-            sid.extend([i] * n)
-        work = [(i, qb) for i in range(n_decode, S) for qb in range(-(-n_new[i] // 128))]
-        bt = []
-        for b in block_lists:
-            bt.extend(list(b) + [0] * (width - len(b)))
         lens = [st + n for st, n in zip(starts, n_new)]
         last = [c - 1 for c in cu[1:]] if logit_rows is None else list(logit_rows)
         slots = [] if slots is None else list(slots)
         long = [i for i in range(S) if n_new[i] > RaggedMeta.STEP_TOKENS] if slots else []
         short = [i for i in range(S) if n_new[i] <= RaggedMeta.STEP_TOKENS] if slots else []
-        chunks, chunk_seqs = [], []
-        for i in long:
-            chunk_seqs += [i, len(chunks)]
-            chunks += [(i, c) for c in range(-(-n_new[i] // RaggedMeta.STATE_CHUNK))]
         # (a sequence is only counted as short if everything before it in the batch is)
         n_short = next((i for i in range(n_decode, S) if n_new[i] > RaggedMeta.SHORT_TOKENS), S)
-        kv = [0]
-        for i in range(n_short, S):
-            kv.append(kv[-1] + lens[i])
-        flat = pos + sid + list(starts) + lens + cu + [x for w in work for x in w] + last + bt + slots + short + chunk_seqs + \
-            [x for w in chunks for x in w] + kv
-        buf = torch.tensor(flat, dtype=torch.int32)
+        kv = list(accumulate(lens[n_short:], initial=0))
+        # everything in one array of 32-bit integers (a decode step is bound by the host: no detour over long lists)
+        flat, sizes = array("i"), []
+
+        def part(values=()):
+            flat.extend(values)
+            sizes.append(len(flat))
+
+        for st, n in zip(starts, n_new):
+            flat.extend((st, ) if n == 1 else range(st, st + n))
+        part()
+        for i, n in enumerate(n_new):
+            flat.extend((i, ) if n == 1 else repeat(i, n))
+        part()
+        part(starts)
+        part(lens)
+        part(cu)
+        for i in range(n_decode, S):
+            for qb in range(-(-n_new[i] // 128)):
+                flat.extend((i, qb))
+        part()
+        part(last)
+        for b in block_lists:
+            flat.extend(b)
+            flat.frombytes(bytes(4 * (width - len(b))))
+        part()
+        part(slots)
+        part(short)
+        chunks, chunk_seqs = [], []
+        for i in long:
+            chunk_seqs += [i, len(chunks) // 2]
+            for c in range(-(-n_new[i] // RaggedMeta.STATE_CHUNK)):
+                chunks += (i, c)
+        part(chunk_seqs)
+        part(chunks)
+        part(kv)
+        buf = torch.frombuffer(flat, dtype=torch.int32)
         if device is not None and torch.device(device).type == "cuda":
             buf = buf.pin_memory().to(device, non_blocking=True)
-        views, o = [], 0
-        for n in (T, T, S, S, S + 1, 2 * len(work), len(last), S * width, len(slots), len(short), len(chunk_seqs),
-                  2 * len(chunks), len(kv)):
-            views.append(buf[o:o + n])
-            o += n
+        views = [buf[a:b] for a, b in zip([0] + sizes, sizes)]
         pos_t, sid_t, st_t, len_t, cu_t, work_t, last_t, bt_t, slot_t, short_t, long_t, chunk_t, kv_t = views
         return RaggedMeta(block_tables=bt_t.view(S, width), start_pos=st_t, seq_lens=len_t, pos_ids=pos_t,
                           seq_ids=sid_t, cu_q=cu_t, work=work_t.view(-1, 2), last_idx=last_t.long(),

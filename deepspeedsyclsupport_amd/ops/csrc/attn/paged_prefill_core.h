@@ -322,7 +322,8 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
         for (int e = 0; e < 4; ++e) { vv[e] = lo[e]; vv[4 + e] = hi[e]; }
         return __builtin_bit_cast(bf16x8_t, vv);
       };
-      if constexpr (EXT) {  // 16 keys at a time: weights as two bf16 terms, the second what the first leaves out
+      // EXT, LATENT: weights as two bf16 terms, the second what the first leaves out
+      if constexpr (LAT) {  // (16 keys at a time: with wide keys the registers are short)
 #pragma unroll
         for (int t = 0; t < 2; ++t)
 #pragma unroll
@@ -348,13 +349,25 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
           for (int ss = 0; ss < 2; ++ss)
 #pragma unroll
             for (int e = 0; e < 8; ++e) pa[t][ss][e] = (bf16)s[t][8 * ss + e];
+        bf16x8_t pl[2][2];
+        if constexpr (EXT) {
+#pragma unroll
+          for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int ss = 0; ss < 2; ++ss)
+#pragma unroll
+              for (int e = 0; e < 8; ++e) pl[t][ss][e] = (bf16)(s[t][8 * ss + e] - (float)pa[t][ss][e]);
+        }
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
           for (int t = 0; t < 2; ++t)
 #pragma unroll
-            for (int ss = 0; ss < 2; ++ss)
-              o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pa[t][ss], v_of(t, ss, dt), o[dt], 0, 0, 0);
+            for (int ss = 0; ss < 2; ++ss) {
+              const bf16x8_t vv = v_of(t, ss, dt);
+              o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pa[t][ss], vv, o[dt], 0, 0, 0);
+              if constexpr (EXT) o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(pl[t][ss], vv, o[dt], 0, 0, 0);
+            }
       }
     }
     if (j + 1 < kt1) stage_store(cur ^ 1);

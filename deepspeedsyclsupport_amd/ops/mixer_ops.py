@@ -65,12 +65,12 @@ def latent_attention(q, lat, ukv, ukt, freq, sink, meta, scale, d, e):
         ql = ops.head_linear(q[:short], ukt, freq, meta.pos_ids[:short])  # [short, H, R + rot]
         if tiled:
             ol = q.new_empty(short, H, R)
+            cu = meta.cu_host
             for a, b in ((0, meta.n_decode), (meta.n_decode, meta.n_short)):  # decodes; short portions
                 if a < b:
-                    cu = meta.cu_host
-                    ops.latent_decode(ql, lat, meta.block_tables, meta.cu_q, meta.start_pos, a, b - a,
-                                      max(cu[i + 1] - cu[i] for i in range(a, b)), cu[a], cu[b], meta.max_len, R, scale, sink,
-                                      ol)
+                    longest = 1 if b == meta.n_decode else max(cu[i + 1] - cu[i] for i in range(a, b))
+                    ops.latent_decode(ql, lat, meta.block_tables, meta.cu_q, meta.start_pos, a, b - a, longest, cu[a], cu[b],
+                                      meta.max_len, R, scale, sink, ol)
         else:
             ol = ops.latent_generic(ql, lat, meta.block_tables, meta.pos_ids, meta.seq_ids, R, scale, sink)
         ops.head_linear(ol, ukv[H * d:].view(H, e, R), out=o[:short])
