@@ -24,7 +24,8 @@ constexpr int CLAMPED_GLU = 5;  // DS_ACT_CLAMPED_GLU
 constexpr int UNARY = 16;       // DS_ACT_UNARY
 
 // x [M, K] . w [N, K]^T for M <= 16 bf16 rows: the vector kernel up to two rows (or where K does not tile), else MFMA.
-// act: an activation code applied to the result. With a limit instead, w is a fused [gate | up] weight and the result its clamped gated activation [M, N / 2].
+// act: an activation code applied to the result. With a limit instead, w is a fused [gate | up] weight and the result its
+// clamped gated activation [M, N / 2].
 Tensor decode_linear(Tensor x, Tensor w, std::optional<double> glu_limit, std::optional<int64_t> act) {
   need(x, "x"); need(w, "w");
   const int64_t N = w.size(0), K = w.size(1), M = x.numel() / K;
@@ -61,8 +62,8 @@ Tensor decode_linear_sh(Tensor x, Tensor wsh, int64_t N, std::optional<double> g
   auto sizes = x.sizes().vec();
   sizes.back() = glu ? N / 2 : N;
   auto y = torch::empty(sizes, x.options());
-  check(ds_skinny_b16_mfma(x.data_ptr(), wsh.data_ptr(), nullptr, glu || act.has_value() ? nullptr : y.data_ptr(), ws.data_ptr<float>(),
-                           (int)M, (int)N, (int)K, stream()), "decode_linear_sh");
+  check(ds_skinny_b16_mfma(x.data_ptr(), wsh.data_ptr(), nullptr, glu || act.has_value() ? nullptr : y.data_ptr(),
+                           ws.data_ptr<float>(), (int)M, (int)N, (int)K, stream()), "decode_linear_sh");
   if (act.has_value())
     check(ds_skinny_finalize_act(ws.data_ptr<float>(), y.data_ptr(), (int)M, (int)N, (int)NP, (int)*act, stream()),
           "decode_linear_sh (activation)");
@@ -78,6 +79,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("act") = py::none());
   m.def("decode_linear_ok", &decode_linear_ok);
   m.def("decode_linear_sh", &decode_linear_sh, py::arg("x"), py::arg("wsh"), py::arg("N"),
-        py::arg("glu_limit") = py::none(),
-        py::arg("act") = py::none());
+        py::arg("glu_limit") = py::none(), py::arg("act") = py::none());
 }
