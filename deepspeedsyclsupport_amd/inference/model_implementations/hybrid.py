@@ -7,6 +7,7 @@ constants as parameters:
 
 * `StreamResidual`    S fp32 residual streams, mixed by small matrices around every sublayer, fused with the pre-norm
 * `PostNormResidual`  one fp32 residual; the sublayers read it as it is and their outputs are RMS-normed before the sum
+* `PreNormResidual`   one fp32 residual with RMS norms on the sublayers' inputs
 * `AttentionMixer`    GQA, key and value widths of their own, per-head query / key RMS norm, score cap, chunked
                       visibility, value mixing with an earlier layer; K / V live in the blocked cache
 * `LatentMixer`       attention over a shared low-rank latent with a rotated key part and a softmax sink; only the latent
@@ -14,8 +15,14 @@ constants as parameters:
 * `DeltaMixer`        gated delta rule behind short convolutions; its fp32 state lives in a slot per sequence
 * `Mamba2Mixer`       state-space recurrence with a scalar decay per head and token behind a short convolution
 * `LightningMixer`    linear attention with a constant decay per head
+* `RotaryAttention`   GQA with projection biases, query / key norms over all heads, partial rotation, chunked visibility and a
+                      softmax sink
+* `MatrixMemory`      recurrence with exponential input and forget gates, a running maximum and a normaliser
+* `Retention`         linear attention with rotated queries and keys and a constant decay per head
+* `ParallelMixer`     two of these on the same input, their weighted outputs summed
 * `ClampedMLP`        gated feed-forward with clamped gate and up branches
 * `GeluMLP`           plain feed-forward with the exact gelu
+* `RoutedMLP`         gated experts, chosen per token among the best groups of experts
 * `TokenSide`         a small embedding per layer and token, gated by the residual
 
 Per sublayer the launches are: residual + norm, one fused input projection, the mixer's kernels, the output projection.
@@ -25,8 +32,9 @@ import math
 import torch
 import torch.nn as nn
 
+from ...ops import expert_ops
 from ...ops import hybrid_ops as ops
-from ...ops import mixer_ops
+from ...ops import mixer_ops, op_builder
 from .transformer import DSInferenceModel, ProjectionLayer
 
 
@@ -101,12 +109,38 @@ class PostNormResidual(nn.Module):
         return x + y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + spec.norm_eps) * self.norm_w
 
 
-RESIDUALS = {"streams": StreamResidual, "post_norm": PostNormResidual}
+class PreNormResidual(nn.Module):
+    """Norm weight of one sublayer's input: x <- x + f(x / rms(x) * w). A sublayer may hand over an `ExpertSum`; it is summed
+    in the pass that adds it."""
+
+    def __init__(self, streams, width, device):
+        super().__init__()
+        self.norm_w = _f32((width, ), 1.0, device)
+
+    @staticmethod
+    def begin(model, ids):
+        spec = model.spec
+        x = torch.empty(ids.numel(), spec.hidden_size, dtype=torch.float32, device=model.embed.device)
+        return x, expert_ops.pre_norm(x, None, model.layers[0].res1.norm_w, spec.norm_eps, ids=ids, embed=model.embed,
+                                      mult=spec.embed_scale)
+
+    def enter(self, spec, x, pending):
+        return expert_ops.pre_norm(x, pending[0], self.norm_w, spec.norm_eps)
+
+    def finish(self, model, x, y, rows):
+        return expert_ops.pre_norm(x, y, model.norm_w, model.spec.norm_eps, rows=rows)
+
+    def peek(self, spec, x, y):
+        return x + (y.sum() if isinstance(y, expert_ops.ExpertSum) else y).float()
+
+
+RESIDUALS = {"streams": StreamResidual, "post_norm": PostNormResidual, "pre_norm": PreNormResidual}
 
 
 class Mixer:
     """What a mixer may leave at its default. `rows`: width of the fused input projection; `out_width`: of its output."""
     extra_projections = ()   # names of weight matrices beside the input and output projection
+    extensions = ()          # native extensions its ops come from
 
     def parameters(self, device):
         """Small fp32 weights, by name."""
@@ -132,6 +166,7 @@ class Mixer:
 class AttentionMixer(Mixer):
     """Sizes and constants of an attention mixer; the weights are the layer's."""
     kind = "attention"
+    extensions = ("ds_hybrid_ops", "ds_attn_ops")
 
     def __init__(self, mx, tp):
         self.H, self.G, self.dk, self.dv = mx["heads"] // tp, mx["kv_heads"] // tp, mx["dim"], mx["vdim"]
@@ -178,6 +213,7 @@ class AttentionMixer(Mixer):
 class DeltaMixer(Mixer):
     """Sizes of a gated-delta-rule mixer; the weights are the layer's."""
     kind = "delta"
+    extensions = ("ds_hybrid_ops", )
 
     def __init__(self, mx, tp):
         if mx["heads"] % mx["kv_heads"] or mx["kv_heads"] % tp:
@@ -217,6 +253,7 @@ class LatentMixer(Mixer):
     beside one rotated key part shared by all heads. The cache holds the latent and that part, one row per token."""
     kind = "latent_attention"
     extra_projections = ("uq_w", )
+    extensions = ("ds_mixer_ops", )
 
     def __init__(self, mx, tp):
         if mx["heads"] % tp:
@@ -269,6 +306,7 @@ class ScanMixer(Mixer):
     """Recurrences S_t = a_t S_(t-1) + b_t k_t v_t^T, o_t = S_t^T q_t + D v_t with a scalar decay per head; the layout of
     the fused projection row tells the kernels where everything is (`mixer_ops.ScanLayout`). Where a tensor-parallel
     split would cut a norm's part, every rank runs all heads and hands its share of the columns on."""
+    extensions = ("ds_mixer_ops", "ds_scan_ops")
 
     def _size(self, layout, parts, tp, split):
         self.lay, self.parts = layout, parts
@@ -369,12 +407,262 @@ class LightningMixer(ScanMixer):
                                                 "sigmoid_after"), layer)
 
 
-MIXERS = {m.kind: m for m in (AttentionMixer, LatentMixer, DeltaMixer, Mamba2Mixer, LightningMixer)}
+class SideMixer(Mixer):
+    """A mixer that reads its columns of a fused projection row (from `first` on) and writes its columns of a fused read-out,
+    so that several can stand side by side in a layer (`ParallelMixer`). `prefix` names its small weights, `mult` is a factor
+    of its output, applied in fp32 ahead of the output projection. Where a tensor-parallel split would cut a norm, every rank
+    runs all heads and hands its share of the columns on."""
+
+    def __init__(self, mx, tp, prefix="", first=0, mult=1.0):
+        self.prefix, self.first, self.mult = prefix, first, float(mult)
+
+    def _columns(self, cols, tp):
+        """`cols`: read-out columns of the heads that run here."""
+        self.cols, self.out_width = cols, cols if self.split or tp == 1 else cols // tp
+        if cols % self.out_width or (not self.split and cols % tp):
+            raise ValueError(f"{cols} columns over {tp} ranks")
+
+    def project(self, lw, r, tp):
+        """This rank's rows of the input projection."""
+        part = (lambda n: _shard(lw[self.prefix + n], r, tp)) if self.split else (lambda n: lw[self.prefix + n])
+        return torch.cat([part(n) for n in self.sections])
+
+    def output(self, lw, r, tp):
+        """This rank's columns of the output projection."""
+        return _shard(lw[self.prefix + "o_w"], r, tp, 1)
+
+    def small(self, lw, r, tp):
+        """The small weights, by name."""
+        return {}
+
+    def shard(self, lw, r, tp):
+        return {"qkv_w": self.project(lw, r, tp), "o_w": self.output(lw, r, tp), **self.small(lw, r, tp)}
+
+    def weight(self, layer, name):
+        return getattr(layer, self.prefix + name)
+
+    def read_out(self, layer, proj, meta, cache, carry, out):
+        """Projection rows [T, all columns of the layer] -> out [T, out_width] (columns of a wider matrix)."""
+        if self.out_width == self.cols:
+            self.heads(layer, proj, meta, cache, carry, out)
+            return
+        whole = proj.new_empty(proj.shape[0], self.cols)
+        self.heads(layer, proj, meta, cache, carry, whole)
+        r = layer.tp_rank * self.out_width
+        out.copy_(whole[:, r:r + self.out_width])
+
+    def run(self, layer, h, meta, cache, carry):
+        proj = layer._linear(h, "qkv_w")
+        out = proj.new_empty(proj.shape[0], self.out_width)
+        self.read_out(layer, proj, meta, cache, carry, out)
+        return out
 
 
-class ClampedMLP:
+class Rotation:
+    """Frequencies of rotated positions: pair i of `dims` / 2 turns by position * base^(-2 i / dims) / factor. The batch's angle
+    table is made once per step for all layers with the same constants."""
+
+    def __init__(self, rot, width):
+        self.dims, self.base = int(rot["dims"]), float(rot["base"])
+        self.factor = float((rot.get("scaling") or {}).get("factor", 1.0))
+        if self.dims % 2 or not 0 <= self.dims <= width:
+            raise ValueError(f"{self.dims} rotated of {width} dimensions")
+
+    def frequencies(self, device):
+        i = torch.arange(self.dims // 2, dtype=torch.float64)
+        return (self.base**(-2 * i / max(self.dims, 1)) / self.factor).to(device)
+
+    def angles(self, freq, meta, carry):
+        if not self.dims:
+            return None
+        tables = carry.setdefault("angles", {})
+        key = (self.dims, self.base, self.factor)
+        if key not in tables:
+            tables[key] = ops.rope_table(meta.pos_ids, freq)
+        return tables[key]
+
+
+class RotaryAttention(SideMixer):
+    """Sizes and constants; the weights are the layer's. The output's factor rides on the cached values."""
+    kind = "rotary_attention"
+    extensions = ("ds_attn_ops", )
+    sections = ("q_w", "k_w", "v_w")
+    split = False          # the query and key norms run over all heads
+
+    def __init__(self, mx, tp, prefix="", first=0, mult=1.0):
+        super().__init__(mx, tp, prefix, first, mult)
+        self.H, self.G, self.dk, self.dv = mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
+        if self.H % self.G:
+            raise ValueError(f"{self.H} query / {self.G} key heads")
+        self.scale, self.chunk = float(mx["scale"]), int((mx.get("mask") or {}).get("size") or 0)
+        self.rot = Rotation(mx["rot"], self.dk)
+        self.rows = (self.H + self.G) * self.dk + self.G * self.dv
+        self._columns(self.H * self.dv, tp)
+
+    def parameters(self, device):
+        p = self.prefix
+        return {p + "bias": _f32((self.rows, ), 0.0, device), p + "q_norm": _f32((self.H * self.dk, ), 1.0, device),
+                p + "k_norm": _f32((self.G * self.dk, ), 1.0, device)}
+
+    def constants(self, device):
+        # a score of zero without a value in every softmax
+        return {self.prefix + "rot_freq": self.rot.frequencies(device), self.prefix + "sink": torch.zeros(self.H, device=device)}
+
+    def small(self, lw, r, tp):
+        p = self.prefix
+        return {p + "bias": torch.cat([lw[p + n] for n in ("q_b", "k_b", "v_b")]), p + "q_norm": lw[p + "q_norm"],
+                p + "k_norm": lw[p + "k_norm"]}
+
+    def kv_geometry(self):
+        return self.G, self.dk, self.dv
+
+    def heads(self, layer, proj, meta, cache, carry, out):
+        w, kc, vc = self.weight, cache.k[layer.layer_idx], cache.v[layer.layer_idx]
+        cs = self.rot.angles(w(layer, "rot_freq"), meta, carry)
+        q = ops.qk_rope_append(proj[:, self.first:self.first + self.rows], w(layer, "bias"), w(layer, "q_norm"),
+                               w(layer, "k_norm"), layer.spec.norm_eps, cs, meta, kc, vc, self.H, self.mult)
+        ops.ragged_attention(q, kc, vc, meta, self.scale, chunk=self.chunk, sink=w(layer, "sink"), out=out)
+
+
+class HeadScan(SideMixer):
+    """A recurrence per head whose read-out is divided by its root mean square head by head: splits by heads."""
+    extensions = ("ds_scan_ops", )
+
+    def _heads(self, mx, tp, width):
+        """`width`: projection rows per head."""
+        H, self.dk, self.dv = mx["heads"], mx["dim"], mx["vdim"]
+        self.split = H % tp == 0
+        self.H = H // tp if self.split else H
+        self.rows = self.H * width
+        self._columns(self.H * self.dv, tp)
+        a, b = self.first + self.H * self.dk, self.first + 2 * self.H * self.dk
+        self.gate = b + self.H * self.dv
+        self.at = dict(q=self.first, k=a, v=b, gate=self.gate, Hk=self.H, H=self.H, dk=self.dk, dv=self.dv)
+
+    def state_geometry(self, dtype):
+        return {"state": ((self.H, self.dv, -(-self.dk // 8) * 8), torch.float32)}
+
+
+class MatrixMemory(HeadScan):
+    kind = "matrix_memory"
+    sections = ("q_w", "k_w", "v_w", "g_w", "i_w", "f_w")
+
+    def __init__(self, mx, tp, prefix="", first=0, mult=1.0):
+        super().__init__(mx, tp, prefix, first, mult)
+        self.cap = float(mx["gate_cap"])
+        self._heads(mx, tp, 2 * mx["dim"] + 2 * mx["vdim"] + 2)
+
+    def parameters(self, device):
+        p = self.prefix
+        return {p + "i_b": _f32((self.H, ), 0.0, device), p + "f_b": _f32((self.H, ), 0.0, device),
+                p + "head_norm": _f32((self.H * self.dv, ), 1.0, device)}
+
+    def small(self, lw, r, tp):
+        p = self.prefix
+        s = (lambda t: _shard(t, r, tp)) if self.split else (lambda t: t)
+        return {p + "i_b": s(lw[p + "i_b"]), p + "f_b": s(lw[p + "f_b"]), p + "head_norm": s(lw[p + "head_norm"]).float() * self.mult}
+
+    def state_geometry(self, dtype):
+        dks = -(-self.dk // 8) * 8
+        return {**super().state_geometry(dtype), "norm": ((self.H, -(-self.dv // 32), dks), torch.float32),
+                "peak": ((self.H, ), torch.float32)}
+
+    def heads(self, layer, proj, meta, cache, carry, out):
+        w = self.weight
+        y = mixer_ops.matrix_memory(proj, mixer_ops.ScanLayout(rows=proj.shape[1], **self.at), cache.state[layer.layer_idx], meta,
+                                    self.gate + self.cols, w(layer, "i_b"), w(layer, "f_b"), self.cap, self.dk**-0.5)
+        mixer_ops.gated_norm(y, proj, self.gate, w(layer, "head_norm"), self.H, layer.spec.norm_eps, "sigmoid_after", out)
+
+
+class Retention(HeadScan):
+    kind = "retention"
+    sections = ("q_w", "k_w", "v_w", "g_w")
+
+    def __init__(self, mx, tp, prefix="", first=0, mult=1.0):
+        super().__init__(mx, tp, prefix, first, mult)
+        if mult != 1.0:
+            raise NotImplementedError("retention as a scaled side: it has no weight to take the factor")
+        if len(mx["decay"]) != mx["heads"]:
+            raise ValueError(f"{len(mx['decay'])} decays for {mx['heads']} heads")
+        self.decay, self.rot = [float(a) for a in mx["decay"]], Rotation(mx["rot"], mx["dim"])
+        self._heads(mx, tp, 2 * mx["dim"] + 2 * mx["vdim"])
+
+    def constants(self, device):
+        # (a decay of zero: its logarithm as a number whose exponential is zero)
+        return {self.prefix + "log_decay": torch.tensor([math.log(a) if a > 0 else -200.0 for a in self.decay], device=device),
+                self.prefix + "rot_freq": self.rot.frequencies(device)}
+
+    def heads(self, layer, proj, meta, cache, carry, out):
+        w = self.weight
+        ld = w(layer, "log_decay")
+        if self.H < len(self.decay):
+            ld = ld[layer.tp_rank * self.H:(layer.tp_rank + 1) * self.H]
+        y = mixer_ops.retention(proj, mixer_ops.ScanLayout(rows=proj.shape[1], **self.at), cache.state[layer.layer_idx]["state"],
+                                meta, ld, self.rot.angles(w(layer, "rot_freq"), meta, carry), self.dk**-0.5)
+        mixer_ops.gated_norm(y, proj, self.gate, None, self.H, layer.spec.norm_eps, "silu_after", out)
+
+
+class ParallelMixer(Mixer):
+    """Attention and a matrix memory on the same input: one fused input projection, read-outs side by side, one output
+    projection that sums them. At most one side keeps keys and values, at most one a state."""
+    kind = "parallel"
+    sides = (("left", RotaryAttention), ("right", MatrixMemory))
+
+    def __init__(self, mx, tp):
+        self.parts, self.rows, self.out_width = [], 0, 0
+        for name, cls in self.sides:
+            side = cls(mx[name], tp, name + "_", self.rows, mx[name + "_scale"])
+            self.parts.append(side)
+            self.rows += side.rows
+            self.out_width += side.out_width
+        self.extensions = tuple(e for s in self.parts for e in s.extensions)
+
+    def _all(self, f):
+        return {k: v for s in self.parts for k, v in f(s).items()}
+
+    def parameters(self, device):
+        return self._all(lambda s: s.parameters(device))
+
+    def constants(self, device):
+        return self._all(lambda s: s.constants(device))
+
+    def shard(self, lw, r, tp):
+        return {"qkv_w": torch.cat([s.project(lw, r, tp) for s in self.parts]),
+                "o_w": torch.cat([s.output(lw, r, tp) for s in self.parts], 1), **self._all(lambda s: s.small(lw, r, tp))}
+
+    def kv_geometry(self):
+        return next((g for g in (s.kv_geometry() for s in self.parts) if g), None)
+
+    def state_geometry(self, dtype):
+        return next((g for g in (s.state_geometry(dtype) for s in self.parts) if g), None)
+
+    def run(self, layer, h, meta, cache, carry):
+        proj = layer._linear(h, "qkv_w")
+        out, at = proj.new_empty(proj.shape[0], self.out_width), 0
+        for s in self.parts:
+            s.read_out(layer, proj, meta, cache, carry, out[:, at:at + s.out_width])
+            at += s.out_width
+        return out
+
+
+MIXERS = {m.kind: m for m in (AttentionMixer, LatentMixer, DeltaMixer, Mamba2Mixer, LightningMixer, RotaryAttention, MatrixMemory,
+                              Retention, ParallelMixer)}
+
+
+class MLP:
+    """What a feed-forward may leave at its default. `rows`: width of the first product's output; `ff`: of the second's input."""
+    projections = ("fc1_w", "fc2_w")   # weights that are quantised / re-laid
+    extensions = ()
+
+    def matrices(self, width):
+        """Shapes of the weight matrices, by name."""
+        return {"fc1_w": (self.rows, width), "fc2_w": (width, self.ff)}
+
+
+class ClampedMLP(MLP):
     """Gated feed-forward whose branches are clamped before the product."""
     kind = "dense"
+    extensions = ("ds_hybrid_ops", )
 
     def __init__(self, ml, tp):
         if ml["ff"] % tp:
@@ -394,9 +682,10 @@ class ClampedMLP:
         return layer._linear(mid, "fc2_w")
 
 
-class GeluMLP:
+class GeluMLP(MLP):
     """Feed-forward without a gate: down gelu(up x), the gelu of the error function."""
     kind = "gelu"
+    extensions = ("ds_mixer_ops", )
 
     def __init__(self, ml, tp):
         if ml["ff"] % tp:
@@ -414,7 +703,39 @@ class GeluMLP:
         return layer._linear(mid, "fc2_w")
 
 
-MLPS = {m.kind: m for m in (ClampedMLP, GeluMLP)}
+class RoutedMLP(MLP):
+    """Mixture of gated (silu) experts. The experts form equal groups; those of the best groups compete, the best are weighted
+    by their softmax over all, divided by its sum. Every rank routes for itself and holds a slice of every expert."""
+    kind = "routed"
+    projections = ()
+    extensions = ("ds_expert_ops", )
+
+    def __init__(self, ml, tp):
+        ro = ml["router"]
+        groups = ro.get("groups") or {}
+        self.E, self.top = int(ro["experts"]), int(ro["top"])
+        self.groups, self.keep = int(groups.get("count", 1)), int(groups.get("keep", 1))
+        if ml["expert"]["ff"] % tp:
+            raise ValueError(f"expert width {ml['expert']['ff']} over {tp} ranks")
+        if self.groups < 1 or self.E % self.groups or not 1 <= self.keep <= self.groups or \
+                not 1 <= self.top <= self.keep * (self.E // self.groups):
+            raise ValueError(f"{self.top} of {self.E} experts, {self.keep} of {self.groups} groups")
+        self.ff = ml["expert"]["ff"] // tp
+
+    def matrices(self, width):
+        return {"router_w": (self.E, width), "fc1_w": (self.E, 2 * self.ff, width), "fc2_w": (self.E, width, self.ff)}
+
+    def shard(self, lw, r, tp):
+        return {"router_w": lw["router_w"], "fc1_w": torch.cat([_shard(lw["experts_gate"], r, tp, 1),
+                                                                _shard(lw["experts_up"], r, tp, 1)], 1),
+                "fc2_w": _shard(lw["experts_down"], r, tp, 2)}
+
+    def run(self, layer, h):
+        y = expert_ops.experts(h, layer.router_w, layer.fc1_w, layer.fc2_w, self.top, self.groups, self.keep)
+        return y if layer.tp == 1 else y.sum()   # ranks exchange plain sums
+
+
+MLPS = {m.kind: m for m in (ClampedMLP, GeluMLP, RoutedMLP)}
 
 
 class TokenSide:
@@ -457,8 +778,8 @@ class DSHybridLayer(ProjectionLayer):
                 raise NotImplementedError(f"layer {layer_idx}: no feed-forward {kind!r}")
             self.mlp = MLPS[kind](ls["mlp"], tp_size)
             self.res2 = residual(spec.streams, W, device)
-            self.fc1_w = _empty((self.mlp.rows, W), dtype, device)
-            self.fc2_w = _empty((W, self.mlp.ff), dtype, device)
+            for name, shape in self.mlp.matrices(W).items():
+                self.register_parameter(name, _empty(shape, dtype, device))
         if spec.token_side:
             self.side = TokenSide(spec.token_side, layer_idx)
             self.res_side = residual(spec.streams, W, device)
@@ -466,7 +787,7 @@ class DSHybridLayer(ProjectionLayer):
             self.side_proj_w = _empty((W, spec.token_side), dtype, device)
 
     def projection_names(self):
-        return ("qkv_w", "o_w") + self.mixer.extra_projections + (("fc1_w", "fc2_w") if self.mlp else ()) + \
+        return ("qkv_w", "o_w") + self.mixer.extra_projections + (self.mlp.projections if self.mlp else ()) + \
             (("side_gate_w", "side_proj_w") if self.side else ())
 
     def _linear(self, x, name, bias=None):
@@ -516,6 +837,9 @@ class DSHybridModel(DSInferenceModel):
 
     def __init__(self, spec, tp_group=None, tp_size=1, tp_rank=0, dtype=torch.bfloat16, device=None):
         super().__init__(spec, tp_group, tp_size, tp_rank, dtype, device)
+        if torch.device(device or "cpu").type == "cuda":  # all at once: in a fresh checkout they compile side by side
+            parts = [p for la in self.layers for p in (la.mixer, la.mlp) if p]
+            op_builder.prepare(sorted({"ds_gemv_ops", *(e for p in parts for e in p.extensions)}))
         self.norm_w = _f32((spec.hidden_size, ), 1.0, device)  # norms read the fp32 residual
         if spec.token_side:
             self.side_embed = _empty((spec.vocab_size, spec.token_side * spec.num_layers), dtype, device)

@@ -68,9 +68,11 @@ class DSModelSpec:
     layer_specs: tuple = ()
     streams: int = 1                 # residual streams (hyper-connections)
     residual_mult: float = 1.0       # factor of every sublayer's output
-    residual: str = "streams"        # "streams" (pre-norm over the streams) | "post_norm" (norms on sublayer outputs)
+    residual: str = "streams"        # "streams" (pre-norm over the streams) | "post_norm" (norms on sublayer outputs) |
+                                     # "pre_norm" (one fp32 residual, RMS norms on sublayer inputs)
     token_side: int = 0              # width of a side embedding per layer and token (0: none)
     logit_scale: float = 1.0
+    embed_scale: float = 1.0         # factor of the embedding rows ("pre_norm" residual)
 
     def __post_init__(self):
         if not self.head_dim:

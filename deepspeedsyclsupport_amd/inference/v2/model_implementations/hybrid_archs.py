@@ -3,11 +3,15 @@ config.json + model.safetensors in this package's own layout, with the layers li
 
 A layer's container is assembled from the tensors its kind has: the mixer's, the feed-forward's if it has one, the
 norms and, for models with residual streams, the mixing matrices."""
-from ...model_implementations.hybrid import DSHybridModel
+from types import SimpleNamespace
+
+import torch
+
+from ...model_implementations.hybrid import DSHybridModel, ParallelMixer
 from ...model_implementations.transformer import DSModelSpec
 from .inference_policy_base import ContainerMap, InferenceV2Policy, register
 from .layer_container_base import LayerContainer
-from .parameter_base import single
+from .parameter_base import ParamList, ParameterBase, single
 
 _MIXER_TENSORS = {  # checkpoint name below `<layer>.mix.` -> canonical key
     "attention": {"q": "q_w", "k": "k_w", "v": "v_w", "o": "o_w", "q.norm": "q_norm", "k.norm": "k_norm"},
@@ -18,8 +22,17 @@ _MIXER_TENSORS = {  # checkpoint name below `<layer>.mix.` -> canonical key
     "mamba2": {"in": "in_w", "conv": "conv_w", "conv.b": "conv_b", "dt_bias": "dt_bias", "A_log": "a_log", "D": "skip",
                "norm": "head_norm", "o": "o_w"},
     "lightning": {"q": "q_w", "k": "k_w", "v": "v_w", "g": "g_w", "o": "o_w", "norm": "head_norm"},
+    "rotary_attention": {"q": "q_w", "k": "k_w", "v": "v_w", "q.b": "q_b", "k.b": "k_b", "v.b": "v_b", "q.norm": "q_norm",
+                         "k.norm": "k_norm", "o": "o_w"},
+    "matrix_memory": {"q": "q_w", "k": "k_w", "v": "v_w", "g": "g_w", "i": "i_w", "i.b": "i_b", "f": "f_w", "f.b": "f_b",
+                      "norm": "head_norm", "o": "o_w"},
+    "retention": {"q": "q_w", "k": "k_w", "v": "v_w", "g": "g_w", "o": "o_w"},
 }
-_MLP_TENSORS = {"dense": {"gate": "gate_w", "up": "up_w", "down": "down_w"}, "gelu": {"up": "up_w", "down": "down_w"}}
+_MIXER_TENSORS["parallel"] = {f"{side}.{n}": f"{side}_{key}" for side, cls in ParallelMixer.sides
+                              for n, key in _MIXER_TENSORS[cls.kind].items()}
+_MLP_TENSORS = {"dense": {"gate": "gate_w", "up": "up_w", "down": "down_w"}, "gelu": {"up": "up_w", "down": "down_w"},
+                "routed": {"router": "router_w"}}
+_EXPERT_TENSORS = {"gate": "experts_gate", "up": "experts_up", "down": "experts_down"}
 _SIDE_TENSORS = {"side.gate": "side_gate_w", "side.proj": "side_proj_w", "side.norm": "side_norm_w"}
 
 
@@ -35,11 +48,29 @@ class _HybridContainer(LayerContainer):
         return [name for name, p in self._params.items() if not p.complete and name not in self.may_lack]
 
 
-def container(name, tensors, may_lack=()):
-    """A container class for {checkpoint tensor: canonical key}."""
-    return type(name, (_HybridContainer, ), {"__annotations__": {key: single(key) for key in tensors.values()},
-                                             "PARAM_MAPPING": {src: f"{key}.params" for src, key in tensors.items()},
-                                             "may_lack": may_lack})
+def _stacked(key, count):
+    """A parameter of `count` tensors that are stacked under `key`."""
+
+    class _Stacked(ParameterBase):
+        params: ParamList("count")
+
+        def __init__(self, model=None, name=None):
+            super().__init__(SimpleNamespace(count=count), name)
+
+        def finalize(self):
+            return {key: torch.stack(list(self.params))}
+
+    return _Stacked
+
+
+def container(name, tensors, may_lack=(), stacked=None, count=0):
+    """A container class for {checkpoint tensor: canonical key}; `stacked`: the same for lists of `count` tensors, the index
+    being the `*` of the name."""
+    lists = stacked or {}
+    return type(name, (_HybridContainer, ), {
+        "__annotations__": {**{key: single(key) for key in tensors.values()}, **{key: _stacked(key, count)
+                                                                                for key in lists.values()}},
+        "PARAM_MAPPING": {src: f"{key}.params" for src, key in {**tensors, **lists}.items()}, "may_lack": may_lack})
 
 
 def layer_container(layer, streams=False, may_lack=(), side=False):
@@ -47,11 +78,14 @@ def layer_container(layer, streams=False, may_lack=(), side=False):
     if layer["type"] not in _MIXER_TENSORS:
         raise NotImplementedError(f"no mixer {layer['type']!r}")
     tensors = {f"mix.{n}": key for n, key in _MIXER_TENSORS[layer["type"]].items()}
+    lists, count = {}, 0
     if layer["mixer"].get("v_mix"):
         tensors["mix.vmix"] = "vmix"
     if layer.get("mlp"):
         if layer["mlp"].get("kind") not in _MLP_TENSORS:
             raise NotImplementedError(f"no feed-forward {layer['mlp'].get('kind')!r}")
+        if layer["mlp"]["kind"] == "routed":
+            lists, count = {f"mlp.e*.{n}": key for n, key in _EXPERT_TENSORS.items()}, layer["mlp"]["router"]["experts"]
         tensors.update({f"mlp.{n}": key for n, key in _MLP_TENSORS[layer["mlp"]["kind"]].items()})
     for q in (1, 2) if layer.get("mlp") else (1, ):
         tensors[f"norm{q}"] = f"norm{q}_w"
@@ -59,11 +93,18 @@ def layer_container(layer, streams=False, may_lack=(), side=False):
             tensors.update({f"hc{q}.{n}": f"hc{q}_{n}" for n in ("in", "out", "mix")})
     if side:
         tensors.update(_SIDE_TENSORS)
-    return container("HybridLayerContainer", tensors, may_lack)
+    return container("HybridLayerContainer", tensors, may_lack, lists, count)
+
+
+def _renamed(layers, kinds):
+    """A config's layers with its names of feed-forwards replaced by the package's."""
+    return [{**la, "mlp": {**la["mlp"], "kind": kinds.get(la["mlp"].get("kind"), la["mlp"].get("kind"))}
+             if la.get("mlp") else None} for la in layers]
 
 
 _TOP_TENSORS = {"embed": "embed", "final.norm": "norm_w", "head": "lm_head"}
 TopContainer = container("HybridTopContainer", _TOP_TENSORS)
+TiedTopContainer = container("HybridTiedTopContainer", {n: k for n, k in _TOP_TENSORS.items() if k != "lm_head"})
 SideTopContainer = container("HybridSideTopContainer", {**_TOP_TENSORS, "side.embed": "side_embed"})
 
 
@@ -105,8 +146,7 @@ class PerelornPolicy(InferenceV2Policy):
 
     def layers(self):
         """The config's layers in the spec's terms: its "dense" feed-forward is the ungated gelu one."""
-        return [{**la, "mlp": {**la["mlp"], "kind": {"dense": "gelu"}.get(la["mlp"].get("kind"), la["mlp"].get("kind"))}
-                 if la.get("mlp") else None} for la in self._model_config.layers]
+        return _renamed(self._model_config.layers, {"dense": "gelu"})
 
     def spec(self):
         c = self._model_config
@@ -121,4 +161,32 @@ class PerelornPolicy(InferenceV2Policy):
         cmap = ContainerMap()
         cmap.set_transformer_params("l", [layer_container(la, side=True)(self._view) for la in self.layers()], sep="")
         cmap.set_non_transformer_params(SideTopContainer(self._view))
+        return cmap
+
+
+@register
+class LefisunPolicy(InferenceV2Policy):
+    """Lefisun: retention layers and layers of chunked rotary attention beside a matrix memory, routed experts, one fp32 residual
+    with norms on the sublayers' inputs, the embedding table as output."""
+    model_types = ("lefisun", )
+    model_class = DSHybridModel
+
+    def layers(self):
+        """The config's layers in the spec's terms."""
+        return _renamed(self._model_config.layers, {"moe": "routed"})
+
+    def spec(self):
+        c, layers = self._model_config, self.layers()
+        first = next((la["mixer"]["left"] for la in layers if la["type"] == "parallel"), layers[0]["mixer"])
+        return DSModelSpec(arch="lefisun", vocab_size=c.vocab, hidden_size=c.width, num_layers=len(c.layers),
+                           num_heads=first["heads"], num_kv_heads=first.get("kv_heads", first["heads"]), head_dim=first["dim"],
+                           intermediate_size=max([la["mlp"]["expert"]["ff"] for la in layers if la["mlp"] and "expert" in
+                                                  la["mlp"]], default=0),
+                           norm="rms", norm_eps=float(c.norm["eps"]), pos="none", tie_embeddings=True,
+                           layer_specs=tuple(layers), residual="pre_norm", embed_scale=float(c.embedding["scale"]))
+
+    def build_container_map(self):
+        cmap = ContainerMap()
+        cmap.set_transformer_params("l", [layer_container(la)(self._view) for la in self.layers()], sep="")
+        cmap.set_non_transformer_params(TiedTopContainer(self._view))
         return cmap

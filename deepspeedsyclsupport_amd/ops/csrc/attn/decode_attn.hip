@@ -14,7 +14,7 @@
 //    last-block merge was measured 2x slower: the device-scope fences it needs write back L2.)
 // Optional ALiBi slopes (BLOOM) are applied on the fly. With a sliding window (Mistral) or chunked visibility only the
 // keys in sight are split and read. A second instantiation takes key and value widths of their own (multiples of 8), a
-// tanh score cap and GQA groups of any size.
+// tanh score cap, a softmax sink per head and GQA groups of any size.
 #include "../include/ds_hip.h"
 
 namespace {
@@ -37,8 +37,8 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
     const float* __restrict__ alibi,     // [Hq] or null
     float* __restrict__ part_acc,        // [B, Hq, S, dv]  (only if S > 1)
     float* __restrict__ part_ml,         // [B, Hq, S, 2]
-    bf16* __restrict__ out,              // [B, Hq, dv]  (written directly when S == 1)
-    int Hq, int Hk, int BS, int max_blocks, int chunk, float scale, int window, int mask_chunk, float softcap, int dk_rt,
+    bf16* __restrict__ out,              // [B, Hq, dv], rows ldo apart (written directly when S == 1)
+    const float* __restrict__ sink, int64_t ldo, int Hq, int Hk, int BS, int max_blocks, int chunk, float scale, int window, int mask_chunk, float softcap, int dk_rt,
     int dv_rt) {
   constexpr bool EXT = DK == 0;
   static_assert(EXT || (DK % 16 == 0 && DK >= 64 && DK <= 256 && DK == DV), "head dim");
@@ -187,7 +187,12 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
       const int hq = h0 + g;
       const float m = red[g * 2], l = red[g * 2 + 1];
       if (S == 1) {
-        out[((int64_t)b * Hq + hq) * dv + idx] = (bf16)(l > 0.f ? s / l : 0.f);
+        float r = l > 0.f ? s / l : 0.f;
+        if (EXT && sink) {  // in the frame of the larger of the two
+          const float mn = fmaxf(m, sink[hq]), f = __expf(m - mn);
+          r = s * f / fmaf(l, f, __expf(sink[hq] - mn));
+        }
+        out[(int64_t)b * ldo + hq * dv + idx] = (bf16)r;
       } else {
         part_acc[(((int64_t)b * Hq + hq) * S + split) * dv + idx] = s;
         if (idx == 0) {
@@ -202,11 +207,13 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
 
 // blockDim.x = D, the value width
 __global__ void __launch_bounds__(256) combine_kernel(const float* __restrict__ part_acc,
-                                                      const float* __restrict__ part_ml, bf16* __restrict__ out, int S) {
+                                                      const float* __restrict__ part_ml, bf16* __restrict__ out,
+                                                      const float* __restrict__ sink, int Hq, int64_t ldo, int S) {
   const int bh = blockIdx.x, d = threadIdx.x, D = blockDim.x;
-  float M = -INFINITY;
+  const float sk = sink ? sink[bh % Hq] : -INFINITY;
+  float M = sk;
   for (int s = 0; s < S; ++s) M = fmaxf(M, part_ml[((int64_t)bh * S + s) * 2]);
-  float num = 0.f, den = 0.f;
+  float num = 0.f, den = sink ? __expf(sk - M) : 0.f;
   for (int s = 0; s < S; ++s) {
     const float m = part_ml[((int64_t)bh * S + s) * 2], l = part_ml[((int64_t)bh * S + s) * 2 + 1];
     if (m == -INFINITY) continue;
@@ -214,7 +221,7 @@ __global__ void __launch_bounds__(256) combine_kernel(const float* __restrict__ 
     num = fmaf(w, part_acc[((int64_t)bh * S + s) * D + d], num);
     den = fmaf(w, l, den);
   }
-  out[(int64_t)bh * D + d] = (bf16)(den > 0.f ? num / den : 0.f);
+  out[bh / Hq * ldo + bh % Hq * D + d] = (bf16)(den > 0.f ? num / den : 0.f);
 }
 
 // Write new K/V rows into the paged cache: k,v [B, n_new, Hk, D] token-major; positions start at seq_lens_before[b].
@@ -334,11 +341,13 @@ extern "C" int ds_paged_decode(const void* q, const void* kc, const void* vc, co
   dim3 grid(B, Hk, splits);
 #define LAUNCH(DD)                                                                                                  \
   hipLaunchKernelGGL((paged_decode_kernel<DD, DD>), grid, dim3(THREADS), lds, s, (const bf16*)q, (const bf16*)kc,       \
-                     (const bf16*)vc, block_table, seq_lens, alibi, part_acc, part_ml, (bf16*)out, Hq, Hk, BS,       \
+                     (const bf16*)vc, block_table, seq_lens, alibi, part_acc, part_ml, (bf16*)out, nullptr,          \
+                     (int64_t)Hq * DD, Hq, Hk, BS,                                                                   \
                      max_blocks, chunk, scale, window, 0, 0.f, DD, DD);                                             \
   DS_CHECK_LAUNCH();                                                                                                \
   if (splits > 1) {                                                                                                 \
-    hipLaunchKernelGGL(combine_kernel, dim3(B * Hq), dim3(DD), 0, s, part_acc, part_ml, (bf16*)out, splits);  \
+    hipLaunchKernelGGL(combine_kernel, dim3(B * Hq), dim3(DD), 0, s, part_acc, part_ml, (bf16*)out, nullptr, Hq, \
+                       (int64_t)Hq * DD, splits);                                                                     \
     DS_CHECK_LAUNCH();                                                                                              \
   }
   if (D == 64) { LAUNCH(64) }
@@ -351,13 +360,15 @@ extern "C" int ds_paged_decode(const void* q, const void* kc, const void* vc, co
   return 0;
 }
 
-// Key / value widths of their own (multiples of 8 up to 256), chunked and / or windowed visibility, score cap. `splits`
+// Key / value widths of their own (multiples of 8 up to 256), chunked and / or windowed visibility, score cap, softmax sink
+// [Hq] (or null), rows of out ldo elements apart. `splits`
 // from ds_paged_decode_splits(B, Hk, span) with span = the most keys in sight.
 extern "C" int ds_paged_decode_ext(const void* q, const void* kc, const void* vc, const int* block_table,
                                    const int* seq_lens, float* part_acc, float* part_ml, void* out, int B, int Hq, int Hk,
                                    int dk, int dv, int BS, int max_blocks, int span, int splits, float scale,
-                                   float softcap, int window, int mask_chunk, hipStream_t s) {
-  if (Hk <= 0 || Hq % Hk || dk % 8 || dv % 8 || dk <= 0 || dv <= 0 || dk > 256 || dv > 256 || splits <= 0)
+                                   float softcap, int window, int mask_chunk, const float* sink, int64_t ldo, hipStream_t s) {
+  if (Hk <= 0 || Hq % Hk || dk % 8 || dv % 8 || dk <= 0 || dv <= 0 || dk > 256 || dv > 256 || splits <= 0 ||
+      ldo < (int64_t)Hq * dv)
     return (int)hipErrorInvalidValue;
   const int chunk = ((span + splits - 1) / splits + 63) / 64 * 64;
   if (chunk > MAX_CHUNK) return (int)hipErrorInvalidValue;
@@ -366,7 +377,7 @@ extern "C" int ds_paged_decode_ext(const void* q, const void* kc, const void* vc
   dim3 grid(B, Hk * ((Hq / Hk + MAXG - 1) / MAXG), splits);
 #define GO(LK, LV)                                                                                                  \
   hipLaunchKernelGGL((paged_decode_kernel<0, 0, LK, LV>), grid, dim3(THREADS), lds, s, (const bf16*)q, (const bf16*)kc, \
-                     (const bf16*)vc, block_table, seq_lens, nullptr, part_acc, part_ml, (bf16*)out, Hq, Hk, BS,     \
+                     (const bf16*)vc, block_table, seq_lens, nullptr, part_acc, part_ml, (bf16*)out, sink, ldo, Hq, Hk, BS,     \
                      max_blocks, chunk, scale, window, mask_chunk, softcap, dk, dv)
 #define ROW(LK)                 \
   {                             \
@@ -381,7 +392,7 @@ extern "C" int ds_paged_decode_ext(const void* q, const void* kc, const void* vc
 #undef GO
   DS_CHECK_LAUNCH();
   if (splits > 1) {
-    hipLaunchKernelGGL(combine_kernel, dim3(B * Hq), dim3(dv), 0, s, part_acc, part_ml, (bf16*)out, splits);
+    hipLaunchKernelGGL(combine_kernel, dim3(B * Hq), dim3(dv), 0, s, part_acc, part_ml, (bf16*)out, sink, Hq, ldo, splits);
     DS_CHECK_LAUNCH();
   }
   return 0;

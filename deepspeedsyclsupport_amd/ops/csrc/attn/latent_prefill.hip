@@ -34,6 +34,7 @@ extern "C" int ds_latent_prefill(const void* q, const void* kv, const void* ctx,
   a.ldk = H * (dn + dv);
   a.ldr = ldr;
   a.rot0 = rot0;
+  a.ldo = (int64_t)H * dv;
 #define DS_ROW(K)                                               \
   {                                                             \
     if (dv <= 32) return launch<K, 32, LATENT>(a, nwork, st);   \

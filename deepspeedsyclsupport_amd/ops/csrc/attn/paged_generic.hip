@@ -17,7 +17,7 @@ __global__ void __launch_bounds__(64) paged_generic_kernel(
     const T* __restrict__ q, const T* __restrict__ kc, const T* __restrict__ vc, T* __restrict__ o,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ pos, const int* __restrict__ seq_ids,
     int H, int G, int dk, int dv, int vrow, int BS, float scale, float softcap, int window, int chunk,
-    const float* __restrict__ sink) {
+    const float* __restrict__ sink, int64_t ldo) {
   __shared__ float qs[MAXD];
   __shared__ float ps[64];
   __shared__ int64_t slot_s[64];
@@ -67,7 +67,7 @@ __global__ void __launch_bounds__(64) paged_generic_kernel(
 #pragma unroll
     for (int i = 0; i < MAXD / 64; ++i) acc[i] *= alpha;
   }
-  T* orow = o + ((int64_t)t * H + h) * dv;
+  T* orow = o + t * ldo + h * dv;
 #pragma unroll
   for (int i = 0; i < MAXD / 64; ++i) {
     const int c = i * 64 + lane;
@@ -79,15 +79,16 @@ __global__ void __launch_bounds__(64) paged_generic_kernel(
 
 extern "C" int ds_paged_generic(const void* q, const void* kc, const void* vc, void* o, const int* bt, int max_blocks,
                                 const int* pos, const int* seq_ids, int tokens, int H, int G, int dk, int dv, int vrow,
-                                int BS, float scale, float softcap, int window, int chunk, const float* sink, int dtype,
-                                hipStream_t st) {
+                                int BS, float scale, float softcap, int window, int chunk, const float* sink, int64_t ldo,
+                                int dtype, hipStream_t st) {
   if (tokens <= 0) return 0;
-  if (G <= 0 || H % G || dk <= 0 || dv <= 0 || vrow < dv || dk > MAXD || dv > MAXD || BS <= 0 || H > 65535)
+  if (G <= 0 || H % G || dk <= 0 || dv <= 0 || vrow < dv || dk > MAXD || dv > MAXD || BS <= 0 || H > 65535 ||
+      ldo < (int64_t)H * dv)
     return (int)hipErrorInvalidValue;
 #define GO(T)                                                                                                        \
   hipLaunchKernelGGL((paged_generic_kernel<T>), dim3(tokens, H), dim3(64), 0, st, (const T*)q, (const T*)kc,         \
                      (const T*)vc, (T*)o, bt, max_blocks, pos, seq_ids, H, G, dk, dv, vrow, BS, scale, softcap, window, chunk, \
-                     sink)
+                     sink, ldo)
   if (dtype == DS_F32) GO(float);
   else if (dtype == DS_BF16) GO(bf16);
   else return (int)hipErrorInvalidValue;

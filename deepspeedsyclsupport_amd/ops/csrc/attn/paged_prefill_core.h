@@ -66,7 +66,7 @@ struct PagedArgs {
   const bf16* q;          // [T, Hq, D]
   const bf16* kc;         // [blocks, Hk, BS, D]
   const bf16* vc;
-  bf16* o;                // [T, Hq, D]
+  bf16* o;                // [T, Hq, D], ldo elements from row to row
   const int* block_table; // [nseq, max_blocks]
   const int* start;       // [nseq] cached tokens before this step
   const int* cu_q;        // [nseq + 1] token offsets of each sequence's new tokens
@@ -80,6 +80,7 @@ struct PagedArgs {
   const int* kv_offs;     // LATENT: first context row of sequence `first`, and of the ones after it
   int first, dn, ldk, ldr, rot0;  // key columns of a head (the rest is rotated), row lengths of kc and of vc, first rotated
                           // column there; kc: the expanded rows, vc: the latents' rows
+  int64_t ldo;            // elements from a token's row of o to the next one's
   float cap_in, cap_out;  // EXT: capped score in log2 units = cap_out * tanh(score * cap_in); cap_out 0: no cap
 };
 
@@ -397,7 +398,7 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
   for (int r = 0; r < 16; ++r) {
     const int qi = q0w + (r & 3) + 8 * (r >> 2) + 4 * h;
     if (qi < n) {
-      bf16* orow = a.o + ((int64_t)(t0 + qi) * a.Hq + hq) * dv + l32;
+      bf16* orow = a.o + (int64_t)(t0 + qi) * a.ldo + hq * dv + l32;
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt)
         if ((!EXT && DV % 32 == 0) || dt * 32 + l32 < dv) orow[dt * 32] = (bf16)(o[dt][r] * iv[r]);

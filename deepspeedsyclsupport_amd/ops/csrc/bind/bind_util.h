@@ -31,4 +31,15 @@ const int* i32(const Tensor& t, int64_t n, const char* name) {
   return t.data_ptr<int>();
 }
 bool has(const OptT& t) { return t.has_value() && t->defined(); }
+[[maybe_unused]] const float* opt_f32(const OptT& t, int64_t n, const char* name) { return has(t) ? f32(*t, n, name) : nullptr; }
+[[maybe_unused]] const double* f64(const Tensor& t, const char* name) {
+  need(t, name);
+  TORCH_CHECK(t.scalar_type() == at::kDouble, name, ": fp64");
+  return t.data_ptr<double>();
+}
+// A matrix whose rows may lie further apart than they are wide
+[[maybe_unused]] void need_rows(const Tensor& t, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.stride(1) == 1 && (t.size(0) <= 1 || t.stride(0) >= t.size(1)), name,
+              " must be a device matrix with contiguous rows");
+}
 }  // namespace

@@ -1,16 +1,11 @@
-// Module of the hybrid decoder's ops: multi-stream residual + norm, QKV epilogue with per-head norms, ragged paged
-// attention with chunked / windowed visibility and score capping, gated delta rule, clamped gated activation. A shared
-// object of its own, so that serving such a model compiles only this and the decode products (gemv_bind.cpp).
+// Module of the ops that only models with residual streams use: multi-stream residual + norm, gated delta rule, clamped
+// gated activation. A shared object of its own, so that serving a model compiles the mechanisms it has and no others.
 #include "bind_util.h"
 
 extern "C" {
 int ds_stream_norm(float*, const void*, const int*, const void*, const int*, int, int, const float*, const float*, float,
                    const float*, const float*, void*, int, float, int, hipStream_t);
 int ds_clamped_glu(const void*, void*, int64_t, int, float, float, float, int, hipStream_t);
-int ds_qk_norm_append(const void*, const float*, const float*, float, const void*, int64_t, const float*, const int*,
-                      const int*, const int*, int, void*, void*, void*, int, int, int, int, int, int, int, hipStream_t);
-int ds_paged_generic(const void*, const void*, const void*, void*, const int*, int, const int*, const int*, int, int, int,
-                     int, int, int, int, float, float, int, int, const float*, int, hipStream_t);
 int ds_delta_prepare(const void*, const float*, const void*, const float*, const float*, const int*, const int*,
                      const int*, const int*, float*, void*, float*, int, int, int, int, int, int, int, hipStream_t);
 int ds_delta_recur(const float*, const void*, const float*, const void*, const float*, float, float*, void*, const int*,
@@ -19,11 +14,6 @@ int64_t ds_delta_chunk_ws(int, int, int, int);
 int ds_delta_chunk(const float*, const void*, const float*, const void*, const float*, float, float*, void*, const int*,
                    int, const int*, int, const int*, const int*, const int*, float*, float*, void*, int, int, int, int,
                    int, int, int, hipStream_t);
-int ds_paged_prefill_ext(const void*, const void*, const void*, void*, const int*, const int*, const int*, const int*, int,
-                         int, int, int, int, int, int, int, int, float, float, hipStream_t);
-int ds_paged_decode_splits(int, int, int);
-int ds_paged_decode_ext(const void*, const void*, const void*, const int*, const int*, float*, float*, void*, int, int,
-                        int, int, int, int, int, int, int, float, float, int, int, hipStream_t);
 }
 
 namespace {
@@ -73,111 +63,6 @@ Tensor clamped_glu(Tensor gu, double limit, double alpha, double shift) {
   check(ds_clamped_glu(gu.data_ptr(), out.data_ptr(), rows, (int)F, (float)limit, (float)alpha, (float)shift, dcode(gu),
                        stream()), "clamped_glu");
   return out;
-}
-
-struct Cache {
-  int G, BS, dk, dv;
-};
-Cache cache_of(const Tensor& kc, const Tensor& vc) {
-  need(kc, "k cache"); need(vc, "v cache");
-  TORCH_CHECK(kc.dim() == 4 && vc.dim() == 4 && kc.size(0) == vc.size(0) && kc.size(1) == vc.size(1) &&
-              kc.size(2) == vc.size(2) && kc.scalar_type() == vc.scalar_type(), "caches [NB, G, BS, dk / dv]");
-  return {(int)kc.size(1), (int)kc.size(2), (int)kc.size(3), (int)vc.size(3)};
-}
-
-// qkv [T, (H + G) dk + G dv] -> q [T, H, dk]; k / v into the caches. vfirst: the same-shaped v columns [T, G dv] (row
-// stride free) of an earlier layer, mixed in with weight `lam` [1].
-Tensor qk_norm_append(Tensor qkv, Tensor qw, Tensor kw, double eps, OptT vfirst, OptT lam, Tensor pos, Tensor seq_ids,
-                      Tensor block_table, Tensor kc, Tensor vc, int64_t H) {
-  need(qkv, "qkv"); need(block_table, "block_table");
-  const Cache c = cache_of(kc, vc);
-  const int64_t N = (H + c.G) * c.dk + (int64_t)c.G * c.dv, T = qkv.numel() / N;
-  TORCH_CHECK(qkv.numel() == T * N && qkv.size(-1) == N, "qk_norm_append: qkv width");
-  TORCH_CHECK(qkv.scalar_type() == kc.scalar_type(), "qk_norm_append: projection and cache types differ");
-  TORCH_CHECK(block_table.dim() == 2 && block_table.scalar_type() == at::kInt, "block_table [S, M] int32");
-  const void* vf = nullptr;
-  int64_t vs = 0;
-  const float* lp = nullptr;
-  if (has(vfirst)) {
-    TORCH_CHECK(vfirst->is_cuda() && vfirst->dim() == 2 && vfirst->size(0) == T && vfirst->size(1) == (int64_t)c.G * c.dv &&
-                vfirst->stride(1) == 1 && vfirst->scalar_type() == qkv.scalar_type(), "vfirst [T, G dv]");
-    vf = vfirst->data_ptr();
-    vs = vfirst->stride(0);
-    lp = f32(*lam, 1, "lambda");
-  }
-  auto q = torch::empty({T, H, c.dk}, qkv.options());
-  check(ds_qk_norm_append(qkv.data_ptr(), f32(qw, c.dk, "q norm"), f32(kw, c.dk, "k norm"), (float)eps, vf, vs, lp,
-                          i32(pos, T, "pos"), i32(seq_ids, T, "seq_ids"), block_table.data_ptr<int>(),
-                          (int)block_table.size(1), q.data_ptr(), kc.data_ptr(), vc.data_ptr(), (int)T, (int)H, c.G, c.dk,
-                          c.dv, c.BS, dcode(qkv), stream()), "qk_norm_append");
-  return q;
-}
-
-// q [T, H, dk] at positions pos of sequences seq_ids -> o [T, H, dv]
-Tensor paged_generic(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor pos, Tensor seq_ids, double scale,
-                     double softcap, int64_t window, int64_t chunk) {
-  need(q, "q"); need(block_table, "block_table");
-  const Cache c = cache_of(kc, vc);
-  const int64_t T = q.size(0), H = q.size(1);
-  TORCH_CHECK(q.dim() == 3 && q.size(2) == c.dk && H % c.G == 0 && q.scalar_type() == kc.scalar_type(), "paged_generic: q");
-  TORCH_CHECK(block_table.dim() == 2 && block_table.scalar_type() == at::kInt, "block_table [S, M] int32");
-  TORCH_CHECK(c.dk <= 1024 && c.dv <= 1024, "paged_generic: head sizes up to 1024");
-  auto o = torch::empty({T, H, c.dv}, q.options());
-  check(ds_paged_generic(q.data_ptr(), kc.data_ptr(), vc.data_ptr(), o.data_ptr(), block_table.data_ptr<int>(),
-                         (int)block_table.size(1), i32(pos, T, "pos"), i32(seq_ids, T, "seq_ids"), (int)T, (int)H, c.G,
-                         c.dk, c.dv, c.dv, c.BS, (float)scale, (float)softcap, (int)window, (int)chunk, nullptr, dcode(q),
-                         stream()), "paged_generic");
-  return o;
-}
-
-bool paged_tiled_ok(int64_t dk, int64_t dv) { return dk % 8 == 0 && dv % 8 == 0 && dk <= 256 && dv <= 256; }
-
-// Prompts and portions: q [T, H, dk] bf16 of every new token; work [n, 2] names (sequence, 128-row block) -> o [T, H, dv]
-// (rows of sequences the list leaves out are not written).
-Tensor paged_prefill(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor start, Tensor cu_q, Tensor work,
-                     double scale, double softcap, int64_t window, int64_t chunk) {
-  need(q, "q"); need(block_table, "block_table");
-  const Cache c = cache_of(kc, vc);
-  const int64_t T = q.size(0), H = q.size(1), S = start.numel();
-  TORCH_CHECK(q.dim() == 3 && q.size(2) == c.dk && H % c.G == 0 && q.scalar_type() == at::kBFloat16 &&
-              kc.scalar_type() == at::kBFloat16 && paged_tiled_ok(c.dk, c.dv), "paged_prefill: q / caches");
-  TORCH_CHECK(block_table.dim() == 2 && block_table.size(0) == S && block_table.scalar_type() == at::kInt, "block_table");
-  TORCH_CHECK(work.dim() == 2 && work.size(1) == 2 && scale > 0, "paged_prefill: work [n, 2], scale > 0");
-  auto o = torch::empty({T, H, c.dv}, q.options());
-  check(ds_paged_prefill_ext(q.data_ptr(), kc.data_ptr(), vc.data_ptr(), o.data_ptr(), block_table.data_ptr<int>(),
-                             i32(start, S, "start"), i32(cu_q, S + 1, "cu_q"), i32(work, work.numel(), "work"),
-                             (int)work.size(0), (int)H, c.G, c.dk, c.dv, c.BS, (int)block_table.size(1), (int)window,
-                             (int)chunk, (float)scale, (float)softcap, stream()), "paged_prefill");
-  return o;
-}
-
-// One new token per sequence: q [B, H, dk] bf16, the first B rows of the tables -> out[:B] of [.., H, dv]
-void paged_decode(Tensor q, Tensor kc, Tensor vc, Tensor block_table, Tensor seq_lens, int64_t max_len, double scale,
-                  double softcap, int64_t window, int64_t chunk, Tensor out) {
-  need(q, "q"); need(block_table, "block_table"); need(out, "out");
-  const Cache c = cache_of(kc, vc);
-  const int64_t B = q.size(0), H = q.size(1);
-  TORCH_CHECK(q.dim() == 3 && q.size(2) == c.dk && H % c.G == 0 && q.scalar_type() == at::kBFloat16 &&
-              kc.scalar_type() == at::kBFloat16 && paged_tiled_ok(c.dk, c.dv), "paged_decode: q / caches");
-  TORCH_CHECK(block_table.dim() == 2 && block_table.size(0) >= B && block_table.scalar_type() == at::kInt &&
-              block_table.size(1) * c.BS >= max_len, "block_table");
-  TORCH_CHECK(out.dim() == 3 && out.size(0) >= B && out.size(1) == H && out.size(2) == c.dv &&
-              out.scalar_type() == at::kBFloat16, "paged_decode: out");
-  int64_t span = max_len;
-  if (window > 0) span = std::min(span, window);
-  if (chunk > 0) span = std::min(span, chunk);
-  const int splits = ds_paged_decode_splits((int)B, c.G, (int)span);
-  Tensor acc, ml;
-  if (splits > 1) {
-    auto fo = q.options().dtype(at::kFloat);
-    acc = torch::empty({B, H, splits, c.dv}, fo);
-    ml = torch::empty({B, H, splits, 2}, fo);
-  }
-  check(ds_paged_decode_ext(q.data_ptr(), kc.data_ptr(), vc.data_ptr(), block_table.data_ptr<int>(),
-                            i32(seq_lens, seq_lens.numel(), "seq_lens"), splits > 1 ? acc.data_ptr<float>() : nullptr,
-                            splits > 1 ? ml.data_ptr<float>() : nullptr, out.data_ptr(), (int)B, (int)H, c.G, c.dk, c.dv,
-                            c.BS, (int)block_table.size(1), (int)span, splits, (float)scale, (float)softcap, (int)window,
-                            (int)chunk, stream()), "paged_decode");
 }
 
 void delta_dims_ok(int64_t Hk, int64_t H, int64_t dk, int64_t dv, int64_t taps) {
@@ -261,12 +146,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("in_"), py::arg("w"), py::arg("eps"), py::arg("ids") = py::none(), py::arg("embed") = py::none(),
         py::arg("rows") = py::none());
   m.def("clamped_glu", &clamped_glu);
-  m.def("qk_norm_append", &qk_norm_append);
-  m.def("paged_generic", &paged_generic);
   m.def("delta_prepare", &delta_prepare);
   m.def("delta_recur", &delta_recur);
   m.def("delta_chunk", &delta_chunk);
-  m.def("paged_tiled_ok", &paged_tiled_ok);
-  m.def("paged_prefill", &paged_prefill);
-  m.def("paged_decode", &paged_decode);
 }

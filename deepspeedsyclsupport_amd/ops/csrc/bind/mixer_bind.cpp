@@ -1,12 +1,10 @@
-// Module of the ops of hybrid decoders without residual streams: norms on sublayer outputs, gated norms, token-side gates,
-// latent attention, recurrences with a scalar decay per head. A shared object of its own, so that serving such a model
-// compiles only this and the decode products (gemv_bind.cpp).
+// Module of the ops of post-norm hybrid decoders: norms on sublayer outputs, token-side gates, latent attention. A shared
+// object of its own, so that serving a model compiles the mechanisms it has and no others.
 #include "bind_util.h"
 
 extern "C" {
 int ds_post_norm(float*, const void*, const float*, const int*, const void*, const int*, int, const float*, float, void*, int,
                  float, int, hipStream_t);
-int ds_gated_norm(const void*, const void*, int64_t, const float*, void*, int64_t, int, int, float, int, int, hipStream_t);
 int ds_gelu(const void*, void*, int64_t, int, hipStream_t);
 int ds_token_gate(const void*, const int*, const void*, int64_t, void*, int64_t, int, int, hipStream_t);
 int ds_latent_prepare(const void*, const float*, const float*, float, const double*, int, const int*, const int*, const int*,
@@ -16,7 +14,7 @@ int ds_head_linear(const void*, const void*, void*, int, int, int, int, int, int
                    hipStream_t);
 int ds_latent_gather(const void*, const int*, int, const int*, int, int, void*, int64_t, int, int, int, hipStream_t);
 int ds_paged_generic(const void*, const void*, const void*, void*, const int*, int, const int*, const int*, int, int, int,
-                     int, int, int, int, float, float, int, int, const float*, int, hipStream_t);
+                     int, int, int, int, float, float, int, int, const float*, int64_t, int, hipStream_t);
 int ds_latent_decode_ok(int, int);
 void ds_latent_decode_plan(int, int, int, int, int, int*, int*);
 int ds_latent_decode(const void*, const void*, void*, float*, float*, const int*, int, const int*, const int*, int, int, int,
@@ -24,22 +22,9 @@ int ds_latent_decode(const void*, const void*, void*, float*, float*, const int*
 int ds_latent_prefill_ok(int, int, int);
 int ds_latent_prefill(const void*, const void*, const void*, void*, const int*, const int*, const int*, int, const int*, int,
                       int, int, int, int, int, int, const float*, float, hipStream_t);
-int ds_scan_prepare(const void*, const float*, const float*, const void*, const float*, const float*, const int*, const int*,
-                    const int*, const int*, void*, void*, float*, const int*, int, int, hipStream_t);
-int ds_scan_recur(const void*, const void*, const float*, const float*, const float*, const void*, float*, void*, const int*,
-                  int, int, const int*, const int*, const int*, void*, const int*, int, int, hipStream_t);
-int ds_scan_chunk_ok(int);
-int ds_scan_chunk(const void*, const void*, const float*, const float*, const float*, const void*, float*, void*, const int*,
-                  int, const int*, const int*, const int*, void*, const int*, int, hipStream_t);
 }
 
 namespace {
-const float* opt_f32(const OptT& t, int64_t n, const char* name) { return has(t) ? f32(*t, n, name) : nullptr; }
-const double* f64(const Tensor& t, const char* name) {
-  need(t, name);
-  TORCH_CHECK(t.scalar_type() == at::kDouble, name, ": fp64");
-  return t.data_ptr<double>();
-}
 void table(const Tensor& bt, int64_t seqs) {
   need(bt, "block_table");
   TORCH_CHECK(bt.dim() == 2 && bt.scalar_type() == at::kInt && bt.size(0) >= seqs, "block_table [S, M] int32");
@@ -62,17 +47,6 @@ Tensor post_norm(Tensor x, OptT y, OptT w, double eps, OptT ids, OptT embed, Opt
                      has(embed) ? i32(*ids, T, "ids") : nullptr, has(embed) ? embed->data_ptr() : nullptr,
                      has(rows) ? i32(*rows, R, "rows") : nullptr, (int)R, has(rows) ? f32(*final_w, W, "final norm") : nullptr,
                      (float)mult, out.data_ptr(), (int)W, (float)eps, dcode(src), stream()), "post_norm");
-  return out;
-}
-
-Tensor gated_norm(Tensor y, Tensor proj, int64_t gate, Tensor w, int64_t parts, double eps, bool before) {
-  need(y, "y"); need(proj, "proj");
-  const int64_t T = y.size(0), C = y.size(1);
-  TORCH_CHECK(y.dim() == 2 && proj.dim() == 2 && proj.size(0) == T && gate >= 0 && gate + C <= proj.size(1) &&
-              proj.scalar_type() == y.scalar_type() && parts > 0 && C % parts == 0, "gated_norm: y [T, C], gate columns of proj");
-  auto out = torch::empty_like(y);
-  check(ds_gated_norm(y.data_ptr(), (const char*)proj.data_ptr() + gate * proj.element_size(), proj.size(1), f32(w, C, "norm"),
-                      out.data_ptr(), T, (int)C, (int)parts, (float)eps, before, dcode(y), stream()), "gated_norm");
   return out;
 }
 
@@ -156,7 +130,7 @@ Tensor latent_generic(Tensor q, Tensor lat, Tensor bt, Tensor pos, Tensor seq_id
   auto o = torch::empty({T, H, R}, q.options());
   check(ds_paged_generic(q.data_ptr(), lat.data_ptr(), lat.data_ptr(), o.data_ptr(), bt.data_ptr<int>(), (int)bt.size(1),
                          i32(pos, T, "pos"), i32(seq_ids, T, "seq_ids"), (int)T, (int)H, 1, c.W, (int)R, c.W, c.BS, (float)scale,
-                         0.f, 0, 0, f32(sink, H, "sink"), dcode(q), stream()), "latent_generic");
+                         0.f, 0, 0, f32(sink, H, "sink"), H * R, dcode(q), stream()), "latent_generic");
   return o;
 }
 
@@ -220,121 +194,10 @@ void latent_prefill(Tensor q, Tensor kv, Tensor ctx, Tensor start, Tensor cu_q, 
                           i32(offs, offs.numel(), "offs"), (int)first, (int)H, (int)d, (int)r, (int)e, (int)ctx.size(1),
                           (int)(ctx.size(1) - r), f32(sink, H, "sink"), (float)scale, stream()), "latent_prefill");
 }
-
-// ---------------------------------------------------------------------------------------------- recurrences
-struct Dims {  // ops/mixer_ops.py: ScanLayout
-  int v[12];
-  int rows() const { return v[0]; }
-  int Hk() const { return v[4]; }
-  int H() const { return v[5]; }
-  int dk() const { return v[6]; }
-  int dv() const { return v[7]; }
-  int taps() const { return v[8]; }
-  int conv() const { return v[9]; }
-  int channels() const { return v[10]; }
-  int dt() const { return v[11]; }
-  int dks() const { return (dk() + 7) / 8 * 8; }
-  int dvs() const { return (dv() + 7) / 8 * 8; }
-};
-Dims dims_of(const std::vector<int64_t>& d) {
-  TORCH_CHECK(d.size() == 12, "scan: 12 dimensions");
-  Dims D;
-  for (int i = 0; i < 12; ++i) D.v[i] = (int)d[i];
-  TORCH_CHECK(D.Hk() > 0 && D.H() > 0 && D.H() % D.Hk() == 0 && D.dk() > 0 && D.dk() <= 512 && D.dv() > 0 && D.taps() >= 1,
-              "scan: head counts / sizes (keys up to 512)");
-  auto inside = [&](int64_t at, int64_t n, int64_t lo, int64_t hi) { return at >= lo && at + n <= hi; };
-  const int64_t nk = (int64_t)D.Hk() * D.dk(), nv = (int64_t)D.H() * D.dv(), lo = D.channels() ? D.conv() : 0,
-                hi = D.channels() ? D.conv() + D.channels() : D.rows();
-  TORCH_CHECK(inside(D.conv(), D.channels(), 0, D.rows()) && inside(D.v[1], nk, lo, hi) && inside(D.v[2], nk, lo, hi) &&
-              inside(D.v[3], nv, lo, hi) && (D.dt() < 0 || inside(D.dt(), D.H(), 0, D.rows())) &&
-              (D.taps() == 1 || D.channels() > 0), "scan: columns outside the projection");
-  return D;
-}
-void conv_ok(const Dims& D, const OptT& cs, const Tensor& proj) {
-  TORCH_CHECK(D.taps() == 1 || (has(cs) && cs->is_cuda() && cs->is_contiguous() && cs->dim() == 3 && cs->size(1) == D.taps() - 1 &&
-              cs->size(2) == D.channels() && cs->scalar_type() == proj.scalar_type()), "scan: conv_state [slots, taps-1, channels]");
-}
-
-// proj [T, rows] -> qk [2, Hk, T, dks], v [H, T, dvs] (storage type), gb [T, 2, H] fp32 or None
-std::tuple<Tensor, Tensor, OptT> scan_prepare(Tensor proj, std::vector<int64_t> dims, OptT conv_w, OptT conv_b, OptT conv_state,
-                                              OptT a_log, OptT dt_bias, Tensor seq_ids, Tensor cu, Tensor start, Tensor slots) {
-  need(proj, "proj");
-  const Dims D = dims_of(dims);
-  const int64_t T = proj.size(0), S = start.numel();
-  TORCH_CHECK(proj.dim() == 2 && proj.size(1) == D.rows(), "scan_prepare: proj [T, rows]");
-  TORCH_CHECK(has(conv_w) == (D.channels() > 0) && has(conv_b) == has(conv_w), "scan_prepare: convolution weights");
-  conv_ok(D, conv_state, proj);
-  // (rows are padded to 16-byte pieces with zeros)
-  auto make = [&](at::IntArrayRef s, bool pad) { return pad ? torch::zeros(s, proj.options()) : torch::empty(s, proj.options()); };
-  Tensor qk = make({2, D.Hk(), T, D.dks()}, D.dks() != D.dk()), v = make({D.H(), T, D.dvs()}, D.dvs() != D.dv());
-  OptT gb;
-  if (D.dt() >= 0) gb = torch::empty({T, 2, D.H()}, proj.options().dtype(at::kFloat));
-  check(ds_scan_prepare(proj.data_ptr(), opt_f32(conv_w, (int64_t)D.channels() * D.taps(), "conv_w"),
-                        opt_f32(conv_b, D.channels(), "conv_b"), D.taps() > 1 ? conv_state->data_ptr() : nullptr,
-                        D.dt() >= 0 ? f32(*a_log, D.H(), "a_log") : nullptr, D.dt() >= 0 ? f32(*dt_bias, D.H(), "dt_bias") : nullptr,
-                        i32(seq_ids, T, "seq_ids"), i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"),
-                        qk.data_ptr(), v.data_ptr(), gb ? gb->data_ptr<float>() : nullptr, D.v, (int)T, dcode(proj), stream()),
-        "scan_prepare");
-  return {qk, v, gb};
-}
-
-struct ScanCheck {
-  ScanCheck(const Dims& D, const Tensor& qk, const Tensor& v, const OptT& gb, const OptT& ld, const Tensor& proj,
-            const Tensor& state, const OptT& conv_state, const Tensor& out) {
-    need(qk, "qk"); need(v, "v"); need(proj, "proj"); need(state, "state"); need(out, "out");
-    const int64_t T = proj.size(0);
-    TORCH_CHECK(proj.size(1) == D.rows() && qk.numel() == 2 * D.Hk() * T * D.dks() && v.numel() == D.H() * T * D.dvs() &&
-                qk.scalar_type() == proj.scalar_type() && v.scalar_type() == proj.scalar_type(), "scan: qk / v");
-    TORCH_CHECK(has(gb) != has(ld), "scan: decays per token or per head");
-    TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == D.H() && state.size(2) == D.dv() &&
-                state.size(3) == D.dks(), "scan: state [slots, H, dv, dks] fp32");
-    TORCH_CHECK(out.numel() == T * D.H() * D.dv() && out.scalar_type() == proj.scalar_type(), "scan: out [T, H dv]");
-    conv_ok(D, conv_state, proj);
-    TORCH_CHECK(D.taps() == 1 || conv_state->size(0) == state.size(0), "scan: slots");
-  }
-};
-
-// Runs the sequences in `list` token by token; writes their rows of out and their state slots
-void recur_list(Tensor qk, Tensor v, OptT gb, OptT log_decay, OptT skip, Tensor proj, const Dims& D, Tensor state,
-                OptT conv_state, Tensor list, int stride, Tensor cu, Tensor start, Tensor slots, Tensor out) {
-  const int64_t T = proj.size(0), S = start.numel();
-  check(ds_scan_recur(qk.data_ptr(), v.data_ptr(), opt_f32(gb, T * 2 * D.H(), "gb"), opt_f32(log_decay, D.H(), "log_decay"),
-                      opt_f32(skip, D.H(), "skip"), proj.data_ptr(), state.data_ptr<float>(),
-                      D.taps() > 1 ? conv_state->data_ptr() : nullptr, i32(list, list.numel(), "list"),
-                      (int)(list.numel() / stride), stride, i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"),
-                      out.data_ptr(), D.v, (int)T, dcode(proj), stream()), "scan_recur");
-}
-
-void scan_recur(Tensor qk, Tensor v, OptT gb, OptT log_decay, OptT skip, Tensor proj, std::vector<int64_t> dims, Tensor state,
-                OptT conv_state, Tensor list, Tensor cu, Tensor start, Tensor slots, Tensor out) {
-  const Dims D = dims_of(dims);
-  ScanCheck(D, qk, v, gb, log_decay, proj, state, conv_state, out);
-  recur_list(qk, v, gb, log_decay, skip, proj, D, state, conv_state, list, 1, cu, start, slots, out);
-}
-
-// The same for long portions, seqs [n, 2]: bf16 by chunks of 64 tokens on the matrix cores; fp32 (and key widths above 256)
-// token by token
-void scan_chunk(Tensor qk, Tensor v, OptT gb, OptT log_decay, OptT skip, Tensor proj, std::vector<int64_t> dims, Tensor state,
-                OptT conv_state, Tensor seqs, Tensor cu, Tensor start, Tensor slots, Tensor out) {
-  const Dims D = dims_of(dims);
-  ScanCheck(D, qk, v, gb, log_decay, proj, state, conv_state, out);
-  TORCH_CHECK(seqs.dim() == 2 && seqs.size(1) == 2, "scan_chunk: seqs [n, 2]");
-  if (proj.scalar_type() != at::kBFloat16 || !ds_scan_chunk_ok(D.dk())) {
-    recur_list(qk, v, gb, log_decay, skip, proj, D, state, conv_state, seqs, 2, cu, start, slots, out);
-    return;
-  }
-  const int64_t T = proj.size(0), S = start.numel();
-  check(ds_scan_chunk(qk.data_ptr(), v.data_ptr(), opt_f32(gb, T * 2 * D.H(), "gb"), opt_f32(log_decay, D.H(), "log_decay"),
-                      opt_f32(skip, D.H(), "skip"), proj.data_ptr(), state.data_ptr<float>(),
-                      D.taps() > 1 ? conv_state->data_ptr() : nullptr, i32(seqs, seqs.numel(), "seqs"), (int)seqs.size(0),
-                      i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"), out.data_ptr(), D.v, (int)T, stream()),
-        "scan_chunk");
-}
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("post_norm", &post_norm);
-  m.def("gated_norm", &gated_norm);
   m.def("gelu", &gelu);
   m.def("token_gate", &token_gate);
   m.def("latent_prepare", &latent_prepare);
@@ -346,7 +209,4 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("latent_decode", &latent_decode);
   m.def("latent_gather", &latent_gather);
   m.def("latent_prefill", &latent_prefill);
-  m.def("scan_prepare", &scan_prepare);
-  m.def("scan_recur", &scan_recur);
-  m.def("scan_chunk", &scan_chunk);
 }

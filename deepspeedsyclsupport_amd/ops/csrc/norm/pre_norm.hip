@@ -1,0 +1,152 @@
+// Plain fp32 residual with RMS norms on the sublayers' inputs, CDNA4 (gfx950). One launch per sublayer boundary:
+//   1. x <- x + y, or x <- x + sum_k w[t, k] y[row(t, k)] (the weighted outputs of a token's experts), or, at the start of the
+//      model, x <- the token's embedding row times a constant;
+//   2. the next sublayer's input x / rms(x) * w in the storage type.
+// With a row list (the rows whose logits are wanted) only those rows are normed and x stays as it is.
+//
+// HBM-bound: every operand is read once with 16-byte accesses, the row stays in registers between the passes; widths that are
+// no multiple of 8 take a plain version that goes over x twice.
+#include "ds_hip.h"
+
+namespace {
+
+struct PreArgs {
+  float* x;            // [T, W]
+  const void* y;       // [T, W] or [T * K, W]
+  const float* yw;     // [T, K] or null
+  const int* yrow;     // [T, K]: rows of y; null: t * K + k
+  int K;
+  const int* ids;      // [T]
+  const void* embed;   // [V, W]
+  float mult;          // of the embedding
+  const int* rows;
+  const float* w;      // [W]
+  void* out;
+  int W;
+  float eps;
+};
+
+// What the sublayer before adds to columns c .. c + 7 of token t
+template <typename T>
+__device__ __forceinline__ void added(const PreArgs& a, int64_t t, int c, float (&v)[8]) {
+  const T* y = (const T*)a.y;
+  if (!a.yw) {
+    Vec8<T>::load(y + t * a.W + c, v);
+    return;
+  }
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v[j] = 0.f;
+#pragma unroll 4
+  for (int k = 0; k < a.K; ++k) {
+    const int64_t e = t * a.K + k, r = a.yrow ? a.yrow[e] : e;
+    float u[8];
+    Vec8<T>::load(y + r * a.W + c, u);
+    const float g = a.yw[e];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] = fmaf(g, u[j], v[j]);
+  }
+}
+
+// NT threads per token, E x 8 elements per thread
+template <typename T, int NT, int E>
+__global__ void __launch_bounds__(NT) pre_norm_kernel(PreArgs a) {
+  __shared__ float red[NT / 64];
+  const int r = blockIdx.x, tid = threadIdx.x, W = a.W;
+  const int64_t src = a.rows ? a.rows[r] : r;
+  float* xr = a.x + src * W;
+  float xv[E][8], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < E; ++i) {
+    const int c = (tid + i * NT) * 8;
+    if (c >= W) continue;
+    if (a.embed) {
+      Vec8<T>::load((const T*)a.embed + (int64_t)a.ids[r] * W + c, xv[i]);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) xv[i][j] *= a.mult;
+    } else {
+      float v[8];
+      Vec8<float>::load(xr + c, xv[i]);
+      added<T>(a, src, c, v);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) xv[i][j] += v[j];
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ss = fmaf(xv[i][j], xv[i][j], ss);
+    if (!a.rows) Vec8<float>::store(xr + c, xv[i]);
+  }
+  const float rs = 1.f / sqrtf(block_sum(ss, red) / (float)W + a.eps);
+#pragma unroll
+  for (int i = 0; i < E; ++i) {
+    const int c = (tid + i * NT) * 8;
+    if (c >= W) continue;
+    float g[8];
+    Vec8<float>::load(a.w + c, g);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) xv[i][j] *= rs * g[j];
+    Vec8<T>::store((T*)a.out + (int64_t)r * W + c, xv[i]);
+  }
+}
+
+// any width
+template <typename T>
+__global__ void __launch_bounds__(256) pre_norm_any_kernel(PreArgs a) {
+  __shared__ float red[4];
+  const int r = blockIdx.x, tid = threadIdx.x, W = a.W;
+  const int64_t src = a.rows ? a.rows[r] : r;
+  const T* y = (const T*)a.y;
+  float* xr = a.x + src * W;
+  auto sum = [&](int c) {
+    if (a.embed) return (float)((const T*)a.embed)[(int64_t)a.ids[r] * W + c] * a.mult;
+    if (!a.yw) return xr[c] + (float)y[src * W + c];
+    float v = xr[c];
+    for (int k = 0; k < a.K; ++k) {
+      const int64_t e = src * a.K + k;
+      v = fmaf(a.yw[e], (float)y[(a.yrow ? a.yrow[e] : e) * W + c], v);
+    }
+    return v;
+  };
+  float ss = 0.f;
+  for (int c = tid; c < W; c += 256) {
+    const float v = sum(c);
+    ss = fmaf(v, v, ss);
+    if (!a.rows) xr[c] = v;
+  }
+  const float rs = 1.f / sqrtf(block_sum(ss, red) / (float)W + a.eps);
+  for (int c = tid; c < W; c += 256)  // (each thread re-reads what it wrote)
+    ((T*)a.out)[(int64_t)r * W + c] = (T)((a.rows ? sum(c) : xr[c]) * rs * a.w[c]);
+}
+
+template <typename T>
+int pre_norm(const PreArgs& a, int n, hipStream_t st) {
+#define GO(NT, E) hipLaunchKernelGGL((pre_norm_kernel<T, NT, E>), dim3(n), dim3(NT), 0, st, a)
+  const int W = a.W;
+  if (W % 8 == 0 && W <= 16384) {
+    if (W <= 512) GO(64, 1);
+    else if (n <= 512 && W <= 4096) GO(512, 1);
+    else if (n <= 512 && W <= 8192) GO(1024, 1);
+    else if (n <= 512) GO(1024, 2);
+    else if (W <= 2048) GO(256, 1);
+    else if (W <= 4096) GO(256, 2);
+    else if (W <= 8192) GO(256, 4);
+    else GO(256, 8);
+  } else {
+    hipLaunchKernelGGL((pre_norm_any_kernel<T>), dim3(n), dim3(256), 0, st, a);
+  }
+#undef GO
+  DS_CHECK_LAUNCH();
+  return 0;
+}
+
+}  // namespace
+
+// y [T, W] (yw null), or y [.., W] with yw [T, K] and optionally yrow [T, K]; or ids and embed, times mult. -> out [n, W]
+extern "C" int ds_pre_norm(float* x, const void* y, const float* yw, const int* yrow, int K, const int* ids, const void* embed,
+                           float mult, const int* rows, int n, const float* w, void* out, int W, float eps, int dtype,
+                           hipStream_t st) {
+  if (n <= 0) return 0;
+  if (W <= 0 || (!y == !embed) || (embed && (!ids || rows)) || (yw && K <= 0)) return (int)hipErrorInvalidValue;
+  const PreArgs a{x, y, yw, yrow, K, ids, embed, mult, rows, w, out, W, eps};
+  if (dtype == DS_F32) return pre_norm<float>(a, n, st);
+  if (dtype == DS_BF16) return pre_norm<bf16>(a, n, st);
+  return (int)hipErrorInvalidValue;
+}

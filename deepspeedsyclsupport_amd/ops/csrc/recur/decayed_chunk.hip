@@ -4,6 +4,8 @@
 // With the running log decay G_i of a chunk (its first token included) and the state S0 the chunk starts from:
 //     o_i = e^{G_i} S0^T q_i + sum_{j <= i} P_ij v_j + D v_i,    P_ij = e^{G_i - G_j} b_j (q_i . k_j)
 //     S   = e^{G_C} S0 + sum_j e^{G_C - G_j} b_j k_j v_j^T
+// (the first two terms of o times a constant). The normaliser's products are the same with a single value column of ones:
+// z . q_i = e^{G_i} z0 . q_i + sum_j P_ij. Every workgroup keeps its own in LDS; it costs a few sums per chunk.
 // One workgroup per (sequence, head, 16 WC value columns) walks the chunks. Two of its 2 WC waves share 16 value columns: each
 // keeps half of the key rows of their state in registers, in the result layout of the matrix instructions. The next state
 // accumulates into it, and the same registers are the left operand of the read-out (a product's k order is free as long as
@@ -86,11 +88,11 @@ __device__ __forceinline__ bf16x8 read_tr(const bf16* base, int pitch, int r, in
 
 // NK: 32-wide steps of the key width (rounded up), even unless the waves of a pair cannot share (NK 1: the second one has
 // no rows); WC: groups of 16 value columns
-template <int NK, int WC>
+template <int NK, int WC, bool NORM>
 __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decayed_chunk_kernel(
     const bf16* __restrict__ qk, const bf16* __restrict__ v, const float* __restrict__ gb,
-    const float* __restrict__ log_decay, const float* __restrict__ skip, const bf16* __restrict__ proj,
-    float* __restrict__ state, bf16* __restrict__ conv_state, const int* __restrict__ seqs, const int* __restrict__ cu,
+    const float* __restrict__ log_decay, const float* __restrict__ skip, float scale, const bf16* __restrict__ proj,
+    float* __restrict__ state, float* __restrict__ zstate, const float* __restrict__ floors, bf16* __restrict__ conv_state, const int* __restrict__ seqs, const int* __restrict__ cu,
     const int* __restrict__ start, const int* __restrict__ slots, bf16* __restrict__ out, ScanDims D) {
   constexpr int NT = 128 * WC, NW = 2 * WC, VT = 16 * WC;
   constexpr int KP = 32 * NK + 8, VP = VT + 8;      // LDS row lengths of q and k, of v
@@ -108,6 +110,10 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
   float* const bs = reinterpret_cast<float*>(Gs + 2 * NW * C);    // [2 NW][C] step sizes
   float* const eg = bs + 2 * NW * C;                              // [2 NW][C] e^{G_i}
   float* const ws = eg + 2 * NW * C;                              // [2 NW][C] e^{G_C - G_j} b_j
+  float* const fl = ws + 2 * NW * C;                              // NORM: [2 NW][C] floors,
+  float* const zs = fl + 2 * NW * C;                              //   [32 NK] normaliser the chunk starts from,
+  float* const zq = zs + 32 * NK;                                 //   [C] its products with the queries,
+  float* const rs = zq + C;                                       //   [4][C] sums of P's rows over 16 columns each
 
   const int vts = (D.dv + VT - 1) / VT, bid = xcd_remap(blockIdx.x, gridDim.x);
   const int vt = bid % vts, h = bid / vts % D.H, seq = seqs[2 * (bid / (vts * D.H))];
@@ -126,6 +132,10 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
     const int k = k_first + 16 * t + 4 * q4;
     S[t] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (!fresh && col < D.dv && k < dks) S[t] = *reinterpret_cast<const f32x4*>(st + k);
+  }
+  if constexpr (NORM) {  // (visible after the first barrier of the loop)
+    const float* zt = zstate + D.z_at(slots[seq], h, v0);
+    for (int k = tid; k < 32 * NK; k += NT) zs[k] = !fresh && k < dks ? zt[k] : 0.f;
   }
   const float sk = skip ? skip[h] : 0.f, ld = log_decay ? log_decay[h] : 0.f;
   const bf16* qbase = qk + D.q_at(g, t0);
@@ -192,11 +202,12 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
     }
   };
   // ---- decays and step sizes of a chunk, a lane per token: every NW chunks each wave prepares one of the next NW
-  float lg = 0.f, lb = 0.f;
+  float lg = 0.f, lb = 0.f, lf = 0.f;
   auto fetch_gb = [&](int c) {
     const int64_t t = t0 + min(c * C + lane, n - 1);
     lg = gb ? gb[t * 2 * D.H + h] : ld;
     lb = gb ? gb[(t * 2 + 1) * D.H + h] : 1.f;
+    if constexpr (NORM) lf = floors[t * D.H + h];
   };
   auto scan_gb = [&](int c) {
     const bool ok = c * C + lane < n;  // rows past the end neither decay nor add anything
@@ -213,6 +224,7 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
     bs[b] = b0;
     eg[b] = __builtin_amdgcn_exp2f((float)G);
     ws[b] = __builtin_amdgcn_exp2f((float)(GC - G)) * b0;
+    if constexpr (NORM) fl[b] = lf;
   };
   fetch(0);
   fetch_gb(w);
@@ -244,6 +256,12 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
         {  // (no branch: behind the diagonal the factor is some number, or infinite)
           const float f = s[r] * (__builtin_amdgcn_exp2f((float)(gi - Gs[cb + j + r])) * bs[cb + j + r]);
           s[r] = j + r <= i ? f : 0.f;
+        }
+        if constexpr (NORM) {
+          float sum = (s[0] + s[1]) + (s[2] + s[3]);
+          sum += __shfl_xor(sum, 16, 64);
+          sum += __shfl_xor(sum, 32, 64);
+          if (q4 == 0) rs[jt * C + i] = sum;
         }
       }
       unsigned a[2], b[2], d[2];
@@ -282,6 +300,20 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
         }
       }
     }
+    if constexpr (NORM) {  // z0 . q: neighbouring lanes share a token, 8 key columns at a time
+      constexpr int LP = NT / C;
+      const int row = tid / LP, part = tid % LP;
+      float a = 0.f;
+      for (int k = 8 * part; k < 32 * NK; k += 8 * LP) {
+        float x[8];
+        Vec8<bf16>::load(Qs + row * KP + k, x);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) a = fmaf(x[e], zs[k + e], a);
+      }
+#pragma unroll
+      for (int o = 1; o < LP; o <<= 1) a += __shfl_xor(a, o, 64);
+      if (part == 0) zq[row] = a;
+    }
     // each wave of a pair finishes two token tiles: the other two go to its partner
 #pragma unroll
     for (int i = 0; i < 2; ++i) Ys[(w * 2 + i) * 64 + lane] = pick(half, y[i], y[2 + i]);
@@ -310,6 +342,28 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       }
     }
     lds_barrier();  // P and the partner's half are complete
+    if constexpr (NORM) {  // next normaliser: neighbouring lanes share a pair of key columns and take every JP-th token
+      constexpr int JP = NT / (16 * NK);
+      const int k = tid / JP * 2, part = tid % JP;
+      float a0 = 0.f, a1 = 0.f;
+#pragma unroll 4
+      for (int j = part; j < C; j += JP) {
+        const bf16x2 x = *reinterpret_cast<const bf16x2*>(Ks + j * KP + k);
+        const float wj = ws[cb + j];
+        a0 = fmaf((float)x[0], wj, a0);
+        a1 = fmaf((float)x[1], wj, a1);
+      }
+#pragma unroll
+      for (int o = 1; o < JP; o <<= 1) {
+        a0 += __shfl_xor(a0, o, 64);
+        a1 += __shfl_xor(a1, o, 64);
+      }
+      if (part == 0) {
+        const float dc = eg[cb + C - 1];
+        zs[k] = fmaf(dc, zs[k], a0);
+        zs[k + 1] = fmaf(dc, zs[k + 1], a1);
+      }
+    }
     // ---- within the chunk, token tiles 2 half and 2 half + 1
 #pragma unroll
     for (int k = 0; k < 2; ++k) {
@@ -323,6 +377,14 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
         acc = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr + 2 * C * PP), acc);
         acc = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr + C * PP), acc);
         acc = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr), acc);
+      }
+      if constexpr (NORM) {
+        const int r = 16 * i + l16;
+        float z = eg[cb + r] * zq[r];
+        for (int jt = 0; jt <= i; ++jt) z += rs[jt * C + r];
+        acc *= scale / (fmaxf(fabsf(z * scale), fl[cb + r]) + 1e-6f);
+      } else {
+        acc *= scale;
       }
       const int t = c * C + 16 * i + l16, cv = v0 + 16 * wc + 4 * q4;
       const bf16x4 vv = *reinterpret_cast<const bf16x4*>(Vs + (16 * i + l16) * VP + 16 * wc + 4 * q4);
@@ -348,25 +410,32 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       if (k < dks) *reinterpret_cast<f32x4*>(st + k) = S[t];
     }
   }
+  if constexpr (NORM) {  // (the loop ends with a barrier) every copy that is about this workgroup's columns
+    for (int cc = 0; cc < VT && v0 + cc < D.dv; cc += Z_COLS) {
+      float* zt = zstate + D.z_at(slots[seq], h, v0 + cc);
+      for (int k = tid; k < dks; k += NT) zt[k] = zs[k];
+    }
+  }
   if (vt == 0 && D.taps > 1)
     advance_windows(conv_state + (int64_t)slots[seq] * (D.taps - 1) * D.channels, proj, t0, n, D, fresh, h);
 }
 
-template <int NK, int WC>
-int launch(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip, const void* proj,
-           float* state, void* conv_state, const int* seqs, int nseq, const int* cu, const int* start, const int* slots,
+template <int NK, int WC, bool NORM>
+int launch(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip, float scale,
+           const void* proj, float* state, float* zstate, const float* floors, void* conv_state, const int* seqs, int nseq, const int* cu, const int* start, const int* slots,
            void* out, const ScanDims& D, hipStream_t st) {
   constexpr int VT = 16 * WC;
-  constexpr int LDS = (2 * C * (32 * NK + 8) + C * (VT + 8) + 3 * C * PP) * 2 + 2 * WC * 2 * 64 * 16 + 4 * WC * C * 20;
+  constexpr int LDS = (2 * C * (32 * NK + 8) + C * (VT + 8) + 3 * C * PP) * 2 + 2 * WC * 2 * 64 * 16 + 4 * WC * C * 20 +
+                      (NORM ? (4 * WC * C + 32 * NK + 5 * C) * 4 : 0);
   static bool attr = false;
   if (!attr) {
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<NK, WC>),
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<NK, WC, NORM>),
                               hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
     attr = true;
   }
-  hipLaunchKernelGGL((decayed_chunk_kernel<NK, WC>), dim3((unsigned)((D.dv + VT - 1) / VT * D.H * nseq)), dim3(128 * WC), LDS,
-                     st, (const bf16*)qk, (const bf16*)v, gb, log_decay, skip, (const bf16*)proj, state, (bf16*)conv_state,
-                     seqs, cu, start, slots, (bf16*)out, D);
+  hipLaunchKernelGGL((decayed_chunk_kernel<NK, WC, NORM>), dim3((unsigned)((D.dv + VT - 1) / VT * D.H * nseq)), dim3(128 * WC), LDS,
+                     st, (const bf16*)qk, (const bf16*)v, gb, log_decay, skip, scale, (const bf16*)proj, state, zstate,
+                     floors, (bf16*)conv_state, seqs, cu, start, slots, (bf16*)out, D);
   DS_CHECK_LAUNCH();
   return 0;
 }
@@ -375,24 +444,33 @@ int launch(const void* qk, const void* v, const float* gb, const float* log_deca
 
 extern "C" int ds_scan_chunk_ok(int dk) { return dk <= 256; }
 
-// bf16 storage, dk up to 256. seqs [nseq, 2]: (sequence, anything)
+// bf16 storage, dk up to 256. seqs [nseq, 2]: (sequence, anything). zstate, floors: as for ds_scan_recur
 extern "C" int ds_scan_chunk(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip,
-                             const void* proj, float* state, void* conv_state, const int* seqs, int nseq, const int* cu,
+                             float scale, const void* proj, float* state, float* zstate, const float* floors,
+                             void* conv_state, const int* seqs, int nseq, const int* cu,
                              const int* start, const int* slots, void* out, const int* dims, int tokens, hipStream_t st) {
   if (nseq <= 0) return 0;
   const ScanDims D{dims[0], dims[1], dims[2], dims[3], dims[4], dims[5], dims[6], dims[7], dims[8], dims[9], dims[10], dims[11],
                    tokens};
-  if (!scan_dims_ok(D) || !ds_scan_chunk_ok(D.dk) || (!gb == !log_decay) || (D.taps > 1 && !conv_state) ||
+  if (!scan_dims_ok(D) || !ds_scan_chunk_ok(D.dk) || (!gb == !log_decay) || (!zstate != !floors) || (D.taps > 1 && !conv_state) ||
       (int64_t)nseq * D.H * ((D.dv + 31) / 32) > INT32_MAX)
     return (int)hipErrorInvalidValue;
   // wide workgroups share q, k and P among more columns; narrow ones where there are too few to fill the chip
   const bool wide = D.dv > 32 && (int64_t)nseq * D.H * ((D.dv + 63) / 64) >= 192;
-#define GO(NK)                                                                                                         \
-  return wide ? launch<NK, 4>(qk, v, gb, log_decay, skip, proj, state, conv_state, seqs, nseq, cu, start, slots, out, D, st) \
-              : launch<NK, 2>(qk, v, gb, log_decay, skip, proj, state, conv_state, seqs, nseq, cu, start, slots, out, D, st)
-  if (D.dk <= 32) GO(1);
-  if (D.dk <= 64) GO(2);
-  if (D.dk <= 128) GO(4);
-  GO(8);
+#define RUN(NK, WC, NORM)                                                                                               \
+  return launch<NK, WC, NORM>(qk, v, gb, log_decay, skip, scale, proj, state, zstate, floors, conv_state, seqs, nseq, cu, start, \
+                              slots, out, D, st)
+#define GO(NK)                             \
+  {                                        \
+    if (zstate && wide) RUN(NK, 4, true);  \
+    if (zstate) RUN(NK, 2, true);          \
+    if (wide) RUN(NK, 4, false);           \
+    RUN(NK, 2, false);                     \
+  }
+  if (D.dk <= 32) GO(1)
+  if (D.dk <= 64) GO(2)
+  if (D.dk <= 128) GO(4)
+  GO(8)
 #undef GO
+#undef RUN
 }

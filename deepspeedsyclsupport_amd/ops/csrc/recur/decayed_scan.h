@@ -5,6 +5,8 @@
 
 namespace {
 
+constexpr int Z_COLS = 32;
+
 // Fused projection row of `rows` columns: q, k [Hk heads of dk], v [H heads of dv] start at columns q, k, v; `channels`
 // columns from `conv` on pass a convolution of `taps`; dt: first of H step-size columns, or -1.
 struct ScanDims {
@@ -15,6 +17,9 @@ struct ScanDims {
   // head by head, [heads, T, width]: tiles of a head's rows spread over the memory channels whatever the head count
   __host__ __device__ int64_t q_at(int g, int64_t t) const { return ((int64_t)g * T + t) * dks(); }
   __host__ __device__ int64_t k_at(int g, int64_t t) const { return ((int64_t)(Hk + g) * T + t) * dks(); }
+  // normaliser of the columns around `col`: a slot holds a copy for every Z_COLS value columns, [H, copies, dks]
+  __host__ __device__ int zc() const { return (dv + Z_COLS - 1) / Z_COLS; }
+  __host__ __device__ int64_t z_at(int64_t slot, int h, int col) const { return ((slot * H + h) * zc() + col / Z_COLS) * dks(); }
   __host__ __device__ int64_t v_at(int h, int64_t t) const { return ((int64_t)h * T + t) * dvs(); }
 };
 

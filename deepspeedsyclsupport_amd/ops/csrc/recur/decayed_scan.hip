@@ -1,13 +1,15 @@
 // Recurrences with a scalar decay per head (state-space duality, linear attention with constant decays), CDNA4 (gfx950).
 //
 // Per head, with a state S [dk, dv] in fp32 that starts at zero:
-//     S <- a S + b k v^T;   o = S^T q + D v
-// with b = softplus(dt + dt_bias), a = exp(-exp(A_log) b) per token, or b = 1 and a constant a. q, k and v are columns of a
-// fused projection row that passed (optionally) a causal convolution with bias and (always) silu; several heads may share
-// q and k.
+//     S <- a S + b k v^T;   o = c S^T q + D v
+// with b = softplus(dt + dt_bias), a = exp(-exp(A_log) b) per token, or any a and b per token (exp_gates.hip), or b = 1 and a
+// constant a; c is a constant. q, k and v are columns of a fused projection row. Several heads may share q and k. With a
+// normaliser, z <- a z + b k runs beside the state and o becomes c S^T q / (max(|c z . q|, floor) + 1e-6), floor per token.
 //
-//  * prepare: a lane per few channels of a tile of consecutive tokens; inputs before the portion come from the sequence's
-//    state slot. Step sizes and log decays leave it in fp32, q / k / v in the storage type (they are activations).
+//  * prepare: q, k and v after (optionally) a causal convolution with bias and silu. A lane per few channels of a tile of
+//    consecutive tokens; inputs before the portion come from the sequence's state slot. Step sizes and log decays leave it in
+//    fp32, q / k / v in the storage type (they are activations).
+//  * split: q, k and v as they are, with (optionally) pairs of columns of q and k turned to their positions.
 //  * recur: one workgroup per (sequence, head, 64 value columns), the state in registers while the portion's tokens pass
 //    one by one: decoding, short portions, and everything in fp32 models. It also moves the convolution's windows on
 //    (prepare, which reads the old ones, has finished by then).
@@ -145,33 +147,85 @@ __global__ void __launch_bounds__(256) scan_prepare_kernel(
   }
 }
 
+// One workgroup per token: the row's q, k and v head by head, pairs (i, i + half) of the first 2 half columns of q and k turned
+// by the token's angles cs [half, 2]
+template <typename T, int V>
+__global__ void __launch_bounds__(256) scan_split_kernel(const T* __restrict__ proj, const float* __restrict__ cs, int half,
+                                                         T* __restrict__ qk, T* __restrict__ v_out, ScanDims D) {
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const T* row = proj + (int64_t)t * D.rows;
+  const float* a = cs + (int64_t)t * half * 2;
+  const int per = (D.dk - half) / V, hv = half / V;  // a head's pairs, then its columns without one
+  for (int i = tid; i < 2 * D.Hk * per; i += 256) {
+    const int g = i / per, j = i % per;
+    const T* src = row + (g < D.Hk ? D.q + g * D.dk : D.k + (g - D.Hk) * D.dk);
+    T* dst = qk + D.q_at(g, t);  // (k's heads lie behind q's)
+    if (j < hv) {
+      const int c = j * V;
+      float u[V], w[V], x[V], y[V];
+      ldv<T, V>(src + c, u);
+      ldv<T, V>(src + half + c, w);
+#pragma unroll
+      for (int e = 0; e < V; ++e) {
+        const float co = a[2 * (c + e)], si = a[2 * (c + e) + 1];
+        x[e] = u[e] * co - w[e] * si;
+        y[e] = w[e] * co + u[e] * si;
+      }
+      stv<T, V>(dst + c, x);
+      stv<T, V>(dst + half + c, y);
+    } else {
+      const int c = half + j * V;
+      float u[V];
+      ldv<T, V>(src + c, u);
+      stv<T, V>(dst + c, u);
+    }
+  }
+  const int pv = D.dv / V;
+  for (int i = tid; i < D.H * pv; i += 256) {
+    const int h = i / pv, c = i % pv * V;
+    float u[V];
+    ldv<T, V>(row + D.v + h * D.dv + c, u);
+    stv<T, V>(v_out + D.v_at(h, t) + c, u);
+  }
+}
+
 constexpr int LPC = 8;     // lanes per value column: lane p holds key rows 4 (p + LPC i) + 0..3
 constexpr int COLS = 64;   // value columns per workgroup
 
-template <typename T, int NV>
+// NORM: with a normaliser
+template <typename T, int NV, bool NORM>
 __global__ void __launch_bounds__(LPC * COLS) scan_recur_kernel(
     const T* __restrict__ qk, const T* __restrict__ v, const float* __restrict__ gb, const float* __restrict__ log_decay,
-    const float* __restrict__ skip, const T* __restrict__ proj, float* __restrict__ state, T* __restrict__ conv_state,
-    const int* __restrict__ list, int lstride, const int* __restrict__ cu, const int* __restrict__ start,
-    const int* __restrict__ slots, T* __restrict__ out, ScanDims D) {
+    const float* __restrict__ skip, float scale, const T* __restrict__ proj, float* __restrict__ state,
+    float* __restrict__ zstate, const float* __restrict__ floors, T* __restrict__ conv_state, const int* __restrict__ list,
+    int lstride, const int* __restrict__ cu, const int* __restrict__ start, const int* __restrict__ slots, T* __restrict__ out,
+    ScanDims D) {
   const int seq = list[blockIdx.x * lstride], h = blockIdx.y, g = h / (D.H / D.Hk), tid = threadIdx.x;
   const int64_t t0 = cu[seq];
   const int n = cu[seq + 1] - (int)t0, col = blockIdx.z * COLS + tid / LPC, p = tid % LPC, dks = D.dks();
   const bool fresh = start[seq] == 0, on = col < D.dv;
   float* st = state + (((int64_t)slots[seq] * D.H + h) * D.dv + min(col, D.dv - 1)) * dks;
-  f32x4 S[NV];
+  // every Z_COLS columns have a copy of the normaliser, so that no workgroup reads what another one writes
+  float* zt = NORM ? zstate + D.z_at(slots[seq], h, min(col, D.dv - 1)) : nullptr;
+  f32x4 S[NV], Z[NORM ? NV : 1];
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
     const int k = 4 * (p + LPC * i);
     S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (!fresh && k < dks) S[i] = *reinterpret_cast<const f32x4*>(st + k);
+    if constexpr (NORM) {
+      Z[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (!fresh && k < dks) Z[i] = *reinterpret_cast<const f32x4*>(zt + k);
+    }
   }
+  // (every column of a copy has read it before its first one writes it: they are of one workgroup)
+  if constexpr (NORM) __syncthreads();
   const float sk = skip ? skip[h] : 0.f, ld = log_decay ? log_decay[h] : 0.f;
   for (int t = 0; t < n; ++t) {
     const int64_t tok = t0 + t;
     const float a = expf(gb ? gb[tok * 2 * D.H + h] : ld), b = gb ? gb[(tok * 2 + 1) * D.H + h] : 1.f;
     const float vv = (float)v[D.v_at(h, tok) + min(col, D.dv - 1)], u = b * vv;
-    float o = 0.f;
+    float o = 0.f, zq = 0.f;
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int k = 4 * (p + LPC * i), kc = min(k, dks - 4);
@@ -183,10 +237,19 @@ __global__ void __launch_bounds__(LPC * COLS) scan_recur_kernel(
       for (int e = 0; e < 4; ++e) {
         S[i][e] = fmaf(kf[e] * z, u, a * S[i][e]);
         o = fmaf(S[i][e], qf[e], o);
+        if constexpr (NORM) {
+          Z[i][e] = fmaf(kf[e] * z, b, a * Z[i][e]);
+          zq = fmaf(Z[i][e], qf[e], zq);
+        }
       }
     }
 #pragma unroll
-    for (int d = 1; d < LPC; d <<= 1) o += __shfl_xor(o, d, 64);
+    for (int d = 1; d < LPC; d <<= 1) {
+      o += __shfl_xor(o, d, 64);
+      if constexpr (NORM) zq += __shfl_xor(zq, d, 64);
+    }
+    o *= scale;
+    if constexpr (NORM) o /= fmaxf(fabsf(zq * scale), floors[tok * D.H + h]) + 1e-6f;
     if (on && p == 0) out[(tok * D.H + h) * D.dv + col] = (T)fmaf(sk, vv, o);
   }
   if (on) {
@@ -194,6 +257,9 @@ __global__ void __launch_bounds__(LPC * COLS) scan_recur_kernel(
     for (int i = 0; i < NV; ++i) {
       const int k = 4 * (p + LPC * i);
       if (k < dks) *reinterpret_cast<f32x4*>(st + k) = S[i];
+      if constexpr (NORM) {
+        if (k < dks && col % Z_COLS == 0) *reinterpret_cast<f32x4*>(zt + k) = Z[i];
+      }
     }
   }
   if (blockIdx.z == 0 && D.taps > 1)
@@ -201,20 +267,27 @@ __global__ void __launch_bounds__(LPC * COLS) scan_recur_kernel(
 }
 
 template <typename T>
-int recur(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip, const void* proj,
-          float* state, void* conv_state, const int* list, int nlist, int lstride, const int* cu, const int* start,
+int recur(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip, float scale,
+          const void* proj, float* state, float* zstate, const float* floors, void* conv_state, const int* list, int nlist, int lstride, const int* cu, const int* start,
           const int* slots, void* out, const ScanDims& D, hipStream_t st) {
   const dim3 grid(nlist, D.H, (D.dv + COLS - 1) / COLS);
   const int nt = D.dv >= COLS ? LPC * COLS : (LPC * D.dv + 63) / 64 * 64, nv = (D.dks() / 4 + LPC - 1) / LPC;
-#define GO(NV)                                                                                                       \
-  hipLaunchKernelGGL((scan_recur_kernel<T, NV>), grid, dim3(nt), 0, st, (const T*)qk, (const T*)v, gb, log_decay, skip,   \
-                     (const T*)proj, state, (T*)conv_state, list, lstride, cu, start, slots, (T*)out, D)
-  if (nv <= 1) GO(1);
-  else if (nv <= 2) GO(2);
-  else if (nv <= 4) GO(4);
-  else if (nv <= 8) GO(8);
-  else GO(16);
+#define RUN(NV, NORM)                                                                                                \
+  hipLaunchKernelGGL((scan_recur_kernel<T, NV, NORM>), grid, dim3(nt), 0, st, (const T*)qk, (const T*)v, gb, log_decay,   \
+                     skip, scale, (const T*)proj, state, zstate, floors, (T*)conv_state, list, lstride, cu, start, slots, \
+                     (T*)out, D)
+#define GO(NV)                  \
+  {                             \
+    if (zstate) RUN(NV, true);  \
+    else RUN(NV, false);        \
+  }
+  if (nv <= 1) GO(1)
+  else if (nv <= 2) GO(2)
+  else if (nv <= 4) GO(4)
+  else if (nv <= 8) GO(8)
+  else GO(16)
 #undef GO
+#undef RUN
   DS_CHECK_LAUNCH();
   return 0;
 }
@@ -266,19 +339,49 @@ extern "C" int ds_scan_prepare(const void* proj, const float* conv_w, const floa
   return (int)hipErrorInvalidValue;
 }
 
-// list: sequences (indices into cu / start / slots) to run, `lstride` entries apart
+// The same tensors straight from the projection's columns (no convolution, no activation), the first 2 half columns of every
+// head of q and k turned by cs [tokens, half, 2] (cos, sin)
+extern "C" int ds_scan_split(const void* proj, const float* cs, int half, void* qk, void* v, const int* dims, int tokens,
+                             int dtype, hipStream_t st) {
+  if (tokens <= 0) return 0;
+  const ScanDims D{dims[0], dims[1], dims[2], dims[3], dims[4], dims[5], dims[6], dims[7], dims[8], dims[9], dims[10], dims[11],
+                   tokens};
+  if (!scan_dims_ok(D) || half < 0 || 2 * half > D.dk || (half && !cs)) return (int)hipErrorInvalidValue;
+  const int all = D.rows | D.q | D.k | D.v | D.dk | D.dv | half;
+#define GO(T, V) \
+  hipLaunchKernelGGL((scan_split_kernel<T, V>), dim3(tokens), dim3(256), 0, st, (const T*)proj, cs, half, (T*)qk, (T*)v, D)
+  if (dtype == DS_F32) {
+    if (all % 4 == 0) GO(float, 4);
+    else GO(float, 1);
+  } else if (dtype == DS_BF16) {
+    if (all % 8 == 0) GO(bf16, 8);
+    else if (all % 4 == 0) GO(bf16, 4);
+    else GO(bf16, 1);
+  } else {
+    return (int)hipErrorInvalidValue;
+  }
+#undef GO
+  DS_CHECK_LAUNCH();
+  return 0;
+}
+
+// list: sequences (indices into cu / start / slots) to run, `lstride` entries apart. zstate (null: no normaliser) [slots, H,
+// ceil(dv / 32), dks] with floors [tokens, H]
 extern "C" int ds_scan_recur(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip,
-                             const void* proj, float* state, void* conv_state, const int* list, int nlist, int lstride,
+                             float scale, const void* proj, float* state, float* zstate, const float* floors,
+                             void* conv_state, const int* list, int nlist, int lstride,
                              const int* cu, const int* start, const int* slots, void* out, const int* dims, int tokens,
                              int dtype, hipStream_t st) {
   if (nlist <= 0) return 0;
   const ScanDims D{dims[0], dims[1], dims[2], dims[3], dims[4], dims[5], dims[6], dims[7], dims[8], dims[9], dims[10], dims[11],
                    tokens};
-  if (!scan_dims_ok(D) || (!gb == !log_decay) || (D.taps > 1 && !conv_state)) return (int)hipErrorInvalidValue;
+  if (!scan_dims_ok(D) || (!gb == !log_decay) || (!zstate != !floors) || (D.taps > 1 && !conv_state))
+    return (int)hipErrorInvalidValue;
   if (dtype == DS_F32)
-    return recur<float>(qk, v, gb, log_decay, skip, proj, state, conv_state, list, nlist, lstride, cu, start, slots, out, D,
-                        st);
+    return recur<float>(qk, v, gb, log_decay, skip, scale, proj, state, zstate, floors, conv_state, list, nlist, lstride, cu,
+                        start, slots, out, D, st);
   if (dtype == DS_BF16)
-    return recur<bf16>(qk, v, gb, log_decay, skip, proj, state, conv_state, list, nlist, lstride, cu, start, slots, out, D, st);
+    return recur<bf16>(qk, v, gb, log_decay, skip, scale, proj, state, zstate, floors, conv_state, list, nlist, lstride, cu,
+                       start, slots, out, D, st);
   return (int)hipErrorInvalidValue;
 }

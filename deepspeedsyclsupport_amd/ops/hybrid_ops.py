@@ -1,13 +1,13 @@
 """Ops of the hybrid decoder (`inference/model_implementations/hybrid.py`): multi-stream residual, attention with
 per-head norms and chunked visibility, gated delta rule, clamped gated activation.
 
-Device tensors run the gfx950 kernels of `ds_hybrid_ops` (fp32 or bf16 storage, fp32 arithmetic); host tensors the
-plain versions in `ops/reference.py`, as everywhere in `ops`."""
+Device tensors run the gfx950 kernels of `ds_hybrid_ops`, `ds_attn_ops` and `ds_gemv_ops` (fp32 or bf16 storage, fp32
+arithmetic); host tensors the plain versions in `ops/reference.py`, as everywhere in `ops`."""
 import torch
 import torch.nn.functional as F
 
 from . import mixer_ops, reference
-from .native import gemv_ops, hybrid_ops, use_native
+from .native import attn_ops, gemv_ops, hybrid_ops, use_native
 
 DECODE_ROWS = 16
 ACTS = {"gelu": 2}  # epilogue codes of the decode products (csrc/gemv/skinny_*.hip)
@@ -27,28 +27,44 @@ def clamped_glu(gu, limit, alpha=1.702, shift=1.0):
 
 
 def qk_norm_append(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H):
-    f = hybrid_ops().qk_norm_append if use_native(qkv) else reference.qk_norm_append
+    f = attn_ops().qk_norm_append if use_native(qkv) else reference.qk_norm_append
     return f(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H)
 
 
-def ragged_attention(q, kc, vc, meta, scale, softcap=0.0, window=0, chunk=0):
-    """q [T, H, dk] of a ragged batch (`RaggedMeta`) over the paged cache, the new tokens already appended."""
+def rope_table(pos, freq):
+    """cos and sin of pos [T] * freq [half] (fp64) -> [T, half, 2] fp32."""
+    return (attn_ops() if use_native(pos) else reference).rope_table(pos, freq)
+
+
+def qk_rope_append(qkv, bias, qw, kw, eps, cs, meta, kc, vc, H, v_mult=1.0):
+    """Rows [q | k | v] (they may be columns of wider ones) plus bias -> q [T, H, dk]; k, and v times `v_mult`, into the paged
+    cache. q and k are divided by the root mean square over all their heads, times qw / kw (None: no norm), then the pairs
+    (i, i + half) of every head's first 2 half columns are turned by cs [T, half, 2] (None: no rotation)."""
+    f = attn_ops().qk_rope_append if use_native(qkv) else reference.qk_rope_append
+    return f(qkv, bias, qw, kw, eps, cs, v_mult, meta.pos_ids, meta.seq_ids, meta.block_tables, kc, vc, H)
+
+
+def ragged_attention(q, kc, vc, meta, scale, softcap=0.0, window=0, chunk=0, sink=None, out=None):
+    """q [T, H, dk] of a ragged batch (`RaggedMeta`) over the paged cache, the new tokens already appended -> [T, H, dv], or
+    into `out` [T, H dv] (it may be columns of a wider matrix). `sink` [H]: exp(sink) joins the denominators."""
+    T, H, dv = q.shape[0], q.shape[1], vc.shape[3]
     args = (meta.block_tables, meta.pos_ids, meta.seq_ids, scale, softcap, window, chunk)
+    if out is None:
+        out = q.new_empty(T, H * dv)
+        return ragged_attention(q, kc, vc, meta, scale, softcap, window, chunk, sink, out).view(T, H, dv)
     if not use_native(q):
-        return reference.paged_attention(q, kc, vc, *args)
-    ops = hybrid_ops()
-    if q.dtype != torch.bfloat16 or not ops.paged_tiled_ok(kc.shape[3], vc.shape[3]):
-        return ops.paged_generic(q, kc, vc, *args)
+        return out.copy_(reference.paged_attention(q, kc, vc, *args, sink).reshape(T, H * dv))
+    ops = attn_ops()
+    if q.dtype != torch.bfloat16 or not ops.paged_tiled_ok(kc.shape[3], dv):
+        return ops.paged_generic(q, kc, vc, *args, sink, out)
     nd = meta.n_decode
     if nd < len(meta.start_host):
-        o = ops.paged_prefill(q, kc, vc, meta.block_tables, meta.start_pos, meta.cu_q, meta.work, scale, softcap, window,
-                              chunk)
-    else:
-        o = q.new_empty(q.shape[0], q.shape[1], vc.shape[3])
+        ops.paged_prefill(q, kc, vc, meta.block_tables, meta.start_pos, meta.cu_q, meta.work, scale, softcap, window, chunk,
+                          sink, out)
     if nd:
         ops.paged_decode(q[:nd], kc, vc, meta.block_tables[:nd], meta.seq_lens[:nd], meta.max_len, scale, softcap, window,
-                         chunk, o)
-    return o
+                         chunk, out, sink)
+    return out
 
 
 def delta_rule(proj, conv_w, a_log, dt_bias, norm_w, eps, state, conv_state, meta, Hk, H, dk, dv):

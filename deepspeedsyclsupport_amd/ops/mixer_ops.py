@@ -1,8 +1,8 @@
 """Ops of hybrid decoders without residual streams (`inference/model_implementations/hybrid.py`): norms on sublayer
 outputs, latent attention, recurrences with a scalar decay per head, gated norms, token-side inputs.
 
-Device tensors run the gfx950 kernels of `ds_mixer_ops` (fp32 or bf16 storage); host tensors the plain versions in
-`ops/reference.py`, as everywhere in `ops`. Residual, norms, angles, scores, softmax, decays and the recurrent state are
+Device tensors run the gfx950 kernels of `ds_mixer_ops` and `ds_scan_ops` (fp32 or bf16 storage); host tensors the plain
+versions in `ops/reference.py`, as everywhere in `ops`. Residual, norms, angles, scores, softmax, decays and the recurrent state are
 fp32 whatever the storage type."""
 from dataclasses import dataclass
 
@@ -10,7 +10,7 @@ import torch
 import torch.nn.functional as F
 
 from . import reference
-from .native import mixer_ops, use_native
+from .native import mixer_ops, scan_ops, use_native
 
 
 def post_norm(x, y, w, eps, ids=None, embed=None, rows=None, final_w=None, mult=1.0):
@@ -32,12 +32,15 @@ def token_gate(g, ids, table, first):
     return f(g, ids, table, first)
 
 
-def gated_norm(y, proj, gate, w, parts, eps, mode):
-    """y [T, C] with the gate columns proj[:, gate:gate + C]. "silu_before": y silu(gate), then every one of `parts` equal
-    parts of a row by its own rms, times w. "sigmoid_after": the parts of y by their rms, times w sigmoid(gate)."""
-    before = {"silu_before": True, "sigmoid_after": False}[mode]
-    f = mixer_ops().gated_norm if use_native(y) else reference.gated_norm
-    return f(y, proj, gate, w, parts, eps, before)
+GATES = {"sigmoid_after": 0, "silu_before": 1, "silu_after": 2}
+
+
+def gated_norm(y, proj, gate, w, parts, eps, mode, out=None):
+    """y [T, C] with the gate columns proj[:, gate:gate + C]: every one of `parts` equal parts of a row by its own rms, times w
+    (None: no weight), times sigmoid(gate) or silu(gate); "silu_before": silu(gate) comes before the norm. `out`: where to
+    write (a matrix that may be columns of a wider one)."""
+    f = scan_ops().gated_norm if use_native(y) else reference.gated_norm
+    return f(y, proj, gate, w, parts, eps, GATES[mode], out)
 
 
 # ------------------------------------------------------------------------------------------------ latent attention
@@ -88,7 +91,7 @@ def latent_attention(q, lat, ukv, ukt, freq, sink, meta, scale, d, e):
 class ScanLayout:
     """Where a fused projection row [rows] holds what. q, k [Hk heads of dk], v [H heads of dv] and the output gate start
     at the given columns. With taps > 1, columns conv .. conv + channels (they hold q, k and v) pass a causal convolution
-    with bias; q, k and v pass silu either way. dt: first of H step-size columns, or -1 (constant decays, step 1)."""
+    with bias. dt: first of H step-size columns, or -1 (decays and steps from elsewhere)."""
     rows: int
     q: int
     k: int
@@ -109,21 +112,52 @@ class ScanLayout:
         return -(-self.dk // 8) * 8
 
 
-def decayed_scan(proj, lay, state, meta, conv_w=None, conv_b=None, conv_state=None, a_log=None, dt_bias=None, skip=None,
-                 log_decay=None):
-    """S_t = a_t S_(t-1) + b_t k_t v_t^T, o_t = S_t^T q_t + skip v_t for every head -> [T, H dv]; state slots
-    [slots, H, dv, dks] fp32 (and the convolution's windows) advance. Step sizes b = softplus(dt + dt_bias) with
-    a = exp(-exp(a_log) b), or b = 1 with a = exp(log_decay).
+    @property
+    def dims(self):
+        return (self.rows, self.q, self.k, self.v, self.Hk, self.H, self.dk, self.dv, self.taps, self.conv, self.channels,
+                self.dt)
 
-    Portions up to `RaggedMeta.STEP_TOKENS` go token by token, longer ones by chunks."""
-    ops = mixer_ops() if use_native(proj) else reference
-    dims = (lay.rows, lay.q, lay.k, lay.v, lay.Hk, lay.H, lay.dk, lay.dv, lay.taps, lay.conv, lay.channels, lay.dt)
-    qk, v, gb = ops.scan_prepare(proj, dims, conv_w, conv_b, conv_state, a_log, dt_bias, meta.seq_ids, meta.cu_q,
-                                 meta.start_pos, meta.slots)
+
+def _scan(ops, proj, lay, qk, v, gb, log_decay, skip, scale, state, zstate, floors, conv_state, meta):
     out = proj.new_empty(proj.shape[0], lay.H * lay.dv)
-    args = (qk, v, gb, log_decay, skip, proj, dims, state, conv_state)
+    args = (qk, v, gb, log_decay, skip, scale, proj, lay.dims, state, zstate, floors, conv_state)
     if meta.seq_list.numel():
         ops.scan_recur(*args, meta.seq_list, meta.cu_q, meta.start_pos, meta.slots, out)
     if meta.chunk_seqs.numel():
         ops.scan_chunk(*args, meta.chunk_seqs, meta.cu_q, meta.start_pos, meta.slots, out)
     return out
+
+
+def decayed_scan(proj, lay, state, meta, conv_w=None, conv_b=None, conv_state=None, a_log=None, dt_bias=None, skip=None,
+                 log_decay=None):
+    """S_t = a_t S_(t-1) + b_t k_t v_t^T, o_t = S_t^T q_t + skip v_t for every head -> [T, H dv]; state slots
+    [slots, H, dv, dks] fp32 (and the convolution's windows) advance. q, k and v pass silu. Step sizes b = softplus(dt +
+    dt_bias) with a = exp(-exp(a_log) b), or b = 1 with a = exp(log_decay).
+
+    Portions up to `RaggedMeta.STEP_TOKENS` go token by token, longer ones by chunks."""
+    ops = scan_ops() if use_native(proj) else reference
+    qk, v, gb = ops.scan_prepare(proj, lay.dims, conv_w, conv_b, conv_state, a_log, dt_bias, meta.seq_ids, meta.cu_q,
+                                 meta.start_pos, meta.slots)
+    return _scan(ops, proj, lay, qk, v, gb, log_decay, skip, 1.0, state, None, None, conv_state, meta)
+
+
+def retention(proj, lay, state, meta, log_decay, cs, scale):
+    """S_t = exp(log_decay) S_(t-1) + k_t v_t^T, o_t = scale S_t^T q_t; the pairs (i, i + half) of every head's first 2 half
+    columns of q and k are turned by cs [T, half, 2] (None: no rotation)."""
+    ops = scan_ops() if use_native(proj) else reference
+    qk, v = ops.scan_split(proj, lay.dims, cs)
+    return _scan(ops, proj, lay, qk, v, None, log_decay, None, scale, state, None, None, None, meta)
+
+
+def matrix_memory(proj, lay, slots, meta, gates, bi, bf, cap, scale):
+    """Exponentially gated recurrence with a normaliser. Gate columns gates, gates + H of the projection give, per head,
+    i = cap tanh((x + bi) / cap) and f = logsigmoid(cap tanh((x + bf) / cap)); m_t = max(f + m_(t-1), i) from m = 0, and
+    S_t = e^(f + m_(t-1) - m_t) S_(t-1) + e^(i - m_t) k v^T, z likewise with k alone, o = c S^T q / (max(|c z . q|, e^-m) + 1e-6)
+    with c = `scale`. `slots`: {"state": [.., H, dv, dks], "norm": [.., H, ceil(dv / 32), dks], "peak": [.., H]}."""
+    ops = scan_ops() if use_native(proj) else reference
+    cu = meta.cu_host
+    longest = max(b - a for a, b in zip(cu, cu[1:]))
+    gb, floors = ops.exp_gates(proj, gates, gates + lay.H, bi, bf, cap, slots["peak"], meta.cu_q, meta.start_pos, meta.slots,
+                               longest)
+    qk, v = ops.scan_split(proj, lay.dims, None)
+    return _scan(ops, proj, lay, qk, v, gb, None, None, scale, slots["state"], slots["norm"], floors, None, meta)

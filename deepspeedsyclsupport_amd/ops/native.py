@@ -20,14 +20,32 @@ def hip_ops():
 
 @functools.lru_cache(None)
 def hybrid_ops():
-    """The gfx950 ops of hybrid decoders with residual streams (a module of its own, see `op_builder.EXTENSIONS`)."""
+    """Residual streams, gated delta rule (the hybrid decoders' ops are modules by mechanism, see `op_builder.EXTENSIONS`)."""
     return op_builder.load("ds_hybrid_ops")
 
 
 @functools.lru_cache(None)
 def mixer_ops():
-    """The gfx950 ops of `ops/mixer_ops.py`."""
+    """Norms on sublayer outputs, latent attention, token-side gates."""
     return op_builder.load("ds_mixer_ops")
+
+
+@functools.lru_cache(None)
+def attn_ops():
+    """Attention over the paged cache in a ragged batch."""
+    return op_builder.load("ds_attn_ops")
+
+
+@functools.lru_cache(None)
+def scan_ops():
+    """Recurrences with a scalar decay per head, gated norms."""
+    return op_builder.load("ds_scan_ops")
+
+
+@functools.lru_cache(None)
+def expert_ops():
+    """Mixture of experts with grouped routing, pre-norm residual."""
+    return op_builder.load("ds_expert_ops")
 
 
 @functools.lru_cache(None)

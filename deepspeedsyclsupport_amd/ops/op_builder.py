@@ -58,8 +58,8 @@ EXTENSIONS = {
         "bindings": ["bind/ds_hip_ops.cpp", "bind/infer_bind.cpp", "bind/moe_bind.cpp", "bind/host_mem.cpp",
                      "bind/comm_bind.cpp", "bind/attn_small_bind.cpp"],
     },
-    # what serving the hybrid decoders (inference/model_implementations/hybrid.py) needs, and nothing else: in a fresh
-    # checkout such a model starts after compiling the decode products and its own mixers' sources only
+    # what serving the hybrid decoders (inference/model_implementations/hybrid.py) needs, mechanism by mechanism: in a fresh
+    # checkout such a model starts after compiling the decode products and the sources of what it is made of
     "ds_gemv_ops": {
         "kind": "hip",
         "kernels": [
@@ -70,7 +70,41 @@ EXTENSIONS = {
         ],
         "bindings": ["bind/gemv_bind.cpp"],
     },
-    # norms on sublayer outputs, latent attention, recurrences with a scalar decay per head
+    # attention over the paged cache: QKV epilogues, prefill, decode
+    "ds_attn_ops": {
+        "kind": "hip",
+        "kernels": [
+            "attn/qk_norm_append.hip",
+            "attn/qk_rope_append.hip",
+            "attn/paged_generic.hip",
+            "attn/paged_prefill.hip",
+            "attn/decode_attn.hip",
+        ],
+        "bindings": ["bind/paged_bind.cpp"],
+    },
+    # recurrences with a scalar decay per head, gated norms
+    "ds_scan_ops": {
+        "kind": "hip",
+        "kernels": [
+            "norm/gated_norm.hip",
+            "recur/exp_gates.hip",
+            "recur/decayed_scan.hip",
+            "recur/decayed_chunk.hip",
+        ],
+        "bindings": ["bind/scan_bind.cpp"],
+    },
+    # mixture of experts with grouped routing, pre-norm residual
+    "ds_expert_ops": {
+        "kind": "hip",
+        "kernels": [
+            "norm/pre_norm.hip",
+            "act/clamped_glu.hip",
+            "moe/expert_route.hip",
+            "moe/expert_gemm.hip",
+        ],
+        "bindings": ["bind/expert_bind.cpp"],
+    },
+    # norms on sublayer outputs, token-side gates, latent attention
     "ds_mixer_ops": {
         "kind": "hip",
         "kernels": [
@@ -80,21 +114,15 @@ EXTENSIONS = {
             "attn/latent_decode.hip",
             "attn/latent_prefill.hip",
             "attn/paged_generic.hip",
-            "recur/decayed_scan.hip",
-            "recur/decayed_chunk.hip",
         ],
         "bindings": ["bind/mixer_bind.cpp"],
     },
-    # residual streams, attention with head norms, gated delta rule
+    # residual streams, gated delta rule
     "ds_hybrid_ops": {
         "kind": "hip",
         "kernels": [
             "norm/stream_norm.hip",
             "act/clamped_glu.hip",
-            "attn/qk_norm_append.hip",
-            "attn/paged_generic.hip",
-            "attn/paged_prefill.hip",
-            "attn/decode_attn.hip",
             "recur/delta_rule.hip",
             "recur/delta_chunk.hip",
         ],
@@ -225,6 +253,14 @@ def build(names=None, verbose=False, jobs=None):
 
 def is_built(name):
     return os.path.exists(so_path(name))
+
+
+def prepare(names):
+    """Build those of the named extensions that are missing, in one go."""
+    with _lock:
+        missing = [n for n in names if n not in _loaded and not is_built(n)]
+        if missing:
+            build(missing)
 
 
 def load(name, build_if_missing=True):

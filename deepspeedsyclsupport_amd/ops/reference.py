@@ -167,7 +167,34 @@ def qk_norm_append(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc,
     return q.to(qkv.dtype)
 
 
-def paged_attention(q, kc, vc, block_table, pos, seq_ids, scale, softcap, window, chunk):
+def rope_table(pos, freq):
+    a = pos.double()[:, None] * freq.double()
+    return torch.stack([a.cos(), a.sin()], -1).float()
+
+
+def _turn_pairs(x, cs):
+    """x [T, heads, d]: pairs (i, i + half) turned by cs [T, half, 2]."""
+    if cs is None:
+        return x
+    h, (c, s) = cs.shape[1], cs[:, None].unbind(-1)
+    u, v = x[..., :h], x[..., h:2 * h]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * h:]], -1)
+
+
+def qk_rope_append(qkv, bias, qw, kw, eps, cs, v_mult, pos, seq_ids, block_table, kc, vc, H):
+    G, BS, dk, dv = kc.shape[1], kc.shape[2], kc.shape[3], vc.shape[3]
+    T = qkv.shape[0]
+    q, k, v = (qkv.float() if bias is None else qkv.float() + bias).split([H * dk, G * dk, G * dv], -1)
+    q, k = (x if w is None else _rms(x, eps) * w for x, w in ((q, qw), (k, kw)))
+    q, k, v = _turn_pairs(q.view(T, H, dk), cs), _turn_pairs(k.view(T, G, dk), cs), v.reshape(T, G, dv) * v_mult
+    slot = pos.long()
+    blk = block_table.long()[seq_ids.long(), slot // BS]
+    kc[blk, :, slot % BS] = k.to(kc.dtype)
+    vc[blk, :, slot % BS] = v.to(vc.dtype)
+    return q.to(qkv.dtype)
+
+
+def paged_attention(q, kc, vc, block_table, pos, seq_ids, scale, softcap, window, chunk, sink=None):
     """q [T, H, dk] at absolute positions -> [T, H, dv]; visible keys [lo(pos), pos] (window / chunk start / 0)."""
     G, BS = kc.shape[1], kc.shape[2]
     out = q.new_empty(q.shape[0], q.shape[1], vc.shape[3])
@@ -181,7 +208,11 @@ def paged_attention(q, kc, vc, block_table, pos, seq_ids, scale, softcap, window
         s = torch.einsum("grd,ngd->grn", qq, k) * scale
         if softcap:
             s = softcap * torch.tanh(s / softcap)
-        out[t] = torch.einsum("grn,ngd->grd", s.softmax(-1), v).reshape(q.shape[1], -1).to(q.dtype)
+        if sink is not None:
+            p = torch.cat([s, sink.view(G, -1, 1)], -1).softmax(-1)[..., :-1]
+        else:
+            p = s.softmax(-1)
+        out[t] = torch.einsum("grn,ngd->grd", p, v).reshape(q.shape[1], -1).to(q.dtype)
     return out
 
 
@@ -257,13 +288,14 @@ def token_gate(g, ids, table, first):
     return (F.gelu(g.float(), approximate="tanh") * e).to(g.dtype)
 
 
-def gated_norm(y, proj, gate, w, parts, eps, before):
+def gated_norm(y, proj, gate, w, parts, eps, mode, out=None):
     T, C = y.shape
     g, v = proj[:, gate:gate + C].float(), y.float()
-    if before:
+    if mode == 1:
         v = v * F.silu(g)
-    v = _rms(v.view(T, parts, C // parts), eps).view(T, C) * w
-    return (v if before else v * torch.sigmoid(g)).to(y.dtype)
+    v = _rms(v.view(T, parts, C // parts), eps).view(T, C) * (1.0 if w is None else w)
+    v = (v * torch.sigmoid(g) if mode == 0 else v * F.silu(g) if mode == 2 else v).to(y.dtype)
+    return v if out is None else out.copy_(v)
 
 
 def _turn(x, freq, pos):
@@ -326,26 +358,96 @@ def scan_prepare(proj, dims, conv_w, conv_b, conv_state, a_log, dt_bias, seq_ids
     return qk, part(D["v"], D["H"], D["dv"]), gb
 
 
-def scan_recur(qk, v, gb, log_decay, skip, proj, dims, state, conv_state, seqs, cu, start, slots, out):
+def scan_split(proj, dims, cs):
+    D = _scan_dims(dims)
+    part = lambda at, n, w: proj[:, at:at + n * w].reshape(-1, n, w)
+    q, k = (_turn_pairs(part(D[c], D["Hk"], D["dk"]).float(), cs).to(proj.dtype) for c in "qk")
+    return torch.stack([q, k], 1), part(D["v"], D["H"], D["dv"])
+
+
+def exp_gates(proj, ci, cf, bi, bf, cap, peak, cu, start, slots, longest):
+    H = bi.numel()
+    i = cap * torch.tanh((proj[:, ci:ci + H].float() + bi) / cap)
+    f = F.logsigmoid(cap * torch.tanh((proj[:, cf:cf + H].float() + bf) / cap))
+    gb, floors = torch.empty(proj.shape[0], 2, H), torch.empty(proj.shape[0], H)
+    for s in range(start.numel()):
+        m = peak[int(slots[s])].clone() if int(start[s]) else torch.zeros(H)
+        for t in range(int(cu[s]), int(cu[s + 1])):
+            new = torch.maximum(f[t] + m, i[t])
+            gb[t, 0], gb[t, 1], floors[t], m = f[t] + m - new, (i[t] - new).exp(), (-new).exp(), new
+        peak[int(slots[s])] = m
+    return gb, floors
+
+
+def scan_recur(qk, v, gb, log_decay, skip, scale, proj, dims, state, zstate, floors, conv_state, seqs, cu, start, slots, out):
     D = _scan_dims(dims)
     T, H, dk = proj.shape[0], D["H"], D["dk"]
     rep, out = H // D["Hk"], out.view(T, H, D["dv"])
     for i in seqs.tolist():
-        a, b, slot = int(cu[i]), int(cu[i + 1]), int(slots[i])
-        S = state[slot, ..., :dk].transpose(1, 2).clone() if int(start[i]) else torch.zeros(H, dk, D["dv"])
+        a, b, slot, old = int(cu[i]), int(cu[i + 1]), int(slots[i]), int(start[i]) > 0
+        S = state[slot, ..., :dk].transpose(1, 2).clone() if old else torch.zeros(H, dk, D["dv"])
+        Z = zstate[slot, :, 0, :dk].clone() if zstate is not None and old else torch.zeros(H, dk)
         for t in range(a, b):
             q, k = qk[t].float().repeat_interleave(rep, 1)
             g, step = (gb[t, 0], gb[t, 1]) if gb is not None else (log_decay, torch.ones(H))
             S = S * g.exp()[:, None, None] + (k * step[:, None])[:, :, None] * v[t].float()[:, None]
-            o = (S * q[:, :, None]).sum(1)
+            o = scale * (S * q[:, :, None]).sum(1)
+            if zstate is not None:
+                Z = Z * g.exp()[:, None] + k * step[:, None]
+                o = o / (torch.maximum((scale * (Z * q).sum(-1)).abs(), floors[t]) + 1e-6)[:, None]
             out[t] = (o if skip is None else o + skip[:, None] * v[t].float()).to(out.dtype)
         state[slot, ..., :dk] = S.transpose(1, 2)
+        if zstate is not None:
+            zstate[slot, ..., :dk] = Z[:, None]
         if conv_state is not None and conv_state.shape[1]:
-            old = conv_state[slot] if int(start[i]) else torch.zeros_like(conv_state[slot])
+            before = conv_state[slot] if old else torch.zeros_like(conv_state[slot])
             new = proj[a:b, D["conv"]:D["conv"] + D["channels"]]
-            conv_state[slot] = torch.cat([old, new])[-(D["taps"] - 1):].clone()
+            conv_state[slot] = torch.cat([before, new])[-(D["taps"] - 1):].clone()
 
 
-def scan_chunk(qk, v, gb, log_decay, skip, proj, dims, state, conv_state, seqs, cu, start, slots, out):
+def scan_chunk(qk, v, gb, log_decay, skip, scale, proj, dims, state, zstate, floors, conv_state, seqs, cu, start, slots, out):
     """Long portions: the same recurrence (the device splits it into chunks)."""
-    scan_recur(qk, v, gb, log_decay, skip, proj, dims, state, conv_state, seqs[:, 0], cu, start, slots, out)
+    scan_recur(qk, v, gb, log_decay, skip, scale, proj, dims, state, zstate, floors, conv_state, seqs[:, 0], cu, start, slots,
+               out)
+
+
+# ---------------------------------------------------------------- pre-norm residual, experts with grouped routing
+def expert_sum(y, w, rows):
+    T, K = w.shape
+    e = y.float()[rows.long().view(-1)] if rows is not None else y.float()
+    return (e.view(T, K, -1) * w[..., None]).sum(1).to(y.dtype)
+
+
+def pre_norm(x, y, yw, yrow, w, eps, ids, embed, mult, rows):
+    if y is None:
+        x.copy_(embed.float()[ids.long()] * mult)
+        return (_rms(x, eps) * w).to(embed.dtype)
+    s = x + (y.float() if yw is None else expert_sum(y.float(), yw, yrow))
+    if rows is not None:
+        return (_rms(s[rows.long()], eps) * w).to(y.dtype)
+    x.copy_(s)
+    return (_rms(s, eps) * w).to(y.dtype)
+
+
+def route(h, router, k, groups, keep):
+    s = (h.float() @ router.float().t()).softmax(-1)
+    T, E = s.shape
+    best = s.view(T, groups, E // groups).amax(-1).topk(keep, -1).indices
+    open_ = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best, True).repeat_interleave(E // groups, 1)
+    w, e = s.masked_fill(~open_, -1.0).topk(k, -1)
+    return e.to(torch.int32), w / (w.sum(-1, keepdim=True) + 1e-20)
+
+
+def silu_mul(gu):
+    g, u = gu.float().chunk(2, -1)
+    return (F.silu(g) * u).to(gu.dtype)
+
+
+def expert_gemm(x, w, experts, div, gated):
+    out = x.new_empty(experts.numel(), w.shape[1] // (2 if gated else 1))
+    e = experts.view(-1).long()
+    for i in e.unique().tolist():
+        r = (e == i).nonzero().view(-1)
+        y = F.linear(x[r // div], w[i])
+        out[r] = silu_mul(y) if gated else y
+    return out

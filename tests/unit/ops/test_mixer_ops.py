@@ -265,15 +265,15 @@ def test_decayed_scan(device, dtype, tol, H, Hk, dk, dv, taps):
 @pytest.mark.parametrize("dk,dv", [(16, 16), (64, 64), (128, 80), (200, 64)])
 def test_chunk_state_is_fp32(dk, dv):
     """The chunked state against fp64, to fp32 precision, from the activations as the device rounds them."""
-    from deepspeedsyclsupport_amd.ops.native import mixer_ops
+    from deepspeedsyclsupport_amd.ops.native import scan_ops
     H, n = 2, 333
     la = scan_layout(H, H, dk, dv, 0)
     proj = rnd(n, la.rows, seed=3).bfloat16()
     ld = torch.tensor([-0.002, -0.3])
     m, _ = meta([(0, n)], "cuda", slots=[0])
     dims = (la.rows, la.q, la.k, la.v, la.Hk, la.H, la.dk, la.dv, la.taps, la.conv, la.channels, la.dt)
-    qk, v_act, _ = mixer_ops().scan_prepare(proj.cuda(), dims, None, None, None, None, None, m.seq_ids, m.cu_q, m.start_pos,
-                                            m.slots)
+    qk, v_act, _ = scan_ops().scan_prepare(proj.cuda(), dims, None, None, None, None, None, m.seq_ids, m.cu_q, m.start_pos,
+                                           m.slots)
     state = torch.zeros(1, H, dv, -(-dk // 8) * 8, device="cuda")
     ops.decayed_scan(proj.cuda(), la, state, m, log_decay=ld.cuda())
     for h in range(H):
