@@ -3,8 +3,11 @@ counts, all through the ragged engine with random bf16 weights: whole-prompt pre
 
 * hybrid: Vopepel layers (gated delta rule, chunked attention, residual streams)
 * perelorn: Perelorn layers (Mamba-2, latent attention, lightning attention, norms on sublayer outputs, token-side input)
+* lefisun: Lefisun layers (chunked rotary attention beside a matrix memory, retention, routed experts); beside it
+  uniform_moe, the Llama-style decoder with the same experts (Mixtral's routing), and the others with a dense feed-forward as
+  wide as the experts of a token together
 
-    python bench.py --workload hybrid [--sizes 2048,4096] [--model-kind hybrid|perelorn|uniform|both|all]
+    python bench.py --workload hybrid [--sizes 2048,4096] [--model-kind hybrid|perelorn|lefisun|uniform|uniform_moe|both|moe|all]
 """
 import json
 import math
@@ -20,7 +23,11 @@ HEAD, CHUNK, STREAMS, VOCAB, SIDE = 128, 2048, 4, 32000, 256
 # Perelorn: the delta layers' places go to Mamba-2 and lightning, attention to latent attention; every layer keeps its
 # feed-forward, so that the projections are of one size
 PERELORN = ("mamba2", "latent_attention", "lightning", "mamba2", "latent_attention", "lightning", "mamba2", "latent_attention")
-KINDS = {"both": ("hybrid", "uniform"), "all": ("hybrid", "perelorn", "uniform")}
+KINDS = {"both": ("hybrid", "uniform"), "moe": ("lefisun", "uniform_moe"),
+         "all": ("hybrid", "perelorn", "uniform", "lefisun", "uniform_moe")}
+# Lefisun: attention of the others' size beside a memory of half its heads, retention in the places of their recurrences
+EXPERTS, TOP, GROUPS, KEEP = 32, 4, 4, 2
+LEFISUN = ("parallel", "retention") * 4
 
 
 def specs(width):
@@ -44,7 +51,20 @@ def specs(width):
     perelorn = DSModelSpec(arch="perelorn", norm="rms", pos="none", residual="post_norm", token_side=SIDE, logit_scale=1.0,
                            layer_specs=tuple({"type": t, "mixer": mixers[t], "mlp": {"kind": "gelu", "ff": s["ff"]}}
                                              for t in PERELORN), **common)
-    return {"hybrid": hybrid, "perelorn": perelorn, "uniform": uniform}
+    ff = s["ff"] // TOP
+    mixers = {"parallel": {"left": {"heads": h, "kv_heads": s["kv"], "dim": HEAD, "vdim": HEAD, "scale": HEAD**-0.5,
+                                    "mask": {"size": CHUNK}, "rot": {"base": 5e5, "dims": HEAD // 2, "scaling": {"factor": 4.0}}},
+                           "right": {"heads": h // 2, "dim": HEAD, "vdim": HEAD, "gate_cap": 15.0},
+                           "left_scale": 0.8, "right_scale": 0.6},
+              "retention": {"heads": h, "dim": HEAD, "vdim": HEAD, "rot": {"base": 1e4, "dims": HEAD},
+                            "decay": [1 - 2**(-5 - 3 * i / h) for i in range(h)]}}
+    mlp = {"kind": "routed", "expert": {"ff": ff}, "router": {"experts": EXPERTS, "top": TOP, "groups": {"count": GROUPS,
+                                                                                                        "keep": KEEP}}}
+    lefisun = DSModelSpec(arch="lefisun", norm="rms", pos="none", residual="pre_norm", tie_embeddings=True,
+                          layer_specs=tuple({"type": t, "mixer": mixers[t], "mlp": mlp} for t in LEFISUN), **common)
+    uniform_moe = DSModelSpec(arch="mixtral", norm="rms", pos="rope", max_positions=16384, num_experts=EXPERTS, moe_top_k=TOP,
+                              **{**common, "intermediate_size": ff})
+    return {"hybrid": hybrid, "perelorn": perelorn, "uniform": uniform, "lefisun": lefisun, "uniform_moe": uniform_moe}
 
 
 def build(spec, device, blocks):

@@ -97,9 +97,11 @@ def layer_container(layer, streams=False, may_lack=(), side=False):
 
 
 def _renamed(layers, kinds):
-    """A config's layers with its names of feed-forwards replaced by the package's."""
-    return [{**la, "mlp": {**la["mlp"], "kind": kinds.get(la["mlp"].get("kind"), la["mlp"].get("kind"))}
-             if la.get("mlp") else None} for la in layers]
+    """A config's layers with its names of feed-forwards replaced by the package's ({config's: package's}, no others)."""
+    for i, la in enumerate(layers):
+        if la.get("mlp") and la["mlp"].get("kind") not in kinds:
+            raise NotImplementedError(f"layer {i}: no feed-forward {la['mlp'].get('kind')!r}")
+    return [{**la, "mlp": {**la["mlp"], "kind": kinds[la["mlp"]["kind"]]} if la.get("mlp") else None} for la in layers]
 
 
 _TOP_TENSORS = {"embed": "embed", "final.norm": "norm_w", "head": "lm_head"}

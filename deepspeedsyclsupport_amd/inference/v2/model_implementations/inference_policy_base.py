@@ -61,8 +61,8 @@ class ContainerMap:
                 idx = int(m.group(1))
                 if idx >= len(self._transformer_params):
                     raise ValueError(f"{name}: layer {idx} is beyond the model's {len(self._transformer_params)}")
-                if not self._transformer_params[idx].set_dependency(m.group(2), parameter) \
-                        and not self._ignored(name):
+                container = self._transformer_params[idx]  # (None: the layer is complete and loaded)
+                if (container is None or not container.set_dependency(m.group(2), parameter)) and not self._ignored(name):
                     raise ValueError(f"Cannot find container for {name}, please double check the Containers/"
                                      f"ContainerMap")
                 return idx

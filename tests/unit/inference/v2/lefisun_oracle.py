@@ -177,3 +177,115 @@ def forward(cfg, weights, tokens, cast=torch.float64, trace=None):
         if trace is not None:
             trace.append(x)
     return project(rms(x, eps) * w["final.norm"], w["embed"])
+
+
+# ------------------------------------------------------------------------------------------------ test models
+CODE = 8   # columns of the residual that `decisive` models keep for the router
+
+
+def random_model(cfg, seed=0, dtype=torch.bfloat16, decisive=False):
+    """Random weights for a config. `decisive`: the last `CODE` columns of the residual belong to the router alone (no sublayer
+    writes them, the embedding does), with values drawn anew until no token comes near a tie in any layer. Rounding then cannot
+    change an expert, so that whole models compare in 16 bits."""
+    g = torch.Generator().manual_seed(seed)
+    W, w = cfg["width"], {}
+
+    def put(name, shape, std=None, mean=0.0):
+        std = std if std is not None else 1 / math.sqrt(shape[-1])
+        w[name] = (torch.randn(shape, generator=g) * std + mean).to(dtype)
+
+    put("embed", (cfg["vocab"], W), 1.0 / cfg["embedding"]["scale"])
+    put("final.norm", (W, ), 0.1, 1.0 / math.sqrt(W))
+    w["final.norm"] *= cfg["embedding"]["scale"]
+    for i, layer in enumerate(cfg["layers"]):
+        p, mx = f"l{i}.", layer["mixer"]
+        put(p + "norm1", (W, ), 0.2, 0.9)
+        if layer["type"] == "parallel":
+            le, ri = mx["left"], mx["right"]
+            q = p + "mix.left."
+            for n, rows in (("q", le["heads"] * le["dim"]), ("k", le["kv_heads"] * le["dim"]), ("v", le["kv_heads"] * le["vdim"])):
+                put(q + n, (rows, W))
+                put(q + n + ".b", (rows, ), 0.5)
+            put(q + "q.norm", (le["heads"] * le["dim"], ), 0.2, 1.0)
+            put(q + "k.norm", (le["kv_heads"] * le["dim"], ), 0.2, 1.0)
+            put(q + "o", (W, le["heads"] * le["vdim"]))
+            q, H = p + "mix.right.", ri["heads"]
+            for n, rows in (("q", H * ri["dim"]), ("k", H * ri["dim"]), ("v", H * ri["vdim"]), ("g", H * ri["vdim"]), ("i", H),
+                            ("f", H)):
+                put(q + n, (rows, W))
+            put(q + "i.b", (H, ), 1.0)
+            put(q + "f.b", (H, ), 1.5, 2.0)
+            put(q + "norm", (H * ri["vdim"], ), 0.2, 1.0)
+            put(q + "o", (W, H * ri["vdim"]))
+        else:
+            H = mx["heads"]
+            for n, rows in (("q", H * mx["dim"]), ("k", H * mx["dim"]), ("v", H * mx["vdim"]), ("g", H * mx["vdim"])):
+                put(p + f"mix.{n}", (rows, W))
+            put(p + "mix.o", (W, H * mx["vdim"]))
+        if layer.get("mlp"):
+            F, E = layer["mlp"]["expert"]["ff"], layer["mlp"]["router"]["experts"]
+            put(p + "norm2", (W, ), 0.2, 0.9)
+            put(p + "mlp.router", (E, W), 1.5 / math.sqrt(W))
+            for e in range(E):
+                put(p + f"mlp.e{e}.gate", (F, W))
+                put(p + f"mlp.e{e}.up", (F, W))
+                put(p + f"mlp.e{e}.down", (W, F))
+    if decisive:
+        _decide(cfg, w, g)
+    return w
+
+
+def _decide(cfg, w, g):
+    routed = [(f"l{i}.", la["mlp"]["router"]) for i, la in enumerate(cfg["layers"]) if la.get("mlp")]
+    for name in w:
+        if name.endswith(("mix.o", "left.o", "right.o", ".down")):
+            w[name][-CODE:] = 0
+    for p, _ in routed:
+        w[p + "mlp.router"] *= 6
+        w[p + "mlp.router"][:, :-CODE] = 0
+    todo = torch.arange(cfg["vocab"])
+    for _ in range(500):
+        w["embed"][todo, -CODE:] = (torch.randn(len(todo), CODE, generator=g) / cfg["embedding"]["scale"]).to(w["embed"].dtype)
+        c = w["embed"][todo, -CODE:].double()
+        near = torch.zeros(len(todo), dtype=torch.bool)
+        for p, r in routed:
+            z = (c * w[p + "norm2"][-CODE:].double()) @ w[p + "mlp.router"][:, -CODE:].double().t()
+            unit = z.std(-1) * 0.05
+            n, (count, keep, top) = len(todo), (r["groups"]["count"], r["groups"]["keep"], r["top"])
+            best = z.view(n, count, -1).max(-1).values.sort(-1, descending=True).values
+            if keep < count:
+                near |= best[:, keep - 1] - best[:, keep] < unit
+            allowed = z.view(n, count, -1).masked_fill((z.view(n, count, -1).max(-1).values < best[:, keep - 1:keep])[..., None],
+                                                       -math.inf).view(n, -1).sort(-1, descending=True).values
+            if top < z.shape[1]:
+                near |= allowed[:, top - 1] - allowed[:, top] < unit
+        todo = todo[near]
+        if not len(todo):
+            return
+    raise AssertionError("no routing without near ties")
+
+
+def parallel_layer(heads=4, kv_heads=2, dim=16, vdim=24, size=40, rot=8, base=1000.0, factor=2.0, scale=None, left_scale=0.7,
+                   right_scale=0.6, r_heads=2, r_dim=16, r_vdim=24, cap=8.0, mlp=None):
+    return {"type": "parallel",
+            "mixer": {"left": {"dim": dim, "heads": heads, "kv_heads": kv_heads, "mask": {"size": size},
+                               "rot": {"base": base, "dims": rot, "scaling": {"factor": factor}},
+                               "scale": scale or dim**-0.5, "vdim": vdim},
+                      "left_scale": left_scale, "right": {"dim": r_dim, "gate_cap": cap, "heads": r_heads, "vdim": r_vdim},
+                      "right_scale": right_scale}, "mlp": mlp}
+
+
+def retention_layer(heads=3, dim=16, vdim=24, decay=None, rot=None, base=5000.0, mlp=None):
+    decay = decay or [1 - 2.0**-(2 * i + 3) for i in range(heads)]
+    return {"type": "retention", "mixer": {"decay": decay, "dim": dim, "heads": heads,
+                                           "rot": {"base": base, "dims": dim if rot is None else rot}, "vdim": vdim}, "mlp": mlp}
+
+
+def moe(experts=6, top=2, count=3, keep=2, ff=32):
+    return {"expert": {"ff": ff}, "kind": "moe", "router": {"experts": experts, "groups": {"count": count, "keep": keep},
+                                                            "top": top}}
+
+
+def config(layers, vocab=97, width=64, scale=1.7, eps=1e-5):
+    return {"architecture": "Lefisun", "embedding": {"scale": scale}, "layers": layers, "norm": {"eps": eps}, "vocab": vocab,
+            "width": width}
