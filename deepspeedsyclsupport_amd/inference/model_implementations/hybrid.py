@@ -658,6 +658,10 @@ class MLP:
         """Shapes of the weight matrices, by name."""
         return {"fc1_w": (self.rows, width), "fc2_w": (width, self.ff)}
 
+    def operand_order(self, layer):
+        """Copies for decoding of weights that are no plain projections."""
+        return {}
+
 
 class ClampedMLP(MLP):
     """Gated feed-forward whose branches are clamped before the product."""
@@ -730,8 +734,16 @@ class RoutedMLP(MLP):
                                                                 _shard(lw["experts_up"], r, tp, 1)], 1),
                 "fc2_w": _shard(lw["experts_down"], r, tp, 2)}
 
+    def operand_order(self, layer):
+        """The expert weights once more as the products read them best, by name (nothing where the sizes forbid it)."""
+        if self.ff % 32:   # (gate and up rows are tiled on their own)
+            return {}
+        both = expert_ops.operand_order(layer.fc1_w.data), expert_ops.operand_order(layer.fc2_w.data)
+        return {} if any(w is None for w in both) else {"experts": both}
+
     def run(self, layer, h):
-        y = expert_ops.experts(h, layer.router_w, layer.fc1_w, layer.fc2_w, self.top, self.groups, self.keep)
+        y = expert_ops.experts(h, layer.router_w, layer.fc1_w, layer.fc2_w, self.top, self.groups, self.keep,
+                               layer.sh.get("experts"))
         return y if layer.tp == 1 else y.sum()   # ranks exchange plain sums
 
 
@@ -802,6 +814,8 @@ class DSHybridLayer(ProjectionLayer):
             return False
         self.sh = {n: Bf16Weight(w.data) for n, w in ((n, getattr(self, n)) for n in self.projection_names())
                    if w.is_cuda and Bf16Weight.supported(w.data)}
+        if self.mlp:
+            self.sh.update(self.mlp.operand_order(self))
         return bool(self.sh)
 
     def shard(self, lw, r, tp):

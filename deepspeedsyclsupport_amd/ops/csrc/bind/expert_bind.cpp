@@ -10,8 +10,9 @@ int ds_route(const void*, const void*, int*, float*, int*, int*, int, int, int, 
 int ds_expert_place(const int*, const int*, const int*, int*, int*, int*, int, int, hipStream_t);
 int ds_expert_spread(const void*, const int*, void*, int, int, int64_t, hipStream_t);
 int ds_expert_few();
+int ds_expert_order_ok(int, int);
 int ds_expert_gemm(const void*, const void*, void*, const int*, const int*, const int*, int, int, int, int, int, int, int, int,
-                   hipStream_t);
+                   int, hipStream_t);
 int ds_expert_sum(const void*, const float*, const int*, void*, int, int, int, int, hipStream_t);
 int ds_clamped_glu(const void*, void*, int64_t, int, float, float, float, int, hipStream_t);
 }
@@ -81,20 +82,21 @@ Tensor expert_spread(Tensor x, Tensor rows) {
 
 int64_t expert_few() { return ds_expert_few(); }
 
+bool expert_order_ok(int64_t N, int64_t K) { return ds_expert_order_ok((int)N, (int)K); }
+
 // x [rows, K], w [E, N or 2 N, K], experts [entries] -> y [entries, N]: y[i] = w[experts[i]] x[i / div], gated: silu(first N
-// rows) times the last N. offs, order: lists from `route`
-Tensor expert_gemm(Tensor x, Tensor w, Tensor experts, OptT offs, OptT order, int64_t div, bool gated) {
+// rows) times the last N. offs, order: lists from `route`. operand: the elements of w are in operand order; tile: many rows per
+// expert (operand order and lists only)
+Tensor expert_gemm(Tensor x, Tensor w, Tensor experts, OptT offs, OptT order, int64_t div, bool gated, bool operand, bool tile) {
   need(x, "x"); need(w, "w");
   const int64_t entries = experts.numel(), E = w.size(0), K = w.size(2), N = w.size(1) / (gated ? 2 : 1);
   TORCH_CHECK(x.dim() == 2 && w.dim() == 3 && x.size(1) == K && x.scalar_type() == w.scalar_type() && E <= 256 &&
               (!gated || w.size(1) % 2 == 0) && div > 0 && entries % div == 0 && x.size(0) == entries / div, "expert_gemm: shapes");
   TORCH_CHECK(has(offs) == has(order), "expert_gemm: lists");
   auto y = torch::empty({entries, N}, x.options());
-  // (a token names an expert at most once)
-  const int64_t most = div > 1 ? x.size(0) : entries / std::max<int64_t>(experts.size(-1), 1);
   check(ds_expert_gemm(x.data_ptr(), w.data_ptr(), y.data_ptr(), i32(experts, entries, "experts"),
                        has(offs) ? i32(*offs, E + 1, "offs") : nullptr, has(order) ? i32(*order, entries, "order") : nullptr,
-                       (int)entries, (int)most, (int)E, (int)N, (int)K, (int)div, gated, dcode(x), stream()), "expert_gemm");
+                       (int)entries, (int)E, (int)N, (int)K, (int)div, gated, operand, tile, dcode(x), stream()), "expert_gemm");
   return y;
 }
 
@@ -125,6 +127,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("route", &route);
   m.def("expert_spread", &expert_spread);
   m.def("expert_few", &expert_few);
+  m.def("expert_order_ok", &expert_order_ok);
   m.def("expert_gemm", &expert_gemm);
   m.def("expert_sum", &expert_sum);
   m.def("silu_mul", &silu_mul);

@@ -11,6 +11,11 @@ namespace {
 
 constexpr int MAXE = 256, MAXK = 64;
 
+template <int N>
+struct Int {
+  static constexpr int value = N;
+};
+
 __device__ __forceinline__ f32x4 mfma(bf16x8 a, bf16x8 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
 }
@@ -122,7 +127,8 @@ __global__ void __launch_bounds__(64 * NW) route_mfma_kernel(const bf16* __restr
                                                              RouteArgs a) {
   constexpr int TOK = 16 * TM, ZP = 16 * ET + 1;
   __shared__ float z[TOK * ZP];
-  __shared__ float gs[NW][MAXE];
+  __shared__ f32x4 red[NW / 2][TM * ET][64];
+  __shared__ float gs[NW][16 * ET];
   __shared__ int hist[MAXE];
   const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, q4 = lane >> 4, w = tid >> 6;
   const int t0 = blockIdx.x * TOK, n = min(TOK, a.T - t0);
@@ -137,38 +143,64 @@ __global__ void __launch_bounds__(64 * NW) route_mfma_kernel(const bf16* __restr
   for (int m = 0; m < TM; ++m) hp[m] = h + (int64_t)(t0 + min(16 * m + l16, n - 1)) * a.W;
 #pragma unroll
   for (int e = 0; e < ET; ++e) wp[e] = rw + (int64_t)min(16 * e + l16, a.E - 1) * a.W;
-  for (int k0 = 32 * w; k0 < a.W; k0 += 32 * NW) {
-    const int k = k0 + 8 * q4, kc = min(k, a.W - 8);
-    bf16x8 x[TM], y[ET];
+  // U steps of 32 of the width: all their loads, then the products
+  auto steps = [&](auto count, int k0, bool tail) {
+    constexpr int U = decltype(count)::value;
+    bf16x8 x[U][TM], y[U][ET];
 #pragma unroll
-    for (int e = 0; e < ET; ++e) y[e] = *reinterpret_cast<const bf16x8*>(wp[e] + kc);
+    for (int u = 0; u < U; ++u) {
+      const int k = k0 + 32 * NW * u + 8 * q4, kc = tail ? min(k, a.W - 8) : k;
 #pragma unroll
-    for (int m = 0; m < TM; ++m) x[m] = *reinterpret_cast<const bf16x8*>(hp[m] + kc);
-    if (k >= a.W) {  // the last step may reach past the width
+      for (int e = 0; e < ET; ++e) y[u][e] = *reinterpret_cast<const bf16x8*>(wp[e] + kc);
 #pragma unroll
-      for (int m = 0; m < TM; ++m)
+      for (int m = 0; m < TM; ++m) x[u][m] = *reinterpret_cast<const bf16x8*>(hp[m] + kc);
+      if (tail && k >= a.W) {  // the last step may reach past the width
 #pragma unroll
-        for (int j = 0; j < 8; ++j) x[m][j] = (bf16)0.f;
+        for (int m = 0; m < TM; ++m)
+#pragma unroll
+          for (int j = 0; j < 8; ++j) x[u][m][j] = (bf16)0.f;
+      }
     }
 #pragma unroll
-    for (int m = 0; m < TM; ++m)
-#pragma unroll
-      for (int e = 0; e < ET; ++e) acc[m][e] = mfma(y[e], x[m], acc[m][e]);
-  }
-  for (int s = 0; s < NW; ++s) {  // the waves' shares, in order
-    if (w == s) {
+    for (int u = 0; u < U; ++u)
 #pragma unroll
       for (int m = 0; m < TM; ++m)
 #pragma unroll
-        for (int e = 0; e < ET; ++e)
+        for (int e = 0; e < ET; ++e) acc[m][e] = mfma(y[u][e], x[u][m], acc[m][e]);
+  };
+  constexpr int U = ET <= 2 ? 8 : ET <= 4 ? 4 : 2;
+  const int whole = a.W / 32;
+  int k = w;
+  for (; k + NW * (U - 1) < whole; k += NW * U) steps(Int<U>{}, 32 * k, false);
+  for (; k < whole; k += NW) steps(Int<1>{}, 32 * k, false);
+  if (a.W % 32 && whole % NW == w) steps(Int<1>{}, 32 * whole, true);
 #pragma unroll
-          for (int r = 0; r < 4; ++r) {  // token 16 m + l16, expert 16 e + 4 q4 + r
-            float* p = z + (16 * m + l16) * ZP + 16 * e + 4 * q4 + r;
-            *p = s ? *p + acc[m][e][r] : acc[m][e][r];
-          }
+  for (int half = NW / 2; half >= 1; half /= 2) {  // the waves' shares, pairwise
+    if (w >= half && w < 2 * half) {
+#pragma unroll
+      for (int m = 0; m < TM; ++m)
+#pragma unroll
+        for (int e = 0; e < ET; ++e) red[w - half][m * ET + e][lane] = acc[m][e];
+    }
+    __syncthreads();
+    if (w < half) {
+#pragma unroll
+      for (int m = 0; m < TM; ++m)
+#pragma unroll
+        for (int e = 0; e < ET; ++e) acc[m][e] += red[w][m * ET + e][lane];
     }
     __syncthreads();
   }
+  if (w == 0) {
+#pragma unroll
+    for (int m = 0; m < TM; ++m)
+#pragma unroll
+      for (int e = 0; e < ET; ++e)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)  // token 16 m + l16, expert 16 e + 4 q4 + r
+          z[(16 * m + l16) * ZP + 16 * e + 4 * q4 + r] = acc[m][e][r];
+  }
+  __syncthreads();
   for (int i = w; i < n; i += NW) choose(z + i * ZP, gs[w], t0 + i, a, a.counts ? hist : nullptr);
   if (a.counts) claim(a, t0, n, hist);
 }
@@ -255,18 +287,21 @@ extern "C" int ds_route(const void* h, const void* router, int* experts, float* 
     return (int)hipErrorInvalidValue;
   const RouteArgs a{T, W, E, K, groups, keep, experts, weights, counts, slots};
   if (dtype == DS_BF16 && W % 8 == 0) {
-#define GO(ET)                                                                                                           \
-  {                                                                                                                      \
-    if (T > 1024 && ET <= 8)                                                                                             \
-      hipLaunchKernelGGL((route_mfma_kernel<ET, 2, 4>), dim3((T + 31) / 32), dim3(256), 0, st, (const bf16*)h, (const bf16*)router, a); \
-    else                                                                                                                 \
-      hipLaunchKernelGGL((route_mfma_kernel<ET, 1, 8>), dim3((T + 15) / 16), dim3(512), 0, st, (const bf16*)h, (const bf16*)router, a); \
-  }
-    if (E <= 16) GO(1)
-    else if (E <= 32) GO(2)
-    else if (E <= 64) GO(4)
-    else if (E <= 128) GO(8)
-    else GO(16)
+#define GO(ET, TM, NW)                                                                                              \
+  hipLaunchKernelGGL((route_mfma_kernel<ET, TM, NW>), dim3((T + 16 * TM - 1) / (16 * TM)), dim3(64 * NW), 0, st,     \
+                     (const bf16*)h, (const bf16*)router, a)
+    const bool wide = T > 4096;
+    if (E <= 16) {
+      if (wide) GO(1, 2, 8);
+      else GO(1, 1, 16);
+    } else if (E <= 32) {
+      if (wide) GO(2, 2, 8);
+      else GO(2, 1, 16);
+    } else if (E <= 64) {
+      if (wide) GO(4, 2, 8);
+      else GO(4, 1, 8);
+    } else if (E <= 128) GO(8, 1, 8);
+    else GO(16, 1, 4);
 #undef GO
   } else if (dtype == DS_BF16) {
     hipLaunchKernelGGL(route_any_kernel<bf16>, dim3(T), dim3(256), 0, st, (const bf16*)h, (const bf16*)router, a);

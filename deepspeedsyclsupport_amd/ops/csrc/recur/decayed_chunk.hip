@@ -305,10 +305,11 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       const int row = tid / LP, part = tid % LP;
       float a = 0.f;
       for (int k = 8 * part; k < 32 * NK; k += 8 * LP) {
-        float x[8];
+        float x[8], y[8];
         Vec8<bf16>::load(Qs + row * KP + k, x);
+        Vec8<float>::load(zs + k, y);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) a = fmaf(x[e], zs[k + e], a);
+        for (int e = 0; e < 8; ++e) a = fmaf(x[e], y[e], a);
       }
 #pragma unroll
       for (int o = 1; o < LP; o <<= 1) a += __shfl_xor(a, o, 64);
@@ -342,26 +343,42 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       }
     }
     lds_barrier();  // P and the partner's half are complete
-    if constexpr (NORM) {  // next normaliser: neighbouring lanes share a pair of key columns and take every JP-th token
-      constexpr int JP = NT / (16 * NK);
-      const int k = tid / JP * 2, part = tid % JP;
-      float a0 = 0.f, a1 = 0.f;
-#pragma unroll 4
-      for (int j = part; j < C; j += JP) {
-        const bf16x2 x = *reinterpret_cast<const bf16x2*>(Ks + j * KP + k);
-        const float wj = ws[cb + j];
-        a0 = fmaf((float)x[0], wj, a0);
-        a1 = fmaf((float)x[1], wj, a1);
-      }
+    if constexpr (NORM) {  // next normaliser: neighbouring lanes share 8 key columns and take every JP-th token
+      constexpr int JP = NT / (4 * NK) < 64 ? NT / (4 * NK) : 64;
+      const int k = tid / JP * 8, part = tid % JP;
+      if (NT / JP <= 4 * NK || k < 32 * NK) {
+        float a[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int o = 1; o < JP; o <<= 1) {
-        a0 += __shfl_xor(a0, o, 64);
-        a1 += __shfl_xor(a1, o, 64);
-      }
-      if (part == 0) {
-        const float dc = eg[cb + C - 1];
-        zs[k] = fmaf(dc, zs[k], a0);
-        zs[k + 1] = fmaf(dc, zs[k + 1], a1);
+        for (int j = 0; j < C / JP; ++j) {
+          float x[8];
+          Vec8<bf16>::load(Ks + (part + j * JP) * KP + k, x);
+          const float wj = ws[cb + part + j * JP];
+#pragma unroll
+          for (int e = 0; e < 8; ++e) a[e] = fmaf(x[e], wj, a[e]);
+        }
+        // sums over the JP lanes: while there are columns to share out, every exchange halves them
+        int n = 8, col = 0;
+#pragma unroll
+        for (int o = JP / 2; o > 0; o /= 2) {
+          const bool up = part & o;
+          if (n > 1) {
+            n /= 2;
+#pragma unroll
+            for (int e = 0; e < n; ++e) {
+              const float keep = up ? a[n + e] : a[e], give = up ? a[e] : a[n + e];
+              a[e] = keep + __shfl_xor(give, o, 64);
+            }
+            if (up) col += n;
+          } else {
+            a[0] += __shfl_xor(a[0], o, 64);
+          }
+        }
+        constexpr int OWN = JP >= 8 ? 1 : 8 / JP;  // columns a lane ends up with; above 8 lanes several hold the same one
+        if (JP <= 8 || part % (JP / 8) == 0) {
+          const float dc = eg[cb + C - 1];
+#pragma unroll
+          for (int e = 0; e < OWN; ++e) zs[k + col + e] = fmaf(dc, zs[k + col + e], a[e]);
+        }
       }
     }
     // ---- within the chunk, token tiles 2 half and 2 half + 1
@@ -381,7 +398,11 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       if constexpr (NORM) {
         const int r = 16 * i + l16;
         float z = eg[cb + r] * zq[r];
-        for (int jt = 0; jt <= i; ++jt) z += rs[jt * C + r];
+#pragma unroll
+        for (int jt = 0; jt < 4; ++jt) {  // (tiles behind the diagonal hold leftovers)
+          const float p = rs[jt * C + r];
+          z += jt <= i ? p : 0.f;
+        }
         acc *= scale / (fmaxf(fabsf(z * scale), fl[cb + r]) + 1e-6f);
       } else {
         acc *= scale;

@@ -33,24 +33,38 @@ def pre_norm(x, y, w, eps, ids=None, embed=None, mult=1.0, rows=None):
     return f(x, y, None, None, w, eps, ids, embed, mult, rows)
 
 
-# From this many rows on the products go to the library's grouped GEMM, over rows copied into expert order
-LIBRARY_ROWS = 1024
+# Average rows per expert from which on the products tile the rows instead of streaming the weights (in operand order)
+TILE_ROWS = 12
+# ... and, where only row-major weights are kept, go to the library's grouped GEMM over rows copied into expert order
+LIBRARY_ROWS = 32
 
 
-def experts(h, router, fc1, fc2, top, groups=1, keep=1):
+def operand_order(w):
+    """Expert weights [E, N, K] as the products on the matrix cores read them (`bf16_gemv.preshuffle16` of every expert), or None
+    where sizes or type do not allow it. N: rows of one expert (gate and up count as one half each)."""
+    from .bf16_gemv import preshuffle16
+    E, N, K = w.shape
+    if w.dtype != torch.bfloat16 or not w.is_cuda or not expert_ops().expert_order_ok(N, K):
+        return None
+    return torch.stack([preshuffle16(e) for e in w]).view(E, N, K)
+
+
+def experts(h, router, fc1, fc2, top, groups=1, keep=1, order=None):
     """Routed gated feed-forwards: h [T, W], router [E, W], fc1 [E, 2 F, W] (gate rows, up rows), fc2 [E, W, F] -> `ExpertSum`.
     The experts of the `keep` best of `groups` equal groups compete; the best `top` are taken, weighted by their softmax over
-    all experts divided by its sum."""
+    all experts divided by its sum. `order`: (fc1, fc2) in operand order, if they are kept."""
     if not use_native(h):
         e, w = reference.route(h, router, top, groups, keep)
         return ExpertSum(reference.expert_gemm(reference.expert_gemm(h, fc1, e, top, True), fc2, e, 1, False), w)
     ops = expert_ops()
-    rows = h.shape[0] * top
-    few = rows <= ops.expert_few() or h.dtype != torch.bfloat16
-    e, w, offs, order, at = ops.route(h, router, top, groups, keep, not few)
-    if rows >= LIBRARY_ROWS and not few and all(n % 128 == 0 for n in (*fc1.shape[1:], fc2.shape[2])):
+    rows, E = h.shape[0] * top, router.shape[0]
+    tile = order is not None and rows >= TILE_ROWS * E
+    few = h.dtype != torch.bfloat16 or (rows <= ops.expert_few() and not tile)
+    e, w, offs, entries, at = ops.route(h, router, top, groups, keep, not few)
+    if order is None and not few and rows >= LIBRARY_ROWS * E and all(n % 128 == 0 for n in (*fc1.shape[1:], fc2.shape[2])):
         ends = offs[1:]
         mid = ops.silu_mul(torch._grouped_mm(ops.expert_spread(h, at), fc1.transpose(1, 2), offs=ends))
         return ExpertSum(torch._grouped_mm(mid, fc2.transpose(1, 2), offs=ends), w, at)
-    mid = ops.expert_gemm(h, fc1, e, offs, order, top, True)
-    return ExpertSum(ops.expert_gemm(mid, fc2, e, offs, order, 1, False), w)
+    (a, b), operand = (order, True) if order else ((fc1, fc2), False)
+    mid = ops.expert_gemm(h, a, e, offs, entries, top, True, operand, tile)
+    return ExpertSum(ops.expert_gemm(mid, b, e, offs, entries, 1, False, operand, tile), w)

@@ -91,21 +91,29 @@ def test_route(device, dtype, tol, E, top, groups, keep, W, T):
 
 
 SIZES = [(12, 3, 64, 96), (8, 2, 40, 24), (4, 1, 256, 200), (9, 4, 136, 72), (16, 6, 320, 128), (5, 2, 33, 27), (64, 8, 128, 64),
-         (32, 3, 256, 128)]
+         (32, 3, 256, 128), (3, 2, 448, 192), (6, 5, 128, 320)]
 
 
 @pytest.mark.parametrize("device,dtype,tol", CASES)
 @pytest.mark.parametrize("E,top,W,F", SIZES)
 @pytest.mark.parametrize("T", [1, 2, 19, 130, 700])
-def test_experts(device, dtype, tol, E, top, W, F, T):
-    """Few rows (lists made in the products), lists, and the library's grouped product; experts without a token."""
+@pytest.mark.parametrize("path", ["rows", "order", "library"])
+def test_experts(device, dtype, tol, E, top, W, F, T, path, monkeypatch):
+    """Weights row by row and in operand order: few rows (lists made in the products), lists streamed, tiles; the library's
+    grouped product; experts without a token."""
     if device == "cpu" and (T > 19 or E > 16):
         pytest.skip("sizes of device kernels")
+    if path != "rows" and (dtype != torch.bfloat16 or W % 64 or F % 64 or (path == "library" and (T < 130 or W % 128 or F % 128))):
+        pytest.skip("no such path at these sizes")
+    if path == "library":
+        monkeypatch.setattr(expert_ops, "LIBRARY_ROWS", 0)
     g = 2 if E % 2 == 0 else 1
     h = rnd(T, W, seed=1).to(dtype)
     r = rnd(E, W, seed=2, scale=2 * W**-0.5).to(dtype)
     fc1, fc2 = rnd(E, 2 * F, W, seed=3, scale=W**-0.5).to(dtype), rnd(E, W, F, seed=4, scale=F**-0.5).to(dtype)
-    got = expert_ops.experts(*(t.to(device) for t in (h, r, fc1, fc2)), top, g, 1 if top <= E // g else g)
+    dev = [t.to(device) for t in (h, r, fc1, fc2)]
+    order = tuple(expert_ops.operand_order(t) for t in dev[2:]) if path == "order" else None
+    got = expert_ops.experts(*dev, top, g, 1 if top <= E // g else g, order)
     e, w = O.route(h.double() @ r.double().t(), top, g, 1 if top <= E // g else g)
     x = h.double()
     want = torch.zeros(T, W).double()
@@ -117,15 +125,18 @@ def test_experts(device, dtype, tol, E, top, W, F, T):
 
 
 @GPU
-def test_experts_any_rows():
+@pytest.mark.parametrize("path", ["rows", "stream", "tile"])
+def test_experts_any_rows(path, monkeypatch):
     """Lists and products over row counts around every border of the paths; a single expert that takes everything."""
-    E, top, W, F = 6, 2, 128, 96
+    E, top, W, F = 6, 2, 128, 192
+    monkeypatch.setattr(expert_ops, "TILE_ROWS", 0 if path == "tile" else 1 << 20)
     r, fc1, fc2 = (rnd(*s, seed=i, scale=0.1).bfloat16().cuda() for i, s in enumerate([(E, W), (E, 2 * F, W), (E, W, F)]))
-    for T in (15, 16, 17, 31, 33, 63, 65, 255, 256, 257, 511, 512, 513):
+    for T in (15, 16, 17, 31, 33, 63, 65, 127, 128, 129, 255, 256, 257, 289, 511, 513):
         h = rnd(T, W, seed=T).bfloat16()
         h[:, 0] = 30.0
         r[:, 0] = torch.tensor([5.0, 0, 0, 2.0, 0, 0]).bfloat16()   # every token: experts 0 and 3
-        got = expert_ops.experts(h.cuda(), r, fc1, fc2, top)
+        order = None if path == "rows" else (expert_ops.operand_order(fc1), expert_ops.operand_order(fc2))
+        got = expert_ops.experts(h.cuda(), r, fc1, fc2, top, order=order)
         x, want = h.double(), 0
         e, w = O.route(x @ r.double().cpu().t(), top, 1, 1)
         assert set(e.view(-1).tolist()) == {0, 3}
