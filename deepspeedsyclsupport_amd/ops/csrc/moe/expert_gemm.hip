@@ -10,7 +10,7 @@
 //  * tile: many rows per expert. 128 entries x 256 weight rows (gated: 128 of either part) per workgroup. Weights are stored in
 //    operand order and every wave has rows of its own, so they go from memory to registers in 512-byte runs, one step of 64
 //    ahead; only the entries' rows pass through LDS (swizzled, two buffers). Two workgroups share a CU. Workgroups walk groups
-//    of 8 column tiles by all row tiles of an expert, so that those at work on an XCD at a time share both operands in its L2.
+//    of 4 column tiles by all row tiles of an expert, so that those at work on an XCD at a time share both operands in its L2.
 //  * any: a workgroup per entry and 64 columns; fp32 and widths that are no multiple of 8.
 #include "ds_hip.h"
 
@@ -210,7 +210,7 @@ __global__ void __launch_bounds__(256) expert_stream_kernel(ExpertArgs a) {
 }
 
 // ------------------------------------------------------------------------------------------------ many rows per expert
-constexpr int BM = 128, BN = 256, GROUP = 8;
+constexpr int BM = 128, BN = 256, GROUP = 4;
 
 template <bool GLU>
 __global__ void __launch_bounds__(256, 2) expert_tile_kernel(ExpertArgs a) {
@@ -307,7 +307,7 @@ __global__ void __launch_bounds__(256, 2) expert_tile_kernel(ExpertArgs a) {
       for (int j = 0; j < 2; ++j)
 #pragma unroll
         for (int m = 0; m < 4; ++m) {
-          if (m >= tiles) break;
+          if (m >= tiles) break;  // (the branch also keeps the operands of later steps out of the registers)
           const bf16x8 x = *reinterpret_cast<const bf16x8*>(&xs[buf][(32 * m + l32) * 64 + 8 * ((4 * j + 2 * hh + h) ^ sw)]);
 #pragma unroll
           for (int t = 0; t < 2; ++t) acc[t][m] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(w[t][h][j], x, acc[t][m], 0, 0, 0);
