@@ -8,15 +8,15 @@ int ds_gated_norm(const void*, const void*, int64_t, const float*, void*, int64_
                   hipStream_t);
 int ds_scan_prepare(const void*, const float*, const float*, const void*, const float*, const float*, const int*, const int*,
                     const int*, const int*, void*, void*, float*, const int*, int, int, hipStream_t);
-int ds_scan_split(const void*, const float*, int, void*, void*, const int*, int, int, hipStream_t);
+int ds_scan_split(const void*, const float*, int, void*, void*, int, const int*, int, int, hipStream_t);
 int ds_exp_gates(const void*, int, int, int, const float*, const float*, float, float*, const int*, const int*, const int*,
                  float*, float*, int, int, int, int, hipStream_t);
 int ds_scan_recur(const void*, const void*, const float*, const float*, const float*, float, const void*, float*, float*,
-                  const float*, void*, const int*, int, int, const int*, const int*, const int*, void*, const int*, int, int,
-                  hipStream_t);
+                  const float*, void*, int, const int*, int, int, const int*, const int*, const int*, void*, const int*, int,
+                  int, hipStream_t);
 int ds_scan_chunk_ok(int);
 int ds_scan_chunk(const void*, const void*, const float*, const float*, const float*, float, const void*, float*, float*,
-                  const float*, void*, const int*, int, const int*, const int*, const int*, void*, const int*, int,
+                  const float*, void*, int, const int*, int, const int*, const int*, const int*, void*, const int*, int,
                   hipStream_t);
 }
 
@@ -94,16 +94,18 @@ std::tuple<Tensor, Tensor, OptT> scan_prepare(Tensor proj, std::vector<int64_t> 
   return {qk, v, gb};
 }
 
-// The same qk and v straight from the projection's columns, the first 2 half of every head of q and k turned by cs [T, half, 2]
+// The same qk and v straight from the projection's columns, the first 2 half of every head of q and k turned by cs [T, half, 2];
+// turned ones in bf16 as sums of two terms: qk [2 terms, 2, Hk, T, dks]
 std::tuple<Tensor, Tensor> scan_split(Tensor proj, std::vector<int64_t> dims, OptT cs) {
   need(proj, "proj");
   const Dims D = dims_of(dims);
   const int64_t T = proj.size(0), half = has(cs) ? cs->numel() / 2 / std::max<int64_t>(T, 1) : 0;
   TORCH_CHECK(proj.dim() == 2 && proj.size(1) == D.rows() && 2 * half <= D.dk(), "scan_split: proj [T, rows]");
   auto make = [&](at::IntArrayRef s, bool pad) { return pad ? torch::zeros(s, proj.options()) : torch::empty(s, proj.options()); };
-  Tensor qk = make({2, D.Hk(), T, D.dks()}, D.dks() != D.dk()), v = make({D.H(), T, D.dvs()}, D.dvs() != D.dv());
+  const int terms = half > 0 && proj.scalar_type() == at::kBFloat16 ? 2 : 1;
+  Tensor qk = make({terms, 2, D.Hk(), T, D.dks()}, D.dks() != D.dk()), v = make({D.H(), T, D.dvs()}, D.dvs() != D.dv());
   check(ds_scan_split(proj.data_ptr(), has(cs) ? f32(*cs, T * half * 2, "angles") : nullptr, (int)half, qk.data_ptr(), v.data_ptr(),
-                      D.v, (int)T, dcode(proj), stream()), "scan_split");
+                      terms, D.v, (int)T, dcode(proj), stream()), "scan_split");
   return {qk, v};
 }
 
@@ -125,12 +127,14 @@ std::tuple<Tensor, Tensor> exp_gates(Tensor proj, int64_t ci, int64_t cf, Tensor
   return {gb, floors};
 }
 
+int terms_of(const Dims& D, const Tensor& qk, int64_t T) { return qk.numel() > 2 * D.Hk() * T * D.dks() ? 2 : 1; }
+
 struct ScanCheck {
   ScanCheck(const Dims& D, const Tensor& qk, const Tensor& v, const OptT& gb, const OptT& ld, const Tensor& proj,
             const Tensor& state, const OptT& conv_state, const OptT& zstate, const OptT& floors, const Tensor& out) {
     need(qk, "qk"); need(v, "v"); need(proj, "proj"); need(state, "state"); need(out, "out");
     const int64_t T = proj.size(0);
-    TORCH_CHECK(proj.size(1) == D.rows() && qk.numel() == 2 * D.Hk() * T * D.dks() && v.numel() == D.H() * T * D.dvs() &&
+    TORCH_CHECK(proj.size(1) == D.rows() && qk.numel() == terms_of(D, qk, T) * 2 * D.Hk() * T * D.dks() && v.numel() == D.H() * T * D.dvs() &&
                 qk.scalar_type() == proj.scalar_type() && v.scalar_type() == proj.scalar_type(), "scan: qk / v");
     TORCH_CHECK(has(gb) != has(ld), "scan: decays per token or per head");
     TORCH_CHECK(state.scalar_type() == at::kFloat && state.dim() == 4 && state.size(1) == D.H() && state.size(2) == D.dv() &&
@@ -138,6 +142,7 @@ struct ScanCheck {
     TORCH_CHECK(out.numel() == T * D.H() * D.dv() && out.scalar_type() == proj.scalar_type(), "scan: out [T, H dv]");
     TORCH_CHECK(has(zstate) == has(floors), "scan: normaliser and floors");
     if (has(zstate)) {
+      TORCH_CHECK(terms_of(D, qk, T) == 1, "scan: a normaliser takes q and k of one term");
       need(*zstate, "normaliser");
       TORCH_CHECK(zstate->scalar_type() == at::kFloat && zstate->dim() == 4 && zstate->size(0) == state.size(0) &&
                   zstate->size(1) == D.H() && zstate->size(2) == (D.dv() + 31) / 32 && zstate->size(3) == D.dks(),
@@ -155,7 +160,7 @@ void recur_list(Tensor qk, Tensor v, OptT gb, OptT log_decay, OptT skip, double 
   check(ds_scan_recur(qk.data_ptr(), v.data_ptr(), opt_f32(gb, T * 2 * D.H(), "gb"), opt_f32(log_decay, D.H(), "log_decay"),
                       opt_f32(skip, D.H(), "skip"), (float)scale, proj.data_ptr(), state.data_ptr<float>(),
                       has(zstate) ? zstate->data_ptr<float>() : nullptr, opt_f32(floors, T * D.H(), "floors"),
-                      D.taps() > 1 ? conv_state->data_ptr() : nullptr, i32(list, list.numel(), "list"),
+                      D.taps() > 1 ? conv_state->data_ptr() : nullptr, terms_of(D, qk, T), i32(list, list.numel(), "list"),
                       (int)(list.numel() / stride), stride, i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"),
                       out.data_ptr(), D.v, (int)T, dcode(proj), stream()), "scan_recur");
 }
@@ -182,7 +187,7 @@ void scan_chunk(Tensor qk, Tensor v, OptT gb, OptT log_decay, OptT skip, double 
   check(ds_scan_chunk(qk.data_ptr(), v.data_ptr(), opt_f32(gb, T * 2 * D.H(), "gb"), opt_f32(log_decay, D.H(), "log_decay"),
                       opt_f32(skip, D.H(), "skip"), (float)scale, proj.data_ptr(), state.data_ptr<float>(),
                       has(zstate) ? zstate->data_ptr<float>() : nullptr, opt_f32(floors, T * D.H(), "floors"),
-                      D.taps() > 1 ? conv_state->data_ptr() : nullptr, i32(seqs, seqs.numel(), "seqs"), (int)seqs.size(0),
+                      D.taps() > 1 ? conv_state->data_ptr() : nullptr, terms_of(D, qk, T), i32(seqs, seqs.numel(), "seqs"), (int)seqs.size(0),
                       i32(cu, S + 1, "cu"), i32(start, S, "start"), i32(slots, S, "slots"), out.data_ptr(), D.v, (int)T, stream()),
         "scan_chunk");
 }

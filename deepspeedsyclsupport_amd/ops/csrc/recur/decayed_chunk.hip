@@ -1,4 +1,4 @@
-// Recurrences with a scalar decay per head over long portions, by chunks of 64 tokens (CDNA4, gfx950). See decayed_scan.hip
+// Recurrences with a scalar decay per head over long portions, by chunks of 64 (or 32) tokens (CDNA4, gfx950). See decayed_scan.hip
 // for the recurrence.
 //
 // With the running log decay G_i of a chunk (its first token included) and the state S0 the chunk starts from:
@@ -11,7 +11,8 @@
 // accumulates into it, and the same registers are the left operand of the read-out (a product's k order is free as long as
 // both sides agree on it). The two halves of the read-out meet in LDS, where the 64 x 64 weights P are shared too.
 //
-// Precision: q, k and v are bf16 activations; everything else is fp32. The bf16 matrix instructions take an fp32 operand
+// Precision: q, k and v are bf16 activations, or q and k (where they were computed on, as by a rotation) sums of two bf16 terms;
+// everything else is fp32. The bf16 matrix instructions take an fp32 operand
 // as three bf16 terms (8 + 8 + 8 mantissa bits, nothing is lost) with fp32 accumulation, so state, weights and decays
 // enter the products as 32-bit numbers at a third of the bf16 rate, five times that of the fp32 instructions. Log decays
 // are summed in fp64: only differences enter, and a strong decay early in a chunk must not cost the later ones their digits.
@@ -20,8 +21,8 @@
 
 namespace {
 
-constexpr int C = 64;
-constexpr int PP = C + 8;  // LDS row length (elements) of the weights
+// tokens per chunk: two terms of wide keys leave room for 32
+constexpr int chunk_of(int NK, int QT) { return QT == 2 && NK > 4 ? 32 : 64; }
 constexpr double LOG2E = 1.4426950408889634073599246810019;
 
 typedef short s16x4_t __attribute__((ext_vector_type(4)));
@@ -87,26 +88,27 @@ __device__ __forceinline__ bf16x8 read_tr(const bf16* base, int pitch, int r, in
 }
 
 // NK: 32-wide steps of the key width (rounded up), even unless the waves of a pair cannot share (NK 1: the second one has
-// no rows); WC: groups of 16 value columns
-template <int NK, int WC, bool NORM>
+// no rows); WC: groups of 16 value columns; NORM: with a normaliser; QT: terms of q and k
+template <int NK, int WC, bool NORM, int QT>
 __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decayed_chunk_kernel(
     const bf16* __restrict__ qk, const bf16* __restrict__ v, const float* __restrict__ gb,
     const float* __restrict__ log_decay, const float* __restrict__ skip, float scale, const bf16* __restrict__ proj,
-    float* __restrict__ state, float* __restrict__ zstate, const float* __restrict__ floors, bf16* __restrict__ conv_state, const int* __restrict__ seqs, const int* __restrict__ cu,
-    const int* __restrict__ start, const int* __restrict__ slots, bf16* __restrict__ out, ScanDims D) {
-  constexpr int NT = 128 * WC, NW = 2 * WC, VT = 16 * WC;
+    float* __restrict__ state, float* __restrict__ zstate, const float* __restrict__ floors, bf16* __restrict__ conv_state,
+    const int* __restrict__ seqs, const int* __restrict__ cu, const int* __restrict__ start, const int* __restrict__ slots, bf16* __restrict__ out, ScanDims D) {
+  constexpr int C = chunk_of(NK, QT), PP = C + 8;   // PP: LDS row length of the weights
+  constexpr int NT = 128 * WC, NW = 2 * WC, VT = 16 * WC, FT = C / 32;  // FT: token tiles a wave finishes
   constexpr int KP = 32 * NK + 8, VP = VT + 8;      // LDS row lengths of q and k, of v
   constexpr int KH = (NK + 1) / 2;                  // steps of a wave's half of the key rows
   constexpr int PQ = C * 4 * NK / NT, PV = (C * VT / 8 + NT - 1) / NT;  // 16-byte pieces per thread of q or k, of v
   static_assert(C * 4 * NK % NT == 0 || NK == 1, "pieces");
   constexpr int PQN = PQ > 0 ? PQ : 1;
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  bf16* const Qs = reinterpret_cast<bf16*>(smem);
-  bf16* const Ks = Qs + C * KP;
-  bf16* const Vs = Ks + C * KP;
+  bf16* const Qs = reinterpret_cast<bf16*>(smem);                 // [QT][C][KP]
+  bf16* const Ks = Qs + QT * C * KP;
+  bf16* const Vs = Ks + QT * C * KP;
   bf16* const Ps = Vs + C * VP;                                   // [3][C][PP]
-  f32x4* const Ys = reinterpret_cast<f32x4*>(Ps + 3 * C * PP);    // [NW][2][64]: halves of the read-out on their way
-  double* const Gs = reinterpret_cast<double*>(Ys + NW * 2 * 64); // [2 NW][C] running log2 decay
+  f32x4* const Ys = reinterpret_cast<f32x4*>(Ps + 3 * C * PP);    // [NW][FT][64]: halves of the read-out on their way
+  double* const Gs = reinterpret_cast<double*>(Ys + NW * FT * 64); // [2 NW][C] running log2 decay
   float* const bs = reinterpret_cast<float*>(Gs + 2 * NW * C);    // [2 NW][C] step sizes
   float* const eg = bs + 2 * NW * C;                              // [2 NW][C] e^{G_i}
   float* const ws = eg + 2 * NW * C;                              // [2 NW][C] e^{G_C - G_j} b_j
@@ -141,11 +143,12 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
   const bf16* qbase = qk + D.q_at(g, t0);
   const bf16* kbase = qk + D.k_at(g, t0);
   const bf16* vbase = v + D.v_at(h, t0) + v0;
+  const int64_t term = 2 * D.Hk * D.T * dks;  // from one term of q and k to the next
   const int vw = min(dvs - v0, VT);    // v columns of this workgroup that exist
   const bool k_full = dks == 32 * NK, v_full = vw == VT;
 
   // ---- a chunk's rows on their way to LDS: 4 NK (q, k) and VT / 8 (v) 16-byte pieces per row
-  bf16x8 rq[PQN], rk[PQN], rv[PV];
+  bf16x8 rq[QT][PQN], rk[QT][PQN], rv[PV];
   auto fetch = [&](int c) {
     const bool whole = (c + 1) * C <= n;
     const int64_t base = (int64_t)c * C * dks, vb = (int64_t)c * C * dvs;
@@ -157,8 +160,11 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       if (!whole) row = min(row, last);
       if (!k_full) ch = min(ch, dks - 8);
       if (PQ > 0 || p < C * 4 * NK) {
-        rq[i] = *reinterpret_cast<const bf16x8*>(qbase + base + row * dks + ch);
-        rk[i] = *reinterpret_cast<const bf16x8*>(kbase + base + row * dks + ch);
+#pragma unroll
+        for (int u = 0; u < QT; ++u) {
+          rq[u][i] = *reinterpret_cast<const bf16x8*>(qbase + u * term + base + row * dks + ch);
+          rk[u][i] = *reinterpret_cast<const bf16x8*>(kbase + u * term + base + row * dks + ch);
+        }
       }
     }
 #pragma unroll
@@ -179,7 +185,10 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
 #pragma unroll
       for (int i = 0; i < PQN; ++i) {
         const int p = tid + i * NT;
-        if (c * C + p / (4 * NK) >= n || p % (4 * NK) * 8 >= dks) rq[i] = rk[i] = z;
+        if (c * C + p / (4 * NK) >= n || p % (4 * NK) * 8 >= dks) {
+#pragma unroll
+          for (int u = 0; u < QT; ++u) rq[u][i] = rk[u][i] = z;
+        }
       }
 #pragma unroll
       for (int i = 0; i < PV; ++i) {
@@ -191,8 +200,11 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
     for (int i = 0; i < PQN; ++i) {
       const int p = tid + i * NT, row = p / (4 * NK), ch = p % (4 * NK) * 8;
       if (PQ > 0 || p < C * 4 * NK) {
-        *reinterpret_cast<bf16x8*>(Qs + row * KP + ch) = rq[i];
-        *reinterpret_cast<bf16x8*>(Ks + row * KP + ch) = rk[i];
+#pragma unroll
+        for (int u = 0; u < QT; ++u) {
+          *reinterpret_cast<bf16x8*>(Qs + (u * C + row) * KP + ch) = rq[u][i];
+          *reinterpret_cast<bf16x8*>(Ks + (u * C + row) * KP + ch) = rk[u][i];
+        }
       }
     }
 #pragma unroll
@@ -201,7 +213,7 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       if (p < C * VT / 8) *reinterpret_cast<bf16x8*>(Vs + p / (VT / 8) * VP + p % (VT / 8) * 8) = rv[i];
     }
   };
-  // ---- decays and step sizes of a chunk, a lane per token: every NW chunks each wave prepares one of the next NW
+  // ---- decays and step sizes of a chunk, a lane per token (the others add nothing): every NW chunks each wave prepares one of the next NW
   float lg = 0.f, lb = 0.f, lf = 0.f;
   auto fetch_gb = [&](int c) {
     const int64_t t = t0 + min(c * C + lane, n - 1);
@@ -210,7 +222,7 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
     if constexpr (NORM) lf = floors[t * D.H + h];
   };
   auto scan_gb = [&](int c) {
-    const bool ok = c * C + lane < n;  // rows past the end neither decay nor add anything
+    const bool ok = lane < C && c * C + lane < n;  // rows past the end neither decay nor add anything
     const float b0 = ok ? lb : 0.f;
     double G = ok ? (double)lg * LOG2E : 0.0;
 #pragma unroll
@@ -219,6 +231,7 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       if (lane >= o) G += p;
     }
     const double GC = __shfl(G, 63, 64);
+    if (lane >= C) return;
     const int b = c % (2 * NW) * C + lane;
     Gs[b] = G;
     bs[b] = b0;
@@ -237,17 +250,25 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
     if (ahead) fetch_gb(c + NW + w);
     lds_barrier();
     // ---- P. The read-out takes pairs of 16 x 16 tiles of a row: 10 tiles up to the diagonal, and 2 behind it that are zero
+    // (32 tokens: 3 and 1)
+    constexpr int PT = C == 64 ? 12 : 4;
 #pragma unroll
-    for (int u = 0; u < (12 + NW - 1) / NW; ++u) {
+    for (int u = 0; u < (PT + NW - 1) / NW; ++u) {
       const int tl = w + u * NW;
-      if (tl >= 12) break;
+      if (tl >= PT) break;
       const int it = tl < 4 ? tl >> 1 : 2 + ((tl - 4) >> 2), jt = tl < 4 ? tl & 1 : (tl - 4) & 3;
       f32x4 s = {0.f, 0.f, 0.f, 0.f};
       if (jt <= it) {
 #pragma unroll
-        for (int kk = 0; kk < NK; ++kk)
-          s = mfma(*reinterpret_cast<const bf16x8*>(Ks + (16 * jt + l16) * KP + 32 * kk + 8 * q4),
-                   *reinterpret_cast<const bf16x8*>(Qs + (16 * it + l16) * KP + 32 * kk + 8 * q4), s);
+        for (int kk = 0; kk < NK; ++kk) {
+          const bf16 *kr = Ks + (16 * jt + l16) * KP + 32 * kk + 8 * q4, *qr = Qs + (16 * it + l16) * KP + 32 * kk + 8 * q4;
+          const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(kr), q0 = *reinterpret_cast<const bf16x8*>(qr);
+          if constexpr (QT == 2) {  // (the product of the second terms is below 2^-16 of the whole)
+            s = mfma(*reinterpret_cast<const bf16x8*>(kr + C * KP), q0, s);
+            s = mfma(k0, *reinterpret_cast<const bf16x8*>(qr + C * KP), s);
+          }
+          s = mfma(k0, q0, s);
+        }
         // lane: row i of P, columns j .. j + 3
         const int i = 16 * it + l16, j = 16 * jt + 4 * q4;
         const double gi = Gs[cb + i];
@@ -273,9 +294,9 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       *reinterpret_cast<uint2*>(p + 2 * C * PP) = uint2{d[0], d[1]};
     }
     // ---- read-out of the state the chunk starts from, this half of the key rows: y^T [16 columns, 64 tokens] = S^T q^T
-    f32x4 y[4];
+    f32x4 y[2 * FT];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) y[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < 2 * FT; ++i) y[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (rows_ok) {
 #pragma unroll
       for (int kk = 0; kk < KH; ++kk) {
@@ -285,15 +306,24 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
         for (int e = 0; e < 8; ++e) x[e] = S[2 * kk + (e >> 2)][e & 3];
         split3(x, s0, s1, s2);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
+        for (int i = 0; i < 2 * FT; ++i) {
           const bf16* qr = Qs + (16 * i + l16) * KP + k_first + 32 * kk + 4 * q4;
-          const bf16x4 lo = *reinterpret_cast<const bf16x4*>(qr), hi = *reinterpret_cast<const bf16x4*>(qr + 16);
-          bf16x8 qb;
+          auto row = [&](const bf16* p) {
+            const bf16x4 lo = *reinterpret_cast<const bf16x4*>(p), hi = *reinterpret_cast<const bf16x4*>(p + 16);
+            bf16x8 q;
 #pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            qb[e] = lo[e];
-            qb[4 + e] = hi[e];
+            for (int e = 0; e < 4; ++e) {
+              q[e] = lo[e];
+              q[4 + e] = hi[e];
+            }
+            return q;
+          };
+          if constexpr (QT == 2) {
+            const bf16x8 qc = row(qr + C * KP);
+            y[i] = mfma(s1, qc, y[i]);
+            y[i] = mfma(s0, qc, y[i]);
           }
+          const bf16x8 qb = row(qr);
           y[i] = mfma(s2, qb, y[i]);
           y[i] = mfma(s1, qb, y[i]);
           y[i] = mfma(s0, qb, y[i]);
@@ -315,18 +345,18 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       for (int o = 1; o < LP; o <<= 1) a += __shfl_xor(a, o, 64);
       if (part == 0) zq[row] = a;
     }
-    // each wave of a pair finishes two token tiles: the other two go to its partner
+    // each wave of a pair finishes half of the token tiles: the others go to its partner
 #pragma unroll
-    for (int i = 0; i < 2; ++i) Ys[(w * 2 + i) * 64 + lane] = pick(half, y[i], y[2 + i]);
+    for (int i = 0; i < FT; ++i) Ys[(w * FT + i) * 64 + lane] = pick(half, y[i], y[FT + i]);
     // this pair's columns of v: lane l16 a column, tokens 32 s + 8 q4 + e
-    bf16x8 vf[2];
+    bf16x8 vf[FT];
 #pragma unroll
-    for (int s = 0; s < 2; ++s) vf[s] = read_tr(Vs, VP, 32 * s + 8 * q4, 32 * s + 8 * q4 + 4, 16 * wc, l16);
+    for (int s = 0; s < FT; ++s) vf[s] = read_tr(Vs, VP, 32 * s + 8 * q4, 32 * s + 8 * q4 + 4, 16 * wc, l16);
     // ---- next state
     if (rows_ok) {
       const float dc = eg[cb + C - 1];
 #pragma unroll
-      for (int s = 0; s < 2; ++s) {
+      for (int s = 0; s < FT; ++s) {
         bf16x8 u0, u1, u2;
         float x[8];
 #pragma unroll
@@ -336,6 +366,11 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
         for (int t = 0; t < 2 * KH; ++t) {
           const bf16x8 kf = read_tr(Ks, KP, 32 * s + 8 * q4, 32 * s + 8 * q4 + 4, k_first + 16 * t, l16);
           if (s == 0) S[t] *= dc;
+          if constexpr (QT == 2) {
+            const bf16x8 kl = read_tr(Ks + C * KP, KP, 32 * s + 8 * q4, 32 * s + 8 * q4 + 4, k_first + 16 * t, l16);
+            S[t] = mfma(kl, u1, S[t]);
+            S[t] = mfma(kl, u0, S[t]);
+          }
           S[t] = mfma(kf, u2, S[t]);
           S[t] = mfma(kf, u1, S[t]);
           S[t] = mfma(kf, u0, S[t]);
@@ -381,15 +416,15 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
         }
       }
     }
-    // ---- within the chunk, token tiles 2 half and 2 half + 1
+    // ---- within the chunk, this wave's token tiles
 #pragma unroll
-    for (int k = 0; k < 2; ++k) {
-      const int i = 2 * half + k;
-      f32x4 acc = pick(half, y[2 + k], y[k]);
-      acc = (acc + Ys[((w ^ 1) * 2 + k) * 64 + lane]) * eg[cb + 16 * i + l16];
+    for (int k = 0; k < FT; ++k) {
+      const int i = FT * half + k;
+      f32x4 acc = pick(half, y[FT + k], y[k]);
+      acc = (acc + Ys[((w ^ 1) * FT + k) * 64 + lane]) * eg[cb + 16 * i + l16];
 #pragma unroll
-      for (int s = 0; s < 2; ++s) {
-        if (s > half) break;
+      for (int s = 0; s < FT; ++s) {
+        if (s > i / 2) break;
         const bf16* pr = Ps + (16 * i + l16) * PP + 32 * s + 8 * q4;
         acc = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr + 2 * C * PP), acc);
         acc = mfma(vf[s], *reinterpret_cast<const bf16x8*>(pr + C * PP), acc);
@@ -441,20 +476,21 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
     advance_windows(conv_state + (int64_t)slots[seq] * (D.taps - 1) * D.channels, proj, t0, n, D, fresh, h);
 }
 
-template <int NK, int WC, bool NORM>
+template <int NK, int WC, bool NORM, int QT>
 int launch(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip, float scale,
            const void* proj, float* state, float* zstate, const float* floors, void* conv_state, const int* seqs, int nseq, const int* cu, const int* start, const int* slots,
            void* out, const ScanDims& D, hipStream_t st) {
-  constexpr int VT = 16 * WC;
-  constexpr int LDS = (2 * C * (32 * NK + 8) + C * (VT + 8) + 3 * C * PP) * 2 + 2 * WC * 2 * 64 * 16 + 4 * WC * C * 20 +
+  constexpr int VT = 16 * WC, C = chunk_of(NK, QT);
+  constexpr int LDS = (2 * QT * C * (32 * NK + 8) + C * (VT + 8) + 3 * C * (C + 8)) * 2 + 2 * WC * C / 32 * 64 * 16 +
+                      4 * WC * C * 20 +
                       (NORM ? (4 * WC * C + 32 * NK + 5 * C) * 4 : 0);
   static bool attr = false;
   if (!attr) {
-    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<NK, WC, NORM>),
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<NK, WC, NORM, QT>),
                               hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
     attr = true;
   }
-  hipLaunchKernelGGL((decayed_chunk_kernel<NK, WC, NORM>), dim3((unsigned)((D.dv + VT - 1) / VT * D.H * nseq)), dim3(128 * WC), LDS,
+  hipLaunchKernelGGL((decayed_chunk_kernel<NK, WC, NORM, QT>), dim3((unsigned)((D.dv + VT - 1) / VT * D.H * nseq)), dim3(128 * WC), LDS,
                      st, (const bf16*)qk, (const bf16*)v, gb, log_decay, skip, scale, (const bf16*)proj, state, zstate,
                      floors, (bf16*)conv_state, seqs, cu, start, slots, (bf16*)out, D);
   DS_CHECK_LAUNCH();
@@ -465,28 +501,31 @@ int launch(const void* qk, const void* v, const float* gb, const float* log_deca
 
 extern "C" int ds_scan_chunk_ok(int dk) { return dk <= 256; }
 
-// bf16 storage, dk up to 256. seqs [nseq, 2]: (sequence, anything). zstate, floors: as for ds_scan_recur
+// bf16 storage, dk up to 256. seqs [nseq, 2]: (sequence, anything). zstate, floors, terms: as for ds_scan_recur
 extern "C" int ds_scan_chunk(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip,
                              float scale, const void* proj, float* state, float* zstate, const float* floors,
-                             void* conv_state, const int* seqs, int nseq, const int* cu,
+                             void* conv_state, int terms, const int* seqs, int nseq, const int* cu,
                              const int* start, const int* slots, void* out, const int* dims, int tokens, hipStream_t st) {
   if (nseq <= 0) return 0;
   const ScanDims D{dims[0], dims[1], dims[2], dims[3], dims[4], dims[5], dims[6], dims[7], dims[8], dims[9], dims[10], dims[11],
                    tokens};
-  if (!scan_dims_ok(D) || !ds_scan_chunk_ok(D.dk) || (!gb == !log_decay) || (!zstate != !floors) || (D.taps > 1 && !conv_state) ||
+  if (!scan_dims_ok(D) || !ds_scan_chunk_ok(D.dk) || (!gb == !log_decay) || (!zstate != !floors) ||
+      terms < 1 || terms > 2 || (terms == 2 && zstate) || (D.taps > 1 && !conv_state) ||
       (int64_t)nseq * D.H * ((D.dv + 31) / 32) > INT32_MAX)
     return (int)hipErrorInvalidValue;
   // wide workgroups share q, k and P among more columns; narrow ones where there are too few to fill the chip
   const bool wide = D.dv > 32 && (int64_t)nseq * D.H * ((D.dv + 63) / 64) >= 192;
-#define RUN(NK, WC, NORM)                                                                                               \
-  return launch<NK, WC, NORM>(qk, v, gb, log_decay, skip, scale, proj, state, zstate, floors, conv_state, seqs, nseq, cu, start, \
-                              slots, out, D, st)
-#define GO(NK)                             \
-  {                                        \
-    if (zstate && wide) RUN(NK, 4, true);  \
-    if (zstate) RUN(NK, 2, true);          \
-    if (wide) RUN(NK, 4, false);           \
-    RUN(NK, 2, false);                     \
+#define RUN(NK, WC, NORM, QT)                                                                                           \
+  return launch<NK, WC, NORM, QT>(qk, v, gb, log_decay, skip, scale, proj, state, zstate, floors, conv_state, seqs, nseq, cu, \
+                                  start, slots, out, D, st)
+#define GO(NK)                                    \
+  {                                               \
+    if (terms == 2 && wide) RUN(NK, 4, false, 2); \
+    if (terms == 2) RUN(NK, 2, false, 2);         \
+    if (zstate && wide) RUN(NK, 4, true, 1);      \
+    if (zstate) RUN(NK, 2, true, 1);              \
+    if (wide) RUN(NK, 4, false, 1);               \
+    RUN(NK, 2, false, 1);                         \
   }
   if (D.dk <= 32) GO(1)
   if (D.dk <= 64) GO(2)

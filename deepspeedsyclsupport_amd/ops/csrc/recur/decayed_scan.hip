@@ -9,7 +9,8 @@
 //  * prepare: q, k and v after (optionally) a causal convolution with bias and silu. A lane per few channels of a tile of
 //    consecutive tokens; inputs before the portion come from the sequence's state slot. Step sizes and log decays leave it in
 //    fp32, q / k / v in the storage type (they are activations).
-//  * split: q, k and v as they are, with (optionally) pairs of columns of q and k turned to their positions.
+//  * split: q, k and v as they are, with (optionally) pairs of columns of q and k turned to their positions. In 16-bit storage
+//    the turned ones leave as the sum of two terms: what enters a recurrence is not rounded to 16 bits again.
 //  * recur: one workgroup per (sequence, head, 64 value columns), the state in registers while the portion's tokens pass
 //    one by one: decoding, short portions, and everything in fp32 models. It also moves the convolution's windows on
 //    (prepare, which reads the old ones, has finished by then).
@@ -148,10 +149,10 @@ __global__ void __launch_bounds__(256) scan_prepare_kernel(
 }
 
 // One workgroup per token: the row's q, k and v head by head, pairs (i, i + half) of the first 2 half columns of q and k turned
-// by the token's angles cs [half, 2]
+// by the token's angles cs [half, 2]; `term` (0: none): from the first terms of q and k to what rounding them left out
 template <typename T, int V>
 __global__ void __launch_bounds__(256) scan_split_kernel(const T* __restrict__ proj, const float* __restrict__ cs, int half,
-                                                         T* __restrict__ qk, T* __restrict__ v_out, ScanDims D) {
+                                                         T* __restrict__ qk, T* __restrict__ v_out, int64_t term, ScanDims D) {
   const int t = blockIdx.x, tid = threadIdx.x;
   const T* row = proj + (int64_t)t * D.rows;
   const float* a = cs + (int64_t)t * half * 2;
@@ -173,11 +174,25 @@ __global__ void __launch_bounds__(256) scan_split_kernel(const T* __restrict__ p
       }
       stv<T, V>(dst + c, x);
       stv<T, V>(dst + half + c, y);
+      if (term) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          x[e] -= (float)(T)x[e];
+          y[e] -= (float)(T)y[e];
+        }
+        stv<T, V>(dst + term + c, x);
+        stv<T, V>(dst + term + half + c, y);
+      }
     } else {
       const int c = half + j * V;
       float u[V];
       ldv<T, V>(src + c, u);
       stv<T, V>(dst + c, u);
+      if (term) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) u[e] = 0.f;
+        stv<T, V>(dst + term + c, u);
+      }
     }
   }
   const int pv = D.dv / V;
@@ -192,8 +207,8 @@ __global__ void __launch_bounds__(256) scan_split_kernel(const T* __restrict__ p
 constexpr int LPC = 8;     // lanes per value column: lane p holds key rows 4 (p + LPC i) + 0..3
 constexpr int COLS = 64;   // value columns per workgroup
 
-// NORM: with a normaliser
-template <typename T, int NV, bool NORM>
+// NORM: with a normaliser; TWO: q and k of two terms
+template <typename T, int NV, bool NORM, bool TWO>
 __global__ void __launch_bounds__(LPC * COLS) scan_recur_kernel(
     const T* __restrict__ qk, const T* __restrict__ v, const float* __restrict__ gb, const float* __restrict__ log_decay,
     const float* __restrict__ skip, float scale, const T* __restrict__ proj, float* __restrict__ state,
@@ -221,6 +236,7 @@ __global__ void __launch_bounds__(LPC * COLS) scan_recur_kernel(
   // (every column of a copy has read it before its first one writes it: they are of one workgroup)
   if constexpr (NORM) __syncthreads();
   const float sk = skip ? skip[h] : 0.f, ld = log_decay ? log_decay[h] : 0.f;
+  const int64_t term = 2 * D.Hk * D.T * dks;
   for (int t = 0; t < n; ++t) {
     const int64_t tok = t0 + t;
     const float a = expf(gb ? gb[tok * 2 * D.H + h] : ld), b = gb ? gb[(tok * 2 + 1) * D.H + h] : 1.f;
@@ -232,6 +248,16 @@ __global__ void __launch_bounds__(LPC * COLS) scan_recur_kernel(
       float kf[4], qf[4];
       ldv<T, 4>(qk + D.k_at(g, tok) + kc, kf);
       ldv<T, 4>(qk + D.q_at(g, tok) + kc, qf);
+      if constexpr (TWO) {
+        float kl[4], ql[4];
+        ldv<T, 4>(qk + term + D.k_at(g, tok) + kc, kl);
+        ldv<T, 4>(qk + term + D.q_at(g, tok) + kc, ql);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          kf[e] += kl[e];
+          qf[e] += ql[e];
+        }
+      }
       const float z = k < dks ? 1.f : 0.f;  // rows past the width stay zero
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
@@ -268,18 +294,19 @@ __global__ void __launch_bounds__(LPC * COLS) scan_recur_kernel(
 
 template <typename T>
 int recur(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip, float scale,
-          const void* proj, float* state, float* zstate, const float* floors, void* conv_state, const int* list, int nlist, int lstride, const int* cu, const int* start,
+          const void* proj, float* state, float* zstate, const float* floors, void* conv_state, int terms, const int* list, int nlist, int lstride, const int* cu, const int* start,
           const int* slots, void* out, const ScanDims& D, hipStream_t st) {
   const dim3 grid(nlist, D.H, (D.dv + COLS - 1) / COLS);
   const int nt = D.dv >= COLS ? LPC * COLS : (LPC * D.dv + 63) / 64 * 64, nv = (D.dks() / 4 + LPC - 1) / LPC;
-#define RUN(NV, NORM)                                                                                                \
-  hipLaunchKernelGGL((scan_recur_kernel<T, NV, NORM>), grid, dim3(nt), 0, st, (const T*)qk, (const T*)v, gb, log_decay,   \
+#define RUN(NV, NORM, TWO)                                                                                                \
+  hipLaunchKernelGGL((scan_recur_kernel<T, NV, NORM, TWO>), grid, dim3(nt), 0, st, (const T*)qk, (const T*)v, gb, log_decay,   \
                      skip, scale, (const T*)proj, state, zstate, floors, (T*)conv_state, list, lstride, cu, start, slots, \
                      (T*)out, D)
-#define GO(NV)                  \
-  {                             \
-    if (zstate) RUN(NV, true);  \
-    else RUN(NV, false);        \
+#define GO(NV)                                 \
+  {                                            \
+    if (zstate) RUN(NV, true, false);          \
+    else if (terms == 2) RUN(NV, false, true); \
+    else RUN(NV, false, false);                \
   }
   if (nv <= 1) GO(1)
   else if (nv <= 2) GO(2)
@@ -340,16 +367,18 @@ extern "C" int ds_scan_prepare(const void* proj, const float* conv_w, const floa
 }
 
 // The same tensors straight from the projection's columns (no convolution, no activation), the first 2 half columns of every
-// head of q and k turned by cs [tokens, half, 2] (cos, sin)
-extern "C" int ds_scan_split(const void* proj, const float* cs, int half, void* qk, void* v, const int* dims, int tokens,
-                             int dtype, hipStream_t st) {
+// head of q and k turned by cs [tokens, half, 2] (cos, sin). terms 2: qk [2, 2, Hk, T, dks] takes q and k as sums of two
+extern "C" int ds_scan_split(const void* proj, const float* cs, int half, void* qk, void* v, int terms, const int* dims,
+                             int tokens, int dtype, hipStream_t st) {
   if (tokens <= 0) return 0;
   const ScanDims D{dims[0], dims[1], dims[2], dims[3], dims[4], dims[5], dims[6], dims[7], dims[8], dims[9], dims[10], dims[11],
                    tokens};
-  if (!scan_dims_ok(D) || half < 0 || 2 * half > D.dk || (half && !cs)) return (int)hipErrorInvalidValue;
+  if (!scan_dims_ok(D) || half < 0 || 2 * half > D.dk || (half && !cs) || terms < 1 || terms > 2)
+    return (int)hipErrorInvalidValue;
+  const int64_t term = terms == 2 ? 2 * (int64_t)D.Hk * D.T * D.dks() : 0;
   const int all = D.rows | D.q | D.k | D.v | D.dk | D.dv | half;
 #define GO(T, V) \
-  hipLaunchKernelGGL((scan_split_kernel<T, V>), dim3(tokens), dim3(256), 0, st, (const T*)proj, cs, half, (T*)qk, (T*)v, D)
+  hipLaunchKernelGGL((scan_split_kernel<T, V>), dim3(tokens), dim3(256), 0, st, (const T*)proj, cs, half, (T*)qk, (T*)v, term, D)
   if (dtype == DS_F32) {
     if (all % 4 == 0) GO(float, 4);
     else GO(float, 1);
@@ -366,22 +395,23 @@ extern "C" int ds_scan_split(const void* proj, const float* cs, int half, void* 
 }
 
 // list: sequences (indices into cu / start / slots) to run, `lstride` entries apart. zstate (null: no normaliser) [slots, H,
-// ceil(dv / 32), dks] with floors [tokens, H]
+// ceil(dv / 32), dks] with floors [tokens, H]; terms: of q and k (ds_scan_split)
 extern "C" int ds_scan_recur(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip,
                              float scale, const void* proj, float* state, float* zstate, const float* floors,
-                             void* conv_state, const int* list, int nlist, int lstride,
+                             void* conv_state, int terms, const int* list, int nlist, int lstride,
                              const int* cu, const int* start, const int* slots, void* out, const int* dims, int tokens,
                              int dtype, hipStream_t st) {
   if (nlist <= 0) return 0;
   const ScanDims D{dims[0], dims[1], dims[2], dims[3], dims[4], dims[5], dims[6], dims[7], dims[8], dims[9], dims[10], dims[11],
                    tokens};
-  if (!scan_dims_ok(D) || (!gb == !log_decay) || (!zstate != !floors) || (D.taps > 1 && !conv_state))
+  if (!scan_dims_ok(D) || (!gb == !log_decay) || (!zstate != !floors) || terms < 1 || terms > 2 || (terms == 2 && zstate) ||
+      (D.taps > 1 && !conv_state))
     return (int)hipErrorInvalidValue;
   if (dtype == DS_F32)
-    return recur<float>(qk, v, gb, log_decay, skip, scale, proj, state, zstate, floors, conv_state, list, nlist, lstride, cu,
-                        start, slots, out, D, st);
+    return recur<float>(qk, v, gb, log_decay, skip, scale, proj, state, zstate, floors, conv_state, terms, list, nlist, lstride,
+                        cu, start, slots, out, D, st);
   if (dtype == DS_BF16)
-    return recur<bf16>(qk, v, gb, log_decay, skip, scale, proj, state, zstate, floors, conv_state, list, nlist, lstride, cu,
-                       start, slots, out, D, st);
+    return recur<bf16>(qk, v, gb, log_decay, skip, scale, proj, state, zstate, floors, conv_state, terms, list, nlist, lstride,
+                       cu, start, slots, out, D, st);
   return (int)hipErrorInvalidValue;
 }

@@ -264,6 +264,8 @@ def _run_portions(f, proj, device, slot):
 @pytest.mark.parametrize("device,dtype,tol", CASES)
 @pytest.mark.parametrize("H,dk,dv", HEADS)
 def test_retention(device, dtype, tol, H, dk, dv):
+    """Portions in reused slots; the state is held to fp64 far below 16-bit precision whatever the storage type: turned keys
+    must not be rounded once more on their way into it."""
     rot, base, first, scale = dk // 2 // 2 * 2, 50.0, 16, dk**-0.5
     la = mixer_ops.ScanLayout(rows=first + H * (2 * dk + 2 * dv), q=first, k=first + H * dk, v=first + 2 * H * dk,
                               gate=first + H * (2 * dk + dv), Hk=H, H=H, dk=dk, dv=dv)
@@ -279,11 +281,37 @@ def test_retention(device, dtype, tol, H, dk, dv):
         x = x.double()
         part = lambda at, w: x[:, at:at + H * w].view(-1, H, w)
         q, k, v = part(la.q, dk), part(la.k, dk), part(la.v, dv)
-        turn = lambda y: O.rotate(y, rot, base).to(dtype).double()
+        turn = lambda y: O.rotate(y, rot, base)
         o = [O.decayed_scan(turn(q[:, h]), turn(k[:, h]) * scale, v[:, h], decay[h]) for h in range(H)]
-        # (rounding a turned query to bf16 may go another way in fp32 than in fp64: that is what tol is for)
         close(got[i], torch.stack(o, 1).reshape(-1, H * dv), tol)
+        for h in range(H):
+            wt = decay[h]**torch.arange(len(x) - 1, -1, -1).double()
+            close(state[slot[i], h, :, :dk], (v[:, h] * wt[:, None]).t() @ turn(k[:, h]), 2e-5)
     assert not state[..., dk:].any()
+
+
+@GPU
+@pytest.mark.parametrize("H,dk,dv,S,n", [(2, 64, 64, 3, 300), (16, 128, 128, 16, 130), (3, 96, 40, 2, 257), (12, 256, 64, 20, 100),
+                                         (2, 256, 96, 1, 200), (1, 24, 16, 2, 129)])
+def test_turned_read_out(H, dk, dv, S, n):
+    """Read-outs of turned keys and queries by chunks (narrow and wide workgroups, both chunk lengths) equal those token by
+    token to well below 16 bits before they are stored."""
+    la = mixer_ops.ScanLayout(rows=H * (2 * dk + dv), q=0, k=H * dk, v=2 * H * dk, gate=0, Hk=H, H=H, dk=dk, dv=dv)
+    proj = rnd(S * n, la.rows, seed=3).bfloat16().cuda()
+    freq = torch.tensor([100.0**(-2 * i / dk) for i in range(dk // 2)], dtype=torch.float64, device="cuda")
+    ld, outs = torch.full((H, ), -0.02, device="cuda"), []
+    for step in (n, 16):
+        state, out = torch.zeros(S, H, dv, dk, device="cuda"), torch.empty(S, n, H * dv, device="cuda")
+        for at in range(0, n, step):
+            c = min(step, n - at)
+            mm, _ = meta([(at, c)] * S, "cuda", slots=range(S))
+            x = proj.view(S, n, -1)[:, at:at + c].reshape(S * c, -1).contiguous()
+            out[:, at:at + c] = mixer_ops.retention(x, la, state, mm, ld, hybrid_ops.rope_table(mm.pos_ids, freq),
+                                                    1.0).view(S, c, -1).float()
+        outs.append((out, state))
+    (a, sa), (b, sb) = outs
+    close(sa, sb.cpu(), 1e-5)
+    assert (a - b).abs().max() <= 2**-8 * a.abs().max() and ((a - b) != 0).float().mean() < 0.05   # single roundings of the output
 
 
 def _gates(la, proj, at, b, cap, H):
