@@ -5,7 +5,7 @@
 //     o_i = e^{G_i} S0^T q_i + sum_{j <= i} P_ij v_j + D v_i,    P_ij = e^{G_i - G_j} b_j (q_i . k_j)
 //     S   = e^{G_C} S0 + sum_j e^{G_C - G_j} b_j k_j v_j^T
 // (the first two terms of o times a constant). The normaliser's products are the same with a single value column of ones:
-// z . q_i = e^{G_i} z0 . q_i + sum_j P_ij. Every workgroup keeps its own in LDS; it costs a few sums per chunk.
+// z . q_i = e^{G_i} z0 . q_i + sum_j P_ij. Every workgroup keeps its own, moved on by one of its pairs of waves.
 // One workgroup per (sequence, head, 16 WC value columns) walks the chunks. Two of its 2 WC waves share 16 value columns: each
 // keeps half of the key rows of their state in registers, in the result layout of the matrix instructions. The next state
 // accumulates into it, and the same registers are the left operand of the read-out (a product's k order is free as long as
@@ -21,8 +21,8 @@
 
 namespace {
 
-// tokens per chunk: two terms of wide keys leave room for 32
-constexpr int chunk_of(int NK, int QT) { return QT == 2 && NK > 4 ? 32 : 64; }
+// Tokens per chunk. 32 where two terms of q and k fill the LDS, or a wide normaliser the registers
+constexpr int chunk_of(int NK, bool NORM, int QT) { return (QT == 2 && NK >= 4) || (NORM && NK > 4) ? 32 : 64; }
 constexpr double LOG2E = 1.4426950408889634073599246810019;
 
 typedef short s16x4_t __attribute__((ext_vector_type(4)));
@@ -62,6 +62,14 @@ __device__ __forceinline__ void split3(const float (&x)[8], bf16x8& a, bf16x8& b
   c = __builtin_bit_cast(bf16x8, w);
 }
 
+// Sum over the lanes that share lane % 16, in all of them
+__device__ __forceinline__ float sum_rows16(float x) {
+  auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false, false);  // rows (0 0 2 2), (1 1 3 3)
+  x = __uint_as_float(a[0]) + __uint_as_float(a[1]);
+  a = __builtin_amdgcn_permlane32_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+  return __uint_as_float(a[0]) + __uint_as_float(a[1]);
+}
+
 // by value: a choice between array elements must not become one between addresses
 __device__ __forceinline__ f32x4 pick(bool c, f32x4 a, f32x4 b) {
   f32x4 r;
@@ -95,7 +103,7 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
     const float* __restrict__ log_decay, const float* __restrict__ skip, float scale, const bf16* __restrict__ proj,
     float* __restrict__ state, float* __restrict__ zstate, const float* __restrict__ floors, bf16* __restrict__ conv_state,
     const int* __restrict__ seqs, const int* __restrict__ cu, const int* __restrict__ start, const int* __restrict__ slots, bf16* __restrict__ out, ScanDims D) {
-  constexpr int C = chunk_of(NK, QT), PP = C + 8;   // PP: LDS row length of the weights
+  constexpr int C = chunk_of(NK, NORM, QT), PP = C + 8;   // PP: LDS row length of the weights
   constexpr int NT = 128 * WC, NW = 2 * WC, VT = 16 * WC, FT = C / 32;  // FT: token tiles a wave finishes
   constexpr int KP = 32 * NK + 8, VP = VT + 8;      // LDS row lengths of q and k, of v
   constexpr int KH = (NK + 1) / 2;                  // steps of a wave's half of the key rows
@@ -113,8 +121,8 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
   float* const eg = bs + 2 * NW * C;                              // [2 NW][C] e^{G_i}
   float* const ws = eg + 2 * NW * C;                              // [2 NW][C] e^{G_C - G_j} b_j
   float* const fl = ws + 2 * NW * C;                              // NORM: [2 NW][C] floors,
-  float* const zs = fl + 2 * NW * C;                              //   [32 NK] normaliser the chunk starts from,
-  float* const zq = zs + 32 * NK;                                 //   [C] its products with the queries,
+  float* const zs = fl + 2 * NW * C;                              //   [2][32 NK] normaliser the chunk starts from,
+  float* const zq = zs + 64 * NK;                                 //   [C] its products with the queries,
   float* const rs = zq + C;                                       //   [4][C] sums of P's rows over 16 columns each
 
   const int vts = (D.dv + VT - 1) / VT, bid = xcd_remap(blockIdx.x, gridDim.x);
@@ -129,6 +137,7 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
   float* st = state + (((int64_t)slots[seq] * D.H + h) * D.dv + min(col, D.dv - 1)) * dks;
 
   f32x4 S[2 * KH];  // rows k_first + 16 t + 4 q4 + 0..3
+  f32x4 Z[NORM ? 2 * KH : 1];
 #pragma unroll
   for (int t = 0; t < 2 * KH; ++t) {
     const int k = k_first + 16 * t + 4 * q4;
@@ -138,6 +147,12 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
   if constexpr (NORM) {  // (visible after the first barrier of the loop)
     const float* zt = zstate + D.z_at(slots[seq], h, v0);
     for (int k = tid; k < 32 * NK; k += NT) zs[k] = !fresh && k < dks ? zt[k] : 0.f;
+#pragma unroll
+    for (int t = 0; t < 2 * KH; ++t) {
+      const int k = k_first + 16 * t + 4 * q4;
+      Z[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (!fresh && k < dks) Z[t] = *reinterpret_cast<const f32x4*>(zt + k);
+    }
   }
   const float sk = skip ? skip[h] : 0.f, ld = log_decay ? log_decay[h] : 0.f;
   const bf16* qbase = qk + D.q_at(g, t0);
@@ -279,9 +294,7 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
           s[r] = j + r <= i ? f : 0.f;
         }
         if constexpr (NORM) {
-          float sum = (s[0] + s[1]) + (s[2] + s[3]);
-          sum += __shfl_xor(sum, 16, 64);
-          sum += __shfl_xor(sum, 32, 64);
+          const float sum = sum_rows16((s[0] + s[1]) + (s[2] + s[3]));
           if (q4 == 0) rs[jt * C + i] = sum;
         }
       }
@@ -330,6 +343,8 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
         }
       }
     }
+    float* const zc = zs + (c & 1) * 32 * NK;        // NORM: this chunk's normaliser, the next one's
+    float* const zn = zs + ((c & 1) ^ 1) * 32 * NK;
     if constexpr (NORM) {  // z0 . q: neighbouring lanes share a token, 8 key columns at a time
       constexpr int LP = NT / C;
       const int row = tid / LP, part = tid % LP;
@@ -337,7 +352,7 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
       for (int k = 8 * part; k < 32 * NK; k += 8 * LP) {
         float x[8], y[8];
         Vec8<bf16>::load(Qs + row * KP + k, x);
-        Vec8<float>::load(zs + k, y);
+        Vec8<float>::load(zc + k, y);
 #pragma unroll
         for (int e = 0; e < 8; ++e) a = fmaf(x[e], y[e], a);
       }
@@ -362,6 +377,12 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
 #pragma unroll
         for (int e = 0; e < 8; ++e) x[e] = (float)vf[s][e] * ws[cb + 32 * s + 8 * q4 + e];
         split3(x, u0, u1, u2);
+        bf16x8 z0, z1, z2;  // the first pair's waves move the normaliser on too, 16 times the same column
+        if (NORM && wc == 0) {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[e] = ws[cb + 32 * s + 8 * q4 + e];
+          split3(x, z0, z1, z2);
+        }
 #pragma unroll
         for (int t = 0; t < 2 * KH; ++t) {
           const bf16x8 kf = read_tr(Ks, KP, 32 * s + 8 * q4, 32 * s + 8 * q4 + 4, k_first + 16 * t, l16);
@@ -374,48 +395,20 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
           S[t] = mfma(kf, u2, S[t]);
           S[t] = mfma(kf, u1, S[t]);
           S[t] = mfma(kf, u0, S[t]);
-        }
-      }
-    }
-    lds_barrier();  // P and the partner's half are complete
-    if constexpr (NORM) {  // next normaliser: neighbouring lanes share 8 key columns and take every JP-th token
-      constexpr int JP = NT / (4 * NK) < 64 ? NT / (4 * NK) : 64;
-      const int k = tid / JP * 8, part = tid % JP;
-      if (NT / JP <= 4 * NK || k < 32 * NK) {
-        float a[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int j = 0; j < C / JP; ++j) {
-          float x[8];
-          Vec8<bf16>::load(Ks + (part + j * JP) * KP + k, x);
-          const float wj = ws[cb + part + j * JP];
-#pragma unroll
-          for (int e = 0; e < 8; ++e) a[e] = fmaf(x[e], wj, a[e]);
-        }
-        // sums over the JP lanes: while there are columns to share out, every exchange halves them
-        int n = 8, col = 0;
-#pragma unroll
-        for (int o = JP / 2; o > 0; o /= 2) {
-          const bool up = part & o;
-          if (n > 1) {
-            n /= 2;
-#pragma unroll
-            for (int e = 0; e < n; ++e) {
-              const float keep = up ? a[n + e] : a[e], give = up ? a[e] : a[n + e];
-              a[e] = keep + __shfl_xor(give, o, 64);
-            }
-            if (up) col += n;
-          } else {
-            a[0] += __shfl_xor(a[0], o, 64);
+          if (NORM && wc == 0) {
+            if (s == 0) Z[t] *= dc;
+            Z[t] = mfma(kf, z2, Z[t]);
+            Z[t] = mfma(kf, z1, Z[t]);
+            Z[t] = mfma(kf, z0, Z[t]);
           }
         }
-        constexpr int OWN = JP >= 8 ? 1 : 8 / JP;  // columns a lane ends up with; above 8 lanes several hold the same one
-        if (JP <= 8 || part % (JP / 8) == 0) {
-          const float dc = eg[cb + C - 1];
-#pragma unroll
-          for (int e = 0; e < OWN; ++e) zs[k + col + e] = fmaf(dc, zs[k + col + e], a[e]);
-        }
       }
     }
+    if (NORM && wc == 0 && rows_ok && l16 == 0) {
+#pragma unroll
+      for (int t = 0; t < 2 * KH; ++t) *reinterpret_cast<f32x4*>(zn + k_first + 16 * t + 4 * q4) = Z[t];
+    }
+    lds_barrier();  // P and the partner's half are complete
     // ---- within the chunk, this wave's token tiles
 #pragma unroll
     for (int k = 0; k < FT; ++k) {
@@ -434,7 +427,7 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
         const int r = 16 * i + l16;
         float z = eg[cb + r] * zq[r];
 #pragma unroll
-        for (int jt = 0; jt < 4; ++jt) {  // (tiles behind the diagonal hold leftovers)
+        for (int jt = 0; jt < C / 16; ++jt) {  // (tiles behind the diagonal hold leftovers)
           const float p = rs[jt * C + r];
           z += jt <= i ? p : 0.f;
         }
@@ -469,7 +462,7 @@ __global__ void __launch_bounds__(128 * WC, (NK <= 4 || WC == 4 ? 2 : 1)) decaye
   if constexpr (NORM) {  // (the loop ends with a barrier) every copy that is about this workgroup's columns
     for (int cc = 0; cc < VT && v0 + cc < D.dv; cc += Z_COLS) {
       float* zt = zstate + D.z_at(slots[seq], h, v0 + cc);
-      for (int k = tid; k < dks; k += NT) zt[k] = zs[k];
+      for (int k = tid; k < dks; k += NT) zt[k] = zs[(nc & 1) * 32 * NK + k];
     }
   }
   if (vt == 0 && D.taps > 1)
@@ -480,10 +473,10 @@ template <int NK, int WC, bool NORM, int QT>
 int launch(const void* qk, const void* v, const float* gb, const float* log_decay, const float* skip, float scale,
            const void* proj, float* state, float* zstate, const float* floors, void* conv_state, const int* seqs, int nseq, const int* cu, const int* start, const int* slots,
            void* out, const ScanDims& D, hipStream_t st) {
-  constexpr int VT = 16 * WC, C = chunk_of(NK, QT);
+  constexpr int VT = 16 * WC, C = chunk_of(NK, NORM, QT);
   constexpr int LDS = (2 * QT * C * (32 * NK + 8) + C * (VT + 8) + 3 * C * (C + 8)) * 2 + 2 * WC * C / 32 * 64 * 16 +
                       4 * WC * C * 20 +
-                      (NORM ? (4 * WC * C + 32 * NK + 5 * C) * 4 : 0);
+                      (NORM ? (4 * WC * C + 64 * NK + 5 * C) * 4 : 0);
   static bool attr = false;
   if (!attr) {
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(&decayed_chunk_kernel<NK, WC, NORM, QT>),
