@@ -8,21 +8,25 @@ constants as parameters:
 * `StreamResidual`    S fp32 residual streams, mixed by small matrices around every sublayer, fused with the pre-norm
 * `PostNormResidual`  one fp32 residual; the sublayers read it as it is and their outputs are RMS-normed before the sum
 * `PreNormResidual`   one fp32 residual with RMS norms on the sublayers' inputs
+* `SandwichResidual`  one fp32 residual with RMS norms on the sublayers' inputs and outputs, and optionally a gate on the outputs
 * `AttentionMixer`    GQA, key and value widths of their own, per-head query / key RMS norm, score cap, chunked
                       visibility, value mixing with an earlier layer; K / V live in the blocked cache
-* `LatentMixer`       attention over a shared low-rank latent with a rotated key part and a softmax sink; only the latent
-                      and that key part are cached
+* `LatentMixer`       attention over a shared low-rank latent with a rotated key part, optionally with a query latent, a softmax
+                      sink and a sliding window; only the latent and that key part are cached
 * `DeltaMixer`        gated delta rule behind short convolutions; its fp32 state lives in a slot per sequence
 * `Mamba2Mixer`       state-space recurrence with a scalar decay per head and token behind a short convolution
 * `LightningMixer`    linear attention with a constant decay per head
 * `RotaryAttention`   GQA with projection biases, query / key norms over all heads, partial rotation, chunked visibility and a
                       softmax sink
+* `WindowAttention`   GQA over a sliding window, queries and keys rotated and then normed head by head, a gate per head
+* `Mamba1Mixer`       selective state space: a decay per channel and state, behind a short convolution
 * `MatrixMemory`      recurrence with exponential input and forget gates, a running maximum and a normaliser
 * `Retention`         linear attention with rotated queries and keys and a constant decay per head
 * `ParallelMixer`     two of these on the same input, their weighted outputs summed
 * `ClampedMLP`        gated feed-forward with clamped gate and up branches
+* `GatedMLP`          gated (silu) feed-forward
 * `GeluMLP`           plain feed-forward with the exact gelu
-* `RoutedMLP`         gated experts, chosen per token among the best groups of experts
+* `RoutedMLP`         experts, chosen per token among the best groups of experts, optionally beside one that every token takes
 * `TokenSide`         a small embedding per layer and token, gated by the residual
 
 Per sublayer the launches are: residual + norm, one fused input projection, the mixer's kernels, the output projection.
@@ -50,11 +54,25 @@ def _shard(t, r, tp, dim=0):
     return t if tp == 1 else t.chunk(tp, dim)[r]
 
 
+def _up8(n):
+    return -(-n // 8) * 8
+
+
+def _fill_rows(w, rows, name):
+    """w [rows, ..] with rows of zeros up to a multiple of 8."""
+    if w.shape[0] != rows:
+        raise ValueError(f"{name} has {w.shape[0]} rows in the checkpoint, {rows} by the configuration")
+    return torch.cat([w, w.new_zeros(_up8(rows) - rows, *w.shape[1:])])
+
+
 class StreamResidual(nn.Module):
     """Mixing weights of one sublayer: in_ [S], mix [S from, S to], out [S] (identity for a plain residual)."""
 
-    def __init__(self, streams, width, device):
+    extensions = ("ds_hybrid_ops", )
+
+    def __init__(self, spec, device, side=False):
         super().__init__()
+        streams, width = spec.streams, spec.hidden_size
         self.norm_w = _f32((width, ), 1.0, device)
         self.in_ = _f32((streams, ), 1.0, device)
         self.out = _f32((streams, ), 1.0, device)
@@ -70,15 +88,15 @@ class StreamResidual(nn.Module):
 
     def enter(self, spec, x, pending):
         """Close the sublayer before (its output and residual weights) and norm this one's input."""
-        y, prev = pending
+        y, prev, _ = pending
         return ops.stream_norm(x, y, prev.mix, prev.out, spec.residual_mult, self.in_, self.norm_w, spec.norm_eps)
 
-    def finish(self, model, x, y, rows):
+    def finish(self, model, x, y, rows, gate=None):
         """Normed output rows of the model; this is the last sublayer's residual."""
         return ops.stream_norm(x, y, self.mix, self.out, model.spec.residual_mult, None, model.norm_w,
                                model.spec.norm_eps, rows=rows)
 
-    def peek(self, spec, x, y):
+    def peek(self, spec, x, y, gate=None):
         """Sum of the streams after this sublayer."""
         return (torch.einsum("st,nsw->ntw", self.mix, x) +
                 spec.residual_mult * self.out[None, :, None] * y[:, None].float()).sum(1)
@@ -87,9 +105,11 @@ class StreamResidual(nn.Module):
 class PostNormResidual(nn.Module):
     """Norm weight of one sublayer's output: x <- x + y / rms(y) * w."""
 
-    def __init__(self, streams, width, device):
+    extensions = ("ds_mixer_ops", )
+
+    def __init__(self, spec, device, side=False):
         super().__init__()
-        self.norm_w = _f32((width, ), 1.0, device)
+        self.norm_w = _f32((spec.hidden_size, ), 1.0, device)
 
     @staticmethod
     def begin(model, ids):
@@ -97,14 +117,14 @@ class PostNormResidual(nn.Module):
         return x, mixer_ops.post_norm(x, None, None, 0.0, ids=ids, embed=model.embed)
 
     def enter(self, spec, x, pending):
-        y, prev = pending
+        y, prev, _ = pending
         return mixer_ops.post_norm(x, y, prev.norm_w, spec.norm_eps)
 
-    def finish(self, model, x, y, rows):
+    def finish(self, model, x, y, rows, gate=None):
         return mixer_ops.post_norm(x, y, self.norm_w, model.spec.norm_eps, rows=rows, final_w=model.norm_w,
                                    mult=model.spec.logit_scale)
 
-    def peek(self, spec, x, y):
+    def peek(self, spec, x, y, gate=None):
         y = y.float()
         return x + y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + spec.norm_eps) * self.norm_w
 
@@ -113,9 +133,11 @@ class PreNormResidual(nn.Module):
     """Norm weight of one sublayer's input: x <- x + f(x / rms(x) * w). A sublayer may hand over an `ExpertSum`; it is summed
     in the pass that adds it."""
 
-    def __init__(self, streams, width, device):
+    extensions = ("ds_expert_ops", )
+
+    def __init__(self, spec, device, side=False):
         super().__init__()
-        self.norm_w = _f32((width, ), 1.0, device)
+        self.norm_w = _f32((spec.hidden_size, ), 1.0, device)
 
     @staticmethod
     def begin(model, ids):
@@ -127,19 +149,52 @@ class PreNormResidual(nn.Module):
     def enter(self, spec, x, pending):
         return expert_ops.pre_norm(x, pending[0], self.norm_w, spec.norm_eps)
 
-    def finish(self, model, x, y, rows):
+    def finish(self, model, x, y, rows, gate=None):
         return expert_ops.pre_norm(x, y, model.norm_w, model.spec.norm_eps, rows=rows)
 
-    def peek(self, spec, x, y):
+    def peek(self, spec, x, y, gate=None):
         return x + (y.sum() if isinstance(y, expert_ops.ExpertSum) else y).float()
 
 
-RESIDUALS = {"streams": StreamResidual, "post_norm": PostNormResidual, "pre_norm": PreNormResidual}
+class SandwichResidual(PreNormResidual):
+    """Norm weights of one sublayer's input and output: x <- x + g / rms(g) * post_w with g = sigmoid(gate + gate_b) * f(h),
+    h = x / rms(x) * norm_w; without `spec.residual_gate`, g = f(h). The gate is a linear map of h. `side`: a sublayer that reads x
+    as it is, without a gate."""
+
+    def __init__(self, spec, device, side=False):
+        super().__init__(spec, device)
+        self.side = side
+        if side:
+            del self.norm_w
+        self.post_w = _f32((spec.hidden_size, ), 1.0, device)
+        if spec.residual_gate and not side:
+            self.gate_b = _f32((spec.hidden_size, ), 0.0, device)
+
+    def _close(self, gate):
+        """How `pre_norm` takes this sublayer's output."""
+        return dict(post_w=self.post_w, gate=gate, gate_b=None if gate is None else self.gate_b)
+
+    def enter(self, spec, x, pending):
+        y, prev, gate = pending
+        return expert_ops.pre_norm(x, y, None if self.side else self.norm_w, spec.norm_eps, **prev._close(gate))
+
+    def finish(self, model, x, y, rows, gate=None):
+        return expert_ops.pre_norm(x, y, model.norm_w, model.spec.norm_eps, rows=rows, **self._close(gate))
+
+    def peek(self, spec, x, y, gate=None):
+        y = (y.sum() if isinstance(y, expert_ops.ExpertSum) else y).float()
+        if gate is not None:
+            y = y * torch.sigmoid(gate.float() + self.gate_b)
+        return x + y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + spec.norm_eps) * self.post_w
+
+
+RESIDUALS = {"streams": StreamResidual, "post_norm": PostNormResidual, "pre_norm": PreNormResidual, "sandwich": SandwichResidual}
 
 
 class Mixer:
     """What a mixer may leave at its default. `rows`: width of the fused input projection; `out_width`: of its output."""
     extra_projections = ()   # names of weight matrices beside the input and output projection
+    strided = False          # takes projection rows that are columns of wider ones
     extensions = ()          # native extensions its ops come from
 
     def parameters(self, device):
@@ -196,7 +251,7 @@ class AttentionMixer(Mixer):
         return self.G, self.dk, self.dv
 
     def run(self, layer, h, meta, cache, carry):
-        qkv = layer._linear(h, "qkv_w")
+        qkv = layer.project(h, carry)
         kc, vc = cache.k[layer.layer_idx], cache.v[layer.layer_idx]
         v_first = None
         if self.v_mix:  # the first mixing layer lends its values to the later ones of the same step
@@ -242,64 +297,186 @@ class DeltaMixer(Mixer):
                                                                                          dtype)}
 
     def run(self, layer, h, meta, cache, carry):
-        proj = layer._linear(h, "qkv_w")
+        proj = layer.project(h, carry)
         st = cache.state[layer.layer_idx]
         return ops.delta_rule(proj, layer.conv_w, layer.a_log, layer.dt_bias, layer.head_norm, layer.spec.norm_eps,
                               st["state"], st["conv"], meta, self.Hk, self.H, self.dk, self.dv)
 
 
+class Rotation:
+    """Frequencies of rotated positions: pair i of `dims` / 2 turns by position * base^(-2 i / dims), slowed down by a scaling:
+
+    * "linear": all by `factor`
+    * "yarn": pairs that turn less than `slow` times within `original` positions by `factor`, those that turn more than `fast`
+      times not at all, with a linear ramp between; cosine and sine grow by `mult`
+
+    Pair i is columns (i, i + dims / 2); "neighbours": (2 i, 2 i + 1). The batch's angle table is made once per step for all
+    layers with the same constants."""
+
+    def __init__(self, rot, width):
+        self.dims, self.base, self.neighbours = int(rot["dims"]), float(rot["base"]), rot.get("pairs") == "neighbours"
+        scaling = rot.get("scaling") or {}
+        self.factor, self.kind = float(scaling.get("factor", 1.0)), scaling.get("type", "linear")
+        if self.dims % 2 or not 0 <= self.dims <= width:
+            raise ValueError(f"{self.dims} rotated of {width} dimensions")
+        if self.kind not in ("linear", "yarn"):
+            raise NotImplementedError(f"no scaling {self.kind!r} of rotated positions")
+        self.mult, self.key = 1.0, (self.dims, self.base, self.factor)
+        if self.kind == "yarn":
+            self.original, self.turns = float(scaling["original"]), (float(scaling["fast"]), float(scaling["slow"]))
+            self.mult = 0.1 * math.log(self.factor) + 1.0
+            self.key += (self.original, *self.turns)
+
+    def _pair_of(self, turns):
+        """The (fractional) pair that turns so many times within the original length."""
+        return self.dims * math.log(self.original / (2 * math.pi * turns)) / (2 * math.log(self.base))
+
+    def frequencies(self, device):
+        i = torch.arange(self.dims // 2, dtype=torch.float64)
+        f = self.base**(-2 * i / max(self.dims, 1))
+        if self.kind == "linear":
+            return (f / self.factor).to(device)
+        lo, hi = max(math.floor(self._pair_of(self.turns[0])), 0), min(math.ceil(self._pair_of(self.turns[1])), self.dims - 1)
+        ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0, 1)
+        return (f / self.factor * ramp + f * (1 - ramp)).to(device)
+
+    def halves(self, w, first=0):
+        """Rows `first` .. of every head of w [heads, rows, ..] reordered so that pairs of neighbours become (i, i + dims / 2):
+        scores do not see an order that queries and keys share."""
+        if not self.neighbours:
+            return w
+        i = torch.arange(self.dims // 2)
+        at = torch.cat([torch.arange(first), first + 2 * i, first + 2 * i + 1, torch.arange(first + self.dims, w.shape[1])])
+        return w[:, at]
+
+    def angles(self, freq, meta, carry):
+        if not self.dims:
+            return None
+        tables = carry.setdefault("angles", {})
+        if self.key not in tables:
+            tables[self.key] = ops.rope_table(meta.pos_ids, freq, self.mult)
+        return tables[self.key]
+
+
 class LatentMixer(Mixer):
-    """Latent attention: queries through a latent of `q_rank`; keys and values are linear maps of a latent of `kv_rank`,
-    beside one rotated key part shared by all heads. The cache holds the latent and that part, one row per token."""
+    """Latent attention: keys and values are linear maps of a latent of `kv_rank`, beside one rotated key part shared by all
+    heads. The cache holds the latent and that part, one row per token. Queries pass a latent of `q_rank`, or none. `sink`: a
+    learned score per head joins the softmax; `mask`: a sliding window."""
     kind = "latent_attention"
-    extra_projections = ("uq_w", )
     extensions = ("ds_mixer_ops", )
+    strided = True
 
     def __init__(self, mx, tp):
         if mx["heads"] % tp:
             raise ValueError(f"{mx['heads']} heads over {tp} ranks")
         self.H, self.d, self.r, self.e = mx["heads"] // tp, mx["dim"], mx["rot_dim"], mx["vdim"]
-        self.q_rank, self.kv_rank = mx["q_rank"], mx["kv_rank"]
-        self.scale, self.base, self.rot = float(mx["scale"]), float(mx["rot"]["base"]), int(mx["rot"]["dims"])
-        if self.rot % 2 or self.rot > self.r:
-            raise ValueError(f"{self.rot} rotated of {self.r} dimensions")
-        self.rows = self.q_rank + self.kv_rank + self.r
+        self.q_rank, self.kv_rank = int(mx.get("q_rank") or 0), mx["kv_rank"]
+        self.scale, self.rot = float(mx["scale"]), Rotation(mx["rot"], mx["rot_dim"])
+        self.window = int((mx.get("mask") or {}).get("size") or 0)
+        self.sink = bool(mx.get("sink", True))
+        self.extra_projections = ("uq_w", ) if self.q_rank else ()
+        self.q_cols = self.q_rank or self.H * (self.d + self.r)
+        self.rows = self.q_cols + self.kv_rank + self.r
         self.out_width = self.H * self.e
 
     def parameters(self, device):
-        return {"q_norm": _f32((self.q_rank, ), 1.0, device), "kv_norm": _f32((self.kv_rank, ), 1.0, device),
-                "sink": _f32((self.H, ), 0.0, device)}
+        p = {"kv_norm": _f32((self.kv_rank, ), 1.0, device)}
+        if self.q_rank:
+            p["q_norm"] = _f32((self.q_rank, ), 1.0, device)
+        if self.sink:
+            p["sink"] = _f32((self.H, ), 0.0, device)
+        return p
 
     def matrices(self, dtype, device):
-        return {"uq_w": _empty((self.H * (self.d + self.r), self.q_rank), dtype, device),
-                "ukv_w": _empty((self.H * (self.d + self.e), self.kv_rank), dtype, device),    # [keys | values]
-                "ukt_w": _empty((self.H, self.kv_rank, self.d), dtype, device)}                # keys, turned over per head
+        m = {"ukv_w": _empty((self.H * (self.d + self.e), self.kv_rank), dtype, device),       # [keys | values]
+             "ukt_w": _empty((self.H, self.kv_rank, self.d), dtype, device)}                   # keys, turned over per head
+        if self.q_rank:
+            m["uq_w"] = _empty((self.H * (self.d + self.r), self.q_rank), dtype, device)
+        return m
 
     def constants(self, device):
-        i = torch.arange(self.rot // 2, dtype=torch.float64)
-        return {"rot_freq": (self.base**(-2 * i / max(self.rot, 1))).to(device)}
+        return {"rot_freq": self.rot.frequencies(device)}
 
     def shard(self, lw, r, tp):
         def s(n, dim=0):
             return _shard(lw[n], r, tp, dim)
 
-        uk = s("uk_w")
-        return {"qkv_w": torch.cat([lw["dq_w"], lw["dkv_w"]]), "uq_w": s("uq_w"), "ukv_w": torch.cat([uk, s("uv_w")]),
-                "ukt_w": uk.view(self.H, self.d, self.kv_rank).transpose(1, 2).contiguous(), "o_w": s("o_w", 1),
-                "q_norm": lw["q_norm"], "kv_norm": lw["kv_norm"], "sink": s("sink")}
+        def queries(n):
+            w = s(n)
+            return self.rot.halves(w.view(self.H, -1, w.shape[1]), self.d).reshape(w.shape)
+
+        uk, dkv = s("uk_w"), lw["dkv_w"]
+        dkv = self.rot.halves(dkv[None], self.kv_rank)[0]
+        out = {"qkv_w": torch.cat([lw["dq_w"] if self.q_rank else queries("q_w"), dkv]), "ukv_w": torch.cat([uk, s("uv_w")]),
+               "ukt_w": uk.view(self.H, self.d, self.kv_rank).transpose(1, 2).contiguous(), "o_w": s("o_w", 1),
+               "kv_norm": lw["kv_norm"]}
+        if self.q_rank:
+            out.update(uq_w=queries("uq_w"), q_norm=lw["q_norm"])
+        if self.sink:
+            out["sink"] = s("sink")
+        return out
 
     def kv_geometry(self):
         return 1, self.kv_rank + self.r, 0
 
     def run(self, layer, h, meta, cache, carry):
-        down = layer._linear(h, "qkv_w")
-        lat = cache.k[layer.layer_idx]
-        cq = mixer_ops.latent_prepare(down, layer.q_norm, layer.kv_norm, layer.spec.norm_eps, layer.rot_freq, meta, lat,
-                                      self.q_rank)
-        q = layer._linear(cq, "uq_w").view(-1, self.H, self.d + self.r)
-        o = mixer_ops.latent_attention(q, lat, layer.ukv_w, layer.ukt_w, layer.rot_freq, layer.sink, meta, self.scale,
-                                       self.d, self.e)
+        proj, lat, Q = layer.project(h, carry), cache.k[layer.layer_idx], self.q_rank
+        cq = mixer_ops.latent_prepare(proj if Q else proj[:, self.q_cols:], layer.q_norm if Q else None, layer.kv_norm,
+                                      layer.spec.norm_eps, layer.rot_freq, meta, lat, Q, self.rot.mult)
+        q = layer._linear(cq, "uq_w") if Q else proj[:, :self.q_cols]
+        o = mixer_ops.latent_attention(q.unflatten(1, (self.H, self.d + self.r)), lat, layer.ukv_w, layer.ukt_w, layer.rot_freq,
+                                       layer.sink if self.sink else None, meta, self.scale, self.d, self.e, self.window,
+                                       self.rot.mult)
         return o.view(h.shape[0], self.out_width)
+
+
+class WindowAttention(Mixer):
+    """Grouped-query attention over a sliding window of `mask.size` keys. Queries and keys are rotated, then divided by their root
+    mean square head by head; every head's output is multiplied by the sigmoid of a linear map of the input."""
+    kind = "window_attention"
+    extensions = ("ds_attn_ops", )
+    strided = True
+
+    def __init__(self, mx, tp):
+        self.H, self.G, self.dk, self.dv = mx["heads"] // tp, mx["kv_heads"] // tp, mx["dim"], mx["vdim"]
+        if mx["heads"] % mx["kv_heads"] or mx["kv_heads"] % tp:
+            raise ValueError(f"{mx['heads']} query / {mx['kv_heads']} key heads over {tp} ranks")
+        self.scale, self.window = float(mx["scale"]), int((mx.get("mask") or {}).get("size") or 0)
+        self.rot = Rotation(mx["rot"], self.dk)
+        self.gate = (self.H + self.G) * self.dk + self.G * self.dv   # first of the gates' columns
+        self.rows = self.gate + self.H
+        self.out_width = self.H * self.dv
+
+    def constants(self, device):
+        return {"rot_freq": self.rot.frequencies(device)}
+
+    def shard(self, lw, r, tp):
+        def s(n):
+            return _shard(lw[n], r, tp)
+
+        def heads(n):   # the kernel turns neighbours
+            w = s(n)
+            return w if self.rot.neighbours else self._interleave(w)
+
+        return {"qkv_w": torch.cat([heads("q_w"), heads("k_w"), s("v_w"), s("g_w")]), "o_w": _shard(lw["o_w"], r, tp, 1)}
+
+    def _interleave(self, w):
+        """Rows (i, i + dims / 2) of every head side by side."""
+        half = self.rot.dims // 2
+        i = torch.arange(half)
+        at = torch.cat([torch.stack([i, i + half], 1).flatten(), torch.arange(2 * half, self.dk)])
+        return w.view(-1, self.dk, w.shape[1])[:, at].reshape(w.shape)
+
+    def kv_geometry(self):
+        return self.G, self.dk, self.dv
+
+    def run(self, layer, h, meta, cache, carry):
+        proj = layer.project(h, carry)
+        kc, vc = cache.k[layer.layer_idx], cache.v[layer.layer_idx]
+        q = ops.qk_norm_append(proj[:, :self.gate], None, None, layer.spec.norm_eps, None, None, meta.pos_ids, meta.seq_ids,
+                               meta.block_tables, kc, vc, self.H, self.rot.angles(layer.rot_freq, meta, carry))
+        o = ops.ragged_attention(q, kc, vc, meta, self.scale, window=self.window, gate=proj[:, self.gate:self.gate + self.H])
+        return o.reshape(h.shape[0], self.out_width)
 
 
 class ScanMixer(Mixer):
@@ -373,7 +550,7 @@ class Mamba2Mixer(ScanMixer):
         return out
 
     def run(self, layer, h, meta, cache, carry):
-        proj = layer._linear(h, "qkv_w")
+        proj = layer.project(h, carry)
         st = cache.state[layer.layer_idx]
         y = mixer_ops.decayed_scan(proj, self.lay, st["state"], meta, conv_w=layer.conv_w, conv_b=layer.conv_b,
                                    conv_state=st.get("conv"), a_log=layer.a_log, dt_bias=layer.dt_bias, skip=layer.skip)
@@ -401,10 +578,57 @@ class LightningMixer(ScanMixer):
                 "o_w": _shard(lw["o_w"], r, tp, 1)}
 
     def run(self, layer, h, meta, cache, carry):
-        proj = layer._linear(h, "qkv_w")
+        proj = layer.project(h, carry)
         y = mixer_ops.decayed_scan(proj, self.lay, cache.state[layer.layer_idx]["state"], meta, log_decay=layer.log_decay)
         return self._share(mixer_ops.gated_norm(y, proj, self.lay.gate, layer.head_norm, self.parts, layer.spec.norm_eps,
                                                 "sigmoid_after"), layer)
+
+
+class Mamba1Mixer(Mixer):
+    """Selective state space: behind a short convolution, every channel carries `state` numbers that decay at rates of their own,
+    with step sizes, inputs and read-outs that depend on the token. The steps come through a bottleneck of `dt_rank`. Every
+    rank of a tensor-parallel group runs all channels (the bottleneck mixes them) and hands its share on."""
+    kind = "mamba1"
+    extra_projections = ("x_w", )
+    extensions = ("ds_selective_ops", )
+    strided = True
+
+    def __init__(self, mx, tp):
+        self.inner, self.N, self.R, self.taps = mx["inner"], mx["state"], mx["dt_rank"], int(mx["conv"])
+        if self.inner % tp:
+            raise ValueError(f"{self.inner} channels over {tp} ranks")
+        self.rows, self.out_width = 2 * self.inner, self.inner // tp
+
+    def parameters(self, device):
+        C = self.inner
+        return {"conv_w": _f32((C, self.taps), 0.0, device), "conv_b": _f32((C, ), 0.0, device),
+                "a_log": _f32((C, self.N), 0.0, device), "dt_bias": _f32((C, ), 0.0, device), "skip": _f32((C, ), 0.0, device)}
+
+    def matrices(self, dtype, device):
+        return {"x_w": _empty((_up8(self.R + 2 * self.N), self.inner), dtype, device),
+                "dt_w": _empty((self.inner, self.R), dtype, device)}
+
+    def shard(self, lw, r, tp):
+        return {"qkv_w": lw["in_w"], "x_w": _fill_rows(lw["x_w"], self.R + 2 * self.N, "mix.x"), "dt_w": lw["dt_w"],
+                "o_w": _shard(lw["o_w"], r, tp, 1), **{n: lw[n] for n in ("conv_w", "conv_b", "a_log", "dt_bias", "skip")}}
+
+    def state_geometry(self, dtype):
+        g = {"state": ((self.inner, -(-self.N // 4) * 4), torch.float32)}
+        if self.taps > 1:
+            g["conv"] = ((self.taps - 1, self.inner), dtype)
+        return g
+
+    def run(self, layer, h, meta, cache, carry):
+        proj, st, C = layer.project(h, carry), cache.state[layer.layer_idx], self.inner
+        x = mixer_ops.causal_conv(proj[:, :C], layer.conv_w, layer.conv_b, st.get("conv"), meta)
+        low = layer._linear(x, "x_w")
+        dt = ops.linear(low[:, :self.R], layer.dt_w)
+        y = mixer_ops.selective_scan(x, dt, low[:, self.R:self.R + 2 * self.N], proj[:, C:2 * C], layer.dt_bias, layer.a_log,
+                                     layer.skip, st["state"], proj[:, :C], st.get("conv"), meta)
+        if self.out_width == C:
+            return y
+        r = layer.tp_rank * self.out_width
+        return y[:, r:r + self.out_width].contiguous()
 
 
 class SideMixer(Mixer):
@@ -452,34 +676,10 @@ class SideMixer(Mixer):
         out.copy_(whole[:, r:r + self.out_width])
 
     def run(self, layer, h, meta, cache, carry):
-        proj = layer._linear(h, "qkv_w")
+        proj = layer.project(h, carry)
         out = proj.new_empty(proj.shape[0], self.out_width)
         self.read_out(layer, proj, meta, cache, carry, out)
         return out
-
-
-class Rotation:
-    """Frequencies of rotated positions: pair i of `dims` / 2 turns by position * base^(-2 i / dims) / factor. The batch's angle
-    table is made once per step for all layers with the same constants."""
-
-    def __init__(self, rot, width):
-        self.dims, self.base = int(rot["dims"]), float(rot["base"])
-        self.factor = float((rot.get("scaling") or {}).get("factor", 1.0))
-        if self.dims % 2 or not 0 <= self.dims <= width:
-            raise ValueError(f"{self.dims} rotated of {width} dimensions")
-
-    def frequencies(self, device):
-        i = torch.arange(self.dims // 2, dtype=torch.float64)
-        return (self.base**(-2 * i / max(self.dims, 1)) / self.factor).to(device)
-
-    def angles(self, freq, meta, carry):
-        if not self.dims:
-            return None
-        tables = carry.setdefault("angles", {})
-        key = (self.dims, self.base, self.factor)
-        if key not in tables:
-            tables[key] = ops.rope_table(meta.pos_ids, freq)
-        return tables[key]
 
 
 class RotaryAttention(SideMixer):
@@ -637,7 +837,7 @@ class ParallelMixer(Mixer):
         return next((g for g in (s.state_geometry(dtype) for s in self.parts) if g), None)
 
     def run(self, layer, h, meta, cache, carry):
-        proj = layer._linear(h, "qkv_w")
+        proj = layer.project(h, carry)
         out, at = proj.new_empty(proj.shape[0], self.out_width), 0
         for s in self.parts:
             s.read_out(layer, proj, meta, cache, carry, out[:, at:at + s.out_width])
@@ -645,13 +845,14 @@ class ParallelMixer(Mixer):
         return out
 
 
-MIXERS = {m.kind: m for m in (AttentionMixer, LatentMixer, DeltaMixer, Mamba2Mixer, LightningMixer, RotaryAttention, MatrixMemory,
-                              Retention, ParallelMixer)}
+MIXERS = {m.kind: m for m in (AttentionMixer, LatentMixer, WindowAttention, DeltaMixer, Mamba1Mixer, Mamba2Mixer, LightningMixer,
+                              RotaryAttention, MatrixMemory, Retention, ParallelMixer)}
 
 
 class MLP:
     """What a feed-forward may leave at its default. `rows`: width of the first product's output; `ff`: of the second's input."""
     projections = ("fc1_w", "fc2_w")   # weights that are quantised / re-laid
+    entry = "fc1_w"                    # the plain projection of the input, which takes the rows of a residual gate along
     extensions = ()
 
     def matrices(self, width):
@@ -678,12 +879,31 @@ class ClampedMLP(MLP):
         return {"fc1_w": torch.cat([_shard(lw["gate_w"], r, tp), _shard(lw["up_w"], r, tp)]),
                 "fc2_w": _shard(lw["down_w"], r, tp, 1)}
 
-    def run(self, layer, h):
-        if "fc1_w" in layer.quant:
-            mid = ops.clamped_glu(layer._linear(h, "fc1_w"), self.limit)
+    def run(self, layer, h, carry):
+        if "fc1_w" in layer.quant or layer.gated:
+            mid = ops.clamped_glu(layer.project(h, carry, self).contiguous(), self.limit)
         else:
             mid = ops.glu_linear(h, layer.fc1_w, layer.sh.get("fc1_w"), self.limit)
         return layer._linear(mid, "fc2_w")
+
+
+class GatedMLP(MLP):
+    """Gated feed-forward: down (silu(gate x) * up x)."""
+    kind = "silu_glu"
+    extensions = ("ds_expert_ops", )
+
+    def __init__(self, ml, tp):
+        if ml["ff"] % tp:
+            raise ValueError(f"feed-forward width {ml['ff']} over {tp} ranks")
+        self.ff = ml["ff"] // tp
+        self.rows = 2 * self.ff
+
+    def shard(self, lw, r, tp):
+        return {"fc1_w": torch.cat([_shard(lw["gate_w"], r, tp), _shard(lw["up_w"], r, tp)]),
+                "fc2_w": _shard(lw["down_w"], r, tp, 1)}
+
+    def run(self, layer, h, carry):
+        return layer._linear(expert_ops.row_act(layer.project(h, carry, self), "silu_glu"), "fc2_w")
 
 
 class GeluMLP(MLP):
@@ -699,40 +919,54 @@ class GeluMLP(MLP):
     def shard(self, lw, r, tp):
         return {"fc1_w": _shard(lw["up_w"], r, tp), "fc2_w": _shard(lw["down_w"], r, tp, 1)}
 
-    def run(self, layer, h):
-        if "fc1_w" in layer.quant:
-            mid = mixer_ops.gelu(layer._linear(h, "fc1_w"))
+    def run(self, layer, h, carry):
+        if "fc1_w" in layer.quant or layer.gated:
+            mid = mixer_ops.gelu(layer.project(h, carry, self).contiguous())
         else:
             mid = ops.linear(h, layer.fc1_w, layer.sh.get("fc1_w"), act="gelu")
         return layer._linear(mid, "fc2_w")
 
 
 class RoutedMLP(MLP):
-    """Mixture of gated (silu) experts. The experts form equal groups; those of the best groups compete, the best are weighted
-    by their softmax over all, divided by its sum. Every rank routes for itself and holds a slice of every expert."""
+    """Mixture of experts: gated (silu) ones, or plain ones with `act` between their two maps. The experts form equal groups; those
+    of the best groups (by their `best` best members) compete, the best are weighted by their scores (the softmax over all, or
+    sigmoids), divided by the scores' sum, times a scale. `shared`: an expert that every token takes. Every rank routes for
+    itself and holds a slice of every expert."""
     kind = "routed"
-    projections = ()
     extensions = ("ds_expert_ops", )
+    entry = "shared1_w"
 
     def __init__(self, ml, tp):
         ro = ml["router"]
         groups = ro.get("groups") or {}
         self.E, self.top = int(ro["experts"]), int(ro["top"])
         self.groups, self.keep = int(groups.get("count", 1)), int(groups.get("keep", 1))
-        if ml["expert"]["ff"] % tp:
-            raise ValueError(f"expert width {ml['expert']['ff']} over {tp} ranks")
+        self.act, self.shared = ml.get("act", "silu_glu"), int((ml.get("shared") or {}).get("ff") or 0)
+        self.how = dict(score=ro.get("score", "softmax"), best=int(groups.get("best", 1)), scale=float(ro.get("scale", 1.0)),
+                        act=self.act)
+        if ml["expert"]["ff"] % tp or self.shared % tp:
+            raise ValueError(f"expert widths {ml['expert']['ff']}, {self.shared} over {tp} ranks")
         if self.groups < 1 or self.E % self.groups or not 1 <= self.keep <= self.groups or \
                 not 1 <= self.top <= self.keep * (self.E // self.groups):
             raise ValueError(f"{self.top} of {self.E} experts, {self.keep} of {self.groups} groups")
-        self.ff = ml["expert"]["ff"] // tp
+        self.ff, self.shared, self.parts = ml["expert"]["ff"] // tp, self.shared // tp, 2 if self.act == "silu_glu" else 1
+        self.rows = self.parts * self.shared
+        self.projections = ("shared1_w", "shared2_w") if self.shared else ()
 
     def matrices(self, width):
-        return {"router_w": (self.E, width), "fc1_w": (self.E, 2 * self.ff, width), "fc2_w": (self.E, width, self.ff)}
+        m = {"router_w": (self.E, width), "fc1_w": (self.E, self.parts * self.ff, width), "fc2_w": (self.E, width, self.ff)}
+        if self.shared:
+            m.update(shared1_w=(self.rows, width), shared2_w=(width, self.shared))
+        return m
 
     def shard(self, lw, r, tp):
-        return {"router_w": lw["router_w"], "fc1_w": torch.cat([_shard(lw["experts_gate"], r, tp, 1),
-                                                                _shard(lw["experts_up"], r, tp, 1)], 1),
-                "fc2_w": _shard(lw["experts_down"], r, tp, 2)}
+        names = ("gate", "up")[2 - self.parts:]
+        out = {"router_w": lw["router_w"], "fc1_w": torch.cat([_shard(lw[f"experts_{n}"], r, tp, 1) for n in names], 1),
+               "fc2_w": _shard(lw["experts_down"], r, tp, 2)}
+        if self.shared:
+            out.update(shared1_w=torch.cat([_shard(lw[f"shared_{n}"], r, tp) for n in names]),
+                       shared2_w=_shard(lw["shared_down"], r, tp, 1))
+        return out
 
     def operand_order(self, layer):
         """The expert weights once more as the products read them best, by name (nothing where the sizes forbid it)."""
@@ -741,23 +975,27 @@ class RoutedMLP(MLP):
         both = expert_ops.operand_order(layer.fc1_w.data), expert_ops.operand_order(layer.fc2_w.data)
         return {} if any(w is None for w in both) else {"experts": both}
 
-    def run(self, layer, h):
+    def run(self, layer, h, carry):
+        first = layer.project(h, carry, self) if self.shared or layer.gated else None
         y = expert_ops.experts(h, layer.router_w, layer.fc1_w, layer.fc2_w, self.top, self.groups, self.keep,
-                               layer.sh.get("experts"))
+                               layer.sh.get("experts"), **self.how)
+        if self.shared:
+            y.base = layer._linear(expert_ops.row_act(first, self.act), "shared2_w")
         return y if layer.tp == 1 else y.sum()   # ranks exchange plain sums
 
 
-MLPS = {m.kind: m for m in (ClampedMLP, GeluMLP, RoutedMLP)}
+MLPS = {m.kind: m for m in (ClampedMLP, GatedMLP, GeluMLP, RoutedMLP)}
 
 
 class TokenSide:
     """Per-layer token input: proj(gelu(gate x) * e), e the layer's part of a side embedding of the token."""
+    extensions = ("ds_mixer_ops", )
 
     def __init__(self, dim, layer_idx):
         self.dim, self.first = dim, layer_idx * dim
 
     def shard(self, lw):
-        return {"side_gate_w": lw["side_gate_w"], "side_proj_w": lw["side_proj_w"], "res_side.norm_w": lw["side_norm_w"]}
+        return {"side_gate_w": lw["side_gate_w"], "side_proj_w": lw["side_proj_w"]}
 
     def run(self, layer, h, carry):
         g = mixer_ops.token_gate(layer._linear(h, "side_gate_w"), carry["ids"], carry["side_embed"], self.first)
@@ -774,10 +1012,10 @@ class DSHybridLayer(ProjectionLayer):
         if ls["type"] not in MIXERS:
             raise NotImplementedError(f"layer {layer_idx}: no mixer {ls['type']!r}")
         residual = RESIDUALS[spec.residual]
-        self.tp_rank = 0
+        self.tp_rank, self.gated = 0, spec.residual_gate
         self.mixer = MIXERS[ls["type"]](ls["mixer"], tp_size)
-        self.res1 = residual(spec.streams, W, device)
-        self.qkv_w = _empty((self.mixer.rows, W), dtype, device)
+        self.res1 = residual(spec, device)
+        self.qkv_w = _empty((self._rows(self.mixer.rows), W), dtype, device)
         self.o_w = _empty((W, self.mixer.out_width), dtype, device)
         for name, p in {**self.mixer.parameters(device), **self.mixer.matrices(dtype, device)}.items():
             self.register_parameter(name, p)
@@ -789,12 +1027,15 @@ class DSHybridLayer(ProjectionLayer):
             if kind not in MLPS:
                 raise NotImplementedError(f"layer {layer_idx}: no feed-forward {kind!r}")
             self.mlp = MLPS[kind](ls["mlp"], tp_size)
-            self.res2 = residual(spec.streams, W, device)
-            for name, shape in self.mlp.matrices(W).items():
+            self.res2 = residual(spec, device)
+            shapes = self.mlp.matrices(W)
+            if self.gated:
+                shapes[self.mlp.entry] = (self._rows(self.mlp.rows), W)
+            for name, shape in shapes.items():
                 self.register_parameter(name, _empty(shape, dtype, device))
         if spec.token_side:
             self.side = TokenSide(spec.token_side, layer_idx)
-            self.res_side = residual(spec.streams, W, device)
+            self.res_side = residual(spec, device, side=True)
             self.side_gate_w = _empty((spec.token_side, W), dtype, device)
             self.side_proj_w = _empty((W, spec.token_side), dtype, device)
 
@@ -802,10 +1043,25 @@ class DSHybridLayer(ProjectionLayer):
         return ("qkv_w", "o_w") + self.mixer.extra_projections + (self.mlp.projections if self.mlp else ()) + \
             (("side_gate_w", "side_proj_w") if self.side else ())
 
+    def _rows(self, own):
+        """Rows of a sublayer's first projection: its own and, behind a whole number of 16-byte pieces, the residual gate's."""
+        return _up8(own) + self.spec.hidden_size if self.gated else own
+
     def _linear(self, x, name, bias=None):
         if name in self.quant:
             return super()._linear(x, name, bias)
         return ops.linear(x, getattr(self, name), self.sh.get(name))
+
+    def project(self, h, carry, mlp=None):
+        """The input projection of the mixer (or the feed-forward). What the residual gate's rows make of h goes to
+        carry["gate"]."""
+        part = mlp or self.mixer
+        y = self._linear(h, mlp.entry if mlp else "qkv_w")
+        if not self.gated:
+            return y
+        carry["gate"] = y[:, _up8(part.rows):]
+        own = y[:, :part.rows]
+        return own if mlp or part.strided else own.contiguous()
 
     def add_decode_layout(self):
         """Shuffled copies of the projections whose shape allows one (see the base class)."""
@@ -825,24 +1081,34 @@ class DSHybridLayer(ProjectionLayer):
             out.update(self.mlp.shard(lw, r, tp))
         if self.side:
             out.update(self.side.shard(lw))
+            out["res_side.post_w" if hasattr(self.res_side, "post_w") else "res_side.norm_w"] = lw["side_norm_w"]
         for q in (1, 2) if self.mlp else (1, ):
             out[f"res{q}.norm_w"] = lw[f"norm{q}_w"]
             for n in ("in", "out", "mix"):
                 if f"hc{q}_{n}" in lw:
                     out[f"res{q}.{'in_' if n == 'in' else n}"] = lw[f"hc{q}_{n}"]
+            if f"post{q}_w" in lw:
+                out[f"res{q}.post_w"] = lw[f"post{q}_w"]
+            if self.gated:
+                name, part, gate = "qkv_w" if q == 1 else self.mlp.entry, self.mixer if q == 1 else self.mlp, lw[f"rg{q}_w"]
+                own = out.get(name, gate.new_empty(0, gate.shape[1]))
+                out[name] = torch.cat([_fill_rows(own, part.rows, name), gate])
+                out[f"res{q}.gate_b"] = lw[f"rg{q}_b"]
         return out
 
     def forward(self, x, pending, meta, cache, carry):
-        """x: the residual, fp32. `pending`: (output, residual weights) of the sublayer before, not yet added, or the
+        """x: the residual, fp32. `pending`: (output, residual weights, gate) of the sublayer before, not yet added, or the
         input of the first layer. Returns this layer's last sublayer as pending."""
         h = pending if torch.is_tensor(pending) else self.res1.enter(self.spec, x, pending)
-        pending = (self._allreduce(self._linear(self.mixer.run(self, h, meta, cache, carry), "o_w")), self.res1)
+        y = self._allreduce(self._linear(self.mixer.run(self, h, meta, cache, carry), "o_w"))
+        pending = (y, self.res1, carry.pop("gate", None))
         if self.mlp:
             h = self.res2.enter(self.spec, x, pending)
-            pending = (self._allreduce(self.mlp.run(self, h)), self.res2)
+            y = self._allreduce(self.mlp.run(self, h, carry))
+            pending = (y, self.res2, carry.pop("gate", None))
         if self.side:
             h = self.res_side.enter(self.spec, x, pending)
-            pending = (self.side.run(self, h, carry), self.res_side)
+            pending = (self.side.run(self, h, carry), self.res_side, None)
         return pending
 
 
@@ -852,7 +1118,7 @@ class DSHybridModel(DSInferenceModel):
     def __init__(self, spec, tp_group=None, tp_size=1, tp_rank=0, dtype=torch.bfloat16, device=None):
         super().__init__(spec, tp_group, tp_size, tp_rank, dtype, device)
         if torch.device(device or "cpu").type == "cuda":  # all at once: in a fresh checkout they compile side by side
-            parts = [p for la in self.layers for p in (la.mixer, la.mlp) if p]
+            parts = [p for la in self.layers for p in (la.mixer, la.mlp, la.side, la.res1) if p]
             op_builder.prepare(sorted({"ds_gemv_ops", *(e for p in parts for e in p.extensions)}))
         self.norm_w = _f32((spec.hidden_size, ), 1.0, device)  # norms read the fp32 residual
         if spec.token_side:
@@ -888,12 +1154,12 @@ class DSHybridModel(DSInferenceModel):
         for layer in self.layers:
             pending = layer(x, pending, meta, self.cache, carry)
             if trace is not None:
-                y, r = pending
-                trace.append(r.peek(spec, x, y))
+                y, r, gate = pending
+                trace.append(r.peek(spec, x, y, gate))
         if meta.last_idx.numel() == 0:
             return tokens.new_empty((0, spec.vocab_size), dtype=self.dtype)
-        y, r = pending
-        return self._logits(r.finish(self, x, y, meta.last_idx.to(torch.int32)))
+        y, r, gate = pending
+        return self._logits(r.finish(self, x, y, meta.last_idx.to(torch.int32), gate))
 
     def _logits(self, h):
         return self._gather_vocab(ops.linear(h, self.lm_head, getattr(self, "lm_head_sh", None)))

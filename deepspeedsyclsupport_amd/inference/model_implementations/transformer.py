@@ -15,7 +15,7 @@ import math
 from array import array
 from dataclasses import dataclass, field
 from itertools import accumulate, repeat
-from typing import List, Optional
+from typing import Dict, List, Optional
 
 import torch
 import torch.nn as nn
@@ -69,7 +69,8 @@ class DSModelSpec:
     streams: int = 1                 # residual streams (hyper-connections)
     residual_mult: float = 1.0       # factor of every sublayer's output
     residual: str = "streams"        # "streams" (pre-norm over the streams) | "post_norm" (norms on sublayer outputs) |
-                                     # "pre_norm" (one fp32 residual, RMS norms on sublayer inputs)
+                                     # "pre_norm" (one fp32 residual, RMS norms on sublayer inputs) | "sandwich" (on both)
+    residual_gate: bool = False      # sublayer outputs times a sigmoid of a linear map of their input ("sandwich")
     token_side: int = 0              # width of a side embedding per layer and token (0: none)
     logit_scale: float = 1.0
     embed_scale: float = 1.0         # factor of the embedding rows ("pre_norm" residual)
@@ -184,10 +185,31 @@ class RaggedMeta:
     n_short: int = 0                 # sequences [0, n_short) are decodes or short portions
     kv_offs: Optional[torch.Tensor] = None   # [S - n_short + 1] offsets of the other sequences' contexts laid end to end
     kv_total: int = 0                # ... and their end
+    seen: Dict[int, tuple] = field(default_factory=dict)   # `contexts` by window
 
     SHORT_TOKENS = 64    # portions up to this long count as short
     STATE_CHUNK = 64     # tokens per chunk of a recurrent layer's parallel form
     STEP_TOKENS = 16     # portions up to this long pass a recurrent layer token by token
+
+    KEY_TILE = 64        # keys per tile of prefill attention
+
+    def contexts(self, window=0):
+        """(offsets, first keys, total) of the long portions' contexts laid end to end, without what no token of the portion
+        sees through a sliding window; a context starts with a whole tile. First keys None: all contexts are whole."""
+        if window not in self.seen:
+            S, tile = len(self.start_host), self.KEY_TILE
+            starts = self.start_host[self.n_short:]
+            first = [max(st - window + 1, 0) // tile * tile if window else 0 for st in starts]
+            if not any(first):
+                self.seen[window] = self.kv_offs, None, self.kv_total
+            else:
+                lens = [self.cu_host[i + 1] - self.cu_host[i] for i in range(self.n_short, S)]
+                offs = list(accumulate((st + n - f for st, n, f in zip(starts, lens, first)), initial=0))
+                buf = torch.tensor(offs + first, dtype=torch.int32)
+                if self.cu_q.is_cuda:
+                    buf = buf.pin_memory().to(self.cu_q.device, non_blocking=True)
+                self.seen[window] = buf[:len(offs)], buf[len(offs):], offs[-1]
+        return self.seen[window]
 
     @staticmethod
     def build(starts, n_new, block_lists, n_decode, block_size, device, slots=None, logit_rows=None):

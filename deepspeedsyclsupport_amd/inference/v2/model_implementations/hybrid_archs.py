@@ -19,6 +19,9 @@ _MIXER_TENSORS = {  # checkpoint name below `<layer>.mix.` -> canonical key
               "k.conv": "k_conv", "v.conv": "v_conv", "A_log": "a_log", "dt_bias": "dt_bias", "norm": "head_norm"},
     "latent_attention": {"dq": "dq_w", "dq.norm": "q_norm", "uq": "uq_w", "dkv": "dkv_w", "dkv.norm": "kv_norm",
                          "uk": "uk_w", "uv": "uv_w", "sink": "sink", "o": "o_w"},
+    "window_attention": {"q": "q_w", "k": "k_w", "v": "v_w", "g": "g_w", "o": "o_w"},
+    "mamba1": {"in": "in_w", "conv": "conv_w", "conv.b": "conv_b", "x": "x_w", "dt": "dt_w", "dt.b": "dt_bias", "A_log": "a_log",
+               "D": "skip", "o": "o_w"},
     "mamba2": {"in": "in_w", "conv": "conv_w", "conv.b": "conv_b", "dt_bias": "dt_bias", "A_log": "a_log", "D": "skip",
                "norm": "head_norm", "o": "o_w"},
     "lightning": {"q": "q_w", "k": "k_w", "v": "v_w", "g": "g_w", "o": "o_w", "norm": "head_norm"},
@@ -31,8 +34,9 @@ _MIXER_TENSORS = {  # checkpoint name below `<layer>.mix.` -> canonical key
 _MIXER_TENSORS["parallel"] = {f"{side}.{n}": f"{side}_{key}" for side, cls in ParallelMixer.sides
                               for n, key in _MIXER_TENSORS[cls.kind].items()}
 _MLP_TENSORS = {"dense": {"gate": "gate_w", "up": "up_w", "down": "down_w"}, "gelu": {"up": "up_w", "down": "down_w"},
-                "routed": {"router": "router_w"}}
-_EXPERT_TENSORS = {"gate": "experts_gate", "up": "experts_up", "down": "experts_down"}
+                "silu_glu": {"gate": "gate_w", "up": "up_w", "down": "down_w"}, "routed": {"router": "router_w"}}
+_EXPERT_TENSORS = ("gate", "up", "down")   # (a plain expert has no gate)
+_SANDWICH_TENSORS = {"norm{}b": "post{}_w", "rg{}": "rg{}_w", "rg{}.b": "rg{}_b"}
 _SIDE_TENSORS = {"side.gate": "side_gate_w", "side.proj": "side_proj_w", "side.norm": "side_norm_w"}
 
 
@@ -73,24 +77,40 @@ def container(name, tensors, may_lack=(), stacked=None, count=0):
         "PARAM_MAPPING": {src: f"{key}.params" for src, key in {**tensors, **lists}.items()}, "may_lack": may_lack})
 
 
-def layer_container(layer, streams=False, may_lack=(), side=False):
-    """Container class of one entry of the spec's layer list."""
+def _mixer_tensors(layer):
+    tensors, mx = dict(_MIXER_TENSORS[layer["type"]]), layer["mixer"]
+    if mx.get("v_mix"):
+        tensors["vmix"] = "vmix"
+    if layer["type"] == "latent_attention":
+        if not mx.get("q_rank"):   # queries straight from the input
+            tensors = {n: key for n, key in tensors.items() if n not in ("dq", "dq.norm", "uq")}
+            tensors["q"] = "q_w"
+        if not mx.get("sink", True):
+            del tensors["sink"]
+    return tensors
+
+
+def layer_container(layer, streams=False, may_lack=(), side=False, sandwich=False):
+    """Container class of one entry of the spec's layer list. `sandwich`: norms on the sublayers' outputs too, and gates."""
     if layer["type"] not in _MIXER_TENSORS:
         raise NotImplementedError(f"no mixer {layer['type']!r}")
-    tensors = {f"mix.{n}": key for n, key in _MIXER_TENSORS[layer["type"]].items()}
+    tensors = {f"mix.{n}": key for n, key in _mixer_tensors(layer).items()}
     lists, count = {}, 0
-    if layer["mixer"].get("v_mix"):
-        tensors["mix.vmix"] = "vmix"
     if layer.get("mlp"):
         if layer["mlp"].get("kind") not in _MLP_TENSORS:
             raise NotImplementedError(f"no feed-forward {layer['mlp'].get('kind')!r}")
         if layer["mlp"]["kind"] == "routed":
-            lists, count = {f"mlp.e*.{n}": key for n, key in _EXPERT_TENSORS.items()}, layer["mlp"]["router"]["experts"]
+            names = _EXPERT_TENSORS[0 if layer["mlp"].get("act", "silu_glu") == "silu_glu" else 1:]
+            lists, count = {f"mlp.e*.{n}": f"experts_{n}" for n in names}, layer["mlp"]["router"]["experts"]
+            if layer["mlp"].get("shared"):
+                tensors.update({f"mlp.shared.{n}": f"shared_{n}" for n in names})
         tensors.update({f"mlp.{n}": key for n, key in _MLP_TENSORS[layer["mlp"]["kind"]].items()})
     for q in (1, 2) if layer.get("mlp") else (1, ):
         tensors[f"norm{q}"] = f"norm{q}_w"
         if streams:
             tensors.update({f"hc{q}.{n}": f"hc{q}_{n}" for n in ("in", "out", "mix")})
+        if sandwich:
+            tensors.update({n.format(q): key.format(q) for n, key in _SANDWICH_TENSORS.items()})
     if side:
         tensors.update(_SIDE_TENSORS)
     return container("HybridLayerContainer", tensors, may_lack, lists, count)
@@ -191,4 +211,50 @@ class LefisunPolicy(InferenceV2Policy):
         cmap = ContainerMap()
         cmap.set_transformer_params("l", [layer_container(la)(self._view) for la in self.layers()], sep="")
         cmap.set_non_transformer_params(TiedTopContainer(self._view))
+        return cmap
+
+
+@register
+class NigilornPolicy(InferenceV2Policy):
+    """Nigilorn: selective state spaces, windowed attention and windowed latent attention between norms on the sublayers' inputs
+    and gated outputs, dense layers and mixtures of plain experts beside a shared one, a token-side input in every layer."""
+    model_types = ("nigilorn", )
+    model_class = DSHybridModel
+
+    def layers(self):
+        """The config's layers in the spec's terms, with what the design fixes: rotation of neighbours and its scaling, no sinks,
+        routing by sigmoids, squared-relu experts."""
+        out = []
+        for i, la in enumerate(_renamed(self._model_config.layers, {"dense": "silu_glu", "moe": "routed"})):
+            kinds = {"attention": "window_attention", "latent_attention": "latent_attention", "mamba1": "mamba1"}
+            if la["type"] not in kinds:
+                raise NotImplementedError(f"layer {i}: no mixer {la['type']!r}")
+            mx, ml = dict(la["mixer"]), la["mlp"]
+            if "rot" in mx:
+                mx["rot"] = {**mx["rot"], "pairs": "neighbours"}
+                if mx["rot"].get("scaling"):
+                    mx["rot"]["scaling"] = {**mx["rot"]["scaling"], "type": "yarn"}
+            if la["type"] == "latent_attention":
+                mx["sink"] = False
+            if ml and ml["kind"] == "routed":
+                groups = ml["router"].get("groups") or {}
+                ml = {**ml, "act": "relu2", "router": {**ml["router"], "score": "sigmoid", "groups": {**groups, "best": 2}}}
+            out.append({"type": kinds[la["type"]], "mixer": mx, "mlp": ml})
+        return out
+
+    def spec(self):
+        c, layers = self._model_config, self.layers()
+        first = next((la["mixer"] for la in layers if la["type"] == "window_attention"), {"heads": 1, "vdim": c.width})
+        widths = [la["mlp"].get("ff") or la["mlp"]["expert"]["ff"] for la in layers if la["mlp"]]
+        return DSModelSpec(arch="nigilorn", vocab_size=c.vocab, hidden_size=c.width, num_layers=len(c.layers),
+                           num_heads=first["heads"], num_kv_heads=first.get("kv_heads", first["heads"]), head_dim=first["vdim"],
+                           intermediate_size=max(widths, default=0), norm="rms", norm_eps=float(c.norm["eps"]), pos="none",
+                           layer_specs=tuple(layers), residual="sandwich", residual_gate=True,
+                           token_side=int(c.token_side["dim"]))
+
+    def build_container_map(self):
+        cmap = ContainerMap()
+        cmap.set_transformer_params("l", [layer_container(la, side=True, sandwich=True)(self._view) for la in self.layers()],
+                                    sep="")
+        cmap.set_non_transformer_params(SideTopContainer(self._view))
         return cmap

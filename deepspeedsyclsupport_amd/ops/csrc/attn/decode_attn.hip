@@ -14,7 +14,7 @@
 //    last-block merge was measured 2x slower: the device-scope fences it needs write back L2.)
 // Optional ALiBi slopes (BLOOM) are applied on the fly. With a sliding window (Mistral) or chunked visibility only the
 // keys in sight are split and read. A second instantiation takes key and value widths of their own (multiples of 8), a
-// tanh score cap, a softmax sink per head and GQA groups of any size.
+// tanh score cap, a softmax sink per head, a gate per token and head, and GQA groups of any size.
 #include "../include/ds_hip.h"
 
 namespace {
@@ -38,7 +38,7 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
     float* __restrict__ part_acc,        // [B, Hq, S, dv]  (only if S > 1)
     float* __restrict__ part_ml,         // [B, Hq, S, 2]
     bf16* __restrict__ out,              // [B, Hq, dv], rows ldo apart (written directly when S == 1)
-    const float* __restrict__ sink, int64_t ldo, int Hq, int Hk, int BS, int max_blocks, int chunk, float scale, int window, int mask_chunk, float softcap, int dk_rt,
+    const float* __restrict__ sink, const bf16* __restrict__ gate, int64_t ldg, int64_t ldo, int Hq, int Hk, int BS, int max_blocks, int chunk, float scale, int window, int mask_chunk, float softcap, int dk_rt,
     int dv_rt) {
   constexpr bool EXT = DK == 0;
   static_assert(EXT || (DK % 16 == 0 && DK >= 64 && DK <= 256 && DK == DV), "head dim");
@@ -192,6 +192,7 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
           const float mn = fmaxf(m, sink[hq]), f = __expf(m - mn);
           r = s * f / fmaf(l, f, __expf(sink[hq] - mn));
         }
+        if (EXT && gate) r /= 1.f + __expf(-(float)gate[b * ldg + hq]);
         out[(int64_t)b * ldo + hq * dv + idx] = (bf16)r;
       } else {
         part_acc[(((int64_t)b * Hq + hq) * S + split) * dv + idx] = s;
@@ -208,7 +209,8 @@ __global__ void __launch_bounds__(THREADS) paged_decode_kernel(
 // blockDim.x = D, the value width
 __global__ void __launch_bounds__(256) combine_kernel(const float* __restrict__ part_acc,
                                                       const float* __restrict__ part_ml, bf16* __restrict__ out,
-                                                      const float* __restrict__ sink, int Hq, int64_t ldo, int S) {
+                                                      const float* __restrict__ sink, const bf16* __restrict__ gate,
+                                                      int64_t ldg, int Hq, int64_t ldo, int S) {
   const int bh = blockIdx.x, d = threadIdx.x, D = blockDim.x;
   const float sk = sink ? sink[bh % Hq] : -INFINITY;
   float M = sk;
@@ -221,6 +223,7 @@ __global__ void __launch_bounds__(256) combine_kernel(const float* __restrict__ 
     num = fmaf(w, part_acc[((int64_t)bh * S + s) * D + d], num);
     den = fmaf(w, l, den);
   }
+  if (gate) den *= 1.f + __expf(-(float)gate[bh / Hq * ldg + bh % Hq]);
   out[bh / Hq * ldo + bh % Hq * D + d] = (bf16)(den > 0.f ? num / den : 0.f);
 }
 
@@ -342,11 +345,11 @@ extern "C" int ds_paged_decode(const void* q, const void* kc, const void* vc, co
 #define LAUNCH(DD)                                                                                                  \
   hipLaunchKernelGGL((paged_decode_kernel<DD, DD>), grid, dim3(THREADS), lds, s, (const bf16*)q, (const bf16*)kc,       \
                      (const bf16*)vc, block_table, seq_lens, alibi, part_acc, part_ml, (bf16*)out, nullptr,          \
-                     (int64_t)Hq * DD, Hq, Hk, BS,                                                                   \
+                     nullptr, 0, (int64_t)Hq * DD, Hq, Hk, BS,                                                                   \
                      max_blocks, chunk, scale, window, 0, 0.f, DD, DD);                                             \
   DS_CHECK_LAUNCH();                                                                                                \
   if (splits > 1) {                                                                                                 \
-    hipLaunchKernelGGL(combine_kernel, dim3(B * Hq), dim3(DD), 0, s, part_acc, part_ml, (bf16*)out, nullptr, Hq, \
+    hipLaunchKernelGGL(combine_kernel, dim3(B * Hq), dim3(DD), 0, s, part_acc, part_ml, (bf16*)out, nullptr, nullptr, 0, Hq, \
                        (int64_t)Hq * DD, splits);                                                                     \
     DS_CHECK_LAUNCH();                                                                                              \
   }
@@ -361,12 +364,13 @@ extern "C" int ds_paged_decode(const void* q, const void* kc, const void* vc, co
 }
 
 // Key / value widths of their own (multiples of 8 up to 256), chunked and / or windowed visibility, score cap, softmax sink
-// [Hq] (or null), rows of out ldo elements apart. `splits`
+// [Hq] (or null), gate [B, Hq] (or null), its rows ldg and rows of out ldo elements apart. `splits`
 // from ds_paged_decode_splits(B, Hk, span) with span = the most keys in sight.
 extern "C" int ds_paged_decode_ext(const void* q, const void* kc, const void* vc, const int* block_table,
                                    const int* seq_lens, float* part_acc, float* part_ml, void* out, int B, int Hq, int Hk,
                                    int dk, int dv, int BS, int max_blocks, int span, int splits, float scale,
-                                   float softcap, int window, int mask_chunk, const float* sink, int64_t ldo, hipStream_t s) {
+                                   float softcap, int window, int mask_chunk, const float* sink, const void* gate,
+                                   int64_t ldg, int64_t ldo, hipStream_t s) {
   if (Hk <= 0 || Hq % Hk || dk % 8 || dv % 8 || dk <= 0 || dv <= 0 || dk > 256 || dv > 256 || splits <= 0 ||
       ldo < (int64_t)Hq * dv)
     return (int)hipErrorInvalidValue;
@@ -377,7 +381,7 @@ extern "C" int ds_paged_decode_ext(const void* q, const void* kc, const void* vc
   dim3 grid(B, Hk * ((Hq / Hk + MAXG - 1) / MAXG), splits);
 #define GO(LK, LV)                                                                                                  \
   hipLaunchKernelGGL((paged_decode_kernel<0, 0, LK, LV>), grid, dim3(THREADS), lds, s, (const bf16*)q, (const bf16*)kc, \
-                     (const bf16*)vc, block_table, seq_lens, nullptr, part_acc, part_ml, (bf16*)out, sink, ldo, Hq, Hk, BS,     \
+                     (const bf16*)vc, block_table, seq_lens, nullptr, part_acc, part_ml, (bf16*)out, sink, (const bf16*)gate, ldg, ldo, Hq, Hk, BS, \
                      max_blocks, chunk, scale, window, mask_chunk, softcap, dk, dv)
 #define ROW(LK)                 \
   {                             \
@@ -392,7 +396,8 @@ extern "C" int ds_paged_decode_ext(const void* q, const void* kc, const void* vc
 #undef GO
   DS_CHECK_LAUNCH();
   if (splits > 1) {
-    hipLaunchKernelGGL(combine_kernel, dim3(B * Hq), dim3(dv), 0, s, part_acc, part_ml, (bf16*)out, sink, Hq, ldo, splits);
+    hipLaunchKernelGGL(combine_kernel, dim3(B * Hq), dim3(dv), 0, s, part_acc, part_ml, (bf16*)out, sink,
+                       (const bf16*)gate, ldg, Hq, ldo, splits);
     DS_CHECK_LAUNCH();
   }
   return 0;

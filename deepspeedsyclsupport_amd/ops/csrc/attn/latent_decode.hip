@@ -9,7 +9,8 @@
 //  * softmax weights go through LDS as two bf16 terms (16 mantissa bits);
 //  * values: O^T += V^T P^T, wave w a quarter of the latent's columns; V^T comes out of the same key tile by transposing
 //    LDS reads.
-// Ranges leave fp32 partial sums that a combine pass merges. The sink joins the denominator once, at the end.
+// Ranges leave fp32 partial sums that a combine pass merges. The sink, if there is one, joins the denominator once, at the end.
+// With a sliding window the ranges start where the sequence's first new token sees its first key.
 #include "ds_hip.h"
 
 namespace {
@@ -36,7 +37,7 @@ struct LatArgs {
   const int* cu;
   const int* start;
   const float* sink;  // [H] or null
-  int first, tok_base, H, R, r, BS, max_blocks, range, splits;
+  int first, tok_base, H, R, r, BS, max_blocks, range, splits, window;
   int64_t rows;  // T H
   float c;       // scale * log2(e)
 };
@@ -57,7 +58,7 @@ __global__ void __launch_bounds__(NT) latent_decode_kernel(LatArgs a) {
   const int st = a.start[s];
   // keys this block may see: up to the last row's position
   const int end = st + min(n - 1, (row0 + rows_b - 1) / a.H) + 1;
-  const int k_lo = split * a.range, k_hi = min(end, k_lo + a.range);
+  const int k_lo = (a.window > 0 ? max(st - a.window + 1, 0) : 0) + split * a.range, k_hi = min(end, k_lo + a.range);
   const int64_t g0 = (int64_t)tok0 * a.H + row0;  // first row in q / out
   if (k_lo >= k_hi) {  // nothing in this range: the combine pass must not read what was never written
     if (a.splits > 1 && tid < rows_b && row0 + tid < nrow) {
@@ -94,9 +95,12 @@ __global__ void __launch_bounds__(NT) latent_decode_kernel(LatArgs a) {
       if (ch < CPR) *reinterpret_cast<bf16x8*>(Ks + krow * KP + ch * 8) = ch < pieces ? kr[i] : zero8;
     }
   };
-  int pos[MR];  // position of this lane's row in every row tile
+  int pos[MR], lo[MR];  // position of this lane's row in every row tile, and the first key it sees
 #pragma unroll
-  for (int m = 0; m < MR; ++m) pos[m] = st + min(row0 + 16 * m + l16, nrow - 1) / a.H;
+  for (int m = 0; m < MR; ++m) {
+    pos[m] = st + min(row0 + 16 * m + l16, nrow - 1) / a.H;
+    lo[m] = a.window > 0 ? pos[m] - a.window + 1 : 0;
+  }
   f32x4 o[MR][NV];
   float m_run[MR], l_run[MR];
 #pragma unroll
@@ -128,7 +132,7 @@ __global__ void __launch_bounds__(NT) latent_decode_kernel(LatArgs a) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int key = k0 + 16 * w + 4 * q4 + j;
-        sc[m][j] = key <= pos[m] && key < k_hi ? sc[m][j] * a.c : -INFINITY;
+        sc[m][j] = key <= pos[m] && key < k_hi && key >= lo[m] ? sc[m][j] * a.c : -INFINITY;
         mx = fmaxf(mx, sc[m][j]);
       }
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -142,20 +146,20 @@ __global__ void __launch_bounds__(NT) latent_decode_kernel(LatArgs a) {
 #pragma unroll
       for (int v = 0; v < 4; ++v) mx = fmaxf(mx, red[v * rows_b + 16 * m + l16]);
       const float use = mx == -INFINITY ? 0.f : mx;
-      const float alpha = exp2f(m_run[m] - use);
+      const float alpha = exp2f(m_run[m] - use);  // (nothing in sight yet: 0, of sums that are 0)
       m_run[m] = mx;
-      bf16x4 hi, lo;
+      bf16x4 hi, rest;
       float sum = 0.f;
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const float p = exp2f(sc[m][j] - use);
         sum += p;
         hi[j] = (bf16)p;
-        lo[j] = (bf16)(p - (float)hi[j]);
+        rest[j] = (bf16)(p - (float)hi[j]);
       }
       l_run[m] = l_run[m] * alpha + sum;
       *reinterpret_cast<bf16x4*>(Ps + (16 * m + l16) * PP + 16 * w + 4 * q4) = hi;
-      *reinterpret_cast<bf16x4*>(Ps + (rows_b + 16 * m + l16) * PP + 16 * w + 4 * q4) = lo;
+      *reinterpret_cast<bf16x4*>(Ps + (rows_b + 16 * m + l16) * PP + 16 * w + 4 * q4) = rest;
       if (!__all(alpha == 1.f)) {
 #pragma unroll
         for (int t = 0; t < NV; ++t) o[m][t] *= alpha;
@@ -307,7 +311,7 @@ extern "C" int ds_latent_decode_ok(int R, int r) {
   return R > 0 && R % 8 == 0 && r >= 0 && r % 8 == 0 && R <= 512 && (R + r) / 8 <= pieces_of(nv_of(R));
 }
 
-// Keys per range and number of ranges for `nseq` sequences of up to max_new tokens and max_len keys
+// Keys per range and number of ranges for `nseq` sequences of up to max_new tokens and max_len keys in sight of them
 extern "C" void ds_latent_decode_plan(int nseq, int max_new, int H, int W, int max_len, int* range, int* splits) {
   const int rows = max_new * H, per = 16 * row_tiles(rows, W), blocks = (rows + per - 1) / per;
   const int tiles = (max_len + BN - 1) / BN;
@@ -325,13 +329,13 @@ extern "C" void ds_latent_decode_plan(int nseq, int max_new, int H, int W, int m
 // batch's token tok_base. q [tokens, H, R + r], lat [blocks, BS, R + r] -> out [tokens, H, R]. acc / ml: workspace of `splits` ranges (unused with one).
 extern "C" int ds_latent_decode(const void* q, const void* lat, void* out, float* acc, float* ml, const int* bt, int max_blocks,
                                 const int* cu, const int* start, int first, int nseq, int max_new, int tok_base, int tokens, int H, int R,
-                                int r, int BS, int range, int splits, const float* sink, float scale, hipStream_t st) {
+                                int r, int BS, int range, int splits, int window, const float* sink, float scale, hipStream_t st) {
   if (nseq <= 0) return 0;
   if (!ds_latent_decode_ok(R, r) || H <= 0 || BS <= 0 || max_blocks <= 0 || range <= 0 || range % BN || splits <= 0 ||
-      splits > MAX_SPLITS || max_new <= 0 || tokens <= 0 || (splits > 1 && (!acc || !ml)))
+      splits > MAX_SPLITS || max_new <= 0 || tokens <= 0 || window < 0 || (splits > 1 && (!acc || !ml)))
     return (int)hipErrorInvalidValue;
   const LatArgs a{(const bf16*)q, (const bf16*)lat, (bf16*)out, acc, ml, bt, cu, start, sink, first, tok_base, H, R, r, BS,
-                  max_blocks, range, splits, (int64_t)tokens * H, scale * LOG2E};
+                  max_blocks, range, splits, window, (int64_t)tokens * H, scale * LOG2E};
   const int mr = row_tiles(max_new * H, R + r);
   const int blocks = (max_new * H + 16 * mr - 1) / (16 * mr);
   if (blocks > 65535) return (int)hipErrorInvalidValue;

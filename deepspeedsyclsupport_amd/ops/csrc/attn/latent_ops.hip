@@ -2,35 +2,41 @@
 //
 // A token is cached as one row [latent c (R) | rotated key part (r)] shared by all heads. Keys and values are linear maps of
 // c per head, so q . k = (W_uk^T q) . c: folding the map into the query leaves attention over the cached rows themselves.
-//  * prepare: the down projection's row [query latent (Q) | c (R) | key part (r)] -> normed query latent; c normed, the key
-//    part rotated to the token's position, both into the paged cache.
+//  * prepare: the down projection's row [query latent (Q, or none) | c (R) | key part (r)], which may be part of a wider one ->
+//    normed query latent; c normed, the key part rotated to the token's position, both into the paged cache.
 //  * head_linear: y[t, h] = W_h x[t, h] for every head, the maps of both directions; optionally the columns behind the map's
 //    (the rotated part of the query) are rotated and carried over.
 //  * rotate_tail: those columns in place, for queries that attend to expanded keys.
 //  * gather: the cached rows of whole contexts laid end to end, operands of the expansion product.
-// Angles are position * frequency in fp64, reduced to one turn, then fp32 sine and cosine.
+// Angles are position * frequency in fp64, reduced to one turn, then fp32 sine and cosine, times a factor.
 #include "ds_hip.h"
 
 namespace {
 
-__device__ __forceinline__ void turn_of(int pos, double freq, float& c, float& s) {
+struct Freq {
+  const double* f;
+  float mult;
+};
+__device__ __forceinline__ void turn_of(int pos, Freq freq, int i, float& c, float& s) {
   constexpr double TAU = 6.283185307179586476925286766559;
-  const double a = (double)pos * freq;
+  const double a = (double)pos * freq.f[i];
   sincosf((float)(a - TAU * rint(a / TAU)), &s, &c);
+  c *= freq.mult;
+  s *= freq.mult;
 }
 
 // One wave per (token, part): part 0 the query latent, part 1 the cached row. V elements per access.
 template <typename T, int V>
 __global__ void __launch_bounds__(256) latent_prepare_kernel(
-    const T* __restrict__ down, const float* __restrict__ qw, const float* __restrict__ kvw, float eps,
-    const double* __restrict__ freq, int half, const int* __restrict__ pos, const int* __restrict__ seq_ids,
+    const T* __restrict__ down, int64_t ld, const float* __restrict__ qw, const float* __restrict__ kvw, float eps,
+    Freq freq, int half, const int* __restrict__ pos, const int* __restrict__ seq_ids,
     const int* __restrict__ bt, int max_blocks, T* __restrict__ lat, T* __restrict__ cq, int tokens, int Q, int R, int r,
     int BS) {
   const int lane = threadIdx.x & 63;
   const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  const int t = (int)(item >> 1), part = (int)(item & 1);
+  const int t = (int)(Q ? item >> 1 : item), part = Q ? (int)(item & 1) : 1;
   if (t >= tokens) return;
-  const T* src = down + (int64_t)t * (Q + R + r) + (part ? Q : 0);
+  const T* src = down + t * ld + (part ? Q : 0);
   const int W = part ? R : Q;
   const float* w = part ? kvw : qw;
   const int p = pos[t];
@@ -60,7 +66,7 @@ __global__ void __launch_bounds__(256) latent_prepare_kernel(
   if (!part) return;
   for (int i = lane; i < half; i += 64) {
     float co, si;
-    turn_of(p, freq[i], co, si);
+    turn_of(p, freq, i, co, si);
     const float u = (float)src[R + i], v = (float)src[R + half + i];
     dst[R + i] = (T)(u * co - v * si);
     dst[R + half + i] = (T)(v * co + u * si);
@@ -70,10 +76,10 @@ __global__ void __launch_bounds__(256) latent_prepare_kernel(
 
 // Item j of the columns behind the map's: pair (j, half + j) turned, or a single column carried over
 template <typename T>
-__device__ __forceinline__ void rotate_one(const T* s, T* d, int j, int half, int p, const double* freq) {
+__device__ __forceinline__ void rotate_one(const T* s, T* d, int j, int half, int p, Freq freq) {
   if (j < half) {
     float co, si;
-    turn_of(p, freq[j], co, si);
+    turn_of(p, freq, j, co, si);
     const float u = (float)s[j], v = (float)s[half + j];
     d[j] = (T)(u * co - v * si);
     d[half + j] = (T)(v * co + u * si);
@@ -85,21 +91,20 @@ __device__ __forceinline__ void rotate_one(const T* s, T* d, int j, int half, in
 // ... of all heads of a token, by a workgroup
 template <typename T>
 __device__ __forceinline__ void rotate_heads(const T* src, int64_t sh, T* dst, int64_t dh, int H, int r, int half, int p,
-                                             const double* freq) {
+                                             Freq freq) {
   const int per = r - half;
   for (int i = threadIdx.x; i < H * per; i += blockDim.x)
     rotate_one(src + i / per * sh, dst + i / per * dh, i % per, half, p, freq);
 }
 
 template <typename T>
-__global__ void __launch_bounds__(256) rotate_tail_kernel(T* __restrict__ q, int64_t row, int d, int r, int H,
-                                                          const double* __restrict__ freq, int half,
-                                                          const int* __restrict__ pos) {
+__global__ void __launch_bounds__(256) rotate_tail_kernel(T* __restrict__ q, int64_t ld, int64_t row, int d, int r, int H,
+                                                          Freq freq, int half, const int* __restrict__ pos) {
   __shared__ float cs[2][256];
   const int t = blockIdx.x, p = pos[t];
-  T* x = q + (int64_t)t * H * row + d;
+  T* x = q + t * ld + d;
   if (half <= 256) {  // one sine and cosine per pair, shared by the heads
-    for (int i = threadIdx.x; i < half; i += 256) turn_of(p, freq[i], cs[0][i], cs[1][i]);
+    for (int i = threadIdx.x; i < half; i += 256) turn_of(p, freq, i, cs[0][i], cs[1][i]);
     __syncthreads();
     for (int i = threadIdx.x; i < H * half; i += 256) {
       const int h = i / half, j = i % half;
@@ -114,13 +119,14 @@ __global__ void __launch_bounds__(256) rotate_tail_kernel(T* __restrict__ q, int
 }
 
 struct HeadArgs {
-  const void* x;     // [T, H, xrow], K columns used
+  const void* x;     // [T, H, xrow], K columns used, ldx elements from token to token
   const void* w;     // [H, N, K]
   void* y;           // [T, H, yrow]
   int T, H, N, K, xrow, yrow;
   int r, half;       // columns K .. K + r of x go to N .. N + r of y, the first 2 half of them rotated
-  const double* freq;
+  Freq freq;
   const int* pos;
+  int64_t ldx;
 };
 
 // TT x 16 tokens, 64 output columns (16 per wave) of one head: W rows as the A operand, tokens as B
@@ -132,7 +138,7 @@ __global__ void __launch_bounds__(256) head_linear_mfma_kernel(HeadArgs a) {
     const int per = a.r - a.half, nt = min(16 * TT, a.T - t0);  // pairs and single columns of a token
     for (int i = threadIdx.x; i < nt * per; i += 256) {
       const int t = t0 + i / per;
-      rotate_one((const bf16*)a.x + ((int64_t)t * a.H + h) * a.xrow + a.K, (bf16*)a.y + ((int64_t)t * a.H + h) * a.yrow + a.N,
+      rotate_one((const bf16*)a.x + t * a.ldx + h * a.xrow + a.K, (bf16*)a.y + ((int64_t)t * a.H + h) * a.yrow + a.N,
                  i % per, a.half, a.pos[t], a.freq);
     }
     return;
@@ -143,7 +149,7 @@ __global__ void __launch_bounds__(256) head_linear_mfma_kernel(HeadArgs a) {
   const bf16* xr[TT];
 #pragma unroll
   for (int i = 0; i < TT; ++i)
-    xr[i] = (const bf16*)a.x + ((int64_t)min(t0 + 16 * i + l16, a.T - 1) * a.H + h) * a.xrow;
+    xr[i] = (const bf16*)a.x + min(t0 + 16 * i + l16, a.T - 1) * a.ldx + h * a.xrow;
   f32x4 acc[TT];
 #pragma unroll
   for (int i = 0; i < TT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -188,7 +194,7 @@ __global__ void __launch_bounds__(256) head_linear_mfma_kernel(HeadArgs a) {
 template <typename T>
 __global__ void __launch_bounds__(256) head_linear_any_kernel(HeadArgs a) {
   const int t = blockIdx.x, h = blockIdx.y;
-  const T* x = (const T*)a.x + ((int64_t)t * a.H + h) * a.xrow;
+  const T* x = (const T*)a.x + t * a.ldx + h * a.xrow;
   T* y = (T*)a.y + ((int64_t)t * a.H + h) * a.yrow;
   for (int n = threadIdx.x; n < a.N; n += 256) {
     const T* w = (const T*)a.w + ((int64_t)h * a.N + n) * a.K;
@@ -201,7 +207,8 @@ __global__ void __launch_bounds__(256) head_linear_any_kernel(HeadArgs a) {
 
 // one wave per context row of 16-byte pieces
 __global__ void __launch_bounds__(256) latent_gather_kernel(const bf16* __restrict__ lat, const int* __restrict__ bt,
-                                                            int max_blocks, const int* __restrict__ offs, int first,
+                                                            int max_blocks, const int* __restrict__ offs,
+                                                            const int* __restrict__ first_keys, int first,
                                                             int nseq, bf16* __restrict__ ctx, int64_t total, int pad,
                                                             int row, int BS) {
   const int64_t i = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -217,7 +224,7 @@ __global__ void __launch_bounds__(256) latent_gather_kernel(const bf16* __restri
   }
   int s = 0;
   while (s + 1 < nseq && i >= offs[s + 1]) ++s;
-  const int p = (int)(i - offs[s]);
+  const int p = (int)(i - offs[s]) + (first_keys ? first_keys[s] : 0);
   const bf16* src = lat + ((int64_t)bt[(int64_t)(first + s) * max_blocks + p / BS] * BS + p % BS) * row;
   for (int c = (threadIdx.x & 63) * 8; c < row; c += 512)
     *reinterpret_cast<bf16x8*>(ctx + i * row + c) = *reinterpret_cast<const bf16x8*>(src + c);
@@ -225,15 +232,18 @@ __global__ void __launch_bounds__(256) latent_gather_kernel(const bf16* __restri
 
 }  // namespace
 
-extern "C" int ds_latent_prepare(const void* down, const float* qw, const float* kvw, float eps, const double* freq, int half,
+// down: rows ld elements apart; Q 0: no query latent (qw, cq unused); cosine and sine times mult
+extern "C" int ds_latent_prepare(const void* down, int64_t ld, const float* qw, const float* kvw, float eps, const double* freq,
+                                 float mult, int half,
                                  const int* pos, const int* seq_ids, const int* bt, int max_blocks, void* lat, void* cq,
                                  int tokens, int Q, int R, int r, int BS, int dtype, hipStream_t st) {
   if (tokens <= 0) return 0;
-  if (Q <= 0 || R <= 0 || r < 0 || half < 0 || 2 * half > r || BS <= 0 || max_blocks <= 0) return (int)hipErrorInvalidValue;
-  const bool vec = Q % 8 == 0 && R % 8 == 0 && r % 8 == 0;
+  if (Q < 0 || (Q && (!qw || !cq)) || ld < (int64_t)Q + R + r || R <= 0 || r < 0 || half < 0 || 2 * half > r || BS <= 0 || max_blocks <= 0) return (int)hipErrorInvalidValue;
+  const bool vec = Q % 8 == 0 && R % 8 == 0 && r % 8 == 0 && ld % 8 == 0 && ((uintptr_t)down & 15) == 0;
+  const int64_t items = (int64_t)tokens * (Q ? 2 : 1);
 #define GO(T, V)                                                                                                      \
-  hipLaunchKernelGGL((latent_prepare_kernel<T, V>), dim3((tokens + 1) / 2), dim3(256), 0, st, (const T*)down, qw, kvw, eps, \
-                     freq, half, pos, seq_ids, bt, max_blocks, (T*)lat, (T*)cq, tokens, Q, R, r, BS)
+  hipLaunchKernelGGL((latent_prepare_kernel<T, V>), dim3((unsigned)((items + 3) / 4)), dim3(256), 0, st, (const T*)down, ld, qw, kvw, \
+                     eps, Freq{freq, mult}, half, pos, seq_ids, bt, max_blocks, (T*)lat, (T*)cq, tokens, Q, R, r, BS)
   if (dtype == DS_F32 && vec) GO(float, 8);
   else if (dtype == DS_F32) GO(float, 1);
   else if (dtype == DS_BF16 && vec) GO(bf16, 8);
@@ -244,29 +254,31 @@ extern "C" int ds_latent_prepare(const void* down, const float* qw, const float*
   return 0;
 }
 
-extern "C" int ds_rotate_tail(void* q, int tokens, int H, int row, int r, const double* freq, int half, const int* pos,
-                              int dtype, hipStream_t st) {
+// ld: elements from token to token
+extern "C" int ds_rotate_tail(void* q, int64_t ld, int tokens, int H, int row, int r, const double* freq, float mult, int half,
+                              const int* pos, int dtype, hipStream_t st) {
   if (tokens <= 0 || half <= 0) return 0;
-  if (H <= 0 || r > row || 2 * half > r) return (int)hipErrorInvalidValue;
+  if (H <= 0 || r > row || 2 * half > r || ld < (int64_t)H * row) return (int)hipErrorInvalidValue;
   if (dtype == DS_F32)
-    hipLaunchKernelGGL((rotate_tail_kernel<float>), dim3(tokens), dim3(256), 0, st, (float*)q, (int64_t)row, row - r, r, H,
-                       freq, half, pos);
+    hipLaunchKernelGGL((rotate_tail_kernel<float>), dim3(tokens), dim3(256), 0, st, (float*)q, ld, (int64_t)row, row - r, r,
+                       H, Freq{freq, mult}, half, pos);
   else if (dtype == DS_BF16)
-    hipLaunchKernelGGL((rotate_tail_kernel<bf16>), dim3(tokens), dim3(256), 0, st, (bf16*)q, (int64_t)row, row - r, r, H, freq,
-                       half, pos);
+    hipLaunchKernelGGL((rotate_tail_kernel<bf16>), dim3(tokens), dim3(256), 0, st, (bf16*)q, ld, (int64_t)row, row - r, r,
+                       H, Freq{freq, mult}, half, pos);
   else return (int)hipErrorInvalidValue;
   DS_CHECK_LAUNCH();
   return 0;
 }
 
-// x [T, H, xrow], w [H, N, K], y [T, H, yrow]; r > 0: columns K .. K + r of x, rotated, behind the N of y
+// x [T, H, xrow] (ldx elements from token to token), w [H, N, K], y [T, H, yrow]; r > 0: columns K .. K + r of x, rotated, behind the N of y
 extern "C" int ds_head_linear(const void* x, const void* w, void* y, int T, int H, int N, int K, int xrow, int yrow, int r,
-                              int half, const double* freq, const int* pos, int dtype, hipStream_t st) {
+                              int64_t ldx, int half, const double* freq, float mult, const int* pos, int dtype, hipStream_t st) {
   if (T <= 0) return 0;
-  if (H <= 0 || H > 65535 || N <= 0 || K <= 0 || xrow < K + r || yrow < N + r || 2 * half > r || (r && (!freq || !pos)))
+  if (H <= 0 || H > 65535 || N <= 0 || K <= 0 || xrow < K + r || yrow < N + r || 2 * half > r || (r && (!freq || !pos)) ||
+      ldx < (int64_t)H * xrow)
     return (int)hipErrorInvalidValue;
-  const HeadArgs a{x, w, y, T, H, N, K, xrow, yrow, r, half, freq, pos};
-  if (dtype == DS_BF16 && K % 8 == 0 && xrow % 8 == 0 && (T + 15) / 16 <= 65535) {
+  const HeadArgs a{x, w, y, T, H, N, K, xrow, yrow, r, half, Freq{freq, mult}, pos, ldx};
+  if (dtype == DS_BF16 && K % 8 == 0 && xrow % 8 == 0 && ldx % 8 == 0 && (((uintptr_t)x | (uintptr_t)w) & 15) == 0 && (T + 15) / 16 <= 65535) {
     const int tiles = (N + 63) / 64 + (r ? 1 : 0);
     if (T <= 16) hipLaunchKernelGGL((head_linear_mfma_kernel<1>), dim3(tiles, H, 1), dim3(256), 0, st, a);
     else if (T <= 64) hipLaunchKernelGGL((head_linear_mfma_kernel<2>), dim3(tiles, H, (T + 31) / 32), dim3(256), 0, st, a);
@@ -282,14 +294,14 @@ extern "C" int ds_head_linear(const void* x, const void* w, void* y, int T, int 
   return 0;
 }
 
-// contexts of sequences first .. first + nseq, offs [nseq + 1] their places in ctx [total + pad, row] (bf16), whose
-// last `pad` rows become zero
-extern "C" int ds_latent_gather(const void* lat, const int* bt, int max_blocks, const int* offs, int first, int nseq, void* ctx,
+// contexts of sequences first .. first + nseq from their first keys on (null: 0), offs [nseq + 1] their places in ctx
+// [total + pad, row] (bf16), whose last `pad` rows become zero
+extern "C" int ds_latent_gather(const void* lat, const int* bt, int max_blocks, const int* offs, const int* first_keys, int first, int nseq, void* ctx,
                                 int64_t total, int pad, int row, int BS, hipStream_t st) {
   if (total <= 0) return 0;
   if (row <= 0 || row % 8 || BS <= 0 || max_blocks <= 0 || nseq <= 0) return (int)hipErrorInvalidValue;
   hipLaunchKernelGGL(latent_gather_kernel, dim3((unsigned)((total + pad + 3) / 4)), dim3(256), 0, st, (const bf16*)lat, bt,
-                     max_blocks, offs, first, nseq, (bf16*)ctx, total, pad, row, BS);
+                     max_blocks, offs, first_keys, first, nseq, (bf16*)ctx, total, pad, row, BS);
   DS_CHECK_LAUNCH();
   return 0;
 }

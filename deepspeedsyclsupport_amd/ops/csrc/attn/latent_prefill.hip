@@ -2,16 +2,18 @@
 // (gfx950): entry point. The kernel is paged_prefill_core.h's.
 #include "paged_prefill_core.h"
 
-// q / o [T, H, dn + r] / [T, H, dv] bf16, rotated; kv [rows, H (dn + dv)]: expanded context rows, keys of all heads, then
+// q / o [T, H, dn + r] (ldq elements from token to token) / [T, H, dv] bf16, rotated; kv [rows, H (dn + dv)]: expanded context rows, keys of all heads, then
 // values; ctx [rows, ldr]: the latents' rows, whose columns rot0 .. rot0 + r are the rotated key part. kv_offs: place of the
-// contexts of sequences first, first + 1, ...; work [nwork, 2] (sequence, 128-row query block). Tiles of 64 keys are
+// contexts of sequences first, first + 1, ..., kv_first: their first keys (multiples of 64, none behind what the window lets the
+// first new token see; null: 0); work [nwork, 2] (sequence, 128-row query block). Tiles of 64 keys are
 // read whole: 64 (finite) rows must exist behind the last context in kv and ctx.
 extern "C" int ds_latent_prefill(const void* q, const void* kv, const void* ctx, void* o, const int* start, const int* cu_q,
-                                 const int* work, int nwork, const int* kv_offs, int first, int H, int dn, int r, int dv,
+                                 const int* work, int nwork, const int* kv_offs, const int* kv_first, int first, int64_t ldq,
+                                 int window, int H, int dn, int r, int dv,
                                  int ldr, int rot0, const float* sink, float scale, hipStream_t st) {
   if (nwork <= 0) return 0;
   const int dk = dn + r;
-  if (H <= 0 || scale <= 0.f || dn <= 0 || r < 0 || dv <= 0 || dn % 8 || r % 8 || dv % 8 || ldr % 8 || rot0 % 8 ||
+  if (ldq % 8 || ((uintptr_t)q & 15) || ldq < (int64_t)H * dk || window < 0 || H <= 0 || scale <= 0.f || dn <= 0 || r < 0 || dv <= 0 || dn % 8 || r % 8 || dv % 8 || ldr % 8 || rot0 % 8 ||
       (int64_t)nwork * H > INT32_MAX)
     return (int)hipErrorInvalidValue;
   PagedArgs a{};
@@ -29,7 +31,10 @@ extern "C" int ds_latent_prefill(const void* q, const void* kv, const void* ctx,
   a.dv = dv;
   a.sink = sink;
   a.kv_offs = kv_offs;
+  a.kv_first = kv_first;
   a.first = first;
+  a.ldq = ldq;
+  a.window = window;
   a.dn = dn;
   a.ldk = H * (dn + dv);
   a.ldr = ldr;

@@ -4,7 +4,8 @@
 // One wave per (token, query head): 64 keys at a time, a lane per key for the scores, then a lane per value column
 // for the weighted sum. Scores, softmax and sums are fp32. A key j is visible to position i if lo(i) <= j <= i, where
 // lo is i - window + 1 (sliding window), the start of i's chunk (chunked attention), or 0. Optional tanh soft cap;
-// optional sink: exp(sink of the head) joins the softmax's denominator. Value rows may lie further apart than their
+// optional sink: exp(sink of the head) joins the softmax's denominator; optional gate: the head's output times the sigmoid of a
+// number per token and head. Value rows may lie further apart than their
 // width: latent attention's values are the first columns of its keys.
 #include "ds_hip.h"
 
@@ -17,7 +18,7 @@ __global__ void __launch_bounds__(64) paged_generic_kernel(
     const T* __restrict__ q, const T* __restrict__ kc, const T* __restrict__ vc, T* __restrict__ o,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ pos, const int* __restrict__ seq_ids,
     int H, int G, int dk, int dv, int vrow, int BS, float scale, float softcap, int window, int chunk,
-    const float* __restrict__ sink, int64_t ldo) {
+    const float* __restrict__ sink, int64_t ldo, const T* __restrict__ gate, int64_t ldg) {
   __shared__ float qs[MAXD];
   __shared__ float ps[64];
   __shared__ int64_t slot_s[64];
@@ -67,6 +68,7 @@ __global__ void __launch_bounds__(64) paged_generic_kernel(
 #pragma unroll
     for (int i = 0; i < MAXD / 64; ++i) acc[i] *= alpha;
   }
+  if (gate) l *= 1.f + expf(-(float)gate[t * ldg + h]);
   T* orow = o + t * ldo + h * dv;
 #pragma unroll
   for (int i = 0; i < MAXD / 64; ++i) {
@@ -80,7 +82,7 @@ __global__ void __launch_bounds__(64) paged_generic_kernel(
 extern "C" int ds_paged_generic(const void* q, const void* kc, const void* vc, void* o, const int* bt, int max_blocks,
                                 const int* pos, const int* seq_ids, int tokens, int H, int G, int dk, int dv, int vrow,
                                 int BS, float scale, float softcap, int window, int chunk, const float* sink, int64_t ldo,
-                                int dtype, hipStream_t st) {
+                                const void* gate, int64_t ldg, int dtype, hipStream_t st) {
   if (tokens <= 0) return 0;
   if (G <= 0 || H % G || dk <= 0 || dv <= 0 || vrow < dv || dk > MAXD || dv > MAXD || BS <= 0 || H > 65535 ||
       ldo < (int64_t)H * dv)
@@ -88,7 +90,7 @@ extern "C" int ds_paged_generic(const void* q, const void* kc, const void* vc, v
 #define GO(T)                                                                                                        \
   hipLaunchKernelGGL((paged_generic_kernel<T>), dim3(tokens, H), dim3(64), 0, st, (const T*)q, (const T*)kc,         \
                      (const T*)vc, (T*)o, bt, max_blocks, pos, seq_ids, H, G, dk, dv, vrow, BS, scale, softcap, window, chunk, \
-                     sink, ldo)
+                     sink, ldo, (const T*)gate, ldg)
   if (dtype == DS_F32) GO(float);
   else if (dtype == DS_BF16) GO(bf16);
   else return (int)hipErrorInvalidValue;

@@ -12,7 +12,8 @@ extern "C" int ds_paged_prefill(const void* q, const void* kc, const void* vc, v
   if (nwork <= 0) return 0;
   if (Hk <= 0 || Hq % Hk || BS <= 0 || max_blocks <= 0 || scale <= 0.f) return (int)hipErrorInvalidValue;
   PagedArgs a{(const bf16*)q, (const bf16*)kc, (const bf16*)vc, (bf16*)o, block_table, start, cu_q, work, alibi,
-              Hq, Hk, BS, max_blocks, window, scale * 1.4426950408889634f, 1.f / scale, D, D, 0, nullptr, nullptr, 0, 0, 0, 0, 0, (int64_t)Hq * D, 0.f, 0.f};
+              Hq, Hk, BS, max_blocks, window, scale * 1.4426950408889634f, 1.f / scale, D, D, 0, nullptr, nullptr, 0, 0, 0, 0, 0, nullptr, (int64_t)Hq * D,
+              (int64_t)Hq * D, nullptr, 0, 0.f, 0.f};
   switch (D) {
     case 64: return launch<64, 64, PLAIN>(a, nwork, st);
     case 80: return launch<80, 80, PLAIN>(a, nwork, st);
@@ -25,11 +26,11 @@ extern "C" int ds_paged_prefill(const void* q, const void* kc, const void* vc, v
 
 // Key width dk and value width dv (multiples of 8 up to 256) of their own, chunked and / or windowed visibility,
 // optional score cap: score = softcap * tanh(scale * q.k / softcap). sink [Hq] or null: exp(sink) joins the softmax's
-// denominator. ldo: elements between the rows of o.
+// denominator. gate [T, Hq] or null: heads come out times its sigmoid. ldo, ldg: elements between the rows of o and gate.
 extern "C" int ds_paged_prefill_ext(const void* q, const void* kc, const void* vc, void* o, const int* block_table,
                                     const int* start, const int* cu_q, const int* work, int nwork, int Hq, int Hk, int dk,
                                     int dv, int BS, int max_blocks, int window, int chunk, float scale, float softcap,
-                                    const float* sink, int64_t ldo, hipStream_t st) {
+                                    const float* sink, const void* gate, int64_t ldg, int64_t ldo, hipStream_t st) {
   if (nwork <= 0) return 0;
   if (Hk <= 0 || Hq % Hk || BS <= 0 || max_blocks <= 0 || scale <= 0.f || dk % 8 || dv % 8 || dk <= 0 || dv <= 0 ||
       ldo < (int64_t)Hq * dv)
@@ -39,7 +40,7 @@ extern "C" int ds_paged_prefill_ext(const void* q, const void* kc, const void* v
   // with a cap the scores leave the capping step in log2 units already
   PagedArgs a{(const bf16*)q, (const bf16*)kc, (const bf16*)vc, (bf16*)o, block_table, start, cu_q, work, nullptr,
               Hq, Hk, BS, max_blocks, window, cap ? 1.f : scale * LOG2E, 1.f / scale, dk, dv, chunk,
-              sink, nullptr, 0, 0, 0, 0, 0, ldo,
+              sink, nullptr, 0, 0, 0, 0, 0, nullptr, ldo, (int64_t)Hq * dk, (const bf16*)gate, ldg,
               cap ? scale / softcap * 2.f * LOG2E : 0.f, cap ? softcap * LOG2E : 0.f};
 #define DS_ROW(K)                                              \
   {                                                            \

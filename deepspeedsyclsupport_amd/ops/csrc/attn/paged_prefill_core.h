@@ -23,7 +23,8 @@
 //  * a third (LATENT) reads keys and values that were expanded from cached latents: rows laid end to end, a sequence's from
 //    kv_offs on, [keys of all heads | values of all heads] per row, with the last key columns (one rotated part for all
 //    heads) in the latent's own row. Its workgroups go head by head, so an XCD's L2 serves one head's keys;
-//  * EXT and LATENT take a softmax sink per head: exp(sink) joins the denominator;
+//  * EXT and LATENT take a softmax sink per head: exp(sink) joins the denominator; EXT a gate per token and head: the output
+//    times its sigmoid;
 //  * the head dim is a template parameter: D / 16 MFMA steps for the scores, ceil(D / 32) output column tiles (D = 80
 //    computes a third, half-used tile over zero-filled LDS columns), LDS rows pitched to 16 (D <= 128) or 32 (D = 256)
 //    16-byte chunks so one swizzle serves every size.
@@ -63,7 +64,7 @@ __device__ __forceinline__ int lds_off(int row, int ch) {
 }
 
 struct PagedArgs {
-  const bf16* q;          // [T, Hq, D]
+  const bf16* q;          // [T, Hq, D], ldq elements from row to row
   const bf16* kc;         // [blocks, Hk, BS, D]
   const bf16* vc;
   bf16* o;                // [T, Hq, D], ldo elements from row to row
@@ -80,7 +81,10 @@ struct PagedArgs {
   const int* kv_offs;     // LATENT: first context row of sequence `first`, and of the ones after it
   int first, dn, ldk, ldr, rot0;  // key columns of a head (the rest is rotated), row lengths of kc and of vc, first rotated
                           // column there; kc: the expanded rows, vc: the latents' rows
-  int64_t ldo;            // elements from a token's row of o to the next one's
+  const int* kv_first;    // LATENT: first key of those contexts (whole tiles into the sequence), or null: 0
+  int64_t ldo, ldq;       // elements from a token's row of o / q to the next one's
+  const bf16* gate;       // EXT: [T, Hq], ldg elements from row to row, or null
+  int64_t ldg;
   float cap_in, cap_out;  // EXT: capped score in log2 units = cap_out * tanh(score * cap_in); cap_out 0: no cap
 };
 
@@ -101,13 +105,14 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
   const int t0 = a.cu_q[seq], n = a.cu_q[seq + 1] - t0, start = a.start[seq], Skv = start + n;
   const int q0 = qb * BM, q0w = q0 + wid * 32;
   const int* bt = LAT ? nullptr : a.block_table + (int64_t)seq * a.max_blocks;
-  const int64_t ctx0 = LAT ? a.kv_offs[seq - a.first] : 0;
+  // (LATENT: the row of key 0, were it there)
+  const int64_t ctx0 = LAT ? a.kv_offs[seq - a.first] - (a.kv_first ? a.kv_first[seq - a.first] : 0) : 0;
   const float slope = a.alibi ? a.alibi[hq] * a.inv_scale : 0.f;
 
   bf16x8_t qf[KC];
   {
     const int qr = min(q0w + l32, n - 1);
-    const bf16* qrow = a.q + ((int64_t)(t0 + qr) * a.Hq + hq) * dk + 8 * h;
+    const bf16* qrow = a.q + (int64_t)(t0 + qr) * a.ldq + hq * dk + 8 * h;
 #pragma unroll
     for (int kk = 0; kk < KC; ++kk) {
       if (!EXT || 16 * kk + 8 * h < dk) {
@@ -124,8 +129,7 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
   int kt1 = min((Skv + BN - 1) / BN, pos_hi / BN + 1);
   // first key a position sees (non-decreasing in the position)
   auto first_key = [&](int p) {
-    if (LAT) return 0;
-    int lo = EXT && a.chunk > 0 ? p / a.chunk * a.chunk : 0;
+    int lo = MODE == EXT_ && a.chunk > 0 ? p / a.chunk * a.chunk : 0;
     if (a.window > 0) lo = max(lo, p - a.window + 1);
     return lo;
   };
@@ -249,7 +253,7 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
         }
       }
       // ALiBi bias, causal diagonal, window, key tail (lane = one query row, r = 32 keys of the 64)
-      const bool need_mask = k0 + BN - 1 > wpos_lo || (!LAT && (k0 + BN > Skv || k0 < lo_whi));
+      const bool need_mask = k0 + BN - 1 > wpos_lo || k0 < lo_whi || (!LAT && k0 + BN > Skv);
       if constexpr (MODE == EXT_) {
         if (a.cap_out > 0.f) {
 #pragma unroll
@@ -266,7 +270,7 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
           for (int r = 0; r < 16; ++r) {
             const int key = k0 + t * 32 + (r & 3) + 8 * (r >> 2) + 4 * h;
             float v = LAT ? s[t][r] : fmaf(slope, (float)(key - pos_lane), s[t][r]);
-            if (LAT ? key > pos_lane : key >= Skv || key > pos_lane || key < lo_lane) v = -INFINITY;
+            if ((!LAT && key >= Skv) || key > pos_lane || key < lo_lane) v = -INFINITY;
             s[t][r] = v;
           }
       }
@@ -383,6 +387,9 @@ __global__ void __launch_bounds__(NTHR, (Cfg<DK, DV>::OCC)) paged_prefill_kernel
       const float mn = fmaxf(m, sk), f = __builtin_amdgcn_exp2f(m - mn);
       inv = f / fmaf(l_tot, f, __builtin_amdgcn_exp2f(sk - mn));
     }
+  }
+  if constexpr (MODE == EXT_) {
+    if (a.gate) inv /= 1.f + __expf(-(float)a.gate[(int64_t)(t0 + min(q0w + l32, n - 1)) * a.ldg + hq]);
   }
   if (lane < 32) scratch[lane] = inv;
   __builtin_amdgcn_wave_barrier();

@@ -1,7 +1,7 @@
 // QKV epilogue of attention layers that norm the query and key projections as a whole and rotate part of every head, CDNA4
 // (gfx950); and the angle tables that such layers share.
 //
-//  * rope_table: cos and sin of position * frequency for every token of the batch. The angle is taken in fp64 and reduced to
+//  * rope_table: cos and sin of position * frequency, times a factor, for every token of the batch. The angle is taken in fp64 and reduced to
 //    one turn before the fp32 functions, so far positions lose nothing. One table serves all heads of all layers with these
 //    frequencies.
 //  * qk_rope_append: one workgroup per token. A projection row [q | k | v] (it may be part of a wider one) gets its biases;
@@ -13,13 +13,13 @@
 namespace {
 
 __global__ void __launch_bounds__(256) rope_table_kernel(const int* __restrict__ pos, const double* __restrict__ freq,
-                                                         f32x2* __restrict__ cs, int64_t items, int half) {
+                                                         f32x2* __restrict__ cs, int64_t items, int half, float mult) {
   constexpr double TAU = 6.283185307179586476925286766559;
   for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < items; i += (int64_t)gridDim.x * 256) {
     const double a = (double)pos[i / half] * freq[i % half];
     float c, s;
     sincosf((float)(a - TAU * rint(a / TAU)), &s, &c);
-    cs[i] = f32x2{c, s};
+    cs[i] = f32x2{c * mult, s * mult};
   }
 }
 
@@ -131,11 +131,12 @@ int launch(const void* qkv, int64_t ld, const float* bias, const float* qw, cons
 
 }  // namespace
 
-// cs [tokens, half, 2]: cos, sin of pos * freq
-extern "C" int ds_rope_table(const int* pos, const double* freq, float* cs, int tokens, int half, hipStream_t st) {
+// cs [tokens, half, 2]: cos, sin of pos * freq, times mult
+extern "C" int ds_rope_table(const int* pos, const double* freq, float* cs, int tokens, int half, float mult, hipStream_t st) {
   if (tokens <= 0 || half <= 0) return 0;
   const int64_t items = (int64_t)tokens * half;
-  hipLaunchKernelGGL(rope_table_kernel, dim3(ds_grid_for(items, 256)), dim3(256), 0, st, pos, freq, (f32x2*)cs, items, half);
+  hipLaunchKernelGGL(rope_table_kernel, dim3(ds_grid_for(items, 256)), dim3(256), 0, st, pos, freq, (f32x2*)cs, items, half,
+                     mult);
   DS_CHECK_LAUNCH();
   return 0;
 }

@@ -1,6 +1,6 @@
 // Products of mixture-of-experts layers, CDNA4 (gfx950). A pair (token, choice) is entry t * K + k: inputs are read from row
 // entry / div, results written to row `entry`, so nothing is copied into expert order and back. The gated form computes
-// silu(gate) up of the same columns in one go.
+// silu(gate) up of the same columns in one go; a plain product may end in a squared relu.
 //
 //  * stream: few rows per expert. bf16 weights are streamed once per tile of up to 64 entries. A workgroup owns 32 weight rows
 //    of an expert (gated: 16 of the gate and the same 16 of the up part); its four waves take alternating 64-wide steps of the
@@ -27,6 +27,12 @@ __device__ __forceinline__ f32x4 mfma(bf16x8 a, bf16x8 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
 }
 __device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.f + expf(-g)) * u; }
+enum : int { NONE = 0, SILU_GLU = 1, RELU2 = 2 };  // activation codes
+__device__ __forceinline__ float plain_act(float x, int act) {
+  if (act != RELU2) return x;
+  x = fmaxf(x, 0.f);
+  return x * x;
+}
 
 struct ExpertArgs {
   const void* x;         // [.., K]
@@ -35,7 +41,7 @@ struct ExpertArgs {
   const int* experts;    // [entries]
   const int* offs;       // [E + 1] and
   const int* order;      // [entries], or null (up to FEW entries)
-  int entries, E, N, K, div;
+  int entries, E, N, K, div, act;
 };
 
 // Operand order of a weight matrix [rows, K] (ops/bf16_gemv.py): 16 x 64 tiles of 1024 elements, tile by tile along K;
@@ -160,6 +166,9 @@ __device__ __forceinline__ void stream_tile(const ExpertArgs& a, const bf16* con
       const f32x4 u = total(MT + j);
 #pragma unroll
       for (int i = 0; i < 4; ++i) v[i] = silu_mul(v[i], u[i]);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = plain_act(v[i], a.act);
     }
     if (r >= cnt) continue;
     bf16* yr = (bf16*)a.y + (int64_t)ents[r] * N + n;
@@ -349,7 +358,7 @@ __global__ void __launch_bounds__(256, 2) expert_tile_kernel(ExpertArgs a) {
         bf16x4 o;
 #pragma unroll
         for (int i = 0; i < 4; ++i)
-          o[i] = (bf16)(GLU ? silu_mul(acc[0][m][4 * q + i], acc[1][m][4 * q + i]) : acc[t][m][4 * q + i]);
+          o[i] = (bf16)(GLU ? silu_mul(acc[0][m][4 * q + i], acc[1][m][4 * q + i]) : plain_act(acc[t][m][4 * q + i], a.act));
         *reinterpret_cast<bf16x4*>(yr + n + 8 * q + 4 * hh) = o;
       }
     }
@@ -372,19 +381,21 @@ __global__ void __launch_bounds__(256) expert_any_kernel(ExpertArgs a) {
     }
     s = wave_sum(s);
     if constexpr (GLU) s = silu_mul(s, wave_sum(u));
+    else s = plain_act(s, a.act);
     if (lane == 0) ((T*)a.y)[i * a.N + n] = (T)s;
   }
 }
 
-// out[t] = sum_k w[t, k] y[row(t, k)]
+// out[t] = sum_k w[t, k] y[row(t, k)] (+ base[t])
 template <typename T>
 __global__ void __launch_bounds__(256) expert_sum_kernel(const T* __restrict__ y, const float* __restrict__ w,
-                                                         const int* __restrict__ rows, T* __restrict__ out, int W, int K) {
+                                                         const int* __restrict__ rows, const T* __restrict__ base,
+                                                         T* __restrict__ out, int W, int K) {
   const int64_t t = blockIdx.x;
   for (int c = threadIdx.x; c < W; c += 256) {
     float v = 0.f;
     for (int k = 0; k < K; ++k) v = fmaf(w[t * K + k], (float)y[(rows ? rows[t * K + k] : t * K + k) * W + c], v);
-    out[t * W + c] = (T)v;
+    out[t * W + c] = (T)(base ? v + (float)base[t * W + c] : v);
   }
 }
 
@@ -393,18 +404,18 @@ __global__ void __launch_bounds__(256) expert_sum_kernel(const T* __restrict__ y
 extern "C" int ds_expert_few() { return FEW; }
 extern "C" int ds_expert_order_ok(int N, int K) { return N % 32 == 0 && K % 64 == 0; }
 
-// y[i] = w[experts[i]] x[i / div] for every entry; gated: silu of the first N rows times the others. offs and order from
+// y[i] = w[experts[i]] x[i / div] for every entry; act SILU_GLU: silu of the first N rows times the others; RELU2: max(., 0)^2. offs and order from
 // ds_expert_place, or null for up to ds_expert_few() entries. operand: the weights are in operand order (N % 32, K % 64 must
 // be 0); then with lists and `tile` the many-rows kernel runs.
 extern "C" int ds_expert_gemm(const void* x, const void* w, void* y, const int* experts, const int* offs, const int* order,
-                              int entries, int E, int N, int K, int div, int gated, int operand, int tile, int dtype,
+                              int entries, int E, int N, int K, int div, int act, int operand, int tile, int dtype,
                               hipStream_t st) {
   if (entries <= 0) return 0;
   if (E <= 0 || E > MAXE || N <= 0 || K <= 0 || div <= 0 || (!offs != !order) || (N + 63) / 64 > 65535)
     return (int)hipErrorInvalidValue;
-  const bool lists = offs != nullptr;
+  const bool lists = offs != nullptr, gated = act == SILU_GLU;
   if (operand && (dtype != DS_BF16 || !ds_expert_order_ok(N, K) || (!lists && entries > FEW))) return (int)hipErrorInvalidValue;
-  const ExpertArgs a{x, w, y, experts, offs, order, entries, E, N, K, div};
+  const ExpertArgs a{x, w, y, experts, offs, order, entries, E, N, K, div, act};
   if (operand && lists && tile) {
     const int per = gated ? BN / 2 : BN;
     const int64_t grid = ((int64_t)entries / BM + E) * ((N + per - 1) / per);
@@ -441,14 +452,16 @@ extern "C" int ds_expert_gemm(const void* x, const void* w, void* y, const int* 
   return 0;
 }
 
-extern "C" int ds_expert_sum(const void* y, const float* w, const int* rows, void* out, int T, int W, int K, int dtype,
+extern "C" int ds_expert_sum(const void* y, const float* w, const int* rows, const void* base, void* out, int T, int W, int K, int dtype,
                              hipStream_t st) {
   if (T <= 0) return 0;
   if (W <= 0 || K <= 0) return (int)hipErrorInvalidValue;
   if (dtype == DS_F32)
-    hipLaunchKernelGGL(expert_sum_kernel<float>, dim3(T), dim3(256), 0, st, (const float*)y, w, rows, (float*)out, W, K);
+    hipLaunchKernelGGL(expert_sum_kernel<float>, dim3(T), dim3(256), 0, st, (const float*)y, w, rows,
+                       (const float*)base, (float*)out, W, K);
   else if (dtype == DS_BF16)
-    hipLaunchKernelGGL(expert_sum_kernel<bf16>, dim3(T), dim3(256), 0, st, (const bf16*)y, w, rows, (bf16*)out, W, K);
+    hipLaunchKernelGGL(expert_sum_kernel<bf16>, dim3(T), dim3(256), 0, st, (const bf16*)y, w, rows,
+                       (const bf16*)base, (bf16*)out, W, K);
   else return (int)hipErrorInvalidValue;
   DS_CHECK_LAUNCH();
   return 0;

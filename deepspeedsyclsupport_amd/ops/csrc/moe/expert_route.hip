@@ -1,8 +1,9 @@
 // Routing of mixture-of-experts layers with grouped experts, CDNA4 (gfx950).
 //
-//  * route: router logits in fp32 (bf16 operands through the matrix cores, or plain fp32 products), softmax over all experts,
-//    the best groups of neighbouring experts (a group is as good as its best member), the best experts within those, weights
-//    divided by their sum. One launch: the logits of a tile of tokens never leave LDS. Ties go to the lower index.
+//  * route: router logits in fp32 (bf16 operands through the matrix cores, or plain fp32 products), scores (the softmax over all
+//    experts, or every expert's sigmoid), the best groups of neighbouring experts (a group is as good as its best member, or its
+//    two best together), the best experts within those, weights divided by their sum, times a constant. One launch: the logits
+//    of a tile of tokens never leave LDS. Ties go to the lower index.
 //  * place: the (token, choice) pairs sorted by expert, as lists for the expert products (expert_gemm.hip). The counts come
 //    from the routing kernel; nothing waits for the host.
 #include "ds_hip.h"
@@ -21,7 +22,8 @@ __device__ __forceinline__ f32x4 mfma(bf16x8 a, bf16x8 b, f32x4 c) {
 }
 
 struct RouteArgs {
-  int T, W, E, K, groups, keep;
+  int T, W, E, K, groups, keep, sigmoid, best;   // best: members that count for a group, 1 or 2
+  float scale;
   int* experts;      // [T, K]
   float* weights;    // [T, K]
   int* counts;       // [E], zero before; null: no lists wanted
@@ -37,24 +39,32 @@ __device__ __forceinline__ void choose(float* z, float* gs, int tok, const Route
     s[i] = lane + 64 * i < E ? z[lane + 64 * i] : -INFINITY;
     mx = fmaxf(mx, s[i]);
   }
-  mx = wave_max(mx);
+  if (a.sigmoid) {
 #pragma unroll
-  for (int i = 0; i < MAXE / 64; ++i) {
-    s[i] = lane + 64 * i < E ? expf(s[i] - mx) : 0.f;
-    den += s[i];
+    for (int i = 0; i < MAXE / 64; ++i) s[i] = 1.f / (1.f + expf(-s[i]));
+  } else {
+    mx = wave_max(mx);
+#pragma unroll
+    for (int i = 0; i < MAXE / 64; ++i) {
+      s[i] = lane + 64 * i < E ? expf(s[i] - mx) : 0.f;
+      den += s[i];
+    }
+    den = wave_sum(den);
+#pragma unroll
+    for (int i = 0; i < MAXE / 64; ++i) s[i] /= den;
   }
-  den = wave_sum(den);
 #pragma unroll
-  for (int i = 0; i < MAXE / 64; ++i) {
-    s[i] /= den;
+  for (int i = 0; i < MAXE / 64; ++i)
     if (lane + 64 * i < E) z[lane + 64 * i] = s[i];
-  }
   __builtin_amdgcn_wave_barrier();
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
   for (int g = lane; g < a.groups; g += 64) {
-    float b = 0.f;
-    for (int e = g * per; e < (g + 1) * per; ++e) b = fmaxf(b, z[e]);
-    gs[g] = b;
+    float b = 0.f, c = 0.f;
+    for (int e = g * per; e < (g + 1) * per; ++e) {
+      c = fmaxf(c, fminf(b, z[e]));
+      b = fmaxf(b, z[e]);
+    }
+    gs[g] = a.best == 2 ? b + c : b;
   }
   __builtin_amdgcn_wave_barrier();
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
@@ -104,7 +114,7 @@ __device__ __forceinline__ void choose(float* z, float* gs, int tok, const Route
   if (lane < a.K) {
     const int64_t i = (int64_t)tok * a.K + lane;
     a.experts[i] = my_e;
-    a.weights[i] = mine / (sum + 1e-20f);
+    a.weights[i] = mine / (sum + 1e-20f) * a.scale;
     if (hist) a.slots[i] = atomicAdd(hist + my_e, 1);  // within the workgroup; the base is added below
   }
 }
@@ -280,12 +290,12 @@ __global__ void __launch_bounds__(256) spread_kernel(const f32x4* __restrict__ x
 
 // h [T, W], router [E, W] -> experts, weights [T, K]; with counts (zero) and slots also the places of all pairs
 extern "C" int ds_route(const void* h, const void* router, int* experts, float* weights, int* counts, int* slots, int T, int W,
-                        int E, int K, int groups, int keep, int dtype, hipStream_t st) {
+                        int E, int K, int groups, int keep, int sigmoid, int best, float scale, int dtype, hipStream_t st) {
   if (T <= 0) return 0;
   if (W <= 0 || E <= 0 || E > MAXE || K <= 0 || K > MAXK || groups <= 0 || E % groups || keep <= 0 || keep > groups ||
-      K > keep * (E / groups) || (!counts != !slots))
+      K > keep * (E / groups) || (!counts != !slots) || best < 1 || best > 2)
     return (int)hipErrorInvalidValue;
-  const RouteArgs a{T, W, E, K, groups, keep, experts, weights, counts, slots};
+  const RouteArgs a{T, W, E, K, groups, keep, sigmoid, best, scale, experts, weights, counts, slots};
   if (dtype == DS_BF16 && W % 8 == 0) {
 #define GO(ET, TM, NW)                                                                                              \
   hipLaunchKernelGGL((route_mfma_kernel<ET, TM, NW>), dim3((T + 16 * TM - 1) / (16 * TM)), dim3(64 * NW), 0, st,     \

@@ -26,14 +26,17 @@ def clamped_glu(gu, limit, alpha=1.702, shift=1.0):
     return f(gu, limit, alpha, shift)
 
 
-def qk_norm_append(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H):
+def qk_norm_append(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H, cs=None):
+    """Rows [q | k | v] (they may be columns of wider ones) -> q [T, H, dk]; k and v into the paged cache. The pairs (2 i, 2 i + 1)
+    of every query and key head's first 2 half columns are turned by cs [T, half, 2] (None: no rotation), then each head is
+    divided by its root mean square, times qw / kw (None: no weight)."""
     f = attn_ops().qk_norm_append if use_native(qkv) else reference.qk_norm_append
-    return f(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H)
+    return f(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H, cs)
 
 
-def rope_table(pos, freq):
-    """cos and sin of pos [T] * freq [half] (fp64) -> [T, half, 2] fp32."""
-    return (attn_ops() if use_native(pos) else reference).rope_table(pos, freq)
+def rope_table(pos, freq, mult=1.0):
+    """cos and sin of pos [T] * freq [half] (fp64), times `mult` -> [T, half, 2] fp32."""
+    return (attn_ops() if use_native(pos) else reference).rope_table(pos, freq, mult)
 
 
 def qk_rope_append(qkv, bias, qw, kw, eps, cs, meta, kc, vc, H, v_mult=1.0):
@@ -44,26 +47,27 @@ def qk_rope_append(qkv, bias, qw, kw, eps, cs, meta, kc, vc, H, v_mult=1.0):
     return f(qkv, bias, qw, kw, eps, cs, v_mult, meta.pos_ids, meta.seq_ids, meta.block_tables, kc, vc, H)
 
 
-def ragged_attention(q, kc, vc, meta, scale, softcap=0.0, window=0, chunk=0, sink=None, out=None):
+def ragged_attention(q, kc, vc, meta, scale, softcap=0.0, window=0, chunk=0, sink=None, out=None, gate=None):
     """q [T, H, dk] of a ragged batch (`RaggedMeta`) over the paged cache, the new tokens already appended -> [T, H, dv], or
-    into `out` [T, H dv] (it may be columns of a wider matrix). `sink` [H]: exp(sink) joins the denominators."""
+    into `out` [T, H dv] (it may be columns of a wider matrix). `sink` [H]: exp(sink) joins the denominators. `gate` [T, H]
+    (columns of a wider matrix): every head's output times the sigmoid of its number."""
     T, H, dv = q.shape[0], q.shape[1], vc.shape[3]
     args = (meta.block_tables, meta.pos_ids, meta.seq_ids, scale, softcap, window, chunk)
     if out is None:
         out = q.new_empty(T, H * dv)
-        return ragged_attention(q, kc, vc, meta, scale, softcap, window, chunk, sink, out).view(T, H, dv)
+        return ragged_attention(q, kc, vc, meta, scale, softcap, window, chunk, sink, out, gate).view(T, H, dv)
     if not use_native(q):
-        return out.copy_(reference.paged_attention(q, kc, vc, *args, sink).reshape(T, H * dv))
+        return out.copy_(reference.paged_attention(q, kc, vc, *args, sink, gate).reshape(T, H * dv))
     ops = attn_ops()
     if q.dtype != torch.bfloat16 or not ops.paged_tiled_ok(kc.shape[3], dv):
-        return ops.paged_generic(q, kc, vc, *args, sink, out)
+        return ops.paged_generic(q, kc, vc, *args, sink, out, gate)
     nd = meta.n_decode
     if nd < len(meta.start_host):
         ops.paged_prefill(q, kc, vc, meta.block_tables, meta.start_pos, meta.cu_q, meta.work, scale, softcap, window, chunk,
-                          sink, out)
+                          sink, out, gate)
     if nd:
         ops.paged_decode(q[:nd], kc, vc, meta.block_tables[:nd], meta.seq_lens[:nd], meta.max_len, scale, softcap, window,
-                         chunk, out, sink)
+                         chunk, out, sink, gate)
     return out
 
 
@@ -87,9 +91,9 @@ def linear(x, w, sh=None, act=None):
     rows up), else the library product. act "gelu": the exact gelu of it (the stream's epilogue, else a pass of its own)."""
     rows = x.numel() // x.shape[-1]
     code = None if act is None else ACTS[act]
-    if sh is not None and x.is_cuda and 2 <= rows <= DECODE_ROWS:
+    if sh is not None and x.is_cuda and x.is_contiguous() and 2 <= rows <= DECODE_ROWS:
         return gemv_ops().decode_linear_sh(x, sh.wsh, sh.shape[0], act=code)
-    if x.is_cuda and x.dtype == torch.bfloat16 and 0 < rows <= DECODE_ROWS and \
+    if x.is_cuda and x.is_contiguous() and x.dtype == torch.bfloat16 and 0 < rows <= DECODE_ROWS and \
             gemv_ops().decode_linear_ok(rows, x.shape[-1]):
         return gemv_ops().decode_linear(x, w, act=code)
     y = F.linear(x, w)

@@ -1,7 +1,8 @@
 """Ops of hybrid decoders without residual streams (`inference/model_implementations/hybrid.py`): norms on sublayer
-outputs, latent attention, recurrences with a scalar decay per head, gated norms, token-side inputs.
+outputs, latent attention, recurrences with a scalar decay per head or a decay per channel and state, gated norms, token-side
+inputs.
 
-Device tensors run the gfx950 kernels of `ds_mixer_ops` and `ds_scan_ops` (fp32 or bf16 storage); host tensors the plain
+Device tensors run the gfx950 kernels of `ds_mixer_ops`, `ds_scan_ops` and `ds_selective_ops` (fp32 or bf16 storage); host tensors the plain
 versions in `ops/reference.py`, as everywhere in `ops`. Residual, norms, angles, scores, softmax, decays and the recurrent state are
 fp32 whatever the storage type."""
 from dataclasses import dataclass
@@ -10,7 +11,7 @@ import torch
 import torch.nn.functional as F
 
 from . import reference
-from .native import mixer_ops, scan_ops, use_native
+from .native import mixer_ops, scan_ops, selective_ops, use_native
 
 
 def post_norm(x, y, w, eps, ids=None, embed=None, rows=None, final_w=None, mult=1.0):
@@ -44,28 +45,32 @@ def gated_norm(y, proj, gate, w, parts, eps, mode, out=None):
 
 
 # ------------------------------------------------------------------------------------------------ latent attention
-def latent_prepare(down, qw, kvw, eps, freq, meta, lat, q_rank):
-    """Projection rows [q latent | kv latent | rotated part] -> normed query latent [T, q_rank]; the normed latent and the
-    rotated part of every token go into the paged cache lat [blocks, 1, block, kv_rank + rot]."""
+def latent_prepare(down, qw, kvw, eps, freq, meta, lat, q_rank, mult=1.0):
+    """Projection rows [q latent | kv latent | rotated part] (they may be columns of wider ones) -> normed query latent
+    [T, q_rank] (q_rank 0: None); the normed latent and the rotated part of every token go into the paged cache lat
+    [blocks, 1, block, kv_rank + rot]. `mult`: factor of cosine and sine."""
     f = mixer_ops().latent_prepare if use_native(down) else reference.latent_prepare
-    return f(down, qw, kvw, eps, freq, meta.pos_ids, meta.seq_ids, meta.block_tables, lat, q_rank)
+    return f(down, qw, kvw, eps, freq, mult, meta.pos_ids, meta.seq_ids, meta.block_tables, lat, q_rank)
 
 
-def latent_attention(q, lat, ukv, ukt, freq, sink, meta, scale, d, e):
-    """q [T, H, d + rot] (not rotated yet) of a ragged batch over the paged latents -> [T, H, e].
+def latent_attention(q, lat, ukv, ukt, freq, sink, meta, scale, d, e, window=0, mult=1.0):
+    """q [T, H, d + rot] (not rotated yet; tokens may lie further apart) of a ragged batch over the paged latents -> [T, H, e].
+    `sink` [H] (or None): exp(sink) joins the denominators. `window`: keys a token sees, itself included (0: all before it).
 
     Decodes and short portions fold the key map into the query and attend to the latents themselves (every cached byte is
-    read once for all heads); longer portions expand keys and values of their context with one product and run tiled
-    attention per head. ukv [H (d + e), kv_rank]: key rows, then value rows; ukt [H, kv_rank, d]: the key map per head."""
+    read once for all heads); longer portions expand keys and values of their context (what the window lets their first token
+    see of it, and on) with one product and run tiled attention per head. ukv [H (d + e), kv_rank]: key rows, then value rows;
+    ukt [H, kv_rank, d]: the key map per head."""
     T, H, R = q.shape[0], q.shape[1], ukt.shape[1]
     if not use_native(q):
-        return reference.latent_attention(q, lat, ukv, freq, sink, meta.block_tables, meta.pos_ids, meta.seq_ids, scale, d, e)
+        return reference.latent_attention(q, lat, ukv, freq, mult, sink, meta.block_tables, meta.pos_ids, meta.seq_ids, scale, d,
+                                          e, window)
     ops = mixer_ops()
     tiled = q.dtype == torch.bfloat16 and ops.latent_tiled_ok(d, q.shape[2] - d, e, R)
     short = meta.cu_host[meta.n_short] if tiled else T
     o = q.new_empty(T, H, e)
     if short:
-        ql = ops.head_linear(q[:short], ukt, freq, meta.pos_ids[:short])  # [short, H, R + rot]
+        ql = ops.head_linear(q[:short], ukt, freq, meta.pos_ids[:short], None, mult)  # [short, H, R + rot]
         if tiled:
             ol = q.new_empty(short, H, R)
             cu = meta.cu_host
@@ -73,16 +78,17 @@ def latent_attention(q, lat, ukv, ukt, freq, sink, meta, scale, d, e):
                 if a < b:
                     longest = 1 if b == meta.n_decode else max(cu[i + 1] - cu[i] for i in range(a, b))
                     ops.latent_decode(ql, lat, meta.block_tables, meta.cu_q, meta.start_pos, a, b - a, longest, cu[a], cu[b],
-                                      meta.max_len, R, scale, sink, ol)
+                                      meta.max_len, R, scale, sink, ol, window)
         else:
-            ol = ops.latent_generic(ql, lat, meta.block_tables, meta.pos_ids, meta.seq_ids, R, scale, sink)
+            ol = ops.latent_generic(ql, lat, meta.block_tables, meta.pos_ids, meta.seq_ids, R, scale, sink, window)
         ops.head_linear(ol, ukv[H * d:].view(H, e, R), out=o[:short])
     if short < T:
-        ctx = ops.latent_gather(lat, meta.block_tables, meta.kv_offs, meta.n_short, meta.kv_total)
+        offs, first_keys, total = meta.contexts(window)
+        ctx = ops.latent_gather(lat, meta.block_tables, offs, first_keys, meta.n_short, total)
         kv = F.linear(ctx[:, :R], ukv)
-        ops.rotate_tail(q[short:], freq, meta.pos_ids[short:], q.shape[2] - d)
-        ops.latent_prefill(q, kv, ctx, meta.start_pos, meta.cu_q, meta.work[meta.n_short - meta.n_decode:], meta.kv_offs,
-                           meta.n_short, meta.kv_total, d, e, scale, sink, o)
+        ops.rotate_tail(q[short:], freq, meta.pos_ids[short:], q.shape[2] - d, mult)
+        ops.latent_prefill(q, kv, ctx, meta.start_pos, meta.cu_q, meta.work[meta.n_short - meta.n_decode:], offs, first_keys,
+                           meta.n_short, total, d, e, scale, sink, o, window)
     return o
 
 
@@ -161,3 +167,21 @@ def matrix_memory(proj, lay, slots, meta, gates, bi, bf, cap, scale):
                                longest)
     qk, v = ops.scan_split(proj, lay.dims, None)
     return _scan(ops, proj, lay, qk, v, gb, None, None, scale, slots["state"], slots["norm"], floors, None, meta)
+
+
+# ------------------------------------------------------------------------------------------------ selective recurrences
+def causal_conv(x, w, b, conv_state, meta):
+    """silu(conv(x) + b): x [T, C] (it may be columns of a wider matrix), w [C, taps] (last column: the current token), inputs
+    before a portion from its slot of conv_state [slots, taps - 1, C]. The slots stay as they are (`selective_scan` moves
+    them on)."""
+    f = (selective_ops() if use_native(x) else reference).causal_conv
+    return f(x, w, b, conv_state, *((meta.seq_ids, ) if use_native(x) else ()), meta.cu_q, meta.start_pos, meta.slots)
+
+
+def selective_scan(x, dt, bc, z, dt_bias, a_log, skip, state, conv_x, conv_state, meta):
+    """A decay per channel and state: with step = softplus(dt + dt_bias) and A = -exp(a_log) [C, N],
+    S[c, n] <- exp(step_c A[c, n]) S[c, n] + step_c x_c B_n, y_c = sum_n S[c, n] C_n + skip_c x_c, out = y silu(z) [T, C]. bc
+    [T, B | C], z [T, C]: columns of wider matrices. state [slots, C, N rounded up to 4] fp32 and conv_state, the last inputs
+    of the convolution conv_x [T, C], advance."""
+    f = (selective_ops() if use_native(x) else reference).selective_scan
+    return f(x, dt, bc, z, dt_bias, a_log, skip, state, conv_x, conv_state, meta.cu_q, meta.start_pos, meta.slots)

@@ -43,8 +43,14 @@ def scan_ops():
 
 
 @functools.lru_cache(None)
+def selective_ops():
+    """Recurrences with a decay per channel and state, short convolutions."""
+    return op_builder.load("ds_selective_ops")
+
+
+@functools.lru_cache(None)
 def expert_ops():
-    """Mixture of experts with grouped routing, pre-norm residual."""
+    """Mixture of experts with grouped routing, residual with norms on sublayer inputs and outputs."""
     return op_builder.load("ds_expert_ops")
 
 

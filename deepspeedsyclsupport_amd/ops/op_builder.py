@@ -93,12 +93,21 @@ EXTENSIONS = {
         ],
         "bindings": ["bind/scan_bind.cpp"],
     },
-    # mixture of experts with grouped routing, pre-norm residual
+    # recurrences with a decay per channel and state, short convolutions
+    "ds_selective_ops": {
+        "kind": "hip",
+        "kernels": [
+            "recur/causal_conv.hip",
+            "recur/selective_scan.hip",
+        ],
+        "bindings": ["bind/selective_bind.cpp"],
+    },
+    # mixture of experts with grouped routing, residual with norms on sublayer inputs and outputs
     "ds_expert_ops": {
         "kind": "hip",
         "kernels": [
             "norm/pre_norm.hip",
-            "act/clamped_glu.hip",
+            "act/row_act.hip",
             "moe/expert_route.hip",
             "moe/expert_gemm.hip",
         ],

@@ -151,13 +151,13 @@ def clamped_glu(gu, limit, alpha, shift):
     return (g * torch.sigmoid(alpha * g) * (u.clamp(-limit, limit) + shift)).to(gu.dtype)
 
 
-def qk_norm_append(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H):
+def qk_norm_append(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc, vc, H, cs=None):
     G, BS, dk, dv = kc.shape[1], kc.shape[2], kc.shape[3], vc.shape[3]
     T = qkv.shape[0]
     q, k, v = qkv.float().split([H * dk, G * dk, G * dv], -1)
-    q, k, v = q.view(T, H, dk), k.view(T, G, dk), v.view(T, G, dv)
-    q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps) * qw
-    k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps) * kw
+    q, k, v = _turn_neighbours(q.view(T, H, dk), cs), _turn_neighbours(k.view(T, G, dk), cs), v.reshape(T, G, dv)
+    q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps) * (1.0 if qw is None else qw)
+    k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps) * (1.0 if kw is None else kw)
     if vfirst is not None:
         v = (1 - lam) * v + lam * vfirst.float().view(T, G, dv)
     slot = pos.long()
@@ -167,9 +167,9 @@ def qk_norm_append(qkv, qw, kw, eps, vfirst, lam, pos, seq_ids, block_table, kc,
     return q.to(qkv.dtype)
 
 
-def rope_table(pos, freq):
+def rope_table(pos, freq, mult):
     a = pos.double()[:, None] * freq.double()
-    return torch.stack([a.cos(), a.sin()], -1).float()
+    return torch.stack([a.cos(), a.sin()], -1).float() * mult
 
 
 def _turn_pairs(x, cs):
@@ -179,6 +179,15 @@ def _turn_pairs(x, cs):
     h, (c, s) = cs.shape[1], cs[:, None].unbind(-1)
     u, v = x[..., :h], x[..., h:2 * h]
     return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * h:]], -1)
+
+
+def _turn_neighbours(x, cs):
+    """x [T, heads, d]: pairs (2 i, 2 i + 1) turned by cs [T, half, 2]."""
+    if cs is None:
+        return x
+    h, (c, s) = cs.shape[1], cs[:, None].unbind(-1)
+    u, v = x[..., 0:2 * h:2], x[..., 1:2 * h:2]
+    return torch.cat([torch.stack([u * c - v * s, v * c + u * s], -1).flatten(-2), x[..., 2 * h:]], -1)
 
 
 def qk_rope_append(qkv, bias, qw, kw, eps, cs, v_mult, pos, seq_ids, block_table, kc, vc, H):
@@ -194,8 +203,9 @@ def qk_rope_append(qkv, bias, qw, kw, eps, cs, v_mult, pos, seq_ids, block_table
     return q.to(qkv.dtype)
 
 
-def paged_attention(q, kc, vc, block_table, pos, seq_ids, scale, softcap, window, chunk, sink=None):
-    """q [T, H, dk] at absolute positions -> [T, H, dv]; visible keys [lo(pos), pos] (window / chunk start / 0)."""
+def paged_attention(q, kc, vc, block_table, pos, seq_ids, scale, softcap, window, chunk, sink=None, gate=None):
+    """q [T, H, dk] at absolute positions -> [T, H, dv]; visible keys [lo(pos), pos] (window / chunk start / 0). `gate` [T, H]:
+    heads come out times its sigmoid."""
     G, BS = kc.shape[1], kc.shape[2]
     out = q.new_empty(q.shape[0], q.shape[1], vc.shape[3])
     for t in range(q.shape[0]):
@@ -212,7 +222,8 @@ def paged_attention(q, kc, vc, block_table, pos, seq_ids, scale, softcap, window
             p = torch.cat([s, sink.view(G, -1, 1)], -1).softmax(-1)[..., :-1]
         else:
             p = s.softmax(-1)
-        out[t] = torch.einsum("grn,ngd->grd", p, v).reshape(q.shape[1], -1).to(q.dtype)
+        o = torch.einsum("grn,ngd->grd", p, v).reshape(q.shape[1], -1)
+        out[t] = (o if gate is None else o * torch.sigmoid(gate[t].float())[:, None]).to(q.dtype)
     return out
 
 
@@ -298,29 +309,29 @@ def gated_norm(y, proj, gate, w, parts, eps, mode, out=None):
     return v if out is None else out.copy_(v)
 
 
-def _turn(x, freq, pos):
-    """Rotate-half on the first 2 len(freq) columns of x [T, .., r] at positions pos [T]."""
+def _turn(x, freq, mult, pos):
+    """Rotate-half on the first 2 len(freq) columns of x [T, .., r] at positions pos [T], cosine and sine times `mult`."""
     h = freq.numel()
     a = (pos.double()[:, None] * freq.double()).view(-1, *[1] * (x.dim() - 2), h)
-    c, s = a.cos().float(), a.sin().float()
+    c, s = a.cos().float() * mult, a.sin().float() * mult
     u, v = x[..., :h], x[..., h:2 * h]
     return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * h:]], -1)
 
 
-def latent_prepare(down, qw, kvw, eps, freq, pos, seq_ids, block_table, lat, q_rank):
+def latent_prepare(down, qw, kvw, eps, freq, mult, pos, seq_ids, block_table, lat, q_rank):
     R, BS = kvw.numel(), lat.shape[2]
     d = down.float()
-    rows = torch.cat([_rms(d[:, q_rank:q_rank + R], eps) * kvw, _turn(d[:, q_rank + R:], freq, pos)], -1)
+    rows = torch.cat([_rms(d[:, q_rank:q_rank + R], eps) * kvw, _turn(d[:, q_rank + R:], freq, mult, pos)], -1)
     slot = pos.long()
     lat[block_table.long()[seq_ids.long(), slot // BS], 0, slot % BS] = rows.to(lat.dtype)
-    return (_rms(d[:, :q_rank], eps) * qw).to(down.dtype)
+    return (_rms(d[:, :q_rank], eps) * qw).to(down.dtype) if q_rank else None
 
 
-def latent_attention(q, lat, ukv, freq, sink, block_table, pos, seq_ids, scale, d, e):
+def latent_attention(q, lat, ukv, freq, mult, sink, block_table, pos, seq_ids, scale, d, e, window=0):
     T, H = q.shape[:2]
     R, BS = ukv.shape[1], lat.shape[2]
     uk, uv = ukv.float().split([H * d, H * e])
-    q = torch.cat([q[..., :d].float(), _turn(q[..., d:].float(), freq, pos)], -1)
+    q = torch.cat([q[..., :d].float(), _turn(q[..., d:].float(), freq, mult, pos)], -1)
     out = q.new_empty(T, H, e, dtype=ukv.dtype)
     for s in seq_ids.unique().tolist():
         rows = (seq_ids == s).nonzero().view(-1)
@@ -329,8 +340,14 @@ def latent_attention(q, lat, ukv, freq, sink, block_table, pos, seq_ids, scale, 
         k = torch.cat([(c[:, :R] @ uk.t()).view(-1, H, d), c[:, None, R:].expand(-1, H, -1)], -1)
         v = (c[:, :R] @ uv.t()).view(-1, H, e)
         sc = torch.einsum("thd,jhd->htj", q[rows], k) * scale
-        sc = sc.masked_fill(j > pos[rows][:, None], float("-inf"))
-        p = torch.cat([sc, sink[:, None, None].expand(-1, rows.numel(), 1)], -1).softmax(-1)[..., :-1]
+        hidden = j > pos[rows][:, None]
+        if window:
+            hidden |= j <= pos[rows][:, None] - window
+        sc = sc.masked_fill(hidden, float("-inf"))
+        if sink is None:
+            p = sc.softmax(-1)
+        else:
+            p = torch.cat([sc, sink[:, None, None].expand(-1, rows.numel(), 1)], -1).softmax(-1)[..., :-1]
         out[rows] = torch.einsum("htj,jhe->the", p, v).to(out.dtype)
     return out
 
@@ -412,42 +429,82 @@ def scan_chunk(qk, v, gb, log_decay, skip, scale, proj, dims, state, zstate, flo
 
 
 # ---------------------------------------------------------------- pre-norm residual, experts with grouped routing
-def expert_sum(y, w, rows):
+def expert_sum(y, w, rows, base=None):
     T, K = w.shape
     e = y.float()[rows.long().view(-1)] if rows is not None else y.float()
-    return (e.view(T, K, -1) * w[..., None]).sum(1).to(y.dtype)
+    s = (e.view(T, K, -1) * w[..., None]).sum(1)
+    return (s if base is None else s + base.float()).to(y.dtype)
 
 
-def pre_norm(x, y, yw, yrow, w, eps, ids, embed, mult, rows):
+def pre_norm(x, y, yw, yrow, base, w, eps, ids, embed, mult, rows, post_w, gate, gate_b):
+    norm = lambda s: s if w is None else _rms(s, eps) * w
     if y is None:
         x.copy_(embed.float()[ids.long()] * mult)
-        return (_rms(x, eps) * w).to(embed.dtype)
-    s = x + (y.float() if yw is None else expert_sum(y.float(), yw, yrow))
+        return norm(x).to(embed.dtype)
+    add = y.float() if yw is None else expert_sum(y.float(), yw, yrow, base)
+    if gate is not None:
+        add = add * torch.sigmoid(gate.float() + gate_b)
+    if post_w is not None:
+        add = _rms(add, eps) * post_w
+    s = x + add
     if rows is not None:
-        return (_rms(s[rows.long()], eps) * w).to(y.dtype)
+        return norm(s[rows.long()]).to(y.dtype)
     x.copy_(s)
-    return (_rms(s, eps) * w).to(y.dtype)
+    return norm(s).to(y.dtype)
 
 
-def route(h, router, k, groups, keep):
-    s = (h.float() @ router.float().t()).softmax(-1)
+def route(h, router, k, groups, keep, score=0, best=1, scale=1.0):
+    z = h.float() @ router.float().t()
+    s = torch.sigmoid(z) if score else z.softmax(-1)
     T, E = s.shape
-    best = s.view(T, groups, E // groups).amax(-1).topk(keep, -1).indices
-    open_ = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best, True).repeat_interleave(E // groups, 1)
+    per = E // groups
+    top = s.view(T, groups, per).topk(min(best, per), -1).values.sum(-1).topk(keep, -1).indices
+    open_ = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, top, True).repeat_interleave(per, 1)
     w, e = s.masked_fill(~open_, -1.0).topk(k, -1)
-    return e.to(torch.int32), w / (w.sum(-1, keepdim=True) + 1e-20)
+    return e.to(torch.int32), w / (w.sum(-1, keepdim=True) + 1e-20) * scale
 
 
-def silu_mul(gu):
-    g, u = gu.float().chunk(2, -1)
-    return (F.silu(g) * u).to(gu.dtype)
+def row_act(x, act):
+    if act == 1:
+        g, u = x.float().chunk(2, -1)
+        return (F.silu(g) * u).to(x.dtype)
+    return x.float().clamp(min=0).square().to(x.dtype) if act == 2 else x
 
 
-def expert_gemm(x, w, experts, div, gated):
-    out = x.new_empty(experts.numel(), w.shape[1] // (2 if gated else 1))
+def expert_gemm(x, w, experts, div, act):
+    out = x.new_empty(experts.numel(), w.shape[1] // (2 if act == 1 else 1))
     e = experts.view(-1).long()
     for i in e.unique().tolist():
         r = (e == i).nonzero().view(-1)
-        y = F.linear(x[r // div], w[i])
-        out[r] = silu_mul(y) if gated else y
+        out[r] = row_act(F.linear(x[r // div], w[i]), act)
+    return out
+
+
+# ---------------------------------------------------------------- recurrences with a decay per channel and state
+def causal_conv(x, w, b, conv_state, cu, start, slots):
+    T, C = x.shape
+    taps, y = w.shape[1], torch.empty(T, C)
+    for i in range(start.numel()):
+        p, q = int(cu[i]), int(cu[i + 1])
+        old = conv_state[int(slots[i])].float() if int(start[i]) and taps > 1 else torch.zeros(taps - 1, C)
+        seq = torch.cat([old, x[p:q].float()])
+        y[p:q] = sum(seq[j:j + q - p] * w[:, j] for j in range(taps)) + b
+    return F.silu(y).to(x.dtype)
+
+
+def selective_scan(x, dt, bc, z, dt_bias, a_log, skip, state, conv_x, conv_state, cu, start, slots):
+    T, C = x.shape
+    N = a_log.shape[1]
+    out, step, A = torch.empty_like(x), F.softplus(dt.float() + dt_bias, threshold=60), -a_log.exp()
+    for i in range(start.numel()):
+        p, q, slot, old = int(cu[i]), int(cu[i + 1]), int(slots[i]), int(start[i]) > 0
+        S = state[slot, :, :N].clone() if old else torch.zeros(C, N)
+        for t in range(p, q):
+            xt, B, Ct = x[t].float(), bc[t, :N].float(), bc[t, N:2 * N].float()
+            S = (step[t][:, None] * A).exp() * S + (step[t] * xt)[:, None] * B
+            out[t] = (((S * Ct).sum(-1) + skip * xt) * F.silu(z[t].float())).to(out.dtype)
+        state[slot, :, :N] = S
+        if conv_state is not None and conv_state.shape[1]:
+            before = conv_state[slot] if old else torch.zeros_like(conv_state[slot])
+            conv_state[slot] = torch.cat([before, conv_x[p:q]])[-conv_state.shape[1]:].clone()
     return out
