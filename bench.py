@@ -44,7 +44,8 @@ def parse():
                     help="train: the flagship training step (default); hybrid: serving throughput of hybrid decoders "
                          "beside the uniform one (benchmarks/hybrid_serving.py)")
     ap.add_argument("--sizes", default="2048,4096", help="--workload hybrid: model widths")
-    ap.add_argument("--model-kind", default="both", choices=["hybrid", "perelorn", "uniform", "lefisun", "uniform_moe", "both", "moe", "all"],
+    ap.add_argument("--model-kind", default="both", choices=["hybrid", "perelorn", "uniform", "lefisun", "uniform_moe",
+                                                           "nigilorn", "both", "moe", "close", "all"],
                     help="--workload hybrid")
     ap.add_argument("--local_rank", type=int, default=0)
     ap.add_argument("--host-dryrun", action="store_true",

@@ -6,8 +6,10 @@ counts, all through the ragged engine with random bf16 weights: whole-prompt pre
 * lefisun: Lefisun layers (chunked rotary attention beside a matrix memory, retention, routed experts); beside it
   uniform_moe, the Llama-style decoder with the same experts (Mixtral's routing), and the others with a dense feed-forward as
   wide as the experts of a token together
+* nigilorn: Nigilorn layers (selective state spaces, windowed attention, windowed latent attention, gated residual with norms on
+  both sides, token-side input, one dense feed-forward, then plain routed experts beside a shared one)
 
-    python bench.py --workload hybrid [--sizes 2048,4096] [--model-kind hybrid|perelorn|lefisun|uniform|uniform_moe|both|moe|all]
+    python bench.py --workload hybrid [--sizes 2048,4096] [--model-kind hybrid|perelorn|lefisun|nigilorn|uniform|uniform_moe|...]
 """
 import json
 import math
@@ -24,10 +26,13 @@ HEAD, CHUNK, STREAMS, VOCAB, SIDE = 128, 2048, 4, 32000, 256
 # feed-forward, so that the projections are of one size
 PERELORN = ("mamba2", "latent_attention", "lightning", "mamba2", "latent_attention", "lightning", "mamba2", "latent_attention")
 KINDS = {"both": ("hybrid", "uniform"), "moe": ("lefisun", "uniform_moe"),
-         "all": ("hybrid", "perelorn", "uniform", "lefisun", "uniform_moe")}
+         "close": ("nigilorn", "perelorn", "lefisun"),   # the last design and those it shares most with
+         "all": ("hybrid", "perelorn", "uniform", "lefisun", "uniform_moe", "nigilorn")}
 # Lefisun: attention of the others' size beside a memory of half its heads, retention in the places of their recurrences
 EXPERTS, TOP, GROUPS, KEEP = 32, 4, 4, 2
 LEFISUN = ("parallel", "retention") * 4
+# Nigilorn: state spaces in the places of the recurrences, the two kinds of attention by turns
+NIGILORN = ("mamba1", "window_attention", "mamba1", "latent_attention") * 2
 
 
 def specs(width):
@@ -64,7 +69,23 @@ def specs(width):
                           layer_specs=tuple({"type": t, "mixer": mixers[t], "mlp": mlp} for t in LEFISUN), **common)
     uniform_moe = DSModelSpec(arch="mixtral", norm="rms", pos="rope", max_positions=16384, num_experts=EXPERTS, moe_top_k=TOP,
                               **{**common, "intermediate_size": ff})
-    return {"hybrid": hybrid, "perelorn": perelorn, "uniform": uniform, "lefisun": lefisun, "uniform_moe": uniform_moe}
+    yarn = {"type": "yarn", "factor": 4.0, "fast": 32.0, "slow": 1.0, "original": 4096}
+    mixers = {"mamba1": {"inner": 2 * width, "state": 16, "dt_rank": width // 16, "conv": 4},
+              "window_attention": {"heads": h, "kv_heads": s["kv"], "dim": HEAD, "vdim": HEAD, "scale": HEAD**-0.5,
+                                   "mask": {"size": CHUNK}, "rot": {"base": 5e5, "dims": HEAD // 2, "pairs": "neighbours",
+                                                                    "scaling": yarn}},
+              "latent_attention": {"heads": h, "dim": HEAD, "rot_dim": 64, "vdim": HEAD, "kv_rank": 512, "sink": False,
+                                   "mask": {"size": CHUNK}, "rot": {"base": 10000.0, "dims": 64, "pairs": "neighbours",
+                                                                    "scaling": yarn}, "scale": (HEAD + 64)**-0.5}}
+    mlp = {**mlp, "act": "relu2", "shared": {"ff": ff},
+           "router": {"experts": EXPERTS, "top": TOP, "score": "sigmoid", "scale": 2.5,
+                      "groups": {"count": GROUPS, "keep": KEEP, "best": 2}}}
+    dense = {"kind": "silu_glu", "ff": s["ff"]}
+    nigilorn = DSModelSpec(arch="nigilorn", norm="rms", pos="none", residual="sandwich", residual_gate=True, token_side=SIDE,
+                           layer_specs=tuple({"type": t, "mixer": mixers[t], "mlp": mlp if i else dense}
+                                             for i, t in enumerate(NIGILORN)), **common)
+    return {"hybrid": hybrid, "perelorn": perelorn, "uniform": uniform, "lefisun": lefisun, "uniform_moe": uniform_moe,
+            "nigilorn": nigilorn}
 
 
 def build(spec, device, blocks):

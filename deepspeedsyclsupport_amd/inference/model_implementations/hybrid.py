@@ -602,7 +602,7 @@ class Mamba1Mixer(Mixer):
     def parameters(self, device):
         C = self.inner
         return {"conv_w": _f32((C, self.taps), 0.0, device), "conv_b": _f32((C, ), 0.0, device),
-                "a_log": _f32((C, self.N), 0.0, device), "dt_bias": _f32((C, ), 0.0, device), "skip": _f32((C, ), 0.0, device)}
+                "decay": _f32((C, self.N), -1.0, device), "dt_bias": _f32((C, ), 0.0, device), "skip": _f32((C, ), 0.0, device)}
 
     def matrices(self, dtype, device):
         return {"x_w": _empty((_up8(self.R + 2 * self.N), self.inner), dtype, device),
@@ -610,7 +610,8 @@ class Mamba1Mixer(Mixer):
 
     def shard(self, lw, r, tp):
         return {"qkv_w": lw["in_w"], "x_w": _fill_rows(lw["x_w"], self.R + 2 * self.N, "mix.x"), "dt_w": lw["dt_w"],
-                "o_w": _shard(lw["o_w"], r, tp, 1), **{n: lw[n] for n in ("conv_w", "conv_b", "a_log", "dt_bias", "skip")}}
+                "o_w": _shard(lw["o_w"], r, tp, 1), "decay": -lw["a_log"].float().exp(),
+                **{n: lw[n] for n in ("conv_w", "conv_b", "dt_bias", "skip")}}
 
     def state_geometry(self, dtype):
         g = {"state": ((self.inner, -(-self.N // 4) * 4), torch.float32)}
@@ -623,7 +624,7 @@ class Mamba1Mixer(Mixer):
         x = mixer_ops.causal_conv(proj[:, :C], layer.conv_w, layer.conv_b, st.get("conv"), meta)
         low = layer._linear(x, "x_w")
         dt = ops.linear(low[:, :self.R], layer.dt_w)
-        y = mixer_ops.selective_scan(x, dt, low[:, self.R:self.R + 2 * self.N], proj[:, C:2 * C], layer.dt_bias, layer.a_log,
+        y = mixer_ops.selective_scan(x, dt, low[:, self.R:self.R + 2 * self.N], proj[:, C:2 * C], layer.dt_bias, layer.decay,
                                      layer.skip, st["state"], proj[:, :C], st.get("conv"), meta)
         if self.out_width == C:
             return y

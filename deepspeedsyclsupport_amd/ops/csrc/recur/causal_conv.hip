@@ -7,8 +7,6 @@
 
 namespace {
 
-constexpr int TILE = 8;  // consecutive tokens of a wave
-
 template <typename T, int V>
 __device__ __forceinline__ void ldv(const T* p, float (&v)[V]) {
   if constexpr (V == 8) Vec8<T>::load(p, v);
@@ -31,8 +29,9 @@ struct ConvArgs {
   int tokens, C, taps;
 };
 
-// TAPS: filter length, the tile's inputs in registers; 0: any length, inputs read per tap. V channels per lane.
-template <typename T, int TAPS, int V>
+// TAPS: filter length, the tile's inputs in registers; 0: any length, inputs read per tap. V channels per lane; TILE: consecutive
+// tokens of a wave (a few decodes spread over the chip one by one).
+template <typename T, int TAPS, int V, int TILE>
 __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
   const int lane = threadIdx.x & 63, parts = (a.C + 64 * V - 1) / (64 * V), taps = TAPS ? TAPS : a.taps;
   const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6), tl = item / parts * TILE;
@@ -98,18 +97,24 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
   }
 }
 
-template <typename T, int V>
+template <typename T, int V, int TILE>
 int launch(const ConvArgs& a, hipStream_t st) {
   const int64_t items = (int64_t)((a.tokens + TILE - 1) / TILE) * ((a.C + 64 * V - 1) / (64 * V));
   const dim3 grid((unsigned)((items + 3) / 4));
   switch (a.taps) {
-    case 2: hipLaunchKernelGGL((causal_conv_kernel<T, 2, V>), grid, dim3(256), 0, st, a); break;
-    case 3: hipLaunchKernelGGL((causal_conv_kernel<T, 3, V>), grid, dim3(256), 0, st, a); break;
-    case 4: hipLaunchKernelGGL((causal_conv_kernel<T, 4, V>), grid, dim3(256), 0, st, a); break;
-    default: hipLaunchKernelGGL((causal_conv_kernel<T, 0, V>), grid, dim3(256), 0, st, a);
+    case 2: hipLaunchKernelGGL((causal_conv_kernel<T, 2, V, TILE>), grid, dim3(256), 0, st, a); break;
+    case 3: hipLaunchKernelGGL((causal_conv_kernel<T, 3, V, TILE>), grid, dim3(256), 0, st, a); break;
+    case 4: hipLaunchKernelGGL((causal_conv_kernel<T, 4, V, TILE>), grid, dim3(256), 0, st, a); break;
+    default: hipLaunchKernelGGL((causal_conv_kernel<T, 0, V, TILE>), grid, dim3(256), 0, st, a);
   }
   DS_CHECK_LAUNCH();
   return 0;
+}
+
+template <typename T>
+int conv(const ConvArgs& a, bool vec, hipStream_t st) {
+  if (!vec) return launch<T, 1, 8>(a, st);
+  return a.tokens <= 512 ? launch<T, 8, 1>(a, st) : launch<T, 8, 8>(a, st);
 }
 
 }  // namespace
@@ -122,7 +127,7 @@ extern "C" int ds_causal_conv(const void* x, int64_t ld, const float* w, const f
   if (C <= 0 || taps < 1 || ld < C || (taps > 1 && !state)) return (int)hipErrorInvalidValue;
   const ConvArgs a{x, ld, w, b, state, seq_ids, cu, start, slots, out, tokens, C, taps};
   const bool vec = C % 8 == 0 && ld % 8 == 0 && (((uintptr_t)x | (uintptr_t)state) & 15) == 0;
-  if (dtype == DS_F32) return vec ? launch<float, 8>(a, st) : launch<float, 1>(a, st);
-  if (dtype == DS_BF16) return vec ? launch<bf16, 8>(a, st) : launch<bf16, 1>(a, st);
+  if (dtype == DS_F32) return conv<float>(a, vec, st);
+  if (dtype == DS_BF16) return conv<bf16>(a, vec, st);
   return (int)hipErrorInvalidValue;
 }

@@ -1,20 +1,23 @@
 // Selective scan: recurrences with a decay of their own per channel and state, CDNA4 (gfx950).
 //
-// Every channel c carries N numbers in fp32 that start at zero. With step = softplus(dt + dt_bias) and A = -exp(A_log):
+// Every channel c carries N numbers in fp32 that start at zero. With step = softplus(dt + dt_bias) and given A[c, n] < 0:
 //     S[c, n] <- exp(step_c A[c, n]) S[c, n] + step_c x_c B_n;   y_c = sum_n S[c, n] C_n + D_c x_c;   out_c = y_c silu(z_c)
-// B and C belong to the token, shared by all channels. One exponential and four multiplications per number and token: bound by
-// the vector unit (the exponential takes a quarter of its rate), so there is nothing for the matrix cores to do.
+// B and C belong to the token, shared by all channels. There is one exponential and four multiplications per number and token
+// and nothing for the matrix cores to do: long portions are bound by the vector unit and by LDS reads, decoding by the state.
 //
-// A workgroup of four waves takes 256 / LP neighbouring channels of one sequence and walks its new tokens, TT at a time. LP lanes
-// share a channel, NPL numbers each, in registers throughout. LP is chosen so that the waves cover the chip: few lanes per
-// channel spend the least on what a channel does once per token, many make a single long sequence parallel.
-//  * stage: step and step * x of every (token, channel) of the tile, B and C, all fp32, into LDS; x and z stay with the thread
-//    that will write the same (token, channel). The next tile's operands are on their way meanwhile.
-//  * walk: token by token without barriers. Partial sums of y meet across the LP lanes; lane i keeps those of token i of LP.
-//  * write: y from LDS, skip and gate applied, in whole rows.
-// Decoding is the same with a tile of one token: it streams the state, 16 bytes per lane. At the end the workgroup moves its
-// channels' convolution windows on (the convolution, which reads the old ones, has finished by then). A sequence whose portion
-// starts at position 0 starts from zero: slots need no clearing between owners.
+//  * scan (long portions): a workgroup of four waves takes 256 / LP neighbouring channels of one sequence and walks its new
+//    tokens, TT at a time. LP lanes share a channel, NPL numbers each, in registers throughout. LP is chosen so that a SIMD gets
+//    two waves at least (a single one issues at little more than half the rate): few lanes per channel spend the least on what
+//    a channel does once per token, many make a single long sequence parallel.
+//      stage: step and step * x of every (token, channel) of the tile, B and C, all fp32, into LDS; x and z stay with the thread
+//        that will write the same (token, channel). The next tile's operands are on their way meanwhile.
+//      walk: token by token without barriers, LDS rows along the tokens, so that a read brings two of them. Shares of y of LP
+//        tokens meet in the lanes whose tokens they are: pairs of lanes trade halves, log2 LP times.
+//      write: y from LDS, skip and gate applied, in whole rows.
+//  * step (decodes, short portions): four numbers per lane, nothing but registers, so that many waves stream the states.
+//
+// At the end the channels' convolution windows move on (the convolution, which reads the old ones, has finished by then). A
+// sequence whose portion starts at position 0 starts from zero: slots need no clearing between owners.
 #include "ds_hip.h"
 
 #include <type_traits>
@@ -25,134 +28,250 @@ constexpr int NT = 256;
 constexpr float LOG2E = 1.4426950408889634f;
 
 struct SelArgs {
-  const void *x, *dt, *bc, *z, *cx;       // x, dt [T, C]; bc [T, B | C], z, cx [T, C]: columns, rows ld* apart
+  const void *x, *dt, *bc, *z, *cx;       // x, dt [T, C]; bc [T, B | C]; z, cx [T, C]: columns, rows ld* apart
   int64_t ldbc, ldz, ldcx;
-  const float *dt_bias, *a_log, *skip;    // [C], [C, N], [C]
+  const float *dt_bias, *decay, *skip;    // [C], [C, N], [C]
   float* state;                           // [slots, C, NS]
   void* conv;                             // [slots, taps - 1, C]: last rows of cx, or null
-  const int *cu, *start, *slots;
+  const int *list, *cu, *start, *slots;   // list: sequences, `stride` apart
   void* out;                              // [T, C]
-  int C, N, NS, taps, seqs;
+  int C, N, NS, taps, seqs, stride;
 };
 
+__device__ __forceinline__ float exp_f(float v) { return __builtin_amdgcn_exp2f(v * LOG2E); }
 // log(1 + e^v) to a few units in the last place: what adding 1 rounds off is put right by the last factor
 __device__ __forceinline__ float softplus_f(float v) {
-  const float u = __expf(-fabsf(v)), w = 1.f + u, d = w - 1.f;
-  return fmaxf(v, 0.f) + (d == 0.f ? u : __logf(w) * (u * __builtin_amdgcn_rcpf(d)));
+  constexpr float LN2 = 0.6931471805599453f;
+  const float u = exp_f(-fabsf(v)), w = 1.f + u, d = w - 1.f;
+  return fmaxf(v, 0.f) + (d == 0.f ? u : __builtin_amdgcn_logf(w) * (LN2 * u * __builtin_amdgcn_rcpf(d)));
 }
-__device__ __forceinline__ float silu_f(float z) { return z * __builtin_amdgcn_rcpf(1.f + __expf(-z)); }
+__device__ __forceinline__ float silu_f(float z) { return z * __builtin_amdgcn_rcpf(1.f + exp_f(-z)); }
 
-// Sum over groups of LP neighbouring lanes, in all of them
+// V neighbouring elements
+template <typename T, int V>
+struct Few {
+  typedef T TV __attribute__((ext_vector_type(2)));
+  T v[V];
+  __device__ __forceinline__ void load(const T* p) {
+    if constexpr (V == 2) *reinterpret_cast<TV*>(v) = *reinterpret_cast<const TV*>(p);
+    else v[0] = p[0];
+  }
+};
+template <typename T, int V>
+__device__ __forceinline__ void store_few(T* p, const float (&f)[V]) {
+  typedef T TV __attribute__((ext_vector_type(2)));
+  if constexpr (V == 2) *reinterpret_cast<TV*>(p) = TV{(T)f[0], (T)f[1]};
+  else p[0] = (T)f[0];
+}
+
+template <int CTRL>
+__device__ __forceinline__ float dpp(float v) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
+}
+constexpr int XOR1 = 0xb1, XOR2 = 0x4e, MIRROR8 = 0x141, MIRROR16 = 0x140;  // lane moves within 4, 8, 16
+
+// p[i]: this lane's share of a sum for token i of LP. Returns the sum over the group of LP lanes of the shares of the lane's own
+// token: in every step pairs of lanes trade halves of what they hold.
 template <int LP>
-__device__ __forceinline__ float group_sum(float v) {
-  auto add = [&](auto sel) {
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), decltype(sel)::value, 0xf, 0xf, true));
+__device__ __forceinline__ float trade(float (&p)[LP], int g) {
+  auto step = [&](auto move, int n) {
+    const bool up = g & n;
+#pragma unroll
+    for (int i = 0; i < n; ++i) {
+      const float keep = up ? p[n + i] : p[i], give = up ? p[i] : p[n + i];
+      p[i] = keep + dpp<decltype(move)::value>(give);
+    }
   };
-  add(std::integral_constant<int, 0xb1>{});                      // quad_perm: lane ^ 1
-  add(std::integral_constant<int, 0x4e>{});                      // quad_perm: lane ^ 2
-  if constexpr (LP >= 8) add(std::integral_constant<int, 0x141>{});   // row_half_mirror: the other quad of 8
-  if constexpr (LP >= 16) add(std::integral_constant<int, 0x140>{});  // row_mirror: the other half of 16
-  return v;
+  if constexpr (LP == 16) step(std::integral_constant<int, MIRROR16>{}, 8);
+  if constexpr (LP >= 8) step(std::integral_constant<int, MIRROR8>{}, 4);
+  step(std::integral_constant<int, XOR2>{}, 2);
+  step(std::integral_constant<int, XOR1>{}, 1);
+  return p[0];
 }
 
-template <typename T, int LP, int NPL>
+// A channel's convolution window: the last taps - 1 of [old window | the portion's inputs]
+template <typename T>
+__device__ __forceinline__ void advance_window(const SelArgs& a, int64_t slot, int t0, int n, bool old, int c) {
+  const int w = a.taps - 1;
+  T* cs = (T*)a.conv + slot * w * a.C + c;
+  for (int j = 0; j < w; ++j) {
+    const int src = n + j;
+    T v = (T)0.f;
+    if (src >= w) v = ((const T*)a.cx)[(int64_t)(t0 + src - w) * a.ldcx + c];
+    else if (old) v = cs[(int64_t)src * a.C];
+    cs[(int64_t)j * a.C] = v;  // ascending: src > j, so nothing is overwritten before it is read
+  }
+}
+
+// V: channels a thread stages and writes
+template <typename T, int LP, int NPL, int V>
 __global__ void __launch_bounds__(NT) selective_scan_kernel(SelArgs a) {
   constexpr int CH = NT / LP, NW = LP * NPL;               // channels; numbers per channel as they are laid out in LDS
   constexpr int TT = LP == 4 || NW > 128 ? 16 : 32;        // tokens of a tile
-  constexpr int PER = TT * CH / NT;                        // (token, channel) pairs per thread
-  __shared__ __attribute__((aligned(16))) f32x2 sx[TT][CH];  // step, step * x
-  __shared__ __attribute__((aligned(16))) f32x2 sb[TT][NW];  // B, C
+  constexpr int CV = CH / V, PR = NT / CV;                 // threads across the channels, tokens they stage at a time
+  constexpr int PER = (TT + PR - 1) / PR;
+  constexpr int U = NPL >= 8 ? 2 : LP / 2 < 4 ? LP / 2 : 4;  // tokens whose operands are read ahead
+  constexpr int ROW = TT + 2;                              // tokens of an LDS row: an odd number of 16-byte pieces
+  constexpr int LANE = NPL * ROW + (NPL % 2 ? 0 : 2);      // a lane's rows of B and C: also odd, so that lanes use all banks
+  __shared__ __attribute__((aligned(16))) f32x2 sx[CH + 1][ROW];  // step, step * x (reads ahead run over the end)
+  __shared__ __attribute__((aligned(16))) f32x2 sb[LP * LANE + ROW];  // B, C
   __shared__ float sy[TT][CH];
   const int blocks = (a.C + CH - 1) / CH, id = xcd_remap(blockIdx.x, gridDim.x);
-  const int seq = id / blocks, c0 = id % blocks * CH, tid = threadIdx.x;
+  const int seq = a.list[id / blocks * a.stride], c0 = id % blocks * CH, tid = threadIdx.x;
   const int t0 = a.cu[seq], n = a.cu[seq + 1] - t0;
+  const int64_t slot = a.slots[seq];
   if (n <= 0) return;
   const bool old = a.start[seq] > 0;
   // ---- this lane's numbers
   const int g = tid % LP, cl = tid / LP, c = min(c0 + cl, a.C - 1), n0 = g * NPL;
   const bool mine = c0 + cl < a.C;
-  float* st = a.state + ((int64_t)a.slots[seq] * a.C + c) * a.NS + n0;
+  float* st = a.state + (slot * a.C + c) * a.NS + n0;
   float S[NPL], A[NPL];
 #pragma unroll
   for (int i = 0; i < NPL; ++i) {
-    const int k = min(n0 + i, a.N - 1);
+    A[i] = 0.f;
     S[i] = 0.f;
-    if (old) S[i] = st[k - n0];
-    A[i] = n0 + i < a.N ? -expf(a.a_log[(int64_t)c * a.N + k]) * LOG2E : 0.f;
-    if (n0 + i >= a.N) S[i] = 0.f;
+    if (n0 + i < a.N) {
+      A[i] = a.decay[(int64_t)c * a.N + n0 + i] * LOG2E;
+      if (old) S[i] = st[i];
+    }
   }
-  // ---- what this thread stages and writes: tokens (tid / CH) + PR j, channel tid % CH
-  constexpr int PR = NT / CH;
-  const int wc = c0 + tid % CH, wcc = min(wc, a.C - 1), wt = tid / CH;
-  const float bias = a.dt_bias[wcc], skip = a.skip[wcc];
-  T xr[PER], dr[PER], zr[PER];
+  // ---- what this thread stages and writes: tokens wt + PR j, channels wc .. wc + V - 1
+  const int wl = tid % CV * V, wt = tid / CV, wc = c0 + wl, wcc = min(wc, a.C - V);
+  const bool on = wc < a.C;
+  float bias[V], skip[V];
+#pragma unroll
+  for (int v = 0; v < V; ++v) {
+    bias[v] = a.dt_bias[wcc + v];
+    skip[v] = a.skip[wcc + v];
+  }
   constexpr int BPER = (TT * NW + NT - 1) / NT;
+  const T *xp = (const T*)a.x + (int64_t)t0 * a.C + wcc, *dp = (const T*)a.dt + (int64_t)t0 * a.C + wcc;
+  const T *zp = (const T*)a.z + t0 * a.ldz + wcc, *bp = (const T*)a.bc + t0 * a.ldbc;
+  int xo[PER], zo[PER], bo[BPER];  // places of a whole tile's operands
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    xo[j] = (wt + PR * j) * a.C;
+    zo[j] = (wt + PR * j) * (int)a.ldz;
+  }
+#pragma unroll
+  for (int j = 0; j < BPER; ++j) {
+    const int e = tid + NT * j;
+    bo[j] = min(e / NW, TT - 1) * (int)a.ldbc + min(e % NW, a.N - 1);
+  }
+  Few<T, V> xr[PER], dr[PER], zr[PER];
   T br[BPER], cr[BPER];
   auto fetch = [&](int k0) {
+    const int last = n - 1 - k0;
+    const T *x = xp + (int64_t)k0 * a.C, *d = dp + (int64_t)k0 * a.C, *z = zp + k0 * a.ldz, *b = bp + k0 * a.ldbc;
+    if (last >= PR * PER - 1 && last >= TT - 1) {
 #pragma unroll
-    for (int j = 0; j < PER; ++j) {
-      const int64_t t = t0 + min(k0 + wt + PR * j, n - 1);
-      xr[j] = ((const T*)a.x)[t * a.C + wcc];
-      dr[j] = ((const T*)a.dt)[t * a.C + wcc];
-      zr[j] = ((const T*)a.z)[t * a.ldz + wcc];
+      for (int j = 0; j < PER; ++j) {
+        xr[j].load(x + xo[j]);
+        dr[j].load(d + xo[j]);
+        zr[j].load(z + zo[j]);
+      }
+#pragma unroll
+      for (int j = 0; j < BPER; ++j) {
+        br[j] = b[bo[j]];
+        cr[j] = b[bo[j] + a.N];
+      }
+    } else {  // rows past the end repeat the last one
+#pragma unroll
+      for (int j = 0; j < PER; ++j) {
+        const int r = min(wt + PR * j, last);
+        xr[j].load(x + r * a.C);
+        dr[j].load(d + r * a.C);
+        zr[j].load(z + r * a.ldz);
+      }
+#pragma unroll
+      for (int j = 0; j < BPER; ++j) {
+        const int e = tid + NT * j;
+        const T* q = b + min(e / NW, last) * a.ldbc + min(e % NW, a.N - 1);
+        br[j] = q[0];
+        cr[j] = q[a.N];
+      }
     }
+  };
+  struct Ahead {  // two tokens at a time
+    f32x4 sd[U / 2], b[U / 2][NPL];
+  };
+  auto read = [&](Ahead& r, int t) {
 #pragma unroll
-    for (int j = 0; j < BPER; ++j) {
-      const int e = tid + NT * j;
-      const T* p = (const T*)a.bc + (int64_t)(t0 + min(k0 + min(e / NW, TT - 1), n - 1)) * a.ldbc + min(e % NW, a.N - 1);
-      br[j] = p[0];
-      cr[j] = p[a.N];
+    for (int u = 0; u < U / 2; ++u) {
+      r.sd[u] = *reinterpret_cast<const f32x4*>(&sx[cl][t + 2 * u]);
+#pragma unroll
+      for (int i = 0; i < NPL; ++i) r.b[u][i] = *reinterpret_cast<const f32x4*>(&sb[g * LANE + i * ROW + t + 2 * u]);
     }
   };
   fetch(0);
   for (int k0 = 0; k0 < n; k0 += TT) {
-    float xs[PER], zs[PER];
+    const int m = min(TT, n - k0);
+    float xs[PER][V], gate[PER][V];
 #pragma unroll
     for (int j = 0; j < PER; ++j) {
-      xs[j] = (float)xr[j];
-      zs[j] = (float)zr[j];
-      const float step = softplus_f((float)dr[j] + bias);
-      sx[wt + PR * j][tid % CH] = f32x2{step, step * xs[j]};
+      const int r = wt + PR * j;
+      f32x2 sd[V];
+#pragma unroll
+      for (int v = 0; v < V; ++v) {
+        xs[j][v] = (float)xr[j].v[v];
+        gate[j][v] = silu_f((float)zr[j].v[v]);
+        float step = softplus_f((float)dr[j].v[v] + bias[v]);
+        step = r < m ? step : 0.f;  // steps of zero leave the numbers as they are
+        sd[v] = f32x2{step, step * xs[j][v]};
+      }
+      if (TT % PR && r >= TT) continue;
+#pragma unroll
+      for (int v = 0; v < V; ++v) sx[wl + v][r] = sd[v];
     }
 #pragma unroll
     for (int j = 0; j < BPER; ++j) {
       const int e = tid + NT * j;
-      if (e < TT * NW) sb[e / NW][e % NW] = e % NW < a.N ? f32x2{(float)br[j], (float)cr[j]} : f32x2{0.f, 0.f};
+      const int i = e % NW;
+      if ((TT * NW) % NT == 0 || e < TT * NW)
+        sb[i / NPL * LANE + i % NPL * ROW + e / NW] = i < a.N ? f32x2{(float)br[j], (float)cr[j]} : f32x2{0.f, 0.f};
     }
     __syncthreads();
     if (k0 + TT < n) fetch(k0 + TT);
-    const int m = min(TT, n - k0);
-    auto token = [&](int t) {
-      const f32x2 sd = sx[t][cl];
-      float y = 0.f;
+    Ahead r[2];
+    read(r[0], 0);
+#pragma unroll 1
+    for (int t = 0; t < m; t += LP) {  // rounds of LP tokens
+      float p[LP];
 #pragma unroll
-      for (int i = 0; i < NPL; ++i) {
-        const f32x2 b = sb[t][n0 + i];
-        S[i] = fmaf(__builtin_amdgcn_exp2f(sd[0] * A[i]), S[i], sd[1] * b[0]);
-        y = fmaf(S[i], b[1], y);
-      }
-      return group_sum<LP>(y);
-    };
-    int t = 0;
-    for (; t + LP <= m; t += LP) {
-      float keep = 0.f;
+      for (int w = 0; w < LP / U; ++w) {
+        read(r[(w + 1) % 2], t + (w + 1) * U);
+        const Ahead& now = r[w % 2];
+        float e[U][NPL];
 #pragma unroll
-      for (int i = 0; i < LP; ++i) {
-        const float y = token(t + i);
-        keep = g == i ? y : keep;
+        for (int u = 0; u < U; ++u)
+#pragma unroll
+          for (int k = 0; k < NPL; ++k) e[u][k] = __builtin_amdgcn_exp2f(now.sd[u / 2][u % 2 * 2] * A[k]);
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+          const float dx = now.sd[u / 2][u % 2 * 2 + 1];
+          float sum = 0.f;
+#pragma unroll
+          for (int k = 0; k < NPL; ++k) {
+            S[k] = fmaf(e[u][k], S[k], dx * now.b[u / 2][k][u % 2 * 2]);
+            const float cn = now.b[u / 2][k][u % 2 * 2 + 1];
+            sum = k ? fmaf(S[k], cn, sum) : S[k] * cn;
+          }
+          p[w * U + u] = sum;
+        }
       }
-      sy[t + g][cl] = keep;
-    }
-    for (; t < m; ++t) {
-      const float y = token(t);
-      if (g == 0) sy[t][cl] = y;
+      sy[t + g][cl] = trade<LP>(p, g);
     }
     __syncthreads();
+    T* out = (T*)a.out + (int64_t)(t0 + k0) * a.C + wcc;
 #pragma unroll
     for (int j = 0; j < PER; ++j) {
       const int r = wt + PR * j;
-      const float y = fmaf(skip, xs[j], sy[r][tid % CH]);
-      if (r < m && wc < a.C) ((T*)a.out)[(int64_t)(t0 + k0 + r) * a.C + wc] = (T)(y * silu_f(zs[j]));
+      if (r >= m || !on) continue;
+      float y[V];
+#pragma unroll
+      for (int v = 0; v < V; ++v) y[v] = fmaf(skip[v], xs[j][v], sy[r][wl + v]) * gate[j][v];
+      store_few<T, V>(out + xo[j], y);
     }
   }
   if (mine) {
@@ -160,21 +279,77 @@ __global__ void __launch_bounds__(NT) selective_scan_kernel(SelArgs a) {
     for (int i = 0; i < NPL; ++i)
       if (n0 + i < a.N) st[i] = S[i];
   }
-  // ---- convolution windows: the last taps - 1 of [old window | the portion's inputs]
-  if (a.conv && tid < CH && c0 + tid < a.C) {
-    const int ch = c0 + tid, w = a.taps - 1;
-    T* cs = (T*)a.conv + (int64_t)a.slots[seq] * w * a.C + ch;
-    for (int j = 0; j < w; ++j) {
-      const int src = n + j;
-      T v = (T)0.f;
-      if (src >= w) v = ((const T*)a.cx)[(int64_t)(t0 + src - w) * a.ldcx + ch];
-      else if (old) v = cs[(int64_t)src * a.C];
-      cs[(int64_t)j * a.C] = v;  // ascending: src > j, so nothing is overwritten before it is read
-    }
-  }
+  if (a.conv && tid < CH && c0 + tid < a.C) advance_window<T>(a, slot, t0, n, old, c0 + tid);
 }
 
-template <typename T, int LP>
+// Four numbers per lane, LP lanes per channel. VEC: N is 4 LP, and B and C lie in 4-element pieces
+template <typename T, int LP, bool VEC>
+__global__ void __launch_bounds__(NT) selective_step_kernel(SelArgs a) {
+  typedef T T4 __attribute__((ext_vector_type(4)));
+  constexpr int CH = NT / LP;
+  const int seq = a.list[blockIdx.y * a.stride], tid = threadIdx.x, g = tid % LP;
+  const int c = min((int)blockIdx.x * CH + tid / LP, a.C - 1), n0 = 4 * g;
+  const bool mine = (int)blockIdx.x * CH + tid / LP < a.C;
+  const int t0 = a.cu[seq], n = a.cu[seq + 1] - t0;
+  const int64_t slot = a.slots[seq];
+  const bool old = a.start[seq] > 0;
+  float* st = a.state + (slot * a.C + c) * a.NS + n0;
+  f32x4 S = {0.f, 0.f, 0.f, 0.f}, A = S;
+  if constexpr (VEC) {
+    A = *reinterpret_cast<const f32x4*>(a.decay + (int64_t)c * a.N + n0);
+    if (old) S = *reinterpret_cast<const f32x4*>(st);
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (n0 + i < a.N) {
+        A[i] = a.decay[(int64_t)c * a.N + n0 + i];
+        if (old) S[i] = st[i];
+      }
+  }
+  const float bias = a.dt_bias[c], skip = a.skip[c];
+  A *= LOG2E;
+  for (int t = t0; t < t0 + n; ++t) {
+    const float x = (float)((const T*)a.x)[(int64_t)t * a.C + c], z = (float)((const T*)a.z)[t * a.ldz + c];
+    const float step = softplus_f((float)((const T*)a.dt)[(int64_t)t * a.C + c] + bias), dx = step * x;
+    const T* b = (const T*)a.bc + t * a.ldbc + n0;
+    f32x4 B = {0.f, 0.f, 0.f, 0.f}, C = B;
+    if constexpr (VEC) {
+      const T4 b4 = *reinterpret_cast<const T4*>(b), c4 = *reinterpret_cast<const T4*>(b + a.N);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        B[i] = (float)b4[i];
+        C[i] = (float)c4[i];
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (n0 + i < a.N) {
+          B[i] = (float)b[i];
+          C[i] = (float)b[a.N + i];
+        }
+    }
+    float y = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      S[i] = fmaf(__builtin_amdgcn_exp2f(step * A[i]), S[i], dx * B[i]);
+      y = fmaf(S[i], C[i], y);
+    }
+#pragma unroll
+    for (int o = LP / 2; o > 0; o >>= 1) y += __shfl_xor(y, o, 64);
+    if (g == 0 && mine) ((T*)a.out)[(int64_t)t * a.C + c] = (T)(fmaf(skip, x, y) * silu_f(z));
+  }
+  if (!mine || n <= 0) return;
+  if constexpr (VEC) {
+    *reinterpret_cast<f32x4*>(st) = S;
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (n0 + i < a.N) st[i] = S[i];
+  }
+  if (a.conv && g == 0) advance_window<T>(a, slot, t0, n, old, c);
+}
+
+template <typename T, int LP, int V>
 int launch(const SelArgs& a, hipStream_t st) {
   constexpr int CH = NT / LP;
   const int64_t grid = (int64_t)((a.C + CH - 1) / CH) * a.seqs;
@@ -182,15 +357,16 @@ int launch(const SelArgs& a, hipStream_t st) {
   const int need = (a.N + LP - 1) / LP;
 #define GO(NPL)                                                                                                    \
   {                                                                                                                \
-    hipLaunchKernelGGL((selective_scan_kernel<T, LP, NPL>), dim3((unsigned)grid), dim3(NT), 0, st, a);             \
+    hipLaunchKernelGGL((selective_scan_kernel<T, LP, NPL, V>), dim3((unsigned)grid), dim3(NT), 0, st, a);          \
     DS_CHECK_LAUNCH();                                                                                             \
     return 0;                                                                                                      \
   }
   if (need <= 1) GO(1)
   if (need <= 2) GO(2)
-  if (need <= 3) GO(3)
   if (need <= 4) GO(4)
-  if (need <= 6) GO(6)
+  if constexpr (LP < 16) {
+    if (need <= 6) GO(6)
+  }
   if (need <= 8) GO(8)
   if constexpr (LP == 16) {
     if (need <= 16) GO(16)
@@ -199,13 +375,31 @@ int launch(const SelArgs& a, hipStream_t st) {
   return (int)hipErrorInvalidValue;
 }
 
+template <typename T, int V>
+int scan(const SelArgs& a, hipStream_t st) {
+  // as few lanes per channel as give the chip's 1024 SIMDs work (a second wave each is worth more than fewer lanes)
+  const int64_t waves = (int64_t)a.C * a.seqs / 16;  // with 4
+  if (a.N <= 32 && waves >= 1536) return launch<T, 4, V>(a, st);
+  if (a.N <= 64 && waves >= 512) return launch<T, 8, V>(a, st);
+  return launch<T, 16, V>(a, st);
+}
+
 template <typename T>
-int choose(const SelArgs& a, bool decode, hipStream_t st) {
-  // waves with 4 lanes per channel; as few lanes as cover the chip's 1024 SIMDs
-  const int64_t waves = (int64_t)a.C * a.seqs / 16;
-  if (a.N <= 32 && (decode || waves >= 1024)) return launch<T, 4>(a, st);
-  if (a.N <= 64 && (decode || waves >= 512)) return launch<T, 8>(a, st);
-  return launch<T, 16>(a, st);
+int step(const SelArgs& a, bool aligned, hipStream_t st) {
+  const int need = (a.N + 3) / 4;
+#define GO(LP)                                                                                                         \
+  if (need <= LP) {                                                                                                    \
+    const dim3 grid((a.C + NT / LP - 1) / (NT / LP), a.seqs);                                                          \
+    if (aligned && a.N == 4 * LP)                                                                                      \
+      hipLaunchKernelGGL((selective_step_kernel<T, LP, true>), grid, dim3(NT), 0, st, a);                              \
+    else                                                                                                               \
+      hipLaunchKernelGGL((selective_step_kernel<T, LP, false>), grid, dim3(NT), 0, st, a);                             \
+    DS_CHECK_LAUNCH();                                                                                                 \
+    return 0;                                                                                                          \
+  }
+  GO(1) GO(2) GO(4) GO(8) GO(16) GO(32) GO(64)
+#undef GO
+  return (int)hipErrorInvalidValue;
 }
 
 }  // namespace
@@ -213,17 +407,31 @@ int choose(const SelArgs& a, bool decode, hipStream_t st) {
 // Numbers per channel a kernel instance holds
 extern "C" int ds_selective_scan_max() { return 256; }
 
-// x, dt [T, C] and, ldbc / ldz / ldcx elements from row to row, bc [T, B | C (N each)], z [T, C], cx [T, C]; state
-// [slots, C, NS]; conv [slots, taps - 1, C] or null. `longest`: most new tokens of a sequence
+// Sequences list[0], list[stride], ... (`seqs` of them). x, dt [T, C] and, ldbc / ldz / ldcx elements from row to row,
+// bc [T, B | C (N each)], z [T, C], cx [T, C]; state [slots, C, NS]; conv [slots, taps - 1, C] or null. `steps`: few tokens each
 extern "C" int ds_selective_scan(const void* x, const void* dt, const void* bc, int64_t ldbc, const void* z, int64_t ldz,
-                                 const float* dt_bias, const float* a_log, const float* skip, float* state, const void* cx,
-                                 int64_t ldcx, void* conv, const int* cu, const int* start, const int* slots, void* out, int seqs,
-                                 int longest, int C, int N, int NS, int taps, int dtype, hipStream_t st) {
+                                 const float* dt_bias, const float* decay, const float* skip, float* state, const void* cx,
+                                 int64_t ldcx, void* conv, const int* list, int seqs, int stride, const int* cu, const int* start,
+                                 const int* slots, void* out, int steps, int C, int N, int NS, int taps, int dtype,
+                                 hipStream_t st) {
   if (seqs <= 0) return 0;
-  if (C <= 0 || N <= 0 || N > ds_selective_scan_max() || NS < N || taps < 1 || (conv && (taps < 2 || !cx)))
+  if (C <= 0 || N <= 0 || N > ds_selective_scan_max() || NS < N || taps < 1 || (conv && (taps < 2 || !cx)) || stride <= 0 ||
+      seqs > 65535)
     return (int)hipErrorInvalidValue;
-  const SelArgs a{x, dt, bc, z, cx, ldbc, ldz, ldcx, dt_bias, a_log, skip, state, conv, cu, start, slots, out, C, N, NS, taps, seqs};
-  if (dtype == DS_F32) return choose<float>(a, longest <= 4, st);
-  if (dtype == DS_BF16) return choose<bf16>(a, longest <= 4, st);
+  // (places within a tile are 32-bit)
+  if (((int64_t)C + ldz + ldbc) * 64 > INT32_MAX) return (int)hipErrorInvalidValue;
+  const SelArgs a{x,    dt,   bc,   z,   cx,    ldbc,  ldz, ldcx, dt_bias, decay, skip, state,
+                  conv, list, cu, start, slots, out, C,   N,    NS,      taps,  seqs, stride};
+  const int el = dtype == DS_F32 ? 4 : 2;
+  if (steps) {
+    const bool aligned = NS % 4 == 0 && ldbc % 4 == 0 && N % 4 == 0 && ((uintptr_t)bc & (4 * el - 1)) == 0 &&
+                         (((uintptr_t)state | (uintptr_t)decay) & 15) == 0;
+    if (dtype == DS_F32) return step<float>(a, aligned, st);
+    if (dtype == DS_BF16) return step<bf16>(a, aligned, st);
+    return (int)hipErrorInvalidValue;
+  }
+  const bool two = C % 2 == 0 && ldz % 2 == 0 && (((uintptr_t)x | (uintptr_t)dt | (uintptr_t)z) & 3) == 0;
+  if (dtype == DS_F32) return scan<float, 1>(a, st);
+  if (dtype == DS_BF16) return two ? scan<bf16, 2>(a, st) : scan<bf16, 1>(a, st);
   return (int)hipErrorInvalidValue;
 }

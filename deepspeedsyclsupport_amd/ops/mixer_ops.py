@@ -178,10 +178,16 @@ def causal_conv(x, w, b, conv_state, meta):
     return f(x, w, b, conv_state, *((meta.seq_ids, ) if use_native(x) else ()), meta.cu_q, meta.start_pos, meta.slots)
 
 
-def selective_scan(x, dt, bc, z, dt_bias, a_log, skip, state, conv_x, conv_state, meta):
-    """A decay per channel and state: with step = softplus(dt + dt_bias) and A = -exp(a_log) [C, N],
-    S[c, n] <- exp(step_c A[c, n]) S[c, n] + step_c x_c B_n, y_c = sum_n S[c, n] C_n + skip_c x_c, out = y silu(z) [T, C]. bc
+def selective_scan(x, dt, bc, z, dt_bias, decay, skip, state, conv_x, conv_state, meta):
+    """A decay per channel and state: with step = softplus(dt + dt_bias) and decay [C, N] < 0,
+    S[c, n] <- exp(step_c decay[c, n]) S[c, n] + step_c x_c B_n, y_c = sum_n S[c, n] C_n + skip_c x_c, out = y silu(z) [T, C]. bc
     [T, B | C], z [T, C]: columns of wider matrices. state [slots, C, N rounded up to 4] fp32 and conv_state, the last inputs
-    of the convolution conv_x [T, C], advance."""
-    f = (selective_ops() if use_native(x) else reference).selective_scan
-    return f(x, dt, bc, z, dt_bias, a_log, skip, state, conv_x, conv_state, meta.cu_q, meta.start_pos, meta.slots)
+    of the convolution conv_x [T, C], advance.
+
+    Portions up to `RaggedMeta.STEP_TOKENS` stream the state token by token, longer ones keep it in registers."""
+    ops, out = selective_ops() if use_native(x) else reference, torch.empty_like(x)
+    args = (x, dt, bc, z, dt_bias, decay, skip, state, conv_x, conv_state)
+    for seqs, steps in ((meta.seq_list, True), (meta.chunk_seqs, False)):
+        if seqs.numel():
+            ops.selective_scan(*args, seqs, meta.cu_q, meta.start_pos, meta.slots, steps, out)
+    return out

@@ -492,19 +492,17 @@ def causal_conv(x, w, b, conv_state, cu, start, slots):
     return F.silu(y).to(x.dtype)
 
 
-def selective_scan(x, dt, bc, z, dt_bias, a_log, skip, state, conv_x, conv_state, cu, start, slots):
-    T, C = x.shape
-    N = a_log.shape[1]
-    out, step, A = torch.empty_like(x), F.softplus(dt.float() + dt_bias, threshold=60), -a_log.exp()
-    for i in range(start.numel()):
+def selective_scan(x, dt, bc, z, dt_bias, decay, skip, state, conv_x, conv_state, seqs, cu, start, slots, steps, out):
+    C, N = decay.shape
+    step = F.softplus(dt.float() + dt_bias, threshold=60)
+    for i in (seqs if steps else seqs[:, 0]).tolist():
         p, q, slot, old = int(cu[i]), int(cu[i + 1]), int(slots[i]), int(start[i]) > 0
         S = state[slot, :, :N].clone() if old else torch.zeros(C, N)
         for t in range(p, q):
             xt, B, Ct = x[t].float(), bc[t, :N].float(), bc[t, N:2 * N].float()
-            S = (step[t][:, None] * A).exp() * S + (step[t] * xt)[:, None] * B
+            S = (step[t][:, None] * decay).exp() * S + (step[t] * xt)[:, None] * B
             out[t] = (((S * Ct).sum(-1) + skip * xt) * F.silu(z[t].float())).to(out.dtype)
         state[slot, :, :N] = S
         if conv_state is not None and conv_state.shape[1]:
             before = conv_state[slot] if old else torch.zeros_like(conv_state[slot])
             conv_state[slot] = torch.cat([before, conv_x[p:q]])[-conv_state.shape[1]:].clone()
-    return out
