@@ -70,11 +70,11 @@ def rotate(x, rot, first=0):
     position * frequency_j and grow by the factor."""
     freq, grow = yarn(rot)
     out = x.clone()
-    for i in range(x.shape[0]):
-        for j, f in enumerate(freq):
-            c, s = grow * math.cos((first + i) * f), grow * math.sin((first + i) * f)
-            u, v = x[i, 2 * j], x[i, 2 * j + 1]
-            out[i, 2 * j], out[i, 2 * j + 1] = u * c - v * s, v * c + u * s
+    for j, f in enumerate(freq):
+        a = torch.arange(first, first + x.shape[0], dtype=torch.float64) * f
+        c, s = (grow * torch.cos(a)).to(x.dtype), (grow * torch.sin(a)).to(x.dtype)
+        u, v = x[:, 2 * j], x[:, 2 * j + 1]
+        out[:, 2 * j], out[:, 2 * j + 1] = u * c - v * s, v * c + u * s
     return out
 
 
@@ -206,3 +206,140 @@ def forward(cfg, weights, tokens, cast=torch.float64, trace=None):
         if trace is not None:
             trace.append(x)
     return project(rms(x, eps) * w["final.norm"], w["head"])
+
+
+# ------------------------------------------------------------------------------------------------ test models
+CODE = 8   # columns of the residual that `decisive` models keep for the router
+
+
+def random_model(cfg, seed=0, dtype=torch.bfloat16, decisive=False):
+    """Random weights for a config. `decisive`: the last `CODE` columns of the residual belong to the router alone (no sublayer
+    writes them, the embedding does), with values drawn anew until no token comes near a tie in any layer. Rounding then cannot
+    change an expert, so that whole models compare in 16 bits."""
+    g = torch.Generator().manual_seed(seed)
+    W, w = cfg["width"], {}
+
+    def put(name, shape, std=None, mean=0.0):
+        std = std if std is not None else 1 / math.sqrt(shape[-1])
+        w[name] = (torch.randn(shape, generator=g) * std + mean).to(dtype)
+
+    put("embed", (cfg["vocab"], W), 1.0)
+    put("head", (cfg["vocab"], W))
+    put("final.norm", (W, ), 0.1, 1.0)
+    sd = cfg["token_side"]["dim"]
+    put("side.embed", (cfg["vocab"], sd * len(cfg["layers"])), 1.0)
+    for i, layer in enumerate(cfg["layers"]):
+        p, mx, ml = f"l{i}.", layer["mixer"], layer.get("mlp")
+        for q in "12" if ml else "1":
+            put(p + f"norm{q}", (W, ), 0.2, 0.9)
+            put(p + f"norm{q}b", (W, ), 0.2, 0.6)
+            put(p + f"rg{q}", (W, W), 1.5 / math.sqrt(W))
+            put(p + f"rg{q}.b", (W, ), 0.7, 0.3)
+        put(p + "side.gate", (sd, W))
+        put(p + "side.proj", (W, sd))
+        put(p + "side.norm", (W, ), 0.1, 0.4)
+        m = p + "mix."
+        if layer["type"] == "mamba1":
+            C, N, R = mx["inner"], mx["state"], mx["dt_rank"]
+            put(m + "in", (2 * C, W))
+            put(m + "conv", (C, mx["conv"]), 0.5)
+            put(m + "conv.b", (C, ), 0.2)
+            put(m + "x", (R + 2 * N, C), 1.5 / math.sqrt(C))
+            put(m + "dt", (C, R), 0.7 / math.sqrt(R))
+            put(m + "dt.b", (C, ), 0.7, -2.0)
+            put(m + "A_log", (C, N), 0.8, -0.3)
+            put(m + "D", (C, ), 0.3, 0.6)
+            put(m + "o", (W, C))
+        elif layer["type"] == "attention":
+            H, G, d, e = mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
+            for n, rows in (("q", H * d), ("k", G * d), ("v", G * e), ("g", H)):
+                put(m + n, (rows, W))
+            put(m + "o", (W, H * e))
+        else:
+            H, d, r, e, R = mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"], mx["kv_rank"]
+            put(m + "q", (H * (d + r), W))
+            put(m + "dkv", (R + r, W))
+            put(m + "dkv.norm", (R, ), 0.2, 1.0)
+            put(m + "uk", (H * d, R))
+            put(m + "uv", (H * e, R))
+            put(m + "o", (W, H * e))
+        if ml and ml["kind"] == "dense":
+            for n, shape in (("gate", (ml["ff"], W)), ("up", (ml["ff"], W)), ("down", (W, ml["ff"]))):
+                put(p + "mlp." + n, shape)
+        elif ml:
+            put(p + "mlp.router", (ml["router"]["experts"], W), 1.5 / math.sqrt(W))
+            for e in [f"e{j}" for j in range(ml["router"]["experts"])] + ["shared"]:
+                F = (ml["shared"] if e == "shared" else ml["expert"])["ff"]
+                put(p + f"mlp.{e}.up", (F, W))
+                put(p + f"mlp.{e}.down", (W, F))
+    if decisive:
+        _decide(cfg, w, g)
+    return w
+
+
+def _decide(cfg, w, g):
+    routed = [(f"l{i}.", la["mlp"]["router"]) for i, la in enumerate(cfg["layers"]) if (la.get("mlp") or {}).get("kind") == "moe"]
+    for name in w:
+        if name.endswith(("norm1b", "norm2b", "side.norm")):
+            w[name][-CODE:] = 0
+    for p, _ in routed:
+        w[p + "mlp.router"] *= 6
+        w[p + "mlp.router"][:, :-CODE] = 0
+    todo = torch.arange(cfg["vocab"])
+    for _ in range(2000):
+        if not len(todo):
+            return
+        w["embed"][todo, -CODE:] = torch.randn(len(todo), CODE, generator=g).to(w["embed"].dtype)
+        c = w["embed"][todo, -CODE:].double()
+        near = torch.zeros(len(todo), dtype=torch.bool)
+        for p, r in routed:
+            count, keep, top = r["groups"]["count"], r["groups"]["keep"], r["top"]
+            full = (c * w[p + "norm2"][-CODE:].double()) @ w[p + "mlp.router"][:, -CODE:].double().t()
+            for shrink in (1.0, 0.6, 0.35, 0.2):   # by how much the norm may have scaled it
+                z = full * shrink
+                unit, n = z.std(-1) * 0.04, len(z)
+                s = sigmoid(z).view(n, count, -1)
+                worth = s.sort(-1, descending=True).values[..., :2].sum(-1)
+                order = worth.sort(-1, descending=True).values
+                if keep < count:
+                    near |= order[:, keep - 1] - order[:, keep] < 0.01
+                allowed = z.view(n, count, -1).masked_fill((worth < order[:, keep - 1:keep])[..., None], -math.inf).view(n, -1)
+                allowed = allowed.sort(-1, descending=True).values
+                if top < z.shape[1]:
+                    near |= allowed[:, top - 1] - allowed[:, top] < unit
+        todo = todo[near]
+    raise AssertionError("no routing without near ties")
+
+
+def rotation(dims, base=1000.0, factor=2.0, original=40, fast=4.0, slow=0.5):
+    return {"base": base, "dims": dims, "scaling": {"factor": factor, "fast": fast, "original": original, "slow": slow}}
+
+
+def mamba_layer(inner=48, state=12, dt_rank=6, conv=4, mlp=None):
+    return {"type": "mamba1", "mixer": {"conv": conv, "dt_rank": dt_rank, "inner": inner, "state": state}, "mlp": mlp}
+
+
+def attention_layer(heads=4, kv_heads=2, dim=16, vdim=24, size=40, rot=None, scale=None, mlp=None):
+    return {"type": "attention", "mixer": {"dim": dim, "heads": heads, "kv_heads": kv_heads, "mask": {"size": size},
+                                           "rot": rot or rotation(dim // 4 * 2), "scale": scale or 1.5 * dim**-0.5,
+                                           "vdim": vdim}, "mlp": mlp}
+
+
+def latent_layer(heads=3, dim=16, rot_dim=8, vdim=24, kv_rank=40, size=40, rot=None, scale=None, mlp=None):
+    return {"type": "latent_attention", "mixer": {"dim": dim, "heads": heads, "kv_rank": kv_rank, "mask": {"size": size},
+                                                  "rot": rot or rotation(rot_dim, 300.0, 3.0), "rot_dim": rot_dim,
+                                                  "scale": scale or 1.5 * (dim + rot_dim)**-0.5, "vdim": vdim}, "mlp": mlp}
+
+
+def dense(ff=40):
+    return {"ff": ff, "kind": "dense"}
+
+
+def moe(experts=6, top=2, count=3, keep=2, ff=32, shared=24, scale=1.7):
+    return {"expert": {"ff": ff}, "kind": "moe", "router": {"experts": experts, "groups": {"count": count, "keep": keep},
+                                                            "scale": scale, "top": top}, "shared": {"ff": shared}}
+
+
+def config(layers, vocab=97, width=64, side=12, eps=1e-5):
+    return {"architecture": "Nigilorn", "layers": layers, "norm": {"eps": eps}, "token_side": {"dim": side}, "vocab": vocab,
+            "width": width}
