@@ -95,8 +95,10 @@ def build(spec, device, blocks):
     torch.manual_seed(0)
     model = model_class(spec)(spec, dtype=torch.bfloat16, device=device)
     with torch.no_grad():
-        for p in model.parameters():
-            if p.dim() >= 2 and p.dtype == torch.bfloat16:
+        for name, p in model.named_parameters():
+            if name.endswith(".decay"):
+                p.copy_(-p.normal_(0, 0.5).exp())   # rates of a selective state space
+            elif p.dim() >= 2 and p.dtype == torch.bfloat16:
                 p.normal_(0, 0.02)
             elif p.dim() == 2 and p.shape[0] == p.shape[1]:
                 p.copy_(torch.eye(p.shape[0]))      # stream mixing
@@ -137,7 +139,9 @@ def measure(spec, device, prompts, batches, context, iters, log):
         out["prefill_tok_s"][f"{n}x{length}"] = round(n * length / t, 1)
         log(f"[bench] {spec.arch} w{spec.hidden_size} prefill {n}x{length}: {t * 1e3:.2f} ms")
     for u in range(max(batches)):
-        eng.put([u], [torch.randint(0, spec.vocab_size, (context, ), generator=g)])
+        logits = eng.put([u], [torch.randint(0, spec.vocab_size, (context, ), generator=g)])
+    if not torch.isfinite(logits.float()).all():
+        raise RuntimeError(f"{spec.arch}: logits are not finite")
     for b in batches:
         one = [torch.tensor([u % spec.vocab_size]) for u in range(b)]
         t = timed(lambda: eng.put(list(range(b)), one), iters * 2)

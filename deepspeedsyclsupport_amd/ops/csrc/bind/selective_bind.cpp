@@ -3,7 +3,7 @@
 #include "bind_util.h"
 
 extern "C" {
-int ds_causal_conv(const void*, int64_t, const float*, const float*, const void*, const int*, const int*, const int*, const int*,
+int ds_causal_conv(const void*, int64_t, const float*, const float*, void*, const int*, const int*, const int*, const int*,
                    void*, int, int, int, int, hipStream_t);
 int ds_selective_scan_max();
 int ds_selective_scan(const void*, const void*, const void*, int64_t, const void*, int64_t, const float*, const float*,
@@ -18,7 +18,8 @@ void window_ok(const OptT& cs, int64_t taps, int64_t C, const Tensor& x) {
               cs->size(2) == C && cs->scalar_type() == x.scalar_type()), "conv_state [slots, taps - 1, C]");
 }
 
-// x [T, C] (it may be columns of a wider matrix), w [C, taps], b [C] -> silu(conv(x) + b) [T, C]
+// x [T, C] (it may be columns of a wider matrix), w [C, taps], b [C] -> silu(conv(x) + b) [T, C]; the windows of portions of one
+// token move on
 Tensor causal_conv(Tensor x, Tensor w, Tensor b, OptT conv_state, Tensor seq_ids, Tensor cu, Tensor start, Tensor slots) {
   need_rows(x, "x");
   TORCH_CHECK(w.dim() == 2 && w.size(0) == x.size(1) && w.size(1) >= 1, "causal_conv: w [C, taps]");
@@ -32,7 +33,8 @@ Tensor causal_conv(Tensor x, Tensor w, Tensor b, OptT conv_state, Tensor seq_ids
 }
 
 // Sequences of `list` ([n], or the first column of [n, 2]): x, dt [T, C], bc [T, 2 N], z [T, C] -> their rows of out [T, C]; their
-// slots of state [slots, C, >= N] and conv_state (last rows of conv_x) advance. steps: few new tokens each
+// slots of state [slots, C, >= N] and, unless causal_conv has moved it on, conv_state (last rows of conv_x) advance. steps: few
+// new tokens each
 void selective_scan(Tensor x, Tensor dt, Tensor bc, Tensor z, Tensor dt_bias, Tensor decay, Tensor skip, Tensor state,
                     Tensor conv_x, OptT conv_state, Tensor list, Tensor cu, Tensor start, Tensor slots, bool steps, Tensor out) {
   need(x, "x"); need(dt, "dt"); need_rows(bc, "bc"); need_rows(z, "z"); need_rows(conv_x, "conv_x"); need(state, "state");

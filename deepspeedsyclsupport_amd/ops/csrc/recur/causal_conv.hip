@@ -1,6 +1,7 @@
 // Short causal convolution per channel with bias and silu, over a ragged batch, CDNA4 (gfx950). Inputs may be columns of a wider
-// matrix; those before a portion come from the sequence's slot of convolution windows, which stays as it is (the recurrence
-// behind the convolution moves it on). A sequence whose portion starts at position 0 has zeros before it.
+// matrix; those before a portion come from the sequence's slot of convolution windows. A sequence whose portion starts at position
+// 0 has zeros before it. The window of a portion of one token moves on here, where it is in registers; other portions are shared
+// by several waves, and the recurrence behind the convolution moves theirs on.
 //
 // HBM-bound: a lane has up to 8 channels of a tile of consecutive tokens, all its inputs in flight at once.
 #include "ds_hip.h"
@@ -23,7 +24,7 @@ struct ConvArgs {
   int64_t ld;
   const float* w;      // [C, taps], last column: the current token
   const float* b;      // [C]
-  const void* state;   // [slots, taps - 1, C]
+  void* state;         // [slots, taps - 1, C]
   const int *seq_ids, *cu, *start, *slots;
   void* out;           // [T, C]
   int tokens, C, taps;
@@ -45,7 +46,9 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
   const int t_hi = min((int)tl + TILE, a.tokens);
   for (int ta = (int)tl; ta < t_hi;) {  // runs of tokens of one sequence
     const int seq = a.seq_ids[ta], first = a.cu[seq], tb = min(t_hi, a.cu[seq + 1]), n = tb - ta, j0 = ta - first;
-    const T* old = a.start[seq] == 0 || taps == 1 ? nullptr : (const T*)a.state + (int64_t)a.slots[seq] * (taps - 1) * a.C + c;
+    T* const window = taps == 1 ? nullptr : (T*)a.state + (int64_t)a.slots[seq] * (taps - 1) * a.C + c;
+    const T* old = a.start[seq] == 0 ? nullptr : window;
+    const bool lone = window && a.cu[seq + 1] - first == 1;
     // the input at place j of the portion (negative: before it); zero tells that there is none
     auto input = [&](int j, float (&v)[V]) {
       const bool none = j < 0 && !old;
@@ -71,6 +74,10 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
           for (int i = 0; i < TAPS; ++i) acc = fmaf(cw[e][i], in[t + i][e], acc);
           y[t][e] = acc;
         }
+      if (lone) {
+#pragma unroll
+        for (int i = 1; i < TAPS; ++i) stv<T, V>(window + (int64_t)(i - 1) * a.C, in[i]);
+      }
     } else {
 #pragma unroll
       for (int t = 0; t < TILE; ++t)
@@ -83,6 +90,13 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
           input(j0 + min(t, n - 1) - (taps - 1) + i, v);
 #pragma unroll
           for (int e = 0; e < V; ++e) y[t][e] = fmaf(w[e * taps + i], v[e], y[t][e]);
+        }
+      }
+      if (lone) {  // (ascending: a row is read before it is written)
+        for (int i = 1; i < taps; ++i) {
+          float v[V];
+          input(i - (taps - 1), v);
+          stv<T, V>(window + (int64_t)(i - 1) * a.C, v);
         }
       }
     }
@@ -120,7 +134,7 @@ int conv(const ConvArgs& a, bool vec, hipStream_t st) {
 }  // namespace
 
 // x [tokens, C], rows ld elements apart -> out [tokens, C] = silu(conv(x) + b); state [slots, taps - 1, C] (unused with one tap)
-extern "C" int ds_causal_conv(const void* x, int64_t ld, const float* w, const float* b, const void* state, const int* seq_ids,
+extern "C" int ds_causal_conv(const void* x, int64_t ld, const float* w, const float* b, void* state, const int* seq_ids,
                               const int* cu, const int* start, const int* slots, void* out, int tokens, int C, int taps,
                               int dtype, hipStream_t st) {
   if (tokens <= 0) return 0;

@@ -16,7 +16,7 @@
 //      write: y from LDS, skip and gate applied, in whole rows.
 //  * step (decodes, short portions): four numbers per lane, nothing but registers, so that many waves stream the states.
 //
-// At the end the channels' convolution windows move on (the convolution, which reads the old ones, has finished by then). A
+// The channels' convolution windows move on as well, but for portions of one token, where the convolution has done it. A
 // sequence whose portion starts at position 0 starts from zero: slots need no clearing between owners.
 #include "ds_hip.h"
 
@@ -92,14 +92,24 @@ __device__ __forceinline__ float trade(float (&p)[LP], int g) {
 // A channel's convolution window: the last taps - 1 of [old window | the portion's inputs]
 template <typename T>
 __device__ __forceinline__ void advance_window(const SelArgs& a, int64_t slot, int t0, int n, bool old, int c) {
+  constexpr int FEW = 4;
   const int w = a.taps - 1;
   T* cs = (T*)a.conv + slot * w * a.C + c;
-  for (int j = 0; j < w; ++j) {
+  auto at = [&](int j) {  // place j of the new window
     const int src = n + j;
-    T v = (T)0.f;
-    if (src >= w) v = ((const T*)a.cx)[(int64_t)(t0 + src - w) * a.ldcx + c];
-    else if (old) v = cs[(int64_t)src * a.C];
-    cs[(int64_t)j * a.C] = v;  // ascending: src > j, so nothing is overwritten before it is read
+    if (src >= w) return ((const T*)a.cx)[(int64_t)(t0 + src - w) * a.ldcx + c];
+    return old ? cs[(int64_t)src * a.C] : (T)0.f;
+  };
+  if (w <= FEW) {  // all loads, then all stores
+    T v[FEW];
+#pragma unroll
+    for (int j = 0; j < FEW; ++j)
+      if (j < w) v[j] = at(j);
+#pragma unroll
+    for (int j = 0; j < FEW; ++j)
+      if (j < w) cs[(int64_t)j * a.C] = v[j];
+  } else {
+    for (int j = 0; j < w; ++j) cs[(int64_t)j * a.C] = at(j);  // ascending: src > j, so nothing is overwritten before it is read
   }
 }
 
@@ -279,74 +289,107 @@ __global__ void __launch_bounds__(NT) selective_scan_kernel(SelArgs a) {
     for (int i = 0; i < NPL; ++i)
       if (n0 + i < a.N) st[i] = S[i];
   }
-  if (a.conv && tid < CH && c0 + tid < a.C) advance_window<T>(a, slot, t0, n, old, c0 + tid);
+  if (a.conv && n > 1 && tid < CH && c0 + tid < a.C) advance_window<T>(a, slot, t0, n, old, c0 + tid);
 }
 
-// Four numbers per lane, LP lanes per channel. VEC: N is 4 LP, and B and C lie in 4-element pieces
-template <typename T, int LP, bool VEC>
+// Four numbers per lane, LP lanes per channel, R sequences at a time. VEC: N is 4 LP, and B and C lie in 4-element pieces
+template <typename T, int LP, bool VEC, int R>
 __global__ void __launch_bounds__(NT) selective_step_kernel(SelArgs a) {
   typedef T T4 __attribute__((ext_vector_type(4)));
   constexpr int CH = NT / LP;
-  const int seq = a.list[blockIdx.y * a.stride], tid = threadIdx.x, g = tid % LP;
-  const int c = min((int)blockIdx.x * CH + tid / LP, a.C - 1), n0 = 4 * g;
-  const bool mine = (int)blockIdx.x * CH + tid / LP < a.C;
-  const int t0 = a.cu[seq], n = a.cu[seq + 1] - t0;
-  const int64_t slot = a.slots[seq];
-  const bool old = a.start[seq] > 0;
-  float* st = a.state + (slot * a.C + c) * a.NS + n0;
-  f32x4 S = {0.f, 0.f, 0.f, 0.f}, A = S;
-  if constexpr (VEC) {
-    A = *reinterpret_cast<const f32x4*>(a.decay + (int64_t)c * a.N + n0);
-    if (old) S = *reinterpret_cast<const f32x4*>(st);
-  } else {
+  const int tid = threadIdx.x, g = tid % LP, n0 = 4 * g, cw = (int)blockIdx.x * CH + tid / LP, c = min(cw, a.C - 1);
+  const bool mine = cw < a.C;
+  int t0[R], n[R], longest = 0;
+  bool old[R];
+  int64_t slot[R];
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (n0 + i < a.N) {
-        A[i] = a.decay[(int64_t)c * a.N + n0 + i];
-        if (old) S[i] = st[i];
-      }
+  for (int r = 0; r < R; ++r) {
+    const int i = (int)blockIdx.y * R + r, seq = a.list[min(i, a.seqs - 1) * a.stride];
+    t0[r] = a.cu[seq];
+    n[r] = i < a.seqs ? a.cu[seq + 1] - t0[r] : 0;
+    old[r] = a.start[seq] > 0;
+    slot[r] = a.slots[seq];
+    longest = max(longest, n[r]);
   }
-  const float bias = a.dt_bias[c], skip = a.skip[c];
-  A *= LOG2E;
-  for (int t = t0; t < t0 + n; ++t) {
-    const float x = (float)((const T*)a.x)[(int64_t)t * a.C + c], z = (float)((const T*)a.z)[t * a.ldz + c];
-    const float step = softplus_f((float)((const T*)a.dt)[(int64_t)t * a.C + c] + bias), dx = step * x;
-    const T* b = (const T*)a.bc + t * a.ldbc + n0;
-    f32x4 B = {0.f, 0.f, 0.f, 0.f}, C = B;
-    if constexpr (VEC) {
-      const T4 b4 = *reinterpret_cast<const T4*>(b), c4 = *reinterpret_cast<const T4*>(b + a.N);
+  auto place = [&](int r) { return a.state + (slot[r] * a.C + c) * a.NS + n0; };
+  f32x4 S[R], A = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        B[i] = (float)b4[i];
-        C[i] = (float)c4[i];
-      }
+  for (int r = 0; r < R; ++r) {
+    S[r] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (!old[r]) continue;
+    if constexpr (VEC) {
+      S[r] = *reinterpret_cast<const f32x4*>(place(r));
     } else {
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        if (n0 + i < a.N) {
-          B[i] = (float)b[i];
-          C[i] = (float)b[a.N + i];
-        }
+        if (n0 + i < a.N) S[r][i] = place(r)[i];
     }
-    float y = 0.f;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      S[i] = fmaf(__builtin_amdgcn_exp2f(step * A[i]), S[i], dx * B[i]);
-      y = fmaf(S[i], C[i], y);
-    }
-#pragma unroll
-    for (int o = LP / 2; o > 0; o >>= 1) y += __shfl_xor(y, o, 64);
-    if (g == 0 && mine) ((T*)a.out)[(int64_t)t * a.C + c] = (T)(fmaf(skip, x, y) * silu_f(z));
   }
-  if (!mine || n <= 0) return;
   if constexpr (VEC) {
-    *reinterpret_cast<f32x4*>(st) = S;
+    A = *reinterpret_cast<const f32x4*>(a.decay + (int64_t)c * a.N + n0);
   } else {
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      if (n0 + i < a.N) st[i] = S[i];
+      if (n0 + i < a.N) A[i] = a.decay[(int64_t)c * a.N + n0 + i];
   }
-  if (a.conv && g == 0) advance_window<T>(a, slot, t0, n, old, c);
+  A *= LOG2E;
+  const float bias = a.dt_bias[c], skip = a.skip[c];
+  for (int k = 0; k < longest; ++k) {
+    float x[R], z[R], step[R];
+    f32x4 B[R], C[R];
+#pragma unroll
+    for (int r = 0; r < R; ++r) {  // (a sequence that is through repeats its last token's operands)
+      const int64_t t = max(t0[r] + min(k, n[r] - 1), 0);
+      x[r] = (float)((const T*)a.x)[t * a.C + c];
+      z[r] = (float)((const T*)a.z)[t * a.ldz + c];
+      step[r] = (float)((const T*)a.dt)[t * a.C + c];
+      const T* b = (const T*)a.bc + t * a.ldbc + n0;
+      B[r] = f32x4{0.f, 0.f, 0.f, 0.f};
+      C[r] = B[r];
+      if constexpr (VEC) {
+        const T4 b4 = *reinterpret_cast<const T4*>(b), c4 = *reinterpret_cast<const T4*>(b + a.N);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          B[r][i] = (float)b4[i];
+          C[r][i] = (float)c4[i];
+        }
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (n0 + i < a.N) {
+            B[r][i] = (float)b[i];
+            C[r][i] = (float)b[a.N + i];
+          }
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      if (k >= n[r]) continue;
+      const float s = softplus_f(step[r] + bias), dx = s * x[r];
+      float y = 0.f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        S[r][i] = fmaf(__builtin_amdgcn_exp2f(s * A[i]), S[r][i], dx * B[r][i]);
+        y = fmaf(S[r][i], C[r][i], y);
+      }
+#pragma unroll
+      for (int o = LP / 2; o > 0; o >>= 1) y += __shfl_xor(y, o, 64);
+      if (g == 0 && mine) ((T*)a.out)[(int64_t)(t0[r] + k) * a.C + c] = (T)(fmaf(skip, x[r], y) * silu_f(z[r]));
+    }
+  }
+  if (!mine) return;
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    if (n[r] <= 0) continue;
+    if constexpr (VEC) {
+      *reinterpret_cast<f32x4*>(place(r)) = S[r];
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (n0 + i < a.N) place(r)[i] = S[r][i];
+    }
+    if (a.conv && n[r] > 1 && g == 0) advance_window<T>(a, slot[r], t0[r], n[r], old[r], c);
+  }
 }
 
 template <typename T, int LP, int V>
@@ -387,18 +430,23 @@ int scan(const SelArgs& a, hipStream_t st) {
 template <typename T>
 int step(const SelArgs& a, bool aligned, hipStream_t st) {
   const int need = (a.N + 3) / 4;
-#define GO(LP)                                                                                                         \
-  if (need <= LP) {                                                                                                    \
-    const dim3 grid((a.C + NT / LP - 1) / (NT / LP), a.seqs);                                                          \
-    if (aligned && a.N == 4 * LP)                                                                                      \
-      hipLaunchKernelGGL((selective_step_kernel<T, LP, true>), grid, dim3(NT), 0, st, a);                              \
-    else                                                                                                               \
-      hipLaunchKernelGGL((selective_step_kernel<T, LP, false>), grid, dim3(NT), 0, st, a);                             \
-    DS_CHECK_LAUNCH();                                                                                                 \
-    return 0;                                                                                                          \
+#define RUN(LP, VEC, R)                                                                                                  \
+  hipLaunchKernelGGL((selective_step_kernel<T, LP, VEC, R>), dim3((a.C + NT / LP - 1) / (NT / LP), (a.seqs + R - 1) / R), \
+                     dim3(NT), 0, st, a)
+#define GO(LP)                                                                                    \
+  if (need <= LP) {                                                                               \
+    if (aligned && a.N == 4 * LP) {                                                               \
+      if ((int64_t)a.C * a.seqs * LP >= (int64_t)2048 * NT) RUN(LP, true, 4);                     \
+      else RUN(LP, true, 1);                                                                      \
+    } else {                                                                                      \
+      RUN(LP, false, 1);                                                                          \
+    }                                                                                             \
+    DS_CHECK_LAUNCH();                                                                            \
+    return 0;                                                                                     \
   }
   GO(1) GO(2) GO(4) GO(8) GO(16) GO(32) GO(64)
 #undef GO
+#undef RUN
   return (int)hipErrorInvalidValue;
 }
 

@@ -172,8 +172,8 @@ def matrix_memory(proj, lay, slots, meta, gates, bi, bf, cap, scale):
 # ------------------------------------------------------------------------------------------------ selective recurrences
 def causal_conv(x, w, b, conv_state, meta):
     """silu(conv(x) + b): x [T, C] (it may be columns of a wider matrix), w [C, taps] (last column: the current token), inputs
-    before a portion from its slot of conv_state [slots, taps - 1, C]. The slots stay as they are (`selective_scan` moves
-    them on)."""
+    before a portion from its slot of conv_state [slots, taps - 1, C]. This op or the `selective_scan` that must follow moves the
+    slots on, whichever does it more cheaply."""
     f = (selective_ops() if use_native(x) else reference).causal_conv
     return f(x, w, b, conv_state, *((meta.seq_ids, ) if use_native(x) else ()), meta.cu_q, meta.start_pos, meta.slots)
 
