@@ -286,7 +286,7 @@ def test_model_widths(tmp_path, dtype, width, vocab):
 
 @GPU
 @pytest.mark.parametrize("attn,latent,mamba", [
-    ((8, 2, 128, 128, 64, 64), (4, 64, 16, 48, 64, 72), (288, 16, 16, 4)),
+    ((8, 2, 128, 128, 64, 64), (4, 56, 16, 48, 80, 75), (288, 16, 16, 4)),
     ((4, 4, 64, 96, 100, 16), (8, 128, 64, 128, 512, 33), (512, 24, 8, 4)),
     ((12, 1, 96, 64, 48, 96), (3, 40, 24, 56, 128, 64), (100, 33, 12, 2)),
     ((2, 1, 256, 256, 80, 128), (20, 24, 8, 16, 256, 20), (64, 128, 24, 3)),
