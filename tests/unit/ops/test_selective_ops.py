@@ -249,8 +249,8 @@ def test_window_latent_attention(device, dtype, tol, dims, window):
     # the kernels turn halves: rows of pairs of neighbours are laid out so
     turned = torch.cat([torch.arange(0, r, 2), torch.arange(1, r, 2)])
     inner = torch.cat([torch.arange(d), d + turned])
-    at = torch.cat([torch.arange(H)[:, None] * (d + r) + inner for _ in (0, )]).flatten()
-    at = torch.cat([at, torch.arange(Q, Q + R), Q + R + turned, torch.arange(Q + R + r, Q + R + r + 8)])
+    heads = (torch.arange(H)[:, None] * (d + r) + inner).flatten()
+    at = torch.cat([heads, torch.arange(Q, Q + R), Q + R + turned, torch.arange(Q + R + r, Q + R + r + 8)])
     rows = [x[:, at].contiguous() for x in rows]
     rotation = Rotation({**rot, "scaling": {**rot["scaling"], "type": "yarn"}}, r)
     freq = rotation.frequencies(device)
